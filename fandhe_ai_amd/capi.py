@@ -86,6 +86,24 @@ class DecoderConfig(C.Structure):
                 ("rope_theta", C.c_double)]
 
 
+MIXER_DELTA, MIXER_LATENT_ATTENTION = 0, 1
+
+
+class LayerConfig(C.Structure):
+    """fa_layer_config: one layer of a layered decoder."""
+    _fields_ = [("mixer", C.c_int32), ("heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32),
+                ("kv_heads", C.c_uint32), ("conv", C.c_uint32), ("q_rank", C.c_uint32), ("kv_rank", C.c_uint32),
+                ("rot_dim", C.c_uint32), ("window", C.c_uint32), ("kv_from", C.c_int32), ("scale", C.c_float),
+                ("rot_base", C.c_double), ("d_ffn", C.c_uint32), ("ffn_limit", C.c_float), ("ffn_alpha", C.c_float)]
+
+
+class LayeredConfig(C.Structure):
+    _fields_ = [("n_layers", C.c_uint32), ("d_model", C.c_uint32), ("vocab", C.c_uint32), ("block_size", C.c_uint32),
+                ("max_blocks_per_seq", C.c_uint32), ("num_blocks", C.c_uint32), ("max_batch", C.c_uint32),
+                ("state_slots", C.c_uint32), ("norm_eps", C.c_float), ("logit_softcap", C.c_float), ("dtype", C.c_int),
+                ("layers", C.POINTER(LayerConfig))]
+
+
 # name -> (restype, argtypes); every symbol the header declares
 SIGNATURES = {
     "fa_last_error_message": (C.c_char_p, []),
@@ -201,6 +219,13 @@ SIGNATURES = {
     "fa_decoder_read_logits": (C.c_int32, [ctx_p, C.c_void_p, f32p]),
     "fa_decoder_logits_buffer": (C.c_int32, [C.c_void_p, C.POINTER(buf_p)]),
     "fa_decoder_read_seq_lens": (C.c_int32, [ctx_p, C.c_void_p, u32p]),
+    "fa_decoder_create_layered": (C.c_int32, [ctx_p, C.POINTER(LayeredConfig), C.POINTER(C.c_void_p)]),
+    "fa_decoder_tensor_count": (C.c_int32, [C.c_void_p, u32p]),
+    "fa_decoder_tensor_info": (C.c_int32, [C.c_void_p, C.c_uint32, C.POINTER(C.c_char_p), C.POINTER(u64), C.POINTER(u64)]),
+    "fa_decoder_set_tensor": (C.c_int32, [ctx_p, C.c_void_p, C.c_char_p, C.c_int, C.c_void_p, u64, u64]),
+    "fa_decoder_set_state_slots": (C.c_int32, [ctx_p, C.c_void_p, u32p]),
+    "fa_decoder_forward": (C.c_int32, [ctx_p, C.c_void_p, u32p, i32p, u64, u32p, f32p]),
+    "fa_decoder_debug_residuals": (C.c_int32, [C.c_void_p, f32p, u64]),
     "fa_set_tuning": (C.c_int32, [C.c_int32, C.c_int32]),
     "fa_timer_create": (C.c_int32, [ctx_p, C.POINTER(C.c_void_p)]),
     "fa_timer_start": (C.c_int32, [ctx_p, C.c_void_p]),

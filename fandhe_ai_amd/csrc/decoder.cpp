@@ -11,6 +11,7 @@
 #include <string>
 #include <vector>
 
+#include "decoder.hpp"
 #include "kernels.hpp"
 #include "runtime.hpp"
 #include "validate.hpp"
@@ -26,54 +27,21 @@ extern int g_weight_prefetch;
 }
 }
 
-struct fa_decoder {
-    uint32_t magic;
-    fa_context *ctx;
-    fa_decoder_config cfg;
-    struct Layer {
-        const fa_buffer *attn_norm = nullptr, *ffn_norm = nullptr;
-        const fa_qweight *wqkv = nullptr, *wo = nullptr, *wgu = nullptr, *wdown = nullptr;
-        fa_buffer *k_pool = nullptr, *v_pool = nullptr;
-    };
-    std::vector<Layer> layers;
-    // The large activation buffers of a prompt pass stay with the decoder from one pass to the next (grow only, until the
-    // decoder goes): the context's pool keeps at most 128 MiB of idle blocks, so buffers of hundreds of megabytes went
-    // back to the driver after every pass and were allocated again for the next (1024 prompt tokens: 12.9 -> 12.3 ms,
-    // 4 x 2048: 71.4 -> 69.1 ms without those calls).  At most kRows rows of them: about 1.8 GB at the benchmark's width.
-    struct KeptBlock {
-        void *ptr = nullptr;
-        uint64_t bytes = 0, cls = 0;
-    };
-    static constexpr int kKept = 8;
-    KeptBlock kept[kKept];
-    const fa_buffer *embed = nullptr, *final_norm = nullptr;
-    const fa_qweight *lm_head = nullptr;
-    uint32_t batch = 0;
-    // resident state and activations
-    fa_buffer *tokens = nullptr, *tables = nullptr, *seq_lens = nullptr, *pos = nullptr, *slots = nullptr;
-    fa_buffer *cos_sin = nullptr, *h = nullptr, *xq = nullptr, *sx = nullptr, *q_bf = nullptr;
-    fa_buffer *attn = nullptr, *act = nullptr, *pmax = nullptr, *logits = nullptr;
-    // captured steps, one per batch size seen (a scheduler changes the batch as requests come and go)
-    std::map<uint32_t, fa_graph *> graphs;
-    int graph_waves = 0;
-    // how the step and the prompt pass pick the next token; rng holds the generator state on the device
-    fa_sampling strategy = FA_SAMPLE_GREEDY;
-    float temperature = 1.0f;
-    uint32_t top_k = 0;
-    fa_buffer *rng = nullptr;
-    // per-row sampling table (k::RowPolicy per row) and whether the pick uses it
-    fa_buffer *policy = nullptr;
-    bool per_row = false;
-    // host mirror of the installed block tables and of the sequence lengths (advanced with every step and
-    // prompt chunk), used to validate that a prompt fits before anything is queued
-    std::vector<uint32_t> host_tables, host_lens;
-};
+namespace fa {
+// logits [batch, vocab] -> next tokens, by the decoder's sampling strategy
+void enqueue_pick(fa_decoder *d, hipStream_t s) {
+    if (d->per_row)
+        k::sample_rows_policy((const float *)d->logits->ptr, (int32_t *)d->tokens->ptr, (k::RowPolicy *)d->policy->ptr,
+                              d->batch, d->cfg.vocab, s);
+    else if (d->strategy == FA_SAMPLE_GREEDY)
+        k::argmax_rows_f32((const float *)d->logits->ptr, (int32_t *)d->tokens->ptr, d->batch, d->cfg.vocab, s);
+    else
+        k::sample_rows((const float *)d->logits->ptr, (int32_t *)d->tokens->ptr, (uint64_t *)d->rng->ptr, d->batch,
+                       d->cfg.vocab, d->strategy == FA_SAMPLE_TOP_K, d->temperature, d->top_k, s);
+}
+}  // namespace fa
 
 namespace {
-
-constexpr uint32_t kDecMagic = 0xFA0DEC01u;
-
-uint64_t round_up(uint64_t v, uint64_t to) { return (v + to - 1) / to * to; }
 
 void drop_graphs(fa_decoder *d) {
     for (auto &g : d->graphs) fa_graph_destroy(d->ctx, g.second);
@@ -82,6 +50,12 @@ void drop_graphs(fa_decoder *d) {
 
 fa_status check_dec(const fa_decoder *d) {
     if (!d || d->magic != kDecMagic) return fail(FA_ERR_INVALID_ARGUMENT, "decoder: not a decoder");
+    return FA_OK;
+}
+
+// entry points of the W8A8 stack that a layered decoder does not have
+fa_status check_llama(const fa_decoder *d, const char *what) {
+    if (d->layered) return fail(FA_ERR_UNSUPPORTED, std::string(what) + ": not for a layered decoder");
     return FA_OK;
 }
 
@@ -103,6 +77,7 @@ fa_status check_vec(const fa_decoder *d, const fa_buffer *b, uint64_t numel, con
 }
 
 void free_all(fa_context *ctx, fa_decoder *d) {
+    if (d->layered) layered_free(ctx, d);
     for (auto &kb : d->kept) {
         if (kb.ptr) pool_free(ctx, kb.ptr, kb.bytes, kb.cls);
         kb = fa_decoder::KeptBlock{};
@@ -118,18 +93,6 @@ void free_all(fa_context *ctx, fa_decoder *d) {
         if (l.v_pool) fa_buffer_free(ctx, l.v_pool);
         l.k_pool = l.v_pool = nullptr;
     }
-}
-
-// logits [batch, vocab] -> next tokens, by the decoder's sampling strategy
-void enqueue_pick(fa_decoder *d, hipStream_t s) {
-    if (d->per_row)
-        k::sample_rows_policy((const float *)d->logits->ptr, (int32_t *)d->tokens->ptr, (k::RowPolicy *)d->policy->ptr,
-                              d->batch, d->cfg.vocab, s);
-    else if (d->strategy == FA_SAMPLE_GREEDY)
-        k::argmax_rows_f32((const float *)d->logits->ptr, (int32_t *)d->tokens->ptr, d->batch, d->cfg.vocab, s);
-    else
-        k::sample_rows((const float *)d->logits->ptr, (int32_t *)d->tokens->ptr, (uint64_t *)d->rng->ptr, d->batch,
-                       d->cfg.vocab, d->strategy == FA_SAMPLE_TOP_K, d->temperature, d->top_k, s);
 }
 
 // Whether the step about to be enqueued (the host lengths already count its token) sees only short contexts: its
@@ -614,6 +577,7 @@ fa_status fa_decoder_set_layer(fa_decoder *d, uint32_t layer, const fa_buffer *a
                                const fa_qweight *wqkv, const fa_qweight *wo, const fa_qweight *wgu,
                                const fa_qweight *wdown) {
     if (fa_status s = check_dec(d)) return s;
+    if (fa_status s = check_llama(d, "decoder_set_layer")) return s;
     const fa_decoder_config &c = d->cfg;
     if (layer >= c.n_layers) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_set_layer: layer out of range");
     const uint64_t D = c.d_model, EQ = (uint64_t)c.n_heads * c.head_dim, EKV = (uint64_t)c.n_kv_heads * c.head_dim;
@@ -637,6 +601,7 @@ fa_status fa_decoder_set_layer(fa_decoder *d, uint32_t layer, const fa_buffer *a
 fa_status fa_decoder_set_head(fa_decoder *d, const fa_buffer *embed, const fa_buffer *final_norm,
                               const fa_qweight *lm_head) {
     if (fa_status s = check_dec(d)) return s;
+    if (fa_status s = check_llama(d, "decoder_set_head")) return s;
     const fa_decoder_config &c = d->cfg;
     if (fa_status s = check_vec(d, embed, (uint64_t)c.vocab * c.d_model, "decoder_set_head: embed")) return s;
     if (fa_status s = check_vec(d, final_norm, c.d_model, "decoder_set_head: final_norm")) return s;
@@ -706,6 +671,7 @@ fa_status fa_decoder_read_row_sampling(fa_context *ctx, fa_decoder *d, fa_row_sa
 
 fa_status fa_decoder_kv_pools(fa_decoder *d, uint32_t layer, fa_buffer **k_pool, fa_buffer **v_pool) {
     if (fa_status s = check_dec(d)) return s;
+    if (fa_status s = check_llama(d, "decoder_kv_pools")) return s;
     if (layer >= d->cfg.n_layers) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_kv_pools: layer out of range");
     if (k_pool) *k_pool = d->layers[layer].k_pool;
     if (v_pool) *v_pool = d->layers[layer].v_pool;
@@ -739,6 +705,7 @@ fa_status fa_decoder_set_sequences(fa_context *ctx, fa_decoder *d, uint32_t batc
         d->batch = 0;
         return fail(FA_ERR_ALLOCATION_FAILED, "decoder_set_sequences: out of host memory");
     }
+    if (d->layered) return layered_sequences_set(ctx, d);
     return FA_OK;
 }
 
@@ -774,16 +741,21 @@ fa_status fa_decoder_step(fa_context *ctx, fa_decoder *d, int32_t use_graph) {
     if (fa_status s = check_dec(d)) return s;
     if (d->ctx != ctx) return fail(FA_ERR_DEVICE_MISMATCH, "decoder_step: decoder belongs to another context");
     if (d->batch == 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_step: no sequences installed");
-    if (!d->embed || !d->final_norm || !d->lm_head) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_step: head weights missing");
-    for (auto &l : d->layers)
-        if (!l.wqkv) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_step: layer weights missing");
-    // attention workspace sized before anything is captured
-    k::PagedShape ps{};
-    ps.batch = d->batch;
-    ps.num_heads = d->cfg.n_heads;
-    ps.num_kv_heads = d->cfg.n_kv_heads;
-    ps.max_blocks_per_seq = d->cfg.max_blocks_per_seq;
-    if (fa_status s = ensure_workspace(ctx, k::paged_decode_workspace_bytes(ps, (uint32_t)g_decode_waves))) return s;
+    if (d->layered) {
+        if (fa_status s = layered_ready(d, "decoder_step")) return s;
+        if (fa_status s = layered_prepare_step(ctx, d)) return s;      // buffers sized before anything is captured
+    } else {
+        if (!d->embed || !d->final_norm || !d->lm_head) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_step: head weights missing");
+        for (auto &l : d->layers)
+            if (!l.wqkv) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_step: layer weights missing");
+        // attention workspace sized before anything is captured
+        k::PagedShape ps{};
+        ps.batch = d->batch;
+        ps.num_heads = d->cfg.n_heads;
+        ps.num_kv_heads = d->cfg.n_kv_heads;
+        ps.max_blocks_per_seq = d->cfg.max_blocks_per_seq;
+        if (fa_status s = ensure_workspace(ctx, k::paged_decode_workspace_bytes(ps, (uint32_t)g_decode_waves))) return s;
+    }
     if (fa_status s = check_step_room(d)) return s;
     // The host mirror of the lengths follows the device-side advance of this step; every return below that has
     // queued nothing takes the advance back.
@@ -792,14 +764,14 @@ fa_status fa_decoder_step(fa_context *ctx, fa_decoder *d, int32_t use_graph) {
     };
     if (!use_graph) {
         advance(1);
-        fa_status es = enqueue_step(ctx, d);
+        fa_status es = d->layered ? layered_enqueue_step(ctx, d) : enqueue_step(ctx, d);
         if (es != FA_OK) advance(-1);
         return es;
     }
     if (d->graph_waves != g_decode_waves) drop_graphs(d);
     // a graph per batch size and kind of step (bit 31: the short-context form, decided on the lengths after this step)
     advance(1);
-    const uint32_t key = d->batch | (step_is_short(d) ? 0x80000000u : 0u);
+    const uint32_t key = d->batch | (!d->layered && step_is_short(d) ? 0x80000000u : 0u);
     advance(-1);
     auto it = d->graphs.find(key);
     if (it == d->graphs.end()) {
@@ -814,7 +786,7 @@ fa_status fa_decoder_step(fa_context *ctx, fa_decoder *d, int32_t use_graph) {
         fa_status cs = fa_graph_capture_begin(ctx);
         fa_graph *g = nullptr;
         if (cs == FA_OK) {
-            fa_status es = enqueue_step(ctx, d);
+            fa_status es = d->layered ? layered_enqueue_step(ctx, d) : enqueue_step(ctx, d);
             cs = fa_graph_capture_end(ctx, &g);
             if (es != FA_OK) {
                 if (g) fa_graph_destroy(ctx, g);
@@ -835,6 +807,27 @@ fa_status fa_decoder_step(fa_context *ctx, fa_decoder *d, int32_t use_graph) {
     return ls;
 }
 
+// Rectangular prompt blocks on a layered decoder: its pass takes rows of any lengths, so padding is dropped here.
+static fa_status layered_rows(fa_context *ctx, fa_decoder *d, const int32_t *tokens, uint32_t l_new, int32_t *picked, float *logits,
+                              const uint32_t *row_lens) {
+    const uint32_t B = d->batch;
+    try {
+        std::vector<uint32_t> counts(B), want;
+        std::vector<int32_t> flat;
+        for (uint32_t b = 0; b < B; ++b) {
+            counts[b] = row_lens ? row_lens[b] : l_new;
+            if (counts[b] == 0 || counts[b] > l_new)
+                return fail(FA_ERR_INVALID_ARGUMENT, "decoder_prefill: row " + std::to_string(b) + " has a length outside 1..=l_max");
+            flat.insert(flat.end(), tokens + (uint64_t)b * l_new, tokens + (uint64_t)b * l_new + counts[b]);
+        }
+        if (!picked) return layered_forward(ctx, d, counts.data(), flat.data(), 0, nullptr, nullptr, nullptr);
+        for (uint32_t r = 0; r < flat.size(); ++r) want.push_back(r);
+        return layered_forward(ctx, d, counts.data(), flat.data(), want.size(), want.data(), logits, picked);
+    } catch (const std::exception &) {
+        return fail(FA_ERR_ALLOCATION_FAILED, "decoder_prefill: out of host memory");
+    }
+}
+
 static fa_status prefill_impl(fa_context *ctx, fa_decoder *d, const int32_t *tokens, uint32_t l_new, int32_t *picked,
                               float *logits, const uint32_t *row_lens = nullptr) {
     const bool verify = picked != nullptr, padded = row_lens != nullptr;
@@ -843,6 +836,10 @@ static fa_status prefill_impl(fa_context *ctx, fa_decoder *d, const int32_t *tok
     if (d->ctx != ctx) return fail(FA_ERR_DEVICE_MISMATCH, "decoder_prefill: decoder belongs to another context");
     if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "decoder_prefill during graph capture");
     if (d->batch == 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_prefill: no sequences installed");
+    if (d->layered) {
+        if (!tokens || l_new == 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_prefill: no tokens");
+        return layered_rows(ctx, d, tokens, l_new, picked, logits, row_lens);
+    }
     if (!d->embed || !d->final_norm || !d->lm_head) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_prefill: head weights missing");
     for (auto &l : d->layers)
         if (!l.wqkv) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_prefill: layer weights missing");
@@ -982,6 +979,10 @@ fa_status fa_decoder_rewind(fa_context *ctx, fa_decoder *d, const uint32_t *seq_
         if (seq_lens[b] > d->host_lens[b])
             return fail(FA_ERR_INVALID_ARGUMENT, "decoder_rewind: row " + std::to_string(b) + " cannot grow (" +
                                                      std::to_string(seq_lens[b]) + " > " + std::to_string(d->host_lens[b]) + ")");
+    if (d->layered && layered_has_state(d))
+        for (uint32_t b = 0; b < d->batch; ++b)
+            if (seq_lens[b] != d->host_lens[b])
+                return fail(FA_ERR_UNSUPPORTED, "decoder_rewind: a recurrent state cannot be cut back");
     if (fa_status s = fa_upload_into(ctx, seq_lens, d->batch, d->seq_lens, 0)) return s;
     std::copy(seq_lens, seq_lens + d->batch, d->host_lens.begin());
     return FA_OK;
@@ -990,6 +991,7 @@ fa_status fa_decoder_rewind(fa_context *ctx, fa_decoder *d, const uint32_t *seq_
 fa_status fa_decoder_debug_step_until(fa_context *ctx, fa_decoder *d, int32_t stop_after) {
     if (fa_status s = check_ctx(ctx)) return s;
     if (fa_status s = check_dec(d)) return s;
+    if (fa_status s = check_llama(d, "decoder_debug_step_until")) return s;
     if (d->ctx != ctx) return fail(FA_ERR_DEVICE_MISMATCH, "decoder_debug_step_until: decoder belongs to another context");
     if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "decoder_debug_step_until during graph capture");
     if (d->batch == 0 || stop_after < 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_debug_step_until: no sequences or negative stage");
@@ -1012,6 +1014,7 @@ fa_status fa_decoder_debug_step_until(fa_context *ctx, fa_decoder *d, int32_t st
 
 fa_status fa_decoder_debug_buffer(fa_decoder *d, int32_t which, fa_buffer **out) {
     if (fa_status s = check_dec(d)) return s;
+    if (fa_status s = check_llama(d, "decoder_debug_buffer")) return s;
     if (!out) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_debug_buffer: null output");
     fa_buffer *table[] = {d->h, d->xq, d->sx, d->q_bf, d->act, d->pmax, d->logits, d->cos_sin, d->slots, d->pos};
     if (which < 0 || which >= (int32_t)(sizeof(table) / sizeof(table[0])))

@@ -125,7 +125,66 @@ __global__ void __launch_bounds__(256)
     }
 }
 
+// A pass over sequences of any numbers of new tokens (none included): rows row_start[b] .. row_start[b + 1] - 1 belong to
+// sequence b and sit at positions seq_lens[b], seq_lens[b] + 1, ...  The lengths advance in a second launch.
+__global__ void __launch_bounds__(256)
+    ragged_prepare_kernel(const uint32_t *__restrict__ row_start, const uint32_t *__restrict__ tables,
+                          const uint32_t *__restrict__ seq_lens, uint32_t *__restrict__ row_seq, int32_t *__restrict__ pos,
+                          uint32_t *__restrict__ kv_slot, int32_t *__restrict__ last_rows, uint32_t batch, uint32_t rows,
+                          uint32_t block_size, uint32_t max_blocks, uint32_t num_blocks) {
+    const uint32_t r = blockIdx.x * 256 + threadIdx.x;
+    if (r >= rows) return;
+    uint32_t lo = 0, hi = batch;                     // the last b with row_start[b] <= r
+    while (hi - lo > 1) {
+        const uint32_t mid = (lo + hi) / 2;
+        if (row_start[mid] <= r) lo = mid;
+        else hi = mid;
+    }
+    const uint32_t p = seq_lens[lo] + (r - row_start[lo]);
+    uint32_t slot = 0xffffffffu;
+    if (p / block_size < max_blocks) {
+        const uint32_t id = tables[(uint64_t)lo * max_blocks + p / block_size];
+        if (id < num_blocks) slot = id * block_size + p % block_size;
+    }
+    row_seq[r] = lo;
+    pos[r] = (int32_t)p;
+    kv_slot[r] = slot;
+    if (r + 1 == row_start[lo + 1]) last_rows[lo] = (int32_t)r;
+}
+
+__global__ void ragged_advance_kernel(const uint32_t *__restrict__ row_start, uint32_t *__restrict__ seq_lens, uint32_t batch) {
+    const uint32_t b = blockIdx.x * blockDim.x + threadIdx.x;
+    if (b < batch) seq_lens[b] += row_start[b + 1] - row_start[b];
+}
+
+__global__ void __launch_bounds__(64)
+    rotation_table_kernel(const int32_t *__restrict__ pos, float *__restrict__ cos_sin, uint32_t dims, double base) {
+    const uint32_t r = blockIdx.x, half = dims / 2;
+    for (uint32_t i = threadIdx.x; i < half; i += 64) {
+        const double ang = (double)pos[r] * pow(base, -2.0 * (double)i / (double)dims);
+        cos_sin[(uint64_t)r * dims + i] = (float)cos(ang);
+        cos_sin[(uint64_t)r * dims + half + i] = (float)sin(ang);
+    }
+}
+
 }  // namespace
+
+void ragged_prepare(const uint32_t *row_start, const uint32_t *tables, const uint32_t *seq_lens, uint32_t *row_seq, int32_t *pos,
+                    uint32_t *kv_slot, int32_t *last_rows, uint32_t batch, uint32_t rows, uint32_t block_size, uint32_t max_blocks,
+                    uint32_t num_blocks, hipStream_t s) {
+    if (rows == 0) return;
+    ragged_prepare_kernel<<<(rows + 255) / 256, 256, 0, s>>>(row_start, tables, seq_lens, row_seq, pos, kv_slot, last_rows, batch, rows,
+                                                             block_size, max_blocks, num_blocks);
+}
+
+void ragged_advance(const uint32_t *row_start, uint32_t *seq_lens, uint32_t batch, hipStream_t s) {
+    ragged_advance_kernel<<<(batch + 63) / 64, 64, 0, s>>>(row_start, seq_lens, batch);
+}
+
+void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t dims, double base, hipStream_t s) {
+    if (rows == 0 || dims == 0) return;
+    rotation_table_kernel<<<rows, 64, 0, s>>>(pos, cos_sin, dims, base);
+}
 
 void prefill_prepare(const uint32_t *tables, const uint32_t *seq_lens, uint32_t *slots, float *cos_sin, uint32_t batch,
                      uint32_t l_chunk, uint32_t block_size, uint32_t max_blocks_per_seq, uint32_t num_blocks,

@@ -220,5 +220,32 @@ void rope_f32(const float *x, const int32_t *pos, float *out, uint64_t rows, uin
     rope_kernel<<<(unsigned)rows, 64, 0, s>>>(x, pos, out, (uint32_t)heads, (uint32_t)head_dim, theta);
 }
 
+namespace {
+template <typename T>
+__global__ void __launch_bounds__(256)
+    gather_rows_any_kernel(const T *__restrict__ table, uint64_t table_rows, uint32_t cols, const int32_t *__restrict__ idx,
+                           float *__restrict__ out) {
+    int64_t src = idx[blockIdx.x];
+    const bool ok = src >= 0 && (uint64_t)src < table_rows;
+    for (uint32_t c = threadIdx.x; c < cols; c += 256) {
+        float v = __uint_as_float(0x7fc00000u);
+        if (ok) {
+            if constexpr (sizeof(T) == 4) v = table[src * cols + c];
+            else v = bf16_to_f32(table[src * cols + c]);
+        }
+        out[(uint64_t)blockIdx.x * cols + c] = v;
+    }
+}
+}  // namespace
+
+void gather_rows_any(const void *table, int table_f32, uint64_t table_rows, uint64_t cols, const int32_t *idx, float *out,
+                     uint64_t rows, hipStream_t s) {
+    if (rows == 0) return;
+    if (table_f32)
+        gather_rows_any_kernel<float><<<(unsigned)rows, 256, 0, s>>>((const float *)table, table_rows, (uint32_t)cols, idx, out);
+    else
+        gather_rows_any_kernel<uint16_t><<<(unsigned)rows, 256, 0, s>>>((const uint16_t *)table, table_rows, (uint32_t)cols, idx, out);
+}
+
 }  // namespace k
 }  // namespace fa

@@ -44,6 +44,39 @@ __global__ void __launch_bounds__(kBlock) rmsnorm_kernel(const float *__restrict
     }
 }
 
+// Layer norm with a weight and no bias: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, two passes over the row held in
+// registers (VPT values per thread).
+template <int VPT, bool OUT_F32>
+__global__ void __launch_bounds__(kBlock)
+    layernorm_kernel(const float *__restrict__ x, const float *__restrict__ w, void *__restrict__ out, uint32_t hidden, uint64_t ld,
+                     float eps) {
+    __shared__ float smem[kWaves];
+    const float *row = x + (uint64_t)blockIdx.x * hidden;
+    float v[VPT], sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const uint32_t c = threadIdx.x + i * kBlock;
+        v[i] = c < hidden ? row[c] : 0.0f;
+        sum += v[i];
+    }
+    const float mean = block_sum<float, kWaves, true>(sum, smem) / (float)hidden;
+    float sq = 0.0f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const float c = threadIdx.x + i * kBlock < hidden ? v[i] - mean : 0.0f;
+        sq = fmaf(c, c, sq);
+    }
+    const float rstd = 1.0f / sqrtf(block_sum<float, kWaves, true>(sq, smem) / (float)hidden + eps);
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const uint32_t c = threadIdx.x + i * kBlock;
+        if (c >= ld) continue;
+        const float y = c < hidden ? (v[i] - mean) * rstd * w[c] : 0.0f;
+        if (OUT_F32) ((float *)out)[blockIdx.x * ld + c] = y;
+        else ((uint16_t *)out)[blockIdx.x * ld + c] = f32_to_bf16(y);
+    }
+}
+
 template <bool IN_BF16>
 __device__ __forceinline__ float load_in(const void *x, uint64_t i) {
     if (IN_BF16) return bf16_to_f32(((const uint16_t *)x)[i]);
@@ -540,6 +573,19 @@ __global__ void zero_f32_kernel(float *p) {
 }
 
 }  // namespace
+
+void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps,
+                    hipStream_t s) {
+    if (rows == 0) return;
+    const uint64_t vpt = (ld + kBlock - 1) / kBlock;
+#define FA_LN(V)                                                                                                              \
+    out_f32 ? layernorm_kernel<V, true><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)                \
+            : layernorm_kernel<V, false><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)
+    if (vpt <= 4) FA_LN(4);
+    else if (vpt <= 16) FA_LN(16);
+    else FA_LN(64);                                  // rows up to 16384
+#undef FA_LN
+}
 
 void rmsnorm_f32(const float *x, const float *w, float *out, uint64_t rows, uint64_t hidden, float eps,
                  hipStream_t s) {

@@ -317,6 +317,121 @@ void paged_attention_prefill_bf16(const uint16_t *q, const uint16_t *k_pool, con
                                   const uint32_t *tables, const uint32_t *seq_lens, const PagedShape &ps,
                                   uint32_t waves_per_cu, void *workspace, void *out, int out_bf16, hipStream_t s);
 
+// ---- plain (unquantized) linears (kern_linear.hip, kern_gemm_mfma.hip) ----------
+// A weight W[n, k] of a bf16 model is kept as tiles of 16 output columns x 32 k (1 KiB, the byte order of the int8
+// tiles: byte ((g*16 + c)*16 + 2j) holds W[16*nt + c][32*kt + 8g + j]), tiles ordered [nt][kt], zeros in the padding; of
+// an f32 model as rows [16 * n_tiles][32 * k_tiles].  A batched weight is `batches` of them behind each other.
+// k_tiles is even (k padded to 64), so that two tiles of a column are one stage of the large-tile GEMM.
+struct LinearWeight {
+    const void *w = nullptr;
+    uint32_t n = 0;              // columns the epilogue may store
+    uint32_t n_tiles = 0, k_tiles = 0, batches = 1;
+};
+// What becomes of y = a W^T (f32):
+struct LinearEpilogue {
+    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4 };
+    int mode = kStore;
+    void *out = nullptr;         // [m, ld_out], f32 or bf16; kResidual: the f32 residual itself
+    int out_f32 = 0;
+    uint32_t ld_out = 0;
+    uint64_t out_batch = 0;      // elements between the outputs of two batch entries
+    uint32_t n_lo = 0xffffffffu; // kStore: columns from n_lo on go to out_hi [m, ld_hi], f32, instead
+    float *out_hi = nullptr;
+    uint32_t ld_hi = 0;
+    const float *scale = nullptr;    // kResidual: out[r, c] += scale[c] * y
+    // kGlu: tiles alternate gate / up; g = min(gate, limit), u = clamp(up, +-limit), out = g sigmoid(alpha g) (u + 1)
+    float limit = 0.0f, alpha = 0.0f;
+    float cap = 0.0f;            // kSoftcap: cap tanh(y / cap); cap <= 0: y
+    const float *gate = nullptr; // kHeadGate: y * sigmoid(gate[r * ld_gate + batch])
+    uint32_t ld_gate = 0;
+};
+// a [m, lda] (batch entry i starts i * a_batch elements further on) with 32 * k_tiles readable, finite elements per row;
+// what lies past the weight's own k meets zero weights.
+void linear_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep,
+                 int num_cus, hipStream_t s);
+void linear_f32(const float *a, uint64_t lda, uint64_t a_batch, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep,
+                hipStream_t s);
+// The large-tile form (kern_gemm_mfma.hip): m >= 256, one batch entry, lda == 32 * k_tiles.
+bool gemm_bf16_big_applies(uint64_t lda, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus);
+void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus, hipStream_t s);
+// Packs `rows` source rows of `cols` values (bf16 bits or f32; element (r, c) at src[r * row_stride + c * col_stride]) into
+// columns dst_row(r) of a weight: dst_row(r) = n0 + (r / group) * pitch + r % group.
+void pack_linear(const void *src, int src_f32, uint64_t row_stride, uint64_t col_stride, uint32_t rows, uint32_t cols, void *dst,
+                 int dst_f32, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch, hipStream_t s);
+
+// ---- layered decoder: rows, norms (kern_decoder.hip, kern_norm_quant.hip) ----------------
+// One pass over sequences of any numbers of new tokens: sequence b owns rows row_start[b] .. row_start[b + 1] - 1.
+struct RaggedRows {
+    const uint32_t *row_start;   // [batch + 1]
+    const uint32_t *row_seq;     // [rows]
+    const int32_t *pos;          // [rows] position of the row's token
+    const uint32_t *kv_slot;     // [rows] cache row of the token, UINT32_MAX when its table has none
+    const uint32_t *state_slot;  // [batch]
+    const uint32_t *tables;      // [batch][max_blocks]
+    uint32_t rows, batch, block_size, max_blocks, num_blocks;
+};
+// Fills row_seq, pos, kv_slot from the resident lengths (before this pass), and last_rows[b].  advance_ragged then
+// adds the new tokens to the lengths.
+void ragged_prepare(const uint32_t *row_start, const uint32_t *tables, const uint32_t *seq_lens, uint32_t *row_seq, int32_t *pos,
+                    uint32_t *kv_slot, int32_t *last_rows, uint32_t batch, uint32_t rows, uint32_t block_size, uint32_t max_blocks,
+                    uint32_t num_blocks, hipStream_t s);
+void ragged_advance(const uint32_t *row_start, uint32_t *seq_lens, uint32_t batch, hipStream_t s);
+// cos_sin [rows, dims] of the rows' positions (cos in the first half, sin in the second), angles formed in double
+void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t dims, double base, hipStream_t s);
+// (x - mean) / sqrt(variance + eps) * w per row; out f32 or bf16 with pitch ld, zeros past hidden
+void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps,
+                    hipStream_t s);
+// embedding rows (bf16 bits or f32) as f32
+void gather_rows_any(const void *table, int table_f32, uint64_t table_rows, uint64_t cols, const int32_t *idx, float *out,
+                     uint64_t rows, hipStream_t s);
+
+// ---- latent attention (kern_latent.hip) -----------------------------------------
+struct LatentShape {
+    uint32_t heads, dim, rot, vdim, q_rank, kv_rank;     // sizes of the configuration
+    uint32_t dim_p, rot_p, rank_p;                       // padded to 32: q rows are [heads][dim_p + rot_p], cache rows and
+                                                         // absorbed queries [rank_p + rot_p], padding zero
+    uint32_t window;                                     // keys p - window + 1 .. p
+    float scale, eps;
+    uint64_t pool_rows;
+};
+// From y [rows, ld] f32 = q latent | kv latent | rotated key part | gates: RMS norm of the q latent -> cq [rows, ld_cq];
+// with a pool: RMS norm of the latent and rotation of the key part -> the token's cache row.
+void latent_prepare(const float *y, uint32_t ld, const float *q_norm, const float *kv_norm, const float *cos_sin, void *cq,
+                    uint32_t ld_cq, void *pool, int is_f32, const LatentShape &sh, const RaggedRows &rr, hipStream_t s);
+// Rotated part of q [rows, heads, dim_p + rot_p] -> dst (pitch dst_pitch per head, at dst_off; may be q itself)
+void latent_rotate_query(const void *q, const float *cos_sin, void *dst, uint32_t dst_pitch, uint32_t dst_off, int is_f32,
+                         const LatentShape &sh, uint32_t rows, hipStream_t s);
+// Attention of absorbed queries qa [rows, heads, rank_p + rot_p] over cached rows: out [rows, heads, rank_p] = softmax-weighted
+// latents.  bf16 with sizes the matrix-core kernel holds: that kernel (workspace for the key splits); otherwise a plain one.
+uint64_t latent_attention_workspace_bytes(const LatentShape &sh, uint32_t rows, uint32_t batch);
+void latent_attention(const void *qa, const void *pool, void *out, int is_f32, const LatentShape &sh, const RaggedRows &rr,
+                      uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
+
+// ---- gated delta rule (kern_delta.hip) --------------------------------------------
+struct DeltaShape {
+    uint32_t heads, kv_heads, dim, vdim, taps;
+    __host__ __device__ uint32_t qkv() const { return 2 * kv_heads * dim + heads * vdim; }       // channels that pass the convolution
+    __host__ __device__ uint32_t vdim_p() const { return (vdim + 3) / 4 * 4; }
+    float eps;
+};
+struct DeltaIo {
+    const void *y;               // [rows, ld_y] q | k | v | g (bf16 or f32)
+    uint32_t ld_y;
+    const float *ba;             // [rows, ld_ba] b | a projections
+    uint32_t ld_ba;
+    const float *conv;           // [qkv][taps]
+    const float *a_log, *dt_bias, *norm;
+    float *state;                // [slots][heads][dim][vdim_p]
+    void *ring;                  // [slots][taps][qkv], input of position p in entry p % taps (type of y)
+    void *out;                   // [rows, ld_out] gated, normed read-outs (type of y)
+    uint32_t ld_out;
+    float *scratch;              // delta_scratch_bytes: chunk form only
+};
+constexpr uint32_t kDeltaMaxDim = 256, kDeltaMaxVdim = 1024;
+uint64_t delta_scratch_bytes(const DeltaShape &sh, uint32_t rows, uint32_t batch);
+// max_new: most new tokens of any sequence of the pass
+void delta_mixer(const DeltaShape &sh, const DeltaIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, hipStream_t s);
+
 // ---- sampling (kern_sampling.hip) ------------------------------------------------
 // one row of a per-row sampling table (the layout of fa_row_sampling)
 struct RowPolicy {

@@ -1,0 +1,799 @@
+// Layered decoders: stacks whose layers are described one by one (fa_layered_config).  Weights, the paged latent caches and
+// the recurrent states live here; sequences, sampling, recorded steps and the entry points are decoder.cpp's.
+// One launch sequence serves decode steps, prompt passes and mixed batches: a pass is a list of rows, each with its
+// sequence, position, cache row and state slot (k::RaggedRows), and every kernel takes any number of rows per sequence.
+#include <algorithm>
+#include <cmath>
+#include <cstring>
+#include <functional>
+#include <new>
+#include <string>
+#include <vector>
+
+#include "decoder.hpp"
+#include "validate.hpp"
+
+namespace fa {
+
+int g_layered_rows = 0;      // rows per internal pass of a prompt (tuning; below 64: the built-in figure)
+
+namespace {
+
+uint32_t pad_to(uint32_t v, uint32_t to) { return (v + to - 1) / to * to; }
+
+struct Tensor {
+    std::string name;
+    uint64_t rows, cols;                              // cols 0: a vector
+    bool set = false;
+    // places the tensor, already on the device as bf16 bits or f32, where the kernels read it
+    std::function<void(const void *src, int src_f32, hipStream_t s)> place;
+};
+
+struct Layer {
+    fa_layer_config cfg;
+    float *norm1 = nullptr, *norm2 = nullptr, *ls1 = nullptr, *ls2 = nullptr;
+    k::LinearWeight in, out, gate_up, down;
+    // latent attention
+    k::LatentShape la{};
+    k::LinearWeight uq, uk, uv;
+    float *q_norm = nullptr, *kv_norm = nullptr;
+    void *pool = nullptr;
+    uint32_t rotation = 0;                            // index of its cos / sin table
+    // delta
+    k::DeltaShape de{};
+    float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *head_norm = nullptr, *state = nullptr;
+    void *ring = nullptr;
+};
+
+// Activations of a pass of up to `rows` rows, one allocation.  Every section keeps its place and element type for the
+// arena's life and starts as zeros: what lies behind a row's own width is always finite.
+struct Arena {
+    void *base = nullptr;
+    uint64_t bytes = 0, cls = 0;
+    uint32_t rows = 0;
+    float *x = nullptr, *y32 = nullptr, *ba = nullptr, *head_x = nullptr, *delta_scratch = nullptr;
+    void *hn = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *olat = nullptr, *o = nullptr, *act = nullptr;
+    uint32_t *row_seq = nullptr, *kv_slot = nullptr, *row_start = nullptr;
+    int32_t *pos = nullptr, *tokens = nullptr, *want = nullptr;
+    std::vector<float *> cos_sin;
+};
+
+}  // namespace
+
+struct LayeredState {
+    fa_layered_config cfg{};
+    std::vector<fa_layer_config> layer_cfgs;
+    std::vector<Layer> layers;
+    std::vector<Tensor> tensors;
+    std::vector<fa_buffer *> owned;
+    std::vector<std::pair<uint32_t, double>> rotations;      // distinct (dims, base)
+    void *embed = nullptr;
+    float *final_norm = nullptr;
+    k::LinearWeight head;
+    fa_buffer *state_slots = nullptr, *unit_starts = nullptr, *last_rows = nullptr;
+    Arena step, pass;
+    bool has_state = false, slots_set = false;
+    // test aid: the next pass copies the residual after every layer here ([layers, rows, d_model])
+    float *trace = nullptr;
+    uint64_t trace_rows = 0;
+    int is_f32 = 0;
+    uint64_t esz = 2;
+};
+
+namespace {
+
+// widest of every activation over the layers
+struct Widths {
+    uint64_t hn = 0, y32 = 0, y = 0, ba = 0, cq = 0, q = 0, qa = 0, olat = 0, o = 0, act = 0;
+};
+
+Widths widths(const LayeredState &L) {
+    Widths w;
+    w.hn = pad_to(L.cfg.d_model, 64);
+    for (const Layer &l : L.layers) {
+        if (l.cfg.mixer == FA_MIXER_DELTA) {
+            w.y = std::max<uint64_t>(w.y, pad_to(l.de.qkv() + l.de.heads * l.de.vdim, 8));
+            w.ba = std::max<uint64_t>(w.ba, 2 * l.de.heads);
+        } else {
+            w.y32 = std::max<uint64_t>(w.y32, pad_to(l.in.n, 4));
+            w.cq = std::max<uint64_t>(w.cq, pad_to(l.la.q_rank, 64));
+            w.q = std::max<uint64_t>(w.q, (uint64_t)l.la.heads * (l.la.dim_p + l.la.rot_p));
+            w.qa = std::max<uint64_t>(w.qa, (uint64_t)l.la.heads * (l.la.rank_p + l.la.rot_p));
+            w.olat = std::max<uint64_t>(w.olat, (uint64_t)l.la.heads * l.la.rank_p);
+        }
+        w.o = std::max<uint64_t>(w.o, pad_to(l.cfg.heads * l.cfg.vdim, 64));
+        if (l.cfg.d_ffn) w.act = std::max<uint64_t>(w.act, pad_to(l.cfg.d_ffn, 64));
+    }
+    return w;
+}
+
+fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t rows) {
+    if (a.rows >= rows) return FA_OK;
+    if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "layered decoder: activations must be sized before a capture");
+    if (a.base) pool_free(ctx, a.base, a.bytes, a.cls);
+    a = Arena();
+    const Widths w = widths(L);
+    const uint64_t R = rows, B = L.cfg.max_batch, E = L.esz;
+    uint64_t total = 0;
+    std::vector<std::pair<void **, uint64_t>> parts;
+    auto add = [&](void **p, uint64_t bytes) {
+        parts.emplace_back(p, total);
+        total += round_up(bytes + 512, 256);          // slack: operand reads may run past a row's own width
+    };
+    a.cos_sin.resize(L.rotations.size());
+    add((void **)&a.x, R * L.cfg.d_model * 4);
+    add((void **)&a.head_x, std::max(R, B) * L.cfg.d_model * 4);
+    add(&a.hn, std::max(R, B) * w.hn * E);
+    add((void **)&a.y32, R * w.y32 * 4);
+    add(&a.y, R * w.y * E);
+    add((void **)&a.ba, R * w.ba * 4);
+    add(&a.cq, R * w.cq * E);
+    add(&a.q, R * w.q * E);
+    add(&a.qa, R * w.qa * E);
+    add(&a.olat, R * w.olat * E);
+    add(&a.o, R * w.o * E);
+    add(&a.act, R * w.act * E);
+    add((void **)&a.row_seq, R * 4);
+    add((void **)&a.kv_slot, R * 4);
+    add((void **)&a.pos, R * 4);
+    add((void **)&a.tokens, R * 4);
+    add((void **)&a.want, std::max(R, B) * 4);
+    add((void **)&a.row_start, (B + 1) * 4);
+    for (size_t i = 0; i < L.rotations.size(); ++i) add((void **)&a.cos_sin[i], R * L.rotations[i].first * 4);
+    uint64_t scratch = 0;
+    for (const Layer &l : L.layers)
+        if (l.cfg.mixer == FA_MIXER_DELTA) scratch = std::max(scratch, k::delta_scratch_bytes(l.de, rows, (uint32_t)B));
+    add((void **)&a.delta_scratch, scratch);
+    if (fa_status s = pool_alloc(ctx, total, &a.base, &a.cls)) {
+        a = Arena();
+        return s;
+    }
+    a.bytes = total;
+    a.rows = rows;
+    for (auto &p : parts) *p.first = (uint8_t *)a.base + p.second;
+    k::fill_u32((uint32_t *)a.base, 0, total / 4, ctx->stream);
+    return after_launch(ctx, "layered decoder activations");
+}
+
+void linear(fa_context *ctx, const LayeredState &L, const void *a, uint64_t lda, uint64_t a_batch, uint64_t m, const k::LinearWeight &w,
+            k::LinearEpilogue ep) {
+    if (L.is_f32) k::linear_f32((const float *)a, lda, a_batch, m, w, ep, ctx->stream);
+    else k::linear_bf16((const uint16_t *)a, lda, a_batch, m, w, ep, ctx->props.multiProcessorCount, ctx->stream);
+}
+
+k::LinearEpilogue store_to(void *out, uint64_t ld, int out_f32) {
+    k::LinearEpilogue e;
+    e.out = out;
+    e.ld_out = (uint32_t)ld;
+    e.out_f32 = out_f32;
+    return e;
+}
+
+// All layers over the rows of a pass whose embeddings are in a.x.
+fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::RaggedRows &rr, uint32_t max_new, uint64_t trace_row0) {
+    LayeredState &L = *d->layered;
+    hipStream_t s = ctx->stream;
+    const uint32_t M = rr.rows, D = L.cfg.d_model, ld_hn = pad_to(D, 64);
+    const float eps = L.cfg.norm_eps;
+    const int f32 = L.is_f32;
+    for (size_t i = 0; i < L.rotations.size(); ++i) k::rotation_table(rr.pos, a.cos_sin[i], M, L.rotations[i].first, L.rotations[i].second, s);
+    for (size_t li = 0; li < L.layers.size(); ++li) {
+        const Layer &l = L.layers[li];
+        k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);
+        const uint32_t ow = l.cfg.heads * l.cfg.vdim, ld_o = pad_to(ow, 64);
+        if (l.cfg.mixer == FA_MIXER_DELTA) {
+            const uint32_t n_lo = l.de.qkv() + ow, ld_y = pad_to(n_lo, 8);
+            k::LinearEpilogue e = store_to(a.y, ld_y, f32);
+            e.n_lo = n_lo;
+            e.out_hi = a.ba;
+            e.ld_hi = 2 * l.de.heads;
+            linear(ctx, L, a.hn, ld_hn, 0, M, l.in, e);
+            k::DeltaIo io{a.y, ld_y, a.ba, 2 * l.de.heads, l.conv, l.a_log, l.dt_bias, l.head_norm, l.state, l.ring, a.o, ld_o, a.delta_scratch};
+            k::delta_mixer(l.de, io, f32, rr, max_new, s);
+        } else {
+            const k::LatentShape &sh = l.la;
+            const uint32_t ld_y = pad_to(l.in.n, 4), ld_cq = pad_to(sh.q_rank, 64), qw = sh.dim_p + sh.rot_p, kw = sh.rank_p + sh.rot_p;
+            const bool own = l.cfg.kv_from < 0;
+            const float *cs = a.cos_sin[l.rotation];
+            void *pool = own ? l.pool : L.layers[l.cfg.kv_from].pool;
+            linear(ctx, L, a.hn, ld_hn, 0, M, l.in, store_to(a.y32, ld_y, 1));
+            k::latent_prepare(a.y32, ld_y, l.q_norm, l.kv_norm, cs, a.cq, ld_cq, own ? pool : nullptr, f32, sh, rr, s);
+            linear(ctx, L, a.cq, ld_cq, 0, M, l.uq, store_to(a.q, (uint64_t)sh.heads * qw, f32));
+            k::LinearEpilogue e = store_to(a.qa, (uint64_t)sh.heads * kw, f32);
+            e.out_batch = kw;
+            linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, l.uk, e);
+            k::latent_rotate_query(a.q, cs, a.qa, kw, sh.rank_p, f32, sh, M, s);
+            k::latent_attention(a.qa, pool, a.olat, f32, sh, rr, max_new, ctx->workspace, ctx->props.multiProcessorCount, s);
+            e = store_to(a.o, ld_o, f32);
+            e.mode = k::LinearEpilogue::kHeadGate;
+            e.out_batch = sh.vdim;
+            e.gate = a.y32 + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
+            e.ld_gate = ld_y;
+            linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, l.uv, e);
+        }
+        k::LinearEpilogue r = store_to(a.x, D, 1);
+        r.mode = k::LinearEpilogue::kResidual;
+        r.scale = l.ls1;
+        linear(ctx, L, a.o, ld_o, 0, M, l.out, r);
+        if (l.cfg.d_ffn) {
+            const uint32_t ld_act = pad_to(l.cfg.d_ffn, 64);
+            k::layernorm_rows(a.x, l.norm2, a.hn, f32, M, D, ld_hn, eps, s);
+            k::LinearEpilogue g = store_to(a.act, ld_act, f32);
+            g.mode = k::LinearEpilogue::kGlu;
+            g.limit = l.cfg.ffn_limit;
+            g.alpha = l.cfg.ffn_alpha;
+            linear(ctx, L, a.hn, ld_hn, 0, M, l.gate_up, g);
+            r.scale = l.ls2;
+            linear(ctx, L, a.act, ld_act, 0, M, l.down, r);
+        }
+        if (L.trace) {
+            hipError_t e = hipMemcpyAsync(L.trace + (li * L.trace_rows + trace_row0) * D, a.x, (uint64_t)M * D * 4, hipMemcpyDeviceToHost, s);
+            if (e == hipSuccess) e = hipStreamSynchronize(s);
+            if (e != hipSuccess) return hip_fail(ctx, e, "residual download", FA_ERR_TRANSFER_FAILED);
+        }
+    }
+    return FA_OK;
+}
+
+// Final norm and head over rows of f32 residuals.
+void enqueue_head(fa_context *ctx, LayeredState &L, Arena &a, const float *x, uint32_t rows, float *logits) {
+    const uint32_t ld_hn = pad_to(L.cfg.d_model, 64);
+    k::layernorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
+    k::LinearEpilogue e = store_to(logits, L.cfg.vocab, 1);
+    e.mode = k::LinearEpilogue::kSoftcap;
+    e.cap = L.cfg.logit_softcap;
+    linear(ctx, L, a.hn, ld_hn, 0, rows, L.head, e);
+}
+
+k::RaggedRows ragged(const fa_decoder *d, const Arena &a, const uint32_t *row_start, uint32_t rows) {
+    const fa_decoder_config &c = d->cfg;
+    return k::RaggedRows{row_start, a.row_seq, a.pos, a.kv_slot, (const uint32_t *)d->layered->state_slots->ptr, (const uint32_t *)d->tables->ptr,
+                         rows, d->batch, c.block_size, c.max_blocks_per_seq, c.num_blocks};
+}
+
+void prepare_rows(fa_context *ctx, fa_decoder *d, Arena &a, const uint32_t *row_start, uint32_t rows) {
+    const fa_decoder_config &c = d->cfg;
+    k::ragged_prepare(row_start, (const uint32_t *)d->tables->ptr, (const uint32_t *)d->seq_lens->ptr, a.row_seq, a.pos, a.kv_slot,
+                      (int32_t *)d->layered->last_rows->ptr, d->batch, rows, c.block_size, c.max_blocks_per_seq, c.num_blocks, ctx->stream);
+    k::ragged_advance(row_start, (uint32_t *)d->seq_lens->ptr, d->batch, ctx->stream);
+}
+
+fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch) {
+    uint64_t need = 0;
+    for (const Layer &l : L.layers)
+        if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) need = std::max(need, k::latent_attention_workspace_bytes(l.la, rows, batch));
+    return need ? ensure_workspace(ctx, need) : FA_OK;
+}
+
+uint64_t pass_rows() { return g_layered_rows >= 64 ? (uint64_t)g_layered_rows : 8192; }
+
+fa_status upload(fa_context *ctx, void *dst, const void *src, uint64_t bytes) {
+    hipError_t e = hipMemcpyAsync(dst, src, bytes, hipMemcpyHostToDevice, ctx->stream);
+    if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
+    return e == hipSuccess ? FA_OK : hip_fail(ctx, e, "upload of a pass", FA_ERR_TRANSFER_FAILED);
+}
+
+}  // namespace
+
+void layered_free(fa_context *ctx, fa_decoder *d) {
+    LayeredState *L = d->layered;
+    for (Arena *a : {&L->step, &L->pass})
+        if (a->base) pool_free(ctx, a->base, a->bytes, a->cls);
+    for (fa_buffer *b : L->owned) fa_buffer_free(ctx, b);
+    delete L;
+    d->layered = nullptr;
+}
+
+fa_status layered_ready(const fa_decoder *d, const char *what) {
+    for (const Tensor &t : d->layered->tensors)
+        if (!t.set) return fail(FA_ERR_INVALID_ARGUMENT, std::string(what) + ": tensor " + t.name + " missing");
+    if (d->layered->has_state && !d->layered->slots_set) return fail(FA_ERR_INVALID_ARGUMENT, std::string(what) + ": state slots missing");
+    return FA_OK;
+}
+
+bool layered_has_state(const fa_decoder *d) { return d->layered->has_state; }
+
+fa_status layered_sequences_set(fa_context *ctx, fa_decoder *d) {
+    LayeredState &L = *d->layered;
+    L.slots_set = d->batch <= L.cfg.state_slots;
+    if (!L.slots_set) return FA_OK;
+    std::vector<uint32_t> iota(d->batch);
+    for (uint32_t b = 0; b < d->batch; ++b) iota[b] = b;
+    return fa_upload_into(ctx, iota.data(), d->batch, L.state_slots, 0);
+}
+
+fa_status layered_prepare_step(fa_context *ctx, fa_decoder *d) {
+    LayeredState &L = *d->layered;
+    if (fa_status s = arena_reserve(ctx, L, L.step, L.cfg.max_batch)) return s;
+    return attention_workspace(ctx, L, d->batch, d->batch);
+}
+
+fa_status layered_enqueue_step(fa_context *ctx, fa_decoder *d) {
+    LayeredState &L = *d->layered;
+    Arena &a = L.step;
+    const uint32_t B = d->batch;
+    const uint32_t *starts = (const uint32_t *)L.unit_starts->ptr;
+    prepare_rows(ctx, d, a, starts, B);
+    k::gather_rows_any(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, (const int32_t *)d->tokens->ptr, a.x, B, ctx->stream);
+    if (fa_status s = enqueue_layers(ctx, d, a, ragged(d, a, starts, B), 1, 0)) return s;
+    enqueue_head(ctx, L, a, a.x, B, (float *)d->logits->ptr);
+    enqueue_pick(d, ctx->stream);
+    return after_launch(ctx, "layered decoder step");
+}
+
+fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts, const int32_t *tokens, uint64_t n_want,
+                          const uint32_t *want, float *logits, int32_t *picked) {
+    LayeredState &L = *d->layered;
+    const fa_decoder_config &c = d->cfg;
+    const uint32_t B = d->batch;
+    if (fa_status s = layered_ready(d, "decoder pass")) return s;
+    uint64_t total = 0;
+    for (uint32_t b = 0; b < B; ++b) {
+        const uint64_t end = (uint64_t)d->host_lens[b] + counts[b];
+        if (end > (uint64_t)c.max_blocks_per_seq * c.block_size)
+            return fail(FA_ERR_INVALID_ARGUMENT, "paged_kv: row " + std::to_string(b) + " has no room for the prompt");
+        for (uint64_t i = 0; i < (end + c.block_size - 1) / c.block_size; ++i)
+            if (d->host_tables[(uint64_t)b * c.max_blocks_per_seq + i] >= c.num_blocks)
+                return fail(FA_ERR_INVALID_ARGUMENT, "paged_kv: row " + std::to_string(b) + " entry " + std::to_string(i) + " is not a valid block id");
+        total += counts[b];
+    }
+    if (total == 0 || total > INT32_MAX) return fail(FA_ERR_INVALID_ARGUMENT, "decoder pass: no tokens");
+    for (uint64_t i = 0; i < total; ++i)
+        if (tokens[i] < 0 || (uint32_t)tokens[i] >= c.vocab) return fail(FA_ERR_INVALID_ARGUMENT, "decoder pass: token id outside the vocabulary");
+    const bool last_only = want == nullptr && picked == nullptr && logits == nullptr;
+    for (uint64_t i = 0; i < n_want; ++i)
+        if (want[i] >= total || (i && want[i] <= want[i - 1]))
+            return fail(FA_ERR_INVALID_ARGUMENT, "decoder pass: wanted places must be ascending and below the number of tokens");
+    if (last_only)
+        for (uint32_t b = 0; b < B; ++b)
+            if (counts[b] == 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder pass: row " + std::to_string(b) + " brings no tokens");
+
+    // the arena grows in powers of two up to a full pass
+    const uint64_t budget = pass_rows();
+    uint32_t cap = 64;
+    while (cap < std::min<uint64_t>(total, budget)) cap *= 2;
+    if (fa_status s = arena_reserve(ctx, L, L.pass, cap)) return s;
+    Arena &a = L.pass;
+    if (fa_status s = attention_workspace(ctx, L, (uint32_t)std::min<uint64_t>(total, budget), B)) return s;
+    // logits of wanted rows: at most kHeadRows at a time
+    constexpr uint32_t kHeadRows = 1024;
+    fa_buffer *lbuf = nullptr, *pbuf = nullptr;
+    if (n_want) {
+        const uint64_t rows = std::min<uint64_t>({n_want, kHeadRows, a.rows});
+        if (fa_status s = make_buffer(ctx, FA_F32, rows * c.vocab, false, &lbuf)) return s;
+        if (picked)
+            if (fa_status s = make_buffer(ctx, FA_I32, rows, false, &pbuf)) {
+                fa_buffer_free(ctx, lbuf);
+                return s;
+            }
+    }
+    auto run = [&]() -> fa_status {
+        std::vector<uint32_t> done(B, 0), starts(B + 1), first(B);
+        std::vector<int32_t> stage, pick_rows;
+        uint64_t w_at = 0, placed = 0, tok0 = 0;
+        for (uint32_t b = 0; b < B; ++b) {
+            first[b] = (uint32_t)tok0;
+            tok0 += counts[b];
+        }
+        while (placed < total) {
+            // sequences in order, each as much as the pass has room for
+            uint32_t rows = 0, max_new = 0;
+            stage.clear();
+            pick_rows.clear();
+            std::vector<int32_t> last(B, -1);
+            const uint64_t w_lo = w_at;
+            for (uint32_t b = 0; b < B; ++b) {
+                starts[b] = rows;
+                const uint32_t n = (uint32_t)std::min<uint64_t>(counts[b] - done[b], budget - rows);
+                const uint32_t g0 = first[b] + done[b];
+                for (uint32_t i = 0; i < n; ++i) stage.push_back(tokens[g0 + i]);
+                while (w_at < n_want && want[w_at] < g0 + n) pick_rows.push_back((int32_t)(rows + want[w_at++] - g0));
+                done[b] += n;
+                rows += n;
+                max_new = std::max(max_new, n);
+                if (n && done[b] == counts[b]) last[b] = (int32_t)rows - 1;
+            }
+            starts[B] = rows;
+            if (fa_status s = upload(ctx, a.row_start, starts.data(), (B + 1) * 4)) return s;
+            if (fa_status s = upload(ctx, a.tokens, stage.data(), (uint64_t)rows * 4)) return s;
+            prepare_rows(ctx, d, a, a.row_start, rows);
+            k::gather_rows_any(L.embed, L.is_f32, c.vocab, c.d_model, a.tokens, a.x, rows, ctx->stream);
+            if (fa_status s = enqueue_layers(ctx, d, a, ragged(d, a, a.row_start, rows), max_new, placed)) return s;
+            for (uint32_t b = 0; b < B; ++b) d->host_lens[b] += starts[b + 1] - starts[b];
+            placed += rows;
+            if (last_only) {
+                // the last rows of the sequences that end in this pass wait in the decoder's own residual rows
+                for (uint32_t b = 0; b < B; ++b)
+                    if (last[b] >= 0) {
+                        hipError_t e = hipMemcpyAsync((float *)d->h->ptr + (uint64_t)b * c.d_model, a.x + (uint64_t)last[b] * c.d_model,
+                                                      (uint64_t)c.d_model * 4, hipMemcpyDeviceToDevice, ctx->stream);
+                        if (e != hipSuccess) return hip_fail(ctx, e, "last rows", FA_ERR_TRANSFER_FAILED);
+                    }
+            }
+            for (uint64_t i = 0; i < pick_rows.size(); i += kHeadRows) {
+                const uint32_t n = (uint32_t)std::min<uint64_t>(pick_rows.size() - i, kHeadRows);
+                if (fa_status s = upload(ctx, a.want, pick_rows.data() + i, (uint64_t)n * 4)) return s;
+                k::gather_rows_f32(a.x, rows, c.d_model, a.want, a.head_x, n, ctx->stream);
+                enqueue_head(ctx, L, a, a.head_x, n, (float *)lbuf->ptr);
+                hipError_t e = hipSuccess;
+                if (logits) e = hipMemcpyAsync(logits + (w_lo + i) * c.vocab, lbuf->ptr, (uint64_t)n * c.vocab * 4, hipMemcpyDeviceToHost, ctx->stream);
+                if (picked && e == hipSuccess) {
+                    k::argmax_rows_f32((const float *)lbuf->ptr, (int32_t *)pbuf->ptr, n, c.vocab, ctx->stream);
+                    e = hipMemcpyAsync(picked + w_lo + i, pbuf->ptr, (uint64_t)n * 4, hipMemcpyDeviceToHost, ctx->stream);
+                }
+                if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
+                if (e != hipSuccess) return hip_fail(ctx, e, "logits download", FA_ERR_TRANSFER_FAILED);
+            }
+        }
+        if (last_only) {
+            enqueue_head(ctx, L, a, (const float *)d->h->ptr, B, (float *)d->logits->ptr);
+            enqueue_pick(d, ctx->stream);
+        }
+        return after_launch(ctx, "layered decoder pass");
+    };
+    fa_status st;
+    try {
+        st = run();
+    } catch (const std::exception &) {
+        st = fail(FA_ERR_ALLOCATION_FAILED, "decoder pass: out of host memory");
+    }
+    L.trace = nullptr;
+    if (lbuf) fa_buffer_free(ctx, lbuf);
+    if (pbuf) fa_buffer_free(ctx, pbuf);
+    return st;
+}
+
+}  // namespace fa
+
+using namespace fa;
+
+namespace {
+
+fa_status check_layered(const fa_decoder *d, const char *what) {
+    if (!d || d->magic != kDecMagic) return fail(FA_ERR_INVALID_ARGUMENT, "decoder: not a decoder");
+    if (!d->layered) return fail(FA_ERR_UNSUPPORTED, std::string(what) + ": layered decoders only");
+    return FA_OK;
+}
+
+fa_status check_layer(const fa_layered_config &c, uint32_t i) {
+    const fa_layer_config &l = c.layers[i];
+    auto bad = [&](const char *why) { return fail(FA_ERR_INVALID_ARGUMENT, "layer " + std::to_string(i) + ": " + why); };
+    if (l.heads == 0 || l.dim == 0 || l.vdim == 0 || l.heads > 1024 || l.dim > 4096 || l.vdim > 4096) return bad("heads, dim and vdim must be positive");
+    if (l.mixer == FA_MIXER_DELTA) {
+        if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
+        if (l.conv == 0 || l.conv > 16) return bad("the convolution takes 1 to 16 taps");
+        if (l.dim > k::kDeltaMaxDim || l.vdim > k::kDeltaMaxVdim) return fail(FA_ERR_UNSUPPORTED, "delta layer: dim above 256 or vdim above 1024");
+        if (c.state_slots == 0) return bad("a recurrent layer needs state slots");
+    } else if (l.mixer == FA_MIXER_LATENT_ATTENTION) {
+        if (l.q_rank == 0 || l.kv_rank == 0) return bad("q_rank and kv_rank must be positive");
+        if (l.rot_dim == 0 || l.rot_dim % 2 != 0) return bad("rot_dim must be positive and even");
+        if (l.window == 0) return bad("the window must be positive");
+        if (!(l.rot_base > 0.0) || !std::isfinite(l.scale)) return bad("bad rotation base or scale");
+        if (l.kv_rank > 2048 || l.rot_dim > 1024) return fail(FA_ERR_UNSUPPORTED, "latent attention: kv_rank above 2048 or rot_dim above 1024");
+        if (l.kv_from >= 0) {
+            if ((uint32_t)l.kv_from >= i) return bad("kv_from must name an earlier layer");
+            const fa_layer_config &j = c.layers[l.kv_from];
+            if (j.mixer != FA_MIXER_LATENT_ATTENTION || j.kv_from >= 0) return bad("kv_from must name a latent attention layer with a cache of its own");
+            if (j.kv_rank != l.kv_rank || j.rot_dim != l.rot_dim || j.rot_base != l.rot_base) return bad("kv_from: the two layers' latents or rotations differ");
+        }
+    } else {
+        return bad("unknown mixer");
+    }
+    if (l.d_ffn && !(l.ffn_limit >= 0.0f && std::isfinite(l.ffn_alpha))) return bad("bad feed-forward constants");
+    return FA_OK;
+}
+
+}  // namespace
+
+extern "C" {
+
+fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cfg, fa_decoder **out) {
+    if (fa_status s = check_ctx(ctx)) return s;
+    if (!cfg || !out || !cfg->layers) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: null argument");
+    if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "decoder_create_layered during graph capture");
+    const fa_layered_config &c = *cfg;
+    if (c.n_layers == 0 || c.d_model == 0 || c.vocab == 0 || c.max_batch == 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: zero dimension");
+    if (c.max_batch > 256) return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: at most 256 sequences per step");
+    if (c.d_model > 16384) return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: d_model above 16384");
+    if (c.dtype != FA_BF16 && c.dtype != FA_F32) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: dtype must be bf16 or f32");
+    if (!std::isfinite(c.norm_eps) || c.norm_eps < 0.0f || !std::isfinite(c.logit_softcap)) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad constants");
+    if (c.block_size == 0 || (c.block_size & (c.block_size - 1)) != 0 || c.block_size > 256 || c.num_blocks == 0)
+        return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: block_size must be a power of two up to 256, num_blocks positive");
+    if (c.max_blocks_per_seq == 0 || (uint64_t)c.max_blocks_per_seq * c.block_size > (uint64_t)INT32_MAX)
+        return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad max_blocks_per_seq");
+    for (uint32_t i = 0; i < c.n_layers; ++i)
+        if (fa_status s = check_layer(c, i)) return s;
+
+    fa_decoder *d = new (std::nothrow) fa_decoder();
+    LayeredState *L = new (std::nothrow) LayeredState();
+    if (!d || !L) {
+        delete d;
+        delete L;
+        return fail(FA_ERR_ALLOCATION_FAILED, "decoder_create_layered: host allocation failed");
+    }
+    d->magic = kDecMagic;
+    d->ctx = ctx;
+    d->layered = L;
+    d->cfg = fa_decoder_config{};
+    d->cfg.n_layers = c.n_layers;
+    d->cfg.d_model = c.d_model;
+    d->cfg.vocab = c.vocab;
+    d->cfg.block_size = c.block_size;
+    d->cfg.max_blocks_per_seq = c.max_blocks_per_seq;
+    d->cfg.num_blocks = c.num_blocks;
+    d->cfg.max_batch = c.max_batch;
+    fa_status st = FA_OK;
+    try {
+        L->layer_cfgs.assign(c.layers, c.layers + c.n_layers);
+        L->cfg = c;
+        L->cfg.layers = L->layer_cfgs.data();
+        L->is_f32 = c.dtype == FA_F32;
+        L->esz = L->is_f32 ? 4 : 2;
+        const int f32 = L->is_f32;
+        auto mk = [&](fa_dtype t, uint64_t n, fa_buffer **b) {
+            if (st == FA_OK) st = make_buffer(ctx, t, n, true, b);
+        };
+        auto own = [&](fa_dtype t, uint64_t n) -> void * {
+            fa_buffer *b = nullptr;
+            mk(t, n, &b);
+            if (b) L->owned.push_back(b);
+            return b ? b->ptr : nullptr;
+        };
+        auto add = [&](const std::string &name, uint64_t rows, uint64_t cols, std::function<void(const void *, int, hipStream_t)> place) {
+            L->tensors.push_back(Tensor{name, rows, cols, false, std::move(place)});
+        };
+        // f32 vector (or small matrix) in row-major order
+        auto vec = [&](const std::string &name, uint64_t rows, uint64_t cols, float *dst) {
+            const uint64_t n = rows * (cols ? cols : 1);
+            add(name, rows, cols, [=](const void *src, int src_f32, hipStream_t s) {
+                if (src_f32) (void)hipMemcpyAsync(dst, src, n * 4, hipMemcpyDeviceToDevice, s);
+                else k::convert_bf16_to_f32((const uint16_t *)src, dst, n, s);
+            });
+        };
+        auto weight = [&](uint32_t n_store, uint32_t n_cols, uint32_t kk, uint32_t batches = 1) {
+            k::LinearWeight w;
+            w.n = n_store;
+            w.n_tiles = (n_cols + 15) / 16;
+            w.k_tiles = pad_to(kk, 64) / 32;
+            w.batches = batches;
+            w.w = own(f32 ? FA_F32 : FA_BF16, (uint64_t)batches * w.n_tiles * 16 * w.k_tiles * 32);
+            return w;
+        };
+        // whole linear [rows, cols] into output columns n0 ..
+        auto lin = [&](const std::string &name, uint32_t rows, uint32_t cols, const k::LinearWeight &w, uint32_t n0, uint32_t group = 0, uint32_t pitch = 0) {
+            add(name, rows, cols, [=](const void *src, int src_f32, hipStream_t s) {
+                k::pack_linear(src, src_f32, cols, 1, rows, cols, (void *)w.w, f32, w.k_tiles, n0, group ? group : 0x40000000u, pitch, s);
+            });
+        };
+        auto row_ptr = [](const void *src, int src_f32, uint64_t elem) { return (const void *)((const uint8_t *)src + elem * (src_f32 ? 4 : 2)); };
+
+        const uint32_t D = c.d_model;
+        L->embed = own(f32 ? FA_F32 : FA_BF16, (uint64_t)c.vocab * D);
+        {
+            void *dst = L->embed;
+            const uint64_t n = (uint64_t)c.vocab * D;
+            add("embed", c.vocab, D, [=](const void *src, int src_f32, hipStream_t s) {
+                if (src_f32 == f32) (void)hipMemcpyAsync(dst, src, n * (f32 ? 4 : 2), hipMemcpyDeviceToDevice, s);
+                else if (f32) k::convert_bf16_to_f32((const uint16_t *)src, (float *)dst, n, s);
+                else k::convert_f32_to_bf16((const float *)src, (uint16_t *)dst, n, s);
+            });
+        }
+        L->layers.resize(c.n_layers);
+        for (uint32_t i = 0; i < c.n_layers; ++i) {
+            Layer &l = L->layers[i];
+            l.cfg = c.layers[i];
+            const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.", f = p + "mlp.";
+            const fa_layer_config &g = l.cfg;
+            const uint32_t H = g.heads, ow = H * g.vdim;
+            l.norm1 = (float *)own(FA_F32, D);
+            l.ls1 = (float *)own(FA_F32, D);
+            vec(p + "norm1", D, 0, l.norm1);
+            vec(p + "ls1", D, 0, l.ls1);
+            if (g.mixer == FA_MIXER_DELTA) {
+                L->has_state = true;
+                l.de = k::DeltaShape{H, g.kv_heads, g.dim, g.vdim, g.conv, c.norm_eps};
+                const uint32_t nq = g.kv_heads * g.dim, ch = l.de.qkv();
+                l.in = weight(ch + ow + 2 * H, ch + ow + 2 * H, D);
+                lin(m + "q", nq, D, l.in, 0);
+                lin(m + "k", nq, D, l.in, nq);
+                lin(m + "v", ow, D, l.in, 2 * nq);
+                lin(m + "g", ow, D, l.in, ch);
+                lin(m + "b", H, D, l.in, ch + ow);
+                lin(m + "a", H, D, l.in, ch + ow + H);
+                l.conv = (float *)own(FA_F32, (uint64_t)ch * g.conv);
+                vec(m + "q.conv", nq, g.conv, l.conv);
+                vec(m + "k.conv", nq, g.conv, l.conv + (uint64_t)nq * g.conv);
+                vec(m + "v.conv", ow, g.conv, l.conv + 2ull * nq * g.conv);
+                l.a_log = (float *)own(FA_F32, H);
+                l.dt_bias = (float *)own(FA_F32, H);
+                l.head_norm = (float *)own(FA_F32, g.vdim);
+                vec(m + "A_log", H, 0, l.a_log);
+                vec(m + "dt_bias", H, 0, l.dt_bias);
+                vec(m + "norm", g.vdim, 0, l.head_norm);
+                l.state = (float *)own(FA_F32, (uint64_t)c.state_slots * H * g.dim * l.de.vdim_p());
+                l.ring = own(f32 ? FA_F32 : FA_BF16, (uint64_t)c.state_slots * g.conv * ch);
+            } else {
+                k::LatentShape &a = l.la;
+                a.heads = H;
+                a.dim = g.dim;
+                a.rot = g.rot_dim;
+                a.vdim = g.vdim;
+                a.q_rank = g.q_rank;
+                a.kv_rank = g.kv_rank;
+                a.dim_p = pad_to(g.dim, 32);
+                a.rot_p = pad_to(g.rot_dim, 32);
+                a.rank_p = pad_to(g.kv_rank, 32);
+                a.window = g.window;
+                a.scale = g.scale;
+                a.eps = c.norm_eps;
+                a.pool_rows = (uint64_t)c.num_blocks * c.block_size;
+                const bool own_kv = g.kv_from < 0;
+                const uint32_t kvn = own_kv ? g.kv_rank + g.rot_dim : 0;
+                l.in = weight(g.q_rank + kvn + H, g.q_rank + kvn + H, D);
+                lin(m + "dq", g.q_rank, D, l.in, 0);
+                l.q_norm = (float *)own(FA_F32, g.q_rank);
+                vec(m + "dq.norm", g.q_rank, 0, l.q_norm);
+                if (own_kv) {
+                    lin(m + "dkv", kvn, D, l.in, g.q_rank);
+                    l.kv_norm = (float *)own(FA_F32, g.kv_rank);
+                    vec(m + "dkv.norm", g.kv_rank, 0, l.kv_norm);
+                    l.pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * (a.rank_p + a.rot_p));
+                }
+                lin(m + "g", H, D, l.in, g.q_rank + kvn);
+                // queries: per head [dim padded][rot padded]
+                const uint32_t qw = a.dim_p + a.rot_p, hd = g.dim + g.rot_dim, qr = g.q_rank, dim = g.dim, rot = g.rot_dim, dim_p = a.dim_p;
+                l.uq = weight(H * qw, H * qw, qr);
+                {
+                    const k::LinearWeight w = l.uq;
+                    add(m + "uq", (uint64_t)H * hd, qr, [=](const void *src, int sf, hipStream_t s) {
+                        for (uint32_t h = 0; h < H; ++h) {
+                            k::pack_linear(row_ptr(src, sf, (uint64_t)h * hd * qr), sf, qr, 1, dim, qr, (void *)w.w, f32, w.k_tiles, h * qw, 0x40000000u, 0, s);
+                            k::pack_linear(row_ptr(src, sf, ((uint64_t)h * hd + dim) * qr), sf, qr, 1, rot, qr, (void *)w.w, f32, w.k_tiles, h * qw + dim_p, 0x40000000u, 0, s);
+                        }
+                    });
+                }
+                // per head, latent = W_uk^T q: the key projection transposed
+                const uint32_t kr = g.kv_rank, vd = g.vdim;
+                l.uk = weight(a.rank_p, a.rank_p, dim, H);
+                {
+                    const k::LinearWeight w = l.uk;
+                    const uint64_t one = (uint64_t)w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
+                    add(m + "uk", (uint64_t)H * dim, kr, [=](const void *src, int sf, hipStream_t s) {
+                        for (uint32_t h = 0; h < H; ++h)
+                            k::pack_linear(row_ptr(src, sf, (uint64_t)h * dim * kr), sf, 1, kr, kr, dim, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
+                    });
+                }
+                l.uv = weight(vd, vd, kr, H);
+                {
+                    const k::LinearWeight w = l.uv;
+                    const uint64_t one = (uint64_t)w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
+                    add(m + "uv", (uint64_t)H * vd, kr, [=](const void *src, int sf, hipStream_t s) {
+                        for (uint32_t h = 0; h < H; ++h)
+                            k::pack_linear(row_ptr(src, sf, (uint64_t)h * vd * kr), sf, kr, 1, vd, kr, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
+                    });
+                }
+                const std::pair<uint32_t, double> r(g.rot_dim, g.rot_base);
+                l.rotation = (uint32_t)(std::find(L->rotations.begin(), L->rotations.end(), r) - L->rotations.begin());
+                if (l.rotation == L->rotations.size()) L->rotations.push_back(r);
+            }
+            l.out = weight(D, D, ow);
+            lin(m + "o", D, ow, l.out, 0);
+            if (g.d_ffn) {
+                l.norm2 = (float *)own(FA_F32, D);
+                l.ls2 = (float *)own(FA_F32, D);
+                vec(p + "norm2", D, 0, l.norm2);
+                vec(p + "ls2", D, 0, l.ls2);
+                // gate and up alternate in tiles of 16 columns
+                l.gate_up = weight(g.d_ffn, 2 * pad_to(g.d_ffn, 16), D);
+                lin(f + "gate", g.d_ffn, D, l.gate_up, 0, 16, 32);
+                lin(f + "up", g.d_ffn, D, l.gate_up, 16, 16, 32);
+                l.down = weight(D, D, g.d_ffn);
+                lin(f + "down", D, g.d_ffn, l.down, 0);
+            }
+        }
+        L->final_norm = (float *)own(FA_F32, D);
+        vec("final.norm", D, 0, L->final_norm);
+        L->head = weight(c.vocab, c.vocab, D);
+        lin("head", c.vocab, D, L->head, 0);
+
+        const uint64_t B = c.max_batch;
+        mk(FA_I32, B, &d->tokens);
+        mk(FA_U32, B * c.max_blocks_per_seq, &d->tables);
+        mk(FA_U32, B, &d->seq_lens);
+        mk(FA_F32, B * D, &d->h);
+        mk(FA_F32, B * c.vocab, &d->logits);
+        mk(FA_U32, 2, &d->rng);
+        mk(FA_U32, 6 * B, &d->policy);
+        for (fa_buffer **b : {&L->state_slots, &L->unit_starts, &L->last_rows}) {
+            mk(FA_U32, B + 1, b);
+            if (*b) L->owned.push_back(*b);
+        }
+        if (st == FA_OK) {
+            std::vector<uint32_t> iota(B + 1);
+            for (uint64_t b = 0; b <= B; ++b) iota[b] = (uint32_t)b;
+            st = fa_upload_into(ctx, iota.data(), B + 1, L->unit_starts, 0);
+        }
+    } catch (const std::exception &) {
+        st = fail(FA_ERR_ALLOCATION_FAILED, "decoder_create_layered: out of host memory");
+    }
+    if (st != FA_OK) {
+        fa_decoder_destroy(ctx, d);
+        return st;
+    }
+    *out = d;
+    return FA_OK;
+}
+
+fa_status fa_decoder_tensor_count(const fa_decoder *d, uint32_t *count) {
+    if (fa_status s = check_layered(d, "decoder_tensor_count")) return s;
+    if (!count) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_tensor_count: null output");
+    *count = (uint32_t)d->layered->tensors.size();
+    return FA_OK;
+}
+
+fa_status fa_decoder_tensor_info(const fa_decoder *d, uint32_t index, const char **name, uint64_t *rows, uint64_t *cols) {
+    if (fa_status s = check_layered(d, "decoder_tensor_info")) return s;
+    if (!name || !rows || !cols || index >= d->layered->tensors.size()) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_tensor_info: bad argument");
+    const Tensor &t = d->layered->tensors[index];
+    *name = t.name.c_str();
+    *rows = t.rows;
+    *cols = t.cols;
+    return FA_OK;
+}
+
+fa_status fa_decoder_set_tensor(fa_context *ctx, fa_decoder *d, const char *name, fa_dtype dtype, const void *data, uint64_t rows, uint64_t cols) {
+    if (fa_status s = check_ctx(ctx)) return s;
+    if (fa_status s = check_layered(d, "decoder_set_tensor")) return s;
+    if (d->ctx != ctx) return fail(FA_ERR_DEVICE_MISMATCH, "decoder_set_tensor: decoder belongs to another context");
+    if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "decoder_set_tensor during graph capture");
+    if (!name || !data) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_set_tensor: null argument");
+    if (dtype != FA_BF16 && dtype != FA_F32) return fail(FA_ERR_INVALID_ARGUMENT, std::string("decoder_set_tensor: ") + name + ": must be bf16 or f32");
+    auto &ts = d->layered->tensors;
+    auto it = std::find_if(ts.begin(), ts.end(), [&](const Tensor &t) { return t.name == name; });
+    if (it == ts.end()) return fail(FA_ERR_INVALID_ARGUMENT, std::string("decoder_set_tensor: no tensor ") + name);
+    if (it->rows != rows || it->cols != cols)
+        return fail(FA_ERR_SHAPE_MISMATCH, std::string("decoder_set_tensor: ") + name + ": expected [" + std::to_string(it->rows) + ", " + std::to_string(it->cols) +
+                                               "], got [" + std::to_string(rows) + ", " + std::to_string(cols) + "]");
+    fa_buffer *tmp = nullptr;
+    if (fa_status s = fa_upload(ctx, dtype, data, rows * (cols ? cols : 1), &tmp)) return s;
+    it->place(tmp->ptr, dtype == FA_F32, ctx->stream);
+    fa_status s = after_launch(ctx, "decoder_set_tensor");
+    fa_buffer_free(ctx, tmp);                            // the stream is in order: a later user is queued behind the copy
+    if (s == FA_OK) it->set = true;
+    return s;
+}
+
+fa_status fa_decoder_set_state_slots(fa_context *ctx, fa_decoder *d, const uint32_t *slots) {
+    if (fa_status s = check_ctx(ctx)) return s;
+    if (fa_status s = check_layered(d, "decoder_set_state_slots")) return s;
+    if (d->ctx != ctx) return fail(FA_ERR_DEVICE_MISMATCH, "decoder_set_state_slots: decoder belongs to another context");
+    if (d->batch == 0 || !slots) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_set_state_slots: no sequences or null slots");
+    for (uint32_t b = 0; b < d->batch; ++b) {
+        if (slots[b] >= d->layered->cfg.state_slots) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_set_state_slots: row " + std::to_string(b) + " has no such slot");
+        for (uint32_t o = 0; o < b; ++o)
+            if (slots[o] == slots[b]) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_set_state_slots: two rows share a slot");
+    }
+    if (fa_status s = fa_upload_into(ctx, slots, d->batch, d->layered->state_slots, 0)) return s;
+    d->layered->slots_set = true;
+    return FA_OK;
+}
+
+fa_status fa_decoder_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts, const int32_t *tokens, uint64_t n_want, const uint32_t *want, float *logits) {
+    if (fa_status s = check_ctx(ctx)) return s;
+    if (fa_status s = check_layered(d, "decoder_forward")) return s;
+    if (d->ctx != ctx) return fail(FA_ERR_DEVICE_MISMATCH, "decoder_forward: decoder belongs to another context");
+    if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "decoder_forward during graph capture");
+    if (d->batch == 0) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_forward: no sequences installed");
+    if (!counts || !tokens || (n_want && (!want || !logits))) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_forward: null argument");
+    static const uint32_t none = 0;
+    return layered_forward(ctx, d, counts, tokens, n_want, want ? want : &none, logits, nullptr);
+}
+
+fa_status fa_decoder_debug_residuals(fa_decoder *d, float *residuals, uint64_t rows) {
+    if (fa_status s = check_layered(d, "decoder_debug_residuals")) return s;
+    d->layered->trace = residuals;
+    d->layered->trace_rows = rows;
+    return FA_OK;
+}
+
+}  // extern "C"

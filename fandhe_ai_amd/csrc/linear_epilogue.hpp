@@ -1,0 +1,71 @@
+// The epilogues of the unquantized linears (LinearEpilogue), shared by their kernels.
+#pragma once
+
+#include "device_utils.hpp"
+#include "kernels.hpp"
+
+namespace fa {
+namespace k {
+
+__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// The value the epilogue makes of y (and, for gate | up, of the up column's y).
+template <int MODE>
+__device__ __forceinline__ float epilogue_value(const LinearEpilogue &ep, uint32_t row, uint32_t batch, float y, float up) {
+    if constexpr (MODE == LinearEpilogue::kGlu) {
+        const float g = fminf(y, ep.limit), u = fminf(fmaxf(up, -ep.limit), ep.limit);
+        return g * sigmoid_f32(ep.alpha * g) * (u + 1.0f);
+    } else if constexpr (MODE == LinearEpilogue::kSoftcap) {
+        return ep.cap > 0.0f ? ep.cap * tanhf(y / ep.cap) : y;
+    } else if constexpr (MODE == LinearEpilogue::kHeadGate) {
+        return y * sigmoid_f32(ep.gate[(uint64_t)row * ep.ld_gate + batch]);
+    } else {
+        return y;
+    }
+}
+
+template <int MODE>
+__device__ __forceinline__ void epilogue_store1(const LinearEpilogue &ep, uint32_t row, uint32_t col, uint32_t batch, float y, float up) {
+    const float v = epilogue_value<MODE>(ep, row, batch, y, up);
+    if constexpr (MODE == LinearEpilogue::kResidual) {
+        float *o = (float *)ep.out + (uint64_t)row * ep.ld_out + col;
+        *o = *o + ep.scale[col] * v;
+        return;
+    }
+    if (MODE == LinearEpilogue::kStore && col >= ep.n_lo) {
+        ep.out_hi[(uint64_t)row * ep.ld_hi + (col - ep.n_lo)] = v;
+        return;
+    }
+    const uint64_t o = batch * ep.out_batch + (uint64_t)row * ep.ld_out + col;
+    if (ep.out_f32) ((float *)ep.out)[o] = v;
+    else ((uint16_t *)ep.out)[o] = dev::f32_to_bf16(v);
+}
+
+// Columns col .. col + 3 of a row (those below n).
+template <int MODE>
+__device__ __forceinline__ void epilogue_store4(const LinearEpilogue &ep, uint32_t row, uint32_t col, uint32_t n, uint32_t batch,
+                                                dev::v4f y, dev::v4f up) {
+    const uint64_t o = batch * ep.out_batch + (uint64_t)row * ep.ld_out + col;
+    const bool whole = col + 4 <= n && ((ep.ld_out | ep.out_batch) & 3) == 0 && (MODE != LinearEpilogue::kStore || col + 4 <= ep.n_lo);
+    if (!whole) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (col + e < n) epilogue_store1<MODE>(ep, row, col + e, batch, y[e], up[e]);
+        return;
+    }
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = epilogue_value<MODE>(ep, row, batch, y[e], up[e]);
+    if constexpr (MODE == LinearEpilogue::kResidual) {
+        dev::v4f *p = (dev::v4f *)((float *)ep.out + o);
+        const dev::v4f r = *p, ls = *(const dev::v4f *)(ep.scale + col);
+        *p = dev::v4f{r[0] + ls[0] * v[0], r[1] + ls[1] * v[1], r[2] + ls[2] * v[2], r[3] + ls[3] * v[3]};
+    } else if (ep.out_f32) {
+        *(dev::v4f *)((float *)ep.out + o) = dev::v4f{v[0], v[1], v[2], v[3]};
+    } else {
+        *(dev::v2u *)((uint16_t *)ep.out + o) = dev::v2u{dev::f32x2_to_bf16x2(v[0], v[1]), dev::f32x2_to_bf16x2(v[2], v[3])};
+    }
+}
+
+}  // namespace k
+}  // namespace fa

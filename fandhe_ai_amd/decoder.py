@@ -12,6 +12,9 @@ lib = capi.lib
 
 
 class Decoder:
+    state_slots = 0                                       # recurrent states the decoder holds; 0: it has none
+    takes_portions = False                                # whether ``forward`` is there
+
     def __init__(self, ops, n_layers, d_model, n_heads, n_kv_heads, d_ffn, vocab, max_blocks_per_seq, num_blocks,
                  max_batch, head_dim=128, block_size=16, rms_eps=1e-5, rope_theta=500000.0):
         self._ops = ops
@@ -138,3 +141,68 @@ class Decoder:
         out = np.empty(self.batch, dtype=np.uint32)
         check(lib.fa_decoder_read_seq_lens(self._ops._ctx, self._h, out.ctypes.data_as(capi.u32p)))
         return out
+
+
+class LayeredDecoder(Decoder):
+    """A decoder whose layers are described one by one (``fa_decoder_create_layered``): unquantized weights in bf16 or
+    f32, per layer a gated delta rule with a recurrent state or latent attention over the paged cache, and an optional
+    feed-forward.  Sequences, steps, prompt passes and sampling are ``Decoder``'s."""
+
+    takes_portions = True
+
+    def __init__(self, ops, d_model, vocab, layers, norm_eps, logit_softcap, max_blocks_per_seq, num_blocks, max_batch,
+                 state_slots=None, dtype=capi.BF16, block_size=16):
+        """layers: one dict of ``capi.LayerConfig`` fields per layer."""
+        self._ops = ops
+        rows = (capi.LayerConfig * len(layers))(*[capi.LayerConfig(**l) for l in layers])
+        recurrent = any(l["mixer"] == capi.MIXER_DELTA for l in layers)
+        slots = max_batch if state_slots is None else state_slots
+        self.cfg = capi.LayeredConfig(len(layers), d_model, vocab, block_size, max_blocks_per_seq, num_blocks, max_batch,
+                                      slots, norm_eps, logit_softcap, dtype, rows)
+        self.state_slots = slots if recurrent else 0
+        self._h = C.c_void_p()
+        check(lib.fa_decoder_create_layered(ops._ctx, C.byref(self.cfg), C.byref(self._h)))
+        self._keep = []
+        self.batch = 0
+
+    def tensors(self):
+        """name -> shape of every weight tensor the decoder takes."""
+        n, name, rows, cols = C.c_uint32(), C.c_char_p(), capi.u64(), capi.u64()
+        check(lib.fa_decoder_tensor_count(self._h, C.byref(n)))
+        out = {}
+        for i in range(n.value):
+            check(lib.fa_decoder_tensor_info(self._h, i, C.byref(name), C.byref(rows), C.byref(cols)))
+            out[name.value.decode()] = (rows.value, cols.value) if cols.value else (rows.value,)
+        return out
+
+    def set_tensor(self, name, array, bf16=False):
+        """array: float32 values, or bf16 bit patterns in uint16 (bf16=True), as the checkpoint stores them."""
+        a = np.ascontiguousarray(array, dtype=np.uint16 if bf16 else np.float32)
+        rows, cols = (a.shape[0], a.shape[1]) if a.ndim == 2 else (a.size, 0)
+        check(lib.fa_decoder_set_tensor(self._ops._ctx, self._h, name.encode(), capi.BF16 if bf16 else capi.F32,
+                                        a.ctypes.data_as(C.c_void_p), rows, cols))
+
+    def set_state_slots(self, slots):
+        s = np.ascontiguousarray(slots, dtype=np.uint32)
+        if s.size != self.batch:
+            raise ValueError("one state slot per installed sequence")
+        check(lib.fa_decoder_set_state_slots(self._ops._ctx, self._h, s.ctypes.data_as(capi.u32p)))
+
+    def forward(self, portions, want=None, residuals=False):
+        """One pass over all installed sequences: portions[b] are row b's next tokens (any number, none included).
+        want[b]: places in portions[b] whose logits are asked for.  Returns the logits [wanted, vocab] in row order (and,
+        with residuals, the residual stream after every layer, [layers, tokens, d_model])."""
+        if len(portions) != self.batch:
+            raise ValueError("one portion per installed sequence")
+        counts = np.array([len(p) for p in portions], dtype=np.uint32)
+        flat = np.array([t for p in portions for t in p], dtype=np.int32)
+        starts = np.concatenate([[0], np.cumsum(counts)]).astype(np.int64)
+        places = np.array([starts[b] + k for b, ks in enumerate(want or []) for k in ks], dtype=np.uint32)
+        logits = np.empty((places.size, self.cfg.vocab), dtype=np.float32)
+        trace = np.empty((self.cfg.n_layers, flat.size, self.cfg.d_model), dtype=np.float32) if residuals else None
+        if residuals:
+            check(lib.fa_decoder_debug_residuals(self._h, trace.ctypes.data_as(capi.f32p), flat.size))
+        check(lib.fa_decoder_forward(self._ops._ctx, self._h, counts.ctypes.data_as(capi.u32p), flat.ctypes.data_as(capi.i32p),
+                                     places.size, places.ctypes.data_as(capi.u32p) if places.size else None,
+                                     logits.ctypes.data_as(capi.f32p) if places.size else None))
+        return (logits, trace) if residuals else logits

@@ -1,0 +1,164 @@
+"""Model registry: a folder with config.json and model.safetensors -> a resident decoder.
+
+``load_model`` picks the design by config.json: its "architecture" (or the first of "architectures") names an entry of
+``ARCHITECTURES``.  A new design registers a function that reads its configuration and weights and returns a decoder;
+what the decoder runs on (pages, rows, state slots) is the caller's ``Capacity``.
+"""
+import json
+import os
+
+from . import capi
+from . import safetensors_io as st
+from .decoder import LayeredDecoder
+
+CONFIG_FILE, WEIGHTS_FILE = "config.json", "model.safetensors"
+
+
+class ConfigError(ValueError):
+    """A configuration that is incomplete or asks for something the framework does not have."""
+
+
+class Capacity:
+    """What a decoder is built to hold: ``max_tokens`` cached tokens over all sequences (whole pages), ``max_batch``
+    sequences per step and ``state_slots`` recurrent states (default: one per row of the batch)."""
+
+    def __init__(self, max_tokens, max_batch=32, state_slots=None, block_size=16):
+        if min(max_tokens, max_batch, block_size) < 1:
+            raise ConfigError("Capacity: sizes must be positive")
+        self.max_tokens, self.max_batch, self.block_size = max_tokens, max_batch, block_size
+        self.state_slots = max_batch if state_slots is None else state_slots
+
+    @property
+    def num_blocks(self):
+        return -(-self.max_tokens // self.block_size)
+
+
+DTYPES = {"bfloat16": capi.BF16, "float32": capi.F32}
+
+# architecture name -> function(ops, config, weights path, dtype name, capacity) -> decoder
+ARCHITECTURES = {}
+
+
+def register(name):
+    def add(fn):
+        ARCHITECTURES[name] = fn
+        return fn
+    return add
+
+
+def read_config(folder):
+    try:
+        with open(os.path.join(folder, CONFIG_FILE)) as f:
+            return json.load(f)
+    except (OSError, ValueError) as e:
+        raise ConfigError("%s: %s" % (CONFIG_FILE, e))
+
+
+def architecture_of(config):
+    name = config.get("architecture") or (config.get("architectures") or [None])[0]
+    if name not in ARCHITECTURES:
+        raise ConfigError("unknown architecture %r (known: %s)" % (name, ", ".join(sorted(ARCHITECTURES))))
+    return name
+
+
+def load_model(ops, folder, dtype="bfloat16", capacity=None):
+    """The decoder of the model in ``folder`` on ``ops``."""
+    if dtype not in DTYPES:
+        raise ConfigError("dtype must be one of %s" % ", ".join(sorted(DTYPES)))
+    config = read_config(folder)
+    build = ARCHITECTURES[architecture_of(config)]
+    return build(ops, config, os.path.join(folder, WEIGHTS_FILE), dtype, capacity or Capacity(8192))
+
+
+# ---- Nugelix: layers of gated delta rule and latent attention ---------------------------------------------------
+
+GLU_ALPHA = 1.702                                          # the feed-forward's gate is g * sigmoid(1.702 g)
+
+
+def _entry(d, key, where):
+    if key not in d:
+        raise ConfigError("%s: %r is missing" % (where, key))
+    return d[key]
+
+
+def nugelix_layers(config):
+    """config.json's layer list as ``capi.LayerConfig`` fields."""
+    out = []
+    for i, layer in enumerate(_entry(config, "layers", CONFIG_FILE)):
+        where = "layer %d" % i
+        kind, mx = _entry(layer, "type", where), _entry(layer, "mixer", where)
+        get = lambda key: _entry(mx, key, where + " mixer")
+        l = {"heads": get("heads"), "dim": get("dim"), "vdim": get("vdim"), "kv_from": -1}
+        if kind == "delta":
+            l.update(mixer=capi.MIXER_DELTA, kv_heads=get("kv_heads"), conv=get("conv"))
+        elif kind == "latent_attention":
+            rot = get("rot")
+            if _entry(rot, "dims", where + " rot") != get("rot_dim"):
+                raise ConfigError("%s: all of the rotated part is rotated, rot.dims must equal rot_dim" % where)
+            l.update(mixer=capi.MIXER_LATENT_ATTENTION, q_rank=get("q_rank"), kv_rank=get("kv_rank"), rot_dim=get("rot_dim"),
+                     window=_entry(get("mask"), "size", where + " mask"), scale=get("scale"),
+                     rot_base=_entry(rot, "base", where + " rot"))
+            if mx.get("kv_from") is not None:
+                l["kv_from"] = mx["kv_from"]
+        else:
+            raise ConfigError("%s: unknown type %r" % (where, kind))
+        mlp = layer.get("mlp")
+        if mlp is not None:
+            if _entry(mlp, "kind", where + " mlp") != "dense":
+                raise ConfigError("%s: unknown feed-forward %r" % (where, mlp["kind"]))
+            l.update(d_ffn=_entry(mlp, "ff", where + " mlp"), ffn_limit=_entry(mlp, "limit", where + " mlp"), ffn_alpha=GLU_ALPHA)
+        out.append(l)
+    return out
+
+
+def build_layered(ops, config, dtype, capacity):
+    """The decoder a Nugelix configuration describes, without weights."""
+    return LayeredDecoder(ops, _entry(config, "width", CONFIG_FILE), _entry(config, "vocab", CONFIG_FILE), nugelix_layers(config),
+                          _entry(_entry(config, "norm", CONFIG_FILE), "eps", "norm"), config.get("logit_softcap") or 0.0,
+                          capacity.num_blocks, capacity.num_blocks, capacity.max_batch, capacity.state_slots, DTYPES[dtype],
+                          capacity.block_size)
+
+
+def install_weights(decoder, typed):
+    """name -> ``safetensors_io.TypedTensor`` into a layered decoder: every tensor it takes, none it does not."""
+    wanted = decoder.tensors()
+    st.require_keys(typed, sorted(wanted))
+    extra = sorted(set(typed) - set(wanted))
+    if extra:
+        raise ConfigError("tensors the configuration has no use for: %s" % ", ".join(extra))
+    for name, shape in wanted.items():
+        t = typed[name]
+        if t.shape != shape:
+            raise st.SafetensorsFormat("%s has shape %s, the configuration needs %s" % (name, t.shape, shape))
+        if t.dtype == "BF16":
+            decoder.set_tensor(name, t.data, bf16=True)
+        else:
+            decoder.set_tensor(name, t.to_f32())
+
+
+@register("Nugelix")
+def _nugelix(ops, config, weights, dtype, capacity):
+    typed = st.load_safetensors_typed(weights)
+    decoder = build_layered(ops, config, dtype, capacity)
+    try:
+        install_weights(decoder, typed)
+    except Exception:
+        decoder.close()
+        raise
+    return decoder
+
+
+# ---- Llama-style checkpoints on the W8A8 decoder ------------------------------------------------------------------
+
+@register("LlamaForCausalLM")
+def _llama(ops, config, weights, dtype, capacity):
+    if dtype != "bfloat16":
+        raise ConfigError("the W8A8 decoder has no float32 form")
+    heads, get = _entry(config, "num_attention_heads", CONFIG_FILE), config.get
+    decoder, store = st.load_decoder(ops, weights, _entry(config, "num_hidden_layers", CONFIG_FILE), heads,
+                                     get("num_key_value_heads") or heads, capacity.num_blocks, capacity.num_blocks,
+                                     min(capacity.max_batch, 64), get("head_dim") or config["hidden_size"] // heads, capacity.block_size,
+                                     get("rms_norm_eps") or 1e-5, get("rope_theta") or 10000.0)
+    ops.synchronize_device()
+    store.free()
+    return decoder

@@ -161,6 +161,8 @@ def generate(decoder, input_ids, config):
     pages = _pages_for(config.max_length, cfg.block_size)
     if b > cfg.max_batch or pages > cfg.max_blocks_per_seq or b * pages > cfg.num_blocks:
         raise InvalidArgument("generate: %d rows of %d tokens do not fit the decoder's batch or page pool" % (b, config.max_length))
+    if getattr(decoder, "state_slots", 0) and b > decoder.state_slots:
+        raise InvalidArgument("generate: %d rows, the decoder holds %d recurrent states" % (b, decoder.state_slots))
     config.validate_top_k_le_vocab(cfg.vocab)
     out = np.empty((b, config.max_length), dtype=np.int32)
     out[:, :prompt_len] = ids
@@ -246,6 +248,8 @@ def generate_speculative(target, draft, input_ids, config, k):
     config.validate()
     if not isinstance(k, int) or k < 1:
         raise InvalidArgument("generate_speculative: k must be at least 1")
+    if getattr(target, "state_slots", 0) or getattr(draft, "state_slots", 0):
+        raise InvalidArgument("generate_speculative: a recurrent state cannot be cut back to the accepted length")
     ids, b, prompt_len, want_rank1 = _prompt_shape(input_ids, "generate_speculative")
     if prompt_len == 0:
         raise InvalidArgument("generate_speculative: the prompt is empty")
@@ -409,7 +413,70 @@ class _Pending:
 
 
 class _Active:
-    __slots__ = ("id", "tokens", "pages", "policy", "config", "want_rank1", "fresh")
+    __slots__ = ("id", "tokens", "pages", "slot", "policy", "config", "want_rank1", "fresh")
+
+
+class PortionBatcher:
+    """Requests whose tokens the caller brings, in portions of any size: a request is admitted with its first portion,
+    takes pages as it grows and, on a decoder with recurrent states, one state slot, and gives them back on ``release``.
+    All portions of one ``feed`` are one batch on the device."""
+
+    def __init__(self, decoder):
+        if not getattr(decoder, "takes_portions", False):
+            raise InvalidArgument("PortionBatcher: the decoder takes no mixed passes of portions")
+        self._dec = decoder
+        self._pages = PageAllocator(decoder.cfg.num_blocks)
+        self._slots = PageAllocator(decoder.state_slots) if decoder.state_slots else None
+        self._live = {}                                    # id -> [tokens fed, pages, state slot]
+
+    def live(self):
+        return sorted(self._live)
+
+    def free_pages(self):
+        return self._pages.free_pages()
+
+    def feed(self, entries):
+        """entries: [(id, tokens, wanted places among them)]; returns the wanted logits, [wanted, vocab], in that
+        order.  Nothing changes when the batch does not fit."""
+        cfg = self._dec.cfg
+        if not 0 < len(entries) <= cfg.max_batch or len({e[0] for e in entries}) != len(entries):
+            raise InvalidArgument("feed: between 1 and %d different requests per step" % cfg.max_batch)
+        for rid, tokens, want in entries:
+            if not len(tokens) or any(not 0 <= t < cfg.vocab for t in tokens):
+                raise InvalidArgument("feed: request %r brings no tokens or tokens outside the vocabulary" % (rid,))
+            if any(not 0 <= w < len(tokens) for w in want) or list(want) != sorted(set(want)):
+                raise InvalidArgument("feed: wanted places of request %r must ascend inside its portion" % (rid,))
+        fresh = [rid for rid, _, _ in entries if rid not in self._live]
+        pages = {}
+        for rid, tokens, _ in entries:
+            fed, held = self._live[rid][:2] if rid in self._live else (0, [])
+            pages[rid] = -(-(fed + len(tokens)) // cfg.block_size) - len(held)
+            if pages[rid] + len(held) > cfg.max_blocks_per_seq:
+                raise InvalidArgument("feed: request %r outgrows a block table" % (rid,))
+        if sum(pages.values()) > self._pages.free_pages() or (self._slots and len(fresh) > self._slots.free_pages()):
+            raise InvalidArgument("feed: the batch does not fit the free pages or state slots")
+        for rid in fresh:
+            self._live[rid] = [0, [], self._slots.take(1)[0] if self._slots else 0]
+        tables = np.full((len(entries), cfg.max_blocks_per_seq), 0xFFFFFFFF, dtype=np.uint32)
+        for b, (rid, _, _) in enumerate(entries):
+            held = self._live[rid][1]
+            held.extend(self._pages.take(pages[rid]))
+            tables[b, :len(held)] = held
+        self._dec.set_sequences(tables, np.array([self._live[rid][0] for rid, _, _ in entries], dtype=np.uint32))
+        if self._slots:
+            self._dec.set_state_slots([self._live[rid][2] for rid, _, _ in entries])
+        logits = self._dec.forward([tokens for _, tokens, _ in entries], [want for _, _, want in entries])
+        for rid, tokens, _ in entries:
+            self._live[rid][0] += len(tokens)
+        return logits
+
+    def release(self, rid):
+        if rid not in self._live:
+            raise InvalidArgument("release: no request %r" % (rid,))
+        _, pages, slot = self._live.pop(rid)
+        self._pages.give_back(pages)
+        if self._slots:
+            self._slots.give_back([slot])
 
 
 class BatchScheduler:
@@ -422,7 +489,11 @@ class BatchScheduler:
         self._dec, self.limits = decoder, limits
         self._queue, self._active, self._finished, self._failed = deque(), [], [], []
         self._next_id = 0
+        slots = getattr(decoder, "state_slots", 0)
+        if slots and limits.max_active > slots:
+            raise InvalidArgument("scheduler: max_active (%d) exceeds the decoder's recurrent states (%d)" % (limits.max_active, slots))
         self._pages = PageAllocator(cfg.num_blocks)
+        self._slots = PageAllocator(slots) if slots else None
         self._resident = None                              # ids whose decode state is installed on the device, in row order
         # what the device was asked to do so far: prompt passes, their rows incl. padding, decode steps and their rows
         self.stats = {"prompt_passes": 0, "prompt_rows": 0, "decode_steps": 0, "decode_rows": 0}
@@ -548,6 +619,7 @@ class BatchScheduler:
             a = _Active()
             a.id, a.tokens, a.config, a.want_rank1, a.fresh = p.id, list(p.prompt), p.config, p.want_rank1, True
             a.pages = self._pages.take(need)
+            a.slot = self._slots.take(1)[0] if self._slots else 0
             state = capi.u64()
             check(lib.fa_rng_state_from_seed(p.config.seed, state))
             a.policy = (state.value, float(p.config.temperature), int(p.config.top_k or 0), int(p.config.strategy.kind))
@@ -559,6 +631,16 @@ class BatchScheduler:
         row[:len(a.pages)] = a.pages
         return row
 
+    def _place(self, rows, lens):
+        self._dec.set_sequences(np.stack([self._table_row(a) for a in rows]), np.array(lens, dtype=np.uint32))
+        if self._slots:
+            self._dec.set_state_slots([a.slot for a in rows])
+
+    def _give_back(self, a):
+        self._pages.give_back(a.pages)
+        if self._slots:
+            self._slots.give_back([a.slot])
+
     def _policy_rows(self, rows):
         arr = (capi.RowSampling * len(rows))()
         for r, a in zip(arr, rows):
@@ -567,8 +649,7 @@ class BatchScheduler:
 
     def _install(self, rows):
         self._pull_resident_state()
-        self._dec.set_sequences(np.stack([self._table_row(a) for a in rows]),
-                                np.array([len(a.tokens) - 1 for a in rows], dtype=np.uint32))
+        self._place(rows, [len(a.tokens) - 1 for a in rows])
         self._dec.set_tokens(np.array([a.tokens[-1] for a in rows], dtype=np.int32))
         self._dec.set_row_sampling(self._policy_rows(rows))
         self._resident = [a.id for a in rows]
@@ -605,7 +686,7 @@ class BatchScheduler:
 
     def _ingest(self, group):
         """One prompt pass for the group; returns the requests whose logits were not finite."""
-        self._dec.set_sequences(np.stack([self._table_row(a) for a in group]), np.zeros(len(group), np.uint32))
+        self._place(group, [0] * len(group))
         self._dec.set_row_sampling(self._policy_rows(group))
         self.stats["prompt_passes"] += 1
         self.stats["prompt_rows"] += len(group) * max(len(a.tokens) for a in group)
@@ -629,13 +710,13 @@ class BatchScheduler:
         if len(a.tokens) < a.config.max_length:
             return 0
         self._finished.append((a.id, self._output(a.tokens, a.want_rank1)))
-        self._pages.give_back(a.pages)
+        self._give_back(a)
         gone.add(a.id)
         return 1
 
     def _fail(self, a, err, gone):
         self._failed.append((a.id, err))
-        self._pages.give_back(a.pages)
+        self._give_back(a)
         gone.add(a.id)
 
     @staticmethod

@@ -563,6 +563,51 @@ fa_status fa_decoder_read_seq_lens(fa_context *ctx, fa_decoder *dec, uint32_t *s
  * (speculative.rs:334-531) keeps the probabilities on the device. */
 fa_status fa_decoder_logits_buffer(fa_decoder *dec, fa_buffer **out);
 
+/* -------------------------------------------------------- layered decoders */
+/* A decoder whose layers are described one by one: pre-norm (layer norm) sublayers with a layer scale, a mixer per
+ * layer (gated delta rule with a recurrent state, or latent attention over the paged cache) and an optional clamped
+ * GLU feed-forward, on unquantized weights.  No counterpart in the reference.  It is an fa_decoder: sequences, tokens,
+ * sampling, steps, prompt passes, verification and the read-outs are the calls above. */
+typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1 } fa_mixer_kind;
+typedef struct {
+    int32_t mixer;                /* fa_mixer_kind */
+    uint32_t heads, dim, vdim;    /* per head: query / key dims (latent attention: the unrotated part), value dims */
+    uint32_t kv_heads, conv;      /* delta: q / k heads, taps of the short convolution (1..=16) */
+    uint32_t q_rank, kv_rank;     /* latent attention: sizes of the two latents */
+    uint32_t rot_dim, window;     /* latent attention: rotated dims (even), visible keys incl. the token's own */
+    int32_t kv_from;              /* latent attention: the earlier layer whose cache is used, -1 for its own */
+    float scale;                  /* latent attention: factor of the scores */
+    double rot_base;
+    uint32_t d_ffn;               /* 0: no feed-forward */
+    float ffn_limit, ffn_alpha;   /* g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + 1) */
+} fa_layer_config;
+typedef struct {
+    uint32_t n_layers, d_model, vocab;
+    uint32_t block_size, max_blocks_per_seq, num_blocks;
+    uint32_t max_batch;           /* sequences of a step or pass: 1..=256 */
+    uint32_t state_slots;         /* recurrent states held at a time */
+    float norm_eps, logit_softcap;        /* softcap 0: none */
+    fa_dtype dtype;               /* FA_BF16: weights, activations and cache in bf16; FA_F32: everything in f32 */
+    const fa_layer_config *layers;        /* [n_layers], copied */
+} fa_layered_config;
+fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cfg, fa_decoder **out);
+/* Number of weight tensors the decoder takes and the i-th one's name and shape (cols 0: a vector). */
+fa_status fa_decoder_tensor_count(const fa_decoder *dec, uint32_t *count);
+fa_status fa_decoder_tensor_info(const fa_decoder *dec, uint32_t index, const char **name, uint64_t *rows, uint64_t *cols);
+/* Installs one of them from host memory (FA_BF16 bits or FA_F32, [rows, cols] row-major, linears as [out, in]);
+ * synchronous.  Steps and passes are refused until all are there. */
+fa_status fa_decoder_set_tensor(fa_context *ctx, fa_decoder *dec, const char *name, fa_dtype dtype, const void *data,
+                                uint64_t rows, uint64_t cols);
+/* State slots [batch] of the installed sequences (host array; after fa_decoder_set_sequences, which assumes slot b
+ * for row b).  A slot needs no clearing: a sequence of length 0 starts from a zero state. */
+fa_status fa_decoder_set_state_slots(fa_context *ctx, fa_decoder *dec, const uint32_t *slots);
+/* One pass over all installed sequences, portions of prompts beside single tokens: counts [batch] (0 allowed) new
+ * tokens per sequence, concatenated in tokens.  want [n_want]: places among the concatenated tokens, ascending, whose
+ * logits [n_want, vocab] are copied to the host (n_want 0: none).  Synchronous when logits are asked for.  Layered
+ * decoders only. */
+fa_status fa_decoder_forward(fa_context *ctx, fa_decoder *dec, const uint32_t *counts, const int32_t *tokens,
+                             uint64_t n_want, const uint32_t *want, float *logits);
+
 #ifdef __cplusplus
 }
 #endif

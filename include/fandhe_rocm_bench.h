@@ -153,6 +153,9 @@ fa_status fa_graph_owned_blocks(const fa_graph *graph, void **ptrs, uint64_t cap
  * [batch, head_dim]; 8 cache slots u32 [batch]; 9 positions i32 [batch]. */
 fa_status fa_decoder_debug_step_until(fa_context *ctx, fa_decoder *dec, int32_t stop_after);
 fa_status fa_decoder_debug_buffer(fa_decoder *dec, int32_t which, fa_buffer **out);
+/* Layered decoders: the next fa_decoder_forward (one internal pass, `rows` tokens) copies the residual stream after every
+ * layer to residuals [n_layers, rows, d_model] (host array, f32). */
+fa_status fa_decoder_debug_residuals(fa_decoder *dec, float *residuals, uint64_t rows);
 
 /* A pair of HIP events recorded on the context's stream (the stream the
  * kernels run on); used by the benchmark to time launches. */

@@ -1,0 +1,150 @@
+"""Oracle: the mechanisms of the layered decoders (gated delta rule, latent attention, clamped GLU feed-forward,
+layer norm with layer scale, soft-capped head), one function per mechanism, in float64 and token by token.
+
+TEST INFRASTRUCTURE ONLY: written from the equations, for whole sequences, without a cache, a batch or any code
+of the product; only tests and the smoke check may import it.
+
+``weights`` maps tensor names to arrays (linear weights [out, in]); ``config`` is the parsed config.json.
+"""
+import numpy as np
+
+
+def sigmoid(z):
+    return 0.5 * (1.0 + np.tanh(0.5 * z))
+
+
+def silu(z):
+    return z * sigmoid(z)
+
+
+def softplus(z):
+    return np.maximum(z, 0.0) + np.log1p(np.exp(-np.abs(z)))
+
+
+def rms_norm(x, w, eps):
+    return x / np.sqrt((x * x).mean(axis=-1, keepdims=True) + eps) * w
+
+
+def layer_norm(x, w, eps):
+    c = x - x.mean(axis=-1, keepdims=True)
+    return c / np.sqrt((c * c).mean(axis=-1, keepdims=True) + eps) * w
+
+
+def unit_vector(x):
+    return x / np.sqrt((x * x).sum(axis=-1, keepdims=True) + 1e-6)
+
+
+def rotate(x, positions, base):
+    """Rotate-half rotary embedding of all of x's last axis; positions has x's first axis."""
+    dims = x.shape[-1]
+    half = dims // 2
+    freq = float(base) ** (-2.0 * np.arange(half) / dims)
+    a = np.asarray(positions, dtype=np.float64)[:, None] * freq
+    a = a.reshape((a.shape[0],) + (1,) * (x.ndim - 2) + (half,))
+    u, v = x[..., :half], x[..., half:]
+    return np.concatenate([u * np.cos(a) - v * np.sin(a), v * np.cos(a) + u * np.sin(a)], axis=-1)
+
+
+def causal_conv(x, taps):
+    """y_t = sum_i taps[:, i] x_{t - (T - 1) + i} per channel; zeros before the start."""
+    n, T = x.shape[0], taps.shape[1]
+    padded = np.concatenate([np.zeros((T - 1, x.shape[1])), x])
+    return sum(padded[i:i + n] * taps[:, i] for i in range(T))
+
+
+def delta_recurrence(q, k, v, beta, log_g):
+    """q, k [T, H, dk] (k a unit vector), v [T, H, dv], beta / log_g [T, H] -> [T, H, dv]; the read-out follows
+    the write."""
+    T, H, dk = q.shape
+    S = np.zeros((H, dk, v.shape[2]))
+    out = np.empty_like(v)
+    for t in range(T):
+        S *= np.exp(log_g[t])[:, None, None]
+        u = beta[t][:, None] * (v[t] - np.einsum("hkv,hk->hv", S, k[t]))
+        S += k[t][:, :, None] * u[:, None, :]
+        out[t] = np.einsum("hkv,hk->hv", S, q[t])
+    return out
+
+
+def delta_mixer(h, w, p, mx, eps):
+    """The gated delta rule layer; p is the tensor prefix, mx its configuration entry."""
+    T = h.shape[0]
+    dim, vdim, heads, kvh = mx["dim"], mx["vdim"], mx["heads"], mx["kv_heads"]
+    q, k, v = (silu(causal_conv(h @ w[p + n].T, w[p + n + ".conv"])) for n in "qkv")
+    share = heads // kvh
+    q = np.repeat(unit_vector(q.reshape(T, kvh, dim)), share, axis=1) * dim ** -0.5
+    k = np.repeat(unit_vector(k.reshape(T, kvh, dim)), share, axis=1)
+    beta = sigmoid(h @ w[p + "b"].T)
+    log_g = -np.exp(w[p + "A_log"]) * softplus(h @ w[p + "a"].T + w[p + "dt_bias"])
+    o = delta_recurrence(q, k, v.reshape(T, heads, vdim), beta, log_g)
+    o = rms_norm(o, w[p + "norm"], eps) * silu(h @ w[p + "g"].T).reshape(T, heads, vdim)
+    return o.reshape(T, heads * vdim) @ w[p + "o"].T
+
+
+def latent_rows(h, w, p, mx, eps):
+    """What a layer with a W_dkv of its own keeps of a token: the normed latent and the rotated shared key part."""
+    y = h @ w[p + "dkv"].T
+    r = mx["kv_rank"]
+    return rms_norm(y[:, :r], w[p + "dkv.norm"], eps), rotate(y[:, r:], np.arange(len(h)), mx["rot"]["base"])
+
+
+def windowed_softmax_attention(q, k, v, scale, window):
+    """q, k [T, H, d], v [T, H, dv]; position i sees j with 0 <= i - j < window."""
+    T = q.shape[0]
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    seen = (j <= i) & (i - j < window)
+    out = np.empty(v.shape)
+    for h in range(q.shape[1]):
+        s = np.where(seen, (q[:, h] @ k[:, h].T) * scale, -np.inf)
+        s = np.exp(s - s.max(axis=1, keepdims=True))
+        out[:, h] = (s / s.sum(axis=1, keepdims=True)) @ v[:, h]
+    return out
+
+
+def latent_mixer(h, kept, w, p, mx, eps):
+    """Latent attention over kept = (latents, rotated key parts), which may be another layer's."""
+    T = h.shape[0]
+    H, dim, rot, vdim = mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"]
+    c, kr = kept
+    q = (rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps) @ w[p + "uq"].T).reshape(T, H, dim + rot)
+    q = np.concatenate([q[..., :dim], rotate(q[..., dim:], np.arange(T), mx["rot"]["base"])], axis=-1)
+    k = (c @ w[p + "uk"].T).reshape(T, H, dim)
+    k = np.concatenate([k, np.repeat(kr[:, None, :], H, axis=1)], axis=-1)
+    v = (c @ w[p + "uv"].T).reshape(T, H, vdim)
+    o = windowed_softmax_attention(q, k, v, mx["scale"], mx["mask"]["size"])
+    o = o * sigmoid(h @ w[p + "g"].T)[:, :, None]
+    return o.reshape(T, H * vdim) @ w[p + "o"].T
+
+
+def clamped_glu(h, w, p, limit):
+    g = np.minimum(h @ w[p + "gate"].T, limit)
+    u = np.clip(h @ w[p + "up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[p + "down"].T
+
+
+def softcap(z, cap):
+    return cap * np.tanh(z / cap)
+
+
+def forward(config, weights, tokens, layers_out=None):
+    """Logits [T, vocab] of one whole sequence; layers_out (a list) receives the residual after every layer."""
+    w = {n: np.asarray(a, dtype=np.float64) for n, a in weights.items()}
+    eps = config["norm"]["eps"]
+    x = w["embed"][np.asarray(tokens, dtype=np.int64)]
+    kept = {}
+    for i, layer in enumerate(config["layers"]):
+        p, mx = "l%d." % i, layer["mixer"]
+        h = layer_norm(x, w[p + "norm1"], eps)
+        if layer["type"] == "delta":
+            y = delta_mixer(h, w, p + "mix.", mx, eps)
+        else:
+            src = mx.get("kv_from", i)
+            if src == i:
+                kept[i] = latent_rows(h, w, p + "mix.", mx, eps)
+            y = latent_mixer(h, kept[src], w, p + "mix.", mx, eps)
+        x = x + y * w[p + "ls1"]
+        if layer["mlp"] is not None:
+            x = x + clamped_glu(layer_norm(x, w[p + "norm2"], eps), w, p + "mlp.", layer["mlp"]["limit"]) * w[p + "ls2"]
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return softcap(layer_norm(x, w["final.norm"], eps) @ w["head"].T, config["logit_softcap"])
