@@ -15,10 +15,12 @@ namespace k {
 extern int g_gemm_f32_form, g_weight_prefetch, g_probe_plain_loads, g_rows_wide;
 extern int g_skinny_ksplit, g_skinny_ksplit_s, g_row_fusion;
 extern int g_rows_kernel;
+extern int g_linear_form, g_latent_form, g_delta_form;
 extern int g_skinny_ntw, g_skinny_waves, g_skinny_astat, g_gemm_small_tiles, g_gemm_waves, g_gemm_ntb, g_gemm_split_fill;
 }
 int g_decode_waves = 0;
 int g_prefill_generic = 0;
+extern int g_layered_rows;
 extern int g_prefill_rows, g_prefill_fused_rows, g_decode_partials_only, g_prefill_block_form, g_prefill_block_waves, g_prefill_block_split, g_prefill_block_cols;
 }  // namespace fa
 
@@ -104,6 +106,10 @@ fa_status fa_set_tuning(int32_t key, int32_t value) {
         case 25: fa::g_prefill_rows = value; return FA_OK;
         case 26: fa::g_prefill_fused_rows = value; return FA_OK;
         case 27: k::g_rows_rope = value; return FA_OK;
+        case 28: fa::g_layered_rows = value; return FA_OK;
+        case 29: k::g_linear_form = value; return FA_OK;
+        case 30: k::g_latent_form = value; return FA_OK;
+        case 31: k::g_delta_form = value; return FA_OK;
     }
     return fail(FA_ERR_INVALID_ARGUMENT, "fa_set_tuning: unknown key");
 }

@@ -13,6 +13,8 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
+int g_delta_form = 0;        // tuning: 1 keeps the token-by-token kernel for prompts, 2 takes the chunk form from two tokens on
+
 namespace {
 
 template <typename T>

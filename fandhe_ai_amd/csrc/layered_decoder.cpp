@@ -385,13 +385,14 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
             for (uint32_t b = 0; b < B; ++b) {
                 starts[b] = rows;
                 const uint32_t n = (uint32_t)std::min<uint64_t>(counts[b] - done[b], budget - rows);
+                if (n == 0) continue;
                 const uint32_t g0 = first[b] + done[b];
                 for (uint32_t i = 0; i < n; ++i) stage.push_back(tokens[g0 + i]);
                 while (w_at < n_want && want[w_at] < g0 + n) pick_rows.push_back((int32_t)(rows + want[w_at++] - g0));
                 done[b] += n;
                 rows += n;
                 max_new = std::max(max_new, n);
-                if (n && done[b] == counts[b]) last[b] = (int32_t)rows - 1;
+                if (done[b] == counts[b]) last[b] = (int32_t)rows - 1;
             }
             starts[B] = rows;
             if (fa_status s = upload(ctx, a.row_start, starts.data(), (B + 1) * 4)) return s;

@@ -1,0 +1,113 @@
+"""Small random layered models for the tests: configuration, bf16-representable weights, the oracle's logits, and a
+decoder holding the same model."""
+import os
+import sys
+
+import numpy as np
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+sys.path.insert(0, os.path.join(ROOT, "oracle"))
+import layered as oracle  # noqa: E402
+
+
+def delta(heads=4, kv_heads=2, dim=24, vdim=20, conv=4, mlp=None):
+    return {"type": "delta", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}, "mlp": mlp}
+
+
+def latent(heads=3, dim=20, rot=12, vdim=28, q_rank=36, kv_rank=44, window=13, scale=None, base=10000.0, kv_from=None, mlp=None):
+    mx = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank, "mask": {"size": window},
+          "rot": {"base": base, "dims": rot}, "scale": (dim + rot) ** -0.5 if scale is None else scale}
+    if kv_from is not None:
+        mx["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": mx, "mlp": mlp}
+
+
+def glu(ff=52, limit=1.5):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def config(layers, width=76, vocab=131, eps=1e-5, softcap=12.0):
+    return {"architecture": "Nugelix", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps}, "logit_softcap": softcap}
+
+
+def bf16_round(a):
+    u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32).view(np.float32)
+
+
+def shapes(cfg):
+    D = cfg["width"]
+    out = {"embed": (cfg["vocab"], D), "head": (cfg["vocab"], D), "final.norm": (D,)}
+    for i, l in enumerate(cfg["layers"]):
+        p, m, mx = "l%d." % i, "l%d.mix." % i, l["mixer"]
+        H, ow = mx["heads"], mx["heads"] * mx["vdim"]
+        out.update({p + "norm1": (D,), p + "ls1": (D,), m + "g": (ow if l["type"] == "delta" else H, D), m + "o": (D, ow)})
+        if l["type"] == "delta":
+            nq = mx["kv_heads"] * mx["dim"]
+            for n, rows in (("q", nq), ("k", nq), ("v", ow)):
+                out[m + n], out[m + n + ".conv"] = (rows, D), (rows, mx["conv"])
+            out.update({m + "b": (H, D), m + "a": (H, D), m + "A_log": (H,), m + "dt_bias": (H,), m + "norm": (mx["vdim"],)})
+        else:
+            r, k, d = mx["q_rank"], mx["kv_rank"], mx["dim"]
+            out.update({m + "dq": (r, D), m + "dq.norm": (r,), m + "uq": (H * (d + mx["rot_dim"]), r),
+                        m + "uk": (H * d, k), m + "uv": (H * mx["vdim"], k)})
+            if "kv_from" not in mx:
+                out.update({m + "dkv": (k + mx["rot_dim"], D), m + "dkv.norm": (k,)})
+        if l["mlp"]:
+            f, ff = p + "mlp.", l["mlp"]["ff"]
+            out.update({p + "norm2": (D,), p + "ls2": (D,), f + "gate": (ff, D), f + "up": (ff, D), f + "down": (D, ff)})
+    return out
+
+
+def weights(cfg, seed=0):
+    """Random weights of a size that makes every mechanism count: decays between almost none and strong, clamps that
+    bite, attention that is not flat."""
+    rng = np.random.default_rng(seed)
+    w = {}
+    for name, shape in sorted(shapes(cfg).items()):
+        leaf = name.split(".")[-1]
+        if leaf == "A_log":
+            a = np.log(rng.uniform(0.02, 4.0, shape))
+        elif leaf == "dt_bias":
+            a = rng.uniform(-3.0, 0.5, shape)
+        elif leaf == "conv":
+            a = rng.normal(0, 0.6, shape)
+        elif "norm" in leaf:
+            a = 1.0 + 0.3 * rng.normal(size=shape)
+        elif leaf in ("ls1", "ls2"):
+            a = rng.uniform(0.3, 1.2, shape) * rng.choice([-1.0, 1.0], shape)
+        elif leaf == "embed":
+            a = rng.normal(size=shape)
+        elif leaf in ("uq", "uk", "gate", "up", "b"):
+            a = rng.normal(size=shape) * 2.0 / np.sqrt(shape[1])
+        else:
+            a = rng.normal(size=shape) * 1.5 / np.sqrt(shape[1])
+        w[name] = bf16_round(a.astype(np.float32))
+    return w
+
+
+def tokens(cfg, n, seed=0):
+    return [int(t) for t in np.random.default_rng(1000 + seed).integers(0, cfg["vocab"], n)]
+
+
+def make_decoder(ops, cfg, w, dtype="float32", max_tokens=512, max_batch=4, state_slots=None, block_size=16, as_bf16=True):
+    from fandhe_ai_amd import models
+    from fandhe_ai_amd.safetensors_io import TypedTensor
+    d = models.build_layered(ops, cfg, dtype, models.Capacity(max_tokens, max_batch, state_slots, block_size))
+    typed = {}
+    for n, a in w.items():
+        if as_bf16:
+            typed[n] = TypedTensor("BF16", a.shape, (a.view(np.uint32) >> 16).astype(np.uint16))
+        else:
+            typed[n] = TypedTensor("F32", a.shape, a)
+    models.install_weights(d, typed)
+    return d
+
+
+def error(got, want):
+    """Largest over the positions of the r.m.s. difference relative to the logits' overall r.m.s. (means taken off)."""
+    got, want = np.asarray(got, np.float64), np.asarray(want, np.float64)
+    d = got - want
+    d -= d.mean(axis=-1, keepdims=True)
+    c = want - want.mean(axis=-1, keepdims=True)
+    return float(np.sqrt((d * d).mean(axis=-1)).max() / np.sqrt((c * c).mean()))
