@@ -104,6 +104,93 @@ def make_tables(rng, ctxs, extra_tokens, bs, num_blocks=None):
     return tables, max_blocks, num_blocks
 
 
+# ------------------------------------------------------------------ layered decoders
+# Nugelix stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward and depth.
+def _nugelix(width, heads, q_rank, window, ff, d_heads, d_kv_heads, repeat):
+    latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff, "limit": 7.0},
+              "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": q_rank, "kv_rank": 512, "mask": {"size": window},
+                        "rot": {"base": 1e6, "dims": 64}, "scale": 192 ** -0.5}}
+    delta = {"type": "delta", "mlp": None, "mixer": {"heads": d_heads, "kv_heads": d_kv_heads, "dim": 128, "vdim": 128, "conv": 4}}
+    return {"architecture": "Nugelix", "width": width, "vocab": 32000, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "layers": [latent, delta, delta, delta] * repeat}
+
+
+LAYERED = {"large": (_nugelix(4096, 32, 1536, 2048, 14336, 32, 16, 2), dict(d_model=4096, n_heads=32, n_kv_heads=8, d_ffn=14336)),
+           "small": (_nugelix(2048, 16, 768, 1024, 8192, 16, 8, 2), dict(d_model=2048, n_heads=16, n_kv_heads=4, d_ffn=8192))}
+
+
+def build_nugelix(fa, be, config, max_tokens, batch):
+    dec = fa.models.build_layered(be, config, "bfloat16", fa.models.Capacity(max_tokens, batch))
+    noise = np.random.default_rng(0).normal(size=1 << 20).astype(np.float32)
+    for name, shape in dec.tensors().items():
+        n, leaf = int(np.prod(shape)), name.split(".")[-1]
+        if "norm" in leaf or leaf in ("ls1", "ls2"):
+            a = np.ones(shape, np.float32)
+        elif leaf in ("A_log", "dt_bias"):
+            a = np.full(shape, -1.0, np.float32)
+        else:
+            a = np.resize(noise, n).reshape(shape) * np.float32(1.0 if leaf == "embed" else shape[1] ** -0.5)
+        dec.set_tensor(name, (a.view(np.uint32) >> 16).astype(np.uint16), bf16=True)
+    return dec
+
+
+def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, llama=True):
+    """Decode and prompt throughput of a Nugelix stack, and of the W8A8 decoder of equal width, feed-forward and depth."""
+    lib = fa.capi.lib
+    config, shape = LAYERED[size]
+    V, layers = config["vocab"], len(config["layers"])
+    rng = np.random.default_rng(1)
+    most = max(decode_batches + tuple(b for b, _ in prompts))
+    out = []
+
+    def measure(model, dec, set_rows):
+        for b, l in prompts:
+            prompt = rng.integers(0, V, size=(b, l)).astype(np.int32)
+            best = None
+            for _ in range(3):
+                set_rows(dec, b, 0)
+                t = Timer(fa, be)
+                t.start()
+                dec.prefill(prompt)
+                ms = t.stop_ms()
+                best = ms if best is None else min(best, ms)
+            out.append(dict(model=model, size=size, phase="prompt", batch=b, tokens=l, ms=best, tokens_per_s=b * l / best * 1e3))
+        for b in decode_batches:
+            set_rows(dec, b, 0)
+            for at in range(0, ctx, 256):                       # real cache contents and states
+                dec.prefill(rng.integers(0, V, size=(b, 256)).astype(np.int32))
+            for _ in range(3):
+                dec.step()
+            t = Timer(fa, be)
+            t.start()
+            for _ in range(steps):
+                dec.step()
+            ms = t.stop_ms() / steps
+            assert (dec.tokens() >= 0).all()
+            out.append(dict(model=model, size=size, phase="decode", batch=b, context=ctx, ms=ms, tokens_per_s=b / ms * 1e3))
+
+    pages = ctx // 16 + 4
+
+    def rows_of(num_blocks):
+        def set_rows(dec, b, length):
+            t = np.full((b, dec.cfg.max_blocks_per_seq), U32MAX, dtype=np.uint32)
+            t[:, :pages] = np.random.default_rng(2).permutation(num_blocks)[:b * pages].reshape(b, pages)
+            dec.set_sequences(t, [length] * b)
+        return set_rows
+
+    dec = build_nugelix(fa, be, config, most * pages * 16, most)
+    measure("nugelix bf16", dec, rows_of(most * pages))
+    dec.close()
+    if llama:
+        cfg = dict(MODEL, n_layers=layers, vocab=V, **shape)
+        h, keep, _, _, num_blocks = build_decoder(fa, be, cfg, most, [ctx] * most, 64)
+        dcfg = fa.capi.DecoderConfig(cfg["n_layers"], cfg["d_model"], cfg["n_heads"], cfg["n_kv_heads"], cfg["head_dim"], cfg["d_ffn"], V,
+                                     cfg["block_size"], (ctx + 65 + 15) // 16 + 1, num_blocks, most, cfg["rms_eps"], cfg["rope_theta"])
+        measure("w8a8", fa.Decoder.from_handle(be, h, dcfg), rows_of(most * pages))
+        lib.fa_decoder_destroy(be._ctx, h)
+    return out
+
+
 # ------------------------------------------------------------------ full step
 def build_decoder(fa, be, cfg, batch, ctxs, steps_total, seed=0, max_batch=None):
     lib = fa.capi.lib
@@ -812,9 +899,13 @@ def main():
                     help="with --only decode-linears: one of the four layer shapes (0 .. 3) instead of all, so that "
                          "a counter run sees launches of one shape only")
     ap.add_argument("--only", choices=("attention", "copy", "linears", "decode-linears", "prefill", "prefill-attention", "mfma",
-                                       "prompt", "stream-floor", "gemm-f32", "l2-path", "single-stream"), default=None,
+                                       "prompt", "stream-floor", "gemm-f32", "l2-path", "single-stream", "layered"), default=None,
                     help="profiling aid: run only the dominant kernel at the workload's shape, or a plain "
                          "copy kernel of known size (counter calibration), a few launches, no JSON line")
+    ap.add_argument("--layered-size", choices=tuple(LAYERED) + ("all",), default="all",
+                    help="with --only layered: the sizes of the Nugelix stack (and of the W8A8 decoder beside it)")
+    ap.add_argument("--layered-phase", choices=("all", "decode", "prompt"), default="all",
+                    help="with --only layered: all, or one shape of one phase of the Nugelix stack (for a kernel trace)")
     a = ap.parse_args()
     if a.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (--gpus 1); nothing here shards across devices")
@@ -841,6 +932,14 @@ def main():
             for r in bench_prefill_attention(fa, be):
                 log("prefill attention 4 x 2048 new tokens, 32/8 heads, %s kernel: %.2f ms, %.1f TFLOP/s" %
                     (r["kernel"], r["ms"], r["tflops"]))
+            be.close()
+            return
+        if a.only == "layered":
+            kw = {"all": {}, "decode": dict(decode_batches=(32,), prompts=(), llama=False),
+                  "prompt": dict(decode_batches=(), prompts=((4, 2048),), llama=False)}[a.layered_phase]
+            for size in LAYERED if a.layered_size == "all" else (a.layered_size,):
+                for r in bench_layered(fa, be, size, **kw):
+                    print(json.dumps(r), flush=True)
             be.close()
             return
         if a.only == "prompt":
