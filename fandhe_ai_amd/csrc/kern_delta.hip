@@ -13,7 +13,7 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
-int g_delta_form = 0;        // tuning: 1 keeps the token-by-token kernel for prompts, 2 takes the chunk form from two tokens on
+int g_delta_form = 0;        // tuning: 1 keeps the token-by-token kernel for prompts
 
 namespace {
 
@@ -153,6 +153,391 @@ __global__ void __launch_bounds__(NT)
     }
 }
 
+// ------------------------------------------------------------------ chunk form
+// Prompts: 32 tokens at a time.  With G_i the running sum of the chunk's log decays, S_0 the state in front of it and
+//     A_ij = beta_i exp(G_i - G_j) (k_i . k_j)  for j < i,      T = (I + A)^-1,
+// the chunk's writes are U = T diag(beta) V - T diag(beta exp G) K S_0, its read-outs
+//     o_i = exp(G_i) S_0^T q_i + sum_{j <= i} exp(G_i - G_j) (q_i . k_j) u_j,
+// and the state behind it exp(G_C) S_0 + sum_j exp(G_C - G_j) k_j u_j^T.  delta_chunk_kernel forms everything that does
+// not need S_0, for all chunks at once; delta_scan_kernel walks a sequence's chunks with the state in registers.  All
+// products run on the f32 matrix instruction v_mfma_f32_16x16x4_f32.
+//
+// Fragments: 16 x 16 tiles kept as one float4 per lane, 1 KiB.  "A order": lane l holds row l % 16, columns 4 (l / 16) + e
+// (the first operand of the instructions e = 0 .. 3, which take the columns 4 g + e of the four lane groups g); "D order":
+// lane l holds column l % 16, rows 4 (l / 16) + e, what the instruction leaves, and what serves unchanged as the second
+// operand of a product over those rows, columns of the first operand in A order.  Per (chunk, head):
+//     [-W: 2 x KT, A][exp(G) Q: 2 x KT, A][(decayed K)^T: KT x 2, A][P: 00, 10, 11, A][T diag(beta) V: 2 x VT, D]
+// with W = T diag(beta exp G) K, P the decayed lower triangle of Q K^T, KT and VT the tiles of dim and vdim.
+constexpr int kChunk = 32;
+constexpr uint32_t kChunkFrom = 12;          // sequences with fewer new tokens stay with the token-by-token kernel
+
+struct ChunkPlan {
+    uint32_t slots, kt, vt;                  // chunk slots of the pass; tiles of dim (a power of two) and vdim
+    uint32_t frags;                          // fragments per (chunk, head)
+};
+ChunkPlan chunk_plan(const DeltaShape &sh, uint32_t rows, uint32_t batch) {
+    ChunkPlan p;
+    p.slots = rows / kChunk + batch + 1;
+    p.kt = 1;
+    while (p.kt * 16 < sh.dim) p.kt *= 2;
+    p.vt = (sh.vdim + 15) / 16;
+    p.frags = 6 * p.kt + 3 + 2 * p.vt;
+    return p;
+}
+// Chunk i of sequence b has slot row_start[b] / 32 + b + i: no two chunks share one.
+__device__ __forceinline__ uint32_t slot_base(const RaggedRows &rr, uint32_t b) { return rr.row_start[b] / kChunk + b; }
+
+__device__ __forceinline__ v4f mfma4(const v4f &a, const v4f &b, v4f c) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], b[e], c, 0, 0, 0);
+    return c;
+}
+
+// silu(convolution) of `cols` channels from c0 on for the chunk's tokens t0 .. into dst [32][pitch]; zeros for tokens past
+// the end and columns up to cols_p.
+template <typename T, int MAXTAPS>
+__device__ __forceinline__ void conv_chunk(float *dst, uint32_t pitch, const T *__restrict__ y, uint32_t ld, const T *__restrict__ ring,
+                                           const float *__restrict__ conv, uint32_t taps, uint32_t channels, uint32_t c0, uint32_t cols,
+                                           uint32_t cols_p, uint64_t row0, uint32_t t0, uint32_t n, uint32_t p0) {
+    for (uint32_t item = threadIdx.x; item < cols_p * 4; item += 256) {
+        const uint32_t col = item % cols_p, tg = item / cols_p * 8;
+        if (col >= cols) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) dst[(tg + j) * pitch + col] = 0.0f;
+            continue;
+        }
+        const uint32_t c = c0 + col;
+        if constexpr (MAXTAPS == 0) {
+            for (uint32_t j = 0; j < 8; ++j) {
+                const uint32_t t = t0 + tg + j;
+                dst[(tg + j) * pitch + col] = t < n ? conv_silu(y, ld, ring, conv, taps, channels, c, row0, t, p0 + t) : 0.0f;
+            }
+        } else {
+            float w[MAXTAPS], x[8 + MAXTAPS - 1];
+#pragma unroll
+            for (int i = 0; i < MAXTAPS; ++i) w[i] = i < (int)taps ? conv[(uint64_t)c * taps + taps - 1 - i] : 0.0f;      // w[back]
+#pragma unroll
+            for (int j = 0; j < 8 + MAXTAPS - 1; ++j) {
+                const int t = (int)(t0 + tg) + j - (MAXTAPS - 1);
+                float v = 0.0f;
+                if (t >= 0) {
+                    if (t < (int)n) v = load_as_f32(y + (row0 + t) * ld + c);
+                } else if ((int)p0 + t >= 0 && -t < (int)taps) {
+                    v = load_as_f32(ring + (uint64_t)((p0 + t) % taps) * channels + c);
+                }
+                x[j] = v;
+            }
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                float acc = 0.0f;
+#pragma unroll
+                for (int i = MAXTAPS - 1; i >= 0; --i) acc = fmaf(w[i], x[j + MAXTAPS - 1 - i], acc);
+                dst[(tg + j) * pitch + col] = t0 + tg + j < n ? silu_f32(acc) : 0.0f;
+            }
+        }
+    }
+}
+
+template <typename T, int KT, int MAXTAPS>
+__global__ void __launch_bounds__(256)
+    delta_chunk_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, float *__restrict__ frags, float *__restrict__ chunk_decay, uint32_t vt,
+                       uint32_t n_frags) {
+    constexpr uint32_t DP = KT * 16, PITCH = DP + 4;
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    float *lk = lds, *lq = lk + 32 * PITCH;          // K; Q, then V in slices of DP columns
+    float *la = lq + 32 * PITCH, *lt = la + 32 * 36; // A and T, pitch 36
+    __shared__ float rq[32], rk[32], beta[32], G[32];
+    // the slot's sequence and chunk
+    uint32_t lo = 0, hi = rr.batch;
+    while (hi - lo > 1) {
+        const uint32_t mid = (lo + hi) / 2;
+        if (slot_base(rr, mid) <= blockIdx.x) lo = mid;
+        else hi = mid;
+    }
+    const uint32_t b = lo, row0 = rr.row_start[b], n = rr.row_start[b + 1] - row0, t0 = (blockIdx.x - slot_base(rr, b)) * kChunk;
+    if (n < kChunkFrom || t0 >= n) return;
+    const uint32_t h = blockIdx.y, hk = h / (sh.heads / sh.kv_heads), dim = sh.dim, vdim = sh.vdim, channels = sh.qkv();
+    const T *y = (const T *)io.y, *ring = (const T *)io.ring + (uint64_t)rr.state_slot[b] * sh.taps * channels;
+    const uint32_t p0 = (uint32_t)rr.pos[row0];
+    const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, lr = lane % 16, g = lane / 16;
+    v4f *out = (v4f *)(frags + ((uint64_t)blockIdx.x * sh.heads + h) * n_frags * 256) + lane;
+    auto put = [&](uint32_t f, const v4f &v) { out[f * 64] = v; };
+
+    conv_chunk<T, MAXTAPS>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, hk * dim, dim, DP, row0, t0, n, p0);
+    conv_chunk<T, MAXTAPS>(lk, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, (sh.kv_heads + hk) * dim, dim, DP, row0, t0, n, p0);
+    if (tid < 64) {                                  // lanes past 31 only keep the scan whole
+        const uint32_t t = t0 + lane;
+        float lg = 0.0f, be = 0.0f;
+        if (lane < 32 && t < n) {
+            const float *ba = io.ba + (uint64_t)(row0 + t) * io.ld_ba;
+            be = sigmoid_f32(ba[h]);
+            lg = log_decay(io.a_log[h], ba[sh.heads + h] + io.dt_bias[h]);
+        }
+#pragma unroll
+        for (int off = 1; off < 32; off <<= 1) {
+            const float o = __shfl_up(lg, off, 64);
+            if (lane >= off) lg += o;
+        }
+        if (lane < 32) {
+            beta[lane] = be;
+            G[lane] = lg;
+        }
+    }
+    __syncthreads();
+    {   // four threads per row of Q and of K
+        const float *row = (tid < 128 ? lq : lk) + ((tid % 128) / 4) * PITCH;
+        float sq = 0.0f;
+        for (uint32_t i = tid % 4; i < DP; i += 4) sq = fmaf(row[i], row[i], sq);
+        sq += __shfl_xor(sq, 1, 64);
+        sq += __shfl_xor(sq, 2, 64);
+        if (tid % 4 == 0) {
+            const float r = 1.0f / sqrtf(sq + 1e-6f);
+            if (tid < 128) rq[tid / 4] = r / sqrtf((float)dim);
+            else rk[(tid - 128) / 4] = r;
+        }
+    }
+    __syncthreads();
+    // (K K^T) tiles 00, 10, 11 and (K Q^T) tiles: wave 0: both 00, 1: KK 10, 2: QK 10, 3: both 11.  Rows of the result are
+    // j (the keys), its column i: D order of the transpose is A order of the matrix.
+    auto dot_tile = [&](const float *rows_j, const float *rows_i) {
+        v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
+        for (uint32_t k = g; k < DP; k += 4)
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(rows_j[lr * PITCH + k], rows_i[lr * PITCH + k], acc, 0, 0, 0);
+        return acc;
+    };
+    const int ti = wave == 0 ? 0 : 1, tj = wave == 3 ? 1 : 0, i_ = ti * 16 + lr;
+    if (wave != 2) {
+        const v4f d = dot_tile(lk + tj * 16 * PITCH, lk + ti * 16 * PITCH);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int j = tj * 16 + 4 * g + e;
+            la[i_ * 36 + j] = j < i_ ? beta[i_] * expf(G[i_] - G[j]) * rk[i_] * rk[j] * d[e] : 0.0f;
+        }
+    }
+    if (wave != 1) {
+        v4f d = dot_tile(lk + tj * 16 * PITCH, lq + ti * 16 * PITCH);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int j = tj * 16 + 4 * g + e;
+            d[e] = j <= i_ ? expf(G[i_] - G[j]) * rq[i_] * rk[j] * d[e] : 0.0f;
+        }
+        put(6 * KT + ti + tj, d);
+    }
+    // exp(G) Q and the decayed K^T
+    for (uint32_t f = wave; f < 2 * KT; f += 4) {
+        const uint32_t rt = f / KT, kt = f % KT, i = rt * 16 + lr;
+        put(2 * KT + f, *(const v4f *)(lq + i * PITCH + kt * 16 + 4 * g) * (expf(G[i]) * rq[i]));
+        const uint32_t dt = f / 2, ct = f % 2;
+        v4f v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const uint32_t j = ct * 16 + 4 * g + e;
+            v[e] = lk[j * PITCH + dt * 16 + lr] * rk[j] * expf(G[31] - G[j]);
+        }
+        put(4 * KT + f, v);
+    }
+    if (tid == 0) chunk_decay[(uint64_t)blockIdx.x * sh.heads + h] = expf(G[31]);
+    __syncthreads();
+    // T = (I + A)^-1: the diagonal blocks column by column (lanes 0 - 15, 16 - 31), then T10 = -T11 A10 T00
+    if (wave == 0) {
+        if (lane < 32) {
+            const int o = (lane / 16) * 16;
+            float x[16];
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                float v = i == lr ? 1.0f : 0.0f;
+#pragma unroll
+                for (int j = 0; j < i; ++j) v = fmaf(-la[(o + i) * 36 + o + j], x[j], v);
+                x[i] = v;
+                lt[(o + i) * 36 + o + lr] = v;
+            }
+        }
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+        __builtin_amdgcn_wave_barrier();
+        v4f x = v4f{0.f, 0.f, 0.f, 0.f}, t00, t10 = x;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) t00[e] = lt[(4 * g + e) * 36 + lr];
+        x = mfma4(*(const v4f *)(la + (16 + lr) * 36 + 4 * g), t00, x);
+        t10 = mfma4(*(const v4f *)(lt + (16 + lr) * 36 + 16 + 4 * g), x, t10);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            lt[(16 + 4 * g + e) * 36 + lr] = -t10[e];
+            lt[(4 * g + e) * 36 + 16 + lr] = 0.0f;
+        }
+    }
+    __syncthreads();
+    // -W^T = -K'^T T^T, K' = diag(beta exp(G) rk) K: the columns of the result are tokens, so its D order is W's A order
+    v4f tf[2][2];                                    // T fragments: second operand of W^T, first operand of T V
+#pragma unroll
+    for (int rt = 0; rt < 2; ++rt)
+#pragma unroll
+        for (int ct = 0; ct < 2; ++ct) {
+            tf[rt][ct] = *(const v4f *)(lt + (rt * 16 + lr) * 36 + ct * 16 + 4 * g);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) tf[rt][ct][e] *= beta[ct * 16 + 4 * g + e];
+        }
+    for (uint32_t f = wave; f < 2 * KT; f += 4) {
+        const uint32_t rt = f / KT, kt = f % KT;
+        v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
+        for (uint32_t ct = 0; ct <= rt; ++ct) {
+            v4f kf;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const uint32_t j = ct * 16 + 4 * g + e;
+                kf[e] = -lk[j * PITCH + kt * 16 + lr] * rk[j] * expf(G[j]);
+            }
+            acc = mfma4(kf, rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], acc);
+        }
+        put(f, acc);
+    }
+    // T diag(beta) V, DP columns of V at a time in Q's place (all reads of Q are behind the barriers above)
+    for (uint32_t v0 = 0; v0 < vdim; v0 += DP) {
+        const uint32_t cols = vdim - v0 < DP ? vdim - v0 : DP, cols_p = (cols + 15) / 16 * 16;
+        if (v0) __syncthreads();
+        conv_chunk<T, MAXTAPS>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, 2 * sh.kv_heads * dim + h * vdim + v0, cols, cols_p, row0, t0, n, p0);
+        __syncthreads();
+        for (uint32_t f = wave; f < 2 * (cols_p / 16); f += 4) {
+            const uint32_t rt = f % 2, nt = f / 2;
+            v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
+            for (uint32_t ct = 0; ct <= rt; ++ct) {
+                v4f vf;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) vf[e] = lq[(ct * 16 + 4 * g + e) * PITCH + nt * 16 + lr];
+                acc = mfma4(rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], vf, acc);
+            }
+            put(6 * KT + 3 + (v0 / 16 + nt) * 2 + rt, acc);
+        }
+    }
+}
+
+// One wavefront per (sequence, head, 16 value columns); state tile kt in D order: rows 16 kt + 4 g + e, column l % 16.
+template <int KT>
+__global__ void __launch_bounds__(256)
+    delta_scan_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, const float *__restrict__ frags, const float *__restrict__ chunk_decay,
+                      float *__restrict__ o, uint32_t vt, uint32_t n_frags) {
+    const int lane = threadIdx.x % 64, wave = threadIdx.x / 64, lr = lane % 16, g = lane / 16;
+    const uint32_t b = blockIdx.z, h = blockIdx.y, nt = blockIdx.x * (blockDim.x / 64) + wave;
+    const uint32_t row0 = rr.row_start[b], n = rr.row_start[b + 1] - row0;
+    if (n < kChunkFrom || nt >= vt) return;
+    const uint32_t dim = sh.dim, vdim = sh.vdim, vp = sh.vdim_p(), col = nt * 16 + lr, slot0 = slot_base(rr, b);
+    float *state = io.state + ((uint64_t)rr.state_slot[b] * sh.heads + h) * dim * vp;
+    const bool fresh = rr.pos[row0] == 0;
+    v4f S[KT];
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const uint32_t d = kt * 16 + 4 * g + e;
+            S[kt][e] = !fresh && d < dim && col < vdim ? state[(uint64_t)d * vp + col] : 0.0f;
+        }
+    const uint32_t chunks = (n + kChunk - 1) / kChunk;
+    v4f wq[4 * KT], kd[2 * KT], pf[3], u0[2];
+    auto base = [&](uint32_t c) { return (const v4f *)(frags + ((uint64_t)(slot0 + c) * sh.heads + h) * n_frags * 256) + lane; };
+    auto load_wq = [&](const v4f *f) {
+#pragma unroll
+        for (int i = 0; i < 4 * KT; ++i) wq[i] = f[i * 64];
+    };
+    auto load_rest = [&](const v4f *f) {
+#pragma unroll
+        for (int i = 0; i < 2 * KT; ++i) kd[i] = f[(4 * KT + i) * 64];
+#pragma unroll
+        for (int i = 0; i < 3; ++i) pf[i] = f[(6 * KT + i) * 64];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) u0[i] = f[(6 * KT + 3 + nt * 2 + i) * 64];
+    };
+    load_wq(base(0));
+    load_rest(base(0));
+    for (uint32_t c = 0; c < chunks; ++c) {
+        const v4f *next = base(c + 1 < chunks ? c + 1 : c);
+        const float decay = chunk_decay[(uint64_t)(slot0 + c) * sh.heads + h];
+        v4f u[2] = {u0[0], u0[1]}, r[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+#pragma unroll
+                for (int rt = 0; rt < 2; ++rt) {
+                    u[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(wq[rt * KT + kt][e], S[kt][e], u[rt], 0, 0, 0);
+                    r[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(wq[(2 + rt) * KT + kt][e], S[kt][e], r[rt], 0, 0, 0);
+                }
+        load_wq(next);
+        r[0] = mfma4(pf[0], u[0], r[0]);
+        r[1] = mfma4(pf[1], u[0], r[1]);
+        r[1] = mfma4(pf[2], u[1], r[1]);
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt) S[kt] *= decay;
+#pragma unroll
+        for (int ct = 0; ct < 2; ++ct)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+#pragma unroll
+                for (int kt = 0; kt < KT; ++kt) S[kt] = __builtin_amdgcn_mfma_f32_16x16x4f32(kd[kt * 2 + ct][e], u[ct][e], S[kt], 0, 0, 0);
+        load_rest(next);
+#pragma unroll
+        for (int rt = 0; rt < 2; ++rt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const uint32_t t = c * kChunk + rt * 16 + 4 * g + e;
+                if (t < n && col < vdim) o[((uint64_t)(row0 + t) * sh.heads + h) * vdim + col] = r[rt][e];
+            }
+    }
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const uint32_t d = kt * 16 + 4 * g + e;
+            if (d < dim && col < vdim) state[(uint64_t)d * vp + col] = S[kt][e];
+        }
+}
+
+// Read-outs of the chunk form: root mean square, weight, gate.  One wavefront per (row, head).
+template <typename T>
+__global__ void __launch_bounds__(256) delta_gate_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, const float *__restrict__ o) {
+    const uint32_t lane = threadIdx.x % 64, r = blockIdx.x, vdim = sh.vdim, b = rr.row_seq[r];
+    if (rr.row_start[b + 1] - rr.row_start[b] < kChunkFrom) return;
+    for (uint32_t h = threadIdx.x / 64; h < sh.heads; h += 4) {
+        const float *x = o + ((uint64_t)r * sh.heads + h) * vdim;
+        float sq = 0.0f;
+        for (uint32_t c = lane; c < vdim; c += 64) sq = fmaf(x[c], x[c], sq);
+        const float ro = 1.0f / sqrtf(wave_sum_dpp(sq) / (float)vdim + sh.eps);
+        const T *gate = (const T *)io.y + (uint64_t)r * io.ld_y + sh.qkv() + h * vdim;
+        for (uint32_t c = lane; c < vdim; c += 64)
+            store_from_f32((T *)io.out + (uint64_t)r * io.ld_out + h * vdim + c, x[c] * ro * io.norm[c] * silu_f32(load_as_f32(gate + c)));
+    }
+}
+
+template <typename T, int KT>
+void launch_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr, const ChunkPlan &p, hipStream_t s) {
+    float *frags = io.scratch, *decay = frags + (uint64_t)p.slots * sh.heads * p.frags * 256, *o = decay + (((uint64_t)p.slots * sh.heads + 63) / 64) * 64;
+    const size_t lds = (2 * 32 * (KT * 16 + 4) + 2 * 32 * 36) * 4;
+    auto chunk = sh.taps <= 4 ? &delta_chunk_kernel<T, KT, 4> : &delta_chunk_kernel<T, KT, 0>;
+    if (lds > 65536) {
+        static bool configured = false;
+        if (!configured) {
+            for (auto f : {&delta_chunk_kernel<T, KT, 4>, &delta_chunk_kernel<T, KT, 0>})
+                (void)hipFuncSetAttribute(reinterpret_cast<const void *>(f), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            configured = true;
+        }
+    }
+    chunk<<<dim3(p.slots, sh.heads), 256, lds, s>>>(sh, io, rr, frags, decay, p.vt, p.frags);
+    // wavefronts of a block share the chunk's fragments through the L1; fewer per block where there are few blocks
+    const uint32_t per = (uint64_t)rr.batch * sh.heads * p.vt <= 512 ? 1 : (uint64_t)rr.batch * sh.heads * p.vt <= 1024 ? 2 : 4;
+    delta_scan_kernel<KT><<<dim3((p.vt + per - 1) / per, sh.heads, rr.batch), per * 64, 0, s>>>(sh, io, rr, frags, decay, o, p.vt, p.frags);
+    delta_gate_kernel<T><<<rr.rows, 256, 0, s>>>(sh, io, rr, o);
+}
+
+template <typename T>
+void run_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr, hipStream_t s) {
+    const ChunkPlan p = chunk_plan(sh, rr.rows, rr.batch);
+    switch (p.kt) {
+        case 1: return launch_chunks<T, 1>(sh, io, rr, p, s);
+        case 2: return launch_chunks<T, 2>(sh, io, rr, p, s);
+        case 4: return launch_chunks<T, 4>(sh, io, rr, p, s);
+        case 8: return launch_chunks<T, 8>(sh, io, rr, p, s);
+        default: return launch_chunks<T, 16>(sh, io, rr, p, s);
+    }
+}
+
 // After a pass with more than one token anywhere: the last `taps` inputs of every sequence enter its ring.
 template <typename T>
 __global__ void __launch_bounds__(256) delta_ring_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr) {
@@ -180,14 +565,23 @@ void mixer(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr, uint32
     uint32_t cg_log2 = 0;
     while ((4u << cg_log2) < sh.vdim) ++cg_log2;
     const int write_ring = max_new == 1;
-    if (cg_log2 <= 6) launch_step<T, 256>(sh, io, rr, cg_log2, write_ring, max_new, s);
-    else launch_step<T, 1024>(sh, io, rr, cg_log2, write_ring, max_new, s);
+    const bool chunks = max_new >= kChunkFrom && g_delta_form != 1;
+    const uint32_t longest = chunks ? kChunkFrom - 1 : max_new;      // sequences of a pass go to one of the two forms by length
+    if (!chunks || rr.batch > 1) {
+        if (cg_log2 <= 6) launch_step<T, 256>(sh, io, rr, cg_log2, write_ring, longest, s);
+        else launch_step<T, 1024>(sh, io, rr, cg_log2, write_ring, longest, s);
+    }
+    if (chunks) run_chunks<T>(sh, io, rr, s);
     if (!write_ring) delta_ring_kernel<T><<<dim3(rr.batch, (sh.qkv() + 255) / 256), 256, 0, s>>>(sh, io, rr);
 }
 
 }  // namespace
 
-uint64_t delta_scratch_bytes(const DeltaShape &sh, uint32_t rows, uint32_t batch) { return 0; }
+uint64_t delta_scratch_bytes(const DeltaShape &sh, uint32_t rows, uint32_t batch) {
+    if (rows < kChunkFrom) return 0;
+    const ChunkPlan p = chunk_plan(sh, rows, batch);
+    return ((uint64_t)p.slots * sh.heads * (p.frags * 256 + 1) + 64 + (uint64_t)rows * sh.heads * sh.vdim) * 4;
+}
 
 void delta_mixer(const DeltaShape &sh, const DeltaIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, hipStream_t s) {
     if (rr.rows == 0) return;
