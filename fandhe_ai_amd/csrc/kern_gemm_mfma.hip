@@ -13,6 +13,7 @@
 #include "device_utils.hpp"
 #include "index_models.hpp"
 #include "kernels.hpp"
+#include "linear_epilogue.hpp"
 
 namespace fa {
 namespace k {
@@ -64,6 +65,19 @@ struct EpiF8 {
     void *out;
     int out_bf16;
     const float *sx, *sw, *bias;      // ... or, when sx is set, one per row and one per column (+ optional bias)
+};
+
+// bf16, large-tile kernel only: the unquantized linears' epilogues (linear_epilogue.hpp).  A bf16 operand moves exactly as
+// int8 does (a stage of 128 bytes is two k tiles of 32 values, 16 bytes per lane); only the instruction differs.
+template <int MODE>
+struct EpiBf16 {
+    LinearEpilogue ep;
+};
+template <typename Epi>
+struct IsBf16 : std::false_type {};
+template <int MODE>
+struct IsBf16<EpiBf16<MODE>> : std::true_type {
+    static constexpr int mode = MODE;
 };
 
 constexpr int BM = 128, BN = 128;      // block tile; 4 wavefronts in 2 x 2, 64 x 64 each
@@ -273,6 +287,9 @@ __global__ void __launch_bounds__(256)
 __device__ __forceinline__ void mfma_acc(v4i &c, const v4i &a, const v4i &b) {
     asm volatile("v_mfma_i32_16x16x64_i8 %0, %1, %2, %0" : "+a"(c) : "v"(a), "v"(b));
 }
+__device__ __forceinline__ void mfma_acc(v4f &c, const v4i &a, const v4i &b) {
+    asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+a"(c) : "v"(a), "v"(b));
+}
 __device__ __forceinline__ void mfma_acc(v4f &c, const v8i &a, const v8i &b) {
     const int unit = 0x7f7f7f7f;                      // block scales 2^0
     asm volatile("v_mfma_scale_f32_16x16x128_f8f6f4 %0, %1, %2, %0, %3, %3 op_sel_hi:[0,0,0]"
@@ -370,6 +387,8 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];   // [3][A_STAGE] then [2][B_STAGE]
 
     constexpr bool SWI = std::is_same<Epi, EpiI8Swiglu>::value, ROPE = std::is_same<Epi, EpiI8QkvRope>::value;
+    constexpr bool BF16 = IsBf16<Epi>::value;
+    static_assert(!BF16 || !FP8, "bf16 operands take the int8 layout");
     static_assert(!SWI || (!FP8 && NTB % 4 == 0), "the SwiGLU form pairs gate and up tiles inside a wavefront");
     static_assert(!ROPE || (!FP8 && NTB == 16), "the RoPE form: a head of 128 dims is the eight column tiles of one wavefront");
     const int tid = threadIdx.x, lane = tid % 64;
@@ -448,13 +467,13 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
                                          (lptr)(lds + ixm::big_b_lds_slice<NTB>(slot, ixm::big_b_tile<NTB, NWAVES>(wave, i), h)), 16, 0, 0);
     };
 
-    typedef typename std::conditional<FP8, v4f, v4i>::type acc_t;
+    typedef typename std::conditional<FP8 || BF16, v4f, v4i>::type acc_t;
     acc_t acc[AI][WNT];
 #pragma unroll
     for (int i = 0; i < AI; ++i)
 #pragma unroll
         for (int j = 0; j < WNT; ++j) {
-            if constexpr (FP8) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
+            if constexpr (FP8 || BF16) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
             else acc[i][j] = v4i{0, 0, 0, 0};
         }
     // the per-tensor scales of the e4m3 epilogue are fetched here, not after the last stage, where the two dependent
@@ -642,7 +661,21 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
     int row_l0, col_l0;                               // block-local row of this lane in row tile 0, first column in tile 0
     ixm::big_out_elem<NTB, WM>(wm, wn, 0, 0, 0, lane, &row_l0, &col_l0);
     const int g = lane / 16;
-    if constexpr (ROPE) {
+    if constexpr (BF16) {
+        constexpr int MODE = IsBf16<Epi>::mode, STEP = MODE == LinearEpilogue::kGlu ? 2 : 1;      // gate, up: neighbouring tiles
+        static_assert(STEP == 1 || WNT % 2 == 0, "a gate tile and its up tile belong to one wavefront");
+#pragma unroll
+        for (int i = 0; i < AI; ++i) {
+            const uint32_t row = m0 + row_l0 + i * 16;
+            if (row >= m) continue;
+#pragma unroll
+            for (int j = 0; j < WNT; j += STEP) {
+                const uint32_t t = nt0 + wn * WNT + j;
+                if (t < n_tiles) epilogue_store4<MODE>(ep.ep, row, t / STEP * 16 + 4 * g, n, 0, acc[i][j], acc[i][j + STEP - 1]);
+            }
+        }
+        return;
+    } else if constexpr (ROPE) {
         // The eight column tiles of this wavefront are head hd = 2 nb + wn of q | k | v; tiles j and j + 4 hold dims d
         // and d + 64 of the rotate-half pairs (four consecutive d per lane).  The arithmetic is rope_append's: dequantize,
         // x0 c - x1 s and x1 c + x0 s with explicit roundings, one rounding to bf16.
@@ -1093,6 +1126,31 @@ static void launch_e4m3(const uint8_t *aq, const uint8_t *w_tiles, const EpiF8 &
     dim3 grid((unsigned)((n_pad / 16 + NT - 1) / NT), (unsigned)((m + BM - 1) / BM));
     gemm_mfma_kernel<true, EpiF8><<<grid, 256, 0, s>>>(aq, w_tiles, (uint32_t)m, (uint32_t)n, (uint32_t)(n_pad / 16),
                                                        (uint32_t)(k_pad / 128), e, nullptr);
+}
+
+namespace {
+template <int MODE>
+void launch_big_bf16(const uint16_t *a, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int ntb, hipStream_t s) {
+    const EpiBf16<MODE> e{ep};
+    if constexpr (MODE != LinearEpilogue::kGlu) {
+        if (ntb == 14) return launch_big_wm<false, 14, 4>((const uint8_t *)a, (const uint8_t *)w.w, m, w.n, w.n_tiles, w.k_tiles / 2, e, s);
+    }
+    launch_big_wm<false, 16, 4>((const uint8_t *)a, (const uint8_t *)w.w, m, w.n, w.n_tiles, w.k_tiles / 2, e, s);
+}
+}  // namespace
+
+bool gemm_bf16_big_applies(uint64_t lda, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus) {
+    return w.batches == 1 && lda == (uint64_t)w.k_tiles * 32 && w.k_tiles % 2 == 0 && pick_big_ntb(m, w.n_tiles, num_cus) != 0;
+}
+
+void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus, hipStream_t s) {
+    const int ntb = pick_big_ntb(m, w.n_tiles, num_cus);
+    switch (ep.mode) {
+        case LinearEpilogue::kResidual: return launch_big_bf16<LinearEpilogue::kResidual>(a, m, w, ep, ntb, s);
+        case LinearEpilogue::kGlu: return launch_big_bf16<LinearEpilogue::kGlu>(a, m, w, ep, ntb, s);
+        case LinearEpilogue::kSoftcap: return launch_big_bf16<LinearEpilogue::kSoftcap>(a, m, w, ep, ntb, s);
+        default: return launch_big_bf16<LinearEpilogue::kStore>(a, m, w, ep, ntb, s);
+    }
 }
 
 }  // namespace k

@@ -13,7 +13,7 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
-int g_linear_form = 0;        // tuning: 1 keeps the 128 x 128 kernel out, 2 keeps the large-tile kernel out
+int g_linear_form = 0;        // tuning: 2 keeps the large-tile kernel out
 
 namespace {
 
@@ -284,7 +284,7 @@ void launch_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
 #undef FA_ROWS
         return;
     }
-    if (g_linear_form != 2 && gemm_bf16_big_applies(lda, m, w, ep, num_cus)) return gemm_bf16_big(a, m, w, ep, num_cus, s);
+    if (MODE != LinearEpilogue::kHeadGate && g_linear_form != 2 && gemm_bf16_big_applies(lda, m, w, ep, num_cus)) return gemm_bf16_big(a, m, w, ep, num_cus, s);
     const dim3 grid((w.n_tiles + 7) / 8, (unsigned)((m + 127) / 128), w.batches);
     linear_tile_kernel<MODE><<<grid, 256, 0, s>>>(a, lda, a_batch, wt, (uint32_t)m, w.n, w.n_tiles, w.k_tiles, ep);
 }
@@ -335,7 +335,5 @@ void pack_linear(const void *src, int src_f32, uint64_t row_stride, uint64_t col
         pack_linear_kernel<uint16_t, uint16_t><<<grid, 256, 0, s>>>((const uint16_t *)src, row_stride, col_stride, rows, cols, (uint16_t *)dst, k_tiles, n0, group, pitch);
 }
 
-bool gemm_bf16_big_applies(uint64_t, uint64_t, const LinearWeight &, const LinearEpilogue &, int) { return false; }
-void gemm_bf16_big(const uint16_t *, uint64_t, const LinearWeight &, const LinearEpilogue &, int, hipStream_t) {}
 }  // namespace k
 }  // namespace fa
