@@ -11,7 +11,8 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
-int g_latent_form = 0;       // tuning: 1 keeps the plain attention kernel
+int g_latent_form = 0;       // tuning: 1 keeps the plain attention kernel, 2 the absorbed form for every pass, 3 takes the
+                             // expanded form wherever it can run
 
 namespace {
 
@@ -142,6 +143,471 @@ __global__ void __launch_bounds__(256)
     }
 }
 
+// ------------------------------------------------------------------ matrix-core pieces
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kKeys = 32;                            // keys per step of the kernels below
+
+typedef short v4s __attribute__((ext_vector_type(4)));
+typedef short v8s __attribute__((ext_vector_type(8)));
+
+// The transposed operand of a 32-key step from rows staged in LDS: lane (g, c) gets dim c of 16 dims for keys 4 g .. 4 g + 3
+// and 16 + 4 g .. + 3, in the order in which the scores of the two key tiles sit in a lane.  rows: LDS element address of
+// (key 0, first dim); pitch in elements.
+__device__ __forceinline__ v8bf transposed_keys(const uint16_t *rows, uint32_t pitch, int lane) {
+    typedef __attribute__((address_space(3))) v4s *lptr;
+    const int g = lane / 16, i = lane % 16;
+    const uint16_t *p = rows + (4 * g + i / 4) * pitch + 4 * (i % 4);
+    const v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lptr)p), hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lptr)(p + 16 * pitch));
+    return __builtin_bit_cast(v8bf, v8s{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
+}
+
+// One online-softmax step of a column (query row): scores of eight keys per lane, lanes with equal lane % 16 share the
+// column.  Returns the factor for what was accumulated before; w receives the weights as two bf16 terms whose sum keeps
+// about 16 bits of them.
+__device__ __forceinline__ float softmax_step(const float (&sc)[8], float &m, float &l, v8bf &w_hi, v8bf &w_lo) {
+    float mx = fmaxf(fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3])), fmaxf(fmaxf(sc[4], sc[5]), fmaxf(sc[6], sc[7])));
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float m_new = fmaxf(m, mx), ref = m_new == -INFINITY ? 0.0f : m_new;
+    const float fix = exp2f(m - ref);
+    float sum = 0.0f;
+    uint32_t hi[4], lo[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const float a = exp2f(sc[2 * i] - ref), b = exp2f(sc[2 * i + 1] - ref);
+        sum += a + b;
+        hi[i] = f32x2_to_bf16x2(a, b);
+        lo[i] = f32x2_to_bf16x2(a - bf16_lo(hi[i]), b - bf16_hi(hi[i]));
+    }
+    l = l * fix + sum;
+    m = m_new;
+    w_hi = __builtin_bit_cast(v8bf, v4u{hi[0], hi[1], hi[2], hi[3]});
+    w_lo = __builtin_bit_cast(v8bf, v4u{lo[0], lo[1], lo[2], lo[3]});
+    return fix;
+}
+
+// ------------------------------------------------------------------ absorbed form
+// Query rows of a sequence are its (token, head) pairs in order; a block of NW wavefronts takes 16 NW of them, every
+// wavefront 16 columns of S^T = K Q^T, and walks its share of the keys any of them sees, 32 at a time.  The cached rows of
+// a step are staged once and serve as keys (all of the row) and, transposed, as values (the latent part).
+// Tile i of sequence b has slot row_start[b] heads / (16 NW) + b + i: no two tiles share one.
+struct StreamParams {
+    const uint16_t *qa, *pool;
+    uint16_t *out;
+    float *part_o, *part_ml;                         // [slot][split][16 NW][rank_p], [slot][split][2][16 NW]
+    uint32_t splits;
+};
+
+template <int NW>
+__device__ __forceinline__ bool stream_tile(const RaggedRows &rr, uint32_t heads, uint32_t slot, uint32_t *b_out, uint32_t *t0, uint32_t *n_rows) {
+    auto base = [&](uint32_t b) { return (uint32_t)((uint64_t)rr.row_start[b] * heads / (16 * NW)) + b; };
+    uint32_t lo = 0, hi = rr.batch;
+    while (hi - lo > 1) {
+        const uint32_t mid = (lo + hi) / 2;
+        if (base(mid) <= slot) lo = mid;
+        else hi = mid;
+    }
+    *b_out = lo;
+    *t0 = (slot - base(lo)) * 16 * NW;
+    *n_rows = (rr.row_start[lo + 1] - rr.row_start[lo]) * heads;
+    return *t0 < *n_rows;
+}
+
+template <int RK, int RO, int NW>
+__global__ void __launch_bounds__(NW * 64)
+    latent_stream_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
+    constexpr int KS = RK + RO, VT = 2 * RK, PITCH = KS * 32 + 8, TPK = NW * 64 / kKeys, PIECES = (KS * 4 + TPK - 1) / TPK;
+    extern __shared__ __attribute__((aligned(16))) uint16_t stage[];        // [2][32][PITCH]
+    uint32_t b, t0, n_rows;
+    if (!stream_tile<NW>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
+    const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, g = lane / 16, c = lane % 16;
+    const uint32_t row0 = rr.row_start[b], H = sh.heads, width = sh.rank_p + sh.rot_p, rk = sh.rank_p / 32, ro = sh.rot_p / 32;
+    const uint32_t *table = rr.tables + (uint64_t)b * rr.max_blocks;
+    const uint32_t last_row = t0 + 16 * NW - 1 < n_rows ? t0 + 16 * NW - 1 : n_rows - 1;
+    const int32_t p0 = rr.pos[row0], p_lo = p0 + (int32_t)(t0 / H), p_hi = p0 + (int32_t)(last_row / H), W = (int32_t)sh.window;
+    int32_t k_lo = p_lo - W + 1 > 0 ? p_lo - W + 1 : 0, k_hi = p_hi + 1;    // keys seen by some column
+    if (p.splits > 1) {
+        const int32_t per = ((k_hi - k_lo + (int32_t)p.splits - 1) / (int32_t)p.splits + kKeys - 1) / kKeys * kKeys;
+        k_lo += (int32_t)blockIdx.y * per;
+        k_hi = k_lo + per < k_hi ? k_lo + per : k_hi;
+    }
+    // this lane's column
+    const uint32_t col = t0 + wave * 16 + c, qr = col < n_rows ? col : n_rows - 1;
+    const int32_t pos = p0 + (int32_t)(qr / H);
+    const uint16_t *q = p.qa + ((uint64_t)row0 * H + qr) * width;
+    v8bf qf[KS];
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+        v4u v = v4u{0, 0, 0, 0};
+        if (s < RK ? (uint32_t)s < rk : (uint32_t)(s - RK) < ro) v = *(const v4u *)(q + (s < RK ? s * 32 : sh.rank_p + (s - RK) * 32) + 8 * g);
+        qf[s] = __builtin_bit_cast(v8bf, v);
+    }
+    // staging: TPK threads per key; piece i of a thread is 16-byte piece part + i TPK of the row
+    const int key = tid / TPK, part = tid % TPK;
+    v4u st[PIECES];
+    auto key_row = [&](int32_t j) -> const uint16_t * {              // null: outside the walk; the pool's end: no page
+        if (j >= k_hi) return nullptr;
+        const uint32_t blk = (uint32_t)j / rr.block_size, id = blk < rr.max_blocks ? table[blk] : 0xffffffffu;
+        return p.pool + (id < rr.num_blocks ? (uint64_t)id * rr.block_size + (uint32_t)j % rr.block_size : sh.pool_rows) * width;
+    };
+    const uint16_t *const no_page = p.pool + sh.pool_rows * width;
+    auto fetch = [&](const uint16_t *src) {
+        const uint32_t fill = src == no_page ? 0x7fc07fc0u : 0u;     // a position without a page: NaN, never a silent zero
+#pragma unroll
+        for (int i = 0; i < PIECES; ++i) {
+            const int pc = part + i * TPK, s = pc / 4;
+            st[i] = v4u{fill, fill, fill, fill};
+            const bool real = pc < KS * 4 && (s < RK ? (uint32_t)s < rk : (uint32_t)(s - RK) < ro);
+            if (!real) st[i] = v4u{0, 0, 0, 0};
+            else if (src && src != no_page) st[i] = *(const v4u *)(src + (s < RK ? s * 32 : sh.rank_p + (s - RK) * 32) + (pc % 4) * 8);
+        }
+    };
+    auto put = [&](int buf) {
+#pragma unroll
+        for (int i = 0; i < PIECES; ++i) {
+            const int pc = part + i * TPK;
+            if (pc < KS * 4) *(v4u *)(stage + (buf * kKeys + key) * PITCH + pc * 8) = st[i];
+        }
+    };
+    float m = -INFINITY, l = 0.0f;
+    v4f o[VT];
+#pragma unroll
+    for (int t = 0; t < VT; ++t) o[t] = v4f{0.f, 0.f, 0.f, 0.f};
+    const uint16_t *next = nullptr;
+    if (k_lo < k_hi) {
+        fetch(key_row(k_lo + key));
+        next = key_row(k_lo + kKeys + key);
+        put(0);
+    }
+    __syncthreads();
+    int buf = 0;
+    for (int32_t k0 = k_lo; k0 < k_hi; k0 += kKeys, buf ^= 1) {
+        const bool more = k0 + kKeys < k_hi;
+        if (more) {
+            fetch(next);
+            next = key_row(k0 + 2 * kKeys + key);
+        }
+        const uint16_t *rows = stage + buf * kKeys * PITCH;
+        float sc[8];
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt) {
+            v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int s = 0; s < KS; ++s)
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const v8bf *)(rows + (kt * 16 + c) * PITCH + s * 32 + 8 * g), qf[s], acc, 0, 0, 0);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int32_t j = k0 + kt * 16 + 4 * g + e;
+                sc[kt * 4 + e] = j <= pos && pos - j < W && j < k_hi ? acc[e] * (sh.scale * kLog2e) : -INFINITY;
+            }
+        }
+        v8bf w_hi, w_lo;
+        const float fix = softmax_step(sc, m, l, w_hi, w_lo);
+        if (__any(fix != 1.0f)) {
+#pragma unroll
+            for (int t = 0; t < VT; ++t) o[t] *= fix;
+        }
+#pragma unroll
+        for (int t = 0; t < VT; ++t) {
+            const v8bf v = transposed_keys(rows + t * 16, PITCH, lane);
+            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_hi, o[t], 0, 0, 0);
+            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_lo, o[t], 0, 0, 0);
+        }
+        if (more) put(buf ^ 1);
+        __syncthreads();
+    }
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (p.splits > 1) {
+        const uint64_t ps = ((uint64_t)blockIdx.x * p.splits + blockIdx.y) * 16 * NW;
+        if (g == 0) {
+            p.part_ml[2 * ps + wave * 16 + c] = m;
+            p.part_ml[2 * ps + 16 * NW + wave * 16 + c] = l;
+        }
+        if (col < n_rows && k_lo < k_hi) {
+#pragma unroll
+            for (int t = 0; t < VT; ++t)
+                if ((uint32_t)t < 2 * rk) *(v4f *)(p.part_o + (ps + wave * 16 + c) * sh.rank_p + t * 16 + 4 * g) = o[t];
+        }
+        return;
+    }
+    if (col >= n_rows) return;
+    const float inv = 1.0f / l;
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+        if ((uint32_t)t < 2 * rk)
+            *(v2u *)(p.out + ((uint64_t)row0 * H + col) * sh.rank_p + t * 16 + 4 * g) =
+                v2u{f32x2_to_bf16x2(o[t][0] * inv, o[t][1] * inv), f32x2_to_bf16x2(o[t][2] * inv, o[t][3] * inv)};
+}
+
+// Adds the splits of a tile's columns: one block per (slot, column).
+template <int NW>
+__global__ void __launch_bounds__(128) latent_merge_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
+    uint32_t b, t0, n_rows;
+    if (!stream_tile<NW>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
+    const uint32_t cl = blockIdx.y, col = t0 + cl;
+    if (col >= n_rows) return;
+    const uint64_t ps = (uint64_t)blockIdx.x * p.splits * 16 * NW;
+    float m = -INFINITY, l = 0.0f;
+    for (uint32_t s = 0; s < p.splits; ++s) m = fmaxf(m, p.part_ml[2 * (ps + (uint64_t)s * 16 * NW) + cl]);
+    for (uint32_t s = 0; s < p.splits; ++s) {
+        const uint64_t at = 2 * (ps + (uint64_t)s * 16 * NW) + cl;
+        const float ls = p.part_ml[at + 16 * NW];    // 0: the split held none of the column's keys
+        if (ls != 0.0f) l += ls * exp2f(p.part_ml[at] - m);
+    }
+    const float inv = 1.0f / l;
+    for (uint32_t d = threadIdx.x * 4; d < sh.rank_p; d += 512) {
+        v4f a = v4f{0.f, 0.f, 0.f, 0.f};
+        for (uint32_t s = 0; s < p.splits; ++s) {
+            const uint64_t at = ps + (uint64_t)s * 16 * NW;
+            const float ms = p.part_ml[2 * at + cl];
+            if (p.part_ml[2 * at + 16 * NW + cl] != 0.0f) a += *(const v4f *)(p.part_o + (at + cl) * sh.rank_p + d) * exp2f(ms - m);
+        }
+        *(v2u *)(p.out + ((uint64_t)rr.row_start[b] * sh.heads + col) * sh.rank_p + d) =
+            v2u{f32x2_to_bf16x2(a[0] * inv, a[1] * inv), f32x2_to_bf16x2(a[2] * inv, a[3] * inv)};
+    }
+}
+
+struct StreamPlan {
+    int nw = 0;                                      // 0: the plain kernel
+    uint32_t slots = 0, splits = 1;
+};
+StreamPlan stream_plan(const LatentShape &sh, uint32_t rows, uint32_t batch, uint32_t longest, int num_cus) {
+    StreamPlan p;
+    if (sh.rank_p > 512 || sh.rot_p > 64 || g_latent_form == 1) return p;
+    p.nw = (uint64_t)longest * sh.heads <= 32 ? 2 : 4;
+    p.slots = (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nw)) + batch + 1;
+    // about one block per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NW)
+    const uint64_t used = std::max<uint64_t>(std::max<uint64_t>((uint64_t)rows * sh.heads / (16 * p.nw), batch), 1);
+    const uint64_t want = ((uint64_t)num_cus + used - 1) / used;
+    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (sh.window + 127) / 128, 64}));
+    return p;
+}
+
+template <int RK, int RO, int NW>
+void launch_stream(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, uint32_t slots, hipStream_t s) {
+    constexpr size_t lds = 2ull * kKeys * ((RK + RO) * 32 + 8) * 2;
+    if constexpr (lds > 65536) {
+        static bool configured = false;
+        if (!configured) {
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_stream_kernel<RK, RO, NW>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            configured = true;
+        }
+    }
+    latent_stream_kernel<RK, RO, NW><<<dim3(slots, p.splits), NW * 64, lds, s>>>(p, sh, rr);
+    if (p.splits > 1) latent_merge_kernel<NW><<<dim3(slots, 16 * NW), 128, 0, s>>>(p, sh, rr);
+}
+template <int RK, int RO>
+void launch_stream_nw(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, const StreamPlan &plan, hipStream_t s) {
+    if (plan.nw == 2) launch_stream<RK, RO, 2>(p, sh, rr, plan.slots, s);
+    else launch_stream<RK, RO, 4>(p, sh, rr, plan.slots, s);
+}
+template <int RK>
+void launch_stream_ro(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, const StreamPlan &plan, hipStream_t s) {
+    if (sh.rot_p <= 32) launch_stream_nw<RK, 1>(p, sh, rr, plan, s);
+    else launch_stream_nw<RK, 2>(p, sh, rr, plan, s);
+}
+
+// ------------------------------------------------------------------ expanded form
+// Prompts: the keys and values of every cached token the pass sees are formed per head (one linear), and attention runs per
+// head on them: per query and key 2 (dim + rot + vdim) operations instead of 2 (2 rank + rot).
+__global__ void __launch_bounds__(256)
+    latent_gather_kernel(const uint16_t *__restrict__ pool, uint16_t *__restrict__ c, uint32_t ld_c, uint16_t *__restrict__ kr, LatentShape sh,
+                         RaggedRows rr, LatentExpand ex) {
+    const uint32_t e = blockIdx.x * 4 + threadIdx.x / 64, lane = threadIdx.x % 64;
+    if (e >= ex.rows) return;
+    uint32_t lo = 0, hi = rr.batch;
+    while (hi - lo > 1) {
+        const uint32_t mid = (lo + hi) / 2;
+        if (ex.start[mid] <= e) lo = mid;
+        else hi = mid;
+    }
+    const uint32_t j = ex.first[lo] + (e - ex.start[lo]), width = sh.rank_p + sh.rot_p, blk = j / rr.block_size;
+    const uint32_t id = blk < rr.max_blocks ? rr.tables[(uint64_t)lo * rr.max_blocks + blk] : 0xffffffffu;
+    const bool ok = id < rr.num_blocks;
+    const uint16_t *src = pool + ((uint64_t)(ok ? id : 0) * rr.block_size + j % rr.block_size) * width;
+    for (uint32_t i = lane * 8; i < ld_c + sh.rot_p; i += 512) {
+        v4u v = ok ? v4u{0, 0, 0, 0} : v4u{0x7fc07fc0u, 0x7fc07fc0u, 0x7fc07fc0u, 0x7fc07fc0u};
+        if (i < ld_c) {
+            if (ok && i < sh.rank_p) v = *(const v4u *)(src + i);
+            *(v4u *)(c + (uint64_t)e * ld_c + i) = v;
+        } else {
+            if (ok) v = *(const v4u *)(src + sh.rank_p + (i - ld_c));
+            *(v4u *)(kr + (uint64_t)e * sh.rot_p + (i - ld_c)) = v;
+        }
+    }
+}
+
+// A block of four wavefronts takes 128 tokens of one (sequence, head), every wavefront 32 columns of S^T = K Q^T, and walks
+// the keys they see 32 at a time; K (unrotated | rotated) and V of a step are staged in LDS, two stages.  D: tiles of 32
+// that hold dim and vdim, RO: of the rotated part.
+template <int D, int RO>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2)))
+    latent_flash_kernel(const uint16_t *__restrict__ q, const uint16_t *__restrict__ kv, const uint16_t *__restrict__ kr,
+                        const float *__restrict__ gate, uint32_t ld_gate, uint16_t *__restrict__ out, uint32_t ld_out, LatentShape sh,
+                        RaggedRows rr, LatentExpand ex) {
+    constexpr int KS = D + RO, VT = 2 * D, KP = KS * 32 + 8, VP = D * 32 + 8, NQ = 2;
+    constexpr int PK = KS * 4 / 8, PV = D * 4 / 8;   // 16-byte pieces per thread and step (eight threads per key); KS even or padded below
+    constexpr int PKR = (KS * 4 + 7) / 8;
+    __shared__ __attribute__((aligned(16))) uint16_t ks[2][kKeys * KP], vs[2][kKeys * VP];
+    static_assert(PV * 8 == D * 4 && PK <= PKR, "eight threads stage a key");
+    // longest walks first: the last tiles of a sequence
+    uint32_t lo = 0, hi = rr.batch;
+    const uint32_t slots = gridDim.x, slot = slots - 1 - blockIdx.x;
+    while (hi - lo > 1) {
+        const uint32_t mid = (lo + hi) / 2;
+        if (rr.row_start[mid] / 128 + mid <= slot) lo = mid;
+        else hi = mid;
+    }
+    const uint32_t b = lo, row0 = rr.row_start[b], n = rr.row_start[b + 1] - row0, t0 = (slot - (row0 / 128 + b)) * 128;
+    if (t0 >= n) return;
+    const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), g = lane / 16, c = lane % 16;
+    const uint32_t h = blockIdx.y, H = sh.heads, qw = sh.dim_p + sh.rot_p, dk = sh.dim_p / 32, ro = sh.rot_p / 32, dv = (sh.vdim + 31) / 32;
+    const uint32_t hw = sh.dim_p + dv * 32;          // one head of an expanded row
+    const int32_t p0 = rr.pos[row0], W = (int32_t)sh.window, first = (int32_t)ex.first[b];
+    const uint32_t t_last = t0 + 127 < n ? t0 + 127 : n - 1;
+    int32_t k_lo = p0 + (int32_t)t0 - W + 1, k_hi = p0 + (int32_t)t_last + 1;
+    k_lo = k_lo > first ? k_lo : first;
+    const uint64_t e0 = (uint64_t)ex.start[b] - (uint64_t)first;     // expanded row of key j: e0 + j
+
+    v8bf qf[NQ][KS];
+    int32_t pos[NQ];
+#pragma unroll
+    for (int qi = 0; qi < NQ; ++qi) {
+        uint32_t t = t0 + wave * 32 + qi * 16 + c;
+        t = t < n ? t : n - 1;
+        pos[qi] = p0 + (int32_t)t;
+        const uint16_t *src = q + ((uint64_t)(row0 + t) * H + h) * qw + 8 * g;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) {
+            v4u v = v4u{0, 0, 0, 0};
+            if (s < D ? (uint32_t)s < dk : (uint32_t)(s - D) < ro) v = *(const v4u *)(src + (s < D ? s * 32 : sh.dim_p + (s - D) * 32));
+            qf[qi][s] = __builtin_bit_cast(v8bf, v);
+        }
+    }
+    const int32_t w_lo_pos = p0 + (int32_t)(t0 + wave * 32 < n ? t0 + wave * 32 : n - 1);
+    const int32_t w_hi_pos = p0 + (int32_t)(t0 + wave * 32 + 31 < n ? t0 + wave * 32 + 31 : n - 1);
+
+    const int key = tid / 8, part = tid % 8;
+    v4u sk[PKR], sv[PV];
+    auto fetch = [&](int32_t k0) {
+        const int32_t j = k0 + key;
+        const bool ok = j < k_hi;
+        const uint64_t e = e0 + (uint64_t)(ok ? j : k_hi - 1);
+        const uint16_t *row = kv + (e * H + h) * hw, *rot = kr + e * sh.rot_p;
+#pragma unroll
+        for (int i = 0; i < PKR; ++i) {
+            const int pc = part + 8 * i, s = pc / 4;
+            sk[i] = v4u{0, 0, 0, 0};
+            if (pc >= KS * 4) continue;
+            if (s < D) {
+                if ((uint32_t)s < dk) sk[i] = *(const v4u *)(row + pc * 8);
+            } else if ((uint32_t)(s - D) < ro) {
+                sk[i] = *(const v4u *)(rot + (pc - D * 4) * 8);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < PV; ++i) {
+            const int pc = part + 8 * i;
+            sv[i] = v4u{0, 0, 0, 0};
+            if ((uint32_t)(pc / 4) < dv) sv[i] = *(const v4u *)(row + sh.dim_p + pc * 8);
+        }
+    };
+    auto put = [&](int buf) {
+#pragma unroll
+        for (int i = 0; i < PKR; ++i)
+            if (part + 8 * i < KS * 4) *(v4u *)&ks[buf][key * KP + (part + 8 * i) * 8] = sk[i];
+#pragma unroll
+        for (int i = 0; i < PV; ++i) *(v4u *)&vs[buf][key * VP + (part + 8 * i) * 8] = sv[i];
+    };
+    float m[NQ], l[NQ];
+    v4f o[NQ][VT];
+#pragma unroll
+    for (int qi = 0; qi < NQ; ++qi) {
+        m[qi] = -INFINITY;
+        l[qi] = 0.0f;
+#pragma unroll
+        for (int t = 0; t < VT; ++t) o[qi][t] = v4f{0.f, 0.f, 0.f, 0.f};
+    }
+    fetch(k_lo);
+    put(0);
+    __syncthreads();
+    int buf = 0;
+    for (int32_t k0 = k_lo; k0 < k_hi; k0 += kKeys, buf ^= 1) {
+        const bool more = k0 + kKeys < k_hi;
+        if (more) fetch(k0 + kKeys);
+        if (k0 <= w_hi_pos && k0 + kKeys > w_lo_pos - W + 1) {       // some column of this wavefront sees some key of the step
+            const bool inside = k0 + kKeys - 1 <= w_lo_pos && k0 > w_hi_pos - W;       // every column sees every key
+            float sc[NQ][8];
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt) {
+                v4f acc[NQ];
+#pragma unroll
+                for (int qi = 0; qi < NQ; ++qi) acc[qi] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int s = 0; s < KS; ++s) {
+                    const v8bf kf = *(const v8bf *)&ks[buf][(kt * 16 + c) * KP + s * 32 + 8 * g];
+#pragma unroll
+                    for (int qi = 0; qi < NQ; ++qi) acc[qi] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[qi][s], acc[qi], 0, 0, 0);
+                }
+#pragma unroll
+                for (int qi = 0; qi < NQ; ++qi)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        float v = acc[qi][e] * (sh.scale * kLog2e);
+                        if (!inside) {
+                            const int32_t j = k0 + kt * 16 + 4 * g + e;
+                            if (j > pos[qi] || pos[qi] - j >= W) v = -INFINITY;
+                        }
+                        sc[qi][kt * 4 + e] = v;
+                    }
+            }
+            v8bf w_hi[NQ], w_lo[NQ];
+#pragma unroll
+            for (int qi = 0; qi < NQ; ++qi) {
+                const float fix = softmax_step(sc[qi], m[qi], l[qi], w_hi[qi], w_lo[qi]);
+                if (__any(fix != 1.0f)) {
+#pragma unroll
+                    for (int t = 0; t < VT; ++t) o[qi][t] *= fix;
+                }
+            }
+#pragma unroll
+            for (int t = 0; t < VT; ++t) {
+                const v8bf v = transposed_keys(&vs[buf][t * 16], VP, lane);
+#pragma unroll
+                for (int qi = 0; qi < NQ; ++qi) {
+                    o[qi][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_hi[qi], o[qi][t], 0, 0, 0);
+                    o[qi][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_lo[qi], o[qi][t], 0, 0, 0);
+                }
+            }
+        }
+        if (more) put(buf ^ 1);
+        __syncthreads();
+    }
+#pragma unroll
+    for (int qi = 0; qi < NQ; ++qi) {
+        float sum = l[qi];
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        const uint32_t t = t0 + wave * 32 + qi * 16 + c;
+        if (t >= n) continue;
+        const float f = 1.0f / (1.0f + expf(-gate[(uint64_t)(row0 + t) * ld_gate + h])) / sum;
+        uint16_t *dst = out + (uint64_t)(row0 + t) * ld_out + h * sh.vdim;
+        const bool vec = (sh.vdim & 3) == 0;
+#pragma unroll
+        for (int dt = 0; dt < VT; ++dt) {
+            const uint32_t d = dt * 16 + 4 * g;
+            if (vec && d < sh.vdim)
+                *(v2u *)(dst + d) = v2u{f32x2_to_bf16x2(o[qi][dt][0] * f, o[qi][dt][1] * f), f32x2_to_bf16x2(o[qi][dt][2] * f, o[qi][dt][3] * f)};
+            else if (!vec) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (d + e < sh.vdim) dst[d + e] = f32_to_bf16(o[qi][dt][e] * f);
+            }
+        }
+    }
+}
+
 }  // namespace
 
 void latent_prepare(const float *y, uint32_t ld, const float *q_norm, const float *kv_norm, const float *cos_sin, void *cq,
@@ -162,17 +628,53 @@ void latent_rotate_query(const void *q, const float *cos_sin, void *dst, uint32_
         latent_rotate_query_kernel<uint16_t><<<rows, 256, 0, s>>>((const uint16_t *)q, cos_sin, (uint16_t *)dst, dst_pitch, dst_off, sh);
 }
 
-uint64_t latent_attention_workspace_bytes(const LatentShape &sh, uint32_t rows, uint32_t batch) { return 0; }
+uint64_t latent_attention_workspace_bytes(const LatentShape &sh, int is_f32, uint32_t rows, uint32_t batch, uint32_t max_new, int num_cus) {
+    if (is_f32) return 0;
+    const StreamPlan p = stream_plan(sh, rows, batch, max_new, num_cus);
+    return p.splits > 1 ? (uint64_t)p.slots * p.splits * 16 * p.nw * (sh.rank_p + 2) * 4 : 0;
+}
 
 void latent_attention(const void *qa, const void *pool, void *out, int is_f32, const LatentShape &sh, const RaggedRows &rr,
                       uint32_t max_new, void *workspace, int num_cus, hipStream_t s) {
     if (rr.rows == 0) return;
+    if (!is_f32) {
+        const StreamPlan plan = stream_plan(sh, rr.rows, rr.batch, max_new, num_cus);
+        if (plan.nw) {
+            StreamParams p{(const uint16_t *)qa, (const uint16_t *)pool, (uint16_t *)out, (float *)workspace, nullptr, plan.splits};
+            if (p.splits > 1) p.part_ml = p.part_o + (uint64_t)plan.slots * plan.splits * 16 * plan.nw * sh.rank_p;
+            if (sh.rank_p <= 64) launch_stream_ro<2>(p, sh, rr, plan, s);
+            else if (sh.rank_p <= 128) launch_stream_ro<4>(p, sh, rr, plan, s);
+            else if (sh.rank_p <= 256) launch_stream_ro<8>(p, sh, rr, plan, s);
+            else launch_stream_ro<16>(p, sh, rr, plan, s);
+            return;
+        }
+    }
     const dim3 grid(rr.rows, sh.heads);
     const size_t lds = (size_t)(sh.rank_p + sh.rot_p) * 4;
     if (is_f32)
         latent_attention_plain_kernel<float><<<grid, 256, lds, s>>>((const float *)qa, (const float *)pool, (float *)out, sh, rr);
     else
         latent_attention_plain_kernel<uint16_t><<<grid, 256, lds, s>>>((const uint16_t *)qa, (const uint16_t *)pool, (uint16_t *)out, sh, rr);
+}
+
+bool latent_expand_applies(const LatentShape &sh) { return sh.dim_p <= 128 && sh.vdim <= 128 && sh.rot_p <= 64 && g_latent_form != 1 && g_latent_form != 2; }
+bool latent_expand_always() { return g_latent_form == 3; }
+
+void latent_gather(const void *pool, void *c, uint32_t ld_c, void *kr, const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s) {
+    if (ex.rows == 0) return;
+    latent_gather_kernel<<<(ex.rows + 3) / 4, 256, 0, s>>>((const uint16_t *)pool, (uint16_t *)c, ld_c, (uint16_t *)kr, sh, rr, ex);
+}
+
+void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, void *out, uint32_t ld_out,
+                               const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s) {
+    const dim3 grid(rr.rows / 128 + rr.batch + 1, sh.heads);
+    const bool wide = sh.dim_p > 64 || sh.vdim > 64, rot2 = sh.rot_p > 32;
+#define FA_FLASH(D_, RO_)                                                                                                                    \
+    latent_flash_kernel<D_, RO_><<<grid, 256, 0, s>>>((const uint16_t *)q, (const uint16_t *)kv, (const uint16_t *)kr, gate, ld_gate, (uint16_t *)out, \
+                                                      ld_out, sh, rr, ex)
+    if (wide) rot2 ? FA_FLASH(4, 2) : FA_FLASH(4, 1);
+    else rot2 ? FA_FLASH(2, 2) : FA_FLASH(2, 1);
+#undef FA_FLASH
 }
 
 }  // namespace k

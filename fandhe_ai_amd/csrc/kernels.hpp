@@ -402,10 +402,24 @@ void latent_prepare(const float *y, uint32_t ld, const float *q_norm, const floa
 void latent_rotate_query(const void *q, const float *cos_sin, void *dst, uint32_t dst_pitch, uint32_t dst_off, int is_f32,
                          const LatentShape &sh, uint32_t rows, hipStream_t s);
 // Attention of absorbed queries qa [rows, heads, rank_p + rot_p] over cached rows: out [rows, heads, rank_p] = softmax-weighted
-// latents.  bf16 with sizes the matrix-core kernel holds: that kernel (workspace for the key splits); otherwise a plain one.
-uint64_t latent_attention_workspace_bytes(const LatentShape &sh, uint32_t rows, uint32_t batch);
+// latents.  bf16 with kv_rank <= 512 and rot <= 64: the matrix-core kernel (workspace for the key splits); otherwise a
+// plain one.  max_new: most new tokens of any sequence.
+uint64_t latent_attention_workspace_bytes(const LatentShape &sh, int is_f32, uint32_t rows, uint32_t batch, uint32_t max_new, int num_cus);
 void latent_attention(const void *qa, const void *pool, void *out, int is_f32, const LatentShape &sh, const RaggedRows &rr,
                       uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
+// The form for prompts (bf16, dim, vdim <= 128, rot <= 64): the keys first[b] .. of every sequence are gathered as rows
+// start[b] .. start[b + 1] - 1 (latents c [rows, ld_c], rotated parts kr [rows, rot_p]), a linear turns the latents into
+// kv [rows, heads, dim_p + vdim padded to 32], and attention runs per head on those; q is [rows, heads, dim_p + rot_p] with its
+// rotated part rotated; the heads' gates (sigmoid) are applied, out [rows, ld_out].
+struct LatentExpand {
+    const uint32_t *start, *first;   // [batch + 1], [batch]
+    uint32_t rows;
+};
+bool latent_expand_applies(const LatentShape &sh);
+bool latent_expand_always();         // tuning: wherever it applies, whatever it costs
+void latent_gather(const void *pool, void *c, uint32_t ld_c, void *kr, const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s);
+void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, void *out, uint32_t ld_out,
+                               const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s);
 
 // ---- gated delta rule (kern_delta.hip) --------------------------------------------
 struct DeltaShape {

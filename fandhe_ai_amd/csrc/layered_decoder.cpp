@@ -35,7 +35,8 @@ struct Layer {
     k::LinearWeight in, out, gate_up, down;
     // latent attention
     k::LatentShape la{};
-    k::LinearWeight uq, uk, uv;
+    k::LinearWeight uq, uk, uv, ukv;                  // ukv: keys and values of all heads from the latent (expanded form)
+    uint32_t window_index = 0;
     float *q_norm = nullptr, *kv_norm = nullptr;
     void *pool = nullptr;
     uint32_t rotation = 0;                            // index of its cos / sin table
@@ -56,6 +57,15 @@ struct Arena {
     uint32_t *row_seq = nullptr, *kv_slot = nullptr, *row_start = nullptr;
     int32_t *pos = nullptr, *tokens = nullptr, *want = nullptr;
     std::vector<float *> cos_sin;
+    // expanded latent attention: latents, rotated parts, keys and values of up to `expand_rows` cached tokens
+    uint32_t expand_rows = 0;
+    void *ec = nullptr, *er = nullptr, *ekv = nullptr;
+    uint32_t *expand_meta = nullptr;                 // per distinct window: start [batch + 1], first [batch]
+};
+
+// Which cached tokens a pass expands, per distinct window; rows 0: the absorbed form is cheaper
+struct ExpandPlan {
+    std::vector<uint32_t> rows, meta;
 };
 
 }  // namespace
@@ -67,6 +77,7 @@ struct LayeredState {
     std::vector<Tensor> tensors;
     std::vector<fa_buffer *> owned;
     std::vector<std::pair<uint32_t, double>> rotations;      // distinct (dims, base)
+    std::vector<uint32_t> windows;                           // distinct windows
     void *embed = nullptr;
     float *final_norm = nullptr;
     k::LinearWeight head;
@@ -107,8 +118,10 @@ Widths widths(const LayeredState &L) {
     return w;
 }
 
-fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t rows) {
-    if (a.rows >= rows) return FA_OK;
+fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t rows, uint32_t expand_rows = 0) {
+    if (a.rows >= rows && a.expand_rows >= expand_rows) return FA_OK;
+    rows = std::max(rows, a.rows);
+    expand_rows = std::max(expand_rows, a.expand_rows);
     if (ctx->capturing) return fail(FA_ERR_CAPTURE_IN_PROGRESS, "layered decoder: activations must be sized before a capture");
     if (a.base) pool_free(ctx, a.base, a.bytes, a.cls);
     a = Arena();
@@ -144,12 +157,25 @@ fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t row
     for (const Layer &l : L.layers)
         if (l.cfg.mixer == FA_MIXER_DELTA) scratch = std::max(scratch, k::delta_scratch_bytes(l.de, rows, (uint32_t)B));
     add((void **)&a.delta_scratch, scratch);
+    uint64_t ec = 0, er = 0, ekv = 0;
+    for (const Layer &l : L.layers)
+        if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) {
+            ec = std::max<uint64_t>(ec, pad_to(l.la.rank_p, 64));
+            er = std::max<uint64_t>(er, l.la.rot_p);
+            ekv = std::max<uint64_t>(ekv, (uint64_t)l.la.heads * (l.la.dim_p + pad_to(l.la.vdim, 32)));
+        }
+    if (L.is_f32) expand_rows = 0;
+    add(&a.ec, expand_rows * ec * E);
+    add(&a.er, expand_rows * er * E);
+    add(&a.ekv, expand_rows * ekv * E);
+    add((void **)&a.expand_meta, L.windows.size() * (2 * B + 1) * 4);
     if (fa_status s = pool_alloc(ctx, total, &a.base, &a.cls)) {
         a = Arena();
         return s;
     }
     a.bytes = total;
     a.rows = rows;
+    a.expand_rows = expand_rows;
     for (auto &p : parts) *p.first = (uint8_t *)a.base + p.second;
     k::fill_u32((uint32_t *)a.base, 0, total / 4, ctx->stream);
     return after_launch(ctx, "layered decoder activations");
@@ -170,7 +196,8 @@ k::LinearEpilogue store_to(void *out, uint64_t ld, int out_f32) {
 }
 
 // All layers over the rows of a pass whose embeddings are in a.x.
-fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::RaggedRows &rr, uint32_t max_new, uint64_t trace_row0) {
+fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::RaggedRows &rr, uint32_t max_new, uint64_t trace_row0,
+                         const ExpandPlan *expand = nullptr) {
     LayeredState &L = *d->layered;
     hipStream_t s = ctx->stream;
     const uint32_t M = rr.rows, D = L.cfg.d_model, ld_hn = pad_to(D, 64);
@@ -199,17 +226,28 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
             linear(ctx, L, a.hn, ld_hn, 0, M, l.in, store_to(a.y32, ld_y, 1));
             k::latent_prepare(a.y32, ld_y, l.q_norm, l.kv_norm, cs, a.cq, ld_cq, own ? pool : nullptr, f32, sh, rr, s);
             linear(ctx, L, a.cq, ld_cq, 0, M, l.uq, store_to(a.q, (uint64_t)sh.heads * qw, f32));
-            k::LinearEpilogue e = store_to(a.qa, (uint64_t)sh.heads * kw, f32);
-            e.out_batch = kw;
-            linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, l.uk, e);
-            k::latent_rotate_query(a.q, cs, a.qa, kw, sh.rank_p, f32, sh, M, s);
-            k::latent_attention(a.qa, pool, a.olat, f32, sh, rr, max_new, ctx->workspace, ctx->props.multiProcessorCount, s);
-            e = store_to(a.o, ld_o, f32);
-            e.mode = k::LinearEpilogue::kHeadGate;
-            e.out_batch = sh.vdim;
-            e.gate = a.y32 + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
-            e.ld_gate = ld_y;
-            linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, l.uv, e);
+            const float *gate = a.y32 + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
+            if (expand && expand->rows[l.window_index]) {
+                const uint32_t *meta = a.expand_meta + (uint64_t)l.window_index * (2 * d->cfg.max_batch + 1);
+                const k::LatentExpand ex{meta, meta + d->cfg.max_batch + 1, expand->rows[l.window_index]};
+                const uint32_t ld_c = pad_to(sh.rank_p, 64);
+                k::latent_rotate_query(a.q, cs, a.q, qw, sh.dim_p, f32, sh, M, s);
+                k::latent_gather(pool, a.ec, ld_c, a.er, sh, rr, ex, s);
+                linear(ctx, L, a.ec, ld_c, 0, ex.rows, l.ukv, store_to(a.ekv, l.ukv.n, f32));
+                k::latent_attention_expanded(a.q, a.ekv, a.er, gate, ld_y, a.o, ld_o, sh, rr, ex, s);
+            } else {
+                k::LinearEpilogue e = store_to(a.qa, (uint64_t)sh.heads * kw, f32);
+                e.out_batch = kw;
+                linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, l.uk, e);
+                k::latent_rotate_query(a.q, cs, a.qa, kw, sh.rank_p, f32, sh, M, s);
+                k::latent_attention(a.qa, pool, a.olat, f32, sh, rr, max_new, ctx->workspace, ctx->props.multiProcessorCount, s);
+                e = store_to(a.o, ld_o, f32);
+                e.mode = k::LinearEpilogue::kHeadGate;
+                e.out_batch = sh.vdim;
+                e.gate = gate;
+                e.ld_gate = ld_y;
+                linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, l.uv, e);
+            }
         }
         k::LinearEpilogue r = store_to(a.x, D, 1);
         r.mode = k::LinearEpilogue::kResidual;
@@ -258,11 +296,51 @@ void prepare_rows(fa_context *ctx, fa_decoder *d, Arena &a, const uint32_t *row_
     k::ragged_advance(row_start, (uint32_t *)d->seq_lens->ptr, d->batch, ctx->stream);
 }
 
-fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch) {
+fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch, uint32_t max_new) {
     uint64_t need = 0;
     for (const Layer &l : L.layers)
-        if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) need = std::max(need, k::latent_attention_workspace_bytes(l.la, rows, batch));
+        if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION)
+            need = std::max(need, k::latent_attention_workspace_bytes(l.la, L.is_f32, rows, batch, max_new, ctx->props.multiProcessorCount));
     return need ? ensure_workspace(ctx, need) : FA_OK;
+}
+
+// The expanded form of a pass, per distinct window: sequence b (lens[b] cached tokens, n[b] new ones) needs the keys its
+// first new token sees onwards.  It is taken where forming keys and values per head costs less than attending over
+// latents, counted in multiply-adds per head.
+ExpandPlan plan_expand(const LayeredState &L, const std::vector<uint32_t> &lens, const std::vector<uint32_t> &n, uint32_t max_batch) {
+    constexpr uint64_t kMaxRows = 1u << 16;
+    ExpandPlan p;
+    p.rows.assign(L.windows.size(), 0);
+    p.meta.assign(L.windows.size() * (2 * (size_t)max_batch + 1), 0);
+    if (L.is_f32) return p;
+    for (size_t w = 0; w < L.windows.size(); ++w) {
+        const Layer *l = nullptr;
+        bool ok = true;
+        for (const Layer &c : L.layers)
+            if (c.cfg.mixer == FA_MIXER_LATENT_ATTENTION && c.window_index == w) {
+                ok = ok && k::latent_expand_applies(c.la);
+                l = &c;
+            }
+        if (!l || !ok) continue;
+        const uint64_t W = L.windows[w];
+        uint64_t rows = 0, fresh = 0;
+        double pairs = 0;
+        uint32_t *start = p.meta.data() + w * (2 * (size_t)max_batch + 1), *first = start + max_batch + 1;
+        for (size_t b = 0; b < n.size(); ++b) {
+            start[b] = (uint32_t)rows;
+            first[b] = lens[b] + 1 > W ? (uint32_t)(lens[b] + 1 - W) : 0;
+            if (n[b] == 0) continue;
+            rows += (uint64_t)lens[b] + n[b] - first[b];
+            fresh += n[b];
+            pairs += (double)n[b] * (double)std::min<uint64_t>(W, lens[b] + (n[b] + 1) / 2);
+        }
+        for (size_t b = n.size(); b <= max_batch; ++b) start[b] = (uint32_t)rows;
+        const double up = (double)l->la.kv_rank * (l->la.dim + l->la.vdim);
+        const double expanded = rows * up + pairs * (l->la.dim + l->la.rot + l->la.vdim);
+        const double absorbed = fresh * up + pairs * (2.0 * l->la.kv_rank + l->la.rot);
+        if (rows <= kMaxRows && (k::latent_expand_always() || (expanded < absorbed && fresh >= 128))) p.rows[w] = (uint32_t)rows;
+    }
+    return p;
 }
 
 uint64_t pass_rows() { return g_layered_rows >= 64 ? (uint64_t)g_layered_rows : 8192; }
@@ -305,7 +383,7 @@ fa_status layered_sequences_set(fa_context *ctx, fa_decoder *d) {
 fa_status layered_prepare_step(fa_context *ctx, fa_decoder *d) {
     LayeredState &L = *d->layered;
     if (fa_status s = arena_reserve(ctx, L, L.step, L.cfg.max_batch)) return s;
-    return attention_workspace(ctx, L, d->batch, d->batch);
+    return attention_workspace(ctx, L, d->batch, d->batch, 1);
 }
 
 fa_status layered_enqueue_step(fa_context *ctx, fa_decoder *d) {
@@ -354,7 +432,6 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
     while (cap < std::min<uint64_t>(total, budget)) cap *= 2;
     if (fa_status s = arena_reserve(ctx, L, L.pass, cap)) return s;
     Arena &a = L.pass;
-    if (fa_status s = attention_workspace(ctx, L, (uint32_t)std::min<uint64_t>(total, budget), B)) return s;
     // logits of wanted rows: at most kHeadRows at a time
     constexpr uint32_t kHeadRows = 1024;
     fa_buffer *lbuf = nullptr, *pbuf = nullptr;
@@ -368,7 +445,7 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
             }
     }
     auto run = [&]() -> fa_status {
-        std::vector<uint32_t> done(B, 0), starts(B + 1), first(B);
+        std::vector<uint32_t> done(B, 0), starts(B + 1), first(B), fresh(B);
         std::vector<int32_t> stage, pick_rows;
         uint64_t w_at = 0, placed = 0, tok0 = 0;
         for (uint32_t b = 0; b < B; ++b) {
@@ -395,11 +472,22 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
                 if (done[b] == counts[b]) last[b] = (int32_t)rows - 1;
             }
             starts[B] = rows;
+            for (uint32_t b = 0; b < B; ++b) fresh[b] = starts[b + 1] - starts[b];
+            const ExpandPlan expand = plan_expand(L, d->host_lens, fresh, c.max_batch);
+            uint32_t e_rows = 0;
+            for (uint32_t r : expand.rows) e_rows = std::max(e_rows, r);
+            if (e_rows) {
+                uint32_t e_cap = 256;
+                while (e_cap < e_rows) e_cap *= 2;
+                if (fa_status s = arena_reserve(ctx, L, a, a.rows, e_cap)) return s;
+                if (fa_status s = upload(ctx, a.expand_meta, expand.meta.data(), expand.meta.size() * 4)) return s;
+            }
+            if (fa_status s = attention_workspace(ctx, L, rows, B, max_new)) return s;
             if (fa_status s = upload(ctx, a.row_start, starts.data(), (B + 1) * 4)) return s;
             if (fa_status s = upload(ctx, a.tokens, stage.data(), (uint64_t)rows * 4)) return s;
             prepare_rows(ctx, d, a, a.row_start, rows);
             k::gather_rows_any(L.embed, L.is_f32, c.vocab, c.d_model, a.tokens, a.x, rows, ctx->stream);
-            if (fa_status s = enqueue_layers(ctx, d, a, ragged(d, a, a.row_start, rows), max_new, placed)) return s;
+            if (fa_status s = enqueue_layers(ctx, d, a, ragged(d, a, a.row_start, rows), max_new, placed, &expand)) return s;
             for (uint32_t b = 0; b < B; ++b) d->host_lens[b] += starts[b + 1] - starts[b];
             placed += rows;
             if (last_only) {
@@ -655,6 +743,9 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 }
                 // per head, latent = W_uk^T q: the key projection transposed
                 const uint32_t kr = g.kv_rank, vd = g.vdim;
+                const uint32_t hw = dim_p + pad_to(vd, 32);
+                if (!f32) l.ukv = weight(H * hw, H * hw, kr);
+                const k::LinearWeight both = l.ukv;
                 l.uk = weight(a.rank_p, a.rank_p, dim, H);
                 {
                     const k::LinearWeight w = l.uk;
@@ -662,6 +753,7 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                     add(m + "uk", (uint64_t)H * dim, kr, [=](const void *src, int sf, hipStream_t s) {
                         for (uint32_t h = 0; h < H; ++h)
                             k::pack_linear(row_ptr(src, sf, (uint64_t)h * dim * kr), sf, 1, kr, kr, dim, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
+                        if (both.w) k::pack_linear(src, sf, kr, 1, H * dim, kr, (void *)both.w, f32, both.k_tiles, 0, dim, hw, s);
                     });
                 }
                 l.uv = weight(vd, vd, kr, H);
@@ -671,8 +763,11 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                     add(m + "uv", (uint64_t)H * vd, kr, [=](const void *src, int sf, hipStream_t s) {
                         for (uint32_t h = 0; h < H; ++h)
                             k::pack_linear(row_ptr(src, sf, (uint64_t)h * vd * kr), sf, kr, 1, vd, kr, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
+                        if (both.w) k::pack_linear(src, sf, kr, 1, H * vd, kr, (void *)both.w, f32, both.k_tiles, dim_p, vd, hw, s);
                     });
                 }
+                l.window_index = (uint32_t)(std::find(L->windows.begin(), L->windows.end(), g.window) - L->windows.begin());
+                if (l.window_index == L->windows.size()) L->windows.push_back(g.window);
                 const std::pair<uint32_t, double> r(g.rot_dim, g.rot_base);
                 l.rotation = (uint32_t)(std::find(L->rotations.begin(), L->rotations.end(), r) - L->rotations.begin());
                 if (l.rotation == L->rotations.size()) L->rotations.push_back(r);
