@@ -51,7 +51,9 @@ __device__ __forceinline__ float conv_silu(const T *__restrict__ y, uint32_t ld,
 // ------------------------------------------------------------------ token by token
 // One block per (sequence, head); the state sits in registers (thread: four neighbouring columns of up to RPT rows) from
 // the first token of the pass to the last.  CG = column groups of four, a power of two.
-template <typename T, int NT, int RPT>
+// FAST (single tokens, at most four taps, no more than 2 NT channels): the inputs of the convolution are requested ahead of
+// the state, so that the convolution runs while the state travels.
+template <typename T, int NT, int RPT, bool FAST>
 __global__ void __launch_bounds__(NT)
     delta_step_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, uint32_t cg_log2, int write_ring, uint32_t max_tokens) {
     constexpr int NW = NT / 64;
@@ -70,24 +72,53 @@ __global__ void __launch_bounds__(NT)
     float *state = io.state + ((uint64_t)rr.state_slot[b] * sh.heads + h) * dim * vp;
     const bool col_ok = cg * 4 < vp;
     const uint32_t p0 = (uint32_t)rr.pos[row0];
+    auto channel = [&](uint32_t i) { return i < dim ? hk * dim + i : i < 2 * dim ? (sh.kv_heads + hk) * dim + (i - dim) : 2 * sh.kv_heads * dim + h * vdim + (i - 2 * dim); };
+    float xin[2][4], win[2][4];
+    if constexpr (FAST) {
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+            const uint32_t i = threadIdx.x + q * NT;
+#pragma unroll
+            for (uint32_t back = 0; back < 4; ++back) {
+                xin[q][back] = win[q][back] = 0.0f;
+                if (i < 2 * dim + vdim && back < sh.taps && back <= p0) {
+                    const uint32_t c = channel(i);
+                    xin[q][back] = load_as_f32(back == 0 ? y + (uint64_t)row0 * io.ld_y + c : ring + (uint64_t)((p0 - back) % sh.taps) * channels + c);
+                    win[q][back] = io.conv[(uint64_t)c * sh.taps + sh.taps - 1 - back];
+                }
+            }
+        }
+        __builtin_amdgcn_sched_barrier(0);
+    }
     v4f S[RPT];
 #pragma unroll
     for (int i = 0; i < RPT; ++i) {
         const uint32_t d = rg + i * RG;
         S[i] = v4f{0.f, 0.f, 0.f, 0.f};
-        if (p0 != 0 && col_ok && d < dim) S[i] = *(const v4f *)(state + (uint64_t)d * vp + cg * 4);
+        if (p0 != 0 && col_ok && d < dim) S[i] = stream_load<true>((const v4f *)(state + (uint64_t)d * vp + cg * 4));
     }
+    __builtin_amdgcn_sched_barrier(0);
     const float a_log = io.a_log[h], dt_bias = io.dt_bias[h];
     for (uint32_t t = 0; t < n_tok; ++t) {
         const uint64_t row = row0 + t;
         const uint32_t p = p0 + t;
         // q, k, v of this head behind the convolution
         float sq = 0.0f, sk = 0.0f;
-        for (uint32_t i = threadIdx.x; i < 2 * dim + CG * 4; i += NT) {
+#pragma unroll
+        for (uint32_t q = 0; q < (FAST ? 2u : 0x40000000u); ++q) {
+            const uint32_t i = threadIdx.x + q * NT;
+            if (i >= 2 * dim + CG * 4) break;
             float v = 0.0f;
             if (i < 2 * dim + vdim) {
-                const uint32_t c = i < dim ? hk * dim + i : i < 2 * dim ? (sh.kv_heads + hk) * dim + (i - dim) : 2 * sh.kv_heads * dim + h * vdim + (i - 2 * dim);
-                v = conv_silu(y, io.ld_y, ring, io.conv, sh.taps, channels, c, row0, t, p);
+                const uint32_t c = channel(i);
+                if constexpr (FAST) {
+                    float acc = 0.0f;
+#pragma unroll
+                    for (int back = 3; back >= 0; --back) acc = fmaf(win[q][back], xin[q][back], acc);
+                    v = silu_f32(acc);
+                } else {
+                    v = conv_silu(y, io.ld_y, ring, io.conv, sh.taps, channels, c, row0, t, p);
+                }
                 if (write_ring && (i >= 2 * dim || h % share == 0)) ring[(uint64_t)(p % sh.taps) * channels + c] = y[row * io.ld_y + c];
             }
             (i < dim ? lq[i] : i < 2 * dim ? lk[i - dim] : lv[i - 2 * dim]) = v;
@@ -125,6 +156,7 @@ __global__ void __launch_bounds__(NT)
         for (int i = 0; i < RPT; ++i) {
             const uint32_t d = rg + i * RG;
             if (d < dim) S[i] += u * (lk[d] * rk);
+            if (t + 1 == n_tok && col_ok && d < dim) __builtin_nontemporal_store(S[i], (v4f *)(state + (uint64_t)d * vp + cg * 4));
         }
         const v4f o = dq + u * kq;
         float so = 0.0f;
@@ -145,11 +177,6 @@ __global__ void __launch_bounds__(NT)
             }
         }
         __syncthreads();                             // q, k, v and the partial sums are overwritten by the next token
-    }
-#pragma unroll
-    for (int i = 0; i < RPT; ++i) {
-        const uint32_t d = rg + i * RG;
-        if (col_ok && d < dim) *(v4f *)(state + (uint64_t)d * vp + cg * 4) = S[i];
     }
 }
 
@@ -554,10 +581,16 @@ void launch_step(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr, 
     const uint32_t rg = NT >> cg_log2, rpt = (sh.dim + rg - 1) / rg;
     const size_t lds = (2 * ((sh.dim + 3) / 4 * 4) + (4u << cg_log2) + 2 * NT * 4) * 4;
     const dim3 grid(rr.batch, sh.heads);
-    if (rpt <= 8) delta_step_kernel<T, NT, 8><<<grid, NT, lds, s>>>(sh, io, rr, cg_log2, write_ring, max_tokens);
-    else if (rpt <= 16) delta_step_kernel<T, NT, 16><<<grid, NT, lds, s>>>(sh, io, rr, cg_log2, write_ring, max_tokens);
-    else if (rpt <= 32) delta_step_kernel<T, NT, 32><<<grid, NT, lds, s>>>(sh, io, rr, cg_log2, write_ring, max_tokens);
-    else delta_step_kernel<T, NT, 64><<<grid, NT, lds, s>>>(sh, io, rr, cg_log2, write_ring, max_tokens);
+    // FAST's channels fit two per thread by the caller's check
+#define FA_STEP(R_)                                                                                                   \
+    fast ? delta_step_kernel<T, NT, R_, true><<<grid, NT, lds, s>>>(sh, io, rr, cg_log2, write_ring, max_tokens)       \
+         : delta_step_kernel<T, NT, R_, false><<<grid, NT, lds, s>>>(sh, io, rr, cg_log2, write_ring, max_tokens)
+    const bool fast = max_tokens == 1 && sh.taps <= 4 && 2 * sh.dim + (4u << cg_log2) <= 2 * NT;
+    if (rpt <= 8) FA_STEP(8);
+    else if (rpt <= 16) FA_STEP(16);
+    else if (rpt <= 32) FA_STEP(32);
+    else FA_STEP(64);
+#undef FA_STEP
 }
 
 template <typename T>

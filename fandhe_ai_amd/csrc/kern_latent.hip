@@ -377,9 +377,9 @@ StreamPlan stream_plan(const LatentShape &sh, uint32_t rows, uint32_t batch, uin
     if (sh.rank_p > 512 || sh.rot_p > 64 || g_latent_form == 1) return p;
     p.nw = (uint64_t)longest * sh.heads <= 32 ? 2 : 4;
     p.slots = (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nw)) + batch + 1;
-    // about one block per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NW)
+    // about two blocks per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NW)
     const uint64_t used = std::max<uint64_t>(std::max<uint64_t>((uint64_t)rows * sh.heads / (16 * p.nw), batch), 1);
-    const uint64_t want = ((uint64_t)num_cus + used - 1) / used;
+    const uint64_t want = (2 * (uint64_t)num_cus + used - 1) / used;
     p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (sh.window + 127) / 128, 64}));
     return p;
 }

@@ -13,7 +13,7 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
-int g_linear_form = 0;        // tuning: 2 keeps the large-tile kernel out
+int g_linear_form = 0;        // tuning: 2 keeps the large-tile kernel out, 3 four column tiles per block
 
 namespace {
 
@@ -24,8 +24,8 @@ template <int MT, int NTW, int NWAVES, int MODE>
 __global__ void __launch_bounds__(NWAVES * 64)
     linear_rows_kernel(const uint16_t *__restrict__ a, uint64_t lda, uint64_t a_batch, const uint8_t *__restrict__ w, uint32_t m,
                        uint32_t n, uint32_t n_tiles, uint32_t k_tiles, LinearEpilogue ep) {
-    static_assert(MODE != LinearEpilogue::kGlu || NTW == 2, "gate and up are neighbouring tiles");
-    constexpr int NT = MT * NTW, D = (MT + NTW >= 5) ? 4 : 8;
+    static_assert(MODE != LinearEpilogue::kGlu || NTW % 2 == 0, "gate and up are neighbouring tiles");
+    constexpr int NT = MT * NTW, D = NTW == 4 || MT == 4 ? 4 : 8;
     __shared__ v4f red[NWAVES][NT][64];
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
     const uint32_t nt0 = blockIdx.x * NTW, batch = blockIdx.y;
@@ -269,10 +269,15 @@ void launch_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
         const int mt = (int)((m + 15) / 16);
         // two tiles per block once one tile each would fill the device twice over
         const bool two = GLU || (uint64_t)w.n_tiles * w.batches >= 2 * (uint64_t)num_cus;
-        const dim3 grid(two ? (w.n_tiles + 1) / 2 : w.n_tiles, w.batches);
+        // wide weights, up to 32 rows: four, so that the activations cross the L2 half as often
+        const bool four = mt <= 2 && g_linear_form != 3 && w.batches == 1 && w.n_tiles >= 3 * (uint64_t)num_cus;
+        const dim3 grid(four ? (w.n_tiles + 3) / 4 : two ? (w.n_tiles + 1) / 2 : w.n_tiles, w.batches);
 #define FA_ROWS(MT_, NTW_)                                                                                             \
     linear_rows_kernel<MT_, NTW_, 8, MODE><<<grid, 512, 0, s>>>(a, lda, a_batch, wt, (uint32_t)m, w.n, w.n_tiles, w.k_tiles, ep)
-        if constexpr (GLU) {
+        if (four) {
+            if (mt == 1) FA_ROWS(1, 4);
+            else FA_ROWS(2, 4);
+        } else if constexpr (GLU) {
             if (mt == 1) FA_ROWS(1, 2);
             else if (mt == 2) FA_ROWS(2, 2);
             else FA_ROWS(4, 2);

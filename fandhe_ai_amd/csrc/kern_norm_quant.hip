@@ -46,30 +46,30 @@ __global__ void __launch_bounds__(kBlock) rmsnorm_kernel(const float *__restrict
 
 // Layer norm with a weight and no bias: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, two passes over the row held in
 // registers (VPT values per thread).
-template <int VPT, bool OUT_F32>
-__global__ void __launch_bounds__(kBlock)
+template <int VPT, bool OUT_F32, int NT = kBlock>
+__global__ void __launch_bounds__(NT)
     layernorm_kernel(const float *__restrict__ x, const float *__restrict__ w, void *__restrict__ out, uint32_t hidden, uint64_t ld,
                      float eps) {
-    __shared__ float smem[kWaves];
+    __shared__ float smem[NT / kWave];
     const float *row = x + (uint64_t)blockIdx.x * hidden;
     float v[VPT], sum = 0.0f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const uint32_t c = threadIdx.x + i * kBlock;
+        const uint32_t c = threadIdx.x + i * NT;
         v[i] = c < hidden ? row[c] : 0.0f;
         sum += v[i];
     }
-    const float mean = block_sum<float, kWaves, true>(sum, smem) / (float)hidden;
+    const float mean = block_sum<float, NT / kWave, true>(sum, smem) / (float)hidden;
     float sq = 0.0f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const float c = threadIdx.x + i * kBlock < hidden ? v[i] - mean : 0.0f;
+        const float c = threadIdx.x + i * NT < hidden ? v[i] - mean : 0.0f;
         sq = fmaf(c, c, sq);
     }
-    const float rstd = 1.0f / sqrtf(block_sum<float, kWaves, true>(sq, smem) / (float)hidden + eps);
+    const float rstd = 1.0f / sqrtf(block_sum<float, NT / kWave, true>(sq, smem) / (float)hidden + eps);
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const uint32_t c = threadIdx.x + i * kBlock;
+        const uint32_t c = threadIdx.x + i * NT;
         if (c >= ld) continue;
         const float y = c < hidden ? (v[i] - mean) * rstd * w[c] : 0.0f;
         if (OUT_F32) ((float *)out)[blockIdx.x * ld + c] = y;
@@ -578,6 +578,11 @@ void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint
                     hipStream_t s) {
     if (rows == 0) return;
     const uint64_t vpt = (ld + kBlock - 1) / kBlock;
+    if (rows <= 256 && ld > 1024 && ld <= 8192) {        // few rows: the row spread over 1024 threads
+        if (out_f32) layernorm_kernel<8, true, 1024><<<(unsigned)rows, 1024, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps);
+        else layernorm_kernel<8, false, 1024><<<(unsigned)rows, 1024, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps);
+        return;
+    }
 #define FA_LN(V)                                                                                                              \
     out_f32 ? layernorm_kernel<V, true><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)                \
             : layernorm_kernel<V, false><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)
