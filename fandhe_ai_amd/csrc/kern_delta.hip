@@ -104,7 +104,7 @@ __global__ void __launch_bounds__(NT)
         const uint32_t p = p0 + t;
         // q, k, v of this head behind the convolution
         float sq = 0.0f, sk = 0.0f;
-#pragma unroll
+#pragma unroll FAST ? 2 : 1
         for (uint32_t q = 0; q < (FAST ? 2u : 0x40000000u); ++q) {
             const uint32_t i = threadIdx.x + q * NT;
             if (i >= 2 * dim + CG * 4) break;

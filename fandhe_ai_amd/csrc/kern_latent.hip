@@ -11,6 +11,7 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
+int g_latent_blocks = 0;     // tuning: blocks per compute unit the split of the keys aims at (default 2)
 int g_latent_form = 0;       // tuning: 1 keeps the plain attention kernel, 2 the absorbed form for every pass, 3 takes the
                              // expanded form wherever it can run
 
@@ -187,20 +188,20 @@ __device__ __forceinline__ float softmax_step(const float (&sc)[8], float &m, fl
 }
 
 // ------------------------------------------------------------------ absorbed form
-// Query rows of a sequence are its (token, head) pairs in order; a block of NW wavefronts takes 16 NW of them, every
-// wavefront 16 columns of S^T = K Q^T, and walks its share of the keys any of them sees, 32 at a time.  The cached rows of
+// Query rows of a sequence are its (token, head) pairs in order; a block takes NQ tiles of 16 of them, a tile being 16
+// columns of S^T = K Q^T, and walks its share of the keys any of them sees, 32 at a time.  The cached rows of
 // a step are staged once and serve as keys (all of the row) and, transposed, as values (the latent part).
-// Tile i of sequence b has slot row_start[b] heads / (16 NW) + b + i: no two tiles share one.
+// Block i of sequence b has slot row_start[b] heads / (16 NQ) + b + i: no two share one.
 struct StreamParams {
     const uint16_t *qa, *pool;
     uint16_t *out;
-    float *part_o, *part_ml;                         // [slot][split][16 NW][rank_p], [slot][split][2][16 NW]
+    float *part_o, *part_ml;                         // [slot][split][16 NQ][rank_p], [slot][split][16 NQ][2]: maximum, sum
     uint32_t splits;
 };
 
-template <int NW>
+template <int NQ>
 __device__ __forceinline__ bool stream_tile(const RaggedRows &rr, uint32_t heads, uint32_t slot, uint32_t *b_out, uint32_t *t0, uint32_t *n_rows) {
-    auto base = [&](uint32_t b) { return (uint32_t)((uint64_t)rr.row_start[b] * heads / (16 * NW)) + b; };
+    auto base = [&](uint32_t b) { return (uint32_t)((uint64_t)rr.row_start[b] * heads / (16 * NQ)) + b; };
     uint32_t lo = 0, hi = rr.batch;
     while (hi - lo > 1) {
         const uint32_t mid = (lo + hi) / 2;
@@ -208,22 +209,26 @@ __device__ __forceinline__ bool stream_tile(const RaggedRows &rr, uint32_t heads
         else hi = mid;
     }
     *b_out = lo;
-    *t0 = (slot - base(lo)) * 16 * NW;
+    *t0 = (slot - base(lo)) * 16 * NQ;
     *n_rows = (rr.row_start[lo + 1] - rr.row_start[lo]) * heads;
     return *t0 < *n_rows;
 }
 
-template <int RK, int RO, int NW>
-__global__ void __launch_bounds__(NW * 64)
+// RK, RO: rank_p and rot_p in units of 32.  DH wavefronts share a column tile: each forms the scores (registers for the
+// whole query row) and sums a 1 / DH share of the latent dims.
+template <int RK, int RO, int NQ, int DH>
+__global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_eu(2)))
     latent_stream_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
-    constexpr int KS = RK + RO, VT = 2 * RK, PITCH = KS * 32 + 8, TPK = NW * 64 / kKeys, PIECES = (KS * 4 + TPK - 1) / TPK;
+    constexpr int KS = RK + RO, VT = 2 * RK / DH, WIDTH = KS * 32, PITCH = WIDTH + 8, TPK = NQ * DH * 64 / kKeys, PIECES = KS * 4 / TPK;
+    static_assert(PIECES * TPK == KS * 4 || TPK > 4, "whole rows");
+    constexpr int NP = (KS * 4 + TPK - 1) / TPK;
     extern __shared__ __attribute__((aligned(16))) uint16_t stage[];        // [2][32][PITCH]
     uint32_t b, t0, n_rows;
-    if (!stream_tile<NW>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
-    const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, g = lane / 16, c = lane % 16;
-    const uint32_t row0 = rr.row_start[b], H = sh.heads, width = sh.rank_p + sh.rot_p, rk = sh.rank_p / 32, ro = sh.rot_p / 32;
+    if (!stream_tile<NQ>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
+    const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), qt = wave / DH, dh = wave % DH, g = lane / 16, c = lane % 16;
+    const uint32_t row0 = rr.row_start[b], H = sh.heads;
     const uint32_t *table = rr.tables + (uint64_t)b * rr.max_blocks;
-    const uint32_t last_row = t0 + 16 * NW - 1 < n_rows ? t0 + 16 * NW - 1 : n_rows - 1;
+    const uint32_t last_row = t0 + 16 * NQ - 1 < n_rows ? t0 + 16 * NQ - 1 : n_rows - 1;
     const int32_t p0 = rr.pos[row0], p_lo = p0 + (int32_t)(t0 / H), p_hi = p0 + (int32_t)(last_row / H), W = (int32_t)sh.window;
     int32_t k_lo = p_lo - W + 1 > 0 ? p_lo - W + 1 : 0, k_hi = p_hi + 1;    // keys seen by some column
     if (p.splits > 1) {
@@ -231,75 +236,73 @@ __global__ void __launch_bounds__(NW * 64)
         k_lo += (int32_t)blockIdx.y * per;
         k_hi = k_lo + per < k_hi ? k_lo + per : k_hi;
     }
-    // this lane's column
-    const uint32_t col = t0 + wave * 16 + c, qr = col < n_rows ? col : n_rows - 1;
-    const int32_t pos = p0 + (int32_t)(qr / H);
-    const uint16_t *q = p.qa + ((uint64_t)row0 * H + qr) * width;
-    v8bf qf[KS];
-#pragma unroll
-    for (int s = 0; s < KS; ++s) {
-        v4u v = v4u{0, 0, 0, 0};
-        if (s < RK ? (uint32_t)s < rk : (uint32_t)(s - RK) < ro) v = *(const v4u *)(q + (s < RK ? s * 32 : sh.rank_p + (s - RK) * 32) + 8 * g);
-        qf[s] = __builtin_bit_cast(v8bf, v);
-    }
-    // staging: TPK threads per key; piece i of a thread is 16-byte piece part + i TPK of the row
-    const int key = tid / TPK, part = tid % TPK;
-    v4u st[PIECES];
-    auto key_row = [&](int32_t j) -> const uint16_t * {              // null: outside the walk; the pool's end: no page
-        if (j >= k_hi) return nullptr;
-        const uint32_t blk = (uint32_t)j / rr.block_size, id = blk < rr.max_blocks ? table[blk] : 0xffffffffu;
-        return p.pool + (id < rr.num_blocks ? (uint64_t)id * rr.block_size + (uint32_t)j % rr.block_size : sh.pool_rows) * width;
-    };
-    const uint16_t *const no_page = p.pool + sh.pool_rows * width;
-    auto fetch = [&](const uint16_t *src) {
-        const uint32_t fill = src == no_page ? 0x7fc07fc0u : 0u;     // a position without a page: NaN, never a silent zero
-#pragma unroll
-        for (int i = 0; i < PIECES; ++i) {
-            const int pc = part + i * TPK, s = pc / 4;
-            st[i] = v4u{fill, fill, fill, fill};
-            const bool real = pc < KS * 4 && (s < RK ? (uint32_t)s < rk : (uint32_t)(s - RK) < ro);
-            if (!real) st[i] = v4u{0, 0, 0, 0};
-            else if (src && src != no_page) st[i] = *(const v4u *)(src + (s < RK ? s * 32 : sh.rank_p + (s - RK) * 32) + (pc % 4) * 8);
+    const uint64_t ps = ((uint64_t)blockIdx.x * p.splits + blockIdx.y) * 16 * NQ + qt * 16 + c;
+    if (k_lo >= k_hi) {                              // a split without keys (never the only one)
+        if (dh == 0 && g == 0) {
+            p.part_ml[2 * ps] = -INFINITY;
+            p.part_ml[2 * ps + 1] = 0.0f;
         }
+        return;
+    }
+    // staging: TPK threads per key, 16 bytes each at a time; keys past the walk repeat its last one (their weight is zero)
+    const int key = tid / TPK, part = tid % TPK;
+    v4u st[NP];
+    bool lost = false;                               // the staged position has no page: NaN, never a silent zero
+    auto page_of = [&](int32_t j) -> uint32_t {
+        j = j < k_hi ? j : k_hi - 1;
+        const uint32_t blk = (uint32_t)j / rr.block_size;
+        return blk < rr.max_blocks ? table[blk] : 0xffffffffu;
+    };
+    auto fetch = [&](int32_t j, uint32_t id) {
+        j = j < k_hi ? j : k_hi - 1;
+        lost = id >= rr.num_blocks;
+        const uint16_t *src = p.pool + ((uint64_t)(lost ? 0 : id) * rr.block_size + (uint32_t)j % rr.block_size) * WIDTH + part * 8;
+#pragma unroll
+        for (int i = 0; i < NP; ++i)
+            if (NP * TPK == KS * 4 || part + i * TPK < KS * 4) st[i] = stream_load<true>((const v4u *)(src + i * TPK * 8));
     };
     auto put = [&](int buf) {
+        if (lost) st[0] = v4u{0x7fc07fc0u, 0x7fc07fc0u, 0x7fc07fc0u, 0x7fc07fc0u};
 #pragma unroll
-        for (int i = 0; i < PIECES; ++i) {
-            const int pc = part + i * TPK;
-            if (pc < KS * 4) *(v4u *)(stage + (buf * kKeys + key) * PITCH + pc * 8) = st[i];
-        }
+        for (int i = 0; i < NP; ++i)
+            if (NP * TPK == KS * 4 || part + i * TPK < KS * 4) *(v4u *)(stage + (buf * kKeys + key) * PITCH + (part + i * TPK) * 8) = st[i];
     };
+    uint32_t id = page_of(k_lo + key);
+    uint32_t id_next = page_of(k_lo + kKeys + key);
+    fetch(k_lo + key, id);
+    // this lane's column
+    const uint32_t col = t0 + qt * 16 + c, qr = col < n_rows ? col : n_rows - 1;
+    const int32_t pos = p0 + (int32_t)(qr / H);
+    const uint16_t *q = p.qa + ((uint64_t)row0 * H + qr) * WIDTH + 8 * g;
+    v8bf qf[KS];
+#pragma unroll
+    for (int s = 0; s < KS; ++s) qf[s] = *(const v8bf *)(q + s * 32);
+    const float factor = sh.scale * kLog2e;
     float m = -INFINITY, l = 0.0f;
     v4f o[VT];
 #pragma unroll
     for (int t = 0; t < VT; ++t) o[t] = v4f{0.f, 0.f, 0.f, 0.f};
-    const uint16_t *next = nullptr;
-    if (k_lo < k_hi) {
-        fetch(key_row(k_lo + key));
-        next = key_row(k_lo + kKeys + key);
-        put(0);
-    }
+    put(0);
     __syncthreads();
     int buf = 0;
     for (int32_t k0 = k_lo; k0 < k_hi; k0 += kKeys, buf ^= 1) {
         const bool more = k0 + kKeys < k_hi;
         if (more) {
-            fetch(next);
-            next = key_row(k0 + 2 * kKeys + key);
+            fetch(k0 + kKeys + key, id_next);
+            id_next = page_of(k0 + 2 * kKeys + key);
         }
         const uint16_t *rows = stage + buf * kKeys * PITCH;
+        v4f acc[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int s = 0; s < KS; ++s)
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt)
+                acc[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const v8bf *)(rows + (kt * 16 + c) * PITCH + s * 32 + 8 * g), qf[s], acc[kt], 0, 0, 0);
         float sc[8];
 #pragma unroll
-        for (int kt = 0; kt < 2; ++kt) {
-            v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int s = 0; s < KS; ++s)
-                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const v8bf *)(rows + (kt * 16 + c) * PITCH + s * 32 + 8 * g), qf[s], acc, 0, 0, 0);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int32_t j = k0 + kt * 16 + 4 * g + e;
-                sc[kt * 4 + e] = j <= pos && pos - j < W && j < k_hi ? acc[e] * (sh.scale * kLog2e) : -INFINITY;
-            }
+        for (int i = 0; i < 8; ++i) {
+            const int32_t j = k0 + (i / 4) * 16 + 4 * g + i % 4;
+            sc[i] = j <= pos && pos - j < W && j < k_hi ? acc[i / 4][i % 4] * factor : -INFINITY;
         }
         v8bf w_hi, w_lo;
         const float fix = softmax_step(sc, m, l, w_hi, w_lo);
@@ -309,7 +312,7 @@ __global__ void __launch_bounds__(NW * 64)
         }
 #pragma unroll
         for (int t = 0; t < VT; ++t) {
-            const v8bf v = transposed_keys(rows + t * 16, PITCH, lane);
+            const v8bf v = transposed_keys(rows + (dh * VT + t) * 16, PITCH, lane);
             o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_hi, o[t], 0, 0, 0);
             o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_lo, o[t], 0, 0, 0);
         }
@@ -319,15 +322,13 @@ __global__ void __launch_bounds__(NW * 64)
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
     if (p.splits > 1) {
-        const uint64_t ps = ((uint64_t)blockIdx.x * p.splits + blockIdx.y) * 16 * NW;
-        if (g == 0) {
-            p.part_ml[2 * ps + wave * 16 + c] = m;
-            p.part_ml[2 * ps + 16 * NW + wave * 16 + c] = l;
+        if (dh == 0 && g == 0) {
+            p.part_ml[2 * ps] = m;
+            p.part_ml[2 * ps + 1] = l;
         }
-        if (col < n_rows && k_lo < k_hi) {
+        if (col < n_rows) {
 #pragma unroll
-            for (int t = 0; t < VT; ++t)
-                if ((uint32_t)t < 2 * rk) *(v4f *)(p.part_o + (ps + wave * 16 + c) * sh.rank_p + t * 16 + 4 * g) = o[t];
+            for (int t = 0; t < VT; ++t) *(v4f *)(p.part_o + ps * (RK * 32) + (dh * VT + t) * 16 + 4 * g) = o[t];
         }
         return;
     }
@@ -335,77 +336,86 @@ __global__ void __launch_bounds__(NW * 64)
     const float inv = 1.0f / l;
 #pragma unroll
     for (int t = 0; t < VT; ++t)
-        if ((uint32_t)t < 2 * rk)
-            *(v2u *)(p.out + ((uint64_t)row0 * H + col) * sh.rank_p + t * 16 + 4 * g) =
-                v2u{f32x2_to_bf16x2(o[t][0] * inv, o[t][1] * inv), f32x2_to_bf16x2(o[t][2] * inv, o[t][3] * inv)};
+        *(v2u *)(p.out + ((uint64_t)row0 * H + col) * (RK * 32) + (dh * VT + t) * 16 + 4 * g) =
+            v2u{f32x2_to_bf16x2(o[t][0] * inv, o[t][1] * inv), f32x2_to_bf16x2(o[t][2] * inv, o[t][3] * inv)};
 }
 
-// Adds the splits of a tile's columns: one block per (slot, column).
-template <int NW>
+// Adds the splits of a tile's columns: one block per (slot, column), four dims per thread.
+constexpr uint32_t kMaxSplits = 64;
+template <int NQ>
 __global__ void __launch_bounds__(128) latent_merge_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
+    __shared__ float w[kMaxSplits];
     uint32_t b, t0, n_rows;
-    if (!stream_tile<NW>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
+    if (!stream_tile<NQ>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
     const uint32_t cl = blockIdx.y, col = t0 + cl;
     if (col >= n_rows) return;
-    const uint64_t ps = (uint64_t)blockIdx.x * p.splits * 16 * NW;
-    float m = -INFINITY, l = 0.0f;
-    for (uint32_t s = 0; s < p.splits; ++s) m = fmaxf(m, p.part_ml[2 * (ps + (uint64_t)s * 16 * NW) + cl]);
-    for (uint32_t s = 0; s < p.splits; ++s) {
-        const uint64_t at = 2 * (ps + (uint64_t)s * 16 * NW) + cl;
-        const float ls = p.part_ml[at + 16 * NW];    // 0: the split held none of the column's keys
-        if (ls != 0.0f) l += ls * exp2f(p.part_ml[at] - m);
-    }
-    const float inv = 1.0f / l;
-    for (uint32_t d = threadIdx.x * 4; d < sh.rank_p; d += 512) {
-        v4f a = v4f{0.f, 0.f, 0.f, 0.f};
-        for (uint32_t s = 0; s < p.splits; ++s) {
-            const uint64_t at = ps + (uint64_t)s * 16 * NW;
-            const float ms = p.part_ml[2 * at + cl];
-            if (p.part_ml[2 * at + 16 * NW + cl] != 0.0f) a += *(const v4f *)(p.part_o + (at + cl) * sh.rank_p + d) * exp2f(ms - m);
+    const uint64_t ps = (uint64_t)blockIdx.x * p.splits * 16 * NQ + cl;      // split s of this column: + s * 16 NQ
+    if (threadIdx.x < 64) {
+        const uint32_t s = threadIdx.x;
+        float ms = -INFINITY, ls = 0.0f;                                     // sum 0: the split holds none of the column's keys
+        if (s < p.splits) {
+            const v2f v = *(const v2f *)(p.part_ml + 2 * (ps + (uint64_t)s * 16 * NQ));
+            ms = v[0];
+            ls = v[1];
         }
-        *(v2u *)(p.out + ((uint64_t)rr.row_start[b] * sh.heads + col) * sh.rank_p + d) =
-            v2u{f32x2_to_bf16x2(a[0] * inv, a[1] * inv), f32x2_to_bf16x2(a[2] * inv, a[3] * inv)};
+        const float m = wave_max(ms), f = ls != 0.0f ? exp2f(ms - m) : 0.0f, l = wave_sum(ls * f);
+        w[s] = f / l;
+    }
+    __syncthreads();
+    for (uint32_t d = threadIdx.x * 4; d < sh.rank_p; d += 512) {
+        const float *src = p.part_o + ps * sh.rank_p + d;
+        v4f a = v4f{0.f, 0.f, 0.f, 0.f};
+        for (uint32_t s0 = 0; s0 < p.splits; s0 += 8) {
+            v4f t[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) t[i] = *(const v4f *)(src + (uint64_t)(s0 + i < p.splits ? s0 + i : p.splits - 1) * 16 * NQ * sh.rank_p);
+#pragma unroll
+            for (int i = 0; i < 8; ++i)
+                if (s0 + i < p.splits && w[s0 + i] != 0.0f) a += t[i] * w[s0 + i];
+        }
+        *(v2u *)(p.out + ((uint64_t)rr.row_start[b] * sh.heads + col) * sh.rank_p + d) = v2u{f32x2_to_bf16x2(a[0], a[1]), f32x2_to_bf16x2(a[2], a[3])};
     }
 }
 
 struct StreamPlan {
-    int nw = 0;                                      // 0: the plain kernel
+    int nq = 0;                                      // 0: the plain kernel
     uint32_t slots = 0, splits = 1;
 };
 StreamPlan stream_plan(const LatentShape &sh, uint32_t rows, uint32_t batch, uint32_t longest, int num_cus) {
     StreamPlan p;
     if (sh.rank_p > 512 || sh.rot_p > 64 || g_latent_form == 1) return p;
-    p.nw = (uint64_t)longest * sh.heads <= 32 ? 2 : 4;
-    p.slots = (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nw)) + batch + 1;
-    // about two blocks per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NW)
-    const uint64_t used = std::max<uint64_t>(std::max<uint64_t>((uint64_t)rows * sh.heads / (16 * p.nw), batch), 1);
-    const uint64_t want = (2 * (uint64_t)num_cus + used - 1) / used;
-    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (sh.window + 127) / 128, 64}));
+    p.nq = (uint64_t)longest * sh.heads <= 32 ? 2 : 4;
+    p.slots = (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nq)) + batch + 1;
+    // about two blocks per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NQ)
+    const uint64_t used = std::max<uint64_t>(std::max<uint64_t>((uint64_t)rows * sh.heads / (16 * p.nq), batch), 1);
+    const uint64_t want = ((uint64_t)(g_latent_blocks ? g_latent_blocks : 2) * num_cus + used - 1) / used;
+    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (sh.window + 127) / 128, kMaxSplits}));
     return p;
 }
 
-template <int RK, int RO, int NW>
+template <int RK, int RO, int NQ>
 void launch_stream(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, uint32_t slots, hipStream_t s) {
+    constexpr int DH = RK == 16 ? 2 : 1;
     constexpr size_t lds = 2ull * kKeys * ((RK + RO) * 32 + 8) * 2;
     if constexpr (lds > 65536) {
         static bool configured = false;
         if (!configured) {
-            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_stream_kernel<RK, RO, NW>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_stream_kernel<RK, RO, NQ, DH>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
             configured = true;
         }
     }
-    latent_stream_kernel<RK, RO, NW><<<dim3(slots, p.splits), NW * 64, lds, s>>>(p, sh, rr);
-    if (p.splits > 1) latent_merge_kernel<NW><<<dim3(slots, 16 * NW), 128, 0, s>>>(p, sh, rr);
+    latent_stream_kernel<RK, RO, NQ, DH><<<dim3(slots, p.splits), NQ * DH * 64, lds, s>>>(p, sh, rr);
+    if (p.splits > 1) latent_merge_kernel<NQ><<<dim3(slots, 16 * NQ), 128, 0, s>>>(p, sh, rr);
 }
 template <int RK, int RO>
-void launch_stream_nw(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, const StreamPlan &plan, hipStream_t s) {
-    if (plan.nw == 2) launch_stream<RK, RO, 2>(p, sh, rr, plan.slots, s);
+void launch_stream_nq(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, const StreamPlan &plan, hipStream_t s) {
+    if (plan.nq == 2) launch_stream<RK, RO, 2>(p, sh, rr, plan.slots, s);
     else launch_stream<RK, RO, 4>(p, sh, rr, plan.slots, s);
 }
 template <int RK>
 void launch_stream_ro(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, const StreamPlan &plan, hipStream_t s) {
-    if (sh.rot_p <= 32) launch_stream_nw<RK, 1>(p, sh, rr, plan, s);
-    else launch_stream_nw<RK, 2>(p, sh, rr, plan, s);
+    if (sh.rot_p <= 32) launch_stream_nq<RK, 1>(p, sh, rr, plan, s);
+    else launch_stream_nq<RK, 2>(p, sh, rr, plan, s);
 }
 
 // ------------------------------------------------------------------ expanded form
@@ -439,18 +449,16 @@ __global__ void __launch_bounds__(256)
 }
 
 // A block of four wavefronts takes 128 tokens of one (sequence, head), every wavefront 32 columns of S^T = K Q^T, and walks
-// the keys they see 32 at a time; K (unrotated | rotated) and V of a step are staged in LDS, two stages.  D: tiles of 32
-// that hold dim and vdim, RO: of the rotated part.
+// the keys they see 32 at a time; K (unrotated | rotated) and V of a step are staged in LDS, two stages.  D, RO:
+// dim_p = v_p and rot_p in units of 32.
 template <int D, int RO>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2)))
     latent_flash_kernel(const uint16_t *__restrict__ q, const uint16_t *__restrict__ kv, const uint16_t *__restrict__ kr,
                         const float *__restrict__ gate, uint32_t ld_gate, uint16_t *__restrict__ out, uint32_t ld_out, LatentShape sh,
                         RaggedRows rr, LatentExpand ex) {
     constexpr int KS = D + RO, VT = 2 * D, KP = KS * 32 + 8, VP = D * 32 + 8, NQ = 2;
-    constexpr int PK = KS * 4 / 8, PV = D * 4 / 8;   // 16-byte pieces per thread and step (eight threads per key); KS even or padded below
-    constexpr int PKR = (KS * 4 + 7) / 8;
+    constexpr int PKR = (KS * 4 + 7) / 8, PV = D * 4 / 8;        // 16-byte pieces per thread and step, eight threads per key
     __shared__ __attribute__((aligned(16))) uint16_t ks[2][kKeys * KP], vs[2][kKeys * VP];
-    static_assert(PV * 8 == D * 4 && PK <= PKR, "eight threads stage a key");
     // longest walks first: the last tiles of a sequence
     uint32_t lo = 0, hi = rr.batch;
     const uint32_t slots = gridDim.x, slot = slots - 1 - blockIdx.x;
@@ -462,8 +470,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     const uint32_t b = lo, row0 = rr.row_start[b], n = rr.row_start[b + 1] - row0, t0 = (slot - (row0 / 128 + b)) * 128;
     if (t0 >= n) return;
     const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), g = lane / 16, c = lane % 16;
-    const uint32_t h = blockIdx.y, H = sh.heads, qw = sh.dim_p + sh.rot_p, dk = sh.dim_p / 32, ro = sh.rot_p / 32, dv = (sh.vdim + 31) / 32;
-    const uint32_t hw = sh.dim_p + dv * 32;          // one head of an expanded row
+    const uint32_t h = blockIdx.y, H = sh.heads, qw = KS * 32;
+    constexpr uint32_t hw = 2 * D * 32;              // one head of an expanded row
     const int32_t p0 = rr.pos[row0], W = (int32_t)sh.window, first = (int32_t)ex.first[b];
     const uint32_t t_last = t0 + 127 < n ? t0 + 127 : n - 1;
     int32_t k_lo = p0 + (int32_t)t0 - W + 1, k_hi = p0 + (int32_t)t_last + 1;
@@ -480,9 +488,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
         const uint16_t *src = q + ((uint64_t)(row0 + t) * H + h) * qw + 8 * g;
 #pragma unroll
         for (int s = 0; s < KS; ++s) {
-            v4u v = v4u{0, 0, 0, 0};
-            if (s < D ? (uint32_t)s < dk : (uint32_t)(s - D) < ro) v = *(const v4u *)(src + (s < D ? s * 32 : sh.dim_p + (s - D) * 32));
-            qf[qi][s] = __builtin_bit_cast(v8bf, v);
+            qf[qi][s] = *(const v8bf *)(src + s * 32);
         }
     }
     const int32_t w_lo_pos = p0 + (int32_t)(t0 + wave * 32 < n ? t0 + wave * 32 : n - 1);
@@ -494,24 +500,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
         const int32_t j = k0 + key;
         const bool ok = j < k_hi;
         const uint64_t e = e0 + (uint64_t)(ok ? j : k_hi - 1);
-        const uint16_t *row = kv + (e * H + h) * hw, *rot = kr + e * sh.rot_p;
+        const uint16_t *row = kv + (e * H + h) * hw, *rot = kr + e * (RO * 32);
 #pragma unroll
         for (int i = 0; i < PKR; ++i) {
-            const int pc = part + 8 * i, s = pc / 4;
-            sk[i] = v4u{0, 0, 0, 0};
-            if (pc >= KS * 4) continue;
-            if (s < D) {
-                if ((uint32_t)s < dk) sk[i] = *(const v4u *)(row + pc * 8);
-            } else if ((uint32_t)(s - D) < ro) {
-                sk[i] = *(const v4u *)(rot + (pc - D * 4) * 8);
-            }
+            const int pc = part + 8 * i;
+            if (pc < KS * 4) sk[i] = *(const v4u *)(pc < D * 4 ? row + pc * 8 : rot + (pc - D * 4) * 8);
         }
 #pragma unroll
-        for (int i = 0; i < PV; ++i) {
-            const int pc = part + 8 * i;
-            sv[i] = v4u{0, 0, 0, 0};
-            if ((uint32_t)(pc / 4) < dv) sv[i] = *(const v4u *)(row + sh.dim_p + pc * 8);
-        }
+        for (int i = 0; i < PV; ++i) sv[i] = *(const v4u *)(row + D * 32 + (part + 8 * i) * 8);
     };
     auto put = [&](int buf) {
 #pragma unroll
@@ -628,10 +624,23 @@ void latent_rotate_query(const void *q, const float *cos_sin, void *dst, uint32_
         latent_rotate_query_kernel<uint16_t><<<rows, 256, 0, s>>>((const uint16_t *)q, cos_sin, (uint16_t *)dst, dst_pitch, dst_off, sh);
 }
 
+void latent_pad(LatentShape &sh) {
+    auto up = [](uint32_t v, std::initializer_list<uint32_t> sizes) {
+        for (uint32_t s : sizes)
+            if (v <= s) return s;
+        return (v + 31) / 32 * 32;
+    };
+    sh.rank_p = up(sh.kv_rank, {64, 128, 256, 512});
+    sh.rot_p = up(sh.rot, {32, 64});
+    sh.dim_p = up(sh.dim, {64, 128});
+    sh.v_p = up(sh.vdim, {64, 128});
+    if (sh.dim_p <= 128 && sh.v_p <= 128) sh.dim_p = sh.v_p = sh.dim_p > sh.v_p ? sh.dim_p : sh.v_p;
+}
+
 uint64_t latent_attention_workspace_bytes(const LatentShape &sh, int is_f32, uint32_t rows, uint32_t batch, uint32_t max_new, int num_cus) {
     if (is_f32) return 0;
     const StreamPlan p = stream_plan(sh, rows, batch, max_new, num_cus);
-    return p.splits > 1 ? (uint64_t)p.slots * p.splits * 16 * p.nw * (sh.rank_p + 2) * 4 : 0;
+    return p.splits > 1 ? (uint64_t)p.slots * p.splits * 16 * p.nq * (sh.rank_p + 2) * 4 : 0;
 }
 
 void latent_attention(const void *qa, const void *pool, void *out, int is_f32, const LatentShape &sh, const RaggedRows &rr,
@@ -639,9 +648,9 @@ void latent_attention(const void *qa, const void *pool, void *out, int is_f32, c
     if (rr.rows == 0) return;
     if (!is_f32) {
         const StreamPlan plan = stream_plan(sh, rr.rows, rr.batch, max_new, num_cus);
-        if (plan.nw) {
+        if (plan.nq) {
             StreamParams p{(const uint16_t *)qa, (const uint16_t *)pool, (uint16_t *)out, (float *)workspace, nullptr, plan.splits};
-            if (p.splits > 1) p.part_ml = p.part_o + (uint64_t)plan.slots * plan.splits * 16 * plan.nw * sh.rank_p;
+            if (p.splits > 1) p.part_ml = p.part_o + (uint64_t)plan.slots * plan.splits * 16 * plan.nq * sh.rank_p;
             if (sh.rank_p <= 64) launch_stream_ro<2>(p, sh, rr, plan, s);
             else if (sh.rank_p <= 128) launch_stream_ro<4>(p, sh, rr, plan, s);
             else if (sh.rank_p <= 256) launch_stream_ro<8>(p, sh, rr, plan, s);
@@ -657,7 +666,9 @@ void latent_attention(const void *qa, const void *pool, void *out, int is_f32, c
         latent_attention_plain_kernel<uint16_t><<<grid, 256, lds, s>>>((const uint16_t *)qa, (const uint16_t *)pool, (uint16_t *)out, sh, rr);
 }
 
-bool latent_expand_applies(const LatentShape &sh) { return sh.dim_p <= 128 && sh.vdim <= 128 && sh.rot_p <= 64 && g_latent_form != 1 && g_latent_form != 2; }
+bool latent_expand_applies(const LatentShape &sh) {
+    return sh.dim_p == sh.v_p && sh.v_p <= 128 && sh.rot_p <= 64 && g_latent_form != 1 && g_latent_form != 2;
+}
 bool latent_expand_always() { return g_latent_form == 3; }
 
 void latent_gather(const void *pool, void *c, uint32_t ld_c, void *kr, const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s) {
@@ -668,7 +679,7 @@ void latent_gather(const void *pool, void *c, uint32_t ld_c, void *kr, const Lat
 void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, void *out, uint32_t ld_out,
                                const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s) {
     const dim3 grid(rr.rows / 128 + rr.batch + 1, sh.heads);
-    const bool wide = sh.dim_p > 64 || sh.vdim > 64, rot2 = sh.rot_p > 32;
+    const bool wide = sh.v_p > 64, rot2 = sh.rot_p > 32;
 #define FA_FLASH(D_, RO_)                                                                                                                    \
     latent_flash_kernel<D_, RO_><<<grid, 256, 0, s>>>((const uint16_t *)q, (const uint16_t *)kv, (const uint16_t *)kr, gate, ld_gate, (uint16_t *)out, \
                                                       ld_out, sh, rr, ex)

@@ -388,12 +388,15 @@ void gather_rows_any(const void *table, int table_f32, uint64_t table_rows, uint
 // ---- latent attention (kern_latent.hip) -----------------------------------------
 struct LatentShape {
     uint32_t heads, dim, rot, vdim, q_rank, kv_rank;     // sizes of the configuration
-    uint32_t dim_p, rot_p, rank_p;                       // padded to 32: q rows are [heads][dim_p + rot_p], cache rows and
-                                                         // absorbed queries [rank_p + rot_p], padding zero
+    uint32_t dim_p, rot_p, rank_p, v_p;                  // padded (latent_pad): q rows are [heads][dim_p + rot_p], cache rows
+                                                         // and absorbed queries [rank_p + rot_p], padding zero
     uint32_t window;                                     // keys p - window + 1 .. p
     float scale, eps;
     uint64_t pool_rows;
 };
+// Sets the padded sizes: those of the matrix-core kernels' instances (rank 64, 128, 256 or 512, rot 32 or 64, dim and vdim
+// both 64 or both 128), multiples of 32 beyond them.
+void latent_pad(LatentShape &sh);
 // From y [rows, ld] f32 = q latent | kv latent | rotated key part | gates: RMS norm of the q latent -> cq [rows, ld_cq];
 // with a pool: RMS norm of the latent and rotation of the key part -> the token's cache row.
 void latent_prepare(const float *y, uint32_t ld, const float *q_norm, const float *kv_norm, const float *cos_sin, void *cq,
@@ -409,7 +412,7 @@ void latent_attention(const void *qa, const void *pool, void *out, int is_f32, c
                       uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
 // The form for prompts (bf16, dim, vdim <= 128, rot <= 64): the keys first[b] .. of every sequence are gathered as rows
 // start[b] .. start[b + 1] - 1 (latents c [rows, ld_c], rotated parts kr [rows, rot_p]), a linear turns the latents into
-// kv [rows, heads, dim_p + vdim padded to 32], and attention runs per head on those; q is [rows, heads, dim_p + rot_p] with its
+// kv [rows, heads, dim_p + v_p], and attention runs per head on those; q is [rows, heads, dim_p + rot_p] with its
 // rotated part rotated; the heads' gates (sigmoid) are applied, out [rows, ld_out].
 struct LatentExpand {
     const uint32_t *start, *first;   // [batch + 1], [batch]

@@ -162,7 +162,7 @@ fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t row
         if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) {
             ec = std::max<uint64_t>(ec, pad_to(l.la.rank_p, 64));
             er = std::max<uint64_t>(er, l.la.rot_p);
-            ekv = std::max<uint64_t>(ekv, (uint64_t)l.la.heads * (l.la.dim_p + pad_to(l.la.vdim, 32)));
+            ekv = std::max<uint64_t>(ekv, (uint64_t)l.la.heads * (l.la.dim_p + l.la.v_p));
         }
     if (L.is_f32) expand_rows = 0;
     add(&a.ec, expand_rows * ec * E);
@@ -709,9 +709,7 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 a.vdim = g.vdim;
                 a.q_rank = g.q_rank;
                 a.kv_rank = g.kv_rank;
-                a.dim_p = pad_to(g.dim, 32);
-                a.rot_p = pad_to(g.rot_dim, 32);
-                a.rank_p = pad_to(g.kv_rank, 32);
+                k::latent_pad(a);
                 a.window = g.window;
                 a.scale = g.scale;
                 a.eps = c.norm_eps;
@@ -743,7 +741,7 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 }
                 // per head, latent = W_uk^T q: the key projection transposed
                 const uint32_t kr = g.kv_rank, vd = g.vdim;
-                const uint32_t hw = dim_p + pad_to(vd, 32);
+                const uint32_t hw = dim_p + a.v_p;
                 if (!f32) l.ukv = weight(H * hw, H * hw, kr);
                 const k::LinearWeight both = l.ukv;
                 l.uk = weight(a.rank_p, a.rank_p, dim, H);
