@@ -33,6 +33,10 @@ __device__ __forceinline__ float log_decay(float a_log, float x) {
     return -expf(a_log) * sp;
 }
 
+// x sigmoid(x) and exp(x) on the hardware's exponential and reciprocal (about one unit in the last place each)
+__device__ __forceinline__ float fast_exp(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+__device__ __forceinline__ float fast_silu(float x) { return x * __builtin_amdgcn_rcpf(1.0f + fast_exp(-x)); }
+
 // Convolution + SiLU of channel c for token t of a sequence (row0: its first row of the pass, p: the token's position).
 // Inputs before the pass come from the slot's ring.
 template <typename T>
@@ -45,7 +49,7 @@ __device__ __forceinline__ float conv_silu(const T *__restrict__ y, uint32_t ld,
         const float x = back <= t ? load_as_f32(y + (row0 + t - back) * ld + c) : load_as_f32(ring + (uint64_t)((p - back) % n_taps) * channels + c);
         acc = fmaf(taps[(uint64_t)c * n_taps + i], x, acc);
     }
-    return silu_f32(acc);
+    return fast_silu(acc);
 }
 
 // ------------------------------------------------------------------ token by token
@@ -115,7 +119,7 @@ __global__ void __launch_bounds__(NT)
                     float acc = 0.0f;
 #pragma unroll
                     for (int back = 3; back >= 0; --back) acc = fmaf(win[q][back], xin[q][back], acc);
-                    v = silu_f32(acc);
+                    v = fast_silu(acc);
                 } else {
                     v = conv_silu(y, io.ld_y, ring, io.conv, sh.taps, channels, c, row0, t, p);
                 }
@@ -172,7 +176,7 @@ __global__ void __launch_bounds__(NT)
                 const uint32_t c = cg * 4 + e;
                 if (c < vdim) {
                     const float gate = load_as_f32(y + row * io.ld_y + channels + h * vdim + c);
-                    store_from_f32((T *)io.out + row * io.ld_out + h * vdim + c, o[e] * ro * io.norm[c] * silu_f32(gate));
+                    store_from_f32((T *)io.out + row * io.ld_out + h * vdim + c, o[e] * ro * io.norm[c] * fast_silu(gate));
                 }
             }
         }
@@ -259,7 +263,7 @@ __device__ __forceinline__ void conv_chunk(float *dst, uint32_t pitch, const T *
                 float acc = 0.0f;
 #pragma unroll
                 for (int i = MAXTAPS - 1; i >= 0; --i) acc = fmaf(w[i], x[j + MAXTAPS - 1 - i], acc);
-                dst[(tg + j) * pitch + col] = t0 + tg + j < n ? silu_f32(acc) : 0.0f;
+                dst[(tg + j) * pitch + col] = t0 + tg + j < n ? fast_silu(acc) : 0.0f;
             }
         }
     }
@@ -273,7 +277,7 @@ __global__ void __launch_bounds__(256)
     extern __shared__ __attribute__((aligned(16))) float lds[];
     float *lk = lds, *lq = lk + 32 * PITCH;          // K; Q, then V in slices of DP columns
     float *la = lq + 32 * PITCH, *lt = la + 32 * 36; // A and T, pitch 36
-    __shared__ float rq[32], rk[32], beta[32], G[32];
+    __shared__ float rq[32], rk[32], beta[32], G[32], qs[32], ks[32], ke[32];   // qs = rq exp(G), ks = rk exp(G), ke = rk exp(G_C - G)
     // the slot's sequence and chunk
     uint32_t lo = 0, hi = rr.batch;
     while (hi - lo > 1) {
@@ -319,8 +323,15 @@ __global__ void __launch_bounds__(256)
         sq += __shfl_xor(sq, 2, 64);
         if (tid % 4 == 0) {
             const float r = 1.0f / sqrtf(sq + 1e-6f);
-            if (tid < 128) rq[tid / 4] = r / sqrtf((float)dim);
-            else rk[(tid - 128) / 4] = r;
+            const int i = (tid % 128) / 4;
+            if (tid < 128) {
+                rq[i] = r / sqrtf((float)dim);
+                qs[i] = rq[i] * expf(G[i]);
+            } else {
+                rk[i] = r;
+                ks[i] = r * expf(G[i]);
+                ke[i] = r * expf(G[31] - G[i]);
+            }
         }
     }
     __syncthreads();
@@ -338,7 +349,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int j = tj * 16 + 4 * g + e;
-            la[i_ * 36 + j] = j < i_ ? beta[i_] * expf(G[i_] - G[j]) * rk[i_] * rk[j] * d[e] : 0.0f;
+            la[i_ * 36 + j] = j < i_ ? beta[i_] * fast_exp(G[i_] - G[j]) * rk[i_] * rk[j] * d[e] : 0.0f;
         }
     }
     if (wave != 1) {
@@ -346,20 +357,20 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int j = tj * 16 + 4 * g + e;
-            d[e] = j <= i_ ? expf(G[i_] - G[j]) * rq[i_] * rk[j] * d[e] : 0.0f;
+            d[e] = j <= i_ ? fast_exp(G[i_] - G[j]) * rq[i_] * rk[j] * d[e] : 0.0f;
         }
         put(6 * KT + ti + tj, d);
     }
     // exp(G) Q and the decayed K^T
     for (uint32_t f = wave; f < 2 * KT; f += 4) {
         const uint32_t rt = f / KT, kt = f % KT, i = rt * 16 + lr;
-        put(2 * KT + f, *(const v4f *)(lq + i * PITCH + kt * 16 + 4 * g) * (expf(G[i]) * rq[i]));
+        put(2 * KT + f, *(const v4f *)(lq + i * PITCH + kt * 16 + 4 * g) * qs[i]);
         const uint32_t dt = f / 2, ct = f % 2;
         v4f v;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const uint32_t j = ct * 16 + 4 * g + e;
-            v[e] = lk[j * PITCH + dt * 16 + lr] * rk[j] * expf(G[31] - G[j]);
+            v[e] = lk[j * PITCH + dt * 16 + lr] * ke[j];
         }
         put(4 * KT + f, v);
     }
@@ -411,7 +422,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const uint32_t j = ct * 16 + 4 * g + e;
-                kf[e] = -lk[j * PITCH + kt * 16 + lr] * rk[j] * expf(G[j]);
+                kf[e] = -lk[j * PITCH + kt * 16 + lr] * ks[j];
             }
             acc = mfma4(kf, rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], acc);
         }
@@ -437,16 +448,22 @@ __global__ void __launch_bounds__(256)
     }
 }
 
+// LDS buffers of delta_scan_kernel: two where two chunks fit
+constexpr int scan_buffers(int kt) { return kt <= 8 ? 2 : 1; }
+
 // One wavefront per (sequence, head, 16 value columns); state tile kt in D order: rows 16 kt + 4 g + e, column l % 16.
 template <int KT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(512)
     delta_scan_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, const float *__restrict__ frags, const float *__restrict__ chunk_decay,
                       float *__restrict__ o, uint32_t vt, uint32_t n_frags) {
-    const int lane = threadIdx.x % 64, wave = threadIdx.x / 64, lr = lane % 16, g = lane / 16;
-    const uint32_t b = blockIdx.z, h = blockIdx.y, nt = blockIdx.x * (blockDim.x / 64) + wave;
+    const int lane = threadIdx.x % 64, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), lr = lane % 16, g = lane / 16;
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const uint32_t b = blockIdx.z, h = blockIdx.y, nt_ = blockIdx.x * (blockDim.x / 64) + wave;
     const uint32_t row0 = rr.row_start[b], n = rr.row_start[b + 1] - row0;
-    if (n < kChunkFrom || nt >= vt) return;
-    const uint32_t dim = sh.dim, vdim = sh.vdim, vp = sh.vdim_p(), col = nt * 16 + lr, slot0 = slot_base(rr, b);
+    if (n < kChunkFrom) return;
+    const bool real = nt_ < vt;                      // a wavefront past the last column tile repeats it and stores nothing
+    const uint32_t nt = real ? nt_ : vt - 1;
+    const uint32_t dim = sh.dim, vp = sh.vdim_p(), col = nt * 16 + lr, slot0 = slot_base(rr, b), vdim = real ? sh.vdim : 0;
     float *state = io.state + ((uint64_t)rr.state_slot[b] * sh.heads + h) * dim * vp;
     const bool fresh = rr.pos[row0] == 0;
     v4f S[KT];
@@ -457,57 +474,76 @@ __global__ void __launch_bounds__(256)
             const uint32_t d = kt * 16 + 4 * g + e;
             S[kt][e] = !fresh && d < dim && col < vdim ? state[(uint64_t)d * vp + col] : 0.0f;
         }
-    const uint32_t chunks = (n + kChunk - 1) / kChunk;
-    v4f wq[4 * KT], kd[2 * KT], pf[3], u0[2];
-    auto base = [&](uint32_t c) { return (const v4f *)(frags + ((uint64_t)(slot0 + c) * sh.heads + h) * n_frags * 256) + lane; };
-    auto load_wq = [&](const v4f *f) {
+    // A chunk's fragments are staged in LDS as they are (one load instruction moves one fragment), those of the next chunk
+    // while this one is multiplied: the shared ones once per block, the values' two per wavefront.
+    const uint32_t chunks = (n + kChunk - 1) / kChunk, waves = blockDim.x / 64;
+    constexpr int SHARED = 6 * KT + 3, NB = scan_buffers(KT);
+    typedef __attribute__((address_space(1))) const void *gptr;
+    typedef __attribute__((address_space(3))) void *lptr;
+    const uint32_t buf_frags = SHARED + 2 * waves;
+    auto stage = [&](uint32_t c, uint32_t buf) {
+        const v4f *f = (const v4f *)(frags + ((uint64_t)(slot0 + c) * sh.heads + h) * n_frags * 256) + lane;
+        float *l = lds + (uint64_t)buf * buf_frags * 256;
+        for (uint32_t i = wave; i < (uint32_t)SHARED; i += waves) __builtin_amdgcn_global_load_lds((gptr)(f + i * 64), (lptr)(l + i * 256), 16, 0, 0);
 #pragma unroll
-        for (int i = 0; i < 4 * KT; ++i) wq[i] = f[i * 64];
+        for (uint32_t i = 0; i < 2; ++i)
+            __builtin_amdgcn_global_load_lds((gptr)(f + (SHARED + nt * 2 + i) * 64), (lptr)(l + (SHARED + wave * 2 + i) * 256), 16, 0, 0);
     };
-    auto load_rest = [&](const v4f *f) {
-#pragma unroll
-        for (int i = 0; i < 2 * KT; ++i) kd[i] = f[(4 * KT + i) * 64];
-#pragma unroll
-        for (int i = 0; i < 3; ++i) pf[i] = f[(6 * KT + i) * 64];
-#pragma unroll
-        for (int i = 0; i < 2; ++i) u0[i] = f[(6 * KT + 3 + nt * 2 + i) * 64];
-    };
-    load_wq(base(0));
-    load_rest(base(0));
+    stage(0, 0);
+    __builtin_amdgcn_s_waitcnt(0x0F70);              // this wavefront's fragments have landed
+    __syncthreads();
     for (uint32_t c = 0; c < chunks; ++c) {
-        const v4f *next = base(c + 1 < chunks ? c + 1 : c);
+        if (NB == 2 && c + 1 < chunks) stage(c + 1, (c + 1) & 1);
+        const v4f *f = (const v4f *)(lds + (uint64_t)(NB == 2 ? c & 1 : 0) * buf_frags * 256) + lane;
         const float decay = chunk_decay[(uint64_t)(slot0 + c) * sh.heads + h];
-        v4f u[2] = {u0[0], u0[1]}, r[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
+        v4f u[2], r[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
+        u[0] = f[(SHARED + wave * 2) * 64];
+        u[1] = f[(SHARED + wave * 2 + 1) * 64];
 #pragma unroll
-        for (int kt = 0; kt < KT; ++kt)
+        for (int kt = 0; kt < KT; ++kt) {
+            v4f a[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) a[i] = f[(i * KT + kt) * 64];
 #pragma unroll
             for (int e = 0; e < 4; ++e)
 #pragma unroll
                 for (int rt = 0; rt < 2; ++rt) {
-                    u[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(wq[rt * KT + kt][e], S[kt][e], u[rt], 0, 0, 0);
-                    r[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(wq[(2 + rt) * KT + kt][e], S[kt][e], r[rt], 0, 0, 0);
+                    u[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[rt][e], S[kt][e], u[rt], 0, 0, 0);
+                    r[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[2 + rt][e], S[kt][e], r[rt], 0, 0, 0);
                 }
-        load_wq(next);
-        r[0] = mfma4(pf[0], u[0], r[0]);
-        r[1] = mfma4(pf[1], u[0], r[1]);
-        r[1] = mfma4(pf[2], u[1], r[1]);
+        }
+        r[0] = mfma4(f[(6 * KT) * 64], u[0], r[0]);
+        r[1] = mfma4(f[(6 * KT + 1) * 64], u[0], r[1]);
+        r[1] = mfma4(f[(6 * KT + 2) * 64], u[1], r[1]);
 #pragma unroll
         for (int kt = 0; kt < KT; ++kt) S[kt] *= decay;
 #pragma unroll
         for (int ct = 0; ct < 2; ++ct)
 #pragma unroll
-            for (int e = 0; e < 4; ++e)
+            for (int k4 = 0; k4 < KT; k4 += (KT < 4 ? KT : 4)) {
+                v4f a[4];
 #pragma unroll
-                for (int kt = 0; kt < KT; ++kt) S[kt] = __builtin_amdgcn_mfma_f32_16x16x4f32(kd[kt * 2 + ct][e], u[ct][e], S[kt], 0, 0, 0);
-        load_rest(next);
+                for (int i = 0; i < (KT < 4 ? KT : 4); ++i) a[i] = f[(4 * KT + (k4 + i) * 2 + ct) * 64];
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+#pragma unroll
+                    for (int i = 0; i < (KT < 4 ? KT : 4); ++i) S[k4 + i] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i][e], u[ct][e], S[k4 + i], 0, 0, 0);
+            }
 #pragma unroll
         for (int rt = 0; rt < 2; ++rt)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const uint32_t t = c * kChunk + rt * 16 + 4 * g + e;
-                if (t < n && col < vdim) o[((uint64_t)(row0 + t) * sh.heads + h) * vdim + col] = r[rt][e];
+                if (t < n && col < vdim) o[((uint64_t)(row0 + t) * sh.heads + h) * sh.vdim + col] = r[rt][e];
             }
+        if (NB == 1) {
+            __syncthreads();
+            if (c + 1 < chunks) stage(c + 1, 0);
+        }
+        __builtin_amdgcn_s_waitcnt(0x0F70);          // the next chunk has landed (the read-outs' stores too)
+        __syncthreads();                             // ... for everybody, and nobody reads this chunk's any more
     }
+    if (!real) return;
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
@@ -529,7 +565,7 @@ __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaShape sh, DeltaIo 
         const float ro = 1.0f / sqrtf(wave_sum_dpp(sq) / (float)vdim + sh.eps);
         const T *gate = (const T *)io.y + (uint64_t)r * io.ld_y + sh.qkv() + h * vdim;
         for (uint32_t c = lane; c < vdim; c += 64)
-            store_from_f32((T *)io.out + (uint64_t)r * io.ld_out + h * vdim + c, x[c] * ro * io.norm[c] * silu_f32(load_as_f32(gate + c)));
+            store_from_f32((T *)io.out + (uint64_t)r * io.ld_out + h * vdim + c, x[c] * ro * io.norm[c] * fast_silu(load_as_f32(gate + c)));
     }
 }
 
@@ -547,9 +583,18 @@ void launch_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr
         }
     }
     chunk<<<dim3(p.slots, sh.heads), 256, lds, s>>>(sh, io, rr, frags, decay, p.vt, p.frags);
-    // wavefronts of a block share the chunk's fragments through the L1; fewer per block where there are few blocks
-    const uint32_t per = (uint64_t)rr.batch * sh.heads * p.vt <= 512 ? 1 : (uint64_t)rr.batch * sh.heads * p.vt <= 1024 ? 2 : 4;
-    delta_scan_kernel<KT><<<dim3((p.vt + per - 1) / per, sh.heads, rr.batch), per * 64, 0, s>>>(sh, io, rr, frags, decay, o, p.vt, p.frags);
+    // wavefronts of a block share a head's fragments; fewer per block where there are few blocks
+    uint32_t waves = 1;
+    while (waves < 8 && waves < p.vt && (uint64_t)rr.batch * sh.heads * ((p.vt + waves - 1) / waves) > 256) waves *= 2;
+    const size_t scan_lds = scan_buffers(KT) * (6 * KT + 3 + 2 * (size_t)waves) * 1024;
+    if constexpr (KT >= 4) {
+        static bool configured = false;
+        if (!configured) {
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&delta_scan_kernel<KT>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            configured = true;
+        }
+    }
+    delta_scan_kernel<KT><<<dim3((p.vt + waves - 1) / waves, sh.heads, rr.batch), waves * 64, scan_lds, s>>>(sh, io, rr, frags, decay, o, p.vt, p.frags);
     delta_gate_kernel<T><<<rr.rows, 256, 0, s>>>(sh, io, rr, o);
 }
 

@@ -197,10 +197,17 @@ struct StreamParams {
     uint16_t *out;
     float *part_o, *part_ml;                         // [slot][split][16 NQ][rank_p], [slot][split][16 NQ][2]: maximum, sum
     uint32_t splits;
+    int direct;                                      // one token per sequence, its heads in one block: block b is sequence b
 };
 
 template <int NQ>
-__device__ __forceinline__ bool stream_tile(const RaggedRows &rr, uint32_t heads, uint32_t slot, uint32_t *b_out, uint32_t *t0, uint32_t *n_rows) {
+__device__ __forceinline__ bool stream_tile(int direct, const RaggedRows &rr, uint32_t heads, uint32_t slot, uint32_t *b_out, uint32_t *t0, uint32_t *n_rows) {
+    if (direct) {
+        *b_out = slot;
+        *t0 = 0;
+        *n_rows = heads;
+        return true;
+    }
     auto base = [&](uint32_t b) { return (uint32_t)((uint64_t)rr.row_start[b] * heads / (16 * NQ)) + b; };
     uint32_t lo = 0, hi = rr.batch;
     while (hi - lo > 1) {
@@ -224,7 +231,7 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
     constexpr int NP = (KS * 4 + TPK - 1) / TPK;
     extern __shared__ __attribute__((aligned(16))) uint16_t stage[];        // [2][32][PITCH]
     uint32_t b, t0, n_rows;
-    if (!stream_tile<NQ>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
+    if (!stream_tile<NQ>(p.direct, rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
     const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), qt = wave / DH, dh = wave % DH, g = lane / 16, c = lane % 16;
     const uint32_t row0 = rr.row_start[b], H = sh.heads;
     const uint32_t *table = rr.tables + (uint64_t)b * rr.max_blocks;
@@ -346,7 +353,7 @@ template <int NQ>
 __global__ void __launch_bounds__(128) latent_merge_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
     __shared__ float w[kMaxSplits];
     uint32_t b, t0, n_rows;
-    if (!stream_tile<NQ>(rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
+    if (!stream_tile<NQ>(p.direct, rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
     const uint32_t cl = blockIdx.y, col = t0 + cl;
     if (col >= n_rows) return;
     const uint64_t ps = (uint64_t)blockIdx.x * p.splits * 16 * NQ + cl;      // split s of this column: + s * 16 NQ
@@ -378,14 +385,15 @@ __global__ void __launch_bounds__(128) latent_merge_kernel(StreamParams p, Laten
 }
 
 struct StreamPlan {
-    int nq = 0;                                      // 0: the plain kernel
+    int nq = 0, direct = 0;                          // nq 0: the plain kernel
     uint32_t slots = 0, splits = 1;
 };
 StreamPlan stream_plan(const LatentShape &sh, uint32_t rows, uint32_t batch, uint32_t longest, int num_cus) {
     StreamPlan p;
     if (sh.rank_p > 512 || sh.rot_p > 64 || g_latent_form == 1) return p;
     p.nq = (uint64_t)longest * sh.heads <= 32 ? 2 : 4;
-    p.slots = (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nq)) + batch + 1;
+    p.direct = longest == 1 && rows == batch && sh.heads <= 16u * p.nq;
+    p.slots = p.direct ? batch : (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nq)) + batch + 1;
     // about two blocks per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NQ)
     const uint64_t used = std::max<uint64_t>(std::max<uint64_t>((uint64_t)rows * sh.heads / (16 * p.nq), batch), 1);
     const uint64_t want = ((uint64_t)(g_latent_blocks ? g_latent_blocks : 2) * num_cus + used - 1) / used;
@@ -649,7 +657,7 @@ void latent_attention(const void *qa, const void *pool, void *out, int is_f32, c
     if (!is_f32) {
         const StreamPlan plan = stream_plan(sh, rr.rows, rr.batch, max_new, num_cus);
         if (plan.nq) {
-            StreamParams p{(const uint16_t *)qa, (const uint16_t *)pool, (uint16_t *)out, (float *)workspace, nullptr, plan.splits};
+            StreamParams p{(const uint16_t *)qa, (const uint16_t *)pool, (uint16_t *)out, (float *)workspace, nullptr, plan.splits, plan.direct};
             if (p.splits > 1) p.part_ml = p.part_o + (uint64_t)plan.slots * plan.splits * 16 * plan.nq * sh.rank_p;
             if (sh.rank_p <= 64) launch_stream_ro<2>(p, sh, rr, plan, s);
             else if (sh.rank_p <= 128) launch_stream_ro<4>(p, sh, rr, plan, s);

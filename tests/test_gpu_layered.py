@@ -48,6 +48,7 @@ MECHANISMS = {
     "delta one head group": [lc.delta(heads=2, kv_heads=2, dim=16, vdim=32, conv=3)],
     "delta one kv head, no convolution history": [lc.delta(heads=5, kv_heads=1, dim=9, vdim=7, conv=1)],
     "delta wide": [lc.delta(heads=2, kv_heads=1, dim=130, vdim=260, conv=2)],
+    "delta 256": [lc.delta(heads=2, kv_heads=1, dim=256, vdim=48, conv=5)],
     "delta 128": [lc.delta(heads=4, kv_heads=2, dim=128, vdim=128, conv=4)],
     "delta with feed-forward": [lc.delta(mlp=lc.glu())],
     "latent": [lc.latent()],
