@@ -162,6 +162,18 @@ __device__ __forceinline__ v8bf transposed_keys(const uint16_t *rows, uint32_t p
     return __builtin_bit_cast(v8bf, v8s{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
 }
 
+// Loads into these registers complete here: inside a loop that has loads of its own in flight, the compiler would otherwise
+// wait for both at the first use of every iteration.
+template <int N>
+__device__ __forceinline__ void hold(v8bf (&r)[N]) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        v4u t = __builtin_bit_cast(v4u, r[i]);
+        asm volatile("" : "+v"(t));
+        r[i] = __builtin_bit_cast(v8bf, t);
+    }
+}
+
 // One online-softmax step of a column (query row): scores of eight keys per lane, lanes with equal lane % 16 share the
 // column.  Returns the factor for what was accumulated before; w receives the weights as two bf16 terms whose sum keeps
 // about 16 bits of them.
@@ -226,9 +238,9 @@ __device__ __forceinline__ bool stream_tile(int direct, const RaggedRows &rr, ui
 template <int RK, int RO, int NQ, int DH>
 __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_eu(2)))
     latent_stream_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
-    constexpr int KS = RK + RO, VT = 2 * RK / DH, WIDTH = KS * 32, PITCH = WIDTH + 8, TPK = NQ * DH * 64 / kKeys, PIECES = KS * 4 / TPK;
-    static_assert(PIECES * TPK == KS * 4 || TPK > 4, "whole rows");
-    constexpr int NP = (KS * 4 + TPK - 1) / TPK;
+    constexpr int KS = RK + RO, VT = 2 * RK / DH, WIDTH = KS * 32, PITCH = WIDTH + 8, TPK = NQ * DH * 64 / kKeys;
+    static_assert(VT % 4 == 0, "value tiles go in groups of four");
+    constexpr int NP = (KS * 4 + TPK - 1) / TPK, KG = 2;
     extern __shared__ __attribute__((aligned(16))) uint16_t stage[];        // [2][32][PITCH]
     uint32_t b, t0, n_rows;
     if (!stream_tile<NQ>(p.direct, rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
@@ -284,6 +296,7 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
     v8bf qf[KS];
 #pragma unroll
     for (int s = 0; s < KS; ++s) qf[s] = *(const v8bf *)(q + s * 32);
+    hold(qf);
     const float factor = sh.scale * kLog2e;
     float m = -INFINITY, l = 0.0f;
     v4f o[VT];
@@ -299,12 +312,28 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
             id_next = page_of(k0 + 2 * kKeys + key);
         }
         const uint16_t *rows = stage + buf * kKeys * PITCH;
+        // operands are read a group ahead of the multiplies that take them
         v4f acc[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
+        v8bf kf[2][KG][2];
+        auto read_keys = [&](int s0, v8bf (&d)[KG][2]) {
 #pragma unroll
-        for (int s = 0; s < KS; ++s)
+            for (int s = 0; s < KG; ++s)
 #pragma unroll
-            for (int kt = 0; kt < 2; ++kt)
-                acc[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const v8bf *)(rows + (kt * 16 + c) * PITCH + s * 32 + 8 * g), qf[s], acc[kt], 0, 0, 0);
+                for (int kt = 0; kt < 2; ++kt)
+                    if (s0 + s < KS) d[s][kt] = *(const v8bf *)(rows + (kt * 16 + c) * PITCH + (s0 + s) * 32 + 8 * g);
+        };
+        read_keys(0, kf[0]);
+#pragma unroll
+        for (int s0 = 0; s0 < KS; s0 += KG) {
+            if (s0 + KG < KS) read_keys(s0 + KG, kf[(s0 / KG + 1) & 1]);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int s = 0; s < KG; ++s)
+#pragma unroll
+                for (int kt = 0; kt < 2; ++kt)
+                    if (s0 + s < KS) acc[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[(s0 / KG) & 1][s][kt], qf[s0 + s], acc[kt], 0, 0, 0);
+            __builtin_amdgcn_sched_barrier(0);
+        }
         float sc[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
@@ -317,11 +346,21 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
 #pragma unroll
             for (int t = 0; t < VT; ++t) o[t] *= fix;
         }
+        v8bf vf[2][4];
 #pragma unroll
-        for (int t = 0; t < VT; ++t) {
-            const v8bf v = transposed_keys(rows + (dh * VT + t) * 16, PITCH, lane);
-            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_hi, o[t], 0, 0, 0);
-            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, w_lo, o[t], 0, 0, 0);
+        for (int i = 0; i < 4; ++i) vf[0][i] = transposed_keys(rows + (dh * VT + i) * 16, PITCH, lane);
+#pragma unroll
+        for (int t = 0; t < VT; t += 4) {
+            if (t + 4 < VT) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) vf[(t / 4 + 1) & 1][i] = transposed_keys(rows + (dh * VT + t + 4 + i) * 16, PITCH, lane);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o[t + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[(t / 4) & 1][i], w_hi, o[t + i], 0, 0, 0);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o[t + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[(t / 4) & 1][i], w_lo, o[t + i], 0, 0, 0);
+            __builtin_amdgcn_sched_barrier(0);
         }
         if (more) put(buf ^ 1);
         __syncthreads();
@@ -499,6 +538,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
             qf[qi][s] = *(const v8bf *)(src + s * 32);
         }
     }
+#pragma unroll
+    for (int qi = 0; qi < NQ; ++qi) hold(qf[qi]);
     const int32_t w_lo_pos = p0 + (int32_t)(t0 + wave * 32 < n ? t0 + wave * 32 : n - 1);
     const int32_t w_hi_pos = p0 + (int32_t)(t0 + wave * 32 + 31 < n ? t0 + wave * 32 + 31 : n - 1);
 
