@@ -11,7 +11,7 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
-int g_latent_blocks = 0;     // tuning: blocks per compute unit the split of the keys aims at (default 2)
+int g_latent_blocks = 0;     // tuning: blocks per compute unit the split of the keys aims at
 int g_latent_form = 0;       // tuning: 1 keeps the plain attention kernel, 2 the absorbed form for every pass, 3 takes the
                              // expanded form wherever it can run
 
@@ -234,17 +234,20 @@ __device__ __forceinline__ bool stream_tile(int direct, const RaggedRows &rr, ui
 }
 
 // RK, RO: rank_p and rot_p in units of 32.  DH wavefronts share a column tile: each forms the scores (registers for the
-// whole query row) and sums a 1 / DH share of the latent dims.
-template <int RK, int RO, int NQ, int DH>
-__global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_eu(2)))
+// whole query row) and sums a 1 / DH share of the latent dims.  GR groups of NQ DH wavefronts take a part of the block's keys
+// each and meet in LDS at the end, which keeps partial results out of memory.
+template <int RK, int RO, int NQ, int DH, int GR>
+__global__ void __launch_bounds__(NQ * DH * GR * 64) __attribute__((amdgpu_waves_per_eu(2)))
     latent_stream_kernel(StreamParams p, LatentShape sh, RaggedRows rr) {
     constexpr int KS = RK + RO, VT = 2 * RK / DH, WIDTH = KS * 32, PITCH = WIDTH + 8, TPK = NQ * DH * 64 / kKeys;
     static_assert(VT % 4 == 0, "value tiles go in groups of four");
     constexpr int NP = (KS * 4 + TPK - 1) / TPK, KG = 2;
-    extern __shared__ __attribute__((aligned(16))) uint16_t stage[];        // [2][32][PITCH]
+    extern __shared__ __attribute__((aligned(16))) uint16_t stage_all[];    // [GR][2][32][PITCH]
     uint32_t b, t0, n_rows;
     if (!stream_tile<NQ>(p.direct, rr, sh.heads, blockIdx.x, &b, &t0, &n_rows)) return;
-    const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), qt = wave / DH, dh = wave % DH, g = lane / 16, c = lane % 16;
+    const int group = GR == 1 ? 0 : __builtin_amdgcn_readfirstlane(threadIdx.x / (NQ * DH * 64)), tid = threadIdx.x % (NQ * DH * 64);
+    const int lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), qt = wave / DH, dh = wave % DH, g = lane / 16, c = lane % 16;
+    uint16_t *stage = stage_all + group * 2 * kKeys * PITCH;
     const uint32_t row0 = rr.row_start[b], H = sh.heads;
     const uint32_t *table = rr.tables + (uint64_t)b * rr.max_blocks;
     const uint32_t last_row = t0 + 16 * NQ - 1 < n_rows ? t0 + 16 * NQ - 1 : n_rows - 1;
@@ -257,23 +260,30 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
     }
     const uint64_t ps = ((uint64_t)blockIdx.x * p.splits + blockIdx.y) * 16 * NQ + qt * 16 + c;
     if (k_lo >= k_hi) {                              // a split without keys (never the only one)
-        if (dh == 0 && g == 0) {
+        if (group == 0 && dh == 0 && g == 0) {
             p.part_ml[2 * ps] = -INFINITY;
             p.part_ml[2 * ps + 1] = 0.0f;
         }
         return;
+    }
+    const int32_t k_last = k_hi - 1;
+    int32_t steps = (k_hi - k_lo + kKeys - 1) / kKeys;
+    if (GR > 1) {                                    // this group's keys; every group runs the same number of steps
+        steps = (steps + GR - 1) / GR;
+        k_lo += group * steps * kKeys;
+        k_hi = k_lo + steps * kKeys < k_hi ? k_lo + steps * kKeys : k_hi;
     }
     // staging: TPK threads per key, 16 bytes each at a time; keys past the walk repeat its last one (their weight is zero)
     const int key = tid / TPK, part = tid % TPK;
     v4u st[NP];
     bool lost = false;                               // the staged position has no page: NaN, never a silent zero
     auto page_of = [&](int32_t j) -> uint32_t {
-        j = j < k_hi ? j : k_hi - 1;
+        j = j <= k_last ? j : k_last;
         const uint32_t blk = (uint32_t)j / rr.block_size;
         return blk < rr.max_blocks ? table[blk] : 0xffffffffu;
     };
     auto fetch = [&](int32_t j, uint32_t id) {
-        j = j < k_hi ? j : k_hi - 1;
+        j = j <= k_last ? j : k_last;
         lost = id >= rr.num_blocks;
         const uint16_t *src = p.pool + ((uint64_t)(lost ? 0 : id) * rr.block_size + (uint32_t)j % rr.block_size) * WIDTH + part * 8;
 #pragma unroll
@@ -305,8 +315,8 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
     put(0);
     __syncthreads();
     int buf = 0;
-    for (int32_t k0 = k_lo; k0 < k_hi; k0 += kKeys, buf ^= 1) {
-        const bool more = k0 + kKeys < k_hi;
+    for (int32_t it = 0, k0 = k_lo; it < steps; ++it, k0 += kKeys, buf ^= 1) {
+        const bool more = it + 1 < steps;
         if (more) {
             fetch(k0 + kKeys + key, id_next);
             id_next = page_of(k0 + 2 * kKeys + key);
@@ -367,6 +377,27 @@ __global__ void __launch_bounds__(NQ * DH * 64) __attribute__((amdgpu_waves_per_
     }
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
+    if constexpr (GR == 2) {
+        constexpr int OP = RK * 32 + 4;              // pitch of an exchanged row
+        static_assert(16 * NQ * (OP * 4 + 8) <= GR * 2 * kKeys * PITCH * 2, "the exchange fits the stages");
+        float *xo = (float *)stage_all, *xm = xo + 16 * NQ * OP;
+        if (group == 1) {
+            if (g == 0) {
+                xm[(qt * 16 + c) * 2] = m;
+                xm[(qt * 16 + c) * 2 + 1] = l;
+            }
+#pragma unroll
+            for (int t = 0; t < VT; ++t) *(v4f *)(xo + (qt * 16 + c) * OP + (dh * VT + t) * 16 + 4 * g) = o[t];
+        }
+        __syncthreads();
+        if (group == 1) return;
+        const float m1 = xm[(qt * 16 + c) * 2], l1 = xm[(qt * 16 + c) * 2 + 1], mx = fmaxf(m, m1), ref = mx == -INFINITY ? 0.0f : mx;
+        const float f0 = exp2f(m - ref), f1 = exp2f(m1 - ref);
+        m = mx;
+        l = l * f0 + l1 * f1;
+#pragma unroll
+        for (int t = 0; t < VT; ++t) o[t] = o[t] * f0 + *(const v4f *)(xo + (qt * 16 + c) * OP + (dh * VT + t) * 16 + 4 * g) * f1;
+    }
     if (p.splits > 1) {
         if (dh == 0 && g == 0) {
             p.part_ml[2 * ps] = m;
@@ -423,6 +454,9 @@ __global__ void __launch_bounds__(128) latent_merge_kernel(StreamParams p, Laten
     }
 }
 
+// Key groups of a block: two for the few query rows of a decode step
+constexpr int stream_groups(int nq) { return nq == 2 ? 2 : 1; }
+
 struct StreamPlan {
     int nq = 0, direct = 0;                          // nq 0: the plain kernel
     uint32_t slots = 0, splits = 1;
@@ -433,25 +467,26 @@ StreamPlan stream_plan(const LatentShape &sh, uint32_t rows, uint32_t batch, uin
     p.nq = (uint64_t)longest * sh.heads <= 32 ? 2 : 4;
     p.direct = longest == 1 && rows == batch && sh.heads <= 16u * p.nq;
     p.slots = p.direct ? batch : (uint32_t)((uint64_t)rows * sh.heads / (16 * p.nq)) + batch + 1;
-    // about two blocks per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NQ)
+    // wavefronts for about two blocks of one key group per compute unit, at least 128 keys each; the number of used slots is close to rows * heads / (16 NQ)
     const uint64_t used = std::max<uint64_t>(std::max<uint64_t>((uint64_t)rows * sh.heads / (16 * p.nq), batch), 1);
-    const uint64_t want = ((uint64_t)(g_latent_blocks ? g_latent_blocks : 2) * num_cus + used - 1) / used;
-    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (sh.window + 127) / 128, kMaxSplits}));
+    const uint64_t per_cu = g_latent_blocks ? g_latent_blocks : 3 - stream_groups(p.nq), least = 128 * stream_groups(p.nq);
+    const uint64_t want = (per_cu * num_cus + used - 1) / used;
+    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (sh.window + least - 1) / least, kMaxSplits}));
     return p;
 }
 
 template <int RK, int RO, int NQ>
 void launch_stream(const StreamParams &p, const LatentShape &sh, const RaggedRows &rr, uint32_t slots, hipStream_t s) {
-    constexpr int DH = RK == 16 ? 2 : 1;
-    constexpr size_t lds = 2ull * kKeys * ((RK + RO) * 32 + 8) * 2;
+    constexpr int DH = RK == 16 ? 2 : 1, GR = stream_groups(NQ);
+    constexpr size_t lds = GR * 2ull * kKeys * ((RK + RO) * 32 + 8) * 2;
     if constexpr (lds > 65536) {
         static bool configured = false;
         if (!configured) {
-            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_stream_kernel<RK, RO, NQ, DH>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_stream_kernel<RK, RO, NQ, DH, GR>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
             configured = true;
         }
     }
-    latent_stream_kernel<RK, RO, NQ, DH><<<dim3(slots, p.splits), NQ * DH * 64, lds, s>>>(p, sh, rr);
+    latent_stream_kernel<RK, RO, NQ, DH, GR><<<dim3(slots, p.splits), NQ * DH * GR * 64, lds, s>>>(p, sh, rr);
     if (p.splits > 1) latent_merge_kernel<NQ><<<dim3(slots, 16 * NQ), 128, 0, s>>>(p, sh, rr);
 }
 template <int RK, int RO>
