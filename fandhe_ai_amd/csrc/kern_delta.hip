@@ -225,58 +225,69 @@ __device__ __forceinline__ v4f mfma4(const v4f &a, const v4f &b, v4f c) {
 }
 
 // silu(convolution) of `cols` channels from c0 on for the chunk's tokens t0 .. into dst [32][pitch]; zeros for tokens past
-// the end and columns up to cols_p.
-template <typename T, int MAXTAPS>
+// the end and columns up to cols_p.  A thread takes TG tokens of two neighbouring channels (one where they are not aligned).
+template <typename T, int MAXTAPS, int TG>
 __device__ __forceinline__ void conv_chunk(float *dst, uint32_t pitch, const T *__restrict__ y, uint32_t ld, const T *__restrict__ ring,
                                            const float *__restrict__ conv, uint32_t taps, uint32_t channels, uint32_t c0, uint32_t cols,
                                            uint32_t cols_p, uint64_t row0, uint32_t t0, uint32_t n, uint32_t p0) {
-    for (uint32_t item = threadIdx.x; item < cols_p * 4; item += 256) {
-        const uint32_t col = item % cols_p, tg = item / cols_p * 8;
-        if (col >= cols) {
+    constexpr uint32_t NG = kChunk / TG;
+    if (MAXTAPS != 0 && ((ld | channels | c0 | cols) & 1) == 0) {
+        constexpr int NX = TG + (MAXTAPS ? MAXTAPS : 1) - 1, MT = MAXTAPS ? MAXTAPS : 1;
+        const uint32_t pairs = cols_p / 2;
+        for (uint32_t item = threadIdx.x; item < pairs * NG; item += 256) {
+            const uint32_t col = item % pairs * 2, tg = item / pairs * TG;
+            const uint32_t c = c0 + (col < cols ? col : 0);
+            v2f w[MT], x[NX];
 #pragma unroll
-            for (int j = 0; j < 8; ++j) dst[(tg + j) * pitch + col] = 0.0f;
-            continue;
-        }
-        const uint32_t c = c0 + col;
-        if constexpr (MAXTAPS == 0) {
-            for (uint32_t j = 0; j < 8; ++j) {
-                const uint32_t t = t0 + tg + j;
-                dst[(tg + j) * pitch + col] = t < n ? conv_silu(y, ld, ring, conv, taps, channels, c, row0, t, p0 + t) : 0.0f;
-            }
-        } else {
-            float w[MAXTAPS], x[8 + MAXTAPS - 1];
-#pragma unroll
-            for (int i = 0; i < MAXTAPS; ++i) w[i] = i < (int)taps ? conv[(uint64_t)c * taps + taps - 1 - i] : 0.0f;      // w[back]
-#pragma unroll
-            for (int j = 0; j < 8 + MAXTAPS - 1; ++j) {
-                const int t = (int)(t0 + tg) + j - (MAXTAPS - 1);
-                float v = 0.0f;
-                if (t >= 0) {
-                    if (t < (int)n) v = load_as_f32(y + (row0 + t) * ld + c);
-                } else if ((int)p0 + t >= 0 && -t < (int)taps) {
-                    v = load_as_f32(ring + (uint64_t)((p0 + t) % taps) * channels + c);
+            for (int j = 0; j < NX; ++j) {
+                const int t = (int)(t0 + tg) + j - (MT - 1);
+                const bool inside = t >= 0 && t < (int)n, before = t < 0 && (int)p0 + t >= 0 && -t < (int)taps;
+                const T *src = before ? ring + (uint64_t)((p0 + t) % taps) * channels + c : y + (row0 + (inside ? t : 0)) * ld + c;
+                v2f v;
+                if constexpr (std::is_same<T, float>::value) {
+                    v = *(const v2f *)src;
+                } else {
+                    const uint32_t u = *(const uint32_t *)src;
+                    v = v2f{bf16_lo(u), bf16_hi(u)};
                 }
-                x[j] = v;
+                x[j] = inside || before ? v : v2f{0.0f, 0.0f};
             }
 #pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                float acc = 0.0f;
+            for (int i = 0; i < MT; ++i)
 #pragma unroll
-                for (int i = MAXTAPS - 1; i >= 0; --i) acc = fmaf(w[i], x[j + MAXTAPS - 1 - i], acc);
-                dst[(tg + j) * pitch + col] = t0 + tg + j < n ? fast_silu(acc) : 0.0f;
+                for (int e = 0; e < 2; ++e) w[i][e] = i < (int)taps ? conv[(uint64_t)(c + e) * taps + taps - 1 - i] : 0.0f;      // w[back]
+#pragma unroll
+            for (int j = 0; j < TG; ++j) {
+                v2f r;
+#pragma unroll
+                for (int e = 0; e < 2; ++e) {
+                    float acc = 0.0f;
+#pragma unroll
+                    for (int i = MT - 1; i >= 0; --i) acc = fmaf(w[i][e], x[j + MT - 1 - i][e], acc);
+                    r[e] = t0 + tg + j < n && col < cols ? fast_silu(acc) : 0.0f;
+                }
+                *(v2f *)(dst + (tg + j) * pitch + col) = r;
             }
+        }
+        return;
+    }
+    for (uint32_t item = threadIdx.x; item < cols_p * NG; item += 256) {
+        const uint32_t col = item % cols_p, tg = item / cols_p * TG;
+        for (uint32_t j = 0; j < TG; ++j) {
+            const uint32_t t = t0 + tg + j;
+            dst[(tg + j) * pitch + col] = t < n && col < cols ? conv_silu(y, ld, ring, conv, taps, channels, c0 + col, row0, t, p0 + t) : 0.0f;
         }
     }
 }
 
+// One block per (chunk, q / k head); the heads that share it are taken one after the other.
 template <typename T, int KT, int MAXTAPS>
 __global__ void __launch_bounds__(256)
-    delta_chunk_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, float *__restrict__ frags, float *__restrict__ chunk_decay, uint32_t vt,
-                       uint32_t n_frags) {
-    constexpr uint32_t DP = KT * 16, PITCH = DP + 4;
+    delta_chunk_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, float *__restrict__ frags, float *__restrict__ chunk_decay, uint32_t n_frags) {
+    constexpr uint32_t DP = KT * 16, PITCH = DP + 4, VS = 64, VPITCH = VS + 4;
     extern __shared__ __attribute__((aligned(16))) float lds[];
-    float *lk = lds, *lq = lk + 32 * PITCH;          // K; Q, then V in slices of DP columns
-    float *la = lq + 32 * PITCH, *lt = la + 32 * 36; // A and T, pitch 36
+    float *lk = lds, *lq = lk + 32 * PITCH, *lv = lq + 32 * PITCH;          // K, Q, 64 columns of V
+    float *la = lv + 32 * VPITCH, *lt = la + 32 * 36;                       // A and T, pitch 36
     __shared__ float rq[32], rk[32], beta[32], G[32], qs[32], ks[32], ke[32];   // qs = rq exp(G), ks = rk exp(G), ke = rk exp(G_C - G)
     // the slot's sequence and chunk
     uint32_t lo = 0, hi = rr.batch;
@@ -287,33 +298,13 @@ __global__ void __launch_bounds__(256)
     }
     const uint32_t b = lo, row0 = rr.row_start[b], n = rr.row_start[b + 1] - row0, t0 = (blockIdx.x - slot_base(rr, b)) * kChunk;
     if (n < kChunkFrom || t0 >= n) return;
-    const uint32_t h = blockIdx.y, hk = h / (sh.heads / sh.kv_heads), dim = sh.dim, vdim = sh.vdim, channels = sh.qkv();
+    const uint32_t hk = blockIdx.y, share = sh.heads / sh.kv_heads, dim = sh.dim, vdim = sh.vdim, channels = sh.qkv();
     const T *y = (const T *)io.y, *ring = (const T *)io.ring + (uint64_t)rr.state_slot[b] * sh.taps * channels;
     const uint32_t p0 = (uint32_t)rr.pos[row0];
     const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, lr = lane % 16, g = lane / 16;
-    v4f *out = (v4f *)(frags + ((uint64_t)blockIdx.x * sh.heads + h) * n_frags * 256) + lane;
-    auto put = [&](uint32_t f, const v4f &v) { out[f * 64] = v; };
 
-    conv_chunk<T, MAXTAPS>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, hk * dim, dim, DP, row0, t0, n, p0);
-    conv_chunk<T, MAXTAPS>(lk, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, (sh.kv_heads + hk) * dim, dim, DP, row0, t0, n, p0);
-    if (tid < 64) {                                  // lanes past 31 only keep the scan whole
-        const uint32_t t = t0 + lane;
-        float lg = 0.0f, be = 0.0f;
-        if (lane < 32 && t < n) {
-            const float *ba = io.ba + (uint64_t)(row0 + t) * io.ld_ba;
-            be = sigmoid_f32(ba[h]);
-            lg = log_decay(io.a_log[h], ba[sh.heads + h] + io.dt_bias[h]);
-        }
-#pragma unroll
-        for (int off = 1; off < 32; off <<= 1) {
-            const float o = __shfl_up(lg, off, 64);
-            if (lane >= off) lg += o;
-        }
-        if (lane < 32) {
-            beta[lane] = be;
-            G[lane] = lg;
-        }
-    }
+    conv_chunk<T, MAXTAPS, 8>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, hk * dim, dim, DP, row0, t0, n, p0);
+    conv_chunk<T, MAXTAPS, 8>(lk, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, (sh.kv_heads + hk) * dim, dim, DP, row0, t0, n, p0);
     __syncthreads();
     {   // four threads per row of Q and of K
         const float *row = (tid < 128 ? lq : lk) + ((tid % 128) / 4) * PITCH;
@@ -323,127 +314,161 @@ __global__ void __launch_bounds__(256)
         sq += __shfl_xor(sq, 2, 64);
         if (tid % 4 == 0) {
             const float r = 1.0f / sqrtf(sq + 1e-6f);
-            const int i = (tid % 128) / 4;
-            if (tid < 128) {
-                rq[i] = r / sqrtf((float)dim);
-                qs[i] = rq[i] * expf(G[i]);
-            } else {
-                rk[i] = r;
-                ks[i] = r * expf(G[i]);
-                ke[i] = r * expf(G[31] - G[i]);
-            }
+            if (tid < 128) rq[tid / 4] = r / sqrtf((float)dim);
+            else rk[(tid - 128) / 4] = r;
         }
     }
-    __syncthreads();
     // (K K^T) tiles 00, 10, 11 and (K Q^T) tiles: wave 0: both 00, 1: KK 10, 2: QK 10, 3: both 11.  Rows of the result are
     // j (the keys), its column i: D order of the transpose is A order of the matrix.
     auto dot_tile = [&](const float *rows_j, const float *rows_i) {
         v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
-        for (uint32_t k = g; k < DP; k += 4)
-            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(rows_j[lr * PITCH + k], rows_i[lr * PITCH + k], acc, 0, 0, 0);
+        rows_j += lr * PITCH + g;
+        rows_i += lr * PITCH + g;
+#pragma unroll
+        for (uint32_t k = 0; k < DP; k += 4) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(rows_j[k], rows_i[k], acc, 0, 0, 0);
         return acc;
     };
     const int ti = wave == 0 ? 0 : 1, tj = wave == 3 ? 1 : 0, i_ = ti * 16 + lr;
-    if (wave != 2) {
-        const v4f d = dot_tile(lk + tj * 16 * PITCH, lk + ti * 16 * PITCH);
+    v4f kk = v4f{0.f, 0.f, 0.f, 0.f}, qk = kk;
+    if (wave != 2) kk = dot_tile(lk + tj * 16 * PITCH, lk + ti * 16 * PITCH);
+    if (wave != 1) qk = dot_tile(lk + tj * 16 * PITCH, lq + ti * 16 * PITCH);
+
+    for (uint32_t h = hk * share; h < (hk + 1) * share; ++h) {
+        v4f *out = (v4f *)(frags + ((uint64_t)blockIdx.x * sh.heads + h) * n_frags * 256) + lane;
+        auto put = [&](uint32_t f, const v4f &v) { out[f * 64] = v; };
+        __syncthreads();                             // norms are there; the previous head's scalars and A, T, V are read
+        if (tid < 64) {                              // lanes past 31 only keep the scan whole
+            const uint32_t t = t0 + lane;
+            float lg = 0.0f, be = 0.0f;
+            if (lane < 32 && t < n) {
+                const float *ba = io.ba + (uint64_t)(row0 + t) * io.ld_ba;
+                be = sigmoid_f32(ba[h]);
+                lg = log_decay(io.a_log[h], ba[sh.heads + h] + io.dt_bias[h]);
+            }
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int j = tj * 16 + 4 * g + e;
-            la[i_ * 36 + j] = j < i_ ? beta[i_] * fast_exp(G[i_] - G[j]) * rk[i_] * rk[j] * d[e] : 0.0f;
-        }
-    }
-    if (wave != 1) {
-        v4f d = dot_tile(lk + tj * 16 * PITCH, lq + ti * 16 * PITCH);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int j = tj * 16 + 4 * g + e;
-            d[e] = j <= i_ ? fast_exp(G[i_] - G[j]) * rq[i_] * rk[j] * d[e] : 0.0f;
-        }
-        put(6 * KT + ti + tj, d);
-    }
-    // exp(G) Q and the decayed K^T
-    for (uint32_t f = wave; f < 2 * KT; f += 4) {
-        const uint32_t rt = f / KT, kt = f % KT, i = rt * 16 + lr;
-        put(2 * KT + f, *(const v4f *)(lq + i * PITCH + kt * 16 + 4 * g) * qs[i]);
-        const uint32_t dt = f / 2, ct = f % 2;
-        v4f v;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const uint32_t j = ct * 16 + 4 * g + e;
-            v[e] = lk[j * PITCH + dt * 16 + lr] * ke[j];
-        }
-        put(4 * KT + f, v);
-    }
-    if (tid == 0) chunk_decay[(uint64_t)blockIdx.x * sh.heads + h] = expf(G[31]);
-    __syncthreads();
-    // T = (I + A)^-1: the diagonal blocks column by column (lanes 0 - 15, 16 - 31), then T10 = -T11 A10 T00
-    if (wave == 0) {
-        if (lane < 32) {
-            const int o = (lane / 16) * 16;
-            float x[16];
-#pragma unroll
-            for (int i = 0; i < 16; ++i) {
-                float v = i == lr ? 1.0f : 0.0f;
-#pragma unroll
-                for (int j = 0; j < i; ++j) v = fmaf(-la[(o + i) * 36 + o + j], x[j], v);
-                x[i] = v;
-                lt[(o + i) * 36 + o + lr] = v;
+            for (int off = 1; off < 32; off <<= 1) {
+                const float o = __shfl_up(lg, off, 64);
+                if (lane >= off) lg += o;
+            }
+            const float last = __shfl(lg, 31, 64);
+            if (lane < 32) {
+                beta[lane] = be;
+                G[lane] = lg;
+                qs[lane] = rq[lane] * expf(lg);
+                ks[lane] = rk[lane] * expf(lg);
+                ke[lane] = rk[lane] * expf(last - lg);
             }
         }
-        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
-        __builtin_amdgcn_wave_barrier();
-        v4f x = v4f{0.f, 0.f, 0.f, 0.f}, t00, t10 = x;
+        __syncthreads();
+        if (wave != 2) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) t00[e] = lt[(4 * g + e) * 36 + lr];
-        x = mfma4(*(const v4f *)(la + (16 + lr) * 36 + 4 * g), t00, x);
-        t10 = mfma4(*(const v4f *)(lt + (16 + lr) * 36 + 16 + 4 * g), x, t10);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            lt[(16 + 4 * g + e) * 36 + lr] = -t10[e];
-            lt[(4 * g + e) * 36 + 16 + lr] = 0.0f;
+            for (int e = 0; e < 4; ++e) {
+                const int j = tj * 16 + 4 * g + e;
+                la[i_ * 36 + j] = j < i_ ? beta[i_] * fast_exp(G[i_] - G[j]) * rk[i_] * rk[j] * kk[e] : 0.0f;
+            }
         }
-    }
-    __syncthreads();
-    // -W^T = -K'^T T^T, K' = diag(beta exp(G) rk) K: the columns of the result are tokens, so its D order is W's A order
-    v4f tf[2][2];                                    // T fragments: second operand of W^T, first operand of T V
+        if (wave != 1) {
+            v4f d;
 #pragma unroll
-    for (int rt = 0; rt < 2; ++rt)
-#pragma unroll
-        for (int ct = 0; ct < 2; ++ct) {
-            tf[rt][ct] = *(const v4f *)(lt + (rt * 16 + lr) * 36 + ct * 16 + 4 * g);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) tf[rt][ct][e] *= beta[ct * 16 + 4 * g + e];
+            for (int e = 0; e < 4; ++e) {
+                const int j = tj * 16 + 4 * g + e;
+                d[e] = j <= i_ ? fast_exp(G[i_] - G[j]) * rq[i_] * rk[j] * qk[e] : 0.0f;
+            }
+            put(6 * KT + ti + tj, d);
         }
-    for (uint32_t f = wave; f < 2 * KT; f += 4) {
-        const uint32_t rt = f / KT, kt = f % KT;
-        v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
-        for (uint32_t ct = 0; ct <= rt; ++ct) {
-            v4f kf;
+        // exp(G) Q and the decayed K^T
+        for (uint32_t f = wave; f < 2 * KT; f += 4) {
+            const uint32_t rt = f / KT, kt = f % KT, i = rt * 16 + lr;
+            put(2 * KT + f, *(const v4f *)(lq + i * PITCH + kt * 16 + 4 * g) * qs[i]);
+            const uint32_t dt = f / 2, ct = f % 2;
+            v4f v;
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const uint32_t j = ct * 16 + 4 * g + e;
-                kf[e] = -lk[j * PITCH + kt * 16 + lr] * ks[j];
+                v[e] = lk[j * PITCH + dt * 16 + lr] * ke[j];
             }
-            acc = mfma4(kf, rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], acc);
+            put(4 * KT + f, v);
         }
-        put(f, acc);
-    }
-    // T diag(beta) V, DP columns of V at a time in Q's place (all reads of Q are behind the barriers above)
-    for (uint32_t v0 = 0; v0 < vdim; v0 += DP) {
-        const uint32_t cols = vdim - v0 < DP ? vdim - v0 : DP, cols_p = (cols + 15) / 16 * 16;
-        if (v0) __syncthreads();
-        conv_chunk<T, MAXTAPS>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, 2 * sh.kv_heads * dim + h * vdim + v0, cols, cols_p, row0, t0, n, p0);
+        if (tid == 0) chunk_decay[(uint64_t)blockIdx.x * sh.heads + h] = expf(G[31]);
+        // the first columns of V, whose loads travel under the inversion
+        const uint32_t vc0 = 2 * sh.kv_heads * dim + h * vdim;
+        auto conv_v = [&](uint32_t v0) {
+            const uint32_t cols = vdim - v0 < VS ? vdim - v0 : VS;
+            conv_chunk<T, MAXTAPS, 4>(lv, VPITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, vc0 + v0, cols, (cols + 15) / 16 * 16, row0, t0, n, p0);
+        };
+        conv_v(0);
         __syncthreads();
-        for (uint32_t f = wave; f < 2 * (cols_p / 16); f += 4) {
-            const uint32_t rt = f % 2, nt = f / 2;
+        // T = (I + A)^-1: the diagonal blocks column by column (lanes 0 - 15, 16 - 31), then T10 = -T11 A10 T00
+        if (wave == 0) {
+            if (lane < 32) {
+                const int o = (lane / 16) * 16;
+                float x[16];
+#pragma unroll
+                for (int i = 0; i < 16; ++i) {
+                    float v = i == lr ? 1.0f : 0.0f;
+#pragma unroll
+                    for (int j = 0; j < i; ++j) v = fmaf(-la[(o + i) * 36 + o + j], x[j], v);
+                    x[i] = v;
+                    lt[(o + i) * 36 + o + lr] = v;
+                }
+            }
+            __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+            __builtin_amdgcn_wave_barrier();
+            v4f x = v4f{0.f, 0.f, 0.f, 0.f}, t00, t10 = x;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) t00[e] = lt[(4 * g + e) * 36 + lr];
+            x = mfma4(*(const v4f *)(la + (16 + lr) * 36 + 4 * g), t00, x);
+            t10 = mfma4(*(const v4f *)(lt + (16 + lr) * 36 + 16 + 4 * g), x, t10);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                lt[(16 + 4 * g + e) * 36 + lr] = -t10[e];
+                lt[(4 * g + e) * 36 + 16 + lr] = 0.0f;
+            }
+        }
+        __syncthreads();
+        // -W^T = -K'^T T^T, K' = diag(beta exp(G) rk) K: the columns of the result are tokens, so its D order is W's A order
+        v4f tf[2][2];                                // T fragments: second operand of W^T, first operand of T V
+#pragma unroll
+        for (int rt = 0; rt < 2; ++rt)
+#pragma unroll
+            for (int ct = 0; ct < 2; ++ct) {
+                tf[rt][ct] = *(const v4f *)(lt + (rt * 16 + lr) * 36 + ct * 16 + 4 * g);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) tf[rt][ct][e] *= beta[ct * 16 + 4 * g + e];
+            }
+        for (uint32_t f = wave; f < 2 * KT; f += 4) {
+            const uint32_t rt = f / KT, kt = f % KT;
             v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
             for (uint32_t ct = 0; ct <= rt; ++ct) {
-                v4f vf;
+                v4f kf;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) vf[e] = lq[(ct * 16 + 4 * g + e) * PITCH + nt * 16 + lr];
-                acc = mfma4(rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], vf, acc);
+                for (int e = 0; e < 4; ++e) {
+                    const uint32_t j = ct * 16 + 4 * g + e;
+                    kf[e] = -lk[j * PITCH + kt * 16 + lr] * ks[j];
+                }
+                acc = mfma4(kf, rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], acc);
             }
-            put(6 * KT + 3 + (v0 / 16 + nt) * 2 + rt, acc);
+            put(f, acc);
+        }
+        // T diag(beta) V
+        for (uint32_t v0 = 0; v0 < vdim; v0 += VS) {
+            if (v0) {
+                __syncthreads();
+                conv_v(v0);
+                __syncthreads();
+            }
+            const uint32_t tiles = ((vdim - v0 < VS ? vdim - v0 : VS) + 15) / 16;
+            for (uint32_t f = wave; f < 2 * tiles; f += 4) {
+                const uint32_t rt = f % 2, nt = f / 2;
+                v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
+                for (uint32_t ct = 0; ct <= rt; ++ct) {
+                    v4f vf;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) vf[e] = lv[(ct * 16 + 4 * g + e) * VPITCH + nt * 16 + lr];
+                    acc = mfma4(rt == 0 ? tf[0][0] : ct == 0 ? tf[1][0] : tf[1][1], vf, acc);
+                }
+                put(6 * KT + 3 + (v0 / 16 + nt) * 2 + rt, acc);
+            }
         }
     }
 }
@@ -489,13 +514,15 @@ __global__ void __launch_bounds__(512)
         for (uint32_t i = 0; i < 2; ++i)
             __builtin_amdgcn_global_load_lds((gptr)(f + (SHARED + nt * 2 + i) * 64), (lptr)(l + (SHARED + wave * 2 + i) * 256), 16, 0, 0);
     };
+    float decay = chunk_decay[(uint64_t)slot0 * sh.heads + h];
     stage(0, 0);
     __builtin_amdgcn_s_waitcnt(0x0F70);              // this wavefront's fragments have landed
     __syncthreads();
     for (uint32_t c = 0; c < chunks; ++c) {
+        // the next decay is asked for ahead of the fragments: its use would otherwise wait for all of them
+        const float next_decay = chunk_decay[(uint64_t)(slot0 + (c + 1 < chunks ? c + 1 : c)) * sh.heads + h];
         if (NB == 2 && c + 1 < chunks) stage(c + 1, (c + 1) & 1);
         const v4f *f = (const v4f *)(lds + (uint64_t)(NB == 2 ? c & 1 : 0) * buf_frags * 256) + lane;
-        const float decay = chunk_decay[(uint64_t)(slot0 + c) * sh.heads + h];
         v4f u[2], r[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
         u[0] = f[(SHARED + wave * 2) * 64];
         u[1] = f[(SHARED + wave * 2 + 1) * 64];
@@ -517,30 +544,40 @@ __global__ void __launch_bounds__(512)
         r[1] = mfma4(f[(6 * KT + 2) * 64], u[1], r[1]);
 #pragma unroll
         for (int kt = 0; kt < KT; ++kt) S[kt] *= decay;
+        constexpr int GK = KT < 4 ? KT : 4, GROUPS = 2 * KT / GK;    // fragments are read a group ahead of the multiplies
+        v4f kd[2][GK];
+        auto read_kd = [&](int q, v4f (&d)[GK]) {
 #pragma unroll
-        for (int ct = 0; ct < 2; ++ct)
+            for (int i = 0; i < GK; ++i) d[i] = f[(4 * KT + (q / 2 * GK + i) * 2 + q % 2) * 64];
+        };
+        read_kd(0, kd[0]);
 #pragma unroll
-            for (int k4 = 0; k4 < KT; k4 += (KT < 4 ? KT : 4)) {
-                v4f a[4];
+        for (int q = 0; q < GROUPS; ++q) {
+            if (q + 1 < GROUPS) read_kd(q + 1, kd[(q + 1) & 1]);
+            __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-                for (int i = 0; i < (KT < 4 ? KT : 4); ++i) a[i] = f[(4 * KT + (k4 + i) * 2 + ct) * 64];
+            for (int e = 0; e < 4; ++e)
 #pragma unroll
-                for (int e = 0; e < 4; ++e)
+                for (int i = 0; i < GK; ++i)
+                    S[q / 2 * GK + i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kd[q & 1][i][e], u[q % 2][e], S[q / 2 * GK + i], 0, 0, 0);
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        auto store = [&]() {
 #pragma unroll
-                    for (int i = 0; i < (KT < 4 ? KT : 4); ++i) S[k4 + i] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i][e], u[ct][e], S[k4 + i], 0, 0, 0);
-            }
+            for (int rt = 0; rt < 2; ++rt)
 #pragma unroll
-        for (int rt = 0; rt < 2; ++rt)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const uint32_t t = c * kChunk + rt * 16 + 4 * g + e;
-                if (t < n && col < vdim) o[((uint64_t)(row0 + t) * sh.heads + h) * sh.vdim + col] = r[rt][e];
-            }
+                for (int e = 0; e < 4; ++e) {
+                    const uint32_t t = c * kChunk + rt * 16 + 4 * g + e;
+                    if (t < n && col < vdim) o[((uint64_t)(row0 + t) * sh.heads + h) * sh.vdim + col] = r[rt][e];
+                }
+        };
         if (NB == 1) {
             __syncthreads();
             if (c + 1 < chunks) stage(c + 1, 0);
         }
-        __builtin_amdgcn_s_waitcnt(0x0F70);          // the next chunk has landed (the read-outs' stores too)
+        __builtin_amdgcn_s_waitcnt(0x0F70);          // the next chunk has landed
+        decay = next_decay;
+        store();                                     // behind that wait: nothing waits for these stores before the next one
         __syncthreads();                             // ... for everybody, and nobody reads this chunk's any more
     }
     if (!real) return;
@@ -572,7 +609,7 @@ __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaShape sh, DeltaIo 
 template <typename T, int KT>
 void launch_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr, const ChunkPlan &p, hipStream_t s) {
     float *frags = io.scratch, *decay = frags + (uint64_t)p.slots * sh.heads * p.frags * 256, *o = decay + (((uint64_t)p.slots * sh.heads + 63) / 64) * 64;
-    const size_t lds = (2 * 32 * (KT * 16 + 4) + 2 * 32 * 36) * 4;
+    const size_t lds = (2 * 32 * (KT * 16 + 4) + 32 * 68 + 2 * 32 * 36) * 4;
     auto chunk = sh.taps <= 4 ? &delta_chunk_kernel<T, KT, 4> : &delta_chunk_kernel<T, KT, 0>;
     if (lds > 65536) {
         static bool configured = false;
@@ -582,7 +619,7 @@ void launch_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr
             configured = true;
         }
     }
-    chunk<<<dim3(p.slots, sh.heads), 256, lds, s>>>(sh, io, rr, frags, decay, p.vt, p.frags);
+    chunk<<<dim3(p.slots, sh.kv_heads), 256, lds, s>>>(sh, io, rr, frags, decay, p.frags);
     // wavefronts of a block share a head's fragments; fewer per block where there are few blocks
     uint32_t waves = 1;
     while (waves < 8 && waves < p.vt && (uint64_t)rr.batch * sh.heads * ((p.vt + waves - 1) / waves) > 256) waves *= 2;
