@@ -134,7 +134,7 @@ def build_nugelix(fa, be, config, max_tokens, batch):
     return dec
 
 
-def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, llama=True):
+def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "w8a8")):
     """Decode and prompt throughput of a Nugelix stack, and of the W8A8 decoder of equal width, feed-forward and depth."""
     lib = fa.capi.lib
     config, shape = LAYERED[size]
@@ -178,10 +178,11 @@ def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1
             dec.set_sequences(t, [length] * b)
         return set_rows
 
-    dec = build_nugelix(fa, be, config, most * pages * 16, most)
-    measure("nugelix bf16", dec, rows_of(most * pages))
-    dec.close()
-    if llama:
+    if "nugelix" in models:
+        dec = build_nugelix(fa, be, config, most * pages * 16, most)
+        measure("nugelix bf16", dec, rows_of(most * pages))
+        dec.close()
+    if "w8a8" in models:
         cfg = dict(MODEL, n_layers=layers, vocab=V, **shape)
         h, keep, _, _, num_blocks = build_decoder(fa, be, cfg, most, [ctx] * most, 64)
         dcfg = fa.capi.DecoderConfig(cfg["n_layers"], cfg["d_model"], cfg["n_heads"], cfg["n_kv_heads"], cfg["head_dim"], cfg["d_ffn"], V,
@@ -905,7 +906,8 @@ def main():
     ap.add_argument("--layered-size", choices=tuple(LAYERED) + ("all",), default="all",
                     help="with --only layered: the sizes of the Nugelix stack (and of the W8A8 decoder beside it)")
     ap.add_argument("--layered-phase", choices=("all", "decode", "prompt"), default="all",
-                    help="with --only layered: all, or one shape of one phase of the Nugelix stack (for a kernel trace)")
+                    help="with --only layered: all, or one shape of one phase (for a kernel trace)")
+    ap.add_argument("--layered-model", choices=("both", "nugelix", "w8a8"), default="both", help="with --only layered: one of the two decoders")
     a = ap.parse_args()
     if a.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (--gpus 1); nothing here shards across devices")
@@ -935,8 +937,9 @@ def main():
             be.close()
             return
         if a.only == "layered":
-            kw = {"all": {}, "decode": dict(decode_batches=(32,), prompts=(), llama=False),
-                  "prompt": dict(decode_batches=(), prompts=((4, 2048),), llama=False)}[a.layered_phase]
+            kw = {"all": {}, "decode": dict(decode_batches=(32,), prompts=()), "prompt": dict(decode_batches=(), prompts=((4, 2048),))}[a.layered_phase]
+            if a.layered_model != "both":
+                kw["models"] = (a.layered_model,)
             for size in LAYERED if a.layered_size == "all" else (a.layered_size,):
                 for r in bench_layered(fa, be, size, **kw):
                     print(json.dumps(r), flush=True)

@@ -308,7 +308,7 @@ fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t r
 // first new token sees onwards.  It is taken where forming keys and values per head costs less than attending over
 // latents, counted in multiply-adds per head.
 ExpandPlan plan_expand(const LayeredState &L, const std::vector<uint32_t> &lens, const std::vector<uint32_t> &n, uint32_t max_batch) {
-    constexpr uint64_t kMaxRows = 1u << 16;
+    constexpr uint64_t kMaxRows = 1u << 17;
     ExpandPlan p;
     p.rows.assign(L.windows.size(), 0);
     p.meta.assign(L.windows.size() * (2 * (size_t)max_batch + 1), 0);
