@@ -86,7 +86,9 @@ class DecoderConfig(C.Structure):
                 ("rope_theta", C.c_double)]
 
 
-MIXER_DELTA, MIXER_LATENT_ATTENTION = 0, 1
+MIXER_DELTA, MIXER_LATENT_ATTENTION, MIXER_ATTENTION = 0, 1, 2
+NORM_INPUT, NORM_OUTPUT = 0, 1
+ATTENTION_BIAS, ATTENTION_QK_NORM = 1, 2
 
 
 class LayerConfig(C.Structure):
@@ -94,14 +96,15 @@ class LayerConfig(C.Structure):
     _fields_ = [("mixer", C.c_int32), ("heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32),
                 ("kv_heads", C.c_uint32), ("conv", C.c_uint32), ("q_rank", C.c_uint32), ("kv_rank", C.c_uint32),
                 ("rot_dim", C.c_uint32), ("window", C.c_uint32), ("kv_from", C.c_int32), ("scale", C.c_float),
-                ("rot_base", C.c_double), ("d_ffn", C.c_uint32), ("ffn_limit", C.c_float), ("ffn_alpha", C.c_float)]
+                ("rot_base", C.c_double), ("d_ffn", C.c_uint32), ("ffn_limit", C.c_float), ("ffn_alpha", C.c_float),
+                ("attention", C.c_uint32), ("experts", C.c_uint32), ("top", C.c_uint32)]
 
 
 class LayeredConfig(C.Structure):
     _fields_ = [("n_layers", C.c_uint32), ("d_model", C.c_uint32), ("vocab", C.c_uint32), ("block_size", C.c_uint32),
                 ("max_blocks_per_seq", C.c_uint32), ("num_blocks", C.c_uint32), ("max_batch", C.c_uint32),
                 ("state_slots", C.c_uint32), ("norm_eps", C.c_float), ("logit_softcap", C.c_float), ("dtype", C.c_int),
-                ("layers", C.POINTER(LayerConfig))]
+                ("layers", C.POINTER(LayerConfig)), ("norm", C.c_int32), ("embed_scale", C.c_float), ("position_base", C.c_double)]
 
 
 # name -> (restype, argtypes); every symbol the header declares

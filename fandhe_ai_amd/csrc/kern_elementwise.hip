@@ -247,5 +247,45 @@ void gather_rows_any(const void *table, int table_f32, uint64_t table_rows, uint
         gather_rows_any_kernel<uint16_t><<<(unsigned)rows, 256, 0, s>>>((const uint16_t *)table, table_rows, (uint32_t)cols, idx, out);
 }
 
+namespace {
+template <typename T>
+__global__ void __launch_bounds__(256)
+    embed_rows_kernel(const T *__restrict__ table, uint64_t table_rows, uint32_t cols, const int32_t *__restrict__ idx, const int32_t *__restrict__ pos,
+                      const double *__restrict__ freq, float scale, float *__restrict__ x, T *__restrict__ hn, uint64_t ld) {
+    const uint64_t r = blockIdx.x;
+    const int64_t src = idx[r];
+    const bool ok = src >= 0 && (uint64_t)src < table_rows;
+    for (uint32_t c = 2 * threadIdx.x; c < ld; c += 512) {           // an entry and its neighbour share an angle
+        double sn = 0.0, cs = 0.0;
+        if (freq && c < cols) sincos((double)pos[r] * freq[c / 2], &sn, &cs);
+#pragma unroll
+        for (uint32_t e = 0; e < 2; ++e) {
+            if (c + e >= ld) continue;
+            float v = 0.0f;
+            if (c + e < cols) {
+                v = __uint_as_float(0x7fc00000u);
+                if (ok) {
+                    if constexpr (sizeof(T) == 4) v = table[src * cols + c + e];
+                    else v = bf16_to_f32(table[src * cols + c + e]);
+                }
+                v = v * scale + (float)(e ? cs : sn);
+                x[r * cols + c + e] = v;
+            }
+            if constexpr (sizeof(T) == 4) hn[r * ld + c + e] = v;
+            else hn[r * ld + c + e] = f32_to_bf16(v);
+        }
+    }
+}
+}  // namespace
+
+void embed_rows(const void *table, int is_f32, uint64_t table_rows, uint64_t cols, const int32_t *idx, const int32_t *pos, const double *freq,
+                float scale, float *x, void *hn, uint64_t ld, uint64_t rows, hipStream_t s) {
+    if (rows == 0) return;
+    if (is_f32)
+        embed_rows_kernel<float><<<(unsigned)rows, 256, 0, s>>>((const float *)table, table_rows, (uint32_t)cols, idx, pos, freq, scale, x, (float *)hn, ld);
+    else
+        embed_rows_kernel<uint16_t><<<(unsigned)rows, 256, 0, s>>>((const uint16_t *)table, table_rows, (uint32_t)cols, idx, pos, freq, scale, x, (uint16_t *)hn, ld);
+}
+
 }  // namespace k
 }  // namespace fa

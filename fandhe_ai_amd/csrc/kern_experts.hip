@@ -1,0 +1,295 @@
+// Sublayers that norm their output, and the routing of sparse feed-forwards: the residual update with its norm, the weighted
+// sum of a row's experts, the router with the choice of experts.  The experts' linears are kern_linear.hip's.
+#include <algorithm>
+
+#include "attention_tiles.hpp"
+#include "device_utils.hpp"
+#include "kernels.hpp"
+
+namespace fa {
+namespace k {
+using namespace fa::dev;
+
+int g_route_form = 0;         // tuning: 1 the router in the residual update whatever the rows, 2 in a launch of its own
+
+namespace {
+
+// The experts of one row from its logits (LDS), by one wavefront: lane i < top returns with the i-th largest logit's expert in
+// `id` and its softmax weight in `weight`.  NaN logits come out as experts in order with NaN weights.
+__device__ __forceinline__ void choose_experts(const float *logits, uint32_t experts, uint32_t top, int lane, uint32_t *id, float *weight) {
+    float v[kMaxExperts / 64];
+    bool bad = false;
+#pragma unroll
+    for (uint32_t i = 0; i < kMaxExperts / 64; ++i) {
+        const uint32_t e = i * 64 + lane;
+        v[i] = e < experts ? logits[e] : -INFINITY;
+        bad = bad || v[i] != v[i];
+        if (v[i] != v[i]) v[i] = -INFINITY;
+    }
+    bad = __any(bad);
+    uint32_t taken = 0;                              // bit i: this lane's value i has been chosen
+    float mine = -INFINITY, first = 0.0f;
+    *id = 0;
+    for (uint32_t t = 0; t < top; ++t) {
+        float best = -INFINITY;
+        uint32_t at = 0xffffffffu;
+#pragma unroll
+        for (uint32_t i = 0; i < kMaxExperts / 64; ++i) {
+            const uint32_t e = i * 64 + lane;
+            if (e < experts && !(taken >> i & 1) && (at == 0xffffffffu || v[i] > best)) {
+                best = v[i];
+                at = e;
+            }
+        }
+        const float top_v = wave_max_dpp(at == 0xffffffffu ? -INFINITY : best);
+        uint32_t cand = at != 0xffffffffu && best == top_v ? at : 0xffffffffu;
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) {
+            const uint32_t o = (uint32_t)__shfl_xor((int)cand, off, 64);
+            cand = o < cand ? o : cand;
+        }
+        if (t == 0) first = top_v;
+        if ((uint32_t)lane == cand % 64) taken |= 1u << (cand / 64);
+        if ((uint32_t)lane == t) {
+            mine = top_v;
+            *id = cand;
+        }
+    }
+    const float e = (uint32_t)lane < top ? expf(mine - first) : 0.0f;
+    const float sum = wave_sum_dpp(e);
+    *weight = bad ? __uint_as_float(0x7fc00000u) : e / sum;
+}
+
+// ------------------------------------------------------------------ residual update
+// One block per row, VPT values of it per thread.
+template <typename T, int VPT, int NT, bool ROUTE>
+__global__ void __launch_bounds__(NT)
+    residual_norm_kernel(ResidualNorm rn, float *__restrict__ x, T *__restrict__ hn, uint32_t hidden, uint64_t ld, RouteIo io) {
+    constexpr int NW = NT / 64;
+    __shared__ float smem[NW], logits[ROUTE ? kMaxExperts : 1];
+    extern __shared__ __attribute__((aligned(16))) uint8_t hs_raw[];     // ROUTE: the row of hn
+    const uint64_t r = blockIdx.x;
+    const int tid = threadIdx.x;
+    if (rn.clear && r == 0)
+        for (uint32_t i = tid; i < rn.n_clear; i += NT) rn.clear[i] = 0;
+    const float *y = rn.y + r * rn.parts * hidden;
+    float v[VPT], xv[VPT], sq = 0.0f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const uint32_t c = tid + i * NT;
+        v[i] = 0.0f;
+        xv[i] = c < hidden ? x[r * hidden + c] : 0.0f;
+        if (!rn.gate) v[i] = c < hidden ? y[c] : 0.0f;
+    }
+    if (rn.gate) {
+        for (uint32_t p = 0; p < rn.parts; ++p) {
+            const float g = rn.gate[r * rn.parts + p];
+#pragma unroll
+            for (int i = 0; i < VPT; ++i) {
+                const uint32_t c = tid + i * NT;
+                if (c < hidden) v[i] = fmaf(g, y[(uint64_t)p * hidden + c], v[i]);
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) sq = fmaf(v[i], v[i], sq);
+    const float rstd = 1.0f / sqrtf(block_sum<float, NW, true, true>(sq, smem) / (float)hidden + rn.eps);
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const uint32_t c = tid + i * NT;
+        if (c >= ld) continue;
+        float o = 0.0f;
+        if (c < hidden) {
+            o = xv[i] + v[i] * rstd * rn.w[c];
+            x[r * hidden + c] = o;
+        }
+        store_from_f32(hn + r * ld + c, o);
+        if constexpr (ROUTE) store_from_f32((T *)hs_raw + c, o);
+    }
+    if constexpr (ROUTE) {
+        const int lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64);
+        const T *h = (const T *)hs_raw;
+        __syncthreads();
+        if constexpr (sizeof(T) == 4) {
+            for (uint32_t e = wave; e < io.experts; e += NW) {
+                const float *w = (const float *)io.w + (uint64_t)e * ld;
+                float acc = 0.0f;
+                for (uint32_t c = lane; c < ld; c += 64) acc = fmaf(w[c], h[c], acc);
+                const float z = wave_sum_dpp(acc);
+                if (lane == 0) logits[e] = z;
+            }
+        } else {
+            // every wavefront its k tiles of all experts; the row is the operand of all sixteen columns
+            float *part = (float *)(hs_raw + ld * sizeof(T));        // [experts padded to 16][NW + 1]
+            const uint32_t k_tiles = (uint32_t)(ld / 32), tiles = (io.experts + 15) / 16;
+            for (uint32_t t = 0; t < tiles; ++t) {
+                const v8bf *w = (const v8bf *)io.w + (uint64_t)t * k_tiles * 64 + lane;
+                v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
+                for (uint32_t s0 = wave; s0 < k_tiles; s0 += NW * 4) {
+                    v8bf wv[4];
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) wv[u] = w[(uint64_t)(s0 + u * NW < k_tiles ? s0 + u * NW : s0) * 64];
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) {
+                        const uint32_t s = s0 + u * NW;
+                        if (s < k_tiles) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u], *(const v8bf *)(h + s * 32 + 8 * (lane / 16)), acc, 0, 0, 0);
+                    }
+                }
+                if (lane % 16 == 0)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) part[(t * 16 + 4 * (lane / 16) + e) * (NW + 1) + wave] = acc[e];
+            }
+            __syncthreads();
+            for (uint32_t e = tid; e < io.experts; e += NT) {
+                float z = 0.0f;
+#pragma unroll
+                for (int q = 0; q < NW; ++q) z += part[e * (NW + 1) + q];
+                logits[e] = z;
+            }
+        }
+        __syncthreads();
+        if (wave == 0) {
+            uint32_t id;
+            float g;
+            choose_experts(logits, io.experts, io.top, lane, &id, &g);
+            if ((uint32_t)lane < io.top) {
+                io.gate[r * io.top + lane] = g;
+                const uint32_t at = atomicAdd(io.count + id, 1u);
+                if (at < io.pitch) io.list[(uint64_t)id * io.pitch + at] = (uint32_t)(r * io.top + lane);
+            }
+        }
+    }
+}
+
+// ------------------------------------------------------------------ router
+// 16 rows per block; its four wavefronts take a quarter of k each and meet in LDS.  ET: tiles of 16 experts.
+template <int ET>
+__global__ void __launch_bounds__(256)
+    route_kernel(const uint16_t *__restrict__ h, uint64_t ld, uint32_t rows, RouteIo io) {
+    extern __shared__ __attribute__((aligned(16))) float part[];         // [4][ET * 16][17]
+    __shared__ uint32_t cnt[kMaxExperts], base[kMaxExperts];
+    __shared__ float logits[16][ET * 16 + 1];
+    const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), g = lane / 16, c = lane % 16;
+    const uint32_t r0 = blockIdx.x * 16, row = r0 + c < rows ? r0 + c : rows - 1;
+    const uint16_t *hp = h + (uint64_t)row * ld + 8 * g, *wp = (const uint16_t *)io.w + lane * 8;
+    v4f acc[ET];
+#pragma unroll
+    for (int t = 0; t < ET; ++t) acc[t] = v4f{0.f, 0.f, 0.f, 0.f};
+    const uint32_t steps = (uint32_t)(ld / 32);
+    constexpr int U = ET == 1 ? 8 : ET == 2 ? 4 : ET == 4 ? 2 : 1;       // k steps whose loads are in flight together
+    for (uint32_t s0 = wave; s0 < steps; s0 += 4 * U) {
+        v8bf hv[U], wv[U][ET];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const uint32_t s = s0 + 4 * u < steps ? s0 + 4 * u : s0;
+            hv[u] = *(const v8bf *)(hp + (uint64_t)s * 32);
+#pragma unroll
+            for (int t = 0; t < ET; ++t) wv[u][t] = *(const v8bf *)(wp + ((uint64_t)t * steps + s) * 512);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (s0 + 4 * u < steps) {
+#pragma unroll
+                for (int t = 0; t < ET; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][t], hv[u], acc[t], 0, 0, 0);
+            }
+    }
+#pragma unroll
+    for (int t = 0; t < ET; ++t)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) part[(wave * ET * 16 + t * 16 + 4 * g + e) * 17 + c] = acc[t][e];
+    for (uint32_t i = tid; i < kMaxExperts; i += 256) cnt[i] = 0;
+    __syncthreads();
+    for (int i = tid; i < ET * 256; i += 256) {
+        const int e = i / 16, rr = i % 16;
+        logits[rr][e] = (part[e * 17 + rr] + part[(ET * 16 + e) * 17 + rr]) + (part[(2 * ET * 16 + e) * 17 + rr] + part[(3 * ET * 16 + e) * 17 + rr]);
+    }
+    __syncthreads();
+    uint32_t id[4], at[4];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+        const uint32_t rr = wave * 4 + q;
+        float w;
+        choose_experts(logits[rr], io.experts, io.top, lane, &id[q], &w);
+        at[q] = 0;
+        if (r0 + rr < rows && (uint32_t)lane < io.top) {
+            io.gate[(uint64_t)(r0 + rr) * io.top + lane] = w;
+            at[q] = atomicAdd(&cnt[id[q]], 1u);
+        }
+    }
+    __syncthreads();
+    for (uint32_t e = tid; e < io.experts; e += 256)
+        if (cnt[e]) base[e] = atomicAdd(io.count + e, cnt[e]);
+    __syncthreads();
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+        const uint32_t rr = wave * 4 + q;
+        if (r0 + rr < rows && (uint32_t)lane < io.top) {
+            const uint32_t p = base[id[q]] + at[q];
+            if (p < io.pitch) io.list[(uint64_t)id[q] * io.pitch + p] = (uint32_t)((r0 + rr) * io.top + lane);
+        }
+    }
+}
+
+template <typename T, bool ROUTE>
+void launch_residual(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
+    const size_t lds = ROUTE ? ld * sizeof(T) + (sizeof(T) == 2 ? (io.experts + 15) / 16 * 16 * 17 * 4 : 0) : 0;
+#define FA_RN(V_, NT_)                                                                                                                    \
+    do {                                                                                                                                  \
+        if (lds > 49152) {                                                                                                                \
+            static bool configured = false;                                                                                               \
+            if (!configured) {                                                                                                            \
+                (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, V_, NT_, ROUTE>),                       \
+                                          hipFuncAttributeMaxDynamicSharedMemorySize, 98304);                                             \
+                configured = true;                                                                                                        \
+            }                                                                                                                             \
+        }                                                                                                                                 \
+        residual_norm_kernel<T, V_, NT_, ROUTE><<<(unsigned)rows, NT_, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);                    \
+    } while (0)
+    if (ld <= 1024) FA_RN(4, 256);
+    else if (rows > 256 && ld <= 4096) FA_RN(16, 256);
+    else if (ld <= 4096) FA_RN(4, 1024);
+    else FA_RN(16, 1024);                            // rows up to 16384
+#undef FA_RN
+}
+
+template <int ET>
+void launch_route(const uint16_t *h, uint64_t rows, uint64_t ld, const RouteIo &io, hipStream_t s) {
+    constexpr int lds = 4 * ET * 16 * 17 * 4;
+    if constexpr (lds + ET * 1024 > 49152) {
+        static bool configured = false;
+        if (!configured) {
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&route_kernel<ET>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+            configured = true;
+        }
+    }
+    route_kernel<ET><<<(unsigned)((rows + 15) / 16), 256, lds, s>>>(h, ld, (uint32_t)rows, io);
+}
+
+}  // namespace
+
+bool residual_norm_routes(int is_f32, uint64_t rows) { return is_f32 || g_route_form == 1 || (rows <= 64 && g_route_form != 2); }
+
+void residual_norm(const ResidualNorm &rn, float *x, void *hn, int is_f32, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo *route,
+                   hipStream_t s) {
+    if (rows == 0) return;
+    if (is_f32) {
+        if (route) launch_residual<float, true>(rn, x, (float *)hn, rows, hidden, ld, *route, s);
+        else launch_residual<float, false>(rn, x, (float *)hn, rows, hidden, ld, RouteIo{}, s);
+    } else {
+        if (route) launch_residual<uint16_t, true>(rn, x, (uint16_t *)hn, rows, hidden, ld, *route, s);
+        else launch_residual<uint16_t, false>(rn, x, (uint16_t *)hn, rows, hidden, ld, RouteIo{}, s);
+    }
+}
+
+void route_rows(const void *h_bf16, uint64_t rows, uint64_t ld, const RouteIo &io, hipStream_t s) {
+    if (rows == 0) return;
+    const uint16_t *p = (const uint16_t *)h_bf16;
+    if (io.experts <= 16) launch_route<1>(p, rows, ld, io, s);
+    else if (io.experts <= 32) launch_route<2>(p, rows, ld, io, s);
+    else if (io.experts <= 64) launch_route<4>(p, rows, ld, io, s);
+    else if (io.experts <= 128) launch_route<8>(p, rows, ld, io, s);
+    else launch_route<16>(p, rows, ld, io, s);
+}
+
+}  // namespace k
+}  // namespace fa

@@ -73,11 +73,25 @@ template <int MODE>
 struct EpiBf16 {
     LinearEpilogue ep;
 };
+// ... on rows grouped by the device (RowGroups): a block finds its group and tile itself, rows are fetched through the list.
+template <int MODE>
+struct EpiBf16Grouped {
+    LinearEpilogue ep;
+    RowGroups rg;
+};
 template <typename Epi>
-struct IsBf16 : std::false_type {};
+struct IsBf16 : std::false_type {
+    static constexpr bool grouped = false;
+};
 template <int MODE>
 struct IsBf16<EpiBf16<MODE>> : std::true_type {
     static constexpr int mode = MODE;
+    static constexpr bool grouped = false;
+};
+template <int MODE>
+struct IsBf16<EpiBf16Grouped<MODE>> : std::true_type {
+    static constexpr int mode = MODE;
+    static constexpr bool grouped = true;
 };
 
 constexpr int BM = 128, BN = 128;      // block tile; 4 wavefronts in 2 x 2, 64 x 64 each
@@ -407,7 +421,23 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
             ks_n = ks_hi - ks_lo;
         }
     }
-    ixm::big_block_tile(tile_id, m_blocks, n_blocks, &mb, &nb);
+    constexpr bool GROUPED = IsBf16<Epi>::grouped;
+    [[maybe_unused]] const uint32_t *list = nullptr;
+    if constexpr (GROUPED) {
+        // consecutive tiles of a group, rows fastest, to one XCD: block ids go round the XCDs
+        const uint32_t total = __builtin_amdgcn_readfirstlane(group_tiles(ep.rg, 256)) * n_blocks, chunk = (total + 7) / 8;
+        uint32_t group;
+        tile_id = blockIdx.x % 8 * chunk + blockIdx.x / 8;
+        if (blockIdx.x / 8 >= chunk || !group_tile(ep.rg, tile_id, 256, n_blocks, &group, &mb, &nb)) return;
+        group = __builtin_amdgcn_readfirstlane(group);
+        mb = __builtin_amdgcn_readfirstlane(mb);
+        nb = __builtin_amdgcn_readfirstlane(nb);
+        m = ep.rg.count[group];
+        list = ep.rg.list + (uint64_t)group * ep.rg.pitch;
+        w_tiles += (uint64_t)group * n_tiles * k_steps * TILE;
+    } else {
+        ixm::big_block_tile(tile_id, m_blocks, n_blocks, &mb, &nb);
+    }
     const uint32_t m0 = mb * 256, nt0 = nb * NTB;
     const uint64_t k_bytes = (uint64_t)k_steps * TK;
 
@@ -435,6 +465,7 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
     for (int i = 0; i < TPW; ++i) {
         uint32_t row = m0 + ixm::big_a_tile<NWAVES>(wave, i) * 16 + ixm::big_a_row(lane);
         row = row < m ? row : m - 1;
+        if constexpr (GROUPED) row = list[row] / ep.rg.a_div;
 #pragma unroll
         for (int x = 0; x < 2; ++x) a_src[i][x] = aq + (uint64_t)row * k_bytes + (uint64_t)ks_lo * TK + ixm::big_a_src_byte<FP8>(lane, x);
         // a block of NTB = 14 has no tiles 14, 15: the wavefronts that would move them repeat tiles
@@ -666,8 +697,9 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
         static_assert(STEP == 1 || WNT % 2 == 0, "a gate tile and its up tile belong to one wavefront");
 #pragma unroll
         for (int i = 0; i < AI; ++i) {
-            const uint32_t row = m0 + row_l0 + i * 16;
+            uint32_t row = m0 + row_l0 + i * 16;
             if (row >= m) continue;
+            if constexpr (GROUPED) row = list[row];
 #pragma unroll
             for (int j = 0; j < WNT; j += STEP) {
                 const uint32_t t = nt0 + wn * WNT + j;
@@ -1151,6 +1183,28 @@ void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const L
         case LinearEpilogue::kSoftcap: return launch_big_bf16<LinearEpilogue::kSoftcap>(a, m, w, ep, ntb, s);
         default: return launch_big_bf16<LinearEpilogue::kStore>(a, m, w, ep, ntb, s);
     }
+}
+
+namespace {
+template <int MODE>
+void launch_big_grouped(const uint16_t *a, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, hipStream_t s) {
+    constexpr int NTB = 16, WM = 4;
+    typedef EpiBf16Grouped<MODE> Epi;
+    const size_t smem = (3 * 16 + 2 * (size_t)NTB) * 2048;
+    static bool configured = false;
+    if (!configured) {
+        (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&gemm_mfma_big_kernel<false, NTB, WM, Epi>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+        configured = true;
+    }
+    const uint32_t nb = (w.n_tiles + NTB - 1) / NTB, tiles = rg.entries / 256 + (rg.groups < rg.entries ? rg.groups : rg.entries);
+    gemm_mfma_big_kernel<false, NTB, WM, Epi><<<(tiles * nb + 7) / 8 * 8, 128 * WM, smem, s>>>((const uint8_t *)a, (const uint8_t *)w.w, 0, w.n, w.n_tiles,
+                                                                                              w.k_tiles / 2, 0, nb, Epi{ep, rg});
+}
+}  // namespace
+
+void gemm_bf16_big_grouped(const uint16_t *a, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, hipStream_t s) {
+    if (ep.mode == LinearEpilogue::kSquaredRelu) launch_big_grouped<LinearEpilogue::kSquaredRelu>(a, w, rg, ep, s);
+    else launch_big_grouped<LinearEpilogue::kStore>(a, w, rg, ep, s);
 }
 
 }  // namespace k

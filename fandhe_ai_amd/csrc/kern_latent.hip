@@ -4,6 +4,7 @@
 #include <algorithm>
 #include <type_traits>
 
+#include "attention_tiles.hpp"
 #include "device_utils.hpp"
 #include "kernels.hpp"
 
@@ -16,17 +17,6 @@ int g_latent_form = 0;       // tuning: 1 keeps the plain attention kernel, 2 th
                              // expanded form wherever it can run
 
 namespace {
-
-template <typename T>
-__device__ __forceinline__ float load_as_f32(const T *p) {
-    if constexpr (std::is_same<T, float>::value) return *p;
-    else return bf16_to_f32(*p);
-}
-template <typename T>
-__device__ __forceinline__ void store_from_f32(T *p, float v) {
-    if constexpr (std::is_same<T, float>::value) *p = v;
-    else *p = f32_to_bf16(v);
-}
 
 // One block per row of y = q latent | kv latent | rotated key part | gates.
 template <typename T>
@@ -142,61 +132,6 @@ __global__ void __launch_bounds__(256)
         const uint32_t d = threadIdx.x + i * 256;
         if (d < sh.rank_p) store_from_f32(out + ((uint64_t)r * sh.heads + h) * sh.rank_p + d, acc[i] / l);
     }
-}
-
-// ------------------------------------------------------------------ matrix-core pieces
-constexpr float kLog2e = 1.4426950408889634f;
-constexpr int kKeys = 32;                            // keys per step of the kernels below
-
-typedef short v4s __attribute__((ext_vector_type(4)));
-typedef short v8s __attribute__((ext_vector_type(8)));
-
-// The transposed operand of a 32-key step from rows staged in LDS: lane (g, c) gets dim c of 16 dims for keys 4 g .. 4 g + 3
-// and 16 + 4 g .. + 3, in the order in which the scores of the two key tiles sit in a lane.  rows: LDS element address of
-// (key 0, first dim); pitch in elements.
-__device__ __forceinline__ v8bf transposed_keys(const uint16_t *rows, uint32_t pitch, int lane) {
-    typedef __attribute__((address_space(3))) v4s *lptr;
-    const int g = lane / 16, i = lane % 16;
-    const uint16_t *p = rows + (4 * g + i / 4) * pitch + 4 * (i % 4);
-    const v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lptr)p), hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lptr)(p + 16 * pitch));
-    return __builtin_bit_cast(v8bf, v8s{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
-}
-
-// Loads into these registers complete here: inside a loop that has loads of its own in flight, the compiler would otherwise
-// wait for both at the first use of every iteration.
-template <int N>
-__device__ __forceinline__ void hold(v8bf (&r)[N]) {
-#pragma unroll
-    for (int i = 0; i < N; ++i) {
-        v4u t = __builtin_bit_cast(v4u, r[i]);
-        asm volatile("" : "+v"(t));
-        r[i] = __builtin_bit_cast(v8bf, t);
-    }
-}
-
-// One online-softmax step of a column (query row): scores of eight keys per lane, lanes with equal lane % 16 share the
-// column.  Returns the factor for what was accumulated before; w receives the weights as two bf16 terms whose sum keeps
-// about 16 bits of them.
-__device__ __forceinline__ float softmax_step(const float (&sc)[8], float &m, float &l, v8bf &w_hi, v8bf &w_lo) {
-    float mx = fmaxf(fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3])), fmaxf(fmaxf(sc[4], sc[5]), fmaxf(sc[6], sc[7])));
-    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float m_new = fmaxf(m, mx), ref = m_new == -INFINITY ? 0.0f : m_new;
-    const float fix = exp2f(m - ref);
-    float sum = 0.0f;
-    uint32_t hi[4], lo[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const float a = exp2f(sc[2 * i] - ref), b = exp2f(sc[2 * i + 1] - ref);
-        sum += a + b;
-        hi[i] = f32x2_to_bf16x2(a, b);
-        lo[i] = f32x2_to_bf16x2(a - bf16_lo(hi[i]), b - bf16_hi(hi[i]));
-    }
-    l = l * fix + sum;
-    m = m_new;
-    w_hi = __builtin_bit_cast(v8bf, v4u{hi[0], hi[1], hi[2], hi[3]});
-    w_lo = __builtin_bit_cast(v8bf, v4u{lo[0], lo[1], lo[2], lo[3]});
-    return fix;
 }
 
 // ------------------------------------------------------------------ absorbed form

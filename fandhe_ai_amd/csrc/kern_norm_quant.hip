@@ -45,8 +45,8 @@ __global__ void __launch_bounds__(kBlock) rmsnorm_kernel(const float *__restrict
 }
 
 // Layer norm with a weight and no bias: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, two passes over the row held in
-// registers (VPT values per thread).
-template <int VPT, bool OUT_F32, int NT = kBlock>
+// registers (VPT values per thread).  RMS: without the mean.
+template <int VPT, bool OUT_F32, bool RMS, int NT = kBlock>
 __global__ void __launch_bounds__(NT)
     layernorm_kernel(const float *__restrict__ x, const float *__restrict__ w, void *__restrict__ out, uint32_t hidden, uint64_t ld,
                      float eps) {
@@ -59,7 +59,7 @@ __global__ void __launch_bounds__(NT)
         v[i] = c < hidden ? row[c] : 0.0f;
         sum += v[i];
     }
-    const float mean = block_sum<float, NT / kWave, true>(sum, smem) / (float)hidden;
+    const float mean = RMS ? 0.0f : block_sum<float, NT / kWave, true>(sum, smem) / (float)hidden;
     float sq = 0.0f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
@@ -574,22 +574,33 @@ __global__ void zero_f32_kernel(float *p) {
 
 }  // namespace
 
-void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps,
-                    hipStream_t s) {
+namespace {
+template <bool RMS>
+void norm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps, hipStream_t s) {
     if (rows == 0) return;
     const uint64_t vpt = (ld + kBlock - 1) / kBlock;
     if (rows <= 256 && ld > 1024 && ld <= 8192) {        // few rows: the row spread over 1024 threads
-        if (out_f32) layernorm_kernel<8, true, 1024><<<(unsigned)rows, 1024, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps);
-        else layernorm_kernel<8, false, 1024><<<(unsigned)rows, 1024, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps);
+        if (out_f32) layernorm_kernel<8, true, RMS, 1024><<<(unsigned)rows, 1024, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps);
+        else layernorm_kernel<8, false, RMS, 1024><<<(unsigned)rows, 1024, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps);
         return;
     }
 #define FA_LN(V)                                                                                                              \
-    out_f32 ? layernorm_kernel<V, true><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)                \
-            : layernorm_kernel<V, false><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)
+    out_f32 ? layernorm_kernel<V, true, RMS><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)           \
+            : layernorm_kernel<V, false, RMS><<<(unsigned)rows, kBlock, 0, s>>>(x, w, out, (uint32_t)hidden, ld, eps)
     if (vpt <= 4) FA_LN(4);
     else if (vpt <= 16) FA_LN(16);
     else FA_LN(64);                                  // rows up to 16384
 #undef FA_LN
+}
+}  // namespace
+
+void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps,
+                    hipStream_t s) {
+    norm_rows<false>(x, w, out, out_f32, rows, hidden, ld, eps, s);
+}
+
+void rmsnorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps, hipStream_t s) {
+    norm_rows<true>(x, w, out, out_f32, rows, hidden, ld, eps, s);
 }
 
 void rmsnorm_f32(const float *x, const float *w, float *out, uint64_t rows, uint64_t hidden, float eps,

@@ -329,7 +329,7 @@ struct LinearWeight {
 };
 // What becomes of y = a W^T (f32):
 struct LinearEpilogue {
-    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4 };
+    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4, kSquaredRelu = 5 };
     int mode = kStore;
     void *out = nullptr;         // [m, ld_out], f32 or bf16; kResidual: the f32 residual itself
     int out_f32 = 0;
@@ -338,6 +338,7 @@ struct LinearEpilogue {
     uint32_t n_lo = 0xffffffffu; // kStore: columns from n_lo on go to out_hi [m, ld_hi], f32, instead
     float *out_hi = nullptr;
     uint32_t ld_hi = 0;
+    const float *bias = nullptr;     // kStore: y + bias[c]
     const float *scale = nullptr;    // kResidual: out[r, c] += scale[c] * y
     // kGlu: tiles alternate gate / up; g = min(gate, limit), u = clamp(up, +-limit), out = g sigmoid(alpha g) (u + 1)
     float limit = 0.0f, alpha = 0.0f;
@@ -351,6 +352,18 @@ void linear_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
                  int num_cus, hipStream_t s);
 void linear_f32(const float *a, uint64_t lda, uint64_t a_batch, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep,
                 hipStream_t s);
+// Rows chosen on the device per batch entry of a weight (the experts of a sparse feed-forward): entry list[g * pitch + i],
+// i < count[g], of group g takes row entry / a_div of the activations and is row `entry` of the output.  Entries are below
+// `entries`, a group holds at most `pitch` of them.
+struct RowGroups {
+    const uint32_t *count = nullptr, *list = nullptr;
+    uint32_t groups = 0, pitch = 0, a_div = 1, entries = 0;
+    uint32_t most = 0;           // entries of a group at most (up to pitch)
+};
+void linear_grouped_bf16(const uint16_t *a, uint64_t lda, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, int num_cus,
+                         hipStream_t s);
+void linear_grouped_f32(const float *a, uint64_t lda, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, hipStream_t s);
+void gemm_bf16_big_grouped(const uint16_t *a, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, hipStream_t s);
 // The large-tile form (kern_gemm_mfma.hip): m >= 256, one batch entry, lda == 32 * k_tiles.
 bool gemm_bf16_big_applies(uint64_t lda, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus);
 void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus, hipStream_t s);
@@ -381,9 +394,65 @@ void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t 
 // (x - mean) / sqrt(variance + eps) * w per row; out f32 or bf16 with pitch ld, zeros past hidden
 void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps,
                     hipStream_t s);
+// The same with x / sqrt(mean(x^2) + eps) * w
+void rmsnorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps, hipStream_t s);
 // embedding rows (bf16 bits or f32) as f32
 void gather_rows_any(const void *table, int table_f32, uint64_t table_rows, uint64_t cols, const int32_t *idx, float *out,
                      uint64_t rows, hipStream_t s);
+
+// x = table[idx] * scale (+ the additive position vector: sin(p freq[i]) in entry 2 i, cos in 2 i + 1; freq null: none) as
+// f32, and the same rounded to the activations' type with pitch ld, zeros past cols.
+void embed_rows(const void *table, int is_f32, uint64_t table_rows, uint64_t cols, const int32_t *idx, const int32_t *pos, const double *freq,
+                float scale, float *x, void *hn, uint64_t ld, uint64_t rows, hipStream_t s);
+
+// ---- sublayers that norm their output (kern_experts.hip) -------------------------
+// Which experts a row takes: router logits in f32 from h in the activations' type (zeros past its width up to ld), the `top` largest (ties: the lower
+// index), a softmax over those; entry row * top + i is appended to the list of its i-th expert.
+struct RouteIo {
+    const void *w = nullptr;     // packed as a LinearWeight of `experts` columns
+    uint32_t experts = 0, top = 0;
+    uint32_t *count = nullptr;   // [experts], zero before
+    uint32_t *list = nullptr;    // [experts][pitch]
+    uint32_t pitch = 0;
+    float *gate = nullptr;       // [rows][top]
+};
+constexpr uint32_t kMaxExperts = 256, kMaxTop = 64;
+void route_rows(const void *h_bf16, uint64_t rows, uint64_t ld, const RouteIo &io, hipStream_t s);
+// x += rmsnorm(y) * w, hn = x in the activations' type (pitch ld, zeros past hidden).  y [rows * parts, hidden] f32; parts > 1
+// (or gate set): y's row is sum_i gate[row][i] y[row * parts + i].  clear (n_clear words): set to zero.  route: the rows'
+// experts are chosen in the same launch (for few rows and in f32; many bf16 rows are faster in a launch of route_rows).
+struct ResidualNorm {
+    const float *y = nullptr, *gate = nullptr;
+    uint32_t parts = 1;
+    const float *w = nullptr;
+    float eps = 0.0f;
+    uint32_t *clear = nullptr, n_clear = 0;
+};
+bool residual_norm_routes(int is_f32, uint64_t rows);
+void residual_norm(const ResidualNorm &rn, float *x, void *hn, int is_f32, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo *route,
+                   hipStream_t s);
+
+// ---- grouped-query attention (kern_attention.hip) --------------------------------
+struct AttentionShape {
+    uint32_t heads, kv_heads, dim, vdim;
+    uint32_t dim_p, v_p;         // padded (attention_pad); q rows are [heads][dim_p], pools [rows][kv_heads][dim_p] and [..][v_p],
+                                 // padding zero in the pools
+    float scale, eps;
+    uint64_t pool_rows;
+    __host__ __device__ uint32_t share() const { return heads / kv_heads; }
+};
+void attention_pad(AttentionShape &sh);
+// From y [rows, ld] f32 = q | k | v: with norms (nullable), RMS norm over the whole of q and of k; q -> [rows, heads, dim_p], k and
+// v -> the token's cache rows (pools null: y holds q only).
+void attention_prepare(const float *y, uint32_t ld, const float *q_norm, const float *k_norm, void *q, void *k_pool, void *v_pool, int is_f32,
+                       const AttentionShape &sh, const RaggedRows &rr, hipStream_t s);
+// Causal softmax attention over the cache -> out [rows, ld_out], heads x vdim.  bf16 with padded sizes up to 256: matrix-core
+// kernels, one for few query rows per sequence (the keys split over blocks that meet in the workspace) and one for many;
+// otherwise a plain one.  min_new / max_new: fewest (not counting none) and most new tokens of any sequence.
+uint64_t attention_workspace_bytes(const AttentionShape &sh, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
+                                   int num_cus);
+void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, int is_f32, const AttentionShape &sh,
+               const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
 
 // ---- latent attention (kern_latent.hip) -----------------------------------------
 struct LatentShape {

@@ -32,7 +32,12 @@ struct Tensor {
 struct Layer {
     fa_layer_config cfg;
     float *norm1 = nullptr, *norm2 = nullptr, *ls1 = nullptr, *ls2 = nullptr;
-    k::LinearWeight in, out, gate_up, down;
+    k::LinearWeight in, out, gate_up, down;           // with experts: gate_up and down hold one batch entry each
+    k::LinearWeight router;
+    // attention; q_norm below
+    k::AttentionShape at{};
+    float *in_bias = nullptr, *k_norm = nullptr;
+    void *k_pool = nullptr, *v_pool = nullptr;
     // latent attention
     k::LatentShape la{};
     k::LinearWeight uq, uk, uv, ukv;                  // ukv: keys and values of all heads from the latent (expanded form)
@@ -52,7 +57,8 @@ struct Arena {
     void *base = nullptr;
     uint64_t bytes = 0, cls = 0;
     uint32_t rows = 0;
-    float *x = nullptr, *y32 = nullptr, *ba = nullptr, *head_x = nullptr, *delta_scratch = nullptr;
+    float *x = nullptr, *y32 = nullptr, *ba = nullptr, *head_x = nullptr, *delta_scratch = nullptr, *gate = nullptr;
+    uint32_t *expert_count = nullptr, *expert_list = nullptr;       // counts are zero between feed-forwards
     void *hn = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *olat = nullptr, *o = nullptr, *act = nullptr;
     uint32_t *row_seq = nullptr, *kv_slot = nullptr, *row_start = nullptr;
     int32_t *pos = nullptr, *tokens = nullptr, *want = nullptr;
@@ -79,6 +85,7 @@ struct LayeredState {
     std::vector<std::pair<uint32_t, double>> rotations;      // distinct (dims, base)
     std::vector<uint32_t> windows;                           // distinct windows
     void *embed = nullptr;
+    double *position_freq = nullptr;                         // additive positions: of every pair of entries
     float *final_norm = nullptr;
     k::LinearWeight head;
     fa_buffer *state_slots = nullptr, *unit_starts = nullptr, *last_rows = nullptr;
@@ -95,7 +102,7 @@ namespace {
 
 // widest of every activation over the layers
 struct Widths {
-    uint64_t hn = 0, y32 = 0, y = 0, ba = 0, cq = 0, q = 0, qa = 0, olat = 0, o = 0, act = 0;
+    uint64_t hn = 0, y32 = 0, y = 0, ba = 0, cq = 0, q = 0, qa = 0, olat = 0, o = 0, act = 0, top = 0, experts = 0;
 };
 
 Widths widths(const LayeredState &L) {
@@ -105,6 +112,9 @@ Widths widths(const LayeredState &L) {
         if (l.cfg.mixer == FA_MIXER_DELTA) {
             w.y = std::max<uint64_t>(w.y, pad_to(l.de.qkv() + l.de.heads * l.de.vdim, 8));
             w.ba = std::max<uint64_t>(w.ba, 2 * l.de.heads);
+        } else if (l.cfg.mixer == FA_MIXER_ATTENTION) {
+            w.y32 = std::max<uint64_t>(w.y32, pad_to(l.in.n, 4));
+            w.q = std::max<uint64_t>(w.q, (uint64_t)l.at.heads * l.at.dim_p);
         } else {
             w.y32 = std::max<uint64_t>(w.y32, pad_to(l.in.n, 4));
             w.cq = std::max<uint64_t>(w.cq, pad_to(l.la.q_rank, 64));
@@ -113,7 +123,11 @@ Widths widths(const LayeredState &L) {
             w.olat = std::max<uint64_t>(w.olat, (uint64_t)l.la.heads * l.la.rank_p);
         }
         w.o = std::max<uint64_t>(w.o, pad_to(l.cfg.heads * l.cfg.vdim, 64));
-        if (l.cfg.d_ffn) w.act = std::max<uint64_t>(w.act, pad_to(l.cfg.d_ffn, 64));
+        const uint64_t parts = l.cfg.experts ? l.cfg.top : 1;
+        if (l.cfg.d_ffn) w.act = std::max<uint64_t>(w.act, parts * pad_to(l.cfg.d_ffn, 64));
+        if (L.cfg.norm == FA_NORM_OUTPUT) w.y32 = std::max<uint64_t>(w.y32, parts * L.cfg.d_model);
+        w.top = std::max<uint64_t>(w.top, l.cfg.experts ? l.cfg.top : 0);
+        w.experts = std::max<uint64_t>(w.experts, l.cfg.experts);
     }
     return w;
 }
@@ -146,6 +160,9 @@ fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t row
     add(&a.olat, R * w.olat * E);
     add(&a.o, R * w.o * E);
     add(&a.act, R * w.act * E);
+    add((void **)&a.gate, R * w.top * 4);
+    add((void **)&a.expert_count, w.experts * 4);
+    add((void **)&a.expert_list, w.experts * R * 4);
     add((void **)&a.row_seq, R * 4);
     add((void **)&a.kv_slot, R * 4);
     add((void **)&a.pos, R * 4);
@@ -195,74 +212,152 @@ k::LinearEpilogue store_to(void *out, uint64_t ld, int out_f32) {
     return e;
 }
 
-// All layers over the rows of a pass whose embeddings are in a.x.
-fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::RaggedRows &rr, uint32_t max_new, uint64_t trace_row0,
+void linear_grouped(fa_context *ctx, const LayeredState &L, const void *a, uint64_t lda, const k::LinearWeight &w, const k::RowGroups &rg,
+                    const k::LinearEpilogue &ep) {
+    if (L.is_f32) k::linear_grouped_f32((const float *)a, lda, w, rg, ep, ctx->stream);
+    else k::linear_grouped_bf16((const uint16_t *)a, lda, w, rg, ep, ctx->props.multiProcessorCount, ctx->stream);
+}
+
+// The new tokens of a pass's sequences, none not counted
+struct Portions {
+    uint32_t min_new, max_new;
+};
+
+// The mixers: from a.hn to a.o (pitch ld_o).
+void enqueue_delta(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const k::RaggedRows &rr, uint32_t max_new, uint32_t ld_hn, uint32_t ld_o) {
+    const uint32_t n_lo = l.in.n - 2 * l.de.heads, ld_y = pad_to(n_lo, 8);
+    k::LinearEpilogue e = store_to(a.y, ld_y, L.is_f32);
+    e.n_lo = n_lo;
+    e.out_hi = a.ba;
+    e.ld_hi = 2 * l.de.heads;
+    linear(ctx, L, a.hn, ld_hn, 0, rr.rows, l.in, e);
+    k::DeltaIo io{a.y, ld_y, a.ba, 2 * l.de.heads, l.conv, l.a_log, l.dt_bias, l.head_norm, l.state, l.ring, a.o, ld_o, a.delta_scratch};
+    k::delta_mixer(l.de, io, L.is_f32, rr, max_new, ctx->stream);
+}
+
+void enqueue_latent(fa_context *ctx, const fa_decoder *d, Arena &a, const Layer &l, const k::RaggedRows &rr, uint32_t max_new, uint32_t ld_hn,
+                    uint32_t ld_o, const ExpandPlan *expand) {
+    LayeredState &L = *d->layered;
+    hipStream_t s = ctx->stream;
+    const int f32 = L.is_f32;
+    const uint32_t M = rr.rows;
+    const k::LatentShape &sh = l.la;
+    const uint32_t ld_y = pad_to(l.in.n, 4), ld_cq = pad_to(sh.q_rank, 64), qw = sh.dim_p + sh.rot_p, kw = sh.rank_p + sh.rot_p;
+    const bool own = l.cfg.kv_from < 0;
+    const float *cs = a.cos_sin[l.rotation];
+    void *pool = own ? l.pool : L.layers[l.cfg.kv_from].pool;
+    linear(ctx, L, a.hn, ld_hn, 0, M, l.in, store_to(a.y32, ld_y, 1));
+    k::latent_prepare(a.y32, ld_y, l.q_norm, l.kv_norm, cs, a.cq, ld_cq, own ? pool : nullptr, f32, sh, rr, s);
+    linear(ctx, L, a.cq, ld_cq, 0, M, l.uq, store_to(a.q, (uint64_t)sh.heads * qw, f32));
+    const float *gate = a.y32 + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
+    if (expand && expand->rows[l.window_index]) {
+        const uint32_t *meta = a.expand_meta + (uint64_t)l.window_index * (2 * d->cfg.max_batch + 1);
+        const k::LatentExpand ex{meta, meta + d->cfg.max_batch + 1, expand->rows[l.window_index]};
+        const uint32_t ld_c = pad_to(sh.rank_p, 64);
+        k::latent_rotate_query(a.q, cs, a.q, qw, sh.dim_p, f32, sh, M, s);
+        k::latent_gather(pool, a.ec, ld_c, a.er, sh, rr, ex, s);
+        linear(ctx, L, a.ec, ld_c, 0, ex.rows, l.ukv, store_to(a.ekv, l.ukv.n, f32));
+        k::latent_attention_expanded(a.q, a.ekv, a.er, gate, ld_y, a.o, ld_o, sh, rr, ex, s);
+    } else {
+        k::LinearEpilogue e = store_to(a.qa, (uint64_t)sh.heads * kw, f32);
+        e.out_batch = kw;
+        linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, l.uk, e);
+        k::latent_rotate_query(a.q, cs, a.qa, kw, sh.rank_p, f32, sh, M, s);
+        k::latent_attention(a.qa, pool, a.olat, f32, sh, rr, max_new, ctx->workspace, ctx->props.multiProcessorCount, s);
+        e = store_to(a.o, ld_o, f32);
+        e.mode = k::LinearEpilogue::kHeadGate;
+        e.out_batch = sh.vdim;
+        e.gate = gate;
+        e.ld_gate = ld_y;
+        linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, l.uv, e);
+    }
+}
+
+void enqueue_attention(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const k::RaggedRows &rr, Portions n, uint32_t ld_hn, uint32_t ld_o) {
+    const k::AttentionShape &sh = l.at;
+    const uint32_t ld_y = pad_to(l.in.n, 4);
+    const bool own = l.cfg.kv_from < 0;
+    const Layer &kv = own ? l : L.layers[l.cfg.kv_from];
+    k::LinearEpilogue e = store_to(a.y32, ld_y, 1);
+    e.bias = l.in_bias;
+    linear(ctx, L, a.hn, ld_hn, 0, rr.rows, l.in, e);
+    k::attention_prepare(a.y32, ld_y, l.q_norm, l.k_norm, a.q, own ? l.k_pool : nullptr, own ? l.v_pool : nullptr, L.is_f32, sh, rr, ctx->stream);
+    k::attention(a.q, kv.k_pool, kv.v_pool, a.o, ld_o, L.is_f32, sh, rr, n.min_new, n.max_new, ctx->workspace, ctx->props.multiProcessorCount, ctx->stream);
+}
+
+// Dense feed-forward: from a.hn to what `out` does with the down projection.
+void enqueue_glu(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t M, uint32_t ld_hn, const k::LinearEpilogue &out) {
+    const uint32_t ld_act = pad_to(l.cfg.d_ffn, 64);
+    k::LinearEpilogue g = store_to(a.act, ld_act, L.is_f32);
+    g.mode = k::LinearEpilogue::kGlu;
+    g.limit = l.cfg.ffn_limit;
+    g.alpha = l.cfg.ffn_alpha;
+    linear(ctx, L, a.hn, ld_hn, 0, M, l.gate_up, g);
+    linear(ctx, L, a.act, ld_act, 0, M, l.down, out);
+}
+
+// Feed-forward of a layer whose sublayers read x and norm their output.  The choice of experts is there (route_rows).
+void enqueue_experts(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t M, uint32_t ld_hn) {
+    const uint32_t D = L.cfg.d_model, ld_act = pad_to(l.cfg.d_ffn, 64), top = l.cfg.top;
+    k::RowGroups rg{a.expert_count, a.expert_list, l.cfg.experts, a.rows, top, M * top};
+    rg.most = M;
+    k::LinearEpilogue up = store_to(a.act, ld_act, L.is_f32);
+    up.mode = k::LinearEpilogue::kSquaredRelu;
+    linear_grouped(ctx, L, a.hn, ld_hn, l.gate_up, rg, up);
+    rg.a_div = 1;
+    linear_grouped(ctx, L, a.act, ld_act, l.down, rg, store_to(a.y32, D, 1));
+}
+
+// All layers over the rows of a pass whose embeddings are in a.x (and, with norms at the output, in a.hn).
+fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::RaggedRows &rr, Portions n, uint64_t trace_row0,
                          const ExpandPlan *expand = nullptr) {
     LayeredState &L = *d->layered;
     hipStream_t s = ctx->stream;
     const uint32_t M = rr.rows, D = L.cfg.d_model, ld_hn = pad_to(D, 64);
     const float eps = L.cfg.norm_eps;
     const int f32 = L.is_f32;
+    const bool at_output = L.cfg.norm == FA_NORM_OUTPUT;
     for (size_t i = 0; i < L.rotations.size(); ++i) k::rotation_table(rr.pos, a.cos_sin[i], M, L.rotations[i].first, L.rotations[i].second, s);
     for (size_t li = 0; li < L.layers.size(); ++li) {
         const Layer &l = L.layers[li];
-        k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);
-        const uint32_t ow = l.cfg.heads * l.cfg.vdim, ld_o = pad_to(ow, 64);
-        if (l.cfg.mixer == FA_MIXER_DELTA) {
-            const uint32_t n_lo = l.de.qkv() + ow, ld_y = pad_to(n_lo, 8);
-            k::LinearEpilogue e = store_to(a.y, ld_y, f32);
-            e.n_lo = n_lo;
-            e.out_hi = a.ba;
-            e.ld_hi = 2 * l.de.heads;
-            linear(ctx, L, a.hn, ld_hn, 0, M, l.in, e);
-            k::DeltaIo io{a.y, ld_y, a.ba, 2 * l.de.heads, l.conv, l.a_log, l.dt_bias, l.head_norm, l.state, l.ring, a.o, ld_o, a.delta_scratch};
-            k::delta_mixer(l.de, io, f32, rr, max_new, s);
-        } else {
-            const k::LatentShape &sh = l.la;
-            const uint32_t ld_y = pad_to(l.in.n, 4), ld_cq = pad_to(sh.q_rank, 64), qw = sh.dim_p + sh.rot_p, kw = sh.rank_p + sh.rot_p;
-            const bool own = l.cfg.kv_from < 0;
-            const float *cs = a.cos_sin[l.rotation];
-            void *pool = own ? l.pool : L.layers[l.cfg.kv_from].pool;
-            linear(ctx, L, a.hn, ld_hn, 0, M, l.in, store_to(a.y32, ld_y, 1));
-            k::latent_prepare(a.y32, ld_y, l.q_norm, l.kv_norm, cs, a.cq, ld_cq, own ? pool : nullptr, f32, sh, rr, s);
-            linear(ctx, L, a.cq, ld_cq, 0, M, l.uq, store_to(a.q, (uint64_t)sh.heads * qw, f32));
-            const float *gate = a.y32 + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
-            if (expand && expand->rows[l.window_index]) {
-                const uint32_t *meta = a.expand_meta + (uint64_t)l.window_index * (2 * d->cfg.max_batch + 1);
-                const k::LatentExpand ex{meta, meta + d->cfg.max_batch + 1, expand->rows[l.window_index]};
-                const uint32_t ld_c = pad_to(sh.rank_p, 64);
-                k::latent_rotate_query(a.q, cs, a.q, qw, sh.dim_p, f32, sh, M, s);
-                k::latent_gather(pool, a.ec, ld_c, a.er, sh, rr, ex, s);
-                linear(ctx, L, a.ec, ld_c, 0, ex.rows, l.ukv, store_to(a.ekv, l.ukv.n, f32));
-                k::latent_attention_expanded(a.q, a.ekv, a.er, gate, ld_y, a.o, ld_o, sh, rr, ex, s);
-            } else {
-                k::LinearEpilogue e = store_to(a.qa, (uint64_t)sh.heads * kw, f32);
-                e.out_batch = kw;
-                linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, l.uk, e);
-                k::latent_rotate_query(a.q, cs, a.qa, kw, sh.rank_p, f32, sh, M, s);
-                k::latent_attention(a.qa, pool, a.olat, f32, sh, rr, max_new, ctx->workspace, ctx->props.multiProcessorCount, s);
-                e = store_to(a.o, ld_o, f32);
-                e.mode = k::LinearEpilogue::kHeadGate;
-                e.out_batch = sh.vdim;
-                e.gate = gate;
-                e.ld_gate = ld_y;
-                linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, l.uv, e);
+        if (!at_output) k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);
+        const uint32_t ld_o = pad_to(l.cfg.heads * l.cfg.vdim, 64);
+        if (l.cfg.mixer == FA_MIXER_DELTA) enqueue_delta(ctx, L, a, l, rr, n.max_new, ld_hn, ld_o);
+        else if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) enqueue_latent(ctx, d, a, l, rr, n.max_new, ld_hn, ld_o, expand);
+        else enqueue_attention(ctx, L, a, l, rr, n, ld_hn, ld_o);
+        if (at_output) {
+            linear(ctx, L, a.o, ld_o, 0, M, l.out, store_to(a.y32, D, 1));
+            k::ResidualNorm rn;
+            rn.y = a.y32;
+            rn.w = l.norm1;
+            rn.eps = eps;
+            k::RouteIo route{l.router.w, l.cfg.experts, l.cfg.top, a.expert_count, a.expert_list, a.rows, a.gate};
+            const bool fused = l.cfg.experts && k::residual_norm_routes(f32, M);
+            k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, fused ? &route : nullptr, s);
+            if (l.cfg.d_ffn) {
+                if (l.cfg.experts) {
+                    if (!fused) k::route_rows(a.hn, M, ld_hn, route, s);
+                    enqueue_experts(ctx, L, a, l, M, ld_hn);
+                    rn.gate = a.gate;
+                    rn.parts = l.cfg.top;
+                    rn.clear = a.expert_count;
+                    rn.n_clear = l.cfg.experts;
+                } else {
+                    enqueue_glu(ctx, L, a, l, M, ld_hn, store_to(a.y32, D, 1));
+                }
+                rn.w = l.norm2;
+                k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
             }
-        }
-        k::LinearEpilogue r = store_to(a.x, D, 1);
-        r.mode = k::LinearEpilogue::kResidual;
-        r.scale = l.ls1;
-        linear(ctx, L, a.o, ld_o, 0, M, l.out, r);
-        if (l.cfg.d_ffn) {
-            const uint32_t ld_act = pad_to(l.cfg.d_ffn, 64);
-            k::layernorm_rows(a.x, l.norm2, a.hn, f32, M, D, ld_hn, eps, s);
-            k::LinearEpilogue g = store_to(a.act, ld_act, f32);
-            g.mode = k::LinearEpilogue::kGlu;
-            g.limit = l.cfg.ffn_limit;
-            g.alpha = l.cfg.ffn_alpha;
-            linear(ctx, L, a.hn, ld_hn, 0, M, l.gate_up, g);
-            r.scale = l.ls2;
-            linear(ctx, L, a.act, ld_act, 0, M, l.down, r);
+        } else {
+            k::LinearEpilogue r = store_to(a.x, D, 1);
+            r.mode = k::LinearEpilogue::kResidual;
+            r.scale = l.ls1;
+            linear(ctx, L, a.o, ld_o, 0, M, l.out, r);
+            if (l.cfg.d_ffn) {
+                k::layernorm_rows(a.x, l.norm2, a.hn, f32, M, D, ld_hn, eps, s);
+                r.scale = l.ls2;
+                enqueue_glu(ctx, L, a, l, M, ld_hn, r);
+            }
         }
         if (L.trace) {
             hipError_t e = hipMemcpyAsync(L.trace + (li * L.trace_rows + trace_row0) * D, a.x, (uint64_t)M * D * 4, hipMemcpyDeviceToHost, s);
@@ -273,10 +368,20 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
     return FA_OK;
 }
 
+// Embeddings of the pass's tokens.
+void enqueue_embed(fa_context *ctx, const LayeredState &L, Arena &a, const int32_t *tokens, const k::RaggedRows &rr) {
+    if (L.cfg.norm == FA_NORM_OUTPUT)
+        k::embed_rows(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, tokens, rr.pos, L.position_freq, L.cfg.embed_scale, a.x, a.hn, pad_to(L.cfg.d_model, 64),
+                      rr.rows, ctx->stream);
+    else
+        k::gather_rows_any(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, tokens, a.x, rr.rows, ctx->stream);
+}
+
 // Final norm and head over rows of f32 residuals.
 void enqueue_head(fa_context *ctx, LayeredState &L, Arena &a, const float *x, uint32_t rows, float *logits) {
     const uint32_t ld_hn = pad_to(L.cfg.d_model, 64);
-    k::layernorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
+    if (L.cfg.norm == FA_NORM_OUTPUT) k::rmsnorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
+    else k::layernorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
     k::LinearEpilogue e = store_to(logits, L.cfg.vocab, 1);
     e.mode = k::LinearEpilogue::kSoftcap;
     e.cap = L.cfg.logit_softcap;
@@ -296,11 +401,15 @@ void prepare_rows(fa_context *ctx, fa_decoder *d, Arena &a, const uint32_t *row_
     k::ragged_advance(row_start, (uint32_t *)d->seq_lens->ptr, d->batch, ctx->stream);
 }
 
-fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch, uint32_t max_new) {
+fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch, Portions n) {
     uint64_t need = 0;
-    for (const Layer &l : L.layers)
+    const int cus = ctx->props.multiProcessorCount;
+    for (const Layer &l : L.layers) {
         if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION)
-            need = std::max(need, k::latent_attention_workspace_bytes(l.la, L.is_f32, rows, batch, max_new, ctx->props.multiProcessorCount));
+            need = std::max(need, k::latent_attention_workspace_bytes(l.la, L.is_f32, rows, batch, n.max_new, cus));
+        else if (l.cfg.mixer == FA_MIXER_ATTENTION)
+            need = std::max(need, k::attention_workspace_bytes(l.at, L.is_f32, batch, n.min_new, n.max_new, L.cfg.max_blocks_per_seq * L.cfg.block_size, cus));
+    }
     return need ? ensure_workspace(ctx, need) : FA_OK;
 }
 
@@ -383,7 +492,7 @@ fa_status layered_sequences_set(fa_context *ctx, fa_decoder *d) {
 fa_status layered_prepare_step(fa_context *ctx, fa_decoder *d) {
     LayeredState &L = *d->layered;
     if (fa_status s = arena_reserve(ctx, L, L.step, L.cfg.max_batch)) return s;
-    return attention_workspace(ctx, L, d->batch, d->batch, 1);
+    return attention_workspace(ctx, L, d->batch, d->batch, Portions{1, 1});
 }
 
 fa_status layered_enqueue_step(fa_context *ctx, fa_decoder *d) {
@@ -392,8 +501,9 @@ fa_status layered_enqueue_step(fa_context *ctx, fa_decoder *d) {
     const uint32_t B = d->batch;
     const uint32_t *starts = (const uint32_t *)L.unit_starts->ptr;
     prepare_rows(ctx, d, a, starts, B);
-    k::gather_rows_any(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, (const int32_t *)d->tokens->ptr, a.x, B, ctx->stream);
-    if (fa_status s = enqueue_layers(ctx, d, a, ragged(d, a, starts, B), 1, 0)) return s;
+    const k::RaggedRows rr = ragged(d, a, starts, B);
+    enqueue_embed(ctx, L, a, (const int32_t *)d->tokens->ptr, rr);
+    if (fa_status s = enqueue_layers(ctx, d, a, rr, Portions{1, 1}, 0)) return s;
     enqueue_head(ctx, L, a, a.x, B, (float *)d->logits->ptr);
     enqueue_pick(d, ctx->stream);
     return after_launch(ctx, "layered decoder step");
@@ -454,7 +564,8 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
         }
         while (placed < total) {
             // sequences in order, each as much as the pass has room for
-            uint32_t rows = 0, max_new = 0;
+            uint32_t rows = 0;
+            Portions portions{0xffffffffu, 0};
             stage.clear();
             pick_rows.clear();
             std::vector<int32_t> last(B, -1);
@@ -468,7 +579,8 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
                 while (w_at < n_want && want[w_at] < g0 + n) pick_rows.push_back((int32_t)(rows + want[w_at++] - g0));
                 done[b] += n;
                 rows += n;
-                max_new = std::max(max_new, n);
+                portions.min_new = std::min(portions.min_new, n);
+                portions.max_new = std::max(portions.max_new, n);
                 if (done[b] == counts[b]) last[b] = (int32_t)rows - 1;
             }
             starts[B] = rows;
@@ -482,12 +594,13 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
                 if (fa_status s = arena_reserve(ctx, L, a, a.rows, e_cap)) return s;
                 if (fa_status s = upload(ctx, a.expand_meta, expand.meta.data(), expand.meta.size() * 4)) return s;
             }
-            if (fa_status s = attention_workspace(ctx, L, rows, B, max_new)) return s;
+            if (fa_status s = attention_workspace(ctx, L, rows, B, portions)) return s;
             if (fa_status s = upload(ctx, a.row_start, starts.data(), (B + 1) * 4)) return s;
             if (fa_status s = upload(ctx, a.tokens, stage.data(), (uint64_t)rows * 4)) return s;
             prepare_rows(ctx, d, a, a.row_start, rows);
-            k::gather_rows_any(L.embed, L.is_f32, c.vocab, c.d_model, a.tokens, a.x, rows, ctx->stream);
-            if (fa_status s = enqueue_layers(ctx, d, a, ragged(d, a, a.row_start, rows), max_new, placed, &expand)) return s;
+            const k::RaggedRows rr = ragged(d, a, a.row_start, rows);
+            enqueue_embed(ctx, L, a, a.tokens, rr);
+            if (fa_status s = enqueue_layers(ctx, d, a, rr, portions, placed, &expand)) return s;
             for (uint32_t b = 0; b < B; ++b) d->host_lens[b] += starts[b + 1] - starts[b];
             placed += rows;
             if (last_only) {
@@ -565,8 +678,24 @@ fa_status check_layer(const fa_layered_config &c, uint32_t i) {
             if (j.mixer != FA_MIXER_LATENT_ATTENTION || j.kv_from >= 0) return bad("kv_from must name a latent attention layer with a cache of its own");
             if (j.kv_rank != l.kv_rank || j.rot_dim != l.rot_dim || j.rot_base != l.rot_base) return bad("kv_from: the two layers' latents or rotations differ");
         }
+    } else if (l.mixer == FA_MIXER_ATTENTION) {
+        if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
+        if (!std::isfinite(l.scale)) return bad("bad scale");
+        if (l.attention & ~(uint32_t)(FA_ATTENTION_BIAS | FA_ATTENTION_QK_NORM)) return bad("unknown attention flags");
+        if (l.kv_from >= 0) {
+            if ((uint32_t)l.kv_from >= i) return bad("kv_from must name an earlier layer");
+            const fa_layer_config &j = c.layers[l.kv_from];
+            if (j.mixer != FA_MIXER_ATTENTION || j.kv_from >= 0) return bad("kv_from must name an attention layer with a cache of its own");
+            if (j.kv_heads != l.kv_heads || j.dim != l.dim || j.vdim != l.vdim) return bad("kv_from: the two layers' key and value sizes differ");
+        }
     } else {
         return bad("unknown mixer");
+    }
+    if (l.experts) {
+        if (l.experts > k::kMaxExperts || l.top > k::kMaxTop) return fail(FA_ERR_UNSUPPORTED, "sparse experts: more than 256, or more than 64 of them per token");
+        if (l.top == 0 || l.top > l.experts || l.d_ffn == 0) return bad("top must be between 1 and experts, d_ffn positive");
+        if (c.norm != FA_NORM_OUTPUT) return fail(FA_ERR_UNSUPPORTED, "sparse experts: with norms at the sublayers' output only");
+        return FA_OK;
     }
     if (l.d_ffn && !(l.ffn_limit >= 0.0f && std::isfinite(l.ffn_alpha))) return bad("bad feed-forward constants");
     return FA_OK;
@@ -586,6 +715,10 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
     if (c.d_model > 16384) return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: d_model above 16384");
     if (c.dtype != FA_BF16 && c.dtype != FA_F32) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: dtype must be bf16 or f32");
     if (!std::isfinite(c.norm_eps) || c.norm_eps < 0.0f || !std::isfinite(c.logit_softcap)) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad constants");
+    if ((c.norm != FA_NORM_INPUT && c.norm != FA_NORM_OUTPUT) || !std::isfinite(c.embed_scale) || !std::isfinite(c.position_base) || c.position_base < 0.0)
+        return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad norm, embed_scale or position_base");
+    if (c.norm == FA_NORM_INPUT && (c.position_base > 0.0 || (c.embed_scale != 0.0f && c.embed_scale != 1.0f)))
+        return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: scaled or positioned embeddings need norms at the sublayers' output");
     if (c.block_size == 0 || (c.block_size & (c.block_size - 1)) != 0 || c.block_size > 256 || c.num_blocks == 0)
         return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: block_size must be a power of two up to 256, num_blocks positive");
     if (c.max_blocks_per_seq == 0 || (uint64_t)c.max_blocks_per_seq * c.block_size > (uint64_t)INT32_MAX)
@@ -616,6 +749,7 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
         L->layer_cfgs.assign(c.layers, c.layers + c.n_layers);
         L->cfg = c;
         L->cfg.layers = L->layer_cfgs.data();
+        if (L->cfg.embed_scale == 0.0f) L->cfg.embed_scale = 1.0f;
         L->is_f32 = c.dtype == FA_F32;
         L->esz = L->is_f32 ? 4 : 2;
         const int f32 = L->is_f32;
@@ -667,6 +801,13 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 else k::convert_f32_to_bf16((const float *)src, (uint16_t *)dst, n, s);
             });
         }
+        if (c.position_base > 0.0) {
+            std::vector<double> freq((D + 1) / 2);
+            for (uint32_t i = 0; i < freq.size(); ++i) freq[i] = std::pow(c.position_base, -2.0 * (double)i / (double)D);
+            L->position_freq = (double *)own(FA_F32, 2 * freq.size());
+            if (st == FA_OK) st = fa_upload_into(ctx, freq.data(), 2 * freq.size(), L->owned.back(), 0);
+        }
+        const bool scaled = c.norm == FA_NORM_INPUT;         // sublayer outputs pass a layer scale
         L->layers.resize(c.n_layers);
         for (uint32_t i = 0; i < c.n_layers; ++i) {
             Layer &l = L->layers[i];
@@ -675,9 +816,11 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             const fa_layer_config &g = l.cfg;
             const uint32_t H = g.heads, ow = H * g.vdim;
             l.norm1 = (float *)own(FA_F32, D);
-            l.ls1 = (float *)own(FA_F32, D);
             vec(p + "norm1", D, 0, l.norm1);
-            vec(p + "ls1", D, 0, l.ls1);
+            if (scaled) {
+                l.ls1 = (float *)own(FA_F32, D);
+                vec(p + "ls1", D, 0, l.ls1);
+            }
             if (g.mixer == FA_MIXER_DELTA) {
                 L->has_state = true;
                 l.de = k::DeltaShape{H, g.kv_heads, g.dim, g.vdim, g.conv, c.norm_eps};
@@ -701,6 +844,28 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 vec(m + "norm", g.vdim, 0, l.head_norm);
                 l.state = (float *)own(FA_F32, (uint64_t)c.state_slots * H * g.dim * l.de.vdim_p());
                 l.ring = own(f32 ? FA_F32 : FA_BF16, (uint64_t)c.state_slots * g.conv * ch);
+            } else if (g.mixer == FA_MIXER_ATTENTION) {
+                k::AttentionShape &a = l.at;
+                a = k::AttentionShape{H, g.kv_heads, g.dim, g.vdim, 0, 0, g.scale, c.norm_eps, (uint64_t)c.num_blocks * c.block_size};
+                k::attention_pad(a);
+                const bool own_kv = g.kv_from < 0, bias = g.attention & FA_ATTENTION_BIAS, norms = g.attention & FA_ATTENTION_QK_NORM;
+                const uint32_t nq = H * g.dim, nk = own_kv ? g.kv_heads * g.dim : 0, nv = own_kv ? g.kv_heads * g.vdim : 0;
+                l.in = weight(nq + nk + nv, nq + nk + nv, D);
+                if (bias) l.in_bias = (float *)own(FA_F32, pad_to(nq + nk + nv, 4));
+                if (norms) l.q_norm = (float *)own(FA_F32, nq);
+                if (norms && own_kv) l.k_norm = (float *)own(FA_F32, nk);
+                const std::pair<const char *, std::pair<uint32_t, uint32_t>> parts[3] = {{"q", {0, nq}}, {"k", {nq, nk}}, {"v", {nq + nk, nv}}};
+                for (const auto &[name, at] : parts) {
+                    if (at.second == 0) continue;
+                    lin(m + name, at.second, D, l.in, at.first);
+                    if (bias) vec(m + name + ".b", at.second, 0, l.in_bias + at.first);
+                }
+                if (l.q_norm) vec(m + "q.norm", nq, 0, l.q_norm);
+                if (l.k_norm) vec(m + "k.norm", nk, 0, l.k_norm);
+                if (own_kv) {
+                    l.k_pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * g.kv_heads * a.dim_p);
+                    l.v_pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * g.kv_heads * a.v_p);
+                }
             } else {
                 k::LatentShape &a = l.la;
                 a.heads = H;
@@ -774,9 +939,29 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             lin(m + "o", D, ow, l.out, 0);
             if (g.d_ffn) {
                 l.norm2 = (float *)own(FA_F32, D);
-                l.ls2 = (float *)own(FA_F32, D);
                 vec(p + "norm2", D, 0, l.norm2);
-                vec(p + "ls2", D, 0, l.ls2);
+                if (scaled) {
+                    l.ls2 = (float *)own(FA_F32, D);
+                    vec(p + "ls2", D, 0, l.ls2);
+                }
+            }
+            if (g.experts) {
+                l.router = weight(g.experts, g.experts, D);
+                lin(f + "router", g.experts, D, l.router, 0);
+                l.gate_up = weight(g.d_ffn, g.d_ffn, D, g.experts);
+                l.down = weight(D, D, g.d_ffn, g.experts);
+                const auto one = [&](const k::LinearWeight &w, uint32_t e) {
+                    k::LinearWeight t = w;
+                    t.batches = 1;
+                    t.w = (uint8_t *)w.w + (uint64_t)e * w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
+                    return t;
+                };
+                for (uint32_t e = 0; e < g.experts; ++e) {
+                    const std::string x = f + "e" + std::to_string(e) + ".";
+                    lin(x + "up", g.d_ffn, D, one(l.gate_up, e), 0);
+                    lin(x + "down", D, g.d_ffn, one(l.down, e), 0);
+                }
+            } else if (g.d_ffn) {
                 // gate and up alternate in tiles of 16 columns
                 l.gate_up = weight(g.d_ffn, 2 * pad_to(g.d_ffn, 16), D);
                 lin(f + "gate", g.d_ffn, D, l.gate_up, 0, 16, 32);

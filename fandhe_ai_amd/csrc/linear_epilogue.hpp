@@ -19,6 +19,9 @@ __device__ __forceinline__ float epilogue_value(const LinearEpilogue &ep, uint32
         return ep.cap > 0.0f ? ep.cap * tanhf(y / ep.cap) : y;
     } else if constexpr (MODE == LinearEpilogue::kHeadGate) {
         return y * sigmoid_f32(ep.gate[(uint64_t)row * ep.ld_gate + batch]);
+    } else if constexpr (MODE == LinearEpilogue::kSquaredRelu) {
+        const float r = fmaxf(y, 0.0f);
+        return r * r;
     } else {
         return y;
     }
@@ -26,7 +29,8 @@ __device__ __forceinline__ float epilogue_value(const LinearEpilogue &ep, uint32
 
 template <int MODE>
 __device__ __forceinline__ void epilogue_store1(const LinearEpilogue &ep, uint32_t row, uint32_t col, uint32_t batch, float y, float up) {
-    const float v = epilogue_value<MODE>(ep, row, batch, y, up);
+    float v = epilogue_value<MODE>(ep, row, batch, y, up);
+    if (MODE == LinearEpilogue::kStore && ep.bias) v += ep.bias[col];
     if constexpr (MODE == LinearEpilogue::kResidual) {
         float *o = (float *)ep.out + (uint64_t)row * ep.ld_out + col;
         *o = *o + ep.scale[col] * v;
@@ -56,6 +60,13 @@ __device__ __forceinline__ void epilogue_store4(const LinearEpilogue &ep, uint32
     float v[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) v[e] = epilogue_value<MODE>(ep, row, batch, y[e], up[e]);
+    if constexpr (MODE == LinearEpilogue::kStore) {
+        if (ep.bias) {
+            const dev::v4f b = *(const dev::v4f *)(ep.bias + col);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] += b[e];
+        }
+    }
     if constexpr (MODE == LinearEpilogue::kResidual) {
         dev::v4f *p = (dev::v4f *)((float *)ep.out + o);
         const dev::v4f r = *p, ls = *(const dev::v4f *)(ep.scale + col);
@@ -65,6 +76,43 @@ __device__ __forceinline__ void epilogue_store4(const LinearEpilogue &ep, uint32
     } else {
         *(dev::v2u *)((uint16_t *)ep.out + o) = dev::v2u{dev::f32x2_to_bf16x2(v[0], v[1]), dev::f32x2_to_bf16x2(v[2], v[3])};
     }
+}
+
+// The t-th tile of `tm` rows over all groups (every group's last tile may be part full): its group and index there; false
+// behind the last one.  `columns` tiles of columns follow each other inside a group, row tiles fastest.  Every wavefront of
+// the block gets the same answer.
+__device__ __forceinline__ bool group_tile(const RowGroups &rg, uint32_t t, uint32_t tm, uint32_t columns, uint32_t *group, uint32_t *row_tile,
+                                           uint32_t *column) {
+    const uint32_t lane = threadIdx.x % 64;
+    uint32_t before = 0;
+    for (uint32_t g0 = 0; g0 < rg.groups; g0 += 64) {
+        const uint32_t own = g0 + lane < rg.groups ? (rg.count[g0 + lane] + tm - 1) / tm : 0;
+        uint32_t incl = own;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const uint32_t o = (uint32_t)__shfl_up((int)incl, off, 64);
+            if (lane >= (uint32_t)off) incl += o;
+        }
+        const uint64_t past = __ballot((before + incl) * columns > t);
+        if (past) {
+            const int first = __builtin_ctzll(past);
+            const uint32_t tiles = dev::lane_value(own, first), start = before + dev::lane_value(incl, first) - tiles;
+            const uint32_t r = t - start * columns;
+            *group = g0 + (uint32_t)first;
+            *row_tile = r % tiles;
+            *column = r / tiles;
+            return true;
+        }
+        before += dev::lane_value(incl, 63);
+    }
+    return false;
+}
+
+__device__ __forceinline__ uint32_t group_tiles(const RowGroups &rg, uint32_t tm) {
+    const uint32_t lane = threadIdx.x % 64;
+    uint32_t own = 0;
+    for (uint32_t g = lane; g < rg.groups; g += 64) own += (rg.count[g] + tm - 1) / tm;
+    return dev::wave_sum(own);
 }
 
 }  // namespace k

@@ -145,20 +145,21 @@ class Decoder:
 
 class LayeredDecoder(Decoder):
     """A decoder whose layers are described one by one (``fa_decoder_create_layered``): unquantized weights in bf16 or
-    f32, per layer a gated delta rule with a recurrent state or latent attention over the paged cache, and an optional
-    feed-forward.  Sequences, steps, prompt passes and sampling are ``Decoder``'s."""
+    f32, per layer a gated delta rule with a recurrent state or attention (latent or grouped-query) over the paged cache,
+    and an optional feed-forward, dense or of sparse experts.  Sequences, steps, prompt passes and sampling are
+    ``Decoder``'s."""
 
     takes_portions = True
 
     def __init__(self, ops, d_model, vocab, layers, norm_eps, logit_softcap, max_blocks_per_seq, num_blocks, max_batch,
-                 state_slots=None, dtype=capi.BF16, block_size=16):
+                 state_slots=None, dtype=capi.BF16, block_size=16, norm=capi.NORM_INPUT, embed_scale=1.0, position_base=0.0):
         """layers: one dict of ``capi.LayerConfig`` fields per layer."""
         self._ops = ops
         rows = (capi.LayerConfig * len(layers))(*[capi.LayerConfig(**l) for l in layers])
         recurrent = any(l["mixer"] == capi.MIXER_DELTA for l in layers)
         slots = max_batch if state_slots is None else state_slots
         self.cfg = capi.LayeredConfig(len(layers), d_model, vocab, block_size, max_blocks_per_seq, num_blocks, max_batch,
-                                      slots, norm_eps, logit_softcap, dtype, rows)
+                                      slots, norm_eps, logit_softcap, dtype, rows, norm, embed_scale, position_base)
         self.state_slots = slots if recurrent else 0
         self._h = C.c_void_p()
         check(lib.fa_decoder_create_layered(ops._ctx, C.byref(self.cfg), C.byref(self._h)))

@@ -111,12 +111,56 @@ def nugelix_layers(config):
     return out
 
 
+def nugelix(config):
+    """A Nugelix configuration as ``LayeredDecoder`` arguments."""
+    return {"d_model": _entry(config, "width", CONFIG_FILE), "vocab": _entry(config, "vocab", CONFIG_FILE), "layers": nugelix_layers(config),
+            "norm_eps": _entry(_entry(config, "norm", CONFIG_FILE), "eps", "norm"), "logit_softcap": config.get("logit_softcap") or 0.0}
+
+
+# ---- Zoferax: grouped-query attention and sparse experts, sublayers normed at their output ------------------------
+
+POSITION_BASE = 10000.0                                    # wavelengths of the additive positions
+
+
+def zoferax_layers(config):
+    """config.json's layer list as ``capi.LayerConfig`` fields."""
+    out = []
+    for i, layer in enumerate(_entry(config, "layers", CONFIG_FILE)):
+        where = "layer %d" % i
+        kind, mx = _entry(layer, "type", where), _entry(layer, "mixer", where)
+        if kind != "attention":
+            raise ConfigError("%s: unknown type %r" % (where, kind))
+        l = {key: _entry(mx, key, where + " mixer") for key in ("heads", "kv_heads", "dim", "vdim", "scale")}
+        l.update(mixer=capi.MIXER_ATTENTION, attention=capi.ATTENTION_BIAS | capi.ATTENTION_QK_NORM, kv_from=-1)
+        if mx.get("kv_from") is not None:
+            l["kv_from"] = mx["kv_from"]
+        mlp = layer.get("mlp")
+        if mlp is not None:
+            if _entry(mlp, "kind", where + " mlp") != "moe":
+                raise ConfigError("%s: unknown feed-forward %r" % (where, mlp["kind"]))
+            router = _entry(mlp, "router", where + " mlp")
+            l.update(d_ffn=_entry(_entry(mlp, "expert", where + " mlp"), "ff", where + " expert"),
+                     experts=_entry(router, "experts", where + " router"), top=_entry(router, "top", where + " router"))
+        out.append(l)
+    return out
+
+
+def zoferax(config):
+    """A Zoferax configuration as ``LayeredDecoder`` arguments."""
+    return {"d_model": _entry(config, "width", CONFIG_FILE), "vocab": _entry(config, "vocab", CONFIG_FILE), "layers": zoferax_layers(config),
+            "norm_eps": _entry(_entry(config, "norm", CONFIG_FILE), "eps", "norm"), "logit_softcap": 0.0, "norm": capi.NORM_OUTPUT,
+            "embed_scale": _entry(_entry(config, "embedding", CONFIG_FILE), "scale", "embedding"), "position_base": POSITION_BASE}
+
+
+# designs made of described layers: architecture name -> function(config) -> LayeredDecoder arguments
+LAYERED = {"Nugelix": nugelix, "Zoferax": zoferax}
+
+
 def build_layered(ops, config, dtype, capacity):
-    """The decoder a Nugelix configuration describes, without weights."""
-    return LayeredDecoder(ops, _entry(config, "width", CONFIG_FILE), _entry(config, "vocab", CONFIG_FILE), nugelix_layers(config),
-                          _entry(_entry(config, "norm", CONFIG_FILE), "eps", "norm"), config.get("logit_softcap") or 0.0,
-                          capacity.num_blocks, capacity.num_blocks, capacity.max_batch, capacity.state_slots, DTYPES[dtype],
-                          capacity.block_size)
+    """The layered decoder a configuration describes, without weights."""
+    return LayeredDecoder(ops, max_blocks_per_seq=capacity.num_blocks, num_blocks=capacity.num_blocks, max_batch=capacity.max_batch,
+                          state_slots=capacity.state_slots, dtype=DTYPES[dtype], block_size=capacity.block_size,
+                          **LAYERED[architecture_of(config)](config))
 
 
 def install_weights(decoder, typed):
@@ -137,7 +181,8 @@ def install_weights(decoder, typed):
 
 
 @register("Nugelix")
-def _nugelix(ops, config, weights, dtype, capacity):
+@register("Zoferax")
+def _layered(ops, config, weights, dtype, capacity):
     typed = st.load_safetensors_typed(weights)
     decoder = build_layered(ops, config, dtype, capacity)
     try:

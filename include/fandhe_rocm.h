@@ -564,22 +564,30 @@ fa_status fa_decoder_read_seq_lens(fa_context *ctx, fa_decoder *dec, uint32_t *s
 fa_status fa_decoder_logits_buffer(fa_decoder *dec, fa_buffer **out);
 
 /* -------------------------------------------------------- layered decoders */
-/* A decoder whose layers are described one by one: pre-norm (layer norm) sublayers with a layer scale, a mixer per
- * layer (gated delta rule with a recurrent state, or latent attention over the paged cache) and an optional clamped
- * GLU feed-forward, on unquantized weights.  No counterpart in the reference.  It is an fa_decoder: sequences, tokens,
+/* A decoder whose layers are described one by one, on unquantized weights: a mixer per layer (gated delta rule with a
+ * recurrent state; latent attention or grouped-query attention over the paged cache) and an optional feed-forward
+ * (clamped GLU, or sparse experts).  No counterpart in the reference.  It is an fa_decoder: sequences, tokens,
  * sampling, steps, prompt passes, verification and the read-outs are the calls above. */
-typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1 } fa_mixer_kind;
+typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1, FA_MIXER_ATTENTION = 2 } fa_mixer_kind;
+/* How sublayers meet the residual stream x.  FA_NORM_INPUT: x += scale * f(layer_norm(x)), a layer scale per channel;
+ * FA_NORM_OUTPUT: x += rms_norm(f(x)).  The final norm is of the same kind. */
+typedef enum { FA_NORM_INPUT = 0, FA_NORM_OUTPUT = 1 } fa_norm_kind;
+/* Attention: projections with biases; RMS norm of the whole query and key projections, over all heads at once. */
+enum { FA_ATTENTION_BIAS = 1, FA_ATTENTION_QK_NORM = 2 };
 typedef struct {
     int32_t mixer;                /* fa_mixer_kind */
     uint32_t heads, dim, vdim;    /* per head: query / key dims (latent attention: the unrotated part), value dims */
-    uint32_t kv_heads, conv;      /* delta: q / k heads, taps of the short convolution (1..=16) */
+    uint32_t kv_heads, conv;      /* delta: q / k heads, taps of the short convolution (1..=16); attention: key / value heads */
     uint32_t q_rank, kv_rank;     /* latent attention: sizes of the two latents */
     uint32_t rot_dim, window;     /* latent attention: rotated dims (even), visible keys incl. the token's own */
-    int32_t kv_from;              /* latent attention: the earlier layer whose cache is used, -1 for its own */
-    float scale;                  /* latent attention: factor of the scores */
+    int32_t kv_from;              /* both attentions: the earlier layer whose cache is used, -1 for its own */
+    float scale;                  /* both attentions: factor of the scores */
     double rot_base;
-    uint32_t d_ffn;               /* 0: no feed-forward */
+    uint32_t d_ffn;               /* 0: no feed-forward; with experts: size of one */
     float ffn_limit, ffn_alpha;   /* g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + 1) */
+    uint32_t attention;           /* attention: FA_ATTENTION_* */
+    uint32_t experts, top;        /* experts > 0 (up to 256): every token takes `top` (up to 64) of them, weighted by a softmax over their
+                                     router logits; an expert is W_down relu(W_up x)^2.  With FA_NORM_OUTPUT only */
 } fa_layer_config;
 typedef struct {
     uint32_t n_layers, d_model, vocab;
@@ -589,6 +597,10 @@ typedef struct {
     float norm_eps, logit_softcap;        /* softcap 0: none */
     fa_dtype dtype;               /* FA_BF16: weights, activations and cache in bf16; FA_F32: everything in f32 */
     const fa_layer_config *layers;        /* [n_layers], copied */
+    int32_t norm;                 /* fa_norm_kind */
+    float embed_scale;            /* factor of the embedding rows; 0: one */
+    double position_base;         /* FA_NORM_OUTPUT, above 0: sin(p base^(-2i / d_model)) is added to entry 2i of the embedding of position p, the
+                                     cosine to entry 2i + 1 */
 } fa_layered_config;
 fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cfg, fa_decoder **out);
 /* Number of weight tensors the decoder takes and the i-th one's name and shape (cols 0: a vector). */

@@ -113,10 +113,14 @@ fa_status fa_probe_l2_path(fa_context *ctx, const fa_buffer *cold, uint64_t cold
  * key 27: prompt passes whose q | k | v projection runs on the weight-stationary kernel: 0: RoPE, the bf16 rounding and
  *        the K / V append in that kernel's epilogue, 1: a pass of their own behind it;
  * layered decoders: key 28: rows per internal pass of a long prompt, from 64 up (smaller: the built-in 8192);
- * key 29: bf16 linears: 2: never the large-tile kernel, 3: never four column tiles per block;
+ * key 29: bf16 linears: 2: never the large-tile kernel, 3: never four column tiles per block; experts' linears: 4: weights
+ *        streamed past the rows, 5: 128 x 128 tiles, 6: large tiles, whatever the number of rows;
  * key 30: latent attention: 1: the plain kernel, 2: the absorbed form for every pass, 3: the expanded form wherever it
  *        can run; key 31: gated delta rule: 1: token by token for prompts too;
- * key 32: blocks per compute unit the key split of the absorbed form aims at. */
+ * key 32: blocks per compute unit the key split of the absorbed form aims at;
+ * key 33: grouped-query attention: 1: the plain kernel, 2: the few-rows kernel for every sequence, 3: the many-rows kernel
+ *        for every sequence; key 34: blocks per compute unit its key split aims at;
+ * key 35: routing of experts: 1: always in the residual update's launch, 2: always in a launch of its own. */
 fa_status fa_set_tuning(int32_t key, int32_t value);
 
 /* What the context found when it was created: xcd_local = 1 when workgroups b and b + 8 of a launch were seen to

@@ -1,5 +1,6 @@
 """Oracle: the mechanisms of the layered decoders (gated delta rule, latent attention, clamped GLU feed-forward,
-layer norm with layer scale, soft-capped head), one function per mechanism, in float64 and token by token.
+layer norm with layer scale, soft-capped head; grouped-query attention with normed projections, sparse experts, additive
+positions, norms on the sublayers' outputs), one function per mechanism, in float64 and token by token.
 
 TEST INFRASTRUCTURE ONLY: written from the equations, for whole sequences, without a cache, a batch or any code
 of the product; only tests and the smoke check may import it.
@@ -126,9 +127,83 @@ def softcap(z, cap):
     return cap * np.tanh(z / cap)
 
 
+def sinusoid(positions, width):
+    """Additive positions: sine in the even entries, cosine in the odd ones, of wavelengths growing to 10000 x 2 pi."""
+    out = np.empty((len(positions), width))
+    for e in range(width):
+        a = np.asarray(positions, dtype=np.float64) * 10000.0 ** (-(e - e % 2) / width)
+        out[:, e] = np.cos(a) if e % 2 else np.sin(a)
+    return out
+
+
+def grouped_kv(h, w, p, mx, eps):
+    """What an attention layer with projections of its own keeps of every token: normed keys [T, G, dim], values
+    [T, G, vdim].  The norm runs over the keys of all heads at once."""
+    G = mx["kv_heads"]
+    k = rms_norm(h @ w[p + "k"].T + w[p + "k.b"], w[p + "k.norm"], eps)
+    v = h @ w[p + "v"].T + w[p + "v.b"]
+    return k.reshape(len(h), G, mx["dim"]), v.reshape(len(h), G, mx["vdim"])
+
+
+def grouped_attention(q, k, v, scale):
+    """q [T, H, d], k [T, G, d], v [T, G, dv]: causal softmax attention, consecutive query heads sharing a key head."""
+    share = q.shape[1] // k.shape[1]
+    return windowed_softmax_attention(q, np.repeat(k, share, axis=1), np.repeat(v, share, axis=1), scale, len(q))
+
+
+def grouped_mixer(h, kept, w, p, mx, eps):
+    """The attention layer over kept = (keys, values), which may be another layer's."""
+    q = rms_norm(h @ w[p + "q"].T + w[p + "q.b"], w[p + "q.norm"], eps)
+    o = grouped_attention(q.reshape(len(h), mx["heads"], mx["dim"]), kept[0], kept[1], mx["scale"])
+    return o.reshape(len(h), -1) @ w[p + "o"].T
+
+
+def route(z, top):
+    """Router logits [T, experts] -> weights [T, experts]: a softmax over the `top` largest, zero elsewhere."""
+    out = np.zeros_like(z)
+    for t, row in enumerate(z):
+        best = np.argsort(-row, kind="stable")[:top]
+        e = np.exp(row[best] - row[best].max())
+        out[t, best] = e / e.sum()
+    return out
+
+
+def squared_relu_expert(h, w, p):
+    return np.maximum(h @ w[p + "up"].T, 0.0) ** 2 @ w[p + "down"].T
+
+
+def sparse_experts(h, w, p, mlp):
+    g = route(h @ w[p + "router"].T, mlp["router"]["top"])
+    y = np.zeros_like(h)
+    for e in range(mlp["router"]["experts"]):
+        rows = np.nonzero(g[:, e])[0]
+        y[rows] += g[rows, e:e + 1] * squared_relu_expert(h[rows], w, p + "e%d." % e)
+    return y
+
+
+def forward_zoferax(config, w, tokens, layers_out=None):
+    """Embedding with additive positions; sublayers read the residual itself and their outputs are normed."""
+    eps = config["norm"]["eps"]
+    x = w["embed"][np.asarray(tokens, dtype=np.int64)] * config["embedding"]["scale"] + sinusoid(np.arange(len(tokens)), config["width"])
+    kept = {}
+    for i, layer in enumerate(config["layers"]):
+        p, mx = "l%d." % i, layer["mixer"]
+        src = mx.get("kv_from", i)
+        if src == i:
+            kept[i] = grouped_kv(x, w, p + "mix.", mx, eps)
+        x = x + rms_norm(grouped_mixer(x, kept[src], w, p + "mix.", mx, eps), w[p + "norm1"], eps)
+        if layer["mlp"] is not None:
+            x = x + rms_norm(sparse_experts(x, w, p + "mlp.", layer["mlp"]), w[p + "norm2"], eps)
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return rms_norm(x, w["final.norm"], eps) @ w["head"].T
+
+
 def forward(config, weights, tokens, layers_out=None):
     """Logits [T, vocab] of one whole sequence; layers_out (a list) receives the residual after every layer."""
     w = {n: np.asarray(a, dtype=np.float64) for n, a in weights.items()}
+    if config["architecture"] == "Zoferax":
+        return forward_zoferax(config, w, tokens, layers_out)
     eps = config["norm"]["eps"]
     x = w["embed"][np.asarray(tokens, dtype=np.int64)]
     kept = {}
