@@ -172,8 +172,20 @@ def squared_relu_expert(h, w, p):
     return np.maximum(h @ w[p + "up"].T, 0.0) ** 2 @ w[p + "down"].T
 
 
-def sparse_experts(h, w, p, mlp):
-    g = route(h @ w[p + "router"].T, mlp["router"]["top"])
+def route_margin(z, top):
+    """How far every row's choice is from another one: the gap between the last chosen logit and the first left out,
+    relative to the row's spread (inf where nothing is left out)."""
+    if top == z.shape[1]:
+        return np.full(len(z), np.inf)
+    s = -np.sort(-z, axis=1)
+    return (s[:, top - 1] - s[:, top]) / (z.std(axis=1) + 1e-30)
+
+
+def sparse_experts(h, w, p, mlp, margins=None):
+    z = h @ w[p + "router"].T
+    g = route(z, mlp["router"]["top"])
+    if margins is not None:
+        margins.append(route_margin(z, mlp["router"]["top"]))
     y = np.zeros_like(h)
     for e in range(mlp["router"]["experts"]):
         rows = np.nonzero(g[:, e])[0]
@@ -181,7 +193,7 @@ def sparse_experts(h, w, p, mlp):
     return y
 
 
-def forward_zoferax(config, w, tokens, layers_out=None):
+def forward_zoferax(config, w, tokens, layers_out=None, margins=None):
     """Embedding with additive positions; sublayers read the residual itself and their outputs are normed."""
     eps = config["norm"]["eps"]
     x = w["embed"][np.asarray(tokens, dtype=np.int64)] * config["embedding"]["scale"] + sinusoid(np.arange(len(tokens)), config["width"])
@@ -193,17 +205,18 @@ def forward_zoferax(config, w, tokens, layers_out=None):
             kept[i] = grouped_kv(x, w, p + "mix.", mx, eps)
         x = x + rms_norm(grouped_mixer(x, kept[src], w, p + "mix.", mx, eps), w[p + "norm1"], eps)
         if layer["mlp"] is not None:
-            x = x + rms_norm(sparse_experts(x, w, p + "mlp.", layer["mlp"]), w[p + "norm2"], eps)
+            x = x + rms_norm(sparse_experts(x, w, p + "mlp.", layer["mlp"], margins), w[p + "norm2"], eps)
         if layers_out is not None:
             layers_out.append(x.copy())
     return rms_norm(x, w["final.norm"], eps) @ w["head"].T
 
 
-def forward(config, weights, tokens, layers_out=None):
-    """Logits [T, vocab] of one whole sequence; layers_out (a list) receives the residual after every layer."""
+def forward(config, weights, tokens, layers_out=None, margins=None):
+    """Logits [T, vocab] of one whole sequence; layers_out (a list) receives the residual after every layer, margins (a
+    list) the routing margins of every layer of sparse experts."""
     w = {n: np.asarray(a, dtype=np.float64) for n, a in weights.items()}
     if config["architecture"] == "Zoferax":
-        return forward_zoferax(config, w, tokens, layers_out)
+        return forward_zoferax(config, w, tokens, layers_out, margins)
     eps = config["norm"]["eps"]
     x = w["embed"][np.asarray(tokens, dtype=np.int64)]
     kept = {}

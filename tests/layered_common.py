@@ -30,12 +30,46 @@ def config(layers, width=76, vocab=131, eps=1e-5, softcap=12.0):
     return {"architecture": "Nugelix", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps}, "logit_softcap": softcap}
 
 
+def attention(heads=6, kv_heads=2, dim=20, vdim=12, scale=None, kv_from=None, mlp=None):
+    mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": 2.0 * dim ** -0.5 if scale is None else scale}
+    if kv_from is not None:
+        mx["kv_from"] = kv_from
+    return {"type": "attention", "mixer": mx, "mlp": mlp}
+
+
+def experts(n=5, top=2, ff=28):
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": n, "top": top}}
+
+
+def zoferax(layers, width=76, vocab=131, eps=1e-5, scale=1.7):
+    return {"architecture": "Zoferax", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps}, "embedding": {"scale": scale}}
+
+
 def bf16_round(a):
     u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
     return ((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32).view(np.float32)
 
 
+def zoferax_shapes(cfg):
+    D = cfg["width"]
+    out = {"embed": (cfg["vocab"], D), "head": (cfg["vocab"], D), "final.norm": (D,)}
+    for i, l in enumerate(cfg["layers"]):
+        p, mx = "l%d." % i, l["mixer"]
+        q, k, v = (mx[h] * mx[d] for h, d in (("heads", "dim"), ("kv_heads", "dim"), ("kv_heads", "vdim")))
+        out.update({p + "norm1": (D,), p + "mix.q": (q, D), p + "mix.q.b": (q,), p + "mix.q.norm": (q,), p + "mix.o": (D, mx["heads"] * mx["vdim"])})
+        if "kv_from" not in mx:
+            out.update({p + "mix.k": (k, D), p + "mix.k.b": (k,), p + "mix.k.norm": (k,), p + "mix.v": (v, D), p + "mix.v.b": (v,)})
+        if l["mlp"]:
+            n, ff = l["mlp"]["router"]["experts"], l["mlp"]["expert"]["ff"]
+            out.update({p + "norm2": (D,), p + "mlp.router": (n, D)})
+            for e in range(n):
+                out.update({p + "mlp.e%d.up" % e: (ff, D), p + "mlp.e%d.down" % e: (D, ff)})
+    return out
+
+
 def shapes(cfg):
+    if cfg["architecture"] == "Zoferax":
+        return zoferax_shapes(cfg)
     D = cfg["width"]
     out = {"embed": (cfg["vocab"], D), "head": (cfg["vocab"], D), "final.norm": (D,)}
     for i, l in enumerate(cfg["layers"]):
@@ -76,7 +110,7 @@ def weights(cfg, seed=0):
             a = 1.0 + 0.3 * rng.normal(size=shape)
         elif leaf in ("ls1", "ls2"):
             a = rng.uniform(0.3, 1.2, shape) * rng.choice([-1.0, 1.0], shape)
-        elif leaf == "embed":
+        elif leaf == "embed" or len(shape) == 1:               # also the projections' biases
             a = rng.normal(size=shape)
         elif leaf in ("uq", "uk", "gate", "up", "b"):
             a = rng.normal(size=shape) * 2.0 / np.sqrt(shape[1])
@@ -102,6 +136,13 @@ def make_decoder(ops, cfg, w, dtype="float32", max_tokens=512, max_batch=4, stat
             typed[n] = TypedTensor("F32", a.shape, a)
     models.install_weights(d, typed)
     return d
+
+
+def decided(cfg, w, toks, least=0.05):
+    """The oracle's logits, and which positions' experts are no close calls (a rounding cannot change them)."""
+    margins = []
+    want = oracle.forward(cfg, w, toks, margins=margins)
+    return want, np.min(margins + [np.full(len(toks), np.inf)], axis=0) >= least
 
 
 def error(got, want):

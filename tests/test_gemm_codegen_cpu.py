@@ -27,7 +27,7 @@ def test_no_accumulator_is_read_before_the_drain():
                os.path.join(tmp, "k.s")]
         subprocess.run(cmd, check=True, capture_output=True, cwd=tmp)
         text = open(os.path.join(tmp, "k.s")).read()
-    kernels = re.findall(r"^(_ZN2fa1k\S*gemm_mfma_big_kernel\w*):[^\n]*\n(.*?)s_endpgm", text, flags=re.S | re.M)
+    kernels = re.findall(r"^(_ZN2fa1k\S*gemm_mfma_big_kernel\w*):[^\n]*\n(.*?)^\.Lfunc_end", text, flags=re.S | re.M)
     assert len(kernels) >= 12, "expected every (type, width, wavefront count) instantiation"
     for name, body in kernels:
         lines = body.split("\n")

@@ -96,11 +96,103 @@ def test_a_planted_mistake_exceeds_the_gpu_tests_tolerance(name):
     assert lc.error(oracle.forward(wrong, w, toks), good) > 30 * 2e-4
 
 
+def test_grouped_attention_shares_heads_and_sees_the_past_only():
+    rng = np.random.default_rng(3)
+    q, k, v = rng.normal(size=(7, 4, 5)), rng.normal(size=(7, 2, 5)), rng.normal(size=(7, 2, 3))
+    got = oracle.grouped_attention(q, k, v, 0.6)
+    for t in range(7):
+        for h in range(4):
+            e = np.exp(0.6 * k[:t + 1, h // 2] @ q[t, h])
+            assert np.allclose(got[t, h], e @ v[:t + 1, h // 2] / e.sum())
+
+
+def test_projection_norm_runs_over_all_heads():
+    rng = np.random.default_rng(4)
+    mx = {"heads": 4, "kv_heads": 2, "dim": 3, "vdim": 2, "scale": 1.0}
+    w = {"k": rng.normal(size=(6, 5)), "k.b": rng.normal(size=6), "k.norm": rng.normal(size=6), "v": rng.normal(size=(4, 5)), "v.b": rng.normal(size=4)}
+    h = rng.normal(size=(3, 5))
+    k, v = oracle.grouped_kv(h, w, "", mx, 1e-3)
+    z = w["k"] @ h[1] + w["k.b"]
+    assert np.allclose(k[1].ravel(), z / np.sqrt((z ** 2).mean() + 1e-3) * w["k.norm"])
+    assert np.allclose(v[2].ravel(), w["v"] @ h[2] + w["v.b"])
+
+
+def test_routing_takes_the_largest_and_weighs_them_among_themselves():
+    z = np.array([[0.0, 3.0, 1.0, 2.0], [5.0, 5.0, -1.0, 4.0]])
+    g = oracle.route(z, 2)
+    assert np.allclose(g[0], [0, 1 / (1 + np.exp(-1)), 0, 1 / (1 + np.exp(1))])
+    assert np.allclose(g[1], [0.5, 0.5, 0, 0])
+    assert np.allclose(oracle.route(z, 4).sum(1), 1) and np.allclose(oracle.route(z, 1)[0], [0, 1, 0, 0])
+    assert np.allclose(oracle.route_margin(z, 2) * z.std(axis=1), [1.0, 1.0]) and np.isinf(oracle.route_margin(z, 4)).all()
+    w = {"router": np.array([[1.0], [0.0]]), "e0.up": np.array([[2.0]]), "e0.down": np.array([[3.0]]), "e1.up": np.array([[-1.0]]), "e1.down": np.array([[1.0]])}
+    y = oracle.sparse_experts(np.array([[2.0], [-2.0]]), w, "", {"router": {"experts": 2, "top": 1}})
+    assert np.allclose(y, [[48.0], [4.0]])
+
+
+def test_additive_positions_closed_form():
+    s = oracle.sinusoid([0, 7, 1000], 6)
+    z = np.exp(1j * np.array([0, 7, 1000])[:, None] * 10000.0 ** (-2.0 * np.arange(3) / 6))
+    assert np.allclose(s[:, 0::2], z.imag) and np.allclose(s[:, 1::2], z.real)
+    assert oracle.sinusoid([5], 3).shape == (1, 3) and np.allclose(oracle.sinusoid([5], 3)[0, 2], np.sin(5 * 10000.0 ** (-2 / 3)))
+
+
+def _change_mixers(cfg, key, value):
+    for l in cfg["layers"]:
+        l["mixer"][key] = value(l["mixer"][key])
+
+
+ZOFERAX_MISTAKES = {
+    "score scale": lambda c: _change_mixers(c, "scale", lambda s: s * 1.05),
+    "norm eps": lambda c: c["norm"].update(eps=0.05),
+    "embedding scale": lambda c: c["embedding"].update(scale=c["embedding"]["scale"] * 1.05),
+    "one expert more": lambda c: [l["mlp"]["router"].update(top=l["mlp"]["router"]["top"] + 1) for l in c["layers"] if l["mlp"]],
+    "cache of the wrong layer": lambda c: c["layers"][2]["mixer"].update(kv_from=1),
+    "feed-forward left out": lambda c: c["layers"][0].update(mlp=None),
+}
+
+
+@pytest.mark.parametrize("name", sorted(ZOFERAX_MISTAKES))
+def test_a_planted_mistake_in_a_zoferax_model_exceeds_the_gpu_tests_tolerance(name):
+    cfg = lc.zoferax([lc.attention(mlp=lc.experts()), lc.attention(mlp=lc.experts(4, 1)), lc.attention(kv_from=0)])
+    w = lc.weights(cfg, 5)
+    toks = lc.tokens(cfg, 40, 5)
+    good = oracle.forward(cfg, w, toks)
+    wrong = copy.deepcopy(cfg)
+    ZOFERAX_MISTAKES[name](wrong)
+    assert lc.error(oracle.forward(wrong, w, toks), good) > 30 * 2e-4
+
+
+@pytest.mark.parametrize("mistake", ["positions", "a key head each", "norm per head", "equal weights", "plain relu", "no bias"])
+def test_another_reading_of_a_zoferax_mechanism_exceeds_the_gpu_tests_tolerance(mistake, monkeypatch):
+    """The oracle with one mechanism computed otherwise."""
+    cfg = lc.zoferax([lc.attention(mlp=lc.experts())])
+    w = lc.weights(cfg, 5)
+    toks = lc.tokens(cfg, 40, 5)
+    good = oracle.forward(cfg, w, toks)
+    if mistake == "positions":
+        sinusoid = oracle.sinusoid
+        monkeypatch.setattr(oracle, "sinusoid", lambda p, width: sinusoid(np.asarray(p) + 1, width))
+    elif mistake == "a key head each":
+        monkeypatch.setattr(oracle, "grouped_attention", lambda q, k, v, s: oracle.windowed_softmax_attention(
+            q, np.tile(k, (1, q.shape[1] // k.shape[1], 1)), np.tile(v, (1, q.shape[1] // v.shape[1], 1)), s, len(q)))
+    elif mistake == "norm per head":
+        norm = oracle.rms_norm
+        monkeypatch.setattr(oracle, "rms_norm", lambda x, g, eps: norm(x, g, eps) if x.shape[-1] == cfg["width"] else norm(x.reshape(len(x), -1, 20), 1.0, eps).reshape(x.shape) * g)
+    elif mistake == "equal weights":
+        route = oracle.route
+        monkeypatch.setattr(oracle, "route", lambda z, top: (route(z, top) > 0) / top)
+    elif mistake == "plain relu":
+        monkeypatch.setattr(oracle, "squared_relu_expert", lambda h, v, p: np.maximum(h @ v[p + "up"].T, 0.0) @ v[p + "down"].T)
+    else:
+        w = dict(w, **{"l0.mix.k.b": np.zeros_like(w["l0.mix.k.b"])})
+    assert lc.error(oracle.forward(cfg, w, toks), good) > 30 * 2e-4
+
+
 # ---- configuration ---------------------------------------------------------------------------------------------
 
 def test_registry_picks_by_architecture_and_rejects_what_it_does_not_know(tmp_path):
     models = _fa().models
-    assert {"Nugelix", "LlamaForCausalLM"} <= set(models.ARCHITECTURES)
+    assert {"Nugelix", "Zoferax", "LlamaForCausalLM"} <= set(models.ARCHITECTURES)
     (tmp_path / "config.json").write_text(json.dumps({"architecture": "Nonesuch"}))
     with pytest.raises(models.ConfigError, match="unknown architecture"):
         models.load_model(None, str(tmp_path))
@@ -134,6 +226,30 @@ def test_layer_list_reads_every_size_and_names_what_is_missing():
     bad["layers"][1]["type"] = "other"
     with pytest.raises(models.ConfigError, match="unknown type"):
         models.nugelix_layers(bad)
+
+
+def test_zoferax_configuration_reads_every_size_and_names_what_is_missing():
+    fa = _fa()
+    models, capi = fa.models, fa.capi
+    cfg = lc.zoferax([lc.attention(heads=12, kv_heads=4, dim=10, vdim=6, scale=0.25, mlp=lc.experts(7, 3, 44)), lc.attention(kv_from=0)], scale=2.5)
+    a = models.zoferax(cfg)
+    assert (a["d_model"], a["vocab"], a["norm"], a["embed_scale"], a["position_base"], a["norm_eps"]) == (76, 131, capi.NORM_OUTPUT, 2.5, 10000.0, 1e-5)
+    l, m = a["layers"]
+    assert (l["mixer"], l["heads"], l["kv_heads"], l["dim"], l["vdim"], l["scale"], l["kv_from"]) == (capi.MIXER_ATTENTION, 12, 4, 10, 6, 0.25, -1)
+    assert (l["d_ffn"], l["experts"], l["top"]) == (44, 7, 3) and m["kv_from"] == 0 and "d_ffn" not in m
+    for path in (("mixer", "kv_heads"), ("mixer", "scale"), ("type",), ("mlp", "kind"), ("mlp", "router", "top"), ("mlp", "expert", "ff")):
+        bad = copy.deepcopy(cfg)
+        at = bad["layers"][0]
+        for key in path[:-1]:
+            at = at[key]
+        del at[path[-1]]
+        with pytest.raises(models.ConfigError, match=path[-1]):
+            models.zoferax(bad)
+    for change in ({"type": "delta"}, {"mlp": {"kind": "dense", "ff": 3}}):
+        bad = copy.deepcopy(cfg)
+        bad["layers"][1].update(change)
+        with pytest.raises(models.ConfigError, match="unknown"):
+            models.zoferax(bad)
 
 
 # ---- batching on a fake decoder ---------------------------------------------------------------------------------
