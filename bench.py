@@ -105,7 +105,8 @@ def make_tables(rng, ctxs, extra_tokens, bs, num_blocks=None):
 
 
 # ------------------------------------------------------------------ layered decoders
-# Nugelix stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward and depth.
+# Nugelix and Zoferax stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward (of the
+# experts: those one token takes) and depth.
 def _nugelix(width, heads, q_rank, window, ff, d_heads, d_kv_heads, repeat):
     latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff, "limit": 7.0},
               "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": q_rank, "kv_rank": 512, "mask": {"size": window},
@@ -115,30 +116,45 @@ def _nugelix(width, heads, q_rank, window, ff, d_heads, d_kv_heads, repeat):
             "layers": [latent, delta, delta, delta] * repeat}
 
 
-LAYERED = {"large": (_nugelix(4096, 32, 1536, 2048, 14336, 32, 16, 2), dict(d_model=4096, n_heads=32, n_kv_heads=8, d_ffn=14336)),
-           "small": (_nugelix(2048, 16, 768, 1024, 8192, 16, 8, 2), dict(d_model=2048, n_heads=16, n_kv_heads=4, d_ffn=8192))}
+def _zoferax(width, heads, kv_heads, vdim, experts, top, ff, layers, shared):
+    def layer(i):
+        mixer = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": vdim, "scale": 128 ** -0.5}
+        if i >= layers - shared:
+            mixer["kv_from"] = layers - shared - 1
+        return {"type": "attention", "mixer": mixer, "mlp": {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}}
+    return {"architecture": "Zoferax", "width": width, "vocab": 32000, "norm": {"eps": 1e-5}, "embedding": {"scale": width ** 0.5},
+            "layers": [layer(i) for i in range(layers)]}
 
 
-def build_nugelix(fa, be, config, max_tokens, batch):
+LAYERED = {"large": dict(nugelix=_nugelix(4096, 32, 1536, 2048, 14336, 32, 16, 2), zoferax=_zoferax(4096, 32, 8, 128, 16, 4, 5376, 8, 3),
+                         w8a8=dict(d_model=4096, n_heads=32, n_kv_heads=8, d_ffn=14336, n_layers=8, vocab=32000)),
+           "small": dict(nugelix=_nugelix(2048, 16, 768, 1024, 8192, 16, 8, 2), zoferax=_zoferax(2048, 16, 4, 64, 16, 4, 3072, 8, 3),
+                         w8a8=dict(d_model=2048, n_heads=16, n_kv_heads=4, d_ffn=8192, n_layers=8, vocab=32000))}
+
+
+def build_layered(fa, be, config, max_tokens, batch):
     dec = fa.models.build_layered(be, config, "bfloat16", fa.models.Capacity(max_tokens, batch))
     noise = np.random.default_rng(0).normal(size=1 << 20).astype(np.float32)
+    made = {}                                                     # equal shapes hold equal values
     for name, shape in dec.tensors().items():
         n, leaf = int(np.prod(shape)), name.split(".")[-1]
-        if "norm" in leaf or leaf in ("ls1", "ls2"):
-            a = np.ones(shape, np.float32)
-        elif leaf in ("A_log", "dt_bias"):
-            a = np.full(shape, -1.0, np.float32)
-        else:
-            a = np.resize(noise, n).reshape(shape) * np.float32(1.0 if leaf == "embed" else shape[1] ** -0.5)
-        dec.set_tensor(name, (a.view(np.uint32) >> 16).astype(np.uint16), bf16=True)
+        kind = "one" if "norm" in leaf or leaf in ("ls1", "ls2") else "minus one" if leaf in ("A_log", "dt_bias") else "embed" if leaf == "embed" else "noise"
+        if (shape, kind) not in made:
+            if kind == "noise" and len(shape) == 2:
+                a = np.resize(noise, n).reshape(shape) * np.float32(shape[1] ** -0.5)
+            elif kind in ("noise", "embed"):
+                a = np.resize(noise, n).reshape(shape)
+            else:
+                a = np.full(shape, 1.0 if kind == "one" else -1.0, np.float32)
+            made[shape, kind] = (a.view(np.uint32) >> 16).astype(np.uint16)
+        dec.set_tensor(name, made[shape, kind], bf16=True)
     return dec
 
 
-def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "w8a8")):
-    """Decode and prompt throughput of a Nugelix stack, and of the W8A8 decoder of equal width, feed-forward and depth."""
+def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "zoferax", "w8a8")):
+    """Decode and prompt throughput of layered stacks, and of the W8A8 decoder of equal width, feed-forward and depth."""
     lib = fa.capi.lib
-    config, shape = LAYERED[size]
-    V, layers = config["vocab"], len(config["layers"])
+    V = LAYERED[size]["w8a8"]["vocab"]
     rng = np.random.default_rng(1)
     most = max(decode_batches + tuple(b for b, _ in prompts))
     out = []
@@ -178,12 +194,13 @@ def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1
             dec.set_sequences(t, [length] * b)
         return set_rows
 
-    if "nugelix" in models:
-        dec = build_nugelix(fa, be, config, most * pages * 16, most)
-        measure("nugelix bf16", dec, rows_of(most * pages))
-        dec.close()
+    for model in ("nugelix", "zoferax"):
+        if model in models:
+            dec = build_layered(fa, be, LAYERED[size][model], most * pages * 16, most)
+            measure(model + " bf16", dec, rows_of(most * pages))
+            dec.close()
     if "w8a8" in models:
-        cfg = dict(MODEL, n_layers=layers, vocab=V, **shape)
+        cfg = dict(MODEL, **LAYERED[size]["w8a8"])
         h, keep, _, _, num_blocks = build_decoder(fa, be, cfg, most, [ctx] * most, 64)
         dcfg = fa.capi.DecoderConfig(cfg["n_layers"], cfg["d_model"], cfg["n_heads"], cfg["n_kv_heads"], cfg["head_dim"], cfg["d_ffn"], V,
                                      cfg["block_size"], (ctx + 65 + 15) // 16 + 1, num_blocks, most, cfg["rms_eps"], cfg["rope_theta"])
@@ -904,10 +921,10 @@ def main():
                     help="profiling aid: run only the dominant kernel at the workload's shape, or a plain "
                          "copy kernel of known size (counter calibration), a few launches, no JSON line")
     ap.add_argument("--layered-size", choices=tuple(LAYERED) + ("all",), default="all",
-                    help="with --only layered: the sizes of the Nugelix stack (and of the W8A8 decoder beside it)")
+                    help="with --only layered: the sizes of the layered stacks (and of the W8A8 decoder beside them)")
     ap.add_argument("--layered-phase", choices=("all", "decode", "prompt"), default="all",
                     help="with --only layered: all, or one shape of one phase (for a kernel trace)")
-    ap.add_argument("--layered-model", choices=("both", "nugelix", "w8a8"), default="both", help="with --only layered: one of the two decoders")
+    ap.add_argument("--layered-model", choices=("all", "nugelix", "zoferax", "w8a8"), default="all", help="with --only layered: one of the decoders")
     a = ap.parse_args()
     if a.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (--gpus 1); nothing here shards across devices")
@@ -938,7 +955,7 @@ def main():
             return
         if a.only == "layered":
             kw = {"all": {}, "decode": dict(decode_batches=(32,), prompts=()), "prompt": dict(decode_batches=(), prompts=((4, 2048),))}[a.layered_phase]
-            if a.layered_model != "both":
+            if a.layered_model != "all":
                 kw["models"] = (a.layered_model,)
             for size in LAYERED if a.layered_size == "all" else (a.layered_size,):
                 for r in bench_layered(fa, be, size, **kw):

@@ -61,11 +61,12 @@ __device__ __forceinline__ void choose_experts(const float *logits, uint32_t exp
 }
 
 // ------------------------------------------------------------------ residual update
-// One block per row, VPT values of it per thread.
-template <typename T, int VPT, int NT, bool ROUTE>
+// One block per row, VPT pieces of it per thread: four values each (VEC, hidden a multiple of four), or one.
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC>
 __global__ void __launch_bounds__(NT)
     residual_norm_kernel(ResidualNorm rn, float *__restrict__ x, T *__restrict__ hn, uint32_t hidden, uint64_t ld, RouteIo io) {
-    constexpr int NW = NT / 64;
+    constexpr int NW = NT / 64, S = VEC ? 4 : 1;
+    typedef float piece __attribute__((ext_vector_type(S)));
     __shared__ float smem[NW], logits[ROUTE ? kMaxExperts : 1];
     extern __shared__ __attribute__((aligned(16))) uint8_t hs_raw[];     // ROUTE: the row of hn
     const uint64_t r = blockIdx.x;
@@ -73,38 +74,57 @@ __global__ void __launch_bounds__(NT)
     if (rn.clear && r == 0)
         for (uint32_t i = tid; i < rn.n_clear; i += NT) rn.clear[i] = 0;
     const float *y = rn.y + r * rn.parts * hidden;
-    float v[VPT], xv[VPT], sq = 0.0f;
+    float *xr = x + r * hidden;
+    piece v[VPT], xv[VPT];
+    float sq = 0.0f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const uint32_t c = tid + i * NT;
-        v[i] = 0.0f;
-        xv[i] = c < hidden ? x[r * hidden + c] : 0.0f;
-        if (!rn.gate) v[i] = c < hidden ? y[c] : 0.0f;
+        const uint32_t c = (tid + i * NT) * S;
+        v[i] = piece(0.0f);
+        xv[i] = c < hidden ? *(const piece *)(xr + c) : piece(0.0f);
+        if (!rn.gate && c < hidden) v[i] = *(const piece *)(y + c);
     }
     if (rn.gate) {
-        for (uint32_t p = 0; p < rn.parts; ++p) {
-            const float g = rn.gate[r * rn.parts + p];
+        for (uint32_t p = 0; p < rn.parts; p += 2) {                     // two parts at a time, in order
+            const bool two = p + 1 < rn.parts;
+            const float g0 = rn.gate[r * rn.parts + p], g1 = two ? rn.gate[r * rn.parts + p + 1] : 0.0f;
+            const float *y0 = y + (uint64_t)p * hidden, *y1 = two ? y0 + hidden : y0;
+            piece t0[VPT], t1[VPT];
 #pragma unroll
             for (int i = 0; i < VPT; ++i) {
-                const uint32_t c = tid + i * NT;
-                if (c < hidden) v[i] = fmaf(g, y[(uint64_t)p * hidden + c], v[i]);
+                const uint32_t c = (tid + i * NT) * S;
+                t0[i] = c < hidden ? *(const piece *)(y0 + c) : piece(0.0f);
+                t1[i] = c < hidden && two ? *(const piece *)(y1 + c) : piece(0.0f);
             }
+#pragma unroll
+            for (int i = 0; i < VPT; ++i)
+#pragma unroll
+                for (int e = 0; e < S; ++e) v[i][e] = fmaf(g1, t1[i][e], fmaf(g0, t0[i][e], v[i][e]));
         }
     }
 #pragma unroll
-    for (int i = 0; i < VPT; ++i) sq = fmaf(v[i], v[i], sq);
+    for (int i = 0; i < VPT; ++i)
+#pragma unroll
+        for (int e = 0; e < S; ++e) sq = fmaf(v[i][e], v[i][e], sq);
     const float rstd = 1.0f / sqrtf(block_sum<float, NW, true, true>(sq, smem) / (float)hidden + rn.eps);
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const uint32_t c = tid + i * NT;
+        const uint32_t c = (tid + i * NT) * S;
         if (c >= ld) continue;
-        float o = 0.0f;
+        piece o = piece(0.0f);
         if (c < hidden) {
-            o = xv[i] + v[i] * rstd * rn.w[c];
-            x[r * hidden + c] = o;
+            const piece w = *(const piece *)(rn.w + c);
+#pragma unroll
+            for (int e = 0; e < S; ++e) o[e] = xv[i][e] + v[i][e] * rstd * w[e];
+            *(piece *)(xr + c) = o;
         }
-        store_from_f32(hn + r * ld + c, o);
-        if constexpr (ROUTE) store_from_f32((T *)hs_raw + c, o);
+        auto put = [&](T *dst) {
+            if constexpr (sizeof(T) == 4) *(piece *)dst = o;
+            else if constexpr (VEC) *(v2u *)dst = v2u{f32x2_to_bf16x2(o[0], o[1]), f32x2_to_bf16x2(o[2], o[3])};
+            else *dst = f32_to_bf16(o[0]);
+        };
+        put(hn + r * ld + c);
+        if constexpr (ROUTE) put((T *)hs_raw + c);
     }
     if constexpr (ROUTE) {
         const int lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64);
@@ -230,26 +250,32 @@ __global__ void __launch_bounds__(256)
     }
 }
 
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC>
+void launch_residual_sized(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
+    const size_t lds = ROUTE ? ld * sizeof(T) + (sizeof(T) == 2 ? (io.experts + 15) / 16 * 16 * 17 * 4 : 0) : 0;
+    if (ROUTE && lds > 49152) {
+        static bool configured = false;
+        if (!configured) {
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, VPT, NT, ROUTE, VEC>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                      98304);
+            configured = true;
+        }
+    }
+    residual_norm_kernel<T, VPT, NT, ROUTE, VEC><<<(unsigned)rows, NT, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);
+}
+
+// rows up to 16384 values
 template <typename T, bool ROUTE>
 void launch_residual(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
-    const size_t lds = ROUTE ? ld * sizeof(T) + (sizeof(T) == 2 ? (io.experts + 15) / 16 * 16 * 17 * 4 : 0) : 0;
-#define FA_RN(V_, NT_)                                                                                                                    \
-    do {                                                                                                                                  \
-        if (lds > 49152) {                                                                                                                \
-            static bool configured = false;                                                                                               \
-            if (!configured) {                                                                                                            \
-                (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, V_, NT_, ROUTE>),                       \
-                                          hipFuncAttributeMaxDynamicSharedMemorySize, 98304);                                             \
-                configured = true;                                                                                                        \
-            }                                                                                                                             \
-        }                                                                                                                                 \
-        residual_norm_kernel<T, V_, NT_, ROUTE><<<(unsigned)rows, NT_, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);                    \
-    } while (0)
-    if (ld <= 1024) FA_RN(4, 256);
-    else if (rows > 256 && ld <= 4096) FA_RN(16, 256);
-    else if (ld <= 4096) FA_RN(4, 1024);
-    else FA_RN(16, 1024);                            // rows up to 16384
-#undef FA_RN
+    if (hidden % 4 == 0) {
+        if (ld <= 1024) launch_residual_sized<T, 1, 256, ROUTE, true>(rn, x, hn, rows, hidden, ld, io, s);
+        else if (rows > 256 && ld <= 4096) launch_residual_sized<T, 4, 256, ROUTE, true>(rn, x, hn, rows, hidden, ld, io, s);
+        else if (ld <= 4096) launch_residual_sized<T, 1, 1024, ROUTE, true>(rn, x, hn, rows, hidden, ld, io, s);
+        else launch_residual_sized<T, 4, 1024, ROUTE, true>(rn, x, hn, rows, hidden, ld, io, s);
+    } else {
+        if (ld <= 1024) launch_residual_sized<T, 4, 256, ROUTE, false>(rn, x, hn, rows, hidden, ld, io, s);
+        else launch_residual_sized<T, 16, 1024, ROUTE, false>(rn, x, hn, rows, hidden, ld, io, s);
+    }
 }
 
 template <int ET>

@@ -355,13 +355,15 @@ void launch_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
     linear_tile_kernel<MODE><<<grid, 256, 0, s>>>(a, lda, a_batch, wt, (uint32_t)m, w.n, w.n_tiles, w.k_tiles, ep, RowGroups{});
 }
 
-// Grouped rows: by the rows a group gets on average.  Few: weights streamed past them; a couple of hundred and more: tiles.
+// Grouped rows: by the rows a group gets on average.  Few: weights streamed past them; a hundred and more: large tiles
+// (16 experts of width 4096 and size 5376, 4 a token, passes of three layers, ms for 32 / 64 / 256 / 512 / 1024 rows: streamed 1.05 /
+// 1.28 / 2.54 / 4.07 / 7.32, 128 x 128 tiles 1.13 / 1.20 / 1.54 / 1.92 / 2.87, large tiles 1.18 / 1.28 / 1.68 / 1.81 / 2.39).
 template <int MODE>
 void launch_grouped_bf16(const uint16_t *a, uint64_t lda, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, int num_cus, hipStream_t s) {
     const uint8_t *wt = (const uint8_t *)w.w;
     const uint64_t mean = rg.entries / rg.groups;
     const int form = g_linear_form;
-    if (form == 4 || (form != 5 && form != 6 && mean <= 48)) {
+    if (form == 4 || (form != 5 && form != 6 && mean <= 10)) {
         const bool two = (uint64_t)w.n_tiles * std::min(rg.groups, rg.entries) >= 2 * (uint64_t)num_cus;
         const dim3 grid(two ? (w.n_tiles + 1) / 2 : w.n_tiles, rg.groups);
 #define FA_ROWS(MT_, NTW_) linear_rows_grouped_kernel<MT_, NTW_, 8, MODE><<<grid, 512, 0, s>>>(a, lda, wt, w.n, w.n_tiles, w.k_tiles, rg, ep)
@@ -371,7 +373,7 @@ void launch_grouped_bf16(const uint16_t *a, uint64_t lda, const LinearWeight &w,
 #undef FA_ROWS
         return;
     }
-    if (form == 6 || (form != 5 && mean >= 192 && lda == (uint64_t)w.k_tiles * 32 && w.n_tiles >= 14)) return gemm_bf16_big_grouped(a, w, rg, ep, s);
+    if (form == 6 || (form != 5 && mean >= 112 && lda == (uint64_t)w.k_tiles * 32 && w.n_tiles >= 14)) return gemm_bf16_big_grouped(a, w, rg, ep, s);
     const uint32_t tiles = rg.entries / 128 + std::min(rg.groups, rg.entries);
     linear_tile_kernel<MODE, true><<<tiles * ((w.n_tiles + 7) / 8), 256, 0, s>>>(a, lda, 0, wt, 0, w.n, w.n_tiles, w.k_tiles, ep, rg);
 }

@@ -34,7 +34,7 @@ def tolerance(dtype):
 def compare(got, want, sure, dtype, what=None):
     """All positions in f32; in bf16 those whose experts are no close calls."""
     keep = np.ones(len(want), bool) if dtype == "float32" else sure
-    assert keep.sum() >= 0.3 * len(want), "too few decided positions"
+    assert keep.sum() >= 0.2 * len(want), "too few decided positions"
     assert lc.error(np.asarray(got)[keep], want[keep]) < tolerance(dtype), what
 
 
