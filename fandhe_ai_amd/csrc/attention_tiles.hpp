@@ -50,20 +50,30 @@ __device__ __forceinline__ void hold(v8bf (&r)[N]) {
     }
 }
 
+// 2^x without the detour for subnormal results (weights that small count as zero)
+__device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
+
+// Maximum over the four lanes with equal lane % 16, in every one of them.
+__device__ __forceinline__ float column_max(float v) {
+    const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);      // rows of 16: 0 0 2 2 and 1 1 3 3
+    v = fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
+    const auto q = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return fmaxf(__uint_as_float(q[0]), __uint_as_float(q[1]));
+}
+
 // One online-softmax step of a column (query row): scores of eight keys per lane, lanes with equal lane % 16 share the
 // column.  Returns the factor for what was accumulated before; w receives the weights as two bf16 terms whose sum keeps
 // about 16 bits of them.
 __device__ __forceinline__ float softmax_step(const float (&sc)[8], float &m, float &l, v8bf &w_hi, v8bf &w_lo) {
     float mx = fmaxf(fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3])), fmaxf(fmaxf(sc[4], sc[5]), fmaxf(sc[6], sc[7])));
-    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    mx = column_max(mx);
     const float m_new = fmaxf(m, mx), ref = m_new == -INFINITY ? 0.0f : m_new;
-    const float fix = exp2f(m - ref);
+    const float fix = exp2_fast(m - ref);
     float sum = 0.0f;
     uint32_t hi[4], lo[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        const float a = exp2f(sc[2 * i] - ref), b = exp2f(sc[2 * i + 1] - ref);
+        const float a = exp2_fast(sc[2 * i] - ref), b = exp2_fast(sc[2 * i + 1] - ref);
         sum += a + b;
         hi[i] = f32x2_to_bf16x2(a, b);
         lo[i] = f32x2_to_bf16x2(a - bf16_lo(hi[i]), b - bf16_hi(hi[i]));

@@ -391,7 +391,7 @@ __global__ void __launch_bounds__(64) attention_merge_kernel(StreamParams p, Att
 // A block of four wavefronts takes 64 NQ columns of one (sequence, key head), every wavefront 16 NQ of them, and walks the keys
 // they see 32 at a time; K and V of a step are staged in LDS, two stages.
 template <int D, int V, int NQ>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2)))
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
     attention_flash_kernel(const uint16_t *__restrict__ q, const uint16_t *__restrict__ k_pool, const uint16_t *__restrict__ v_pool,
                            uint16_t *__restrict__ out, uint32_t ld_out, uint32_t max_cols, AttentionShape sh, RaggedRows rr) {
     constexpr int VT = 2 * V, KP = D * 32 + 8, VP = V * 32 + 8, PK = D / 2, PV = V / 2, BC = 64 * NQ;
