@@ -328,8 +328,10 @@ void launch_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
     if (m <= 64) {
         constexpr bool GLU = MODE == LinearEpilogue::kGlu;
         const int mt = (int)((m + 15) / 16);
-        // two tiles per block once one tile each would fill the device twice over
-        const bool two = GLU || (uint64_t)w.n_tiles * w.batches >= 2 * (uint64_t)num_cus;
+        // two tiles per block once one tile each would fill the device twice over; beyond 16 rows, where the registers allow
+        // one block per compute unit, as soon as one tile each does not fit it at once
+        const uint64_t tiles = (uint64_t)w.n_tiles * w.batches;
+        const bool two = GLU || tiles >= 2 * (uint64_t)num_cus || (mt > 1 && tiles > (uint64_t)num_cus);
         // wide weights, up to 32 rows: four, so that the activations cross the L2 half as often
         const bool four = mt <= 2 && g_linear_form != 3 && w.batches == 1 && w.n_tiles >= 3 * (uint64_t)num_cus;
         const dim3 grid(four ? (w.n_tiles + 3) / 4 : two ? (w.n_tiles + 1) / 2 : w.n_tiles, w.batches);

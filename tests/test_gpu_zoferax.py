@@ -269,23 +269,20 @@ def standing_out(heads, kv_heads, dim, vdim, n, at):
     return cfg, w, toks
 
 
-STANDING_OUT = [(4, 2, 16, 16, 400, (0,)), (4, 1, 16, 8, 420, (63, 300)), (8, 2, 64, 32, 330, (64,)), (2, 1, 128, 128, 700, (31, 511)), (4, 4, 200, 96, 150, (32, 33))]
+STANDING_OUT = [(4, 2, 16, 16, 400, (0,)), (4, 1, 16, 8, 420, (63, 300)), (6, 2, 64, 40, 330, (64,)), (2, 1, 128, 128, 700, (31, 511)), (4, 4, 200, 96, 150, (32, 33))]
 
 
-@pytest.mark.parametrize("form", [0, 1, 2, 3])
 @pytest.mark.parametrize("case", STANDING_OUT, ids=lambda c: "%d heads of %d %d" % (c[0], c[2], c[3]))
-@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("dtype,form", [("float32", 0), ("bfloat16", 0), ("bfloat16", 1), ("bfloat16", 2), ("bfloat16", 3)])
 def test_a_key_that_stands_out(dtype, case, form, tune):
     """The first token, tokens at page and tile borders, keys hundreds of tokens away: seen from their own position on and
     not before, in prompts, portions and decoding, in the layer itself and in one that uses its cache."""
-    if form and dtype == "float32":
-        pytest.skip("f32 has one form")
     tune(33, form)
     cfg, w, toks = standing_out(*case)
     want = oracle.forward(cfg, w, toks)
-    other = list(toks)
-    other[case[5][-1]] = 5
-    assert lc.error(oracle.forward(cfg, w, other)[-1:], want[-1:]) > 0.1 or len(case[5]) > 1
+    hidden = oracle.forward(cfg, w, [5 if t == 39 else t for t in toks])
+    for p in (case[5][0], len(toks) - 1):                     # far beyond the tolerance: at its own place and at the far end
+        assert lc.error(hidden[p:p + 1], want[p:p + 1]) > 0.3
     dec = lc.make_decoder(ops(), cfg, w, dtype, max_tokens=768)
     assert lc.error(whole(dec, toks), want) < tolerance(dtype)
     for cut in (1, case[5][-1] + 1, len(toks) - 40):
