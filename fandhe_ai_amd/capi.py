@@ -86,25 +86,33 @@ class DecoderConfig(C.Structure):
                 ("rope_theta", C.c_double)]
 
 
-MIXER_DELTA, MIXER_LATENT_ATTENTION, MIXER_ATTENTION = 0, 1, 2
-NORM_INPUT, NORM_OUTPUT = 0, 1
-ATTENTION_BIAS, ATTENTION_QK_NORM = 1, 2
+MIXER_DELTA, MIXER_LATENT_ATTENTION, MIXER_ATTENTION, MIXER_LIGHTNING = 0, 1, 2, 3
+NORM_INPUT, NORM_OUTPUT, NORM_BOTH = 0, 1, 2
+ATTENTION_BIAS, ATTENTION_QK_NORM, ATTENTION_HEAD_NORM, ATTENTION_HEAD_UNIT, ATTENTION_KEY_VALUES = 1, 2, 4, 8, 16
+ATTENTION_GATE, ATTENTION_SINK = 32, 64
+GLU_CLAMPED, GLU_SILU = 0, 1
 
 
 class LayerConfig(C.Structure):
     """fa_layer_config: one layer of a layered decoder."""
-    _fields_ = [("mixer", C.c_int32), ("heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32),
-                ("kv_heads", C.c_uint32), ("conv", C.c_uint32), ("q_rank", C.c_uint32), ("kv_rank", C.c_uint32),
-                ("rot_dim", C.c_uint32), ("window", C.c_uint32), ("kv_from", C.c_int32), ("scale", C.c_float),
-                ("rot_base", C.c_double), ("d_ffn", C.c_uint32), ("ffn_limit", C.c_float), ("ffn_alpha", C.c_float),
-                ("attention", C.c_uint32), ("experts", C.c_uint32), ("top", C.c_uint32)]
+
+
+LayerConfig._fields_ = [("mixer", C.c_int32), ("heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32),
+                        ("kv_heads", C.c_uint32), ("conv", C.c_uint32), ("q_rank", C.c_uint32), ("kv_rank", C.c_uint32),
+                        ("rot_dim", C.c_uint32), ("window", C.c_uint32), ("kv_from", C.c_int32), ("scale", C.c_float),
+                        ("rot_base", C.c_double), ("d_ffn", C.c_uint32), ("ffn_limit", C.c_float), ("ffn_alpha", C.c_float),
+                        ("attention", C.c_uint32), ("experts", C.c_uint32), ("top", C.c_uint32), ("glu", C.c_int32),
+                        ("rot_interleaved", C.c_uint32), ("rot_factor", C.c_double), ("rot_low", C.c_double), ("rot_high", C.c_double),
+                        ("rot_original", C.c_double), ("ungated", C.c_uint32), ("decay_rank", C.c_uint32), ("gate_rank", C.c_uint32),
+                        ("decay", f32p), ("right", C.POINTER(LayerConfig)), ("left_scale", C.c_float), ("right_scale", C.c_float)]
 
 
 class LayeredConfig(C.Structure):
     _fields_ = [("n_layers", C.c_uint32), ("d_model", C.c_uint32), ("vocab", C.c_uint32), ("block_size", C.c_uint32),
                 ("max_blocks_per_seq", C.c_uint32), ("num_blocks", C.c_uint32), ("max_batch", C.c_uint32),
                 ("state_slots", C.c_uint32), ("norm_eps", C.c_float), ("logit_softcap", C.c_float), ("dtype", C.c_int),
-                ("layers", C.POINTER(LayerConfig)), ("norm", C.c_int32), ("embed_scale", C.c_float), ("position_base", C.c_double)]
+                ("layers", C.POINTER(LayerConfig)), ("norm", C.c_int32), ("embed_scale", C.c_float), ("position_base", C.c_double),
+                ("logit_scale", C.c_float)]
 
 
 # name -> (restype, argtypes); every symbol the header declares

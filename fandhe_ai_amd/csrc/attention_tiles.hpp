@@ -21,6 +21,11 @@ __device__ __forceinline__ void store_from_f32(T *p, float v) {
     else *p = f32_to_bf16(v);
 }
 
+// The i-th pair of a rotation of 2 half entries: neighbours, or half the entries apart
+__device__ __forceinline__ uint2 rotation_pair(uint32_t i, uint32_t half, uint32_t interleaved) {
+    return interleaved ? make_uint2(2 * i, 2 * i + 1) : make_uint2(i, i + half);
+}
+
 constexpr float kLog2e = 1.4426950408889634f;
 constexpr int kKeys = 32;                            // keys per step of the kernels below
 

@@ -1,5 +1,5 @@
 // Grouped-query attention over paged keys and values for ragged passes: consecutive query heads share a key / value head, keys
-// and values have sizes of their own, positions enter through the causal mask only.
+// and values have sizes of their own; causal, in a window or over everything.
 // The query rows of a (sequence, key head) are its (token, head in group) pairs in order; they are the columns of
 // S^T = K Q^T, in tiles of 16.
 #include <algorithm>
@@ -67,6 +67,104 @@ __global__ void __launch_bounds__(NT)
     place(row + nq + nk, nv, sh.vdim, sh.v_p, 1.0f, nullptr, v_pool + slot * sh.kv_heads * sh.v_p);
 }
 
+// Norms per head and rotation.  One block per row; groups of 2^group_log2 lanes take one head at a time.  VEC: sizes, pitches and
+// the rotated part's halves allow four values at a time.
+struct PrepareHeads {
+    const float *q_norm, *k_norm, *cos_sin;
+    int norms, key_values;
+};
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(256)
+    attention_prepare_heads_kernel(const float *__restrict__ y, uint32_t ld, PrepareHeads ph, T *__restrict__ q, T *__restrict__ k_pool, T *__restrict__ v_pool,
+                                   AttentionShape sh, const uint32_t *__restrict__ kv_slot, uint32_t group_log2) {
+    constexpr uint32_t S = VEC ? 4 : 1;
+    typedef float piece __attribute__((ext_vector_type(S)));
+    const uint32_t r = blockIdx.x, H = sh.heads, G = sh.kv_heads, lanes = 1u << group_log2, lane = threadIdx.x & (lanes - 1);
+    const float *row = y + (uint64_t)r * ld, *cs = ph.cos_sin + (uint64_t)r * sh.rot;
+    const uint64_t slot = kv_slot[r];
+    const uint32_t half = sh.rot / 2;
+    auto put = [&](T *dst, const piece &v) {
+        if constexpr (sizeof(T) == 4) *(piece *)dst = v;
+        else if constexpr (VEC) *(v2u *)dst = v2u{f32x2_to_bf16x2(v[0], v[1]), f32x2_to_bf16x2(v[2], v[3])};
+        else *dst = f32_to_bf16(v[0]);
+    };
+    const uint32_t units = H + (slot < sh.pool_rows ? (ph.key_values ? G : 2 * G) : 0);
+    for (uint32_t u = threadIdx.x >> group_log2; u < units; u += 256u >> group_log2) {
+        if (u >= H + G) {                            // a value head
+            const uint32_t g = u - H - G;
+            const float *src = row + (H + G) * sh.dim + g * sh.vdim;
+            for (uint32_t i = lane * S; i < sh.vdim; i += lanes * S) put(v_pool + (slot * G + g) * sh.v_p + i, *(const piece *)(src + i));
+            continue;
+        }
+        const float *src = row + u * sh.dim, *w = u < H ? ph.q_norm : ph.k_norm;
+        T *dst = u < H ? q + ((uint64_t)r * H + u) * sh.dim_p : k_pool + (slot * G + (u - H)) * sh.dim_p;
+        float f = 1.0f;
+        if (ph.norms) {
+            float sq = 0.0f;
+            for (uint32_t i = lane * S; i < sh.dim; i += lanes * S) {
+                const piece v = *(const piece *)(src + i);
+#pragma unroll
+                for (int e = 0; e < (int)S; ++e) sq = fmaf(v[e], v[e], sq);
+            }
+            for (uint32_t off = lanes / 2; off > 0; off >>= 1) sq += __shfl_xor(sq, (int)off, 64);
+            f = 1.0f / sqrtf(sq / (float)sh.dim + sh.eps);
+        }
+        auto normed = [&](uint32_t i) {
+            piece v = *(const piece *)(src + i) * f;
+            if (w) v *= *(const piece *)(w + i);
+            return v;
+        };
+        for (uint32_t i = lane * S; i < sh.dim; i += lanes * S) {
+            piece v = normed(i);
+            if (i < sh.rot) {
+                if (sh.interleaved) {
+                    if constexpr (VEC) {
+                        const float c0 = cs[i / 2], c1 = cs[i / 2 + 1], s0 = cs[half + i / 2], s1 = cs[half + i / 2 + 1];
+                        v = piece{v[0] * c0 - v[1] * s0, v[1] * c0 + v[0] * s0, v[2] * c1 - v[3] * s1, v[3] * c1 + v[2] * s1};
+                    } else {
+                        const float c = cs[i / 2], s = cs[half + i / 2], o = normed(i ^ 1)[0];
+                        v[0] = i & 1 ? v[0] * c + o * s : v[0] * c - o * s;
+                    }
+                } else {
+                    const bool second = i >= half;
+                    const uint32_t p = second ? i - half : i;
+                    const piece o = normed(second ? p : p + half), c = *(const piece *)(cs + p), s = *(const piece *)(cs + half + p);
+                    v = second ? v * c + o * s : v * c - o * s;
+                }
+            }
+            put(dst + i, v);
+        }
+        if (u >= H && ph.key_values)
+            for (uint32_t i = lane * S; i < sh.vdim; i += lanes * S) put(v_pool + (slot * G + (u - H)) * sh.v_p + i, *(const piece *)(src + i));
+    }
+}
+
+// ------------------------------------------------------------------ output
+// Four values of an output head, d .. d + 3: gate, scale, rounding.
+struct OutputPlace {
+    uint16_t *dst;
+    const uint16_t *gate;
+};
+__device__ __forceinline__ float gate_value(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ void store_columns(const OutputPlace &at, uint32_t d, uint32_t vdim, v4f o) {
+    if ((vdim & 3) == 0) {
+        if (d >= vdim) return;
+        if (at.gate) {
+            const v2u g = *(const v2u *)(at.gate + d);
+            o *= v4f{gate_value(bf16_lo(g[0])), gate_value(bf16_hi(g[0])), gate_value(bf16_lo(g[1])), gate_value(bf16_hi(g[1]))};
+        }
+        *(v2u *)(at.dst + d) = v2u{f32x2_to_bf16x2(o[0], o[1]), f32x2_to_bf16x2(o[2], o[3])};
+        return;
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+        if (d + e < vdim) at.dst[d + e] = f32_to_bf16(at.gate ? o[e] * gate_value(bf16_to_f32(at.gate[d + e])) : o[e]);
+}
+// (row, head) of the output
+__device__ __forceinline__ OutputPlace output_place(uint16_t *out, uint32_t ld_out, const AttentionOutput &ao, const AttentionShape &sh, uint64_t row, uint32_t head) {
+    return OutputPlace{out + row * ld_out + head * sh.vdim, ao.gate ? (const uint16_t *)ao.gate + row * ao.ld_gate + head * sh.vdim : nullptr};
+}
+
 // ------------------------------------------------------------------ plain form: any sizes, f32 or bf16
 // One block per (row, head).  Keys are taken 256 at a time, one per thread for the scores, with a running maximum and sum;
 // the threads then own value dims.
@@ -74,7 +172,7 @@ constexpr uint32_t kPlainMaxV = 4096;
 template <typename T>
 __global__ void __launch_bounds__(256)
     attention_plain_kernel(const T *__restrict__ q, const T *__restrict__ k_pool, const T *__restrict__ v_pool, T *__restrict__ out, uint32_t ld_out,
-                           AttentionShape sh, RaggedRows rr) {
+                           AttentionOutput ao, AttentionShape sh, RaggedRows rr) {
     extern __shared__ float lq[];                    // the query row
     __shared__ float w[256], smem[4];
     __shared__ uint32_t ids[256];
@@ -88,7 +186,8 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
     for (uint32_t i = 0; i < kPlainMaxV / 256; ++i) acc[i] = 0.0f;
     bool lost = false;                               // a position without a page: NaN, never a silent zero
-    for (int32_t j0 = 0; j0 <= p; j0 += 256) {
+    const int32_t first = p - (int32_t)sh.window + 1 > 0 ? p - (int32_t)sh.window + 1 : 0;
+    for (int32_t j0 = first; j0 <= p; j0 += 256) {
         __syncthreads();
         const int32_t j = j0 + (int32_t)threadIdx.x;
         float s = -INFINITY;
@@ -123,11 +222,27 @@ __global__ void __launch_bounds__(256)
         }
     }
     if (__syncthreads_or(lost)) l = __uint_as_float(0x7fc00000u);
+    float f = 1.0f;                                  // of what was summed
+    if (ao.sink) {
+        const float sink = ao.sink[h], mc = fmaxf(m, sink);
+        f = expf(m - mc);
+        l = l * f + expf(sink - mc);
+    }
+    f = f / l * ao.scale;
+    const T *gate = ao.gate ? (const T *)ao.gate + (uint64_t)r * ao.ld_gate + h * sh.vdim : nullptr;
 #pragma unroll
     for (uint32_t i = 0; i < kPlainMaxV / 256; ++i) {
         const uint32_t d = threadIdx.x + i * 256;
-        if (d < sh.vdim) store_from_f32(out + (uint64_t)r * ld_out + h * sh.vdim + d, acc[i] / l);
+        if (d < sh.vdim) store_from_f32(out + (uint64_t)r * ld_out + h * sh.vdim + d, gate ? acc[i] * f * gate_value(load_as_f32(gate + d)) : acc[i] * f);
     }
+}
+
+// Factor of what a column summed with maximum m (of scores in powers of two) and sum l of the weights: the sink takes its share
+// of the softmax here.
+__device__ __forceinline__ float final_factor(const AttentionOutput &ao, uint32_t head, float m, float l) {
+    if (!ao.sink) return ao.scale / l;
+    const float sink = ao.sink[head] * kLog2e, mx = fmaxf(m, sink), f = exp2f(m - mx);
+    return ao.scale * f / (l * f + exp2f(sink - mx));
 }
 
 // ------------------------------------------------------------------ few query rows
@@ -138,20 +253,11 @@ struct StreamParams {
     const uint16_t *q, *k_pool, *v_pool;
     uint16_t *out;
     uint32_t ld_out;
+    AttentionOutput ao;
     float *part_o, *part_ml;                         // [sequence tile][key head][split][16 NQ][v_p], .. [2]: maximum, sum
     uint32_t splits, tiles;                          // tiles of 16 NQ columns per sequence
     uint32_t max_cols;                               // sequences with more columns (and more than one token) are another launch's
 };
-
-__device__ __forceinline__ void store_columns(uint16_t *dst, uint32_t d, uint32_t vdim, v4f o) {
-    if ((vdim & 3) == 0 && d < vdim) {
-        *(v2u *)(dst + d) = v2u{f32x2_to_bf16x2(o[0], o[1]), f32x2_to_bf16x2(o[2], o[3])};
-        return;
-    }
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-        if (d + e < vdim) dst[d + e] = f32_to_bf16(o[e]);
-}
 
 // D, V: dim_p and v_p in units of 32.
 template <int D, int V, int NQ, int NW>
@@ -166,11 +272,12 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
     const uint32_t *table = rr.tables + (uint64_t)b * rr.max_blocks;
     const int32_t p0 = rr.pos[row0];
     const uint32_t last_col = c0 + 16 * NQ - 1 < n_cols ? c0 + 16 * NQ - 1 : n_cols - 1;
-    int32_t k_lo = 0, k_hi = p0 + (int32_t)(last_col / S) + 1;
+    const int32_t W = (int32_t)sh.window, p_lo = p0 + (int32_t)(c0 / S);
+    int32_t k_lo = p_lo - W + 1 > 0 ? p_lo - W + 1 : 0, k_hi = p0 + (int32_t)(last_col / S) + 1;      // keys seen by some column
     const uint64_t part = (((uint64_t)blockIdx.x * G + kh) * p.splits + blockIdx.z) * 16 * NQ;
     if (p.splits > 1) {
-        const int32_t unit = kKeys * NW / 2, per = ((k_hi + (int32_t)p.splits - 1) / (int32_t)p.splits + unit - 1) / unit * unit;
-        k_lo = (int32_t)blockIdx.z * per;
+        const int32_t unit = kKeys * NW / 2, per = ((k_hi - k_lo + (int32_t)p.splits - 1) / (int32_t)p.splits + unit - 1) / unit * unit;
+        k_lo += (int32_t)blockIdx.z * per;
         k_hi = k_lo + per < k_hi ? k_lo + per : k_hi;
         if (k_lo >= k_hi) {                          // a split without keys (never the only one)
             if (tid < 16 * NQ) {
@@ -263,7 +370,7 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int32_t j = k0 + kt * 16 + 4 * g + e;
-                    sc[qi][kt * 4 + e] = j <= pos[qi] && j < k_hi ? acc[qi][e] * factor : -INFINITY;
+                    sc[qi][kt * 4 + e] = j <= pos[qi] && pos[qi] - j < W && j < k_hi ? acc[qi][e] * factor : -INFINITY;
                 }
         }
         __builtin_amdgcn_sched_barrier(0);
@@ -347,10 +454,11 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
                 for (int t = 0; t < VT; ++t) *(v4f *)(p.part_o + at * (V * 32) + t * 16 + 4 * g) = o[qi][t];
             }
         } else if (col < n_cols) {
-            uint16_t *dst = p.out + (uint64_t)(row0 + col / S) * p.ld_out + (kh * S + col % S) * sh.vdim;
-            const float inv = 1.0f / l[qi];
+            const uint32_t head = kh * S + col % S;
+            const OutputPlace at = output_place(p.out, p.ld_out, p.ao, sh, row0 + col / S, head);
+            const float f = final_factor(p.ao, head, m[qi], l[qi]);
 #pragma unroll
-            for (int t = 0; t < VT; ++t) store_columns(dst, t * 16 + 4 * g, sh.vdim, o[qi][t] * inv);
+            for (int t = 0; t < VT; ++t) store_columns(at, t * 16 + 4 * g, sh.vdim, o[qi][t] * f);
         }
     }
 }
@@ -368,8 +476,9 @@ __global__ void __launch_bounds__(64) attention_merge_kernel(StreamParams p, Att
         ms = v[0];
         ls = v[1];
     }
-    const float m = wave_max_dpp(ms), f = ls != 0.0f ? exp2f(ms - m) : 0.0f, w = f / wave_sum_dpp(ls * f);
-    uint16_t *dst = p.out + (uint64_t)(row0 + col / S) * p.ld_out + (kh * S + col % S) * sh.vdim;
+    const uint32_t head = kh * S + col % S;
+    const float m = wave_max_dpp(ms), f = ls != 0.0f ? exp2f(ms - m) : 0.0f, w = f * final_factor(p.ao, head, m, wave_sum_dpp(ls * f));
+    const OutputPlace out = output_place(p.out, p.ld_out, p.ao, sh, row0 + col / S, head);
     for (uint32_t d = lane * 4; d < sh.v_p; d += 256) {
         const float *src = p.part_o + at * sh.v_p + d;
         v4f a = v4f{0.f, 0.f, 0.f, 0.f};
@@ -383,7 +492,7 @@ __global__ void __launch_bounds__(64) attention_merge_kernel(StreamParams p, Att
                 if (ws != 0.0f) a += t[i] * ws;
             }
         }
-        store_columns(dst, d, sh.vdim, a);
+        store_columns(out, d, sh.vdim, a);
     }
 }
 
@@ -393,7 +502,7 @@ __global__ void __launch_bounds__(64) attention_merge_kernel(StreamParams p, Att
 template <int D, int V, int NQ>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
     attention_flash_kernel(const uint16_t *__restrict__ q, const uint16_t *__restrict__ k_pool, const uint16_t *__restrict__ v_pool,
-                           uint16_t *__restrict__ out, uint32_t ld_out, uint32_t max_cols, AttentionShape sh, RaggedRows rr) {
+                           uint16_t *__restrict__ out, uint32_t ld_out, AttentionOutput ao, uint32_t max_cols, AttentionShape sh, RaggedRows rr) {
     constexpr int VT = 2 * V, KP = D * 32 + 8, VP = V * 32 + 8, PK = D / 2, PV = V / 2, BC = 64 * NQ;
     extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
     uint16_t *ks = lds, *vs = lds + 2 * kKeys * KP;  // [2][32][KP], [2][32][VP]
@@ -413,7 +522,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
     const uint32_t *table = rr.tables + (uint64_t)b * rr.max_blocks;
     const int32_t p0 = rr.pos[row0];
     auto pos_of = [&](uint32_t col) { return p0 + (int32_t)((col < n_cols ? col : n_cols - 1) / S); };
-    const int32_t k_hi = pos_of(c0 + BC - 1) + 1;
+    const int32_t W = (int32_t)sh.window, k_hi = pos_of(c0 + BC - 1) + 1, p_lo = pos_of(c0), k_lo = p_lo - W + 1 > 0 ? p_lo - W + 1 : 0;
     v8bf qf[NQ][D];
     int32_t pos[NQ];
 #pragma unroll
@@ -464,20 +573,20 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
 #pragma unroll
         for (int t = 0; t < VT; ++t) o[qi][t] = v4f{0.f, 0.f, 0.f, 0.f};
     }
-    uint32_t id = page_of(key);
-    fetch(key, id);
-    id = page_of(kKeys + key);
+    uint32_t id = page_of(k_lo + key);
+    fetch(k_lo + key, id);
+    id = page_of(k_lo + kKeys + key);
     put(0);
     __syncthreads();
     int buf = 0;
-    for (int32_t k0 = 0; k0 < k_hi; k0 += kKeys, buf ^= 1) {
+    for (int32_t k0 = k_lo; k0 < k_hi; k0 += kKeys, buf ^= 1) {
         const bool more = k0 + kKeys < k_hi;
         if (more) {
             fetch(k0 + kKeys + key, id);
             id = page_of(k0 + 2 * kKeys + key);
         }
-        if (k0 <= w_hi_pos) {                        // some column of this wavefront sees some key of the step
-            const bool inside = k0 + kKeys - 1 <= w_lo_pos;          // every column sees every key
+        if (k0 <= w_hi_pos && k0 + kKeys > w_lo_pos - W + 1) {       // some column of this wavefront sees some key of the step
+            const bool inside = k0 + kKeys - 1 <= w_lo_pos && k0 > w_hi_pos - W;       // every column sees every key
             const uint16_t *kb = ks + buf * kKeys * KP, *vb = vs + buf * kKeys * VP;
             float sc[NQ][8];
 #pragma unroll
@@ -496,7 +605,10 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         float v = acc[qi][e] * factor;
-                        if (!inside && k0 + kt * 16 + 4 * g + e > pos[qi]) v = -INFINITY;
+                        if (!inside) {
+                            const int32_t j = k0 + kt * 16 + 4 * g + e;
+                            if (j > pos[qi] || pos[qi] - j >= W) v = -INFINITY;
+                        }
                         sc[qi][kt * 4 + e] = v;
                     }
             }
@@ -529,10 +641,11 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
         sum += __shfl_xor(sum, 32, 64);
         const uint32_t col = c0 + (wave * NQ + qi) * 16 + c;
         if (col >= n_cols) continue;
-        const float f = 1.0f / sum;
-        uint16_t *dst = out + (uint64_t)(row0 + col / S) * ld_out + (kh * S + col % S) * sh.vdim;
+        const uint32_t head = kh * S + col % S;
+        const float f = final_factor(ao, head, m[qi], sum);
+        const OutputPlace at = output_place(out, ld_out, ao, sh, row0 + col / S, head);
 #pragma unroll
-        for (int t = 0; t < VT; ++t) store_columns(dst, t * 16 + 4 * g, sh.vdim, o[qi][t] * f);
+        for (int t = 0; t < VT; ++t) store_columns(at, t * 16 + 4 * g, sh.vdim, o[qi][t] * f);
     }
 }
 
@@ -560,7 +673,8 @@ AttentionPlan attention_plan(const AttentionShape &sh, int is_f32, uint32_t batc
     p.tiles = (uint32_t)((most + 16 * p.nq - 1) / (16 * p.nq));
     const uint64_t blocks = (uint64_t)batch * ((uint64_t)(S * (uint64_t)std::max(1u, min_new) + 16 * p.nq - 1) / (16 * p.nq)) * sh.kv_heads;
     const uint64_t want = ((uint64_t)(g_attention_blocks ? g_attention_blocks : 1) * num_cus + blocks / 2) / std::max<uint64_t>(blocks, 1);
-    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (max_ctx + 511) / 512, kMaxSplits}));
+    const uint64_t span = std::min<uint64_t>(max_ctx, (uint64_t)sh.window + most / S);
+    p.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({want, (span + 511) / 512, kMaxSplits}));
     return p;
 }
 
@@ -600,7 +714,7 @@ void launch_matrix(const AttentionPlan &plan, const StreamParams &p, const Atten
             }
         }
         const dim3 grid((uint32_t)((uint64_t)rr.rows * sh.share() / (64 * NQ)) + rr.batch, sh.kv_heads);
-        attention_flash_kernel<D, V, NQ><<<grid, 256, lds, s>>>(p.q, p.k_pool, p.v_pool, p.out, p.ld_out, plan.max_cols, sh, rr);
+        attention_flash_kernel<D, V, NQ><<<grid, 256, lds, s>>>(p.q, p.k_pool, p.v_pool, p.out, p.ld_out, p.ao, plan.max_cols, sh, rr);
     }
 }
 template <int D>
@@ -637,26 +751,45 @@ void attention_prepare(const float *y, uint32_t ld, const float *q_norm, const f
 #undef FA_PREP
 }
 
+void attention_prepare_heads(const float *y, uint32_t ld, bool norms, const float *q_norm, const float *k_norm, const float *cos_sin, bool key_values, void *q,
+                             void *k_pool, void *v_pool, int is_f32, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s) {
+    if (rr.rows == 0) return;
+    const bool vec = sh.dim % 4 == 0 && sh.vdim % 4 == 0 && ld % 4 == 0 && sh.rot % (sh.interleaved ? 4 : 8) == 0;
+    uint32_t group_log2 = 0;
+    while (group_log2 < 6 && ((vec ? 4u : 1u) << group_log2) < sh.dim) ++group_log2;
+    const PrepareHeads ph{q_norm, k_norm, cos_sin, norms, key_values};
+#define FA_PREP(T_, VEC_) \
+    attention_prepare_heads_kernel<T_, VEC_><<<rr.rows, 256, 0, s>>>(y, ld, ph, (T_ *)q, (T_ *)k_pool, (T_ *)v_pool, sh, rr.kv_slot, group_log2)
+    if (is_f32) {
+        if (vec) FA_PREP(float, true);
+        else FA_PREP(float, false);
+    } else {
+        if (vec) FA_PREP(uint16_t, true);
+        else FA_PREP(uint16_t, false);
+    }
+#undef FA_PREP
+}
+
 uint64_t attention_workspace_bytes(const AttentionShape &sh, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
                                    int num_cus) {
     const AttentionPlan p = attention_plan(sh, is_f32, batch, min_new, max_new, max_ctx, num_cus);
     return p.splits > 1 ? (uint64_t)batch * p.tiles * sh.kv_heads * p.splits * 16 * p.nq * (sh.v_p + 2) * 4 : 0;
 }
 
-void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, int is_f32, const AttentionShape &sh,
-               const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s) {
+void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, const AttentionOutput &ao, int is_f32,
+               const AttentionShape &sh, const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s) {
     if (rr.rows == 0) return;
     const AttentionPlan plan = attention_plan(sh, is_f32, rr.batch, min_new, max_new, rr.max_blocks * rr.block_size, num_cus);
     if (plan.plain) {
         const dim3 grid(rr.rows, sh.heads);
         if (is_f32)
-            attention_plain_kernel<float><<<grid, 256, sh.dim * 4, s>>>((const float *)q, (const float *)k_pool, (const float *)v_pool, (float *)out, ld_out, sh, rr);
+            attention_plain_kernel<float><<<grid, 256, sh.dim * 4, s>>>((const float *)q, (const float *)k_pool, (const float *)v_pool, (float *)out, ld_out, ao, sh, rr);
         else
             attention_plain_kernel<uint16_t><<<grid, 256, sh.dim * 4, s>>>((const uint16_t *)q, (const uint16_t *)k_pool, (const uint16_t *)v_pool,
-                                                                           (uint16_t *)out, ld_out, sh, rr);
+                                                                           (uint16_t *)out, ld_out, ao, sh, rr);
         return;
     }
-    StreamParams p{(const uint16_t *)q, (const uint16_t *)k_pool, (const uint16_t *)v_pool, (uint16_t *)out, ld_out, (float *)workspace, nullptr, plan.splits,
+    StreamParams p{(const uint16_t *)q, (const uint16_t *)k_pool, (const uint16_t *)v_pool, (uint16_t *)out, ld_out, ao, (float *)workspace, nullptr, plan.splits,
                    plan.tiles, plan.max_cols};
     if (p.splits > 1) p.part_ml = p.part_o + (uint64_t)rr.batch * plan.tiles * sh.kv_heads * plan.splits * 16 * plan.nq * sh.v_p;
     if (sh.dim_p == 64) launch_matrix_v<2>(plan, p, sh, rr, s);

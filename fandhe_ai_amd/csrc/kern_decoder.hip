@@ -158,10 +158,10 @@ __global__ void ragged_advance_kernel(const uint32_t *__restrict__ row_start, ui
 }
 
 __global__ void __launch_bounds__(64)
-    rotation_table_kernel(const int32_t *__restrict__ pos, float *__restrict__ cos_sin, uint32_t dims, double base) {
+    rotation_table_kernel(const int32_t *__restrict__ pos, float *__restrict__ cos_sin, uint32_t dims, const double *__restrict__ freq) {
     const uint32_t r = blockIdx.x, half = dims / 2;
     for (uint32_t i = threadIdx.x; i < half; i += 64) {
-        const double ang = (double)pos[r] * pow(base, -2.0 * (double)i / (double)dims);
+        const double ang = (double)pos[r] * freq[i];
         cos_sin[(uint64_t)r * dims + i] = (float)cos(ang);
         cos_sin[(uint64_t)r * dims + half + i] = (float)sin(ang);
     }
@@ -181,9 +181,9 @@ void ragged_advance(const uint32_t *row_start, uint32_t *seq_lens, uint32_t batc
     ragged_advance_kernel<<<(batch + 63) / 64, 64, 0, s>>>(row_start, seq_lens, batch);
 }
 
-void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t dims, double base, hipStream_t s) {
+void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t dims, const double *freq, hipStream_t s) {
     if (rows == 0 || dims == 0) return;
-    rotation_table_kernel<<<rows, 64, 0, s>>>(pos, cos_sin, dims, base);
+    rotation_table_kernel<<<rows, 64, 0, s>>>(pos, cos_sin, dims, freq);
 }
 
 void prefill_prepare(const uint32_t *tables, const uint32_t *seq_lens, uint32_t *slots, float *cos_sin, uint32_t batch,

@@ -62,12 +62,13 @@ __device__ __forceinline__ void choose_experts(const float *logits, uint32_t exp
 
 // ------------------------------------------------------------------ residual update
 // One block per row, VPT pieces of it per thread: four values each (VEC, hidden a multiple of four), or one.
-template <typename T, int VPT, int NT, bool ROUTE, bool VEC>
+// LAYER: layer norm of the output, and of the new x for the next sublayer.
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC, bool LAYER>
 __global__ void __launch_bounds__(NT)
     residual_norm_kernel(ResidualNorm rn, float *__restrict__ x, T *__restrict__ hn, uint32_t hidden, uint64_t ld, RouteIo io) {
     constexpr int NW = NT / 64, S = VEC ? 4 : 1;
     typedef float piece __attribute__((ext_vector_type(S)));
-    __shared__ float smem[NW], logits[ROUTE ? kMaxExperts : 1];
+    __shared__ float smem[LAYER ? 4 : 1][NW], logits[ROUTE ? kMaxExperts : 1];
     extern __shared__ __attribute__((aligned(16))) uint8_t hs_raw[];     // ROUTE: the row of hn
     const uint64_t r = blockIdx.x;
     const int tid = threadIdx.x;
@@ -76,7 +77,6 @@ __global__ void __launch_bounds__(NT)
     const float *y = rn.y + r * rn.parts * hidden;
     float *xr = x + r * hidden;
     piece v[VPT], xv[VPT];
-    float sq = 0.0f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
         const uint32_t c = (tid + i * NT) * S;
@@ -102,11 +102,52 @@ __global__ void __launch_bounds__(NT)
                 for (int e = 0; e < S; ++e) v[i][e] = fmaf(g1, t1[i][e], fmaf(g0, t0[i][e], v[i][e]));
         }
     }
+    // of the row behind v: its mean is taken off, the root of the mean square returned inverted
+    auto center = [&](piece (&t)[VPT], float *s_mean, float *s_var) {
+        if constexpr (LAYER) {
+            float sum = 0.0f;
 #pragma unroll
-    for (int i = 0; i < VPT; ++i)
+            for (int i = 0; i < VPT; ++i)
 #pragma unroll
-        for (int e = 0; e < S; ++e) sq = fmaf(v[i][e], v[i][e], sq);
-    const float rstd = 1.0f / sqrtf(block_sum<float, NW, true, true>(sq, smem) / (float)hidden + rn.eps);
+                for (int e = 0; e < S; ++e) sum += t[i][e];
+            const float mean = block_sum<float, NW, true, true>(sum, s_mean) / (float)hidden;
+#pragma unroll
+            for (int i = 0; i < VPT; ++i)
+                if ((uint32_t)(tid + i * NT) * S < hidden) t[i] -= mean;
+        }
+        float q = 0.0f;
+#pragma unroll
+        for (int i = 0; i < VPT; ++i)
+#pragma unroll
+            for (int e = 0; e < S; ++e) q = fmaf(t[i][e], t[i][e], q);
+        return 1.0f / sqrtf(block_sum<float, NW, true, true>(q, s_var) / (float)hidden + rn.eps);
+    };
+    const float rstd = LAYER ? center(v, smem[LAYER], smem[0]) : center(v, nullptr, smem[0]);
+    if constexpr (LAYER) {
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const uint32_t c = (tid + i * NT) * S;
+            if (c >= hidden) continue;
+            const piece w = *(const piece *)(rn.w + c);
+#pragma unroll
+            for (int e = 0; e < S; ++e) xv[i][e] += v[i][e] * rstd * w[e];
+            *(piece *)(xr + c) = xv[i];
+        }
+        if (!rn.next) return;
+        const float r2 = center(xv, smem[LAYER ? 2 : 0], smem[LAYER ? 3 : 0]);
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const uint32_t c = (tid + i * NT) * S;
+            if (c >= ld) continue;
+            piece o = piece(0.0f);
+            if (c < hidden) o = xv[i] * r2 * *(const piece *)(rn.next + c);
+            T *dst = hn + r * ld + c;
+            if constexpr (sizeof(T) == 4) *(piece *)dst = o;
+            else if constexpr (VEC) *(v2u *)dst = v2u{f32x2_to_bf16x2(o[0], o[1]), f32x2_to_bf16x2(o[2], o[3])};
+            else *dst = f32_to_bf16(o[0]);
+        }
+        return;
+    }
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
         const uint32_t c = (tid + i * NT) * S;
@@ -250,18 +291,24 @@ __global__ void __launch_bounds__(256)
     }
 }
 
-template <typename T, int VPT, int NT, bool ROUTE, bool VEC>
-void launch_residual_sized(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC, bool LAYER>
+void launch_residual_kind(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
     const size_t lds = ROUTE ? ld * sizeof(T) + (sizeof(T) == 2 ? (io.experts + 15) / 16 * 16 * 17 * 4 : 0) : 0;
     if (ROUTE && lds > 49152) {
         static bool configured = false;
         if (!configured) {
-            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, VPT, NT, ROUTE, VEC>), hipFuncAttributeMaxDynamicSharedMemorySize,
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, VPT, NT, ROUTE, VEC, LAYER>), hipFuncAttributeMaxDynamicSharedMemorySize,
                                       98304);
             configured = true;
         }
     }
-    residual_norm_kernel<T, VPT, NT, ROUTE, VEC><<<(unsigned)rows, NT, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);
+    residual_norm_kernel<T, VPT, NT, ROUTE, VEC, LAYER><<<(unsigned)rows, NT, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);
+}
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC>
+void launch_residual_sized(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
+    if constexpr (!ROUTE)
+        if (rn.layer) return launch_residual_kind<T, VPT, NT, false, VEC, true>(rn, x, hn, rows, hidden, ld, io, s);
+    launch_residual_kind<T, VPT, NT, ROUTE, VEC, false>(rn, x, hn, rows, hidden, ld, io, s);
 }
 
 // rows up to 16384 values

@@ -693,7 +693,7 @@ __global__ void __launch_bounds__(128 * WM) __attribute__((amdgpu_waves_per_eu(W
     ixm::big_out_elem<NTB, WM>(wm, wn, 0, 0, 0, lane, &row_l0, &col_l0);
     const int g = lane / 16;
     if constexpr (BF16) {
-        constexpr int MODE = IsBf16<Epi>::mode, STEP = MODE == LinearEpilogue::kGlu ? 2 : 1;      // gate, up: neighbouring tiles
+        constexpr int MODE = IsBf16<Epi>::mode, STEP = is_glu(MODE) ? 2 : 1;      // gate, up: neighbouring tiles
         static_assert(STEP == 1 || WNT % 2 == 0, "a gate tile and its up tile belong to one wavefront");
 #pragma unroll
         for (int i = 0; i < AI; ++i) {
@@ -1164,7 +1164,7 @@ namespace {
 template <int MODE>
 void launch_big_bf16(const uint16_t *a, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int ntb, hipStream_t s) {
     const EpiBf16<MODE> e{ep};
-    if constexpr (MODE != LinearEpilogue::kGlu) {
+    if constexpr (!is_glu(MODE)) {
         if (ntb == 14) return launch_big_wm<false, 14, 4>((const uint8_t *)a, (const uint8_t *)w.w, m, w.n, w.n_tiles, w.k_tiles / 2, e, s);
     }
     launch_big_wm<false, 16, 4>((const uint8_t *)a, (const uint8_t *)w.w, m, w.n, w.n_tiles, w.k_tiles / 2, e, s);
@@ -1180,6 +1180,7 @@ void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const L
     switch (ep.mode) {
         case LinearEpilogue::kResidual: return launch_big_bf16<LinearEpilogue::kResidual>(a, m, w, ep, ntb, s);
         case LinearEpilogue::kGlu: return launch_big_bf16<LinearEpilogue::kGlu>(a, m, w, ep, ntb, s);
+        case LinearEpilogue::kSiluGlu: return launch_big_bf16<LinearEpilogue::kSiluGlu>(a, m, w, ep, ntb, s);
         case LinearEpilogue::kSoftcap: return launch_big_bf16<LinearEpilogue::kSoftcap>(a, m, w, ep, ntb, s);
         default: return launch_big_bf16<LinearEpilogue::kStore>(a, m, w, ep, ntb, s);
     }

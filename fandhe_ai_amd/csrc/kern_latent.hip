@@ -45,9 +45,10 @@ __global__ void __launch_bounds__(256)
     const uint32_t half = sh.rot / 2;
     const float *cs = cos_sin + (uint64_t)r * sh.rot;
     for (uint32_t i = threadIdx.x; i < half; i += 256) {
-        const float u = kr[i], v = kr[i + half];
-        store_from_f32(dst + sh.rank_p + i, u * cs[i] - v * cs[half + i]);
-        store_from_f32(dst + sh.rank_p + half + i, v * cs[i] + u * cs[half + i]);
+        const uint2 at = rotation_pair(i, half, sh.interleaved);
+        const float u = kr[at.x], v = kr[at.y];
+        store_from_f32(dst + sh.rank_p + at.x, u * cs[i] - v * cs[half + i]);
+        store_from_f32(dst + sh.rank_p + at.y, v * cs[i] + u * cs[half + i]);
     }
 }
 
@@ -62,9 +63,10 @@ __global__ void __launch_bounds__(256)
         const T *src = q + ((uint64_t)r * sh.heads + h) * (sh.dim_p + sh.rot_p) + sh.dim_p;
         T *o = dst + ((uint64_t)r * sh.heads + h) * dst_pitch + dst_off;
         if (d < rh) {
-            const float u = load_as_f32(src + d), v = load_as_f32(src + d + rh);
-            store_from_f32(o + d, u * cs[d] - v * cs[rh + d]);
-            store_from_f32(o + d + rh, v * cs[d] + u * cs[rh + d]);
+            const uint2 at = rotation_pair(d, rh, sh.interleaved);
+            const float u = load_as_f32(src + at.x), v = load_as_f32(src + at.y);
+            store_from_f32(o + at.x, u * cs[d] - v * cs[rh + d]);
+            store_from_f32(o + at.y, v * cs[d] + u * cs[rh + d]);
         } else {                                     // the padding behind the two halves
             store_from_f32(o + rh + d, 0.0f);
             store_from_f32(o + sh.rot_p - 1 - (d - rh), 0.0f);
@@ -471,8 +473,8 @@ __global__ void __launch_bounds__(256)
 template <int D, int RO>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2)))
     latent_flash_kernel(const uint16_t *__restrict__ q, const uint16_t *__restrict__ kv, const uint16_t *__restrict__ kr,
-                        const float *__restrict__ gate, uint32_t ld_gate, uint16_t *__restrict__ out, uint32_t ld_out, LatentShape sh,
-                        RaggedRows rr, LatentExpand ex) {
+                        const float *__restrict__ gate, uint32_t ld_gate, float out_scale, uint16_t *__restrict__ out, uint32_t ld_out,
+                        LatentShape sh, RaggedRows rr, LatentExpand ex) {
     constexpr int KS = D + RO, VT = 2 * D, KP = KS * 32 + 8, VP = D * 32 + 8, NQ = 2;
     constexpr int PKR = (KS * 4 + 7) / 8, PV = D * 4 / 8;        // 16-byte pieces per thread and step, eight threads per key
     __shared__ __attribute__((aligned(16))) uint16_t ks[2][kKeys * KP], vs[2][kKeys * VP];
@@ -606,7 +608,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
         sum += __shfl_xor(sum, 32, 64);
         const uint32_t t = t0 + wave * 32 + qi * 16 + c;
         if (t >= n) continue;
-        const float f = 1.0f / (1.0f + expf(-gate[(uint64_t)(row0 + t) * ld_gate + h])) / sum;
+        const float f = gate ? out_scale / (1.0f + expf(-gate[(uint64_t)(row0 + t) * ld_gate + h])) / sum : out_scale / sum;
         uint16_t *dst = out + (uint64_t)(row0 + t) * ld_out + h * sh.vdim;
         const bool vec = (sh.vdim & 3) == 0;
 #pragma unroll
@@ -695,13 +697,13 @@ void latent_gather(const void *pool, void *c, uint32_t ld_c, void *kr, const Lat
     latent_gather_kernel<<<(ex.rows + 3) / 4, 256, 0, s>>>((const uint16_t *)pool, (uint16_t *)c, ld_c, (uint16_t *)kr, sh, rr, ex);
 }
 
-void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, void *out, uint32_t ld_out,
-                               const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s) {
+void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, float out_scale, void *out,
+                               uint32_t ld_out, const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s) {
     const dim3 grid(rr.rows / 128 + rr.batch + 1, sh.heads);
     const bool wide = sh.v_p > 64, rot2 = sh.rot_p > 32;
 #define FA_FLASH(D_, RO_)                                                                                                                    \
-    latent_flash_kernel<D_, RO_><<<grid, 256, 0, s>>>((const uint16_t *)q, (const uint16_t *)kv, (const uint16_t *)kr, gate, ld_gate, (uint16_t *)out, \
-                                                      ld_out, sh, rr, ex)
+    latent_flash_kernel<D_, RO_><<<grid, 256, 0, s>>>((const uint16_t *)q, (const uint16_t *)kv, (const uint16_t *)kr, gate, ld_gate, out_scale, \
+                                                      (uint16_t *)out, ld_out, sh, rr, ex)
     if (wide) rot2 ? FA_FLASH(4, 2) : FA_FLASH(4, 1);
     else rot2 ? FA_FLASH(2, 2) : FA_FLASH(2, 1);
 #undef FA_FLASH

@@ -26,7 +26,7 @@ template <int MT, int NTW, int NWAVES, int MODE, typename RowOf>
 __device__ __forceinline__ void linear_rows(const uint16_t *__restrict__ a, uint64_t lda, const uint8_t *__restrict__ w_batch, uint32_t m,
                                             uint32_t n, uint32_t n_tiles, uint32_t k_tiles, uint32_t batch, const LinearEpilogue &ep, v4f *red_all,
                                             RowOf row_of) {
-    static_assert(MODE != LinearEpilogue::kGlu || NTW % 2 == 0, "gate and up are neighbouring tiles");
+    static_assert(!is_glu(MODE) || NTW % 2 == 0, "gate and up are neighbouring tiles");
     constexpr int NT = MT * NTW, D = NTW == 4 || MT == 4 ? 4 : 8;
     v4f(*red)[NT][64] = (v4f(*)[NT][64])red_all;
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
@@ -92,14 +92,14 @@ __device__ __forceinline__ void linear_rows(const uint16_t *__restrict__ a, uint
         for (int q = 1; q < NWAVES; ++q) r += red[q][t][lane];
         return r;
     };
-    constexpr int STEP = MODE == LinearEpilogue::kGlu ? 2 : 1;
+    constexpr int STEP = is_glu(MODE) ? 2 : 1;
     for (int t = wave * STEP; t < NT; t += NWAVES * STEP) {
         const int i = t / NTW, j = t % NTW;
         const uint32_t row = i * 16 + lane % 16;
         if (row >= m || nt0 + j >= n_tiles) continue;
         const v4f x = total(t);
         const v4f up = STEP == 2 ? total(t + 1) : x;
-        const uint32_t tile = MODE == LinearEpilogue::kGlu ? (nt0 + j) / 2 : nt0 + j;
+        const uint32_t tile = is_glu(MODE) ? (nt0 + j) / 2 : nt0 + j;
         epilogue_store4<MODE>(ep, row_of(row).y, tile * 16 + 4 * (lane / 16), n, batch, x, up);
     }
 }
@@ -223,7 +223,7 @@ __global__ void __launch_bounds__(256)
         if (more) put(buf ^ 1);
         __syncthreads();
     }
-    constexpr int STEP = MODE == LinearEpilogue::kGlu ? 2 : 1;
+    constexpr int STEP = is_glu(MODE) ? 2 : 1;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         uint32_t row = m0 + (wm * 4 + i) * 16 + lane % 16;
@@ -233,7 +233,7 @@ __global__ void __launch_bounds__(256)
         for (int j = 0; j < 4; j += STEP) {
             const uint32_t nt = nt0 + wn * 4 + j;
             if (nt >= n_tiles) continue;
-            const uint32_t tile = MODE == LinearEpilogue::kGlu ? nt / 2 : nt;
+            const uint32_t tile = is_glu(MODE) ? nt / 2 : nt;
             epilogue_store4<MODE>(ep, row, tile * 16 + 4 * (lane / 16), n, GROUPED ? 0 : batch, acc[i][j], acc[i][j + STEP - 1]);
         }
     }
@@ -282,7 +282,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
                 for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_fmaf(as[q][ty * 4 + i], bs[q][tx + 16 * j], acc[i][j]);
     }
-    constexpr int STEP = MODE == LinearEpilogue::kGlu ? 2 : 1;
+    constexpr int STEP = is_glu(MODE) ? 2 : 1;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         uint32_t row = m0 + ty * 4 + i;
@@ -292,7 +292,7 @@ __global__ void __launch_bounds__(256)
         for (int j = 0; j < 4; j += STEP) {
             const uint32_t nt = n0 / 16 + j;
             if (nt >= n_tiles) continue;
-            const uint32_t col = (MODE == LinearEpilogue::kGlu ? nt / 2 : nt) * 16 + tx;
+            const uint32_t col = (is_glu(MODE) ? nt / 2 : nt) * 16 + tx;
             if (col < n) epilogue_store1<MODE>(ep, row, col, GROUPED ? 0 : batch, acc[i][j], acc[i][j + STEP - 1]);
         }
     }
@@ -301,22 +301,23 @@ __global__ void __launch_bounds__(256)
 template <typename SRC, typename DST>
 __global__ void __launch_bounds__(256)
     pack_linear_kernel(const SRC *__restrict__ src, uint64_t row_stride, uint64_t col_stride, uint32_t rows, uint32_t cols,
-                       DST *__restrict__ dst, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch) {
+                       DST *__restrict__ dst, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch, uint32_t k0) {
     const uint64_t total = (uint64_t)rows * cols;
     for (uint64_t i = (uint64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (uint64_t)gridDim.x * 256) {
         const uint32_t r = (uint32_t)(i / cols), c = (uint32_t)(i % cols);
         const uint32_t nr = n0 + (r / group) * pitch + r % group;
         const SRC v = src[r * row_stride + c * col_stride];
+        const uint32_t kc = k0 + c;
         if constexpr (sizeof(DST) == 4) {
             float f;
             if constexpr (sizeof(SRC) == 4) f = v;
             else f = bf16_to_f32(v);
-            dst[(uint64_t)nr * k_tiles * 32 + c] = f;
+            dst[(uint64_t)nr * k_tiles * 32 + kc] = f;
         } else {
             uint16_t h;
             if constexpr (sizeof(SRC) == 4) h = f32_to_bf16(v);
             else h = v;
-            dst[((uint64_t)(nr / 16) * k_tiles + c / 32) * 512 + (((c % 32) / 8) * 16 + nr % 16) * 8 + c % 8] = h;
+            dst[((uint64_t)(nr / 16) * k_tiles + kc / 32) * 512 + (((kc % 32) / 8) * 16 + nr % 16) * 8 + kc % 8] = h;
         }
     }
 }
@@ -326,7 +327,7 @@ void launch_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
                  int num_cus, hipStream_t s) {
     const uint8_t *wt = (const uint8_t *)w.w;
     if (m <= 64) {
-        constexpr bool GLU = MODE == LinearEpilogue::kGlu;
+        constexpr bool GLU = is_glu(MODE);
         const int mt = (int)((m + 15) / 16);
         // two tiles per block once one tile each would fill the device twice over; beyond 16 rows, where the registers allow
         // one block per compute unit, as soon as one tile each does not fit it at once
@@ -400,6 +401,7 @@ void linear_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
     switch (ep.mode) {
         case LinearEpilogue::kResidual: return launch_bf16<LinearEpilogue::kResidual>(a, lda, a_batch, m, w, ep, num_cus, s);
         case LinearEpilogue::kGlu: return launch_bf16<LinearEpilogue::kGlu>(a, lda, a_batch, m, w, ep, num_cus, s);
+        case LinearEpilogue::kSiluGlu: return launch_bf16<LinearEpilogue::kSiluGlu>(a, lda, a_batch, m, w, ep, num_cus, s);
         case LinearEpilogue::kSoftcap: return launch_bf16<LinearEpilogue::kSoftcap>(a, lda, a_batch, m, w, ep, num_cus, s);
         case LinearEpilogue::kHeadGate: return launch_bf16<LinearEpilogue::kHeadGate>(a, lda, a_batch, m, w, ep, num_cus, s);
         default: return launch_bf16<LinearEpilogue::kStore>(a, lda, a_batch, m, w, ep, num_cus, s);
@@ -411,6 +413,7 @@ void linear_f32(const float *a, uint64_t lda, uint64_t a_batch, uint64_t m, cons
     switch (ep.mode) {
         case LinearEpilogue::kResidual: return launch_f32<LinearEpilogue::kResidual>(a, lda, a_batch, m, w, ep, s);
         case LinearEpilogue::kGlu: return launch_f32<LinearEpilogue::kGlu>(a, lda, a_batch, m, w, ep, s);
+        case LinearEpilogue::kSiluGlu: return launch_f32<LinearEpilogue::kSiluGlu>(a, lda, a_batch, m, w, ep, s);
         case LinearEpilogue::kSoftcap: return launch_f32<LinearEpilogue::kSoftcap>(a, lda, a_batch, m, w, ep, s);
         case LinearEpilogue::kHeadGate: return launch_f32<LinearEpilogue::kHeadGate>(a, lda, a_batch, m, w, ep, s);
         default: return launch_f32<LinearEpilogue::kStore>(a, lda, a_batch, m, w, ep, s);
@@ -431,18 +434,18 @@ void linear_grouped_f32(const float *a, uint64_t lda, const LinearWeight &w, con
 }
 
 void pack_linear(const void *src, int src_f32, uint64_t row_stride, uint64_t col_stride, uint32_t rows, uint32_t cols, void *dst,
-                 int dst_f32, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch, hipStream_t s) {
+                 int dst_f32, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch, hipStream_t s, uint32_t k0) {
     const uint64_t total = (uint64_t)rows * cols;
     if (total == 0) return;
     const unsigned grid = (unsigned)std::min<uint64_t>((total + 255) / 256, 8192);
     if (src_f32 && dst_f32)
-        pack_linear_kernel<float, float><<<grid, 256, 0, s>>>((const float *)src, row_stride, col_stride, rows, cols, (float *)dst, k_tiles, n0, group, pitch);
+        pack_linear_kernel<float, float><<<grid, 256, 0, s>>>((const float *)src, row_stride, col_stride, rows, cols, (float *)dst, k_tiles, n0, group, pitch, k0);
     else if (src_f32)
-        pack_linear_kernel<float, uint16_t><<<grid, 256, 0, s>>>((const float *)src, row_stride, col_stride, rows, cols, (uint16_t *)dst, k_tiles, n0, group, pitch);
+        pack_linear_kernel<float, uint16_t><<<grid, 256, 0, s>>>((const float *)src, row_stride, col_stride, rows, cols, (uint16_t *)dst, k_tiles, n0, group, pitch, k0);
     else if (dst_f32)
-        pack_linear_kernel<uint16_t, float><<<grid, 256, 0, s>>>((const uint16_t *)src, row_stride, col_stride, rows, cols, (float *)dst, k_tiles, n0, group, pitch);
+        pack_linear_kernel<uint16_t, float><<<grid, 256, 0, s>>>((const uint16_t *)src, row_stride, col_stride, rows, cols, (float *)dst, k_tiles, n0, group, pitch, k0);
     else
-        pack_linear_kernel<uint16_t, uint16_t><<<grid, 256, 0, s>>>((const uint16_t *)src, row_stride, col_stride, rows, cols, (uint16_t *)dst, k_tiles, n0, group, pitch);
+        pack_linear_kernel<uint16_t, uint16_t><<<grid, 256, 0, s>>>((const uint16_t *)src, row_stride, col_stride, rows, cols, (uint16_t *)dst, k_tiles, n0, group, pitch, k0);
 }
 
 }  // namespace k

@@ -329,7 +329,7 @@ struct LinearWeight {
 };
 // What becomes of y = a W^T (f32):
 struct LinearEpilogue {
-    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4, kSquaredRelu = 5 };
+    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4, kSquaredRelu = 5, kSiluGlu = 6 };
     int mode = kStore;
     void *out = nullptr;         // [m, ld_out], f32 or bf16; kResidual: the f32 residual itself
     int out_f32 = 0;
@@ -342,6 +342,8 @@ struct LinearEpilogue {
     const float *scale = nullptr;    // kResidual: out[r, c] += scale[c] * y
     // kGlu: tiles alternate gate / up; g = min(gate, limit), u = clamp(up, +-limit), out = g sigmoid(alpha g) (u + 1)
     float limit = 0.0f, alpha = 0.0f;
+    // kSiluGlu: gate sigmoid(gate) up, tiles as kGlu's
+    float factor = 1.0f;         // kStore, kSoftcap, kHeadGate: of y, ahead of everything else
     float cap = 0.0f;            // kSoftcap: cap tanh(y / cap); cap <= 0: y
     const float *gate = nullptr; // kHeadGate: y * sigmoid(gate[r * ld_gate + batch])
     uint32_t ld_gate = 0;
@@ -368,9 +370,9 @@ void gemm_bf16_big_grouped(const uint16_t *a, const LinearWeight &w, const RowGr
 bool gemm_bf16_big_applies(uint64_t lda, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus);
 void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const LinearEpilogue &ep, int num_cus, hipStream_t s);
 // Packs `rows` source rows of `cols` values (bf16 bits or f32; element (r, c) at src[r * row_stride + c * col_stride]) into
-// columns dst_row(r) of a weight: dst_row(r) = n0 + (r / group) * pitch + r % group.
+// columns dst_row(r) of a weight: dst_row(r) = n0 + (r / group) * pitch + r % group, from its input k0 on.
 void pack_linear(const void *src, int src_f32, uint64_t row_stride, uint64_t col_stride, uint32_t rows, uint32_t cols, void *dst,
-                 int dst_f32, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch, hipStream_t s);
+                 int dst_f32, uint32_t k_tiles, uint32_t n0, uint32_t group, uint32_t pitch, hipStream_t s, uint32_t k0 = 0);
 
 // ---- layered decoder: rows, norms (kern_decoder.hip, kern_norm_quant.hip) ----------------
 // One pass over sequences of any numbers of new tokens: sequence b owns rows row_start[b] .. row_start[b + 1] - 1.
@@ -389,8 +391,9 @@ void ragged_prepare(const uint32_t *row_start, const uint32_t *tables, const uin
                     uint32_t *kv_slot, int32_t *last_rows, uint32_t batch, uint32_t rows, uint32_t block_size, uint32_t max_blocks,
                     uint32_t num_blocks, hipStream_t s);
 void ragged_advance(const uint32_t *row_start, uint32_t *seq_lens, uint32_t batch, hipStream_t s);
-// cos_sin [rows, dims] of the rows' positions (cos in the first half, sin in the second), angles formed in double
-void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t dims, double base, hipStream_t s);
+// cos_sin [rows, dims] of the rows' positions (cos in the first half, sin in the second) for the frequencies freq [dims / 2],
+// angles formed in double
+void rotation_table(const int32_t *pos, float *cos_sin, uint32_t rows, uint32_t dims, const double *freq, hipStream_t s);
 // (x - mean) / sqrt(variance + eps) * w per row; out f32 or bf16 with pitch ld, zeros past hidden
 void layernorm_rows(const float *x, const float *w, void *out, int out_f32, uint64_t rows, uint64_t hidden, uint64_t ld, float eps,
                     hipStream_t s);
@@ -418,7 +421,8 @@ struct RouteIo {
 };
 constexpr uint32_t kMaxExperts = 256, kMaxTop = 64;
 void route_rows(const void *h_bf16, uint64_t rows, uint64_t ld, const RouteIo &io, hipStream_t s);
-// x += rmsnorm(y) * w, hn = x in the activations' type (pitch ld, zeros past hidden).  y [rows * parts, hidden] f32; parts > 1
+// x += norm(y) * w, hn = x in the activations' type (pitch ld, zeros past hidden).  The norm is RMS norm, or with `layer` layer
+// norm, hn then being layernorm(x) * next (next null: hn is left alone).  y [rows * parts, hidden] f32; parts > 1
 // (or gate set): y's row is sum_i gate[row][i] y[row * parts + i].  clear (n_clear words): set to zero.  route: the rows'
 // experts are chosen in the same launch (for few rows and in f32; many bf16 rows are faster in a launch of route_rows).
 struct ResidualNorm {
@@ -427,6 +431,8 @@ struct ResidualNorm {
     const float *w = nullptr;
     float eps = 0.0f;
     uint32_t *clear = nullptr, n_clear = 0;
+    bool layer = false;
+    const float *next = nullptr;
 };
 bool residual_norm_routes(int is_f32, uint64_t rows);
 void residual_norm(const ResidualNorm &rn, float *x, void *hn, int is_f32, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo *route,
@@ -439,20 +445,36 @@ struct AttentionShape {
                                  // padding zero in the pools
     float scale, eps;
     uint64_t pool_rows;
+    uint32_t window;             // keys p - window + 1 .. p
+    uint32_t rot, interleaved;   // leading entries of every query and key head that are rotated; their pairs
     __host__ __device__ uint32_t share() const { return heads / kv_heads; }
 };
+constexpr uint32_t kWholeContext = 0x7fffffff;       // a window that holds every earlier token
 void attention_pad(AttentionShape &sh);
 // From y [rows, ld] f32 = q | k | v: with norms (nullable), RMS norm over the whole of q and of k; q -> [rows, heads, dim_p], k and
 // v -> the token's cache rows (pools null: y holds q only).
 void attention_prepare(const float *y, uint32_t ld, const float *q_norm, const float *k_norm, void *q, void *k_pool, void *v_pool, int is_f32,
                        const AttentionShape &sh, const RaggedRows &rr, hipStream_t s);
+// The form with norms per head and rotation: q, k of a head x / sqrt(mean(x^2) + eps) * w with norms (weights [dim], shared by the
+// heads; null: 1), then their first sh.rot entries turned by cos_sin [rows, rot].  key_values: y = q | k, and the projected keys
+// are the values.
+void attention_prepare_heads(const float *y, uint32_t ld, bool norms, const float *q_norm, const float *k_norm, const float *cos_sin, bool key_values, void *q,
+                             void *k_pool, void *v_pool, int is_f32, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s);
+// What happens to the softmax and its result: sink [heads]: a score without key and value (null: none); gate [rows, ld_gate] in
+// the activations' type, heads x vdim: the output times its sigmoid (null: none); and times scale.
+struct AttentionOutput {
+    const float *sink = nullptr;
+    const void *gate = nullptr;
+    uint32_t ld_gate = 0;
+    float scale = 1.0f;
+};
 // Causal softmax attention over the cache -> out [rows, ld_out], heads x vdim.  bf16 with padded sizes up to 256: matrix-core
 // kernels, one for few query rows per sequence (the keys split over blocks that meet in the workspace) and one for many;
 // otherwise a plain one.  min_new / max_new: fewest (not counting none) and most new tokens of any sequence.
 uint64_t attention_workspace_bytes(const AttentionShape &sh, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
                                    int num_cus);
-void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, int is_f32, const AttentionShape &sh,
-               const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
+void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, const AttentionOutput &ao, int is_f32,
+               const AttentionShape &sh, const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
 
 // ---- latent attention (kern_latent.hip) -----------------------------------------
 struct LatentShape {
@@ -460,6 +482,7 @@ struct LatentShape {
     uint32_t dim_p, rot_p, rank_p, v_p;                  // padded (latent_pad): q rows are [heads][dim_p + rot_p], cache rows
                                                          // and absorbed queries [rank_p + rot_p], padding zero
     uint32_t window;                                     // keys p - window + 1 .. p
+    uint32_t interleaved;                                // pairs of the rotation: 1 neighbours, 0 half the rotated part apart
     float scale, eps;
     uint64_t pool_rows;
 };
@@ -482,7 +505,7 @@ void latent_attention(const void *qa, const void *pool, void *out, int is_f32, c
 // The form for prompts (bf16, dim, vdim <= 128, rot <= 64): the keys first[b] .. of every sequence are gathered as rows
 // start[b] .. start[b + 1] - 1 (latents c [rows, ld_c], rotated parts kr [rows, rot_p]), a linear turns the latents into
 // kv [rows, heads, dim_p + v_p], and attention runs per head on those; q is [rows, heads, dim_p + rot_p] with its
-// rotated part rotated; the heads' gates (sigmoid) are applied, out [rows, ld_out].
+// rotated part rotated; the heads' gates (sigmoid; null: none) and out_scale are applied, out [rows, ld_out].
 struct LatentExpand {
     const uint32_t *start, *first;   // [batch + 1], [batch]
     uint32_t rows;
@@ -490,28 +513,41 @@ struct LatentExpand {
 bool latent_expand_applies(const LatentShape &sh);
 bool latent_expand_always();         // tuning: wherever it applies, whatever it costs
 void latent_gather(const void *pool, void *c, uint32_t ld_c, void *kr, const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s);
-void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, void *out, uint32_t ld_out,
+void latent_attention_expanded(const void *q, const void *kv, const void *kr, const float *gate, uint32_t ld_gate, float out_scale, void *out, uint32_t ld_out,
                                const LatentShape &sh, const RaggedRows &rr, const LatentExpand &ex, hipStream_t s);
 
-// ---- gated delta rule (kern_delta.hip) --------------------------------------------
+// ---- linear recurrences (kern_delta.hip) ------------------------------------------
+enum class Recurrence {
+    kDelta,                      // gated delta rule, a decay per head
+    kChannelDelta,               // gated delta rule, a decay per head and key channel
+    kLightning                   // S <- decay S + k v^T with constant decays; q and k as projected, behind silu
+};
 struct DeltaShape {
-    uint32_t heads, kv_heads, dim, vdim, taps;
+    Recurrence kind;
+    uint32_t heads, kv_heads, dim, vdim, taps;           // taps 0: no convolution
+    uint32_t norm_all, gate_sigmoid;                     // read-outs: norm over all heads instead of each; sigmoid gate instead of silu
     __host__ __device__ uint32_t qkv() const { return 2 * kv_heads * dim + heads * vdim; }       // channels that pass the convolution
     __host__ __device__ uint32_t vdim_p() const { return (vdim + 3) / 4 * 4; }
     float eps;
 };
 struct DeltaIo {
-    const void *y;               // [rows, ld_y] q | k | v | g (bf16 or f32)
+    const void *y;               // [rows, ld_y] q | k | v (bf16 or f32)
     uint32_t ld_y;
-    const float *ba;             // [rows, ld_ba] b | a projections
-    uint32_t ld_ba;
+    const void *gate;            // [rows, ld_gate] heads x vdim (type of y)
+    uint32_t ld_gate;
+    const float *beta;           // [rows, ld_beta], one per head, ahead of its sigmoid
+    uint32_t ld_beta;
+    const float *decay;          // [rows, ld_decay], per head (x dim), ahead of dt_bias; lightning: [heads], the decays
+    uint32_t ld_decay;
     const float *conv;           // [qkv][taps]
-    const float *a_log, *dt_bias, *norm;
+    const float *a_log, *dt_bias, *norm;         // norm [vdim], or [heads x vdim] with norm_all
     float *state;                // [slots][heads][dim][vdim_p]
     void *ring;                  // [slots][taps][qkv], input of position p in entry p % taps (type of y)
-    void *out;                   // [rows, ld_out] gated, normed read-outs (type of y)
+    void *out;                   // [rows, ld_out] gated, normed read-outs times out_scale (type of y)
     uint32_t ld_out;
+    float out_scale;
     float *scratch;              // delta_scratch_bytes: chunk form only
+    float *raw;                  // [rows, heads x vdim] read-outs: chunk form and norm_all
 };
 constexpr uint32_t kDeltaMaxDim = 256, kDeltaMaxVdim = 1024;
 uint64_t delta_scratch_bytes(const DeltaShape &sh, uint32_t rows, uint32_t batch);

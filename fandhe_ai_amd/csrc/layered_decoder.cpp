@@ -29,14 +29,18 @@ struct Tensor {
     std::function<void(const void *src, int src_f32, hipStream_t s)> place;
 };
 
-struct Layer {
+// What mixes the tokens of a layer.  Its projections of the layer's input are columns of the layer's `in`: those that stay in the
+// activations' type start at column lo_at of Arena::y, f32 ones at hi_at of Arena::y32.  Its output is columns o_at .. of Arena::o.
+struct Mixer {
     fa_layer_config cfg;
-    float *norm1 = nullptr, *norm2 = nullptr, *ls1 = nullptr, *ls2 = nullptr;
-    k::LinearWeight in, out, gate_up, down;           // with experts: gate_up and down hold one batch entry each
-    k::LinearWeight router;
+    std::string prefix;                               // of its tensors
+    uint32_t lo = 0, lo_at = 0, hi = 0, hi_at = 0, o_at = 0;
+    float out_scale = 1.0f;
+    uint32_t out_width() const { return cfg.heads * cfg.vdim; }
     // attention; q_norm below
     k::AttentionShape at{};
-    float *in_bias = nullptr, *k_norm = nullptr;
+    uint32_t gate_at = 0;                             // column of its `lo` part where the gate starts
+    float *k_norm = nullptr, *sink = nullptr;
     void *k_pool = nullptr, *v_pool = nullptr;
     // latent attention
     k::LatentShape la{};
@@ -45,11 +49,52 @@ struct Layer {
     float *q_norm = nullptr, *kv_norm = nullptr;
     void *pool = nullptr;
     uint32_t rotation = 0;                            // index of its cos / sin table
-    // delta
+    // delta, lightning
     k::DeltaShape de{};
-    float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *head_norm = nullptr, *state = nullptr;
+    float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *head_norm = nullptr, *state = nullptr, *decay = nullptr;
     void *ring = nullptr;
+    // low-rank gates and decays: their inner values start at column rank_at of the `lo` part (decay first, gate from its padded
+    // rank on); one weight with zeros in the other's place makes both
+    k::LinearWeight low_rank;
+    uint32_t rank_at = 0;
 };
+
+bool recurrent(const fa_layer_config &c) { return c.mixer == FA_MIXER_DELTA || c.mixer == FA_MIXER_LIGHTNING; }
+
+struct Layer {
+    fa_layer_config cfg;
+    std::vector<Mixer> mixers;                        // one, or two side by side
+    uint32_t lo = 0, hi = 0, o_width = 0;             // columns of in (lo a multiple of eight) and inputs of out, all mixers
+    float *norm1 = nullptr, *norm2 = nullptr, *post1 = nullptr, *post2 = nullptr;     // post: layer scale, or norm of the output
+    float *in_bias = nullptr;                         // attention alone in its layer
+    k::LinearWeight in, out, gate_up, down;           // with experts: gate_up and down hold one batch entry each
+    k::LinearWeight router;
+};
+
+// A rotation's frequencies follow from these
+struct Rotation {
+    uint32_t dims;
+    double base, factor, low, high, original;
+    bool operator==(const Rotation &o) const {
+        return dims == o.dims && base == o.base && factor == o.factor && low == o.low && high == o.high && original == o.original;
+    }
+};
+Rotation rotation_of(const fa_layer_config &c) {
+    if (!(c.rot_factor > 0.0)) return Rotation{c.rot_dim, c.rot_base, 0.0, 0.0, 0.0, 0.0};
+    return Rotation{c.rot_dim, c.rot_base, c.rot_factor, c.rot_low, c.rot_high, c.rot_original};
+}
+std::vector<double> frequencies(const Rotation &r) {
+    std::vector<double> f(r.dims / 2);
+    for (uint32_t i = 0; i < f.size(); ++i) {
+        f[i] = std::pow(r.base, -2.0 * (double)i / (double)r.dims);
+        if (r.factor > 0.0) {
+            const double turns = r.original * f[i] / (2.0 * 3.14159265358979323846);
+            const double ramp = turns < r.low ? 0.0 : turns > r.high ? 1.0 : (turns - r.low) / (r.high - r.low);
+            f[i] = (1.0 - ramp) * f[i] / r.factor + ramp * f[i];
+        }
+    }
+    return f;
+}
 
 // Activations of a pass of up to `rows` rows, one allocation.  Every section keeps its place and element type for the
 // arena's life and starts as zeros: what lies behind a row's own width is always finite.
@@ -57,9 +102,9 @@ struct Arena {
     void *base = nullptr;
     uint64_t bytes = 0, cls = 0;
     uint32_t rows = 0;
-    float *x = nullptr, *y32 = nullptr, *ba = nullptr, *head_x = nullptr, *delta_scratch = nullptr, *gate = nullptr;
+    float *x = nullptr, *y32 = nullptr, *head_x = nullptr, *delta_scratch = nullptr, *raw = nullptr, *decay = nullptr, *gate = nullptr;
     uint32_t *expert_count = nullptr, *expert_list = nullptr;       // counts are zero between feed-forwards
-    void *hn = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *olat = nullptr, *o = nullptr, *act = nullptr;
+    void *hn = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *olat = nullptr, *o = nullptr, *act = nullptr, *low_gate = nullptr;
     uint32_t *row_seq = nullptr, *kv_slot = nullptr, *row_start = nullptr;
     int32_t *pos = nullptr, *tokens = nullptr, *want = nullptr;
     std::vector<float *> cos_sin;
@@ -78,11 +123,11 @@ struct ExpandPlan {
 
 struct LayeredState {
     fa_layered_config cfg{};
-    std::vector<fa_layer_config> layer_cfgs;
     std::vector<Layer> layers;
     std::vector<Tensor> tensors;
     std::vector<fa_buffer *> owned;
-    std::vector<std::pair<uint32_t, double>> rotations;      // distinct (dims, base)
+    std::vector<Rotation> rotations;                         // distinct ones
+    std::vector<double *> rotation_freq;
     std::vector<uint32_t> windows;                           // distinct windows
     void *embed = nullptr;
     double *position_freq = nullptr;                         // additive positions: of every pair of entries
@@ -102,30 +147,35 @@ namespace {
 
 // widest of every activation over the layers
 struct Widths {
-    uint64_t hn = 0, y32 = 0, y = 0, ba = 0, cq = 0, q = 0, qa = 0, olat = 0, o = 0, act = 0, top = 0, experts = 0;
+    uint64_t hn = 0, y32 = 0, y = 0, cq = 0, q = 0, qa = 0, olat = 0, o = 0, act = 0, top = 0, experts = 0, raw = 0, decay = 0, low_gate = 0;
 };
 
 Widths widths(const LayeredState &L) {
     Widths w;
     w.hn = pad_to(L.cfg.d_model, 64);
     for (const Layer &l : L.layers) {
-        if (l.cfg.mixer == FA_MIXER_DELTA) {
-            w.y = std::max<uint64_t>(w.y, pad_to(l.de.qkv() + l.de.heads * l.de.vdim, 8));
-            w.ba = std::max<uint64_t>(w.ba, 2 * l.de.heads);
-        } else if (l.cfg.mixer == FA_MIXER_ATTENTION) {
-            w.y32 = std::max<uint64_t>(w.y32, pad_to(l.in.n, 4));
-            w.q = std::max<uint64_t>(w.q, (uint64_t)l.at.heads * l.at.dim_p);
-        } else {
-            w.y32 = std::max<uint64_t>(w.y32, pad_to(l.in.n, 4));
-            w.cq = std::max<uint64_t>(w.cq, pad_to(l.la.q_rank, 64));
-            w.q = std::max<uint64_t>(w.q, (uint64_t)l.la.heads * (l.la.dim_p + l.la.rot_p));
-            w.qa = std::max<uint64_t>(w.qa, (uint64_t)l.la.heads * (l.la.rank_p + l.la.rot_p));
-            w.olat = std::max<uint64_t>(w.olat, (uint64_t)l.la.heads * l.la.rank_p);
+        w.y = std::max<uint64_t>(w.y, l.lo);
+        w.y32 = std::max<uint64_t>(w.y32, pad_to(l.hi, 4));
+        w.o = std::max<uint64_t>(w.o, pad_to(l.o_width, 64));
+        for (const Mixer &m : l.mixers) {
+            if (recurrent(m.cfg)) {
+                w.raw = std::max<uint64_t>(w.raw, m.out_width());
+                if (m.low_rank.w) {
+                    w.decay = std::max<uint64_t>(w.decay, pad_to(m.de.heads * m.de.dim, 4));
+                    w.low_gate = std::max<uint64_t>(w.low_gate, pad_to(m.out_width(), 8));
+                }
+            } else if (m.cfg.mixer == FA_MIXER_ATTENTION) {
+                w.q = std::max<uint64_t>(w.q, (uint64_t)m.at.heads * m.at.dim_p);
+            } else {
+                w.cq = std::max<uint64_t>(w.cq, pad_to(m.la.q_rank, 64));
+                w.q = std::max<uint64_t>(w.q, (uint64_t)m.la.heads * (m.la.dim_p + m.la.rot_p));
+                w.qa = std::max<uint64_t>(w.qa, (uint64_t)m.la.heads * (m.la.rank_p + m.la.rot_p));
+                w.olat = std::max<uint64_t>(w.olat, (uint64_t)m.la.heads * m.la.rank_p);
+            }
         }
-        w.o = std::max<uint64_t>(w.o, pad_to(l.cfg.heads * l.cfg.vdim, 64));
         const uint64_t parts = l.cfg.experts ? l.cfg.top : 1;
         if (l.cfg.d_ffn) w.act = std::max<uint64_t>(w.act, parts * pad_to(l.cfg.d_ffn, 64));
-        if (L.cfg.norm == FA_NORM_OUTPUT) w.y32 = std::max<uint64_t>(w.y32, parts * L.cfg.d_model);
+        if (L.cfg.norm != FA_NORM_INPUT) w.y32 = std::max<uint64_t>(w.y32, parts * L.cfg.d_model);
         w.top = std::max<uint64_t>(w.top, l.cfg.experts ? l.cfg.top : 0);
         w.experts = std::max<uint64_t>(w.experts, l.cfg.experts);
     }
@@ -153,7 +203,9 @@ fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t row
     add(&a.hn, std::max(R, B) * w.hn * E);
     add((void **)&a.y32, R * w.y32 * 4);
     add(&a.y, R * w.y * E);
-    add((void **)&a.ba, R * w.ba * 4);
+    add((void **)&a.raw, R * w.raw * 4);
+    add((void **)&a.decay, R * w.decay * 4);
+    add(&a.low_gate, R * w.low_gate * E);
     add(&a.cq, R * w.cq * E);
     add(&a.q, R * w.q * E);
     add(&a.qa, R * w.qa * E);
@@ -169,18 +221,20 @@ fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t row
     add((void **)&a.tokens, R * 4);
     add((void **)&a.want, std::max(R, B) * 4);
     add((void **)&a.row_start, (B + 1) * 4);
-    for (size_t i = 0; i < L.rotations.size(); ++i) add((void **)&a.cos_sin[i], R * L.rotations[i].first * 4);
+    for (size_t i = 0; i < L.rotations.size(); ++i) add((void **)&a.cos_sin[i], R * L.rotations[i].dims * 4);
     uint64_t scratch = 0;
     for (const Layer &l : L.layers)
-        if (l.cfg.mixer == FA_MIXER_DELTA) scratch = std::max(scratch, k::delta_scratch_bytes(l.de, rows, (uint32_t)B));
+        for (const Mixer &m : l.mixers)
+            if (recurrent(m.cfg)) scratch = std::max(scratch, k::delta_scratch_bytes(m.de, rows, (uint32_t)B));
     add((void **)&a.delta_scratch, scratch);
     uint64_t ec = 0, er = 0, ekv = 0;
     for (const Layer &l : L.layers)
-        if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) {
-            ec = std::max<uint64_t>(ec, pad_to(l.la.rank_p, 64));
-            er = std::max<uint64_t>(er, l.la.rot_p);
-            ekv = std::max<uint64_t>(ekv, (uint64_t)l.la.heads * (l.la.dim_p + l.la.v_p));
-        }
+        for (const Mixer &m : l.mixers)
+            if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION) {
+                ec = std::max<uint64_t>(ec, pad_to(m.la.rank_p, 64));
+                er = std::max<uint64_t>(er, m.la.rot_p);
+                ekv = std::max<uint64_t>(ekv, (uint64_t)m.la.heads * (m.la.dim_p + m.la.v_p));
+            }
     if (L.is_f32) expand_rows = 0;
     add(&a.ec, expand_rows * ec * E);
     add(&a.er, expand_rows * er * E);
@@ -223,73 +277,137 @@ struct Portions {
     uint32_t min_new, max_new;
 };
 
-// The mixers: from a.hn to a.o (pitch ld_o).
-void enqueue_delta(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const k::RaggedRows &rr, uint32_t max_new, uint32_t ld_hn, uint32_t ld_o) {
-    const uint32_t n_lo = l.in.n - 2 * l.de.heads, ld_y = pad_to(n_lo, 8);
-    k::LinearEpilogue e = store_to(a.y, ld_y, L.is_f32);
-    e.n_lo = n_lo;
-    e.out_hi = a.ba;
-    e.ld_hi = 2 * l.de.heads;
-    linear(ctx, L, a.hn, ld_hn, 0, rr.rows, l.in, e);
-    k::DeltaIo io{a.y, ld_y, a.ba, 2 * l.de.heads, l.conv, l.a_log, l.dt_bias, l.head_norm, l.state, l.ring, a.o, ld_o, a.delta_scratch};
-    k::delta_mixer(l.de, io, L.is_f32, rr, max_new, ctx->stream);
+// Element `at` of an activation section in the activations' type
+void *element(const LayeredState &L, void *base, uint64_t at) { return (uint8_t *)base + at * L.esz; }
+
+// The layer's input a.hn -> what its mixers read, a.y and a.y32.
+void enqueue_in(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t rows, uint32_t ld_hn) {
+    k::LinearEpilogue e = l.lo ? store_to(a.y, l.lo, L.is_f32) : store_to(a.y32, pad_to(l.hi, 4), 1);
+    if (l.lo) {
+        e.n_lo = l.lo;
+        e.out_hi = a.y32;
+        e.ld_hi = pad_to(l.hi, 4);
+    }
+    e.bias = l.in_bias;
+    linear(ctx, L, a.hn, ld_hn, 0, rows, l.in, e);
 }
 
-void enqueue_latent(fa_context *ctx, const fa_decoder *d, Arena &a, const Layer &l, const k::RaggedRows &rr, uint32_t max_new, uint32_t ld_hn,
+// The mixers: from a.y and a.y32 to their columns of a.o (pitch ld_o).
+void enqueue_recurrence(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const Mixer &m, const k::RaggedRows &rr, uint32_t max_new, uint32_t ld_o) {
+    const k::DeltaShape &sh = m.de;
+    const uint32_t ld_hi = pad_to(l.hi, 4), ow = m.out_width();
+    k::DeltaIo io{};
+    io.y = element(L, a.y, m.lo_at);
+    io.ld_y = l.lo;
+    io.gate = element(L, a.y, m.lo_at + m.gate_at);
+    io.ld_gate = l.lo;
+    io.beta = a.y32 + m.hi_at;
+    io.ld_beta = ld_hi;
+    if (m.low_rank.w) {
+        k::LinearEpilogue e = store_to(a.low_gate, pad_to(ow, 8), L.is_f32);
+        e.n_lo = pad_to(ow, 8);
+        e.out_hi = a.decay;
+        e.ld_hi = pad_to(sh.heads * sh.dim, 4);
+        linear(ctx, L, element(L, a.y, m.lo_at + m.rank_at), l.lo, 0, rr.rows, m.low_rank, e);
+        io.gate = a.low_gate;
+        io.ld_gate = e.ld_out;
+        io.decay = a.decay;
+        io.ld_decay = e.ld_hi;
+    } else {
+        io.decay = sh.kind == k::Recurrence::kLightning ? m.decay : io.beta + sh.heads;
+        io.ld_decay = ld_hi;
+    }
+    io.conv = m.conv;
+    io.a_log = m.a_log;
+    io.dt_bias = m.dt_bias;
+    io.norm = m.head_norm;
+    io.state = m.state;
+    io.ring = m.ring;
+    io.out = element(L, a.o, m.o_at);
+    io.ld_out = ld_o;
+    io.out_scale = m.out_scale;
+    io.scratch = a.delta_scratch;
+    io.raw = a.raw;
+    k::delta_mixer(sh, io, L.is_f32, rr, max_new, ctx->stream);
+}
+
+void enqueue_latent(fa_context *ctx, const fa_decoder *d, Arena &a, const Layer &l, const Mixer &m, const k::RaggedRows &rr, uint32_t max_new,
                     uint32_t ld_o, const ExpandPlan *expand) {
     LayeredState &L = *d->layered;
     hipStream_t s = ctx->stream;
     const int f32 = L.is_f32;
     const uint32_t M = rr.rows;
-    const k::LatentShape &sh = l.la;
-    const uint32_t ld_y = pad_to(l.in.n, 4), ld_cq = pad_to(sh.q_rank, 64), qw = sh.dim_p + sh.rot_p, kw = sh.rank_p + sh.rot_p;
-    const bool own = l.cfg.kv_from < 0;
-    const float *cs = a.cos_sin[l.rotation];
-    void *pool = own ? l.pool : L.layers[l.cfg.kv_from].pool;
-    linear(ctx, L, a.hn, ld_hn, 0, M, l.in, store_to(a.y32, ld_y, 1));
-    k::latent_prepare(a.y32, ld_y, l.q_norm, l.kv_norm, cs, a.cq, ld_cq, own ? pool : nullptr, f32, sh, rr, s);
-    linear(ctx, L, a.cq, ld_cq, 0, M, l.uq, store_to(a.q, (uint64_t)sh.heads * qw, f32));
-    const float *gate = a.y32 + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
-    if (expand && expand->rows[l.window_index]) {
-        const uint32_t *meta = a.expand_meta + (uint64_t)l.window_index * (2 * d->cfg.max_batch + 1);
-        const k::LatentExpand ex{meta, meta + d->cfg.max_batch + 1, expand->rows[l.window_index]};
+    const k::LatentShape &sh = m.la;
+    const uint32_t ld_y = pad_to(l.hi, 4), ld_cq = pad_to(sh.q_rank, 64), qw = sh.dim_p + sh.rot_p, kw = sh.rank_p + sh.rot_p;
+    const bool own = m.cfg.kv_from < 0;
+    const float *cs = a.cos_sin[m.rotation], *y = a.y32 + m.hi_at;
+    void *pool = own ? m.pool : L.layers[m.cfg.kv_from].mixers[0].pool, *o = element(L, a.o, m.o_at);
+    k::latent_prepare(y, ld_y, m.q_norm, m.kv_norm, cs, a.cq, ld_cq, own ? pool : nullptr, f32, sh, rr, s);
+    linear(ctx, L, a.cq, ld_cq, 0, M, m.uq, store_to(a.q, (uint64_t)sh.heads * qw, f32));
+    const float *gate = m.cfg.ungated ? nullptr : y + sh.q_rank + (own ? sh.kv_rank + sh.rot : 0);
+    if (expand && expand->rows[m.window_index]) {
+        const uint32_t *meta = a.expand_meta + (uint64_t)m.window_index * (2 * d->cfg.max_batch + 1);
+        const k::LatentExpand ex{meta, meta + d->cfg.max_batch + 1, expand->rows[m.window_index]};
         const uint32_t ld_c = pad_to(sh.rank_p, 64);
         k::latent_rotate_query(a.q, cs, a.q, qw, sh.dim_p, f32, sh, M, s);
         k::latent_gather(pool, a.ec, ld_c, a.er, sh, rr, ex, s);
-        linear(ctx, L, a.ec, ld_c, 0, ex.rows, l.ukv, store_to(a.ekv, l.ukv.n, f32));
-        k::latent_attention_expanded(a.q, a.ekv, a.er, gate, ld_y, a.o, ld_o, sh, rr, ex, s);
+        linear(ctx, L, a.ec, ld_c, 0, ex.rows, m.ukv, store_to(a.ekv, m.ukv.n, f32));
+        k::latent_attention_expanded(a.q, a.ekv, a.er, gate, ld_y, m.out_scale, o, ld_o, sh, rr, ex, s);
     } else {
         k::LinearEpilogue e = store_to(a.qa, (uint64_t)sh.heads * kw, f32);
         e.out_batch = kw;
-        linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, l.uk, e);
+        linear(ctx, L, a.q, (uint64_t)sh.heads * qw, qw, M, m.uk, e);
         k::latent_rotate_query(a.q, cs, a.qa, kw, sh.rank_p, f32, sh, M, s);
         k::latent_attention(a.qa, pool, a.olat, f32, sh, rr, max_new, ctx->workspace, ctx->props.multiProcessorCount, s);
-        e = store_to(a.o, ld_o, f32);
-        e.mode = k::LinearEpilogue::kHeadGate;
+        e = store_to(o, ld_o, f32);
+        if (gate) e.mode = k::LinearEpilogue::kHeadGate;
+        e.factor = m.out_scale;
         e.out_batch = sh.vdim;
         e.gate = gate;
         e.ld_gate = ld_y;
-        linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, l.uv, e);
+        linear(ctx, L, a.olat, (uint64_t)sh.heads * sh.rank_p, sh.rank_p, M, m.uv, e);
     }
 }
 
-void enqueue_attention(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const k::RaggedRows &rr, Portions n, uint32_t ld_hn, uint32_t ld_o) {
-    const k::AttentionShape &sh = l.at;
-    const uint32_t ld_y = pad_to(l.in.n, 4);
-    const bool own = l.cfg.kv_from < 0;
-    const Layer &kv = own ? l : L.layers[l.cfg.kv_from];
-    k::LinearEpilogue e = store_to(a.y32, ld_y, 1);
-    e.bias = l.in_bias;
-    linear(ctx, L, a.hn, ld_hn, 0, rr.rows, l.in, e);
-    k::attention_prepare(a.y32, ld_y, l.q_norm, l.k_norm, a.q, own ? l.k_pool : nullptr, own ? l.v_pool : nullptr, L.is_f32, sh, rr, ctx->stream);
-    k::attention(a.q, kv.k_pool, kv.v_pool, a.o, ld_o, L.is_f32, sh, rr, n.min_new, n.max_new, ctx->workspace, ctx->props.multiProcessorCount, ctx->stream);
+void enqueue_attention(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const Mixer &m, const k::RaggedRows &rr, Portions n, uint32_t ld_o) {
+    const k::AttentionShape &sh = m.at;
+    const uint32_t ld_y = pad_to(l.hi, 4), flags = m.cfg.attention;
+    const bool own = m.cfg.kv_from < 0;
+    const Mixer &kv = own ? m : L.layers[m.cfg.kv_from].mixers[0];
+    const float *y = a.y32 + m.hi_at;
+    const bool norms = flags & (FA_ATTENTION_HEAD_NORM | FA_ATTENTION_HEAD_UNIT), key_values = flags & FA_ATTENTION_KEY_VALUES;
+    if (norms || key_values || sh.rot)
+        k::attention_prepare_heads(y, ld_y, norms, m.q_norm, m.k_norm, sh.rot ? a.cos_sin[m.rotation] : nullptr, key_values, a.q, m.k_pool, m.v_pool, L.is_f32,
+                                   sh, rr, ctx->stream);
+    else
+        k::attention_prepare(y, ld_y, m.q_norm, m.k_norm, a.q, m.k_pool, m.v_pool, L.is_f32, sh, rr, ctx->stream);
+    k::AttentionOutput ao;
+    ao.sink = m.sink;
+    if (flags & FA_ATTENTION_GATE) {
+        ao.gate = element(L, a.y, m.lo_at + m.gate_at);
+        ao.ld_gate = l.lo;
+    }
+    ao.scale = m.out_scale;
+    k::attention(a.q, kv.k_pool, kv.v_pool, element(L, a.o, m.o_at), ld_o, ao, L.is_f32, sh, rr, n.min_new, n.max_new, ctx->workspace,
+                 ctx->props.multiProcessorCount, ctx->stream);
+}
+
+void enqueue_mixers(fa_context *ctx, fa_decoder *d, Arena &a, const Layer &l, const k::RaggedRows &rr, Portions n, uint32_t ld_hn, uint32_t ld_o,
+                    const ExpandPlan *expand) {
+    LayeredState &L = *d->layered;
+    enqueue_in(ctx, L, a, l, rr.rows, ld_hn);
+    for (const Mixer &m : l.mixers) {
+        if (recurrent(m.cfg)) enqueue_recurrence(ctx, L, a, l, m, rr, n.max_new, ld_o);
+        else if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION) enqueue_latent(ctx, d, a, l, m, rr, n.max_new, ld_o, expand);
+        else enqueue_attention(ctx, L, a, l, m, rr, n, ld_o);
+    }
 }
 
 // Dense feed-forward: from a.hn to what `out` does with the down projection.
 void enqueue_glu(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t M, uint32_t ld_hn, const k::LinearEpilogue &out) {
     const uint32_t ld_act = pad_to(l.cfg.d_ffn, 64);
     k::LinearEpilogue g = store_to(a.act, ld_act, L.is_f32);
-    g.mode = k::LinearEpilogue::kGlu;
+    g.mode = l.cfg.glu == FA_GLU_SILU ? k::LinearEpilogue::kSiluGlu : k::LinearEpilogue::kGlu;
     g.limit = l.cfg.ffn_limit;
     g.alpha = l.cfg.ffn_alpha;
     linear(ctx, L, a.hn, ld_hn, 0, M, l.gate_up, g);
@@ -316,21 +434,19 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
     const uint32_t M = rr.rows, D = L.cfg.d_model, ld_hn = pad_to(D, 64);
     const float eps = L.cfg.norm_eps;
     const int f32 = L.is_f32;
-    const bool at_output = L.cfg.norm == FA_NORM_OUTPUT;
-    for (size_t i = 0; i < L.rotations.size(); ++i) k::rotation_table(rr.pos, a.cos_sin[i], M, L.rotations[i].first, L.rotations[i].second, s);
+    for (size_t i = 0; i < L.rotations.size(); ++i) k::rotation_table(rr.pos, a.cos_sin[i], M, L.rotations[i].dims, L.rotation_freq[i], s);
+    if (L.cfg.norm == FA_NORM_BOTH) k::layernorm_rows(a.x, L.layers[0].norm1, a.hn, f32, M, D, ld_hn, eps, s);
     for (size_t li = 0; li < L.layers.size(); ++li) {
         const Layer &l = L.layers[li];
-        if (!at_output) k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);
-        const uint32_t ld_o = pad_to(l.cfg.heads * l.cfg.vdim, 64);
-        if (l.cfg.mixer == FA_MIXER_DELTA) enqueue_delta(ctx, L, a, l, rr, n.max_new, ld_hn, ld_o);
-        else if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION) enqueue_latent(ctx, d, a, l, rr, n.max_new, ld_hn, ld_o, expand);
-        else enqueue_attention(ctx, L, a, l, rr, n, ld_hn, ld_o);
-        if (at_output) {
+        if (L.cfg.norm == FA_NORM_INPUT) k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);
+        const uint32_t ld_o = pad_to(l.o_width, 64);
+        enqueue_mixers(ctx, d, a, l, rr, n, ld_hn, ld_o, expand);
+        k::ResidualNorm rn;
+        rn.y = a.y32;
+        rn.eps = eps;
+        if (L.cfg.norm == FA_NORM_OUTPUT) {
             linear(ctx, L, a.o, ld_o, 0, M, l.out, store_to(a.y32, D, 1));
-            k::ResidualNorm rn;
-            rn.y = a.y32;
             rn.w = l.norm1;
-            rn.eps = eps;
             k::RouteIo route{l.router.w, l.cfg.experts, l.cfg.top, a.expert_count, a.expert_list, a.rows, a.gate};
             const bool fused = l.cfg.experts && k::residual_norm_routes(f32, M);
             k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, fused ? &route : nullptr, s);
@@ -348,14 +464,28 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
                 rn.w = l.norm2;
                 k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
             }
+        } else if (L.cfg.norm == FA_NORM_BOTH) {
+            // a residual update norms the new stream for the sublayer that comes next; the head norms its own rows
+            const float *next_layer = li + 1 < L.layers.size() ? L.layers[li + 1].norm1 : nullptr;
+            linear(ctx, L, a.o, ld_o, 0, M, l.out, store_to(a.y32, D, 1));
+            rn.layer = true;
+            rn.w = l.post1;
+            rn.next = l.cfg.d_ffn ? l.norm2 : next_layer;
+            k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+            if (l.cfg.d_ffn) {
+                enqueue_glu(ctx, L, a, l, M, ld_hn, store_to(a.y32, D, 1));
+                rn.w = l.post2;
+                rn.next = next_layer;
+                k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+            }
         } else {
             k::LinearEpilogue r = store_to(a.x, D, 1);
             r.mode = k::LinearEpilogue::kResidual;
-            r.scale = l.ls1;
+            r.scale = l.post1;
             linear(ctx, L, a.o, ld_o, 0, M, l.out, r);
             if (l.cfg.d_ffn) {
                 k::layernorm_rows(a.x, l.norm2, a.hn, f32, M, D, ld_hn, eps, s);
-                r.scale = l.ls2;
+                r.scale = l.post2;
                 enqueue_glu(ctx, L, a, l, M, ld_hn, r);
             }
         }
@@ -384,6 +514,7 @@ void enqueue_head(fa_context *ctx, LayeredState &L, Arena &a, const float *x, ui
     else k::layernorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
     k::LinearEpilogue e = store_to(logits, L.cfg.vocab, 1);
     e.mode = k::LinearEpilogue::kSoftcap;
+    e.factor = L.cfg.logit_scale;
     e.cap = L.cfg.logit_softcap;
     linear(ctx, L, a.hn, ld_hn, 0, rows, L.head, e);
 }
@@ -404,12 +535,13 @@ void prepare_rows(fa_context *ctx, fa_decoder *d, Arena &a, const uint32_t *row_
 fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch, Portions n) {
     uint64_t need = 0;
     const int cus = ctx->props.multiProcessorCount;
-    for (const Layer &l : L.layers) {
-        if (l.cfg.mixer == FA_MIXER_LATENT_ATTENTION)
-            need = std::max(need, k::latent_attention_workspace_bytes(l.la, L.is_f32, rows, batch, n.max_new, cus));
-        else if (l.cfg.mixer == FA_MIXER_ATTENTION)
-            need = std::max(need, k::attention_workspace_bytes(l.at, L.is_f32, batch, n.min_new, n.max_new, L.cfg.max_blocks_per_seq * L.cfg.block_size, cus));
-    }
+    for (const Layer &l : L.layers)
+        for (const Mixer &m : l.mixers) {
+            if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION)
+                need = std::max(need, k::latent_attention_workspace_bytes(m.la, L.is_f32, rows, batch, n.max_new, cus));
+            else if (m.cfg.mixer == FA_MIXER_ATTENTION)
+                need = std::max(need, k::attention_workspace_bytes(m.at, L.is_f32, batch, n.min_new, n.max_new, L.cfg.max_blocks_per_seq * L.cfg.block_size, cus));
+        }
     return need ? ensure_workspace(ctx, need) : FA_OK;
 }
 
@@ -423,13 +555,14 @@ ExpandPlan plan_expand(const LayeredState &L, const std::vector<uint32_t> &lens,
     p.meta.assign(L.windows.size() * (2 * (size_t)max_batch + 1), 0);
     if (L.is_f32) return p;
     for (size_t w = 0; w < L.windows.size(); ++w) {
-        const Layer *l = nullptr;
+        const Mixer *l = nullptr;
         bool ok = true;
         for (const Layer &c : L.layers)
-            if (c.cfg.mixer == FA_MIXER_LATENT_ATTENTION && c.window_index == w) {
-                ok = ok && k::latent_expand_applies(c.la);
-                l = &c;
-            }
+            for (const Mixer &m : c.mixers)
+                if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION && m.window_index == w) {
+                    ok = ok && k::latent_expand_applies(m.la);
+                    l = &m;
+                }
         if (!l || !ok) continue;
         const uint64_t W = L.windows[w];
         uint64_t rows = 0, fresh = 0;
@@ -657,39 +790,71 @@ fa_status check_layered(const fa_decoder *d, const char *what) {
     return FA_OK;
 }
 
+// One mixer; alone: it is the only one of its layer.
+fa_status check_mixer(const fa_layered_config &c, const fa_layer_config &l, uint32_t i, bool alone) {
+    auto bad = [&](const char *why) { return fail(FA_ERR_INVALID_ARGUMENT, "layer " + std::to_string(i) + ": " + why); };
+    if (l.heads == 0 || l.dim == 0 || l.vdim == 0 || l.heads > 1024 || l.dim > 4096 || l.vdim > 4096) return bad("heads, dim and vdim must be positive");
+    if (l.mixer == FA_MIXER_DELTA || l.mixer == FA_MIXER_LIGHTNING) {
+        if (l.dim > k::kDeltaMaxDim || l.vdim > k::kDeltaMaxVdim) return fail(FA_ERR_UNSUPPORTED, "delta layer: dim above 256 or vdim above 1024");
+        if (c.state_slots == 0) return bad("a recurrent layer needs state slots");
+        if (l.mixer == FA_MIXER_LIGHTNING) {
+            if (!l.decay) return bad("lightning attention needs its decays");
+            for (uint32_t h = 0; h < l.heads; ++h)
+                if (!(l.decay[h] >= 0.0f && l.decay[h] <= 1.0f)) return bad("decays must be between 0 and 1");
+            return FA_OK;
+        }
+        if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
+        if (l.conv == 0 || l.conv > 16) return bad("the convolution takes 1 to 16 taps");
+        if ((l.decay_rank == 0) != (l.gate_rank == 0)) return bad("low-rank decays and gates go together");
+        if (l.decay_rank > 65536 || l.gate_rank > 65536) return bad("bad ranks");
+        return FA_OK;
+    }
+    if (!std::isfinite(l.scale)) return bad("bad scale");
+    if (l.mixer == FA_MIXER_LATENT_ATTENTION) {
+        if (l.q_rank == 0 || l.kv_rank == 0) return bad("q_rank and kv_rank must be positive");
+        if (l.rot_dim == 0 || l.rot_dim % 2 != 0) return bad("rot_dim must be positive and even");
+        if (l.kv_rank > 2048 || l.rot_dim > 1024) return fail(FA_ERR_UNSUPPORTED, "latent attention: kv_rank above 2048 or rot_dim above 1024");
+    } else if (l.mixer == FA_MIXER_ATTENTION) {
+        if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
+        const uint32_t per_head = FA_ATTENTION_HEAD_NORM | FA_ATTENTION_HEAD_UNIT, all = FA_ATTENTION_BIAS | FA_ATTENTION_QK_NORM | per_head |
+                                                                                        FA_ATTENTION_KEY_VALUES | FA_ATTENTION_GATE | FA_ATTENTION_SINK;
+        if (l.attention & ~all) return bad("unknown attention flags");
+        if ((l.attention & per_head) == per_head) return bad("one kind of norm per head");
+        const bool heads_form = (l.attention & (per_head | FA_ATTENTION_KEY_VALUES)) || l.rot_dim;
+        if (heads_form && (l.attention & FA_ATTENTION_QK_NORM)) return fail(FA_ERR_UNSUPPORTED, "attention: norms over all heads beside norms per head, keys as values or rotation");
+        if ((l.attention & FA_ATTENTION_BIAS) && (!alone || (l.attention & FA_ATTENTION_GATE))) return fail(FA_ERR_UNSUPPORTED, "attention: biases beside a gate or a second mixer");
+        if ((l.attention & FA_ATTENTION_KEY_VALUES) && l.vdim != l.dim) return bad("keys as values need vdim = dim");
+        if (l.rot_dim % 2 != 0 || l.rot_dim > l.dim) return bad("rot_dim must be even and at most dim");
+        if (heads_form && l.kv_from >= 0) return fail(FA_ERR_UNSUPPORTED, "attention: an earlier layer's cache beside norms per head, keys as values or rotation");
+    } else {
+        return bad("unknown mixer");
+    }
+    if (l.rot_dim && !(l.rot_base > 0.0)) return bad("bad rotation base");
+    if (l.rot_dim && l.rot_factor > 0.0 && !(std::isfinite(l.rot_factor) && l.rot_high > l.rot_low && l.rot_original > 0.0)) return bad("bad rotation scaling");
+    if (l.kv_from < 0) return FA_OK;
+    if (!alone) return fail(FA_ERR_UNSUPPORTED, "two mixers side by side: caches of their own only");
+    if ((uint32_t)l.kv_from >= i) return bad("kv_from must name an earlier layer");
+    const fa_layer_config &j = c.layers[l.kv_from];
+    if (j.right) return fail(FA_ERR_UNSUPPORTED, "kv_from names a layer of two mixers");
+    if (j.mixer != l.mixer || j.kv_from >= 0) return bad("kv_from must name an attention layer of the same kind with a cache of its own");
+    if (l.mixer == FA_MIXER_LATENT_ATTENTION) {
+        if (j.kv_rank != l.kv_rank || j.rot_interleaved != l.rot_interleaved || !(rotation_of(j) == rotation_of(l)))
+            return bad("kv_from: the two layers' latents or rotations differ");
+    } else {
+        if (j.kv_heads != l.kv_heads || j.dim != l.dim || j.vdim != l.vdim) return bad("kv_from: the two layers' key and value sizes differ");
+        if (j.rot_dim || (j.attention & (FA_ATTENTION_HEAD_NORM | FA_ATTENTION_HEAD_UNIT | FA_ATTENTION_KEY_VALUES)))
+            return fail(FA_ERR_UNSUPPORTED, "kv_from names a layer with norms per head, keys as values or rotation");
+    }
+    return FA_OK;
+}
+
 fa_status check_layer(const fa_layered_config &c, uint32_t i) {
     const fa_layer_config &l = c.layers[i];
     auto bad = [&](const char *why) { return fail(FA_ERR_INVALID_ARGUMENT, "layer " + std::to_string(i) + ": " + why); };
-    if (l.heads == 0 || l.dim == 0 || l.vdim == 0 || l.heads > 1024 || l.dim > 4096 || l.vdim > 4096) return bad("heads, dim and vdim must be positive");
-    if (l.mixer == FA_MIXER_DELTA) {
-        if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
-        if (l.conv == 0 || l.conv > 16) return bad("the convolution takes 1 to 16 taps");
-        if (l.dim > k::kDeltaMaxDim || l.vdim > k::kDeltaMaxVdim) return fail(FA_ERR_UNSUPPORTED, "delta layer: dim above 256 or vdim above 1024");
-        if (c.state_slots == 0) return bad("a recurrent layer needs state slots");
-    } else if (l.mixer == FA_MIXER_LATENT_ATTENTION) {
-        if (l.q_rank == 0 || l.kv_rank == 0) return bad("q_rank and kv_rank must be positive");
-        if (l.rot_dim == 0 || l.rot_dim % 2 != 0) return bad("rot_dim must be positive and even");
-        if (l.window == 0) return bad("the window must be positive");
-        if (!(l.rot_base > 0.0) || !std::isfinite(l.scale)) return bad("bad rotation base or scale");
-        if (l.kv_rank > 2048 || l.rot_dim > 1024) return fail(FA_ERR_UNSUPPORTED, "latent attention: kv_rank above 2048 or rot_dim above 1024");
-        if (l.kv_from >= 0) {
-            if ((uint32_t)l.kv_from >= i) return bad("kv_from must name an earlier layer");
-            const fa_layer_config &j = c.layers[l.kv_from];
-            if (j.mixer != FA_MIXER_LATENT_ATTENTION || j.kv_from >= 0) return bad("kv_from must name a latent attention layer with a cache of its own");
-            if (j.kv_rank != l.kv_rank || j.rot_dim != l.rot_dim || j.rot_base != l.rot_base) return bad("kv_from: the two layers' latents or rotations differ");
-        }
-    } else if (l.mixer == FA_MIXER_ATTENTION) {
-        if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
-        if (!std::isfinite(l.scale)) return bad("bad scale");
-        if (l.attention & ~(uint32_t)(FA_ATTENTION_BIAS | FA_ATTENTION_QK_NORM)) return bad("unknown attention flags");
-        if (l.kv_from >= 0) {
-            if ((uint32_t)l.kv_from >= i) return bad("kv_from must name an earlier layer");
-            const fa_layer_config &j = c.layers[l.kv_from];
-            if (j.mixer != FA_MIXER_ATTENTION || j.kv_from >= 0) return bad("kv_from must name an attention layer with a cache of its own");
-            if (j.kv_heads != l.kv_heads || j.dim != l.dim || j.vdim != l.vdim) return bad("kv_from: the two layers' key and value sizes differ");
-        }
-    } else {
-        return bad("unknown mixer");
+    if (fa_status s = check_mixer(c, l, i, !l.right)) return s;
+    if (l.right) {
+        if (fa_status s = check_mixer(c, *l.right, i, false)) return s;
+        if (!std::isfinite(l.left_scale) || !std::isfinite(l.right_scale)) return bad("bad scale of a mixer");
     }
     if (l.experts) {
         if (l.experts > k::kMaxExperts || l.top > k::kMaxTop) return fail(FA_ERR_UNSUPPORTED, "sparse experts: more than 256, or more than 64 of them per token");
@@ -697,7 +862,8 @@ fa_status check_layer(const fa_layered_config &c, uint32_t i) {
         if (c.norm != FA_NORM_OUTPUT) return fail(FA_ERR_UNSUPPORTED, "sparse experts: with norms at the sublayers' output only");
         return FA_OK;
     }
-    if (l.d_ffn && !(l.ffn_limit >= 0.0f && std::isfinite(l.ffn_alpha))) return bad("bad feed-forward constants");
+    if (l.glu != FA_GLU_CLAMPED && l.glu != FA_GLU_SILU) return bad("unknown gated linear unit");
+    if (l.d_ffn && l.glu == FA_GLU_CLAMPED && !(l.ffn_limit >= 0.0f && std::isfinite(l.ffn_alpha))) return bad("bad feed-forward constants");
     return FA_OK;
 }
 
@@ -715,9 +881,10 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
     if (c.d_model > 16384) return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: d_model above 16384");
     if (c.dtype != FA_BF16 && c.dtype != FA_F32) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: dtype must be bf16 or f32");
     if (!std::isfinite(c.norm_eps) || c.norm_eps < 0.0f || !std::isfinite(c.logit_softcap)) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad constants");
-    if ((c.norm != FA_NORM_INPUT && c.norm != FA_NORM_OUTPUT) || !std::isfinite(c.embed_scale) || !std::isfinite(c.position_base) || c.position_base < 0.0)
-        return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad norm, embed_scale or position_base");
-    if (c.norm == FA_NORM_INPUT && (c.position_base > 0.0 || (c.embed_scale != 0.0f && c.embed_scale != 1.0f)))
+    if (c.norm < FA_NORM_INPUT || c.norm > FA_NORM_BOTH || !std::isfinite(c.embed_scale) || !std::isfinite(c.position_base) || c.position_base < 0.0 ||
+        !std::isfinite(c.logit_scale))
+        return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad norm, embed_scale, position_base or logit_scale");
+    if (c.norm != FA_NORM_OUTPUT && (c.position_base > 0.0 || (c.embed_scale != 0.0f && c.embed_scale != 1.0f)))
         return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: scaled or positioned embeddings need norms at the sublayers' output");
     if (c.block_size == 0 || (c.block_size & (c.block_size - 1)) != 0 || c.block_size > 256 || c.num_blocks == 0)
         return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: block_size must be a power of two up to 256, num_blocks positive");
@@ -746,9 +913,9 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
     d->cfg.max_batch = c.max_batch;
     fa_status st = FA_OK;
     try {
-        L->layer_cfgs.assign(c.layers, c.layers + c.n_layers);
         L->cfg = c;
-        L->cfg.layers = L->layer_cfgs.data();
+        L->cfg.layers = nullptr;                             // the caller's; every layer keeps its own
+        if (L->cfg.logit_scale == 0.0f) L->cfg.logit_scale = 1.0f;
         if (L->cfg.embed_scale == 0.0f) L->cfg.embed_scale = 1.0f;
         L->is_f32 = c.dtype == FA_F32;
         L->esz = L->is_f32 ? 4 : 2;
@@ -783,9 +950,10 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             return w;
         };
         // whole linear [rows, cols] into output columns n0 ..
-        auto lin = [&](const std::string &name, uint32_t rows, uint32_t cols, const k::LinearWeight &w, uint32_t n0, uint32_t group = 0, uint32_t pitch = 0) {
+        auto lin = [&](const std::string &name, uint32_t rows, uint32_t cols, const k::LinearWeight &w, uint32_t n0, uint32_t group = 0, uint32_t pitch = 0,
+                       uint32_t k0 = 0) {
             add(name, rows, cols, [=](const void *src, int src_f32, hipStream_t s) {
-                k::pack_linear(src, src_f32, cols, 1, rows, cols, (void *)w.w, f32, w.k_tiles, n0, group ? group : 0x40000000u, pitch, s);
+                k::pack_linear(src, src_f32, cols, 1, rows, cols, (void *)w.w, f32, w.k_tiles, n0, group ? group : 0x40000000u, pitch, s, k0);
             });
         };
         auto row_ptr = [](const void *src, int src_f32, uint64_t elem) { return (const void *)((const uint8_t *)src + elem * (src_f32 ? 4 : 2)); };
@@ -807,142 +975,230 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             L->position_freq = (double *)own(FA_F32, 2 * freq.size());
             if (st == FA_OK) st = fa_upload_into(ctx, freq.data(), 2 * freq.size(), L->owned.back(), 0);
         }
-        const bool scaled = c.norm == FA_NORM_INPUT;         // sublayer outputs pass a layer scale
+        // what sublayer outputs pass on their way to the residual: a layer scale or a second norm
+        const char *post[3][2] = {{"ls1", "ls2"}, {nullptr, nullptr}, {"norm1b", "norm2b"}};
+        const uint32_t max_ctx = (uint32_t)std::min<uint64_t>((uint64_t)c.max_blocks_per_seq * c.block_size, k::kWholeContext);
+        auto rotation = [&](Mixer &m) {
+            const Rotation r = rotation_of(m.cfg);
+            m.rotation = (uint32_t)(std::find(L->rotations.begin(), L->rotations.end(), r) - L->rotations.begin());
+            if (m.rotation < L->rotations.size()) return;
+            L->rotations.push_back(r);
+            const std::vector<double> f = frequencies(r);
+            L->rotation_freq.push_back((double *)own(FA_F32, 2 * f.size()));
+            if (st == FA_OK) st = fa_upload_into(ctx, f.data(), 2 * f.size(), L->owned.back(), 0);
+        };
+        // How many columns of `in` a mixer takes, in its own order: first those kept in the activations' type, then the f32 ones.
+        auto measure = [&](Mixer &m) {
+            const fa_layer_config &g = m.cfg;
+            const uint32_t ow = m.out_width();
+            if (recurrent(g)) {
+                const bool lightning = g.mixer == FA_MIXER_LIGHTNING, low_rank = g.decay_rank && !lightning;
+                const k::Recurrence kind = lightning ? k::Recurrence::kLightning : low_rank ? k::Recurrence::kChannelDelta : k::Recurrence::kDelta;
+                m.de = k::DeltaShape{kind, g.heads, lightning ? g.heads : g.kv_heads, g.dim, g.vdim, lightning ? 0 : g.conv, lightning, lightning || low_rank, c.norm_eps};
+                m.gate_at = m.de.qkv();
+                m.rank_at = pad_to(m.de.qkv(), 8);
+                m.lo = low_rank ? m.rank_at + pad_to(g.decay_rank, 8) + g.gate_rank : m.gate_at + ow;
+                m.hi = lightning ? 0 : low_rank ? g.heads : 2 * g.heads;
+            } else if (g.mixer == FA_MIXER_ATTENTION) {
+                const bool own_kv = g.kv_from < 0;
+                m.hi = g.heads * g.dim + (own_kv ? g.kv_heads * g.dim + (g.attention & FA_ATTENTION_KEY_VALUES ? 0 : g.kv_heads * g.vdim) : 0);
+                m.lo = g.attention & FA_ATTENTION_GATE ? ow : 0;
+            } else {
+                m.hi = g.q_rank + (g.kv_from < 0 ? g.kv_rank + g.rot_dim : 0) + (g.ungated ? 0 : g.heads);
+            }
+        };
+        auto set_recurrence = [&](Mixer &m, const Layer &l) {
+            const fa_layer_config &g = m.cfg;
+            const uint32_t H = g.heads, ow = m.out_width(), nq = m.de.kv_heads * g.dim, ch = m.de.qkv(), lo = m.lo_at, hi = l.lo + m.hi_at;
+            L->has_state = true;
+            lin(m.prefix + "q", nq, D, l.in, lo);
+            lin(m.prefix + "k", nq, D, l.in, lo + nq);
+            lin(m.prefix + "v", ow, D, l.in, lo + 2 * nq);
+            const uint32_t n_norm = m.de.norm_all ? ow : g.vdim;
+            m.head_norm = (float *)own(FA_F32, n_norm);
+            vec(m.prefix + "norm", n_norm, 0, m.head_norm);
+            m.state = (float *)own(FA_F32, (uint64_t)c.state_slots * H * g.dim * m.de.vdim_p());
+            if (m.de.kind == k::Recurrence::kLightning) {
+                lin(m.prefix + "g", ow, D, l.in, lo + m.gate_at);
+                m.decay = (float *)own(FA_F32, H);
+                if (st == FA_OK) st = fa_upload_into(ctx, g.decay, H, L->owned.back(), 0);
+                return;
+            }
+            lin(m.prefix + "b", H, D, l.in, hi);
+            m.conv = (float *)own(FA_F32, (uint64_t)ch * g.conv);
+            vec(m.prefix + "q.conv", nq, g.conv, m.conv);
+            vec(m.prefix + "k.conv", nq, g.conv, m.conv + (uint64_t)nq * g.conv);
+            vec(m.prefix + "v.conv", ow, g.conv, m.conv + 2ull * nq * g.conv);
+            m.ring = own(f32 ? FA_F32 : FA_BF16, (uint64_t)c.state_slots * g.conv * ch);
+            const uint32_t n_decay = g.decay_rank ? H * g.dim : H;
+            m.a_log = (float *)own(FA_F32, H);
+            m.dt_bias = (float *)own(FA_F32, n_decay);
+            vec(m.prefix + "A_log", H, 0, m.a_log);
+            vec(m.prefix + "dt_bias", n_decay, 0, m.dt_bias);
+            if (g.decay_rank) {
+                const uint32_t gate_k = pad_to(g.decay_rank, 8), decay_n = pad_to(ow, 8);
+                m.low_rank = weight(decay_n + n_decay, decay_n + n_decay, gate_k + g.gate_rank);
+                lin(m.prefix + "a1", g.decay_rank, D, l.in, lo + m.rank_at);
+                lin(m.prefix + "g1", g.gate_rank, D, l.in, lo + m.rank_at + gate_k);
+                lin(m.prefix + "a2", n_decay, g.decay_rank, m.low_rank, decay_n);
+                lin(m.prefix + "g2", ow, g.gate_rank, m.low_rank, 0, 0, 0, gate_k);
+            } else {
+                lin(m.prefix + "g", ow, D, l.in, lo + m.gate_at);
+                lin(m.prefix + "a", H, D, l.in, hi + H);
+            }
+        };
+        auto set_attention = [&](Mixer &m, Layer &l) {
+            const fa_layer_config &g = m.cfg;
+            const uint32_t H = g.heads, hi = l.lo + m.hi_at;
+            k::AttentionShape &a = m.at;
+            a = k::AttentionShape{H, g.kv_heads, g.dim, g.vdim, 0, 0, g.scale, c.norm_eps, (uint64_t)c.num_blocks * c.block_size,
+                                  g.window ? std::min(g.window, k::kWholeContext) : k::kWholeContext, g.rot_dim, g.rot_interleaved ? 1u : 0u};
+            k::attention_pad(a);
+            const bool own_kv = g.kv_from < 0, bias = g.attention & FA_ATTENTION_BIAS, norms = g.attention & FA_ATTENTION_QK_NORM;
+            const uint32_t nq = H * g.dim, nk = own_kv ? g.kv_heads * g.dim : 0, nv = m.hi - nq - nk;
+            if (bias) l.in_bias = (float *)own(FA_F32, pad_to(nq + nk + nv, 4));
+            const std::pair<const char *, std::pair<uint32_t, uint32_t>> parts[3] = {{"q", {0, nq}}, {"k", {nq, nk}}, {"v", {nq + nk, nv}}};
+            for (const auto &[name, at] : parts) {
+                if (at.second == 0) continue;
+                lin(m.prefix + name, at.second, D, l.in, hi + at.first);
+                if (bias) vec(m.prefix + name + ".b", at.second, 0, l.in_bias + at.first);
+            }
+            auto norm = [&](const char *name, uint32_t n) {
+                float *p = (float *)own(FA_F32, n);
+                vec(m.prefix + name, n, 0, p);
+                return p;
+            };
+            if (norms) m.q_norm = norm("q.norm", nq);
+            if (norms && own_kv) m.k_norm = norm("k.norm", nk);
+            if (g.attention & FA_ATTENTION_HEAD_NORM) {
+                m.q_norm = norm("q.norm", g.dim);
+                m.k_norm = norm("k.norm", g.dim);
+            }
+            if (g.attention & FA_ATTENTION_SINK) m.sink = norm("sink", H);
+            if (g.attention & FA_ATTENTION_GATE) lin(m.prefix + "g", m.out_width(), D, l.in, m.lo_at + m.gate_at);
+            if (g.rot_dim) rotation(m);
+            if (own_kv) {
+                m.k_pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * g.kv_heads * a.dim_p);
+                m.v_pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * g.kv_heads * a.v_p);
+            }
+        };
+        auto set_latent = [&](Mixer &m, const Layer &l) {
+            const fa_layer_config &g = m.cfg;
+            const uint32_t H = g.heads, hi = l.lo + m.hi_at;
+            k::LatentShape &a = m.la;
+            a.heads = H;
+            a.dim = g.dim;
+            a.rot = g.rot_dim;
+            a.vdim = g.vdim;
+            a.q_rank = g.q_rank;
+            a.kv_rank = g.kv_rank;
+            k::latent_pad(a);
+            a.window = g.window ? std::min(g.window, max_ctx) : max_ctx;
+            a.interleaved = g.rot_interleaved ? 1 : 0;
+            a.scale = g.scale;
+            a.eps = c.norm_eps;
+            a.pool_rows = (uint64_t)c.num_blocks * c.block_size;
+            const bool own_kv = g.kv_from < 0;
+            const uint32_t kvn = own_kv ? g.kv_rank + g.rot_dim : 0;
+            lin(m.prefix + "dq", g.q_rank, D, l.in, hi);
+            m.q_norm = (float *)own(FA_F32, g.q_rank);
+            vec(m.prefix + "dq.norm", g.q_rank, 0, m.q_norm);
+            if (own_kv) {
+                lin(m.prefix + "dkv", kvn, D, l.in, hi + g.q_rank);
+                m.kv_norm = (float *)own(FA_F32, g.kv_rank);
+                vec(m.prefix + "dkv.norm", g.kv_rank, 0, m.kv_norm);
+                m.pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * (a.rank_p + a.rot_p));
+            }
+            if (!g.ungated) lin(m.prefix + "g", H, D, l.in, hi + g.q_rank + kvn);
+            // queries: per head [dim padded][rot padded]
+            const uint32_t qw = a.dim_p + a.rot_p, hd = g.dim + g.rot_dim, qr = g.q_rank, dim = g.dim, rot = g.rot_dim, dim_p = a.dim_p;
+            m.uq = weight(H * qw, H * qw, qr);
+            {
+                const k::LinearWeight w = m.uq;
+                add(m.prefix + "uq", (uint64_t)H * hd, qr, [=](const void *src, int sf, hipStream_t s) {
+                    for (uint32_t h = 0; h < H; ++h) {
+                        k::pack_linear(row_ptr(src, sf, (uint64_t)h * hd * qr), sf, qr, 1, dim, qr, (void *)w.w, f32, w.k_tiles, h * qw, 0x40000000u, 0, s);
+                        k::pack_linear(row_ptr(src, sf, ((uint64_t)h * hd + dim) * qr), sf, qr, 1, rot, qr, (void *)w.w, f32, w.k_tiles, h * qw + dim_p, 0x40000000u, 0, s);
+                    }
+                });
+            }
+            // per head, latent = W_uk^T q: the key projection transposed
+            const uint32_t kr = g.kv_rank, vd = g.vdim;
+            const uint32_t hw = dim_p + a.v_p;
+            if (!f32) m.ukv = weight(H * hw, H * hw, kr);
+            const k::LinearWeight both = m.ukv;
+            m.uk = weight(a.rank_p, a.rank_p, dim, H);
+            {
+                const k::LinearWeight w = m.uk;
+                const uint64_t one = (uint64_t)w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
+                add(m.prefix + "uk", (uint64_t)H * dim, kr, [=](const void *src, int sf, hipStream_t s) {
+                    for (uint32_t h = 0; h < H; ++h)
+                        k::pack_linear(row_ptr(src, sf, (uint64_t)h * dim * kr), sf, 1, kr, kr, dim, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
+                    if (both.w) k::pack_linear(src, sf, kr, 1, H * dim, kr, (void *)both.w, f32, both.k_tiles, 0, dim, hw, s);
+                });
+            }
+            m.uv = weight(vd, vd, kr, H);
+            {
+                const k::LinearWeight w = m.uv;
+                const uint64_t one = (uint64_t)w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
+                add(m.prefix + "uv", (uint64_t)H * vd, kr, [=](const void *src, int sf, hipStream_t s) {
+                    for (uint32_t h = 0; h < H; ++h)
+                        k::pack_linear(row_ptr(src, sf, (uint64_t)h * vd * kr), sf, kr, 1, vd, kr, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
+                    if (both.w) k::pack_linear(src, sf, kr, 1, H * vd, kr, (void *)both.w, f32, both.k_tiles, dim_p, vd, hw, s);
+                });
+            }
+            m.window_index = (uint32_t)(std::find(L->windows.begin(), L->windows.end(), a.window) - L->windows.begin());
+            if (m.window_index == L->windows.size()) L->windows.push_back(a.window);
+            rotation(m);
+        };
         L->layers.resize(c.n_layers);
         for (uint32_t i = 0; i < c.n_layers; ++i) {
             Layer &l = L->layers[i];
             l.cfg = c.layers[i];
-            const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.", f = p + "mlp.";
-            const fa_layer_config &g = l.cfg;
-            const uint32_t H = g.heads, ow = H * g.vdim;
+            const std::string p = "l" + std::to_string(i) + ".", f = p + "mlp.";
+            const fa_layer_config g = l.cfg;
             l.norm1 = (float *)own(FA_F32, D);
             vec(p + "norm1", D, 0, l.norm1);
-            if (scaled) {
-                l.ls1 = (float *)own(FA_F32, D);
-                vec(p + "ls1", D, 0, l.ls1);
+            if (post[c.norm][0]) {
+                l.post1 = (float *)own(FA_F32, D);
+                vec(p + post[c.norm][0], D, 0, l.post1);
             }
-            if (g.mixer == FA_MIXER_DELTA) {
-                L->has_state = true;
-                l.de = k::DeltaShape{H, g.kv_heads, g.dim, g.vdim, g.conv, c.norm_eps};
-                const uint32_t nq = g.kv_heads * g.dim, ch = l.de.qkv();
-                l.in = weight(ch + ow + 2 * H, ch + ow + 2 * H, D);
-                lin(m + "q", nq, D, l.in, 0);
-                lin(m + "k", nq, D, l.in, nq);
-                lin(m + "v", ow, D, l.in, 2 * nq);
-                lin(m + "g", ow, D, l.in, ch);
-                lin(m + "b", H, D, l.in, ch + ow);
-                lin(m + "a", H, D, l.in, ch + ow + H);
-                l.conv = (float *)own(FA_F32, (uint64_t)ch * g.conv);
-                vec(m + "q.conv", nq, g.conv, l.conv);
-                vec(m + "k.conv", nq, g.conv, l.conv + (uint64_t)nq * g.conv);
-                vec(m + "v.conv", ow, g.conv, l.conv + 2ull * nq * g.conv);
-                l.a_log = (float *)own(FA_F32, H);
-                l.dt_bias = (float *)own(FA_F32, H);
-                l.head_norm = (float *)own(FA_F32, g.vdim);
-                vec(m + "A_log", H, 0, l.a_log);
-                vec(m + "dt_bias", H, 0, l.dt_bias);
-                vec(m + "norm", g.vdim, 0, l.head_norm);
-                l.state = (float *)own(FA_F32, (uint64_t)c.state_slots * H * g.dim * l.de.vdim_p());
-                l.ring = own(f32 ? FA_F32 : FA_BF16, (uint64_t)c.state_slots * g.conv * ch);
-            } else if (g.mixer == FA_MIXER_ATTENTION) {
-                k::AttentionShape &a = l.at;
-                a = k::AttentionShape{H, g.kv_heads, g.dim, g.vdim, 0, 0, g.scale, c.norm_eps, (uint64_t)c.num_blocks * c.block_size};
-                k::attention_pad(a);
-                const bool own_kv = g.kv_from < 0, bias = g.attention & FA_ATTENTION_BIAS, norms = g.attention & FA_ATTENTION_QK_NORM;
-                const uint32_t nq = H * g.dim, nk = own_kv ? g.kv_heads * g.dim : 0, nv = own_kv ? g.kv_heads * g.vdim : 0;
-                l.in = weight(nq + nk + nv, nq + nk + nv, D);
-                if (bias) l.in_bias = (float *)own(FA_F32, pad_to(nq + nk + nv, 4));
-                if (norms) l.q_norm = (float *)own(FA_F32, nq);
-                if (norms && own_kv) l.k_norm = (float *)own(FA_F32, nk);
-                const std::pair<const char *, std::pair<uint32_t, uint32_t>> parts[3] = {{"q", {0, nq}}, {"k", {nq, nk}}, {"v", {nq + nk, nv}}};
-                for (const auto &[name, at] : parts) {
-                    if (at.second == 0) continue;
-                    lin(m + name, at.second, D, l.in, at.first);
-                    if (bias) vec(m + name + ".b", at.second, 0, l.in_bias + at.first);
-                }
-                if (l.q_norm) vec(m + "q.norm", nq, 0, l.q_norm);
-                if (l.k_norm) vec(m + "k.norm", nk, 0, l.k_norm);
-                if (own_kv) {
-                    l.k_pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * g.kv_heads * a.dim_p);
-                    l.v_pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * g.kv_heads * a.v_p);
-                }
-            } else {
-                k::LatentShape &a = l.la;
-                a.heads = H;
-                a.dim = g.dim;
-                a.rot = g.rot_dim;
-                a.vdim = g.vdim;
-                a.q_rank = g.q_rank;
-                a.kv_rank = g.kv_rank;
-                k::latent_pad(a);
-                a.window = g.window;
-                a.scale = g.scale;
-                a.eps = c.norm_eps;
-                a.pool_rows = (uint64_t)c.num_blocks * c.block_size;
-                const bool own_kv = g.kv_from < 0;
-                const uint32_t kvn = own_kv ? g.kv_rank + g.rot_dim : 0;
-                l.in = weight(g.q_rank + kvn + H, g.q_rank + kvn + H, D);
-                lin(m + "dq", g.q_rank, D, l.in, 0);
-                l.q_norm = (float *)own(FA_F32, g.q_rank);
-                vec(m + "dq.norm", g.q_rank, 0, l.q_norm);
-                if (own_kv) {
-                    lin(m + "dkv", kvn, D, l.in, g.q_rank);
-                    l.kv_norm = (float *)own(FA_F32, g.kv_rank);
-                    vec(m + "dkv.norm", g.kv_rank, 0, l.kv_norm);
-                    l.pool = own(f32 ? FA_F32 : FA_BF16, a.pool_rows * (a.rank_p + a.rot_p));
-                }
-                lin(m + "g", H, D, l.in, g.q_rank + kvn);
-                // queries: per head [dim padded][rot padded]
-                const uint32_t qw = a.dim_p + a.rot_p, hd = g.dim + g.rot_dim, qr = g.q_rank, dim = g.dim, rot = g.rot_dim, dim_p = a.dim_p;
-                l.uq = weight(H * qw, H * qw, qr);
-                {
-                    const k::LinearWeight w = l.uq;
-                    add(m + "uq", (uint64_t)H * hd, qr, [=](const void *src, int sf, hipStream_t s) {
-                        for (uint32_t h = 0; h < H; ++h) {
-                            k::pack_linear(row_ptr(src, sf, (uint64_t)h * hd * qr), sf, qr, 1, dim, qr, (void *)w.w, f32, w.k_tiles, h * qw, 0x40000000u, 0, s);
-                            k::pack_linear(row_ptr(src, sf, ((uint64_t)h * hd + dim) * qr), sf, qr, 1, rot, qr, (void *)w.w, f32, w.k_tiles, h * qw + dim_p, 0x40000000u, 0, s);
-                        }
-                    });
-                }
-                // per head, latent = W_uk^T q: the key projection transposed
-                const uint32_t kr = g.kv_rank, vd = g.vdim;
-                const uint32_t hw = dim_p + a.v_p;
-                if (!f32) l.ukv = weight(H * hw, H * hw, kr);
-                const k::LinearWeight both = l.ukv;
-                l.uk = weight(a.rank_p, a.rank_p, dim, H);
-                {
-                    const k::LinearWeight w = l.uk;
-                    const uint64_t one = (uint64_t)w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
-                    add(m + "uk", (uint64_t)H * dim, kr, [=](const void *src, int sf, hipStream_t s) {
-                        for (uint32_t h = 0; h < H; ++h)
-                            k::pack_linear(row_ptr(src, sf, (uint64_t)h * dim * kr), sf, 1, kr, kr, dim, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
-                        if (both.w) k::pack_linear(src, sf, kr, 1, H * dim, kr, (void *)both.w, f32, both.k_tiles, 0, dim, hw, s);
-                    });
-                }
-                l.uv = weight(vd, vd, kr, H);
-                {
-                    const k::LinearWeight w = l.uv;
-                    const uint64_t one = (uint64_t)w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
-                    add(m + "uv", (uint64_t)H * vd, kr, [=](const void *src, int sf, hipStream_t s) {
-                        for (uint32_t h = 0; h < H; ++h)
-                            k::pack_linear(row_ptr(src, sf, (uint64_t)h * vd * kr), sf, kr, 1, vd, kr, (uint8_t *)w.w + h * one, f32, w.k_tiles, 0, 0x40000000u, 0, s);
-                        if (both.w) k::pack_linear(src, sf, kr, 1, H * vd, kr, (void *)both.w, f32, both.k_tiles, dim_p, vd, hw, s);
-                    });
-                }
-                l.window_index = (uint32_t)(std::find(L->windows.begin(), L->windows.end(), g.window) - L->windows.begin());
-                if (l.window_index == L->windows.size()) L->windows.push_back(g.window);
-                const std::pair<uint32_t, double> r(g.rot_dim, g.rot_base);
-                l.rotation = (uint32_t)(std::find(L->rotations.begin(), L->rotations.end(), r) - L->rotations.begin());
-                if (l.rotation == L->rotations.size()) L->rotations.push_back(r);
+            l.mixers.resize(g.right ? 2 : 1);
+            l.mixers[0].cfg = g;
+            l.mixers[0].prefix = p + (g.right ? "mix.left." : "mix.");
+            if (g.right) {
+                l.mixers[0].out_scale = g.left_scale;
+                l.mixers[1].out_scale = g.right_scale;
+                l.mixers[1].cfg = *g.right;
+                l.mixers[1].prefix = p + "mix.right.";
             }
-            l.out = weight(D, D, ow);
-            lin(m + "o", D, ow, l.out, 0);
+            for (Mixer &m : l.mixers) {
+                measure(m);
+                m.lo_at = l.lo;
+                m.hi_at = l.hi;
+                m.o_at = l.o_width = pad_to(l.o_width, 8);
+                l.lo = pad_to(l.lo + m.lo, 8);
+                l.hi = pad_to(l.hi + m.hi, &m == &l.mixers.back() ? 1 : 4);
+                l.o_width += m.out_width();
+            }
+            l.in = weight(l.lo + l.hi, l.lo + l.hi, D);
+            l.out = weight(D, D, l.o_width);
+            for (Mixer &m : l.mixers) {
+                if (recurrent(m.cfg)) set_recurrence(m, l);
+                else if (m.cfg.mixer == FA_MIXER_ATTENTION) set_attention(m, l);
+                else set_latent(m, l);
+                lin(m.prefix + "o", D, m.out_width(), l.out, 0, 0, 0, m.o_at);
+                m.cfg.right = nullptr;                       // the caller's
+                m.cfg.decay = nullptr;
+            }
+            l.cfg.right = nullptr;
+            l.cfg.decay = nullptr;
             if (g.d_ffn) {
                 l.norm2 = (float *)own(FA_F32, D);
                 vec(p + "norm2", D, 0, l.norm2);
-                if (scaled) {
-                    l.ls2 = (float *)own(FA_F32, D);
-                    vec(p + "ls2", D, 0, l.ls2);
+                if (post[c.norm][1]) {
+                    l.post2 = (float *)own(FA_F32, D);
+                    vec(p + post[c.norm][1], D, 0, l.post2);
                 }
             }
             if (g.experts) {

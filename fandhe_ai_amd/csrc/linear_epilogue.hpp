@@ -15,17 +15,25 @@ __device__ __forceinline__ float epilogue_value(const LinearEpilogue &ep, uint32
     if constexpr (MODE == LinearEpilogue::kGlu) {
         const float g = fminf(y, ep.limit), u = fminf(fmaxf(up, -ep.limit), ep.limit);
         return g * sigmoid_f32(ep.alpha * g) * (u + 1.0f);
+    } else if constexpr (MODE == LinearEpilogue::kSiluGlu) {
+        return y * sigmoid_f32(y) * up;
     } else if constexpr (MODE == LinearEpilogue::kSoftcap) {
+        y *= ep.factor;
         return ep.cap > 0.0f ? ep.cap * tanhf(y / ep.cap) : y;
     } else if constexpr (MODE == LinearEpilogue::kHeadGate) {
-        return y * sigmoid_f32(ep.gate[(uint64_t)row * ep.ld_gate + batch]);
+        return y * ep.factor * sigmoid_f32(ep.gate[(uint64_t)row * ep.ld_gate + batch]);
     } else if constexpr (MODE == LinearEpilogue::kSquaredRelu) {
         const float r = fmaxf(y, 0.0f);
         return r * r;
+    } else if constexpr (MODE == LinearEpilogue::kStore) {
+        return y * ep.factor;
     } else {
         return y;
     }
 }
+
+// Modes whose column tiles alternate gate and up
+constexpr bool is_glu(int mode) { return mode == LinearEpilogue::kGlu || mode == LinearEpilogue::kSiluGlu; }
 
 template <int MODE>
 __device__ __forceinline__ void epilogue_store1(const LinearEpilogue &ep, uint32_t row, uint32_t col, uint32_t batch, float y, float up) {
@@ -51,6 +59,10 @@ __device__ __forceinline__ void epilogue_store4(const LinearEpilogue &ep, uint32
                                                 dev::v4f y, dev::v4f up) {
     const uint64_t o = batch * ep.out_batch + (uint64_t)row * ep.ld_out + col;
     const bool whole = col + 4 <= n && ((ep.ld_out | ep.out_batch) & 3) == 0 && (MODE != LinearEpilogue::kStore || col + 4 <= ep.n_lo);
+    if (MODE == LinearEpilogue::kStore && col >= ep.n_lo && col + 4 <= n && ((ep.n_lo | ep.ld_hi) & 3) == 0 && !ep.bias) {
+        *(dev::v4f *)(ep.out_hi + (uint64_t)row * ep.ld_hi + (col - ep.n_lo)) = y * ep.factor;
+        return;
+    }
     if (!whole) {
 #pragma unroll
         for (int e = 0; e < 4; ++e)

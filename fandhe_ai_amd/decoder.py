@@ -145,26 +145,36 @@ class Decoder:
 
 class LayeredDecoder(Decoder):
     """A decoder whose layers are described one by one (``fa_decoder_create_layered``): unquantized weights in bf16 or
-    f32, per layer a gated delta rule with a recurrent state or attention (latent or grouped-query) over the paged cache,
-    and an optional feed-forward, dense or of sparse experts.  Sequences, steps, prompt passes and sampling are
-    ``Decoder``'s."""
+    f32, per layer one mixer or two side by side (gated delta rule or lightning attention with a recurrent state, attention,
+    latent or grouped-query, over the paged cache), and an optional feed-forward, dense or of sparse experts.  Sequences,
+    steps, prompt passes and sampling are ``Decoder``'s."""
 
     takes_portions = True
 
     def __init__(self, ops, d_model, vocab, layers, norm_eps, logit_softcap, max_blocks_per_seq, num_blocks, max_batch,
-                 state_slots=None, dtype=capi.BF16, block_size=16, norm=capi.NORM_INPUT, embed_scale=1.0, position_base=0.0):
-        """layers: one dict of ``capi.LayerConfig`` fields per layer."""
+                 state_slots=None, dtype=capi.BF16, block_size=16, norm=capi.NORM_INPUT, embed_scale=1.0, position_base=0.0,
+                 logit_scale=1.0):
+        """layers: one dict of ``capi.LayerConfig`` fields per layer (``right``: such a dict, ``decay``: a list)."""
         self._ops = ops
-        rows = (capi.LayerConfig * len(layers))(*[capi.LayerConfig(**l) for l in layers])
-        recurrent = any(l["mixer"] == capi.MIXER_DELTA for l in layers)
+        rows = (capi.LayerConfig * len(layers))(*[self._layer(l) for l in layers])
+        recurrent = any(m["mixer"] in (capi.MIXER_DELTA, capi.MIXER_LIGHTNING) for l in layers for m in (l, l.get("right") or l))
         slots = max_batch if state_slots is None else state_slots
         self.cfg = capi.LayeredConfig(len(layers), d_model, vocab, block_size, max_blocks_per_seq, num_blocks, max_batch,
-                                      slots, norm_eps, logit_softcap, dtype, rows, norm, embed_scale, position_base)
+                                      slots, norm_eps, logit_softcap, dtype, rows, norm, embed_scale, position_base, logit_scale)
         self.state_slots = slots if recurrent else 0
         self._h = C.c_void_p()
         check(lib.fa_decoder_create_layered(ops._ctx, C.byref(self.cfg), C.byref(self._h)))
         self._keep = []
         self.batch = 0
+
+    @classmethod
+    def _layer(cls, fields):
+        f = dict(fields)
+        if f.get("decay") is not None:
+            f["decay"] = (C.c_float * len(f["decay"]))(*f["decay"])
+        if f.get("right") is not None:
+            f["right"] = C.pointer(cls._layer(f["right"]))
+        return capi.LayerConfig(**f)
 
     def tensors(self):
         """name -> shape of every weight tensor the decoder takes."""

@@ -6,6 +6,7 @@ what the decoder runs on (pages, rows, state slots) is the caller's ``Capacity``
 """
 import json
 import os
+import re
 
 from . import capi
 from . import safetensors_io as st
@@ -152,22 +153,101 @@ def zoferax(config):
             "embed_scale": _entry(_entry(config, "embedding", CONFIG_FILE), "scale", "embedding"), "position_base": POSITION_BASE}
 
 
-# designs made of described layers: architecture name -> function(config) -> LayeredDecoder arguments
-LAYERED = {"Nugelix": nugelix, "Zoferax": zoferax}
+# ---- Bubetar: attention beside a recurrence, latent attention; sublayers normed on both sides ---------------------
+
+def _rotation(mx, where, interleaved):
+    """The rotation of a mixer's queries and keys as ``capi.LayerConfig`` fields."""
+    rot = _entry(mx, "rot", where)
+    out = {"rot_dim": _entry(rot, "dims", where + " rot"), "rot_base": _entry(rot, "base", where + " rot"), "rot_interleaved": int(interleaved)}
+    if rot.get("scaling"):
+        for key in ("factor", "low", "high", "original"):
+            out["rot_" + key] = _entry(rot["scaling"], key, where + " rot scaling")
+    return out
 
 
-def build_layered(ops, config, dtype, capacity):
-    """The layered decoder a configuration describes, without weights."""
+def _attention(mx, where, flags, interleaved):
+    l = {key: _entry(mx, key, where) for key in ("heads", "kv_heads", "dim", "vdim", "scale")}
+    l.update(_rotation(mx, where, interleaved), mixer=capi.MIXER_ATTENTION, attention=flags, kv_from=-1)
+    if mx.get("mask"):
+        l["window"] = _entry(mx["mask"], "size", where + " mask")
+    return l
+
+
+def _lightning(mx, where):
+    l = {key: _entry(mx, key, where) for key in ("heads", "dim", "vdim", "decay")}
+    if len(l["decay"]) != l["heads"]:
+        raise ConfigError("%s: one decay per head" % where)
+    return dict(l, mixer=capi.MIXER_LIGHTNING, kv_from=-1)
+
+
+def _channel_delta(mx, where, prefix, shapes):
+    """The ranks of the decays' and gates' projections are their weights' own."""
+    l = {key: _entry(mx, key, where) for key in ("heads", "kv_heads", "dim", "vdim", "conv")}
+    for field, name in (("decay_rank", prefix + "a1"), ("gate_rank", prefix + "g1")):
+        if name not in shapes:
+            raise ConfigError("%s: tensor %s is missing" % (where, name))
+        l[field] = shapes[name][0]
+    return dict(l, mixer=capi.MIXER_DELTA, kv_from=-1)
+
+
+def bubetar_layers(config, shapes):
+    """config.json's layer list as ``capi.LayerConfig`` fields; shapes: of the weights."""
+    out = []
+    for i, layer in enumerate(_entry(config, "layers", CONFIG_FILE)):
+        where = "layer %d" % i
+        kind, mx = _entry(layer, "type", where), _entry(layer, "mixer", where)
+        at = where + " mixer"
+        if kind in ("parallel", "parallel_2"):
+            left, right = _entry(mx, "left", at), _entry(mx, "right", at)
+            if kind == "parallel":
+                l = _attention(left, at + " left", capi.ATTENTION_HEAD_NORM | capi.ATTENTION_GATE, True)
+                r = _lightning(right, at + " right")
+            else:
+                l = _attention(left, at + " left", capi.ATTENTION_HEAD_UNIT | capi.ATTENTION_KEY_VALUES | capi.ATTENTION_SINK, False)
+                r = _channel_delta(right, at + " right", "l%d.mix.right." % i, shapes)
+            l.update(right=r, left_scale=_entry(mx, "left_scale", at), right_scale=_entry(mx, "right_scale", at))
+        elif kind == "latent_attention":
+            l = {key: _entry(mx, key, at) for key in ("heads", "dim", "vdim", "q_rank", "kv_rank", "scale")}
+            l.update(_rotation(mx, at, True), mixer=capi.MIXER_LATENT_ATTENTION, ungated=1, kv_from=-1)
+            if l["rot_dim"] != _entry(mx, "rot_dim", at):
+                raise ConfigError("%s: all of the rotated part is rotated, rot.dims must equal rot_dim" % at)
+        else:
+            raise ConfigError("%s: unknown type %r" % (where, kind))
+        mlp = layer.get("mlp")
+        if mlp is not None:
+            if _entry(mlp, "kind", where + " mlp") != "dense":
+                raise ConfigError("%s: unknown feed-forward %r" % (where, mlp["kind"]))
+            l.update(d_ffn=_entry(mlp, "ff", where + " mlp"), glu=capi.GLU_SILU)
+        out.append(l)
+    return out
+
+
+def bubetar(config, shapes):
+    """A Bubetar configuration as ``LayeredDecoder`` arguments."""
+    scale = config.get("logit_scale")
+    return {"d_model": _entry(config, "width", CONFIG_FILE), "vocab": _entry(config, "vocab", CONFIG_FILE), "layers": bubetar_layers(config, shapes),
+            "norm_eps": _entry(_entry(config, "norm", CONFIG_FILE), "eps", "norm"), "norm": capi.NORM_BOTH,
+            "logit_softcap": config.get("logit_softcap") or 0.0, "logit_scale": 1.0 if scale is None else scale}
+
+
+# designs made of described layers: architecture name -> function(config, shapes of the weights) -> LayeredDecoder arguments
+LAYERED = {"Nugelix": lambda config, shapes: nugelix(config), "Zoferax": lambda config, shapes: zoferax(config), "Bubetar": bubetar}
+
+
+def build_layered(ops, config, dtype, capacity, shapes=None):
+    """The layered decoder a configuration describes, without weights.  shapes: tensor name -> shape, for designs some of whose
+    sizes only the weights tell."""
     return LayeredDecoder(ops, max_blocks_per_seq=capacity.num_blocks, num_blocks=capacity.num_blocks, max_batch=capacity.max_batch,
                           state_slots=capacity.state_slots, dtype=DTYPES[dtype], block_size=capacity.block_size,
-                          **LAYERED[architecture_of(config)](config))
+                          **LAYERED[architecture_of(config)](config, shapes or {}))
 
 
 def install_weights(decoder, typed):
-    """name -> ``safetensors_io.TypedTensor`` into a layered decoder: every tensor it takes, none it does not."""
+    """name -> ``safetensors_io.TypedTensor`` into a layered decoder: every tensor it takes, none it does not (norms of a
+    feed-forward that a layer has not are passed over)."""
     wanted = decoder.tensors()
     st.require_keys(typed, sorted(wanted))
-    extra = sorted(set(typed) - set(wanted))
+    extra = sorted(n for n in set(typed) - set(wanted) if not re.fullmatch(r"l\d+\.norm2b?", n))
     if extra:
         raise ConfigError("tensors the configuration has no use for: %s" % ", ".join(extra))
     for name, shape in wanted.items():
@@ -182,9 +262,10 @@ def install_weights(decoder, typed):
 
 @register("Nugelix")
 @register("Zoferax")
+@register("Bubetar")
 def _layered(ops, config, weights, dtype, capacity):
     typed = st.load_safetensors_typed(weights)
-    decoder = build_layered(ops, config, dtype, capacity)
+    decoder = build_layered(ops, config, dtype, capacity, {n: t.shape for n, t in typed.items()})
     try:
         install_weights(decoder, typed)
     except Exception:

@@ -564,30 +564,52 @@ fa_status fa_decoder_read_seq_lens(fa_context *ctx, fa_decoder *dec, uint32_t *s
 fa_status fa_decoder_logits_buffer(fa_decoder *dec, fa_buffer **out);
 
 /* -------------------------------------------------------- layered decoders */
-/* A decoder whose layers are described one by one, on unquantized weights: a mixer per layer (gated delta rule with a
- * recurrent state; latent attention or grouped-query attention over the paged cache) and an optional feed-forward
- * (clamped GLU, or sparse experts).  No counterpart in the reference.  It is an fa_decoder: sequences, tokens,
- * sampling, steps, prompt passes, verification and the read-outs are the calls above. */
-typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1, FA_MIXER_ATTENTION = 2 } fa_mixer_kind;
+/* A decoder whose layers are described one by one, on unquantized weights: per layer one mixer or two side by side (gated
+ * delta rule or lightning attention with a recurrent state; latent attention or grouped-query attention over the paged
+ * cache) and an optional feed-forward (a gated linear unit, or sparse experts).  No counterpart in the reference.  It is an
+ * fa_decoder: sequences, tokens, sampling, steps, prompt passes, verification and the read-outs are the calls above. */
+typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1, FA_MIXER_ATTENTION = 2, FA_MIXER_LIGHTNING = 3 } fa_mixer_kind;
 /* How sublayers meet the residual stream x.  FA_NORM_INPUT: x += scale * f(layer_norm(x)), a layer scale per channel;
- * FA_NORM_OUTPUT: x += rms_norm(f(x)).  The final norm is of the same kind. */
-typedef enum { FA_NORM_INPUT = 0, FA_NORM_OUTPUT = 1 } fa_norm_kind;
-/* Attention: projections with biases; RMS norm of the whole query and key projections, over all heads at once. */
-enum { FA_ATTENTION_BIAS = 1, FA_ATTENTION_QK_NORM = 2 };
-typedef struct {
+ * FA_NORM_OUTPUT: x += rms_norm(f(x)); FA_NORM_BOTH: x += layer_norm(f(layer_norm(x))).  The final norm is of the same
+ * kind (layer norm for the last). */
+typedef enum { FA_NORM_INPUT = 0, FA_NORM_OUTPUT = 1, FA_NORM_BOTH = 2 } fa_norm_kind;
+/* Attention: projections with biases; RMS norm of the whole query and key projections, over all heads at once; RMS norm per
+ * head with a weight [dim] that the heads share (before the rotation), or without a weight; the projected keys are the
+ * values (vdim = dim); the heads' outputs times the sigmoid of a further projection; a learned score per head that has no
+ * key and no value and takes its share of the softmax. */
+enum { FA_ATTENTION_BIAS = 1, FA_ATTENTION_QK_NORM = 2, FA_ATTENTION_HEAD_NORM = 4, FA_ATTENTION_HEAD_UNIT = 8, FA_ATTENTION_KEY_VALUES = 16,
+       FA_ATTENTION_GATE = 32, FA_ATTENTION_SINK = 64 };
+/* The feed-forward's gated linear unit.  Clamped: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + 1);
+ * silu: gate sigmoid(gate) up. */
+typedef enum { FA_GLU_CLAMPED = 0, FA_GLU_SILU = 1 } fa_glu_kind;
+typedef struct fa_layer_config {
     int32_t mixer;                /* fa_mixer_kind */
     uint32_t heads, dim, vdim;    /* per head: query / key dims (latent attention: the unrotated part), value dims */
     uint32_t kv_heads, conv;      /* delta: q / k heads, taps of the short convolution (1..=16); attention: key / value heads */
     uint32_t q_rank, kv_rank;     /* latent attention: sizes of the two latents */
-    uint32_t rot_dim, window;     /* latent attention: rotated dims (even), visible keys incl. the token's own */
+    uint32_t rot_dim, window;     /* rotated dims (even): latent attention's rotated part; attention: the first ones of every query and key
+                                     head, 0 for none.  Visible keys incl. the token's own; 0: all earlier ones */
     int32_t kv_from;              /* both attentions: the earlier layer whose cache is used, -1 for its own */
     float scale;                  /* both attentions: factor of the scores */
     double rot_base;
     uint32_t d_ffn;               /* 0: no feed-forward; with experts: size of one */
-    float ffn_limit, ffn_alpha;   /* g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + 1) */
+    float ffn_limit, ffn_alpha;   /* FA_GLU_CLAMPED */
     uint32_t attention;           /* attention: FA_ATTENTION_* */
     uint32_t experts, top;        /* experts > 0 (up to 256): every token takes `top` (up to 64) of them, weighted by a softmax over their
                                      router logits; an expert is W_down relu(W_up x)^2.  With FA_NORM_OUTPUT only */
+    int32_t glu;                  /* fa_glu_kind */
+    uint32_t rot_interleaved;     /* pairs of the rotation: 0: i and i + rot_dim / 2, 1: 2i and 2i + 1 */
+    /* rot_factor > 0: frequencies of fewer than rot_low turns within rot_original positions are divided by it, of more than
+       rot_high turns kept, with a linear ramp between */
+    double rot_factor, rot_low, rot_high, rot_original;
+    uint32_t ungated;             /* latent attention: without the gate per head */
+    uint32_t decay_rank, gate_rank;       /* delta, both or neither: decays per head and key channel and output gates (then sigmoid instead of
+                                     silu) per value channel, from projections of these ranks */
+    const float *decay;           /* lightning: [heads], copied */
+    const struct fa_layer_config *right;  /* a second mixer beside this one, reading the same input (its feed-forward, norms and `right`
+                                     unused); the outputs are added as left_scale, right_scale times each.  Tensors are then
+                                     named mix.left.* and mix.right.* */
+    float left_scale, right_scale;
 } fa_layer_config;
 typedef struct {
     uint32_t n_layers, d_model, vocab;
@@ -601,6 +623,7 @@ typedef struct {
     float embed_scale;            /* factor of the embedding rows; 0: one */
     double position_base;         /* FA_NORM_OUTPUT, above 0: sin(p base^(-2i / d_model)) is added to entry 2i of the embedding of position p, the
                                      cosine to entry 2i + 1 */
+    float logit_scale;            /* factor of the logits ahead of the soft cap; 0: one */
 } fa_layered_config;
 fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cfg, fa_decoder **out);
 /* Number of weight tensors the decoder takes and the i-th one's name and shape (cols 0: a vector). */

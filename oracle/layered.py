@@ -1,6 +1,8 @@
 """Oracle: the mechanisms of the layered decoders (gated delta rule, latent attention, clamped GLU feed-forward,
 layer norm with layer scale, soft-capped head; grouped-query attention with normed projections, sparse experts, additive
-positions, norms on the sublayers' outputs), one function per mechanism, in float64 and token by token.
+positions, norms on the sublayers' outputs; two mixers side by side, rotations of either layout with scaled frequencies, norms
+per head, output gates, sinks, lightning attention, the delta rule with a decay per channel, norms on both sides of a
+sublayer), one function per mechanism, in float64 and token by token.
 
 TEST INFRASTRUCTURE ONLY: written from the equations, for whole sequences, without a cache, a batch or any code
 of the product; only tests and the smoke check may import it.
@@ -211,12 +213,170 @@ def forward_zoferax(config, w, tokens, layers_out=None, margins=None):
     return rms_norm(x, w["final.norm"], eps) @ w["head"].T
 
 
+# ---- Bubetar ---------------------------------------------------------------------------------------------------
+
+def scaled_frequencies(freq, scaling):
+    """Rotation frequencies stretched for long contexts: long waves are slowed down by the factor, short ones stay, with a
+    ramp between the two wavelengths original / high and original / low."""
+    out = np.empty_like(freq)
+    for i, f in enumerate(freq):
+        turns = scaling["original"] * f / (2.0 * np.pi)              # of the wave within the original context
+        if turns > scaling["high"]:
+            out[i] = f
+        elif turns < scaling["low"]:
+            out[i] = f / scaling["factor"]
+        else:
+            s = (turns - scaling["low"]) / (scaling["high"] - scaling["low"])
+            out[i] = (1.0 - s) * f / scaling["factor"] + s * f
+    return out
+
+
+def rotate_leading(x, positions, rot, interleaved):
+    """Rotates the first rot["dims"] entries of x's last axis; x [T, heads, d].  Pairs are neighbours (interleaved) or half the
+    rotated part apart."""
+    dims = rot["dims"]
+    freq = float(rot["base"]) ** (-2.0 * np.arange(dims // 2) / dims)
+    if rot.get("scaling"):
+        freq = scaled_frequencies(freq, rot["scaling"])
+    first = np.arange(0, dims, 2) if interleaved else np.arange(dims // 2)
+    second = first + 1 if interleaved else first + dims // 2
+    out = np.array(x)
+    for t, p in enumerate(positions):
+        turn = np.exp(1j * p * freq)
+        z = (x[t][:, first] + 1j * x[t][:, second]) * turn
+        out[t][:, first], out[t][:, second] = z.real, z.imag
+    return out
+
+
+def sink_attention(q, k, v, scale, window=None, sink=None):
+    """Causal attention with shared key heads; window None: every earlier token.  sink [H]: a score without key and value."""
+    T, H = q.shape[:2]
+    share = H // k.shape[1]
+    out = np.empty((T, H, v.shape[2]))
+    for t in range(T):
+        lo = 0 if window is None else max(0, t - window + 1)
+        for h in range(H):
+            s = k[lo:t + 1, h // share] @ q[t, h] * scale
+            m = s.max() if sink is None else max(s.max(), sink[h])
+            e = np.exp(s - m)
+            total = e.sum() + (0.0 if sink is None else np.exp(sink[h] - m))
+            out[t, h] = e @ v[lo:t + 1, h // share] / total
+    return out
+
+
+def gated_attention_mixer(h, w, p, mx, eps):
+    """Normed, rotated queries and keys; the heads' outputs pass a gate read from the same input."""
+    T, H, G, d = len(h), mx["heads"], mx["kv_heads"], mx["dim"]
+    q = rms_norm((h @ w[p + "q"].T).reshape(T, H, d), w[p + "q.norm"], eps)
+    k = rms_norm((h @ w[p + "k"].T).reshape(T, G, d), w[p + "k.norm"], eps)
+    q, k = (rotate_leading(a, range(T), mx["rot"], True) for a in (q, k))
+    o = sink_attention(q, k, (h @ w[p + "v"].T).reshape(T, G, mx["vdim"]), mx["scale"])
+    return (o.reshape(T, -1) * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def key_value_attention_mixer(h, w, p, mx, eps):
+    """The projected keys are the values; queries and keys are rotated, then normed without a weight; window and sink."""
+    T, H, G, d = len(h), mx["heads"], mx["kv_heads"], mx["dim"]
+    q, k = (h @ w[p + "q"].T).reshape(T, H, d), (h @ w[p + "k"].T).reshape(T, G, d)
+    qr, kr = (rms_norm(rotate_leading(a, range(T), mx["rot"], False), 1.0, eps) for a in (q, k))
+    o = sink_attention(qr, kr, k, mx["scale"], mx["mask"]["size"], w[p + "sink"])
+    return o.reshape(T, -1) @ w[p + "o"].T
+
+
+def lightning_recurrence(q, k, v, decay):
+    """S <- decay S + k v^T, o = S^T q per head; q, k [T, H, dk], v [T, H, dv]."""
+    S = np.zeros((q.shape[1], q.shape[2], v.shape[2]))
+    out = np.empty(v.shape)
+    for t in range(len(q)):
+        for h in range(len(S)):
+            S[h] = decay[h] * S[h] + np.outer(k[t, h], v[t, h])
+            out[t, h] = q[t, h] @ S[h]
+    return out
+
+
+def lightning_mixer(h, w, p, mx, eps):
+    T, H = len(h), mx["heads"]
+    q, k, v = (silu(h @ w[p + n].T).reshape(T, H, -1) for n in "qkv")
+    o = lightning_recurrence(q, k, v, mx["decay"]).reshape(T, -1)
+    return (rms_norm(o, w[p + "norm"], eps) * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def channel_delta_recurrence(q, k, v, beta, log_g):
+    """The delta rule with log decays [T, H, dk]: one per head and row of the state."""
+    S = np.zeros((q.shape[1], q.shape[2], v.shape[2]))
+    out = np.empty(v.shape)
+    for t in range(len(q)):
+        for h in range(len(S)):
+            S[h] *= np.exp(log_g[t, h])[:, None]
+            u = beta[t, h] * (v[t, h] - k[t, h] @ S[h])
+            S[h] += np.outer(k[t, h], u)
+            out[t, h] = q[t, h] @ S[h]
+    return out
+
+
+def channel_delta_mixer(h, w, p, mx, eps):
+    T, dim, vdim, heads, kvh = len(h), mx["dim"], mx["vdim"], mx["heads"], mx["kv_heads"]
+    q, k, v = (silu(causal_conv(h @ w[p + n].T, w[p + n + ".conv"])) for n in "qkv")
+    own = np.arange(heads) // (heads // kvh)
+    q = unit_vector(q.reshape(T, kvh, dim))[:, own] * dim ** -0.5
+    k = unit_vector(k.reshape(T, kvh, dim))[:, own]
+    beta = sigmoid(h @ w[p + "b"].T)
+    a = softplus(h @ w[p + "a1"].T @ w[p + "a2"].T + w[p + "dt_bias"]).reshape(T, heads, dim)
+    o = channel_delta_recurrence(q, k, v.reshape(T, heads, vdim), beta, -np.exp(w[p + "A_log"])[None, :, None] * a)
+    o = rms_norm(o, w[p + "norm"], eps).reshape(T, -1) * sigmoid(h @ w[p + "g1"].T @ w[p + "g2"].T)
+    return o @ w[p + "o"].T
+
+
+def plain_latent_mixer(h, w, p, mx, eps):
+    """Latent attention without a gate over all earlier tokens, the rotated parts in pairs of neighbours."""
+    T, H, dim, r = len(h), mx["heads"], mx["dim"], mx["kv_rank"]
+    q = (rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps) @ w[p + "uq"].T).reshape(T, H, -1)
+    y = h @ w[p + "dkv"].T
+    c = rms_norm(y[:, :r], w[p + "dkv.norm"], eps)
+    kr = rotate_leading(y[:, None, r:], range(T), mx["rot"], True)
+    q = np.concatenate([q[..., :dim], rotate_leading(q[..., dim:], range(T), mx["rot"], True)], axis=-1)
+    k = np.concatenate([(c @ w[p + "uk"].T).reshape(T, H, dim), np.repeat(kr, H, axis=1)], axis=-1)
+    o = sink_attention(q, k, (c @ w[p + "uv"].T).reshape(T, H, -1), mx["scale"])
+    return o.reshape(T, -1) @ w[p + "o"].T
+
+
+def side_by_side(h, w, p, mx, eps, left, right):
+    return mx["left_scale"] * left(h, w, p + "left.", mx["left"], eps) + mx["right_scale"] * right(h, w, p + "right.", mx["right"], eps)
+
+
+def silu_glu(h, w, p):
+    return (silu(h @ w[p + "gate"].T) * (h @ w[p + "up"].T)) @ w[p + "down"].T
+
+
+def forward_bubetar(config, w, tokens, layers_out=None):
+    """Every sublayer is normed on both sides; scaled, soft-capped logits."""
+    eps = config["norm"]["eps"]
+    x = w["embed"][np.asarray(tokens, dtype=np.int64)]
+    for i, layer in enumerate(config["layers"]):
+        p, mx = "l%d." % i, layer["mixer"]
+        h = layer_norm(x, w[p + "norm1"], eps)
+        if layer["type"] == "parallel":
+            y = side_by_side(h, w, p + "mix.", mx, eps, gated_attention_mixer, lightning_mixer)
+        elif layer["type"] == "parallel_2":
+            y = side_by_side(h, w, p + "mix.", mx, eps, key_value_attention_mixer, channel_delta_mixer)
+        else:
+            y = plain_latent_mixer(h, w, p + "mix.", mx, eps)
+        x = x + layer_norm(y, w[p + "norm1b"], eps)
+        if layer["mlp"] is not None:
+            x = x + layer_norm(silu_glu(layer_norm(x, w[p + "norm2"], eps), w, p + "mlp."), w[p + "norm2b"], eps)
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return softcap(layer_norm(x, w["final.norm"], eps) @ w["head"].T * config["logit_scale"], config["logit_softcap"])
+
+
 def forward(config, weights, tokens, layers_out=None, margins=None):
     """Logits [T, vocab] of one whole sequence; layers_out (a list) receives the residual after every layer, margins (a
     list) the routing margins of every layer of sparse experts."""
     w = {n: np.asarray(a, dtype=np.float64) for n, a in weights.items()}
     if config["architecture"] == "Zoferax":
         return forward_zoferax(config, w, tokens, layers_out, margins)
+    if config["architecture"] == "Bubetar":
+        return forward_bubetar(config, w, tokens, layers_out)
     eps = config["norm"]["eps"]
     x = w["embed"][np.asarray(tokens, dtype=np.int64)]
     kept = {}

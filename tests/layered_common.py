@@ -45,6 +45,58 @@ def zoferax(layers, width=76, vocab=131, eps=1e-5, scale=1.7):
     return {"architecture": "Zoferax", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps}, "embedding": {"scale": scale}}
 
 
+def rotation(dims, base=10000.0, scaling=None):
+    rot = {"base": base, "dims": dims}
+    if scaling:
+        rot["scaling"] = dict(zip(("factor", "low", "high", "original"), scaling))
+    return rot
+
+
+def beside(left, right, kind, scales, mlp):
+    return {"type": kind, "mixer": {"left": left, "right": right, "left_scale": scales[0], "right_scale": scales[1]}, "mlp": mlp}
+
+
+def gated_left(heads=6, kv_heads=2, dim=20, vdim=12, rot=12, scale=None, base=3000.0):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "rot": rotation(rot, base), "scale": 1.4 * dim ** -0.5 if scale is None else scale}
+
+
+def lightning_right(heads=3, dim=20, vdim=28, decay=None):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "decay": [1.0 - 0.7 ** (2 * h + 1) for h in range(heads)] if decay is None else decay}
+
+
+def key_value_left(heads=6, kv_heads=3, dim=20, rot=16, window=11, scale=None, base=5000.0, scaling=(6.0, 1.0, 3.0, 90)):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "rot": rotation(rot, base, scaling), "mask": {"size": window},
+            "scale": 1.3 * dim ** -0.5 if scale is None else scale}
+
+
+def channel_right(heads=4, kv_heads=2, dim=20, vdim=12, conv=4):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}
+
+
+def parallel(left=None, right=None, scales=(0.7, 1.3), mlp=None):
+    return beside(left or gated_left(), right or lightning_right(), "parallel", scales, mlp)
+
+
+def parallel_2(left=None, right=None, scales=(1.4, 0.6), mlp=None):
+    return beside(left or key_value_left(), right or channel_right(), "parallel_2", scales, mlp)
+
+
+def open_latent(heads=3, dim=20, rot=12, vdim=28, q_rank=36, kv_rank=44, scale=None, base=10000.0, mlp=None):
+    l = latent(heads, dim, rot, vdim, q_rank, kv_rank, 1, scale, base, None, mlp)
+    del l["mixer"]["mask"]
+    return l
+
+
+def dense(ff=52):
+    return {"kind": "dense", "ff": ff}
+
+
+def bubetar(layers, width=76, vocab=131, eps=1e-5, softcap=12.0, scale=0.8, ranks=(10, 14)):
+    """ranks: of the low-rank decays and gates, which only the weights' shapes tell."""
+    return {"architecture": "Bubetar", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps}, "logit_scale": scale, "logit_softcap": softcap,
+            "_ranks": ranks}
+
+
 def bf16_round(a):
     u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
     return ((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32).view(np.float32)
@@ -67,7 +119,37 @@ def zoferax_shapes(cfg):
     return out
 
 
+def bubetar_shapes(cfg):
+    D = cfg["width"]
+    out = {"embed": (cfg["vocab"], D), "head": (cfg["vocab"], D), "final.norm": (D,)}
+    for i, l in enumerate(cfg["layers"]):
+        p, mx = "l%d." % i, l["mixer"]
+        out.update({p + "norm1": (D,), p + "norm1b": (D,)})
+        if l["type"] == "latent_attention":
+            m, H, r, k, d = p + "mix.", mx["heads"], mx["q_rank"], mx["kv_rank"], mx["dim"]
+            out.update({m + "dq": (r, D), m + "dq.norm": (r,), m + "uq": (H * (d + mx["rot_dim"]), r), m + "dkv": (k + mx["rot_dim"], D),
+                        m + "dkv.norm": (k,), m + "uk": (H * d, k), m + "uv": (H * mx["vdim"], k), m + "o": (D, H * mx["vdim"])})
+        else:
+            a, b, m, n = mx["left"], mx["right"], p + "mix.left.", p + "mix.right."
+            H, G, d, wide = a["heads"], a["kv_heads"], a["dim"], b["heads"] * b["vdim"]
+            out.update({m + "q": (H * d, D), m + "k": (G * d, D), m + "o": (D, H * a["vdim"]), n + "v": (wide, D), n + "o": (D, wide)})
+            if l["type"] == "parallel":
+                out.update({m + "v": (G * a["vdim"], D), m + "q.norm": (d,), m + "k.norm": (d,), m + "g": (H * a["vdim"], D), n + "q": (b["heads"] * b["dim"], D),
+                            n + "k": (b["heads"] * b["dim"], D), n + "g": (wide, D), n + "norm": (wide,)})
+            else:
+                (ra, rg), nq, nd = cfg["_ranks"], b["kv_heads"] * b["dim"], b["heads"] * b["dim"]
+                out.update({m + "sink": (H,), n + "q": (nq, D), n + "k": (nq, D), n + "q.conv": (nq, b["conv"]), n + "k.conv": (nq, b["conv"]),
+                            n + "v.conv": (wide, b["conv"]), n + "b": (b["heads"], D), n + "A_log": (b["heads"],), n + "dt_bias": (nd,), n + "norm": (b["vdim"],),
+                            n + "a1": (ra, D), n + "a2": (nd, ra), n + "g1": (rg, D), n + "g2": (wide, rg)})
+        if l["mlp"]:
+            f, ff = p + "mlp.", l["mlp"]["ff"]
+            out.update({p + "norm2": (D,), p + "norm2b": (D,), f + "gate": (ff, D), f + "up": (ff, D), f + "down": (D, ff)})
+    return out
+
+
 def shapes(cfg):
+    if cfg["architecture"] == "Bubetar":
+        return bubetar_shapes(cfg)
     if cfg["architecture"] == "Zoferax":
         return zoferax_shapes(cfg)
     D = cfg["width"]
@@ -127,7 +209,7 @@ def tokens(cfg, n, seed=0):
 def make_decoder(ops, cfg, w, dtype="float32", max_tokens=512, max_batch=4, state_slots=None, block_size=16, as_bf16=True):
     from fandhe_ai_amd import models
     from fandhe_ai_amd.safetensors_io import TypedTensor
-    d = models.build_layered(ops, cfg, dtype, models.Capacity(max_tokens, max_batch, state_slots, block_size))
+    d = models.build_layered(ops, cfg, dtype, models.Capacity(max_tokens, max_batch, state_slots, block_size), shapes(cfg))
     typed = {}
     for n, a in w.items():
         if as_bf16:
