@@ -105,8 +105,8 @@ def make_tables(rng, ctxs, extra_tokens, bs, num_blocks=None):
 
 
 # ------------------------------------------------------------------ layered decoders
-# Nugelix and Zoferax stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward (of the
-# experts: those one token takes) and depth.
+# Nugelix, Zoferax and Bubetar stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward
+# (of the experts: those one token takes) and depth.
 def _nugelix(width, heads, q_rank, window, ff, d_heads, d_kv_heads, repeat):
     latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff, "limit": 7.0},
               "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": q_rank, "kv_rank": 512, "mask": {"size": window},
@@ -126,14 +126,34 @@ def _zoferax(width, heads, kv_heads, vdim, experts, top, ff, layers, shared):
             "layers": [layer(i) for i in range(layers)]}
 
 
+LOW_RANK = 128                                                # of Bubetar's decays and gates
+
+
+def _bubetar(width, heads, kv_heads, q_rank, window, ff, repeat):
+    mlp, rot = {"kind": "dense", "ff": ff}, lambda dims, **more: dict(base=1e6, dims=dims, **more)
+    heads_of = {"heads": heads, "dim": 128, "vdim": 128}
+    grouped = dict(heads_of, kv_heads=kv_heads, scale=128 ** -0.5)
+    lightning = dict(heads_of, decay=[1.0 - 2.0 ** (-1.0 - 8.0 * h / heads) for h in range(heads)])
+    scaled = rot(64, scaling={"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192})
+    layers = [{"type": "parallel", "mlp": mlp, "mixer": {"left": dict(grouped, rot=rot(64)), "right": lightning, "left_scale": 0.8, "right_scale": 1.1}},
+              {"type": "parallel_2", "mlp": mlp, "mixer": {"left": dict(grouped, rot=scaled, mask={"size": window}), "right": dict(heads_of, kv_heads=heads // 2, conv=4),
+                                                           "left_scale": 0.8, "right_scale": 1.1}}]
+    latent = {"type": "latent_attention", "mlp": mlp, "mixer": dict(heads_of, rot_dim=64, q_rank=q_rank, kv_rank=512, rot=rot(64), scale=192 ** -0.5)}
+    return {"architecture": "Bubetar", "width": width, "vocab": 32000, "norm": {"eps": 1e-6}, "logit_scale": 0.5, "logit_softcap": 30.0,
+            "layers": (layers + [latent, latent]) * repeat}
+
+
 LAYERED = {"large": dict(nugelix=_nugelix(4096, 32, 1536, 2048, 14336, 32, 16, 2), zoferax=_zoferax(4096, 32, 8, 128, 16, 4, 5376, 8, 3),
+                         bubetar=_bubetar(4096, 32, 8, 1536, 2048, 14336, 2),
                          w8a8=dict(d_model=4096, n_heads=32, n_kv_heads=8, d_ffn=14336, n_layers=8, vocab=32000)),
            "small": dict(nugelix=_nugelix(2048, 16, 768, 1024, 8192, 16, 8, 2), zoferax=_zoferax(2048, 16, 4, 64, 16, 4, 3072, 8, 3),
+                         bubetar=_bubetar(2048, 16, 4, 768, 1024, 8192, 2),
                          w8a8=dict(d_model=2048, n_heads=16, n_kv_heads=4, d_ffn=8192, n_layers=8, vocab=32000))}
 
 
 def build_layered(fa, be, config, max_tokens, batch):
-    dec = fa.models.build_layered(be, config, "bfloat16", fa.models.Capacity(max_tokens, batch))
+    ranks = {"l%d.mix.right.%s" % (i, n): (LOW_RANK, config["width"]) for i in range(len(config["layers"])) for n in ("a1", "g1")}
+    dec = fa.models.build_layered(be, config, "bfloat16", fa.models.Capacity(max_tokens, batch), ranks)
     noise = np.random.default_rng(0).normal(size=1 << 20).astype(np.float32)
     made = {}                                                     # equal shapes hold equal values
     for name, shape in dec.tensors().items():
@@ -151,7 +171,7 @@ def build_layered(fa, be, config, max_tokens, batch):
     return dec
 
 
-def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "zoferax", "w8a8")):
+def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "zoferax", "bubetar", "w8a8")):
     """Decode and prompt throughput of layered stacks, and of the W8A8 decoder of equal width, feed-forward and depth."""
     lib = fa.capi.lib
     V = LAYERED[size]["w8a8"]["vocab"]
@@ -194,7 +214,7 @@ def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1
             dec.set_sequences(t, [length] * b)
         return set_rows
 
-    for model in ("nugelix", "zoferax"):
+    for model in ("nugelix", "zoferax", "bubetar"):
         if model in models:
             dec = build_layered(fa, be, LAYERED[size][model], most * pages * 16, most)
             measure(model + " bf16", dec, rows_of(most * pages))
@@ -924,7 +944,7 @@ def main():
                     help="with --only layered: the sizes of the layered stacks (and of the W8A8 decoder beside them)")
     ap.add_argument("--layered-phase", choices=("all", "decode", "prompt"), default="all",
                     help="with --only layered: all, or one shape of one phase (for a kernel trace)")
-    ap.add_argument("--layered-model", choices=("all", "nugelix", "zoferax", "w8a8"), default="all", help="with --only layered: one of the decoders")
+    ap.add_argument("--layered-model", choices=("all", "nugelix", "zoferax", "bubetar", "w8a8"), default="all", help="with --only layered: one of the decoders")
     a = ap.parse_args()
     if a.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (--gpus 1); nothing here shards across devices")

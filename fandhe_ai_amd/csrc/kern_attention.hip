@@ -67,8 +67,8 @@ __global__ void __launch_bounds__(NT)
     place(row + nq + nk, nv, sh.vdim, sh.v_p, 1.0f, nullptr, v_pool + slot * sh.kv_heads * sh.v_p);
 }
 
-// Norms per head and rotation.  One block per row; groups of 2^group_log2 lanes take one head at a time.  VEC: sizes, pitches and
-// the rotated part's halves allow four values at a time.
+// Norms per head and rotation.  One block per row, or several where there are few rows; groups of 2^group_log2 lanes take one head
+// at a time.  VEC: sizes, pitches and the rotated part's halves allow four values at a time.
 struct PrepareHeads {
     const float *q_norm, *k_norm, *cos_sin;
     int norms, key_values;
@@ -89,7 +89,8 @@ __global__ void __launch_bounds__(256)
         else *dst = f32_to_bf16(v[0]);
     };
     const uint32_t units = H + (slot < sh.pool_rows ? (ph.key_values ? G : 2 * G) : 0);
-    for (uint32_t u = threadIdx.x >> group_log2; u < units; u += 256u >> group_log2) {
+    const uint32_t groups = 256u >> group_log2;
+    for (uint32_t u = blockIdx.y * groups + (threadIdx.x >> group_log2); u < units; u += gridDim.y * groups) {
         if (u >= H + G) {                            // a value head
             const uint32_t g = u - H - G;
             const float *src = row + (H + G) * sh.dim + g * sh.vdim;
@@ -237,6 +238,9 @@ __global__ void __launch_bounds__(256)
     }
 }
 
+// Whether position p sees key j: 0 <= p - j < W
+__device__ __forceinline__ bool seen(int32_t p, int32_t j, int32_t W) { return (uint32_t)(p - j) < (uint32_t)W; }
+
 // Factor of what a column summed with maximum m (of scores in powers of two) and sum l of the weights: the sink takes its share
 // of the softmax here.
 __device__ __forceinline__ float final_factor(const AttentionOutput &ao, uint32_t head, float m, float l) {
@@ -370,7 +374,7 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int32_t j = k0 + kt * 16 + 4 * g + e;
-                    sc[qi][kt * 4 + e] = j <= pos[qi] && pos[qi] - j < W && j < k_hi ? acc[qi][e] * factor : -INFINITY;
+                    sc[qi][kt * 4 + e] = seen(pos[qi], j, W) && j < k_hi ? acc[qi][e] * factor : -INFINITY;
                 }
         }
         __builtin_amdgcn_sched_barrier(0);
@@ -605,10 +609,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         float v = acc[qi][e] * factor;
-                        if (!inside) {
-                            const int32_t j = k0 + kt * 16 + 4 * g + e;
-                            if (j > pos[qi] || pos[qi] - j >= W) v = -INFINITY;
-                        }
+                        if (!inside && !seen(pos[qi], k0 + kt * 16 + 4 * g + e, W)) v = -INFINITY;
                         sc[qi][kt * 4 + e] = v;
                     }
             }
@@ -758,8 +759,10 @@ void attention_prepare_heads(const float *y, uint32_t ld, bool norms, const floa
     uint32_t group_log2 = 0;
     while (group_log2 < 6 && ((vec ? 4u : 1u) << group_log2) < sh.dim) ++group_log2;
     const PrepareHeads ph{q_norm, k_norm, cos_sin, norms, key_values};
+    const uint32_t groups = 256u >> group_log2, units = sh.heads + 2 * sh.kv_heads;
+    const dim3 grid(rr.rows, rr.rows <= 256 ? (units + groups - 1) / groups : 1);
 #define FA_PREP(T_, VEC_) \
-    attention_prepare_heads_kernel<T_, VEC_><<<rr.rows, 256, 0, s>>>(y, ld, ph, (T_ *)q, (T_ *)k_pool, (T_ *)v_pool, sh, rr.kv_slot, group_log2)
+    attention_prepare_heads_kernel<T_, VEC_><<<grid, 256, 0, s>>>(y, ld, ph, (T_ *)q, (T_ *)k_pool, (T_ *)v_pool, sh, rr.kv_slot, group_log2)
     if (is_f32) {
         if (vec) FA_PREP(float, true);
         else FA_PREP(float, false);

@@ -266,7 +266,7 @@ __device__ __forceinline__ v4f mfma4(const v4f &a, const v4f &b, v4f c) {
 
 // silu(convolution) of `cols` channels from c0 on for the chunk's tokens t0 .. into dst [32][pitch]; zeros for tokens past
 // the end and columns up to cols_p.  A thread takes TG tokens of two neighbouring channels (one where they are not aligned).
-template <typename T, int MAXTAPS, int TG>
+template <typename T, int MAXTAPS, int TG, int NT = 256>
 __device__ __forceinline__ void conv_chunk(float *dst, uint32_t pitch, const T *__restrict__ y, uint32_t ld, const T *__restrict__ ring,
                                            const float *__restrict__ conv, uint32_t taps, uint32_t channels, uint32_t c0, uint32_t cols,
                                            uint32_t cols_p, uint64_t row0, uint32_t t0, uint32_t n, uint32_t p0) {
@@ -274,7 +274,7 @@ __device__ __forceinline__ void conv_chunk(float *dst, uint32_t pitch, const T *
     if (MAXTAPS != 0 && ((ld | channels | c0 | cols) & 1) == 0) {
         constexpr int NX = TG + (MAXTAPS ? MAXTAPS : 1) - 1, MT = MAXTAPS ? MAXTAPS : 1;
         const uint32_t pairs = cols_p / 2;
-        for (uint32_t item = threadIdx.x; item < pairs * NG; item += 256) {
+        for (uint32_t item = threadIdx.x; item < pairs * NG; item += NT) {
             const uint32_t col = item % pairs * 2, tg = item / pairs * TG;
             const uint32_t c = c0 + (col < cols ? col : 0);
             v2f w[MT], x[NX];
@@ -312,7 +312,7 @@ __device__ __forceinline__ void conv_chunk(float *dst, uint32_t pitch, const T *
         }
         return;
     }
-    for (uint32_t item = threadIdx.x; item < cols_p * NG; item += 256) {
+    for (uint32_t item = threadIdx.x; item < cols_p * NG; item += NT) {
         const uint32_t col = item % cols_p, tg = item / cols_p * TG;
         for (uint32_t j = 0; j < TG; ++j) {
             const uint32_t t = t0 + tg + j;
@@ -530,9 +530,11 @@ __global__ void __launch_bounds__(256)
 // Decays per channel: G [32][dim].  One block per (chunk, head).  exp(G_i - G_j) is formed from differences that are never
 // positive, however strong the decays: pair by pair inside the two diagonal blocks of A and P, and through the last token of the
 // first half for the block below the diagonal, exp(G_i - G_15) exp(G_15 - G_j).  G is kept in powers of two.
+constexpr int kChannelThreads = 512;
 template <typename T, int KT, int MAXTAPS>
-__global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, float *__restrict__ frags, uint32_t n_frags) {
+__global__ void __launch_bounds__(kChannelThreads) channel_chunk_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, float *__restrict__ frags, uint32_t n_frags) {
     constexpr Recurrence KIND = Recurrence::kChannelDelta;
+    constexpr int NT = kChannelThreads, NW = NT / 64;
     constexpr uint32_t DP = KT * 16, PITCH = DP + 4, VS = 64, VPITCH = VS + 4;
     extern __shared__ __attribute__((aligned(16))) float lds[];
     float *lk = lds, *lq = lk + 32 * PITCH, *lg = lq + 32 * PITCH, *lv = lg + 32 * PITCH;      // K, Q, G, 64 columns of V
@@ -553,10 +555,10 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
     v4f *out = (v4f *)(frags + ((uint64_t)blockIdx.x * sh.heads + h) * n_frags * 256) + lane;
     auto put = [&](uint32_t f, const v4f &v) { out[f * 64] = v; };
 
-    conv_chunk<T, MAXTAPS, 8>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, hk * dim, dim, DP, row0, t0, n, p0);
-    conv_chunk<T, MAXTAPS, 8>(lk, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, (sh.kv_heads + hk) * dim, dim, DP, row0, t0, n, p0);
+    conv_chunk<T, MAXTAPS, 8, NT>(lq, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, hk * dim, dim, DP, row0, t0, n, p0);
+    conv_chunk<T, MAXTAPS, 8, NT>(lk, PITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, (sh.kv_heads + hk) * dim, dim, DP, row0, t0, n, p0);
     const float a = -expf(io.a_log[h]) * kLog2e;
-    for (uint32_t i = tid; i < 32 * DP; i += 256) {
+    for (uint32_t i = tid; i < 32 * DP; i += NT) {
         const uint32_t t = i / DP, d = i % DP;
         float v = 0.0f;
         if (t0 + t < n && d < dim) v = fast_log2_decay(a, io.decay[(uint64_t)(row0 + t0 + t) * io.ld_decay + h * dim + d] + io.dt_bias[h * dim + d]);
@@ -564,20 +566,20 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
     }
     if (tid < 32) beta[tid] = t0 + tid < n ? sigmoid_f32(io.beta[(uint64_t)(row0 + t0 + tid) * io.ld_beta + h]) : 0.0f;
     __syncthreads();
-    {   // four threads per row of Q and of K
-        const float *row = (tid < 128 ? lq : lk) + ((tid % 128) / 4) * PITCH;
+    {   // eight threads per row of Q and of K
+        const float *row = (tid < 256 ? lq : lk) + ((tid % 256) / 8) * PITCH;
         float sq = 0.0f;
-        for (uint32_t i = tid % 4; i < DP; i += 4) sq = fmaf(row[i], row[i], sq);
-        sq += __shfl_xor(sq, 1, 64);
-        sq += __shfl_xor(sq, 2, 64);
-        if (tid % 4 == 0) {
+        for (uint32_t i = tid % 8; i < DP; i += 8) sq = fmaf(row[i], row[i], sq);
+#pragma unroll
+        for (int off = 1; off < 8; off <<= 1) sq += __shfl_xor(sq, off, 64);
+        if (tid % 8 == 0) {
             const float r = 1.0f / sqrtf(sq + 1e-6f);
-            if (tid < 128) rq[tid / 4] = r / sqrtf((float)dim);
-            else rk[(tid - 128) / 4] = r;
+            if (tid < 256) rq[tid / 8] = r / sqrtf((float)dim);
+            else rk[(tid - 256) / 8] = r;
         }
     }
     __syncthreads();
-    for (uint32_t d = tid; d < DP; d += 256) {       // running sums, eight tokens read at a time
+    for (uint32_t d = tid; d < DP; d += NT) {       // running sums, eight tokens read at a time
         float G = 0.0f;
 #pragma unroll
         for (uint32_t t1 = 0; t1 < 32; t1 += 8) {
@@ -588,20 +590,21 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
             for (uint32_t t = 0; t < 8; ++t) lg[(t1 + t) * PITCH + d] = G += v[t];
         }
     }
-    for (uint32_t i = tid; i < 32 * DP / 4; i += 256) {
+    for (uint32_t i = tid; i < 32 * DP / 4; i += NT) {
         const uint32_t t = i / (DP / 4), d = i % (DP / 4) * 4;
         *(v4f *)(lq + t * PITCH + d) *= rq[t];
         *(v4f *)(lk + t * PITCH + d) *= rk[t];
     }
     __syncthreads();
-    // diagonal blocks: wavefronts 0, 2 the first half of the channels of block 0, 1, wavefronts 1, 3 the second half; a lane takes
-    // two rows by two columns
-    const int blk = wave / 2, ti = lane / 8, tj = lane % 8, i0 = blk * 16 + 2 * ti, j0 = blk * 16 + 2 * tj;
+    // diagonal blocks: wavefronts 0 - 3 a quarter of the channels each of block 0, 4 - 7 of block 1; a lane takes two rows by two
+    // columns
+    const int blk = wave / 4, part = wave % 4, ti = lane / 8, tj = lane % 8, i0 = blk * 16 + 2 * ti, j0 = blk * 16 + 2 * tj;
     v4f kk = v4f{0.f, 0.f, 0.f, 0.f}, qk = kk;       // (i0, j0), (i0, j0 + 1), (i0 + 1, j0), (i0 + 1, j0 + 1)
     if (tj <= ti) {
         const bool diagonal = ti == tj;
-#pragma unroll 2
-        for (uint32_t d = (wave % 2) * (DP / 2); d < (wave % 2 + 1) * (DP / 2); d += 4) {
+#pragma unroll DP >= 32 ? 2 : 1
+        for (uint32_t dd = 0; dd < DP / 4; dd += 4) {
+            const uint32_t d = part * (DP / 4) + dd;
             const v4f gi0 = *(const v4f *)(lg + i0 * PITCH + d), gi1 = *(const v4f *)(lg + (i0 + 1) * PITCH + d);
             const v4f gj0 = *(const v4f *)(lg + j0 * PITCH + d), gj1 = *(const v4f *)(lg + (j0 + 1) * PITCH + d);
             const v4f kj0 = *(const v4f *)(lk + j0 * PITCH + d), kj1 = *(const v4f *)(lk + (j0 + 1) * PITCH + d);
@@ -623,36 +626,41 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
             }
         }
     }
-    if (wave % 2 == 1) {
+    if (part != 0) {                                 // parts 1: in A and P themselves, 2 and 3: in the columns of V
+        float *pa = part == 1 ? la : lv + (part - 2) * 1024, *pp = part == 1 ? lt : pa + 512;
 #pragma unroll
         for (int c = 0; c < 4; ++c) {
-            la[(i0 + c / 2) * 36 + j0 + c % 2] = kk[c];
-            lt[(i0 + c / 2) * 36 + j0 + c % 2] = qk[c];
+            const int i = 2 * ti + c / 2, j = 2 * tj + c % 2, at = part == 1 ? (blk * 16 + i) * 36 + blk * 16 + j : blk * 256 + i * 16 + j;
+            pa[at] = kk[c];
+            pp[at] = qk[c];
         }
-        // the block below the diagonal: wavefront 1 of A, 3 of P; the result's rows are keys, its column is a row of the block
-        const float *lx = wave == 1 ? lk : lq;
+    }
+    if (part == 3) {
+        // the block below the diagonal: wavefront 3 of A, 7 of P; the result's rows are keys, its column is a row of the block
+        const float *lx = wave == 3 ? lk : lq;
         v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
-        for (uint32_t k = g; k < DP; k += 4) {
+        for (uint32_t k0 = 0; k0 < DP; k0 += 4) {
+            const uint32_t k = k0 + g;
             const float ref = lg[15 * PITCH + k];
             const float kj = lk[lr * PITCH + k] * exp2_fast(ref - lg[lr * PITCH + k]);
             const float xi = lx[(16 + lr) * PITCH + k] * exp2_fast(lg[(16 + lr) * PITCH + k] - ref);
             acc = __builtin_amdgcn_mfma_f32_16x16x4f32(kj, xi, acc, 0, 0, 0);
         }
-        float *dst = (wave == 1 ? la : lt) + (16 + lr) * 36 + 4 * g;
-        *(v4f *)dst = wave == 1 ? acc * beta[16 + lr] : acc;
+        float *dst = (wave == 3 ? la : lt) + (16 + lr) * 36 + 4 * g;
+        *(v4f *)dst = wave == 3 ? acc * beta[16 + lr] : acc;
     }
     __syncthreads();
-    if (wave % 2 == 0) {
+    if (part == 0) {
 #pragma unroll
         for (int c = 0; c < 4; ++c) {
-            const int i = i0 + c / 2, j = j0 + c % 2;
-            la[i * 36 + j] = j < i ? beta[i] * (kk[c] + la[i * 36 + j]) : 0.0f;
-            lt[i * 36 + j] = j <= i ? qk[c] + lt[i * 36 + j] : 0.0f;
+            const int i = i0 + c / 2, j = j0 + c % 2, at = blk * 256 + (2 * ti + c / 2) * 16 + 2 * tj + c % 2;
+            la[i * 36 + j] = j < i ? beta[i] * ((kk[c] + la[i * 36 + j]) + (lv[at] + lv[1024 + at])) : 0.0f;
+            lt[i * 36 + j] = j <= i ? (qk[c] + lt[i * 36 + j]) + (lv[512 + at] + lv[1536 + at]) : 0.0f;
         }
     }
     // exp(G) Q, the decayed K^T, the chunk's decays
-    for (uint32_t f = wave; f < 2 * KT; f += 4) {
+    for (uint32_t f = wave; f < 2 * KT; f += NW) {
         const uint32_t rt = f / KT, kt = f % KT, i = rt * 16 + lr;
         const v4f q = *(const v4f *)(lq + i * PITCH + kt * 16 + 4 * g), G = *(const v4f *)(lg + i * PITCH + kt * 16 + 4 * g);
         put(frag_q(KIND, KT) + f, v4f{q[0] * exp2_fast(G[0]), q[1] * exp2_fast(G[1]), q[2] * exp2_fast(G[2]), q[3] * exp2_fast(G[3])});
@@ -666,15 +674,16 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
         }
         put(frag_k(KIND, KT) + f, v);
     }
-    frags[(((uint64_t)blockIdx.x * sh.heads + h) * n_frags + frag_p(KIND, KT) + 3) * 256 + tid] = tid < (int)DP ? exp2_fast(lg[31 * PITCH + tid]) : 0.0f;
+    if (tid < 256)
+        frags[(((uint64_t)blockIdx.x * sh.heads + h) * n_frags + frag_p(KIND, KT) + 3) * 256 + tid] = tid < (int)DP ? exp2_fast(lg[31 * PITCH + tid]) : 0.0f;
     const uint32_t vc0 = 2 * sh.kv_heads * dim + h * vdim;
     auto conv_v = [&](uint32_t v0) {
         const uint32_t cols = vdim - v0 < VS ? vdim - v0 : VS;
-        conv_chunk<T, MAXTAPS, 4>(lv, VPITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, vc0 + v0, cols, (cols + 15) / 16 * 16, row0, t0, n, p0);
+        conv_chunk<T, MAXTAPS, 4, NT>(lv, VPITCH, y, io.ld_y, ring, io.conv, sh.taps, channels, vc0 + v0, cols, (cols + 15) / 16 * 16, row0, t0, n, p0);
     };
+    __syncthreads();                                 // the partial sums are read
     conv_v(0);
-    __syncthreads();
-    if (wave > 0) {                                  // P: 00, 10, 11
+    if (wave > 0 && wave < 4) {                      // P: 00, 10, 11
         const int ri = wave == 1 ? 0 : 1, ci = wave == 3 ? 1 : 0;
         put(frag_p(KIND, KT) + wave - 1, *(const v4f *)(lt + (ri * 16 + lr) * 36 + ci * 16 + 4 * g));
     }
@@ -684,7 +693,7 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
     // -W^T = -K'^T T^T, K' = diag(beta) (exp(G) K): the columns of the result are tokens, so its D order is W's A order
     v4f tf[2][2];
     load_scaled_inverse(tf, lt, beta, lr, g);
-    for (uint32_t f = wave; f < 2 * KT; f += 4) {
+    for (uint32_t f = wave; f < 2 * KT; f += NW) {
         const uint32_t rt = f / KT, kt = f % KT;
         v4f acc = v4f{0.f, 0.f, 0.f, 0.f};
         for (uint32_t ct = 0; ct <= rt; ++ct) {
@@ -705,7 +714,7 @@ __global__ void __launch_bounds__(256) channel_chunk_kernel(DeltaShape sh, Delta
             __syncthreads();
         }
         const uint32_t tiles = ((vdim - v0 < VS ? vdim - v0 : VS) + 15) / 16;
-        for (uint32_t f = wave; f < 2 * tiles; f += 4)
+        for (uint32_t f = wave; f < 2 * tiles; f += NW)
             put(shared_frags(KIND, KT) + (v0 / 16 + f / 2) * 2 + f % 2, value_tile(tf, lv, VPITCH, f % 2, f / 2, lr, g));
     }
 }
@@ -909,7 +918,37 @@ __global__ void __launch_bounds__(512)
         }
 }
 
-// Read-outs of the chunk form: root mean square, weight, gate.  One wavefront per (row, head).
+// Four read-outs, or one: weight, gate, scale, rounding.
+template <typename T, typename P>
+__device__ __forceinline__ void store_gated(const DeltaShape &sh, P v, const T *gate, T *out) {
+    if constexpr (sizeof(P) == 16 && sizeof(T) == 2) {
+        const v2u u = *(const v2u *)gate;
+        v *= P{output_gate(sh.gate_sigmoid, bf16_lo(u[0])), output_gate(sh.gate_sigmoid, bf16_hi(u[0])), output_gate(sh.gate_sigmoid, bf16_lo(u[1])),
+               output_gate(sh.gate_sigmoid, bf16_hi(u[1]))};
+        *(v2u *)out = v2u{f32x2_to_bf16x2(v[0], v[1]), f32x2_to_bf16x2(v[2], v[3])};
+    } else {
+#pragma unroll
+        for (int e = 0; e < (int)(sizeof(P) / 4); ++e) store_from_f32(out + e, v[e] * output_gate(sh.gate_sigmoid, load_as_f32(gate + e)));
+    }
+}
+
+// Read-outs of the chunk form: root mean square, weight, gate.  One wavefront per (row, head); two heads with 32 lanes each where
+// four values per lane make a head (HALVES).
+template <typename T>
+__global__ void __launch_bounds__(256) delta_gate_halves_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr) {
+    const uint32_t c = threadIdx.x % 32 * 4, r = blockIdx.x, vdim = sh.vdim, b = rr.row_seq[r];
+    if (rr.row_start[b + 1] - rr.row_start[b] < kChunkFrom) return;          // done token by token
+    const v4f w = c < vdim ? *(const v4f *)(io.norm + c) * io.out_scale : v4f{0.f, 0.f, 0.f, 0.f};
+    for (uint32_t h = threadIdx.x / 32; h < sh.heads; h += 8) {
+        const uint64_t at = (uint64_t)r * sh.heads * vdim + h * vdim + c;
+        const v4f x = c < vdim ? *(const v4f *)(io.raw + at) : v4f{0.f, 0.f, 0.f, 0.f};
+        float sq = row16_sum(fmaf(x[0], x[0], fmaf(x[1], x[1], fmaf(x[2], x[2], x[3] * x[3]))));
+        sq += __shfl_xor(sq, 16, 64);
+        if (c < vdim)
+            store_gated(sh, x * (1.0f / sqrtf(sq / (float)vdim + sh.eps)) * w, (const T *)io.gate + (uint64_t)r * io.ld_gate + h * vdim + c,
+                        (T *)io.out + (uint64_t)r * io.ld_out + h * vdim + c);
+    }
+}
 template <typename T>
 __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaShape sh, DeltaIo io, RaggedRows rr, const float *__restrict__ o) {
     const uint32_t lane = threadIdx.x % 64, r = blockIdx.x, vdim = sh.vdim, b = rr.row_seq[r];
@@ -945,22 +984,7 @@ __global__ void __launch_bounds__(NT) delta_gate_all_kernel(DeltaShape sh, Delta
     }
     const float ro = io.out_scale / sqrtf(block_sum<float, NT / 64, true, true>(sq, smem) / (float)n + sh.eps);
     for (uint32_t c = threadIdx.x * S; c < n; c += NT * S) {
-        piece v = *(const piece *)(x + c) * ro * *(const piece *)(io.norm + c), z;
-        if constexpr (VEC && sizeof(T) == 2) {
-            const v2u u = *(const v2u *)(gate + c);
-            z = piece{bf16_lo(u[0]), bf16_hi(u[0]), bf16_lo(u[1]), bf16_hi(u[1])};
-        } else {
-#pragma unroll
-            for (int e = 0; e < (int)S; ++e) z[e] = load_as_f32(gate + c + e);
-        }
-#pragma unroll
-        for (int e = 0; e < (int)S; ++e) v[e] *= output_gate(sh.gate_sigmoid, z[e]);
-        if constexpr (VEC && sizeof(T) == 2) {
-            *(v2u *)(out + c) = v2u{f32x2_to_bf16x2(v[0], v[1]), f32x2_to_bf16x2(v[2], v[3])};
-        } else {
-#pragma unroll
-            for (int e = 0; e < (int)S; ++e) store_from_f32(out + c + e, v[e]);
-        }
+        store_gated(sh, *(const piece *)(x + c) * ro * *(const piece *)(io.norm + c), gate + c, out + c);
     }
 }
 
@@ -999,7 +1023,7 @@ void launch_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr
     } else if constexpr (KIND == Recurrence::kChannelDelta) {
         configure(&channel_chunk_kernel<T, KT, 4>, &channel_chunk_kernel<T, KT, 0>);
         auto chunk = sh.taps <= 4 ? &channel_chunk_kernel<T, KT, 4> : &channel_chunk_kernel<T, KT, 0>;
-        chunk<<<dim3(p.slots, sh.heads), 256, lds, s>>>(sh, io, rr, frags, p.frags);
+        chunk<<<dim3(p.slots, sh.heads), kChannelThreads, lds, s>>>(sh, io, rr, frags, p.frags);
     } else {
         configure(&lightning_chunk_kernel<T, KT>);
         lightning_chunk_kernel<T, KT><<<dim3(p.slots, sh.heads), 256, lds, s>>>(sh, io, rr, frags, decay, p.frags);
@@ -1014,7 +1038,9 @@ void launch_chunks(const DeltaShape &sh, const DeltaIo &io, const RaggedRows &rr
         scan_configured = true;
     }
     delta_scan_kernel<KT, KIND><<<dim3((p.vt + waves - 1) / waves, sh.heads, rr.batch), waves * 64, scan_lds, s>>>(sh, io, rr, frags, decay, io.raw, p.vt, p.frags);
-    if (!sh.norm_all) delta_gate_kernel<T><<<rr.rows, 256, 0, s>>>(sh, io, rr, io.raw);
+    if (sh.norm_all) return;                         // the whole pass's rows at the end
+    if (sh.vdim <= 128 && ((sh.vdim | io.ld_gate | io.ld_out) & 3) == 0) delta_gate_halves_kernel<T><<<rr.rows, 256, 0, s>>>(sh, io, rr);
+    else delta_gate_kernel<T><<<rr.rows, 256, 0, s>>>(sh, io, rr, io.raw);
 }
 
 template <typename T, Recurrence KIND>

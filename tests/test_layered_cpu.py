@@ -188,11 +188,136 @@ def test_another_reading_of_a_zoferax_mechanism_exceeds_the_gpu_tests_tolerance(
     assert lc.error(oracle.forward(cfg, w, toks), good) > 30 * 2e-4
 
 
+# ---- Bubetar ------------------------------------------------------------------------------------------------------
+
+def test_leading_rotation_of_either_layout_and_scaled_frequencies():
+    rng = np.random.default_rng(6)
+    x, pos = rng.normal(size=(4, 2, 10)), [0, 1, 7, 5000]
+    for interleaved in (True, False):
+        got = oracle.rotate_leading(x, pos, {"base": 50.0, "dims": 6}, interleaved)
+        assert np.allclose(got[..., 6:], x[..., 6:]) and np.allclose(got[0], x[0])
+        u, v = (np.arange(0, 6, 2), np.arange(1, 6, 2)) if interleaved else (np.arange(3), np.arange(3, 6))
+        for i in range(3):
+            a = np.array(pos) * 50.0 ** (-i / 3.0)
+            c, s = np.cos(a)[:, None], np.sin(a)[:, None]
+            assert np.allclose(got[..., u[i]], x[..., u[i]] * c - x[..., v[i]] * s) and np.allclose(got[..., v[i]], x[..., v[i]] * c + x[..., u[i]] * s)
+    assert np.allclose(oracle.rotate_leading(x, pos, {"base": 50.0, "dims": 10}, False), oracle.rotate(x, pos, 50.0))
+    turns = np.array([0.1, 1.0, 2.5, 4.0, 9.0])
+    f = oracle.scaled_frequencies(turns * 2 * np.pi / 64, {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 64}) * 64 / (2 * np.pi)
+    assert np.allclose(f, [0.1 / 8, 1.0 / 8, 2.5 * (0.5 / 8 + 0.5), 4.0, 9.0])
+
+
+def test_sink_takes_a_share_and_a_window_forgets():
+    rng = np.random.default_rng(7)
+    q, k, v = rng.normal(size=(6, 4, 5)), rng.normal(size=(6, 2, 5)), rng.normal(size=(6, 2, 3))
+    assert np.allclose(oracle.sink_attention(q, k, v, 0.6), oracle.grouped_attention(q, k, v, 0.6))
+    sink = rng.normal(size=4)
+    got = oracle.sink_attention(q, k, v, 0.6, 3, sink)
+    for t in range(6):
+        lo = max(0, t - 2)
+        for h in range(4):
+            e = np.exp(0.6 * k[lo:t + 1, h // 2] @ q[t, h])
+            assert np.allclose(got[t, h], e @ v[lo:t + 1, h // 2] / (e.sum() + np.exp(sink[h])))
+    assert np.allclose(oracle.sink_attention(q, k, v, 0.6, 1), np.repeat(v, 2, axis=1))
+
+
+def test_lightning_is_decayed_linear_attention():
+    rng = np.random.default_rng(8)
+    q, k, v, g = rng.normal(size=(7, 2, 4)), rng.normal(size=(7, 2, 4)), rng.normal(size=(7, 2, 3)), [0.6, 1.0]
+    got = oracle.lightning_recurrence(q, k, v, g)
+    for t in range(7):
+        for h in range(2):
+            assert np.allclose(got[t, h], sum(g[h] ** (t - s) * (q[t, h] @ k[s, h]) * v[s, h] for s in range(t + 1)))
+
+
+def test_channel_decays_reduce_to_one_decay_and_act_on_key_channels():
+    rng = np.random.default_rng(9)
+    q, k, v = rng.normal(size=(7, 2, 4)), oracle.unit_vector(rng.normal(size=(7, 2, 4))), rng.normal(size=(7, 2, 3))
+    beta, lg = rng.uniform(size=(7, 2)), -rng.uniform(size=(7, 2))
+    assert np.allclose(oracle.channel_delta_recurrence(q, k, v, beta, np.repeat(lg[:, :, None], 4, axis=2)), oracle.delta_recurrence(q, k, v, beta, lg))
+    # one write along two channels, then reads of each of them: every channel has faded by its own product
+    k, q = np.zeros((4, 1, 2)), np.zeros((4, 1, 2))
+    k[0, 0] = 0.6, 0.8
+    q[:, 0, 0] = 1.0
+    q[3, 0] = 0.0, 1.0
+    lg = -rng.uniform(size=(4, 1, 2))
+    got = oracle.channel_delta_recurrence(q, k, v[:4, :1], np.ones((4, 1)), lg)[:, 0]
+    assert np.allclose(got[2], 0.6 * np.exp(lg[1:3, 0, 0].sum()) * v[0, 0]) and np.allclose(got[3], 0.8 * np.exp(lg[1:4, 0, 1].sum()) * v[0, 0])
+
+
+def _mixers(c, kind):
+    return [l["mixer"] for l in c["layers"] if l["type"] == kind]
+
+
+BUBETAR_MISTAKES = {
+    "scale of the left mixer": lambda c: [m.update(left_scale=m["left_scale"] * 1.05) for m in _mixers(c, "parallel")],
+    "scale of the right mixer": lambda c: [m.update(right_scale=m["right_scale"] * 1.05) for m in _mixers(c, "parallel_2")],
+    "scores, gated": lambda c: [m["left"].update(scale=m["left"]["scale"] * 1.05) for m in _mixers(c, "parallel")],
+    "scores, key values": lambda c: [m["left"].update(scale=m["left"]["scale"] * 1.05) for m in _mixers(c, "parallel_2")],
+    "scores, latent": lambda c: [m.update(scale=m["scale"] * 1.05) for m in _mixers(c, "latent_attention")],
+    "rotation base": lambda c: [m["left"]["rot"].update(base=m["left"]["rot"]["base"] * 2) for m in _mixers(c, "parallel")],
+    "rotated part": lambda c: [m["left"]["rot"].update(dims=m["left"]["rot"]["dims"] - 2) for m in _mixers(c, "parallel_2")],
+    "no stretch": lambda c: [m["left"]["rot"].pop("scaling") for m in _mixers(c, "parallel_2")],
+    "stretch of another context": lambda c: [m["left"]["rot"]["scaling"].update(original=60) for m in _mixers(c, "parallel_2")],
+    "window one longer": lambda c: [m["left"]["mask"].update(size=m["left"]["mask"]["size"] + 1) for m in _mixers(c, "parallel_2")],
+    "window one shorter": lambda c: [m["left"]["mask"].update(size=m["left"]["mask"]["size"] - 1) for m in _mixers(c, "parallel_2")],
+    "decays of other heads": lambda c: [m["right"]["decay"].reverse() for m in _mixers(c, "parallel")],
+    "logit scale": lambda c: c.update(logit_scale=c["logit_scale"] * 1.1),
+    "soft cap": lambda c: c.update(logit_softcap=c["logit_softcap"] * 1.1),
+    "norm eps": lambda c: c["norm"].update(eps=0.05),
+    "feed-forward left out": lambda c: c["layers"][0].update(mlp=None),
+}
+
+
+def _bubetar():
+    cfg = lc.bubetar([lc.parallel(mlp=lc.dense()), lc.parallel_2(), lc.open_latent()], softcap=4.0)
+    return cfg, lc.weights(cfg, 5), lc.tokens(cfg, 40, 5)
+
+
+@pytest.mark.parametrize("name", sorted(BUBETAR_MISTAKES))
+def test_a_planted_mistake_in_a_bubetar_model_exceeds_the_gpu_tests_tolerance(name):
+    cfg, w, toks = _bubetar()
+    good = oracle.forward(cfg, w, toks)
+    wrong = copy.deepcopy(cfg)
+    BUBETAR_MISTAKES[name](wrong)
+    assert lc.error(oracle.forward(wrong, w, toks), good) > 30 * 2e-4
+
+
+@pytest.mark.parametrize("mistake", ["pairs of the other layout", "values behind the rotation", "a scaled sink", "no sink", "read before the write", "one decay for all channels",
+                                     "norm per head", "the state forgotten", "relu"])
+def test_another_reading_of_a_bubetar_mechanism_exceeds_the_gpu_tests_tolerance(mistake, monkeypatch):
+    cfg, w, toks = _bubetar()
+    good = oracle.forward(cfg, w, toks)
+    rotate, attend, light, channel = oracle.rotate_leading, oracle.sink_attention, oracle.lightning_recurrence, oracle.channel_delta_recurrence
+    if mistake == "pairs of the other layout":
+        monkeypatch.setattr(oracle, "rotate_leading", lambda x, p, rot, interleaved: rotate(x, p, rot, not interleaved))
+    elif mistake == "values behind the rotation":
+        monkeypatch.setattr(oracle, "sink_attention", lambda q, k, v, s, window=None, sink=None: attend(q, k, v if sink is None else k, s, window, sink))
+    elif mistake == "a scaled sink":
+        monkeypatch.setattr(oracle, "sink_attention", lambda q, k, v, s, window=None, sink=None: attend(q, k, v, s, window, None if sink is None else sink * s))
+    elif mistake == "no sink":
+        monkeypatch.setattr(oracle, "sink_attention", lambda q, k, v, s, window=None, sink=None: attend(q, k, v, s, window))
+    elif mistake == "read before the write":
+        monkeypatch.setattr(oracle, "lightning_recurrence", lambda q, k, v, d: light(q, k, v, d) - (q * k).sum(-1, keepdims=True) * v)
+    elif mistake == "one decay for all channels":
+        monkeypatch.setattr(oracle, "channel_delta_recurrence", lambda q, k, v, b, g: channel(q, k, v, b, np.repeat(g.mean(2, keepdims=True), g.shape[2], axis=2)))
+    elif mistake == "norm per head":
+        norm = oracle.rms_norm
+        n = cfg["layers"][0]["mixer"]["right"]
+        monkeypatch.setattr(oracle, "rms_norm", lambda x, g, eps: norm(x, g, eps) if x.shape[-1] != n["heads"] * n["vdim"] else
+                            norm(x.reshape(len(x), n["heads"], -1), 1.0, eps).reshape(x.shape) * g)
+    elif mistake == "the state forgotten":
+        monkeypatch.setattr(oracle, "lightning_recurrence", lambda q, k, v, d: np.concatenate([light(q[:20], k[:20], v[:20], d), light(q[20:], k[20:], v[20:], d)]))
+    else:
+        monkeypatch.setattr(oracle, "silu_glu", lambda h, v, p: (np.maximum(h @ v[p + "gate"].T, 0.0) * (h @ v[p + "up"].T)) @ v[p + "down"].T)
+    assert lc.error(oracle.forward(cfg, w, toks), good) > 30 * 2e-4
+
+
 # ---- configuration ---------------------------------------------------------------------------------------------
 
 def test_registry_picks_by_architecture_and_rejects_what_it_does_not_know(tmp_path):
     models = _fa().models
-    assert {"Nugelix", "Zoferax", "LlamaForCausalLM"} <= set(models.ARCHITECTURES)
+    assert {"Nugelix", "Zoferax", "Bubetar", "LlamaForCausalLM"} <= set(models.ARCHITECTURES)
     (tmp_path / "config.json").write_text(json.dumps({"architecture": "Nonesuch"}))
     with pytest.raises(models.ConfigError, match="unknown architecture"):
         models.load_model(None, str(tmp_path))
@@ -250,6 +375,46 @@ def test_zoferax_configuration_reads_every_size_and_names_what_is_missing():
         bad["layers"][1].update(change)
         with pytest.raises(models.ConfigError, match="unknown"):
             models.zoferax(bad)
+
+
+def test_bubetar_configuration_reads_every_size_and_names_what_is_missing():
+    fa = _fa()
+    models, capi = fa.models, fa.capi
+    cfg = lc.bubetar([lc.parallel(mlp=lc.dense(44)), lc.parallel_2(), lc.open_latent()], scale=0.3, ranks=(7, 11))
+    shapes = lc.shapes(cfg)
+    a = models.bubetar(cfg, shapes)
+    assert (a["d_model"], a["vocab"], a["norm"], a["logit_scale"], a["logit_softcap"], a["norm_eps"]) == (76, 131, capi.NORM_BOTH, 0.3, 12.0, 1e-5)
+    p, q, l = a["layers"]
+    assert (p["mixer"], p["heads"], p["kv_heads"], p["dim"], p["vdim"], p["rot_dim"], p["rot_base"], p["rot_interleaved"]) == (capi.MIXER_ATTENTION, 6, 2, 20, 12, 12, 3000.0, 1)
+    assert p["attention"] == capi.ATTENTION_HEAD_NORM | capi.ATTENTION_GATE and p.get("window", 0) == 0 and "rot_factor" not in p
+    assert (p["left_scale"], p["right_scale"], p["d_ffn"], p["glu"]) == (0.7, 1.3, 44, capi.GLU_SILU)
+    r = p["right"]
+    assert (r["mixer"], r["heads"], r["dim"], r["vdim"], len(r["decay"])) == (capi.MIXER_LIGHTNING, 3, 20, 28, 3)
+    assert q["attention"] == capi.ATTENTION_HEAD_UNIT | capi.ATTENTION_KEY_VALUES | capi.ATTENTION_SINK and (q["window"], q["rot_interleaved"]) == (11, 0)
+    assert (q["rot_factor"], q["rot_low"], q["rot_high"], q["rot_original"]) == (6.0, 1.0, 3.0, 90) and q.get("d_ffn", 0) == 0
+    r = q["right"]
+    assert (r["mixer"], r["kv_heads"], r["conv"], r["decay_rank"], r["gate_rank"]) == (capi.MIXER_DELTA, 2, 4, 7, 11)
+    assert (l["mixer"], l["ungated"], l["q_rank"], l["kv_rank"], l["rot_dim"], l.get("window", 0), l["rot_interleaved"]) == (capi.MIXER_LATENT_ATTENTION, 1, 36, 44, 12, 0, 1)
+    for layer, path in ((0, ("mixer", "left", "scale")), (0, ("mixer", "right", "decay")), (0, ("mixer", "left_scale")), (1, ("mixer", "right", "conv")),
+                        (1, ("mixer", "left", "rot", "scaling", "low")), (2, ("mixer", "q_rank")), (2, ("mixer", "rot", "dims")), (0, ("mlp", "ff")), (1, ("type",))):
+        bad = copy.deepcopy(cfg)
+        at = bad["layers"][layer]
+        for key in path[:-1]:
+            at = at[key]
+        del at[path[-1]]
+        with pytest.raises(models.ConfigError, match=path[-1]):
+            models.bubetar(bad, shapes)
+    with pytest.raises(models.ConfigError, match="a1"):
+        models.bubetar(cfg, {})
+    for change, word in (({"type": "other"}, "unknown type"), ({"mlp": {"kind": "moe"}}, "unknown feed-forward")):
+        bad = copy.deepcopy(cfg)
+        bad["layers"][2].update(change)
+        with pytest.raises(models.ConfigError, match=word):
+            models.bubetar(bad, shapes)
+    bad = copy.deepcopy(cfg)
+    bad["layers"][0]["mixer"]["right"]["decay"].pop()
+    with pytest.raises(models.ConfigError, match="decay"):
+        models.bubetar(bad, shapes)
 
 
 # ---- batching on a fake decoder ---------------------------------------------------------------------------------
