@@ -223,7 +223,8 @@ __global__ void __launch_bounds__(NT)
 }
 
 // ------------------------------------------------------------------ router
-// 16 rows per block; its four wavefronts take a quarter of k each and meet in LDS.  ET: tiles of 16 experts.
+// 16 rows per block; its four wavefronts take a quarter of k each and meet in LDS.  ET: tiles of 16 experts, those past the
+// weight's last one repeat it (nobody looks at their logits).
 template <int ET>
 __global__ void __launch_bounds__(256)
     route_kernel(const uint16_t *__restrict__ h, uint64_t ld, uint32_t rows, RouteIo io) {
@@ -236,7 +237,7 @@ __global__ void __launch_bounds__(256)
     v4f acc[ET];
 #pragma unroll
     for (int t = 0; t < ET; ++t) acc[t] = v4f{0.f, 0.f, 0.f, 0.f};
-    const uint32_t steps = (uint32_t)(ld / 32);
+    const uint32_t steps = (uint32_t)(ld / 32), last_tile = (io.experts + 15) / 16 - 1;
     constexpr int U = ET == 1 ? 8 : ET == 2 ? 4 : ET == 4 ? 2 : 1;       // k steps whose loads are in flight together
     for (uint32_t s0 = wave; s0 < steps; s0 += 4 * U) {
         v8bf hv[U], wv[U][ET];
@@ -245,7 +246,7 @@ __global__ void __launch_bounds__(256)
             const uint32_t s = s0 + 4 * u < steps ? s0 + 4 * u : s0;
             hv[u] = *(const v8bf *)(hp + (uint64_t)s * 32);
 #pragma unroll
-            for (int t = 0; t < ET; ++t) wv[u][t] = *(const v8bf *)(wp + ((uint64_t)t * steps + s) * 512);
+            for (int t = 0; t < ET; ++t) wv[u][t] = *(const v8bf *)(wp + ((uint64_t)((uint32_t)t < last_tile ? t : last_tile) * steps + s) * 512);
         }
 #pragma unroll
         for (int u = 0; u < U; ++u)
