@@ -135,11 +135,11 @@ def _bubetar(width, heads, kv_heads, q_rank, window, ff, repeat):
     grouped = dict(heads_of, kv_heads=kv_heads, scale=128 ** -0.5)
     lightning = dict(heads_of, decay=[1.0 - 2.0 ** (-1.0 - 8.0 * h / heads) for h in range(heads)])
     scaled = rot(64, scaling={"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192})
-    layers = [{"type": "parallel", "mlp": mlp, "mixer": {"left": dict(grouped, rot=rot(64)), "right": lightning, "left_scale": 0.8, "right_scale": 1.1}},
+    layers = [{"type": "parallel", "mlp": mlp, "mixer": {"left": dict(grouped, rot=rot(64)), "right": lightning, "left_scale": 1.0, "right_scale": 0.7}},
               {"type": "parallel_2", "mlp": mlp, "mixer": {"left": dict(grouped, rot=scaled, mask={"size": window}), "right": dict(heads_of, kv_heads=heads // 2, conv=4),
-                                                           "left_scale": 0.8, "right_scale": 1.1}}]
+                                                           "left_scale": 1.0, "right_scale": 0.7}}]
     latent = {"type": "latent_attention", "mlp": mlp, "mixer": dict(heads_of, rot_dim=64, q_rank=q_rank, kv_rank=512, rot=rot(64), scale=192 ** -0.5)}
-    return {"architecture": "Bubetar", "width": width, "vocab": 32000, "norm": {"eps": 1e-6}, "logit_scale": 0.5, "logit_softcap": 30.0,
+    return {"architecture": "Bubetar", "width": width, "vocab": 32000, "norm": {"eps": 1e-5}, "logit_scale": 0.7, "logit_softcap": 20.0,
             "layers": (layers + [latent, latent]) * repeat}
 
 
