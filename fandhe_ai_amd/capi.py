@@ -86,11 +86,12 @@ class DecoderConfig(C.Structure):
                 ("rope_theta", C.c_double)]
 
 
-MIXER_DELTA, MIXER_LATENT_ATTENTION, MIXER_ATTENTION, MIXER_LIGHTNING = 0, 1, 2, 3
-NORM_INPUT, NORM_OUTPUT, NORM_BOTH = 0, 1, 2
+MIXER_DELTA, MIXER_LATENT_ATTENTION, MIXER_ATTENTION, MIXER_LIGHTNING, MIXER_MINGRU = range(5)
+NORM_INPUT, NORM_OUTPUT, NORM_BOTH, NORM_INPUT_RMS = range(4)
 ATTENTION_BIAS, ATTENTION_QK_NORM, ATTENTION_HEAD_NORM, ATTENTION_HEAD_UNIT, ATTENTION_KEY_VALUES = 1, 2, 4, 8, 16
-ATTENTION_GATE, ATTENTION_SINK = 32, 64
-GLU_CLAMPED, GLU_SILU = 0, 1
+ATTENTION_GATE, ATTENTION_SINK, ATTENTION_SIGMOID, ATTENTION_HEAD_GATE = 32, 64, 128, 256
+GLU_CLAMPED, GLU_SILU, FFN_XIELU = 0, 1, 2
+ROUTE_CHOSEN, ROUTE_SCORED = 0, 1
 
 
 class LayerConfig(C.Structure):
@@ -104,7 +105,9 @@ LayerConfig._fields_ = [("mixer", C.c_int32), ("heads", C.c_uint32), ("dim", C.c
                         ("attention", C.c_uint32), ("experts", C.c_uint32), ("top", C.c_uint32), ("glu", C.c_int32),
                         ("rot_interleaved", C.c_uint32), ("rot_factor", C.c_double), ("rot_low", C.c_double), ("rot_high", C.c_double),
                         ("rot_original", C.c_double), ("ungated", C.c_uint32), ("decay_rank", C.c_uint32), ("gate_rank", C.c_uint32),
-                        ("decay", f32p), ("right", C.POINTER(LayerConfig)), ("left_scale", C.c_float), ("right_scale", C.c_float)]
+                        ("decay", f32p), ("right", C.POINTER(LayerConfig)), ("left_scale", C.c_float), ("right_scale", C.c_float),
+                        ("distance", C.c_float), ("q_temp", C.c_float), ("q_temp_every", C.c_uint32), ("route", C.c_int32),
+                        ("identity", C.c_uint32), ("groups", C.c_uint32), ("groups_kept", C.c_uint32), ("route_scale", C.c_float)]
 
 
 class LayeredConfig(C.Structure):

@@ -90,5 +90,18 @@ __device__ __forceinline__ float softmax_step(const float (&sc)[8], float &m, fl
     return fix;
 }
 
+// The weights of a step that no softmax normalizes: sigmoids of scores in powers of two (-inf: 0), as the same two bf16 terms.
+__device__ __forceinline__ void sigmoid_step(const float (&sc)[8], v8bf &w_hi, v8bf &w_lo) {
+    uint32_t hi[4], lo[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const float a = __builtin_amdgcn_rcpf(1.0f + exp2_fast(-sc[2 * i])), b = __builtin_amdgcn_rcpf(1.0f + exp2_fast(-sc[2 * i + 1]));
+        hi[i] = f32x2_to_bf16x2(a, b);
+        lo[i] = f32x2_to_bf16x2(a - bf16_lo(hi[i]), b - bf16_hi(hi[i]));
+    }
+    w_hi = __builtin_bit_cast(v8bf, v4u{hi[0], hi[1], hi[2], hi[3]});
+    w_lo = __builtin_bit_cast(v8bf, v4u{lo[0], lo[1], lo[2], lo[3]});
+}
+
 }  // namespace k
 }  // namespace fa

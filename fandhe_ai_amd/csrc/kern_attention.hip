@@ -1,5 +1,5 @@
 // Grouped-query attention over paged keys and values for ragged passes: consecutive query heads share a key / value head, keys
-// and values have sizes of their own; causal, in a window or over everything.
+// and values have sizes of their own; causal, in a window or over everything; softmax weights, or sigmoids of the scores.
 // The query rows of a (sequence, key head) are its (token, head in group) pairs in order; they are the columns of
 // S^T = K Q^T, in tiles of 16.
 #include <algorithm>
@@ -76,7 +76,7 @@ struct PrepareHeads {
 template <typename T, bool VEC>
 __global__ void __launch_bounds__(256)
     attention_prepare_heads_kernel(const float *__restrict__ y, uint32_t ld, PrepareHeads ph, T *__restrict__ q, T *__restrict__ k_pool, T *__restrict__ v_pool,
-                                   AttentionShape sh, const uint32_t *__restrict__ kv_slot, uint32_t group_log2) {
+                                   AttentionShape sh, const uint32_t *__restrict__ kv_slot, const int32_t *__restrict__ pos, uint32_t group_log2) {
     constexpr uint32_t S = VEC ? 4 : 1;
     typedef float piece __attribute__((ext_vector_type(S)));
     const uint32_t r = blockIdx.x, H = sh.heads, G = sh.kv_heads, lanes = 1u << group_log2, lane = threadIdx.x & (lanes - 1);
@@ -110,6 +110,7 @@ __global__ void __launch_bounds__(256)
             for (uint32_t off = lanes / 2; off > 0; off >>= 1) sq += __shfl_xor(sq, (int)off, 64);
             f = 1.0f / sqrtf(sq / (float)sh.dim + sh.eps);
         }
+        if (u < H && sh.q_temp != 0.0f) f *= 1.0f + sh.q_temp * logf((float)(((uint32_t)pos[r] + 1) / sh.q_temp_every) + 1.0f);
         auto normed = [&](uint32_t i) {
             piece v = *(const piece *)(src + i) * f;
             if (w) v *= *(const piece *)(w + i);
@@ -147,6 +148,10 @@ struct OutputPlace {
     const uint16_t *gate;
 };
 __device__ __forceinline__ float gate_value(float z) { return 1.0f / (1.0f + expf(-z)); }
+// What a (row, head) is multiplied by as a whole
+__device__ __forceinline__ float output_scale(const AttentionOutput &ao, uint64_t row, uint32_t head) {
+    return ao.head_gate ? ao.scale * gate_value(ao.head_gate[row * ao.ld_head_gate + head]) : ao.scale;
+}
 __device__ __forceinline__ void store_columns(const OutputPlace &at, uint32_t d, uint32_t vdim, v4f o) {
     if ((vdim & 3) == 0) {
         if (d >= vdim) return;
@@ -167,8 +172,8 @@ __device__ __forceinline__ OutputPlace output_place(uint16_t *out, uint32_t ld_o
 }
 
 // ------------------------------------------------------------------ plain form: any sizes, f32 or bf16
-// One block per (row, head).  Keys are taken 256 at a time, one per thread for the scores, with a running maximum and sum;
-// the threads then own value dims.
+// One block per (row, head).  Keys are taken 256 at a time, one per thread for the scores, with a running maximum and sum (of a
+// softmax); the threads then own value dims.
 constexpr uint32_t kPlainMaxV = 4096;
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -188,6 +193,7 @@ __global__ void __launch_bounds__(256)
     for (uint32_t i = 0; i < kPlainMaxV / 256; ++i) acc[i] = 0.0f;
     bool lost = false;                               // a position without a page: NaN, never a silent zero
     const int32_t first = p - (int32_t)sh.window + 1 > 0 ? p - (int32_t)sh.window + 1 : 0;
+    const float slope = ao.slope ? ao.slope[h] : 0.0f, bias = ao.bias ? ao.bias[h] : 0.0f;
     for (int32_t j0 = first; j0 <= p; j0 += 256) {
         __syncthreads();
         const int32_t j = j0 + (int32_t)threadIdx.x;
@@ -200,18 +206,25 @@ __global__ void __launch_bounds__(256)
                 const T *key = kp + (uint64_t)slot * kw;
                 float d = 0.0f;
                 for (uint32_t i = 0; i < sh.dim; ++i) d = fmaf(lq[i], load_as_f32(key + i), d);
-                s = d * sh.scale;
+                s = d * sh.scale - slope * (float)(p - j) + bias;
             } else {
                 s = __uint_as_float(0x7fc00000u);
             }
         }
         ids[threadIdx.x] = slot;
         lost = lost || s != s;
-        const float mc = fmaxf(m, block_max<4, true>(s, smem));
-        const float e = j <= p ? expf(s - mc) : 0.0f, fix = expf(m - mc);
-        w[threadIdx.x] = e;
-        l = l * fix + block_sum<float, 4, true>(e, smem);        // its barriers publish w and ids
-        m = mc;
+        float fix = 1.0f;
+        if (ao.sigmoid) {
+            w[threadIdx.x] = j <= p ? gate_value(s) : 0.0f;
+            __syncthreads();
+        } else {
+            const float mc = fmaxf(m, block_max<4, true>(s, smem));
+            const float e = j <= p ? expf(s - mc) : 0.0f;
+            fix = expf(m - mc);
+            w[threadIdx.x] = e;
+            l = l * fix + block_sum<float, 4, true>(e, smem);    // its barriers publish w and ids
+            m = mc;
+        }
         const int32_t n = p - j0 + 1 < 256 ? p - j0 + 1 : 256;
 #pragma unroll
         for (uint32_t i = 0; i < kPlainMaxV / 256; ++i) {
@@ -222,6 +235,7 @@ __global__ void __launch_bounds__(256)
             acc[i] = a;
         }
     }
+    if (ao.sigmoid) l = 1.0f;
     if (__syncthreads_or(lost)) l = __uint_as_float(0x7fc00000u);
     float f = 1.0f;                                  // of what was summed
     if (ao.sink) {
@@ -229,7 +243,7 @@ __global__ void __launch_bounds__(256)
         f = expf(m - mc);
         l = l * f + expf(sink - mc);
     }
-    f = f / l * ao.scale;
+    f = f / l * output_scale(ao, r, h);
     const T *gate = ao.gate ? (const T *)ao.gate + (uint64_t)r * ao.ld_gate + h * sh.vdim : nullptr;
 #pragma unroll
     for (uint32_t i = 0; i < kPlainMaxV / 256; ++i) {
@@ -242,12 +256,23 @@ __global__ void __launch_bounds__(256)
 __device__ __forceinline__ bool seen(int32_t p, int32_t j, int32_t W) { return (uint32_t)(p - j) < (uint32_t)W; }
 
 // Factor of what a column summed with maximum m (of scores in powers of two) and sum l of the weights: the sink takes its share
-// of the softmax here.
-__device__ __forceinline__ float final_factor(const AttentionOutput &ao, uint32_t head, float m, float l) {
-    if (!ao.sink) return ao.scale / l;
+// of the softmax here.  Sigmoid weights: l is 1 or NaN in every part of the sum.
+__device__ __forceinline__ float final_factor(const AttentionOutput &ao, uint64_t row, uint32_t head, float m, float l) {
+    const float scale = output_scale(ao, row, head);
+    if (ao.sigmoid) return l == l ? scale : l;
+    if (!ao.sink) return scale / l;
     const float sink = ao.sink[head] * kLog2e, mx = fmaxf(m, sink), f = exp2f(m - mx);
-    return ao.scale * f / (l * f + exp2f(sink - mx));
+    return scale * f / (l * f + exp2f(sink - mx));
 }
+
+// The scores of a column as sigmoid weights need them, in powers of two: factor a - slope distance + bias
+struct ColumnBias {
+    float slope, bias;
+};
+__device__ __forceinline__ ColumnBias column_bias(const AttentionOutput &ao, uint32_t head) {
+    return ColumnBias{ao.slope ? ao.slope[head] * kLog2e : 0.0f, ao.bias ? ao.bias[head] * kLog2e : 0.0f};
+}
+__device__ __forceinline__ float biased(float score, const ColumnBias &cb, int32_t distance) { return fmaf(-cb.slope, (float)distance, score + cb.bias); }
 
 // ------------------------------------------------------------------ few query rows
 // A block takes NQ column tiles of one (sequence, key head) and a share of the keys; its wavefronts walk that share 32 keys
@@ -264,7 +289,7 @@ struct StreamParams {
 };
 
 // D, V: dim_p and v_p in units of 32.
-template <int D, int V, int NQ, int NW>
+template <int D, int V, int NQ, int NW, bool SIGMOID>
 __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams p, AttentionShape sh, RaggedRows rr) {
     constexpr int VT = 2 * V, VP = V * 32 + 8, OP = V * 32 + 4;
     constexpr int CPR = V * 4, RPI = 64 / CPR, NV = kKeys / RPI;      // 16-byte pieces of a value row, rows per load, loads per step
@@ -328,6 +353,7 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
     v8bf qf[NQ][D];
     int32_t pos[NQ];
     float m[NQ], l[NQ];
+    ColumnBias cb[NQ];
     v4f o[NQ][VT];
     const bool any = first < k_hi;
     uint32_t id0 = 0, id1 = 0;
@@ -342,8 +368,9 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
         const uint16_t *src = p.q + ((uint64_t)(row0 + t) * sh.heads + kh * S + qc % S) * (D * 32) + 8 * g;
 #pragma unroll
         for (int s = 0; s < D; ++s) qf[qi][s] = *(const v8bf *)(src + s * 32);
-        m[qi] = -INFINITY;
-        l[qi] = 0.0f;
+        m[qi] = SIGMOID ? 0.0f : -INFINITY;
+        l[qi] = SIGMOID ? 1.0f : 0.0f;
+        if constexpr (SIGMOID) cb[qi] = column_bias(p.ao, kh * S + qc % S);
 #pragma unroll
         for (int t2 = 0; t2 < VT; ++t2) o[qi][t2] = v4f{0.f, 0.f, 0.f, 0.f};
     }
@@ -374,7 +401,9 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int32_t j = k0 + kt * 16 + 4 * g + e;
-                    sc[qi][kt * 4 + e] = seen(pos[qi], j, W) && j < k_hi ? acc[qi][e] * factor : -INFINITY;
+                    float v = acc[qi][e] * factor;
+                    if constexpr (SIGMOID) v = biased(v, cb[qi], pos[qi] - j);
+                    sc[qi][kt * 4 + e] = seen(pos[qi], j, W) && j < k_hi ? v : -INFINITY;
                 }
         }
         __builtin_amdgcn_sched_barrier(0);
@@ -387,10 +416,14 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
         v8bf w_hi[NQ], w_lo[NQ];
 #pragma unroll
         for (int qi = 0; qi < NQ; ++qi) {
-            const float fix = softmax_step(sc[qi], m[qi], l[qi], w_hi[qi], w_lo[qi]);
-            if (__any(fix != 1.0f)) {
+            if constexpr (SIGMOID) {
+                sigmoid_step(sc[qi], w_hi[qi], w_lo[qi]);
+            } else {
+                const float fix = softmax_step(sc[qi], m[qi], l[qi], w_hi[qi], w_lo[qi]);
+                if (__any(fix != 1.0f)) {
 #pragma unroll
-                for (int t = 0; t < VT; ++t) o[qi][t] *= fix;
+                    for (int t = 0; t < VT; ++t) o[qi][t] *= fix;
+                }
             }
         }
 #pragma unroll
@@ -408,8 +441,10 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
     }
 #pragma unroll
     for (int qi = 0; qi < NQ; ++qi) {
-        l[qi] += __shfl_xor(l[qi], 16, 64);
-        l[qi] += __shfl_xor(l[qi], 32, 64);
+        if constexpr (!SIGMOID) {
+            l[qi] += __shfl_xor(l[qi], 16, 64);
+            l[qi] += __shfl_xor(l[qi], 32, 64);
+        }
         if (__any(lost != 0)) l[qi] = __uint_as_float(0x7fc00000u);  // a position without a page: NaN, never a silent zero
     }
     // pairs of wavefronts meet, half of them left over every time
@@ -435,9 +470,9 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
             for (int qi = 0; qi < NQ; ++qi) {
                 const int at = wave * 16 * NQ + qi * 16 + c;
                 const float m1 = xm[at * 2], l1 = xm[at * 2 + 1], mx = fmaxf(m[qi], m1), ref = mx == -INFINITY ? 0.0f : mx;
-                const float f0 = exp2f(m[qi] - ref), f1 = exp2f(m1 - ref);
+                const float f0 = SIGMOID ? 1.0f : exp2f(m[qi] - ref), f1 = SIGMOID ? 1.0f : exp2f(m1 - ref);
                 m[qi] = mx;
-                l[qi] = l[qi] * f0 + l1 * f1;
+                l[qi] = SIGMOID ? l[qi] * l1 : l[qi] * f0 + l1 * f1;
 #pragma unroll
                 for (int t = 0; t < VT; ++t) o[qi][t] = o[qi][t] * f0 + *(const v4f *)(xo + at * OP + t * 16 + 4 * g) * f1;
             }
@@ -460,7 +495,7 @@ __global__ void __launch_bounds__(NW * 64) attention_stream_kernel(StreamParams 
         } else if (col < n_cols) {
             const uint32_t head = kh * S + col % S;
             const OutputPlace at = output_place(p.out, p.ld_out, p.ao, sh, row0 + col / S, head);
-            const float f = final_factor(p.ao, head, m[qi], l[qi]);
+            const float f = final_factor(p.ao, row0 + col / S, head, m[qi], l[qi]);
 #pragma unroll
             for (int t = 0; t < VT; ++t) store_columns(at, t * 16 + 4 * g, sh.vdim, o[qi][t] * f);
         }
@@ -481,7 +516,7 @@ __global__ void __launch_bounds__(64) attention_merge_kernel(StreamParams p, Att
         ls = v[1];
     }
     const uint32_t head = kh * S + col % S;
-    const float m = wave_max_dpp(ms), f = ls != 0.0f ? exp2f(ms - m) : 0.0f, w = f * final_factor(p.ao, head, m, wave_sum_dpp(ls * f));
+    const float m = wave_max_dpp(ms), f = ls != 0.0f ? exp2f(ms - m) : 0.0f, w = f * final_factor(p.ao, row0 + col / S, head, m, wave_sum_dpp(ls * f));
     const OutputPlace out = output_place(p.out, p.ld_out, p.ao, sh, row0 + col / S, head);
     for (uint32_t d = lane * 4; d < sh.v_p; d += 256) {
         const float *src = p.part_o + at * sh.v_p + d;
@@ -503,7 +538,7 @@ __global__ void __launch_bounds__(64) attention_merge_kernel(StreamParams p, Att
 // ------------------------------------------------------------------ many query rows
 // A block of four wavefronts takes 64 NQ columns of one (sequence, key head), every wavefront 16 NQ of them, and walks the keys
 // they see 32 at a time; K and V of a step are staged in LDS, two stages.
-template <int D, int V, int NQ>
+template <int D, int V, int NQ, bool SIGMOID>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
     attention_flash_kernel(const uint16_t *__restrict__ q, const uint16_t *__restrict__ k_pool, const uint16_t *__restrict__ v_pool,
                            uint16_t *__restrict__ out, uint32_t ld_out, AttentionOutput ao, uint32_t max_cols, AttentionShape sh, RaggedRows rr) {
@@ -529,10 +564,12 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
     const int32_t W = (int32_t)sh.window, k_hi = pos_of(c0 + BC - 1) + 1, p_lo = pos_of(c0), k_lo = p_lo - W + 1 > 0 ? p_lo - W + 1 : 0;
     v8bf qf[NQ][D];
     int32_t pos[NQ];
+    ColumnBias cb[NQ];
 #pragma unroll
     for (int qi = 0; qi < NQ; ++qi) {
         const uint32_t col = c0 + (wave * NQ + qi) * 16 + c, qc = col < n_cols ? col : n_cols - 1;
         pos[qi] = pos_of(col);
+        if constexpr (SIGMOID) cb[qi] = column_bias(ao, kh * S + qc % S);
         const uint16_t *src = q + ((uint64_t)(row0 + qc / S) * sh.heads + kh * S + qc % S) * (D * 32) + 8 * g;
 #pragma unroll
         for (int s = 0; s < D; ++s) qf[qi][s] = *(const v8bf *)(src + s * 32);
@@ -609,6 +646,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         float v = acc[qi][e] * factor;
+                        if constexpr (SIGMOID) v = biased(v, cb[qi], pos[qi] - (k0 + kt * 16 + 4 * g + e));
                         if (!inside && !seen(pos[qi], k0 + kt * 16 + 4 * g + e, W)) v = -INFINITY;
                         sc[qi][kt * 4 + e] = v;
                     }
@@ -616,10 +654,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
             v8bf w_hi[NQ], w_lo[NQ];
 #pragma unroll
             for (int qi = 0; qi < NQ; ++qi) {
-                const float fix = softmax_step(sc[qi], m[qi], l[qi], w_hi[qi], w_lo[qi]);
-                if (__any(fix != 1.0f)) {
+                if constexpr (SIGMOID) {
+                    sigmoid_step(sc[qi], w_hi[qi], w_lo[qi]);
+                } else {
+                    const float fix = softmax_step(sc[qi], m[qi], l[qi], w_hi[qi], w_lo[qi]);
+                    if (__any(fix != 1.0f)) {
 #pragma unroll
-                    for (int t = 0; t < VT; ++t) o[qi][t] *= fix;
+                        for (int t = 0; t < VT; ++t) o[qi][t] *= fix;
+                    }
                 }
             }
 #pragma unroll
@@ -637,13 +679,15 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3)))
     }
 #pragma unroll
     for (int qi = 0; qi < NQ; ++qi) {
-        float sum = l[qi];
-        sum += __shfl_xor(sum, 16, 64);
-        sum += __shfl_xor(sum, 32, 64);
+        float sum = SIGMOID ? 1.0f : l[qi];
+        if constexpr (!SIGMOID) {
+            sum += __shfl_xor(sum, 16, 64);
+            sum += __shfl_xor(sum, 32, 64);
+        }
         const uint32_t col = c0 + (wave * NQ + qi) * 16 + c;
         if (col >= n_cols) continue;
         const uint32_t head = kh * S + col % S;
-        const float f = final_factor(ao, head, m[qi], sum);
+        const float f = final_factor(ao, row0 + col / S, head, m[qi], sum);
         const OutputPlace at = output_place(out, ld_out, ao, sh, row0 + col / S, head);
 #pragma unroll
         for (int t = 0; t < VT; ++t) store_columns(at, t * 16 + 4 * g, sh.vdim, o[qi][t] * f);
@@ -657,9 +701,9 @@ struct AttentionPlan {
     int nq = 1;
     uint32_t tiles = 1, splits = 1;
 };
-AttentionPlan attention_plan(const AttentionShape &sh, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx, int num_cus) {
+AttentionPlan attention_plan(const AttentionShape &sh, const AttentionOutput &ao, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx, int num_cus) {
     AttentionPlan p;
-    if (is_f32 || sh.dim_p > 256 || sh.v_p > 256 || g_attention_form == 1) {
+    if (is_f32 || sh.dim_p > 256 || sh.v_p > 256 || g_attention_form == 1 || (ao.slope && !ao.sigmoid)) {
         p.plain = true;
         return p;
     }
@@ -681,7 +725,7 @@ AttentionPlan attention_plan(const AttentionShape &sh, int is_f32, uint32_t batc
 
 constexpr int stream_waves(int d, int v) { return d == 8 || v == 8 ? 4 : 8; }
 
-template <int D, int V, int NQ>
+template <int D, int V, int NQ, bool SIGMOID>
 void launch_stream(const StreamParams &p, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s) {
     constexpr int NW = stream_waves(D, V);
     constexpr size_t stage = (size_t)NW * kKeys * (V * 32 + 8) * 2, meet = (size_t)NW / 2 * 16 * NQ * ((V * 32 + 4) * 4 + 8);
@@ -690,19 +734,19 @@ void launch_stream(const StreamParams &p, const AttentionShape &sh, const Ragged
     if constexpr (lds > 65536) {
         static bool configured = false;
         if (!configured) {
-            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&attention_stream_kernel<D, V, NQ, NW>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&attention_stream_kernel<D, V, NQ, NW, SIGMOID>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
             configured = true;
         }
     }
-    attention_stream_kernel<D, V, NQ, NW><<<dim3(rr.batch * p.tiles, sh.kv_heads, p.splits), NW * 64, lds, s>>>(p, sh, rr);
+    attention_stream_kernel<D, V, NQ, NW, SIGMOID><<<dim3(rr.batch * p.tiles, sh.kv_heads, p.splits), NW * 64, lds, s>>>(p, sh, rr);
     if (p.splits > 1) attention_merge_kernel<<<dim3(rr.batch * p.tiles, sh.kv_heads, 16 * NQ), 64, 0, s>>>(p, sh, rr, 16 * NQ);
 }
 
-template <int D, int V>
-void launch_matrix(const AttentionPlan &plan, const StreamParams &p, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s) {
+template <int D, int V, bool SIGMOID>
+void launch_matrix_kind(const AttentionPlan &plan, const StreamParams &p, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s) {
     if (plan.stream) {
-        if (plan.nq == 1) launch_stream<D, V, 1>(p, sh, rr, s);
-        else launch_stream<D, V, 2>(p, sh, rr, s);
+        if (plan.nq == 1) launch_stream<D, V, 1, SIGMOID>(p, sh, rr, s);
+        else launch_stream<D, V, 2, SIGMOID>(p, sh, rr, s);
     }
     if (plan.flash) {
         constexpr int NQ = D == 8 || V == 8 ? 1 : 2;
@@ -710,13 +754,18 @@ void launch_matrix(const AttentionPlan &plan, const StreamParams &p, const Atten
         if constexpr (lds > 65536) {
             static bool configured = false;
             if (!configured) {
-                (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&attention_flash_kernel<D, V, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+                (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&attention_flash_kernel<D, V, NQ, SIGMOID>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
                 configured = true;
             }
         }
         const dim3 grid((uint32_t)((uint64_t)rr.rows * sh.share() / (64 * NQ)) + rr.batch, sh.kv_heads);
-        attention_flash_kernel<D, V, NQ><<<grid, 256, lds, s>>>(p.q, p.k_pool, p.v_pool, p.out, p.ld_out, p.ao, plan.max_cols, sh, rr);
+        attention_flash_kernel<D, V, NQ, SIGMOID><<<grid, 256, lds, s>>>(p.q, p.k_pool, p.v_pool, p.out, p.ld_out, p.ao, plan.max_cols, sh, rr);
     }
+}
+template <int D, int V>
+void launch_matrix(const AttentionPlan &plan, const StreamParams &p, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s) {
+    if (p.ao.sigmoid) launch_matrix_kind<D, V, true>(plan, p, sh, rr, s);
+    else launch_matrix_kind<D, V, false>(plan, p, sh, rr, s);
 }
 template <int D>
 void launch_matrix_v(const AttentionPlan &plan, const StreamParams &p, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s) {
@@ -762,7 +811,7 @@ void attention_prepare_heads(const float *y, uint32_t ld, bool norms, const floa
     const uint32_t groups = 256u >> group_log2, units = sh.heads + 2 * sh.kv_heads;
     const dim3 grid(rr.rows, rr.rows <= 256 ? (units + groups - 1) / groups : 1);
 #define FA_PREP(T_, VEC_) \
-    attention_prepare_heads_kernel<T_, VEC_><<<grid, 256, 0, s>>>(y, ld, ph, (T_ *)q, (T_ *)k_pool, (T_ *)v_pool, sh, rr.kv_slot, group_log2)
+    attention_prepare_heads_kernel<T_, VEC_><<<grid, 256, 0, s>>>(y, ld, ph, (T_ *)q, (T_ *)k_pool, (T_ *)v_pool, sh, rr.kv_slot, rr.pos, group_log2)
     if (is_f32) {
         if (vec) FA_PREP(float, true);
         else FA_PREP(float, false);
@@ -773,16 +822,16 @@ void attention_prepare_heads(const float *y, uint32_t ld, bool norms, const floa
 #undef FA_PREP
 }
 
-uint64_t attention_workspace_bytes(const AttentionShape &sh, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
+uint64_t attention_workspace_bytes(const AttentionShape &sh, const AttentionOutput &ao, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
                                    int num_cus) {
-    const AttentionPlan p = attention_plan(sh, is_f32, batch, min_new, max_new, max_ctx, num_cus);
+    const AttentionPlan p = attention_plan(sh, ao, is_f32, batch, min_new, max_new, max_ctx, num_cus);
     return p.splits > 1 ? (uint64_t)batch * p.tiles * sh.kv_heads * p.splits * 16 * p.nq * (sh.v_p + 2) * 4 : 0;
 }
 
 void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, const AttentionOutput &ao, int is_f32,
                const AttentionShape &sh, const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s) {
     if (rr.rows == 0) return;
-    const AttentionPlan plan = attention_plan(sh, is_f32, rr.batch, min_new, max_new, rr.max_blocks * rr.block_size, num_cus);
+    const AttentionPlan plan = attention_plan(sh, ao, is_f32, rr.batch, min_new, max_new, rr.max_blocks * rr.block_size, num_cus);
     if (plan.plain) {
         const dim3 grid(rr.rows, sh.heads);
         if (is_f32)

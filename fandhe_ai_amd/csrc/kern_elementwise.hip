@@ -271,6 +271,7 @@ __global__ void __launch_bounds__(256)
                 v = v * scale + (float)(e ? cs : sn);
                 x[r * cols + c + e] = v;
             }
+            if (!hn) continue;
             if constexpr (sizeof(T) == 4) hn[r * ld + c + e] = v;
             else hn[r * ld + c + e] = f32_to_bf16(v);
         }

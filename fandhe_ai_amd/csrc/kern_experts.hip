@@ -1,5 +1,5 @@
-// Sublayers that norm their output, and the routing of sparse feed-forwards: the residual update with its norm, the weighted
-// sum of a row's experts, the router with the choice of experts.  The experts' linears are kern_linear.hip's.
+// Residual updates with the norms around them, and the routing of sparse feed-forwards: the weighted sum of a row's experts, the
+// router with the choice of experts.  The experts' linears are kern_linear.hip's.
 #include <algorithm>
 
 #include "attention_tiles.hpp"
@@ -60,15 +60,123 @@ __device__ __forceinline__ void choose_experts(const float *logits, uint32_t exp
     *weight = bad ? __uint_as_float(0x7fc00000u) : e / sum;
 }
 
+// The scored choice: softmax over all outputs, the `top` largest s + correction out of the best groups.  Lane i < top returns with
+// the i-th chosen output in `id` and its weight in `weight`.  row: the logits (LDS), overwritten; open: LDS of the wavefront, a
+// flag per group.
+__device__ __forceinline__ void choose_scored(float *row, uint32_t *open, const RouteIo &io, int lane, uint32_t *id, float *weight) {
+    constexpr uint32_t N = kMaxExperts / 64;
+    float s[N], c[N], mx = -INFINITY, sum = 0.0f;
+    bool bad = false;
+#pragma unroll
+    for (uint32_t i = 0; i < N; ++i) {
+        const uint32_t e = i * 64 + lane;
+        s[i] = e < io.experts ? row[e] : -INFINITY;
+        bad = bad || s[i] != s[i];
+        mx = fmaxf(mx, s[i]);
+    }
+    bad = __any(bad);
+    mx = wave_max_dpp(mx);
+#pragma unroll
+    for (uint32_t i = 0; i < N; ++i) {
+        s[i] = i * 64 + lane < io.experts ? expf(s[i] - mx) : 0.0f;
+        sum += s[i];
+    }
+    sum = wave_sum_dpp(sum);
+    const uint32_t size = io.experts / io.groups;
+    const bool all = io.keep >= io.groups;
+#pragma unroll
+    for (uint32_t i = 0; i < N; ++i) {
+        const uint32_t e = i * 64 + lane;
+        s[i] /= sum;
+        c[i] = bad || e >= io.experts ? 0.0f : s[i] + io.correction[e];
+        if (!all && e < io.experts) row[e] = c[i];
+    }
+    if (!all) {
+        __builtin_amdgcn_wave_barrier();
+        float best[N];                               // of the groups lane, lane + 64, ..
+#pragma unroll
+        for (uint32_t i = 0; i < N; ++i) {
+            best[i] = -INFINITY;
+            const uint32_t g = i * 64 + lane;
+            if (g < io.groups)
+                for (uint32_t j = 0; j < size; ++j) best[i] = fmaxf(best[i], row[g * size + j]);
+        }
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (uint32_t i = 0; i < N; ++i)
+            if (i * 64 + lane < io.groups) row[i * 64 + lane] = best[i];
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (uint32_t i = 0; i < N; ++i) {
+            const uint32_t g = i * 64 + lane;
+            if (g >= io.groups) continue;
+            uint32_t ahead = 0;
+            for (uint32_t o = 0; o < io.groups; ++o) ahead += row[o] > best[i] || (row[o] == best[i] && o < g);
+            open[g] = ahead < io.keep;
+        }
+        __builtin_amdgcn_wave_barrier();
+    }
+    uint32_t taken = 0;                              // bit i: this lane's value i cannot be chosen (any more)
+#pragma unroll
+    for (uint32_t i = 0; i < N; ++i) {
+        const uint32_t e = i * 64 + lane;
+        if (e >= io.experts || (!all && !open[e / size])) taken |= 1u << i;
+    }
+    float mine = 0.0f;
+    *id = 0;
+    for (uint32_t t = 0; t < io.top; ++t) {
+        float best = -INFINITY, best_s = 0.0f;
+        uint32_t at = 0xffffffffu;
+#pragma unroll
+        for (uint32_t i = 0; i < N; ++i)
+            if (!(taken >> i & 1) && (at == 0xffffffffu || c[i] > best)) {
+                best = c[i];
+                best_s = s[i];
+                at = i * 64 + lane;
+            }
+        const float top_c = wave_max_dpp(best);
+        uint32_t cand = at != 0xffffffffu && best == top_c ? at : 0xffffffffu;
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) {
+            const uint32_t o = (uint32_t)__shfl_xor((int)cand, off, 64);
+            cand = o < cand ? o : cand;
+        }
+        const float cand_s = __shfl(best_s, (int)(cand % 64), 64);
+        if ((uint32_t)lane == cand % 64) taken |= 1u << (cand / 64);
+        if ((uint32_t)lane == t) {
+            mine = cand_s;
+            *id = cand;
+        }
+    }
+    const float total = wave_sum_dpp(mine) + 1e-20f;
+    *weight = bad ? __uint_as_float(0x7fc00000u) : mine / total * io.scale;
+}
+
+// The experts of row r from its logits (LDS): gates stored; true in the lanes whose expert has a list.
+__device__ __forceinline__ bool choose_row(float *logits, uint32_t *open, const RouteIo &io, uint64_t r, bool store, int lane, uint32_t *id) {
+    float w;
+    if (io.scored) choose_scored(logits, open, io, lane, id, &w);
+    else choose_experts(logits, io.experts, io.top, lane, id, &w);
+    const bool own = (uint32_t)lane < io.top, listed = own && *id < io.experts - io.identity;
+    if (io.identity_gate) {
+        const float sum = wave_sum_dpp(own && !listed ? w : 0.0f);
+        if (store && lane == 0) io.identity_gate[r] = sum;
+    }
+    if (store && own) io.gate[r * io.top + lane] = listed ? w : 0.0f;
+    return listed;
+}
+
 // ------------------------------------------------------------------ residual update
 // One block per row, VPT pieces of it per thread: four values each (VEC, hidden a multiple of four), or one.
-// LAYER: layer norm of the output, and of the new x for the next sublayer.
-template <typename T, int VPT, int NT, bool ROUTE, bool VEC, bool LAYER>
+// KIND: ResidualNorm::Kind.
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC, int KIND>
 __global__ void __launch_bounds__(NT)
     residual_norm_kernel(ResidualNorm rn, float *__restrict__ x, T *__restrict__ hn, uint32_t hidden, uint64_t ld, RouteIo io) {
     constexpr int NW = NT / 64, S = VEC ? 4 : 1;
+    constexpr bool LAYER = KIND == ResidualNorm::kBoth, INPUT = KIND == ResidualNorm::kInput;
     typedef float piece __attribute__((ext_vector_type(S)));
     __shared__ float smem[LAYER ? 4 : 1][NW], logits[ROUTE ? kMaxExperts : 1];
+    __shared__ uint32_t open[ROUTE ? kMaxExperts : 1];
     extern __shared__ __attribute__((aligned(16))) uint8_t hs_raw[];     // ROUTE: the row of hn
     const uint64_t r = blockIdx.x;
     const int tid = threadIdx.x;
@@ -82,7 +190,7 @@ __global__ void __launch_bounds__(NT)
         const uint32_t c = (tid + i * NT) * S;
         v[i] = piece(0.0f);
         xv[i] = c < hidden ? *(const piece *)(xr + c) : piece(0.0f);
-        if (!rn.gate && c < hidden) v[i] = *(const piece *)(y + c);
+        if (!rn.gate && (!INPUT || rn.y) && c < hidden) v[i] = *(const piece *)(y + c);
     }
     if (rn.gate) {
         for (uint32_t p = 0; p < rn.parts; p += 2) {                     // two parts at a time, in order
@@ -93,14 +201,43 @@ __global__ void __launch_bounds__(NT)
 #pragma unroll
             for (int i = 0; i < VPT; ++i) {
                 const uint32_t c = (tid + i * NT) * S;
-                t0[i] = c < hidden ? *(const piece *)(y0 + c) : piece(0.0f);
-                t1[i] = c < hidden && two ? *(const piece *)(y1 + c) : piece(0.0f);
+                t0[i] = c < hidden && g0 != 0.0f ? *(const piece *)(y0 + c) : piece(0.0f);
+                t1[i] = c < hidden && g1 != 0.0f ? *(const piece *)(y1 + c) : piece(0.0f);
             }
 #pragma unroll
             for (int i = 0; i < VPT; ++i)
 #pragma unroll
                 for (int e = 0; e < S; ++e) v[i][e] = fmaf(g1, t1[i][e], fmaf(g0, t0[i][e], v[i][e]));
         }
+        const float gi = rn.identity_gate ? rn.identity_gate[r] : 0.0f;
+        if (gi != 0.0f) {
+#pragma unroll
+            for (int i = 0; i < VPT; ++i) {
+                const uint32_t c = (tid + i * NT) * S;
+                if (c >= hidden) continue;
+                const T *h = hn + r * ld + c;
+                piece t;
+                if constexpr (sizeof(T) == 4) {
+                    t = *(const piece *)h;
+                } else if constexpr (VEC) {
+                    const v2u b = *(const v2u *)h;
+                    t = piece{bf16_lo(b[0]), bf16_hi(b[0]), bf16_lo(b[1]), bf16_hi(b[1])};
+                } else {
+                    t = piece(bf16_to_f32(*h));
+                }
+#pragma unroll
+                for (int e = 0; e < S; ++e) v[i][e] = fmaf(gi, t[e], v[i][e]);
+            }
+        }
+    }
+    if constexpr (INPUT) {
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const uint32_t c = (tid + i * NT) * S;
+            xv[i] += v[i];
+            if (rn.y && c < hidden) *(piece *)(xr + c) = xv[i];
+        }
+        if (!rn.next) return;
     }
     // of the row behind v: its mean is taken off, the root of the mean square returned inverted
     auto center = [&](piece (&t)[VPT], float *s_mean, float *s_var) {
@@ -122,7 +259,7 @@ __global__ void __launch_bounds__(NT)
             for (int e = 0; e < S; ++e) q = fmaf(t[i][e], t[i][e], q);
         return 1.0f / sqrtf(block_sum<float, NW, true, true>(q, s_var) / (float)hidden + rn.eps);
     };
-    const float rstd = LAYER ? center(v, smem[LAYER], smem[0]) : center(v, nullptr, smem[0]);
+    const float rstd = LAYER ? center(v, smem[LAYER], smem[0]) : center(INPUT ? xv : v, nullptr, smem[0]);
     if constexpr (LAYER) {
 #pragma unroll
         for (int i = 0; i < VPT; ++i) {
@@ -153,7 +290,9 @@ __global__ void __launch_bounds__(NT)
         const uint32_t c = (tid + i * NT) * S;
         if (c >= ld) continue;
         piece o = piece(0.0f);
-        if (c < hidden) {
+        if (INPUT) {
+            if (c < hidden) o = xv[i] * rstd * *(const piece *)(rn.next + c);
+        } else if (c < hidden) {
             const piece w = *(const piece *)(rn.w + c);
 #pragma unroll
             for (int e = 0; e < S; ++e) o[e] = xv[i][e] + v[i][e] * rstd * w[e];
@@ -211,10 +350,7 @@ __global__ void __launch_bounds__(NT)
         __syncthreads();
         if (wave == 0) {
             uint32_t id;
-            float g;
-            choose_experts(logits, io.experts, io.top, lane, &id, &g);
-            if ((uint32_t)lane < io.top) {
-                io.gate[r * io.top + lane] = g;
+            if (choose_row(logits, open, io, r, true, lane, &id)) {
                 const uint32_t at = atomicAdd(io.count + id, 1u);
                 if (at < io.pitch) io.list[(uint64_t)id * io.pitch + at] = (uint32_t)(r * io.top + lane);
             }
@@ -229,7 +365,7 @@ template <int ET>
 __global__ void __launch_bounds__(256)
     route_kernel(const uint16_t *__restrict__ h, uint64_t ld, uint32_t rows, RouteIo io) {
     extern __shared__ __attribute__((aligned(16))) float part[];         // [4][ET * 16][17]
-    __shared__ uint32_t cnt[kMaxExperts], base[kMaxExperts];
+    __shared__ uint32_t cnt[kMaxExperts], base[kMaxExperts], open[4][kMaxExperts];
     __shared__ float logits[16][ET * 16 + 1];
     const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), g = lane / 16, c = lane % 16;
     const uint32_t r0 = blockIdx.x * 16, row = r0 + c < rows ? r0 + c : rows - 1;
@@ -267,49 +403,47 @@ __global__ void __launch_bounds__(256)
     }
     __syncthreads();
     uint32_t id[4], at[4];
+    bool listed[4];
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
         const uint32_t rr = wave * 4 + q;
-        float w;
-        choose_experts(logits[rr], io.experts, io.top, lane, &id[q], &w);
-        at[q] = 0;
-        if (r0 + rr < rows && (uint32_t)lane < io.top) {
-            io.gate[(uint64_t)(r0 + rr) * io.top + lane] = w;
-            at[q] = atomicAdd(&cnt[id[q]], 1u);
-        }
+        const bool there = r0 + rr < rows;
+        listed[q] = choose_row(logits[rr], open[wave], io, r0 + rr, there, lane, &id[q]) && there;
+        at[q] = listed[q] ? atomicAdd(&cnt[id[q]], 1u) : 0;
     }
     __syncthreads();
-    for (uint32_t e = tid; e < io.experts; e += 256)
+    for (uint32_t e = tid; e < io.experts - io.identity; e += 256)
         if (cnt[e]) base[e] = atomicAdd(io.count + e, cnt[e]);
     __syncthreads();
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
         const uint32_t rr = wave * 4 + q;
-        if (r0 + rr < rows && (uint32_t)lane < io.top) {
+        if (listed[q]) {
             const uint32_t p = base[id[q]] + at[q];
             if (p < io.pitch) io.list[(uint64_t)id[q] * io.pitch + p] = (uint32_t)((r0 + rr) * io.top + lane);
         }
     }
 }
 
-template <typename T, int VPT, int NT, bool ROUTE, bool VEC, bool LAYER>
+template <typename T, int VPT, int NT, bool ROUTE, bool VEC, int KIND>
 void launch_residual_kind(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
     const size_t lds = ROUTE ? ld * sizeof(T) + (sizeof(T) == 2 ? (io.experts + 15) / 16 * 16 * 17 * 4 : 0) : 0;
     if (ROUTE && lds > 49152) {
         static bool configured = false;
         if (!configured) {
-            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, VPT, NT, ROUTE, VEC, LAYER>), hipFuncAttributeMaxDynamicSharedMemorySize,
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&residual_norm_kernel<T, VPT, NT, ROUTE, VEC, KIND>), hipFuncAttributeMaxDynamicSharedMemorySize,
                                       98304);
             configured = true;
         }
     }
-    residual_norm_kernel<T, VPT, NT, ROUTE, VEC, LAYER><<<(unsigned)rows, NT, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);
+    residual_norm_kernel<T, VPT, NT, ROUTE, VEC, KIND><<<(unsigned)rows, NT, lds, s>>>(rn, x, hn, (uint32_t)hidden, ld, io);
 }
 template <typename T, int VPT, int NT, bool ROUTE, bool VEC>
 void launch_residual_sized(const ResidualNorm &rn, float *x, T *hn, uint64_t rows, uint64_t hidden, uint64_t ld, const RouteIo &io, hipStream_t s) {
     if constexpr (!ROUTE)
-        if (rn.layer) return launch_residual_kind<T, VPT, NT, false, VEC, true>(rn, x, hn, rows, hidden, ld, io, s);
-    launch_residual_kind<T, VPT, NT, ROUTE, VEC, false>(rn, x, hn, rows, hidden, ld, io, s);
+        if (rn.kind == ResidualNorm::kBoth) return launch_residual_kind<T, VPT, NT, false, VEC, ResidualNorm::kBoth>(rn, x, hn, rows, hidden, ld, io, s);
+    if (rn.kind == ResidualNorm::kInput) launch_residual_kind<T, VPT, NT, ROUTE, VEC, ResidualNorm::kInput>(rn, x, hn, rows, hidden, ld, io, s);
+    else launch_residual_kind<T, VPT, NT, ROUTE, VEC, ResidualNorm::kOutput>(rn, x, hn, rows, hidden, ld, io, s);
 }
 
 // rows up to 16384 values
@@ -354,6 +488,14 @@ void residual_norm(const ResidualNorm &rn, float *x, void *hn, int is_f32, uint6
         else launch_residual<uint16_t, false>(rn, x, (uint16_t *)hn, rows, hidden, ld, RouteIo{}, s);
     }
 }
+
+namespace {
+__global__ void xielu_constants_kernel(const float *pq, float *act) {
+    const float z = pq[threadIdx.x];
+    act[threadIdx.x] = fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))) + (threadIdx.x ? 0.5f : 0.0f);
+}
+}  // namespace
+void xielu_constants(const float *pq, float *act, hipStream_t s) { xielu_constants_kernel<<<1, 2, 0, s>>>(pq, act); }
 
 void route_rows(const void *h_bf16, uint64_t rows, uint64_t ld, const RouteIo &io, hipStream_t s) {
     if (rows == 0) return;

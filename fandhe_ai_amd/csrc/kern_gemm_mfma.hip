@@ -1181,6 +1181,7 @@ void gemm_bf16_big(const uint16_t *a, uint64_t m, const LinearWeight &w, const L
         case LinearEpilogue::kResidual: return launch_big_bf16<LinearEpilogue::kResidual>(a, m, w, ep, ntb, s);
         case LinearEpilogue::kGlu: return launch_big_bf16<LinearEpilogue::kGlu>(a, m, w, ep, ntb, s);
         case LinearEpilogue::kSiluGlu: return launch_big_bf16<LinearEpilogue::kSiluGlu>(a, m, w, ep, ntb, s);
+        case LinearEpilogue::kXielu: return launch_big_bf16<LinearEpilogue::kXielu>(a, m, w, ep, ntb, s);
         case LinearEpilogue::kSoftcap: return launch_big_bf16<LinearEpilogue::kSoftcap>(a, m, w, ep, ntb, s);
         default: return launch_big_bf16<LinearEpilogue::kStore>(a, m, w, ep, ntb, s);
     }
@@ -1205,6 +1206,7 @@ void launch_big_grouped(const uint16_t *a, const LinearWeight &w, const RowGroup
 
 void gemm_bf16_big_grouped(const uint16_t *a, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, hipStream_t s) {
     if (ep.mode == LinearEpilogue::kSquaredRelu) launch_big_grouped<LinearEpilogue::kSquaredRelu>(a, w, rg, ep, s);
+    else if (ep.mode == LinearEpilogue::kSiluGlu) launch_big_grouped<LinearEpilogue::kSiluGlu>(a, w, rg, ep, s);
     else launch_big_grouped<LinearEpilogue::kStore>(a, w, rg, ep, s);
 }
 

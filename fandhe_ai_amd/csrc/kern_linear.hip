@@ -364,15 +364,22 @@ void launch_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
 template <int MODE>
 void launch_grouped_bf16(const uint16_t *a, uint64_t lda, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, int num_cus, hipStream_t s) {
     const uint8_t *wt = (const uint8_t *)w.w;
-    const uint64_t mean = rg.entries / rg.groups;
+    constexpr bool GLU = is_glu(MODE);
+    const uint64_t mean = (rg.likely ? rg.likely : rg.entries) / rg.groups;
     const int form = g_linear_form;
     if (form == 4 || (form != 5 && form != 6 && mean <= 10)) {
-        const bool two = (uint64_t)w.n_tiles * std::min(rg.groups, rg.entries) >= 2 * (uint64_t)num_cus;
+        const bool two = GLU || (uint64_t)w.n_tiles * std::min(rg.groups, rg.entries) >= 2 * (uint64_t)num_cus;
         const dim3 grid(two ? (w.n_tiles + 1) / 2 : w.n_tiles, rg.groups);
 #define FA_ROWS(MT_, NTW_) linear_rows_grouped_kernel<MT_, NTW_, 8, MODE><<<grid, 512, 0, s>>>(a, lda, wt, w.n, w.n_tiles, w.k_tiles, rg, ep)
-        if (rg.most <= 16) two ? FA_ROWS(1, 2) : FA_ROWS(1, 1);
-        else if (mean <= 8) two ? FA_ROWS(2, 2) : FA_ROWS(2, 1);
-        else two ? FA_ROWS(4, 2) : FA_ROWS(4, 1);
+        if constexpr (GLU) {
+            if (rg.most <= 16) FA_ROWS(1, 2);
+            else if (mean <= 8) FA_ROWS(2, 2);
+            else FA_ROWS(4, 2);
+        } else {
+            if (rg.most <= 16) two ? FA_ROWS(1, 2) : FA_ROWS(1, 1);
+            else if (mean <= 8) two ? FA_ROWS(2, 2) : FA_ROWS(2, 1);
+            else two ? FA_ROWS(4, 2) : FA_ROWS(4, 1);
+        }
 #undef FA_ROWS
         return;
     }
@@ -404,6 +411,7 @@ void linear_bf16(const uint16_t *a, uint64_t lda, uint64_t a_batch, uint64_t m, 
         case LinearEpilogue::kSiluGlu: return launch_bf16<LinearEpilogue::kSiluGlu>(a, lda, a_batch, m, w, ep, num_cus, s);
         case LinearEpilogue::kSoftcap: return launch_bf16<LinearEpilogue::kSoftcap>(a, lda, a_batch, m, w, ep, num_cus, s);
         case LinearEpilogue::kHeadGate: return launch_bf16<LinearEpilogue::kHeadGate>(a, lda, a_batch, m, w, ep, num_cus, s);
+        case LinearEpilogue::kXielu: return launch_bf16<LinearEpilogue::kXielu>(a, lda, a_batch, m, w, ep, num_cus, s);
         default: return launch_bf16<LinearEpilogue::kStore>(a, lda, a_batch, m, w, ep, num_cus, s);
     }
 }
@@ -416,6 +424,7 @@ void linear_f32(const float *a, uint64_t lda, uint64_t a_batch, uint64_t m, cons
         case LinearEpilogue::kSiluGlu: return launch_f32<LinearEpilogue::kSiluGlu>(a, lda, a_batch, m, w, ep, s);
         case LinearEpilogue::kSoftcap: return launch_f32<LinearEpilogue::kSoftcap>(a, lda, a_batch, m, w, ep, s);
         case LinearEpilogue::kHeadGate: return launch_f32<LinearEpilogue::kHeadGate>(a, lda, a_batch, m, w, ep, s);
+        case LinearEpilogue::kXielu: return launch_f32<LinearEpilogue::kXielu>(a, lda, a_batch, m, w, ep, s);
         default: return launch_f32<LinearEpilogue::kStore>(a, lda, a_batch, m, w, ep, s);
     }
 }
@@ -424,12 +433,14 @@ void linear_grouped_bf16(const uint16_t *a, uint64_t lda, const LinearWeight &w,
                          hipStream_t s) {
     if (rg.entries == 0 || rg.groups == 0) return;
     if (ep.mode == LinearEpilogue::kSquaredRelu) launch_grouped_bf16<LinearEpilogue::kSquaredRelu>(a, lda, w, rg, ep, num_cus, s);
+    else if (ep.mode == LinearEpilogue::kSiluGlu) launch_grouped_bf16<LinearEpilogue::kSiluGlu>(a, lda, w, rg, ep, num_cus, s);
     else launch_grouped_bf16<LinearEpilogue::kStore>(a, lda, w, rg, ep, num_cus, s);
 }
 
 void linear_grouped_f32(const float *a, uint64_t lda, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, hipStream_t s) {
     if (rg.entries == 0 || rg.groups == 0) return;
     if (ep.mode == LinearEpilogue::kSquaredRelu) launch_grouped_f32<LinearEpilogue::kSquaredRelu>(a, lda, w, rg, ep, s);
+    else if (ep.mode == LinearEpilogue::kSiluGlu) launch_grouped_f32<LinearEpilogue::kSiluGlu>(a, lda, w, rg, ep, s);
     else launch_grouped_f32<LinearEpilogue::kStore>(a, lda, w, rg, ep, s);
 }
 

@@ -329,7 +329,7 @@ struct LinearWeight {
 };
 // What becomes of y = a W^T (f32):
 struct LinearEpilogue {
-    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4, kSquaredRelu = 5, kSiluGlu = 6 };
+    enum Mode { kStore = 0, kResidual = 1, kGlu = 2, kSoftcap = 3, kHeadGate = 4, kSquaredRelu = 5, kSiluGlu = 6, kXielu = 7 };
     int mode = kStore;
     void *out = nullptr;         // [m, ld_out], f32 or bf16; kResidual: the f32 residual itself
     int out_f32 = 0;
@@ -339,10 +339,11 @@ struct LinearEpilogue {
     float *out_hi = nullptr;
     uint32_t ld_hi = 0;
     const float *bias = nullptr;     // kStore: y + bias[c]
-    const float *scale = nullptr;    // kResidual: out[r, c] += scale[c] * y
+    const float *scale = nullptr;    // kResidual: out[r, c] += scale[c] * y (null: y)
     // kGlu: tiles alternate gate / up; g = min(gate, limit), u = clamp(up, +-limit), out = g sigmoid(alpha g) (u + 1)
     float limit = 0.0f, alpha = 0.0f;
     // kSiluGlu: gate sigmoid(gate) up, tiles as kGlu's
+    const float *act = nullptr;  // kXielu: act[0] y^2 + y / 2 above 0, act[1] (e^y - 1 - y) + y / 2 below
     float factor = 1.0f;         // kStore, kSoftcap, kHeadGate: of y, ahead of everything else
     float cap = 0.0f;            // kSoftcap: cap tanh(y / cap); cap <= 0: y
     const float *gate = nullptr; // kHeadGate: y * sigmoid(gate[r * ld_gate + batch])
@@ -361,6 +362,7 @@ struct RowGroups {
     const uint32_t *count = nullptr, *list = nullptr;
     uint32_t groups = 0, pitch = 0, a_div = 1, entries = 0;
     uint32_t most = 0;           // entries of a group at most (up to pitch)
+    uint32_t likely = 0;         // entries of all groups to be expected (0: `entries`); tuning only
 };
 void linear_grouped_bf16(const uint16_t *a, uint64_t lda, const LinearWeight &w, const RowGroups &rg, const LinearEpilogue &ep, int num_cus,
                          hipStream_t s);
@@ -404,34 +406,46 @@ void gather_rows_any(const void *table, int table_f32, uint64_t table_rows, uint
                      uint64_t rows, hipStream_t s);
 
 // x = table[idx] * scale (+ the additive position vector: sin(p freq[i]) in entry 2 i, cos in 2 i + 1; freq null: none) as
-// f32, and the same rounded to the activations' type with pitch ld, zeros past cols.
+// f32, and the same rounded to the activations' type with pitch ld, zeros past cols (hn null: not).
 void embed_rows(const void *table, int is_f32, uint64_t table_rows, uint64_t cols, const int32_t *idx, const int32_t *pos, const double *freq,
                 float scale, float *x, void *hn, uint64_t ld, uint64_t rows, hipStream_t s);
 
-// ---- sublayers that norm their output (kern_experts.hip) -------------------------
-// Which experts a row takes: router logits in f32 from h in the activations' type (zeros past its width up to ld), the `top` largest (ties: the lower
-// index), a softmax over those; entry row * top + i is appended to the list of its i-th expert.
+// ---- residual updates with norms, routing (kern_experts.hip) ----------------------
+// Which experts a row takes: router logits in f32 from h in the activations' type (zeros past its width up to ld), and the `top` largest (ties:
+// the lower index) weighted by a softmax over those; or, scored, as FA_ROUTE_SCORED says.  Entry row * top + i is appended to the list
+// of its i-th expert.  The last `identity` outputs have no list: their entries get gate 0, the sum of their weights goes to
+// identity_gate.
 struct RouteIo {
     const void *w = nullptr;     // packed as a LinearWeight of `experts` columns
-    uint32_t experts = 0, top = 0;
-    uint32_t *count = nullptr;   // [experts], zero before
-    uint32_t *list = nullptr;    // [experts][pitch]
+    uint32_t experts = 0, top = 0;       // experts: all outputs of the router
+    uint32_t *count = nullptr;   // [experts - identity], zero before
+    uint32_t *list = nullptr;    // [experts - identity][pitch]
     uint32_t pitch = 0;
     float *gate = nullptr;       // [rows][top]
+    int scored = 0;
+    const float *correction = nullptr;   // [experts]
+    uint32_t identity = 0, groups = 1, keep = 1;
+    float scale = 1.0f;
+    float *identity_gate = nullptr;      // [rows]; null: no identity experts
 };
 constexpr uint32_t kMaxExperts = 256, kMaxTop = 64;
 void route_rows(const void *h_bf16, uint64_t rows, uint64_t ld, const RouteIo &io, hipStream_t s);
-// x += norm(y) * w, hn = x in the activations' type (pitch ld, zeros past hidden).  The norm is RMS norm, or with `layer` layer
-// norm, hn then being layernorm(x) * next (next null: hn is left alone).  y [rows * parts, hidden] f32; parts > 1
-// (or gate set): y's row is sum_i gate[row][i] y[row * parts + i].  clear (n_clear words): set to zero.  route: the rows'
-// experts are chosen in the same launch (for few rows and in f32; many bf16 rows are faster in a launch of route_rows).
+// The residual update of a sublayer's output y and the norm that comes with it:
+//   kOutput  x += rmsnorm(y) w, hn = x
+//   kBoth    x += layernorm(y) w, hn = layernorm(x) next
+//   kInput   x += y, hn = rmsnorm(x) next; y null: x as it is
+// hn in the activations' type (pitch ld, zeros past hidden); next null: hn is left alone.  y [rows * parts, hidden] f32; parts > 1 (or
+// gate set): y's row is sum_i gate[row][i] y[row * parts + i], parts of gate 0 not read, with identity_gate [rows] that times the row
+// of hn added.  clear (n_clear words): set to zero.  route: the rows' experts are chosen in the same launch (for few
+// rows and in f32; many bf16 rows are faster in a launch of route_rows).
 struct ResidualNorm {
-    const float *y = nullptr, *gate = nullptr;
+    enum Kind { kOutput = 0, kBoth = 1, kInput = 2 };
+    Kind kind = kOutput;
+    const float *y = nullptr, *gate = nullptr, *identity_gate = nullptr;
     uint32_t parts = 1;
     const float *w = nullptr;
     float eps = 0.0f;
     uint32_t *clear = nullptr, n_clear = 0;
-    bool layer = false;
     const float *next = nullptr;
 };
 bool residual_norm_routes(int is_f32, uint64_t rows);
@@ -447,6 +461,8 @@ struct AttentionShape {
     uint64_t pool_rows;
     uint32_t window;             // keys p - window + 1 .. p
     uint32_t rot, interleaved;   // leading entries of every query and key head that are rotated; their pairs
+    float q_temp;                // 0: none
+    uint32_t q_temp_every;
     __host__ __device__ uint32_t share() const { return heads / kv_heads; }
 };
 constexpr uint32_t kWholeContext = 0x7fffffff;       // a window that holds every earlier token
@@ -457,21 +473,26 @@ void attention_prepare(const float *y, uint32_t ld, const float *q_norm, const f
                        const AttentionShape &sh, const RaggedRows &rr, hipStream_t s);
 // The form with norms per head and rotation: q, k of a head x / sqrt(mean(x^2) + eps) * w with norms (weights [dim], shared by the
 // heads; null: 1), then their first sh.rot entries turned by cos_sin [rows, rot].  key_values: y = q | k, and the projected keys
-// are the values.
+// are the values.  Queries times 1 + sh.q_temp ln(floor((p + 1) / sh.q_temp_every) + 1) at position p.
 void attention_prepare_heads(const float *y, uint32_t ld, bool norms, const float *q_norm, const float *k_norm, const float *cos_sin, bool key_values, void *q,
                              void *k_pool, void *v_pool, int is_f32, const AttentionShape &sh, const RaggedRows &rr, hipStream_t s);
-// What happens to the softmax and its result: sink [heads]: a score without key and value (null: none); gate [rows, ld_gate] in
-// the activations' type, heads x vdim: the output times its sigmoid (null: none); and times scale.
+// What happens to the scores and their result: slope [heads]: the score less slope times the key's distance (null: none); sigmoid: the
+// weights are the sigmoids of score + bias[head], as they are, instead of a softmax; sink [heads]: a score without key and
+// value in the softmax (null: none); gate [rows, ld_gate] in the activations' type, heads x vdim: the output times its
+// sigmoid (null: none); head_gate [rows, ld_head_gate], f32: the same with one number per head; and times scale.
 struct AttentionOutput {
-    const float *sink = nullptr;
+    const float *slope = nullptr, *bias = nullptr, *sink = nullptr;
+    bool sigmoid = false;
     const void *gate = nullptr;
     uint32_t ld_gate = 0;
+    const float *head_gate = nullptr;
+    uint32_t ld_head_gate = 0;
     float scale = 1.0f;
 };
-// Causal softmax attention over the cache -> out [rows, ld_out], heads x vdim.  bf16 with padded sizes up to 256: matrix-core
+// Causal attention over the cache -> out [rows, ld_out], heads x vdim.  bf16 with padded sizes up to 256: matrix-core
 // kernels, one for few query rows per sequence (the keys split over blocks that meet in the workspace) and one for many;
-// otherwise a plain one.  min_new / max_new: fewest (not counting none) and most new tokens of any sequence.
-uint64_t attention_workspace_bytes(const AttentionShape &sh, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
+// otherwise, and for a softmax over scores with slopes, a plain one.  min_new / max_new: fewest (not counting none) and most new tokens of any sequence.
+uint64_t attention_workspace_bytes(const AttentionShape &sh, const AttentionOutput &ao, int is_f32, uint32_t batch, uint32_t min_new, uint32_t max_new, uint32_t max_ctx,
                                    int num_cus);
 void attention(const void *q, const void *k_pool, const void *v_pool, void *out, uint32_t ld_out, const AttentionOutput &ao, int is_f32,
                const AttentionShape &sh, const RaggedRows &rr, uint32_t min_new, uint32_t max_new, void *workspace, int num_cus, hipStream_t s);
@@ -553,6 +574,27 @@ constexpr uint32_t kDeltaMaxDim = 256, kDeltaMaxVdim = 1024;
 uint64_t delta_scratch_bytes(const DeltaShape &sh, uint32_t rows, uint32_t batch);
 // max_new: most new tokens of any sequence of the pass
 void delta_mixer(const DeltaShape &sh, const DeltaIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, hipStream_t s);
+
+// ---- minimal gated recurrence (kern_gated.hip) ------------------------------------
+// S <- (1 - z) S + z c per channel, z = sigmoid(zu[0 ..] + z_bias), u = zu[width ..] + u_bias, c = u + 1/2 from u = 0 on and sigmoid(u) below;
+// out = S silu(gate) out_scale.
+struct GatedIo {
+    const float *zu;             // [rows, ld_zu]: z and u ahead of their biases, `width` each
+    uint32_t ld_zu;
+    const float *z_bias, *u_bias;        // [width]
+    const void *gate;            // [rows, ld_gate], type of out
+    uint32_t ld_gate;
+    float *state;                // [slots][gated_pitch(width)]
+    void *out;                   // [rows, ld_out], bf16 or f32
+    uint32_t ld_out;
+    float out_scale;
+};
+constexpr uint32_t gated_pitch(uint32_t width) { return (width + 3) / 4 * 4; }
+// max_new: most new tokens of any sequence of the pass
+void gated_mixer(uint32_t width, const GatedIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, hipStream_t s);
+
+// act[0] = softplus(pq[0]), act[1] = 1/2 + softplus(pq[1]): what kXielu reads
+void xielu_constants(const float *pq, float *act, hipStream_t s);
 
 // ---- sampling (kern_sampling.hip) ------------------------------------------------
 // one row of a per-row sampling table (the layout of fa_row_sampling)

@@ -40,7 +40,8 @@ struct Mixer {
     // attention; q_norm below
     k::AttentionShape at{};
     uint32_t gate_at = 0;                             // column of its `lo` part where the gate starts
-    float *k_norm = nullptr, *sink = nullptr;
+    float *k_norm = nullptr, *sink = nullptr, *slope = nullptr, *score_bias = nullptr;
+    uint32_t head_gate_at = 0;                        // column of its `hi` part where the gates per head start
     void *k_pool = nullptr, *v_pool = nullptr;
     // latent attention
     k::LatentShape la{};
@@ -53,12 +54,15 @@ struct Mixer {
     k::DeltaShape de{};
     float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *head_norm = nullptr, *state = nullptr, *decay = nullptr;
     void *ring = nullptr;
+    // minimal gated recurrence: biases of z and u; state above
+    float *z_bias = nullptr, *u_bias = nullptr;
     // low-rank gates and decays: their inner values start at column rank_at of the `lo` part (decay first, gate from its padded
     // rank on); one weight with zeros in the other's place makes both
     k::LinearWeight low_rank;
     uint32_t rank_at = 0;
 };
 
+// States that are matrices per head (DeltaShape)
 bool recurrent(const fa_layer_config &c) { return c.mixer == FA_MIXER_DELTA || c.mixer == FA_MIXER_LIGHTNING; }
 
 struct Layer {
@@ -69,6 +73,9 @@ struct Layer {
     float *in_bias = nullptr;                         // attention alone in its layer
     k::LinearWeight in, out, gate_up, down;           // with experts: gate_up and down hold one batch entry each
     k::LinearWeight router;
+    float *correction = nullptr;                      // of the experts' scores
+    float *act = nullptr;                             // xIELU: the two factors, and the two numbers they come from
+    uint32_t lists() const { return cfg.experts - cfg.identity; }        // experts with tensors
 };
 
 // A rotation's frequencies follow from these
@@ -102,7 +109,7 @@ struct Arena {
     void *base = nullptr;
     uint64_t bytes = 0, cls = 0;
     uint32_t rows = 0;
-    float *x = nullptr, *y32 = nullptr, *head_x = nullptr, *delta_scratch = nullptr, *raw = nullptr, *decay = nullptr, *gate = nullptr;
+    float *x = nullptr, *y32 = nullptr, *head_x = nullptr, *delta_scratch = nullptr, *raw = nullptr, *decay = nullptr, *gate = nullptr, *identity_gate = nullptr;
     uint32_t *expert_count = nullptr, *expert_list = nullptr;       // counts are zero between feed-forwards
     void *hn = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *olat = nullptr, *o = nullptr, *act = nullptr, *low_gate = nullptr;
     uint32_t *row_seq = nullptr, *kv_slot = nullptr, *row_start = nullptr;
@@ -166,7 +173,7 @@ Widths widths(const LayeredState &L) {
                 }
             } else if (m.cfg.mixer == FA_MIXER_ATTENTION) {
                 w.q = std::max<uint64_t>(w.q, (uint64_t)m.at.heads * m.at.dim_p);
-            } else {
+            } else if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION) {
                 w.cq = std::max<uint64_t>(w.cq, pad_to(m.la.q_rank, 64));
                 w.q = std::max<uint64_t>(w.q, (uint64_t)m.la.heads * (m.la.dim_p + m.la.rot_p));
                 w.qa = std::max<uint64_t>(w.qa, (uint64_t)m.la.heads * (m.la.rank_p + m.la.rot_p));
@@ -175,7 +182,7 @@ Widths widths(const LayeredState &L) {
         }
         const uint64_t parts = l.cfg.experts ? l.cfg.top : 1;
         if (l.cfg.d_ffn) w.act = std::max<uint64_t>(w.act, parts * pad_to(l.cfg.d_ffn, 64));
-        if (L.cfg.norm != FA_NORM_INPUT) w.y32 = std::max<uint64_t>(w.y32, parts * L.cfg.d_model);
+        if (L.cfg.norm != FA_NORM_INPUT && (L.cfg.norm != FA_NORM_INPUT_RMS || l.cfg.experts)) w.y32 = std::max<uint64_t>(w.y32, parts * L.cfg.d_model);
         w.top = std::max<uint64_t>(w.top, l.cfg.experts ? l.cfg.top : 0);
         w.experts = std::max<uint64_t>(w.experts, l.cfg.experts);
     }
@@ -213,6 +220,7 @@ fa_status arena_reserve(fa_context *ctx, LayeredState &L, Arena &a, uint32_t row
     add(&a.o, R * w.o * E);
     add(&a.act, R * w.act * E);
     add((void **)&a.gate, R * w.top * 4);
+    add((void **)&a.identity_gate, w.top ? R * 4 : 0);
     add((void **)&a.expert_count, w.experts * 4);
     add((void **)&a.expert_list, w.experts * R * 4);
     add((void **)&a.row_seq, R * 4);
@@ -369,6 +377,40 @@ void enqueue_latent(fa_context *ctx, const fa_decoder *d, Arena &a, const Layer 
     }
 }
 
+void enqueue_gated(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const Mixer &m, const k::RaggedRows &rr, uint32_t max_new, uint32_t ld_o) {
+    k::GatedIo io{};
+    io.zu = a.y32 + m.hi_at;
+    io.ld_zu = pad_to(l.hi, 4);
+    io.z_bias = m.z_bias;
+    io.u_bias = m.u_bias;
+    io.gate = element(L, a.y, m.lo_at);
+    io.ld_gate = l.lo;
+    io.state = m.state;
+    io.out = element(L, a.o, m.o_at);
+    io.ld_out = ld_o;
+    io.out_scale = m.out_scale;
+    k::gated_mixer(m.cfg.vdim, io, L.is_f32, rr, max_new, ctx->stream);
+}
+
+// What an attention mixer does to its scores and to their result; y: its f32 columns
+k::AttentionOutput attention_output(const LayeredState &L, const Arena &a, const Layer &l, const Mixer &m) {
+    k::AttentionOutput ao;
+    ao.slope = m.slope;
+    ao.bias = m.score_bias;
+    ao.sigmoid = m.cfg.attention & FA_ATTENTION_SIGMOID;
+    ao.sink = m.sink;
+    if (m.cfg.attention & FA_ATTENTION_GATE) {
+        ao.gate = element(L, a.y, m.lo_at + m.gate_at);
+        ao.ld_gate = l.lo;
+    }
+    if (m.cfg.attention & FA_ATTENTION_HEAD_GATE) {
+        ao.head_gate = a.y32 + m.hi_at + m.head_gate_at;
+        ao.ld_head_gate = pad_to(l.hi, 4);
+    }
+    ao.scale = m.out_scale;
+    return ao;
+}
+
 void enqueue_attention(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, const Mixer &m, const k::RaggedRows &rr, Portions n, uint32_t ld_o) {
     const k::AttentionShape &sh = m.at;
     const uint32_t ld_y = pad_to(l.hi, 4), flags = m.cfg.attention;
@@ -376,19 +418,12 @@ void enqueue_attention(fa_context *ctx, LayeredState &L, Arena &a, const Layer &
     const Mixer &kv = own ? m : L.layers[m.cfg.kv_from].mixers[0];
     const float *y = a.y32 + m.hi_at;
     const bool norms = flags & (FA_ATTENTION_HEAD_NORM | FA_ATTENTION_HEAD_UNIT), key_values = flags & FA_ATTENTION_KEY_VALUES;
-    if (norms || key_values || sh.rot)
+    if (norms || key_values || sh.rot || sh.q_temp != 0.0f)
         k::attention_prepare_heads(y, ld_y, norms, m.q_norm, m.k_norm, sh.rot ? a.cos_sin[m.rotation] : nullptr, key_values, a.q, m.k_pool, m.v_pool, L.is_f32,
                                    sh, rr, ctx->stream);
     else
         k::attention_prepare(y, ld_y, m.q_norm, m.k_norm, a.q, m.k_pool, m.v_pool, L.is_f32, sh, rr, ctx->stream);
-    k::AttentionOutput ao;
-    ao.sink = m.sink;
-    if (flags & FA_ATTENTION_GATE) {
-        ao.gate = element(L, a.y, m.lo_at + m.gate_at);
-        ao.ld_gate = l.lo;
-    }
-    ao.scale = m.out_scale;
-    k::attention(a.q, kv.k_pool, kv.v_pool, element(L, a.o, m.o_at), ld_o, ao, L.is_f32, sh, rr, n.min_new, n.max_new, ctx->workspace,
+    k::attention(a.q, kv.k_pool, kv.v_pool, element(L, a.o, m.o_at), ld_o, attention_output(L, a, l, m), L.is_f32, sh, rr, n.min_new, n.max_new, ctx->workspace,
                  ctx->props.multiProcessorCount, ctx->stream);
 }
 
@@ -398,32 +433,57 @@ void enqueue_mixers(fa_context *ctx, fa_decoder *d, Arena &a, const Layer &l, co
     enqueue_in(ctx, L, a, l, rr.rows, ld_hn);
     for (const Mixer &m : l.mixers) {
         if (recurrent(m.cfg)) enqueue_recurrence(ctx, L, a, l, m, rr, n.max_new, ld_o);
+        else if (m.cfg.mixer == FA_MIXER_MINGRU) enqueue_gated(ctx, L, a, l, m, rr, n.max_new, ld_o);
         else if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION) enqueue_latent(ctx, d, a, l, m, rr, n.max_new, ld_o, expand);
         else enqueue_attention(ctx, L, a, l, m, rr, n, ld_o);
     }
 }
 
 // Dense feed-forward: from a.hn to what `out` does with the down projection.
-void enqueue_glu(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t M, uint32_t ld_hn, const k::LinearEpilogue &out) {
+void enqueue_dense(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t M, uint32_t ld_hn, const k::LinearEpilogue &out) {
     const uint32_t ld_act = pad_to(l.cfg.d_ffn, 64);
     k::LinearEpilogue g = store_to(a.act, ld_act, L.is_f32);
-    g.mode = l.cfg.glu == FA_GLU_SILU ? k::LinearEpilogue::kSiluGlu : k::LinearEpilogue::kGlu;
+    g.mode = l.cfg.glu == FA_GLU_SILU ? k::LinearEpilogue::kSiluGlu : l.cfg.glu == FA_FFN_XIELU ? k::LinearEpilogue::kXielu : k::LinearEpilogue::kGlu;
+    g.act = l.act;
     g.limit = l.cfg.ffn_limit;
     g.alpha = l.cfg.ffn_alpha;
     linear(ctx, L, a.hn, ld_hn, 0, M, l.gate_up, g);
     linear(ctx, L, a.act, ld_act, 0, M, l.down, out);
 }
 
-// Feed-forward of a layer whose sublayers read x and norm their output.  The choice of experts is there (route_rows).
+k::RouteIo route_io(const Arena &a, const Layer &l) {
+    k::RouteIo io{l.router.w, l.cfg.experts, l.cfg.top, a.expert_count, a.expert_list, a.rows, a.gate};
+    io.scored = l.cfg.route == FA_ROUTE_SCORED;
+    io.correction = l.correction;
+    io.identity = l.cfg.identity;
+    io.groups = l.cfg.groups ? l.cfg.groups : 1;
+    io.keep = l.cfg.groups ? l.cfg.groups_kept : 1;
+    io.scale = l.cfg.route_scale;
+    io.identity_gate = l.cfg.identity ? a.identity_gate : nullptr;
+    return io;
+}
+
+// Sparse feed-forward: from a.hn to the rows' experts' outputs in a.y32.  The choice of experts is there (route_rows).
 void enqueue_experts(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, uint32_t M, uint32_t ld_hn) {
     const uint32_t D = L.cfg.d_model, ld_act = pad_to(l.cfg.d_ffn, 64), top = l.cfg.top;
-    k::RowGroups rg{a.expert_count, a.expert_list, l.cfg.experts, a.rows, top, M * top};
+    k::RowGroups rg{a.expert_count, a.expert_list, l.lists(), a.rows, top, M * top};
     rg.most = M;
+    rg.likely = (uint32_t)((uint64_t)M * top * l.lists() / l.cfg.experts);
     k::LinearEpilogue up = store_to(a.act, ld_act, L.is_f32);
-    up.mode = k::LinearEpilogue::kSquaredRelu;
+    up.mode = l.cfg.glu == FA_GLU_SILU ? k::LinearEpilogue::kSiluGlu : k::LinearEpilogue::kSquaredRelu;
     linear_grouped(ctx, L, a.hn, ld_hn, l.gate_up, rg, up);
     rg.a_div = 1;
     linear_grouped(ctx, L, a.act, ld_act, l.down, rg, store_to(a.y32, D, 1));
+}
+
+// The residual update after the experts
+void add_experts(k::ResidualNorm &rn, const Arena &a, const Layer &l) {
+    rn.y = a.y32;
+    rn.gate = a.gate;
+    rn.identity_gate = l.cfg.identity ? a.identity_gate : nullptr;
+    rn.parts = l.cfg.top;
+    rn.clear = a.expert_count;
+    rn.n_clear = l.lists();
 }
 
 // All layers over the rows of a pass whose embeddings are in a.x (and, with norms at the output, in a.hn).
@@ -436,6 +496,7 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
     const int f32 = L.is_f32;
     for (size_t i = 0; i < L.rotations.size(); ++i) k::rotation_table(rr.pos, a.cos_sin[i], M, L.rotations[i].dims, L.rotation_freq[i], s);
     if (L.cfg.norm == FA_NORM_BOTH) k::layernorm_rows(a.x, L.layers[0].norm1, a.hn, f32, M, D, ld_hn, eps, s);
+    if (L.cfg.norm == FA_NORM_INPUT_RMS) k::rmsnorm_rows(a.x, L.layers[0].norm1, a.hn, f32, M, D, ld_hn, eps, s);
     for (size_t li = 0; li < L.layers.size(); ++li) {
         const Layer &l = L.layers[li];
         if (L.cfg.norm == FA_NORM_INPUT) k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);
@@ -447,19 +508,16 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
         if (L.cfg.norm == FA_NORM_OUTPUT) {
             linear(ctx, L, a.o, ld_o, 0, M, l.out, store_to(a.y32, D, 1));
             rn.w = l.norm1;
-            k::RouteIo route{l.router.w, l.cfg.experts, l.cfg.top, a.expert_count, a.expert_list, a.rows, a.gate};
+            const k::RouteIo route = route_io(a, l);
             const bool fused = l.cfg.experts && k::residual_norm_routes(f32, M);
             k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, fused ? &route : nullptr, s);
             if (l.cfg.d_ffn) {
                 if (l.cfg.experts) {
                     if (!fused) k::route_rows(a.hn, M, ld_hn, route, s);
                     enqueue_experts(ctx, L, a, l, M, ld_hn);
-                    rn.gate = a.gate;
-                    rn.parts = l.cfg.top;
-                    rn.clear = a.expert_count;
-                    rn.n_clear = l.cfg.experts;
+                    add_experts(rn, a, l);
                 } else {
-                    enqueue_glu(ctx, L, a, l, M, ld_hn, store_to(a.y32, D, 1));
+                    enqueue_dense(ctx, L, a, l, M, ld_hn, store_to(a.y32, D, 1));
                 }
                 rn.w = l.norm2;
                 k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
@@ -468,15 +526,41 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
             // a residual update norms the new stream for the sublayer that comes next; the head norms its own rows
             const float *next_layer = li + 1 < L.layers.size() ? L.layers[li + 1].norm1 : nullptr;
             linear(ctx, L, a.o, ld_o, 0, M, l.out, store_to(a.y32, D, 1));
-            rn.layer = true;
+            rn.kind = k::ResidualNorm::kBoth;
             rn.w = l.post1;
             rn.next = l.cfg.d_ffn ? l.norm2 : next_layer;
             k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
             if (l.cfg.d_ffn) {
-                enqueue_glu(ctx, L, a, l, M, ld_hn, store_to(a.y32, D, 1));
+                enqueue_dense(ctx, L, a, l, M, ld_hn, store_to(a.y32, D, 1));
                 rn.w = l.post2;
                 rn.next = next_layer;
                 k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+            }
+        } else if (L.cfg.norm == FA_NORM_INPUT_RMS) {
+            // outputs are added where they are made, a sparse feed-forward's with the norm for the sublayer that comes next
+            const float *next_layer = li + 1 < L.layers.size() ? L.layers[li + 1].norm1 : nullptr;
+            k::LinearEpilogue r = store_to(a.x, D, 1);
+            r.mode = k::LinearEpilogue::kResidual;
+            linear(ctx, L, a.o, ld_o, 0, M, l.out, r);
+            rn.kind = k::ResidualNorm::kInput;
+            rn.y = nullptr;
+            rn.next = l.cfg.d_ffn ? l.norm2 : next_layer;
+            if (l.cfg.experts) {
+                const k::RouteIo route = route_io(a, l);
+                const bool fused = k::residual_norm_routes(f32, M);
+                k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, fused ? &route : nullptr, s);
+                if (!fused) k::route_rows(a.hn, M, ld_hn, route, s);
+                enqueue_experts(ctx, L, a, l, M, ld_hn);
+                add_experts(rn, a, l);
+                rn.next = next_layer;
+                k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+            } else {
+                if (rn.next) k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+                if (l.cfg.d_ffn) {
+                    enqueue_dense(ctx, L, a, l, M, ld_hn, r);
+                    rn.next = next_layer;
+                    if (rn.next) k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+                }
             }
         } else {
             k::LinearEpilogue r = store_to(a.x, D, 1);
@@ -486,7 +570,7 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
             if (l.cfg.d_ffn) {
                 k::layernorm_rows(a.x, l.norm2, a.hn, f32, M, D, ld_hn, eps, s);
                 r.scale = l.post2;
-                enqueue_glu(ctx, L, a, l, M, ld_hn, r);
+                enqueue_dense(ctx, L, a, l, M, ld_hn, r);
             }
         }
         if (L.trace) {
@@ -500,9 +584,9 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
 
 // Embeddings of the pass's tokens.
 void enqueue_embed(fa_context *ctx, const LayeredState &L, Arena &a, const int32_t *tokens, const k::RaggedRows &rr) {
-    if (L.cfg.norm == FA_NORM_OUTPUT)
-        k::embed_rows(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, tokens, rr.pos, L.position_freq, L.cfg.embed_scale, a.x, a.hn, pad_to(L.cfg.d_model, 64),
-                      rr.rows, ctx->stream);
+    if (L.cfg.norm == FA_NORM_OUTPUT || L.cfg.norm == FA_NORM_INPUT_RMS)
+        k::embed_rows(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, tokens, rr.pos, L.position_freq, L.cfg.embed_scale, a.x,
+                      L.cfg.norm == FA_NORM_OUTPUT ? a.hn : nullptr, pad_to(L.cfg.d_model, 64), rr.rows, ctx->stream);
     else
         k::gather_rows_any(L.embed, L.is_f32, L.cfg.vocab, L.cfg.d_model, tokens, a.x, rr.rows, ctx->stream);
 }
@@ -510,7 +594,7 @@ void enqueue_embed(fa_context *ctx, const LayeredState &L, Arena &a, const int32
 // Final norm and head over rows of f32 residuals.
 void enqueue_head(fa_context *ctx, LayeredState &L, Arena &a, const float *x, uint32_t rows, float *logits) {
     const uint32_t ld_hn = pad_to(L.cfg.d_model, 64);
-    if (L.cfg.norm == FA_NORM_OUTPUT) k::rmsnorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
+    if (L.cfg.norm == FA_NORM_OUTPUT || L.cfg.norm == FA_NORM_INPUT_RMS) k::rmsnorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
     else k::layernorm_rows(x, L.final_norm, a.hn, L.is_f32, rows, L.cfg.d_model, ld_hn, L.cfg.norm_eps, ctx->stream);
     k::LinearEpilogue e = store_to(logits, L.cfg.vocab, 1);
     e.mode = k::LinearEpilogue::kSoftcap;
@@ -532,7 +616,7 @@ void prepare_rows(fa_context *ctx, fa_decoder *d, Arena &a, const uint32_t *row_
     k::ragged_advance(row_start, (uint32_t *)d->seq_lens->ptr, d->batch, ctx->stream);
 }
 
-fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t rows, uint32_t batch, Portions n) {
+fa_status attention_workspace(fa_context *ctx, const LayeredState &L, const Arena &a, uint32_t rows, uint32_t batch, Portions n) {
     uint64_t need = 0;
     const int cus = ctx->props.multiProcessorCount;
     for (const Layer &l : L.layers)
@@ -540,7 +624,7 @@ fa_status attention_workspace(fa_context *ctx, const LayeredState &L, uint32_t r
             if (m.cfg.mixer == FA_MIXER_LATENT_ATTENTION)
                 need = std::max(need, k::latent_attention_workspace_bytes(m.la, L.is_f32, rows, batch, n.max_new, cus));
             else if (m.cfg.mixer == FA_MIXER_ATTENTION)
-                need = std::max(need, k::attention_workspace_bytes(m.at, L.is_f32, batch, n.min_new, n.max_new, L.cfg.max_blocks_per_seq * L.cfg.block_size, cus));
+                need = std::max(need, k::attention_workspace_bytes(m.at, attention_output(L, a, l, m), L.is_f32, batch, n.min_new, n.max_new, L.cfg.max_blocks_per_seq * L.cfg.block_size, cus));
         }
     return need ? ensure_workspace(ctx, need) : FA_OK;
 }
@@ -625,7 +709,7 @@ fa_status layered_sequences_set(fa_context *ctx, fa_decoder *d) {
 fa_status layered_prepare_step(fa_context *ctx, fa_decoder *d) {
     LayeredState &L = *d->layered;
     if (fa_status s = arena_reserve(ctx, L, L.step, L.cfg.max_batch)) return s;
-    return attention_workspace(ctx, L, d->batch, d->batch, Portions{1, 1});
+    return attention_workspace(ctx, L, L.step, d->batch, d->batch, Portions{1, 1});
 }
 
 fa_status layered_enqueue_step(fa_context *ctx, fa_decoder *d) {
@@ -727,7 +811,7 @@ fa_status layered_forward(fa_context *ctx, fa_decoder *d, const uint32_t *counts
                 if (fa_status s = arena_reserve(ctx, L, a, a.rows, e_cap)) return s;
                 if (fa_status s = upload(ctx, a.expand_meta, expand.meta.data(), expand.meta.size() * 4)) return s;
             }
-            if (fa_status s = attention_workspace(ctx, L, rows, B, portions)) return s;
+            if (fa_status s = attention_workspace(ctx, L, a, rows, B, portions)) return s;
             if (fa_status s = upload(ctx, a.row_start, starts.data(), (B + 1) * 4)) return s;
             if (fa_status s = upload(ctx, a.tokens, stage.data(), (uint64_t)rows * 4)) return s;
             prepare_rows(ctx, d, a, a.row_start, rows);
@@ -793,6 +877,11 @@ fa_status check_layered(const fa_decoder *d, const char *what) {
 // One mixer; alone: it is the only one of its layer.
 fa_status check_mixer(const fa_layered_config &c, const fa_layer_config &l, uint32_t i, bool alone) {
     auto bad = [&](const char *why) { return fail(FA_ERR_INVALID_ARGUMENT, "layer " + std::to_string(i) + ": " + why); };
+    if (l.mixer == FA_MIXER_MINGRU) {
+        if (l.heads != 1 || l.vdim == 0 || l.vdim > 65536) return bad("a minimal gated recurrence has one head of a width up to 65536");
+        if (c.state_slots == 0) return bad("a recurrent layer needs state slots");
+        return FA_OK;
+    }
     if (l.heads == 0 || l.dim == 0 || l.vdim == 0 || l.heads > 1024 || l.dim > 4096 || l.vdim > 4096) return bad("heads, dim and vdim must be positive");
     if (l.mixer == FA_MIXER_DELTA || l.mixer == FA_MIXER_LIGHTNING) {
         if (l.dim > k::kDeltaMaxDim || l.vdim > k::kDeltaMaxVdim) return fail(FA_ERR_UNSUPPORTED, "delta layer: dim above 256 or vdim above 1024");
@@ -817,12 +906,15 @@ fa_status check_mixer(const fa_layered_config &c, const fa_layer_config &l, uint
     } else if (l.mixer == FA_MIXER_ATTENTION) {
         if (l.kv_heads == 0 || l.heads % l.kv_heads != 0) return bad("heads must be a multiple of kv_heads");
         const uint32_t per_head = FA_ATTENTION_HEAD_NORM | FA_ATTENTION_HEAD_UNIT, all = FA_ATTENTION_BIAS | FA_ATTENTION_QK_NORM | per_head |
-                                                                                        FA_ATTENTION_KEY_VALUES | FA_ATTENTION_GATE | FA_ATTENTION_SINK;
+                                                                                        FA_ATTENTION_KEY_VALUES | FA_ATTENTION_GATE | FA_ATTENTION_SINK | FA_ATTENTION_SIGMOID |
+                                                                                        FA_ATTENTION_HEAD_GATE;
         if (l.attention & ~all) return bad("unknown attention flags");
         if ((l.attention & per_head) == per_head) return bad("one kind of norm per head");
-        const bool heads_form = (l.attention & (per_head | FA_ATTENTION_KEY_VALUES)) || l.rot_dim;
-        if (heads_form && (l.attention & FA_ATTENTION_QK_NORM)) return fail(FA_ERR_UNSUPPORTED, "attention: norms over all heads beside norms per head, keys as values or rotation");
-        if ((l.attention & FA_ATTENTION_BIAS) && (!alone || (l.attention & FA_ATTENTION_GATE))) return fail(FA_ERR_UNSUPPORTED, "attention: biases beside a gate or a second mixer");
+        if ((l.attention & FA_ATTENTION_SIGMOID) && (l.attention & FA_ATTENTION_SINK)) return bad("a sink needs a softmax");
+        if (!std::isfinite(l.distance) || !std::isfinite(l.q_temp) || (l.q_temp != 0.0f && l.q_temp_every == 0)) return bad("bad distance or query temperature");
+        const bool heads_form = (l.attention & (per_head | FA_ATTENTION_KEY_VALUES)) || l.rot_dim || l.q_temp != 0.0f;
+        if (heads_form && (l.attention & FA_ATTENTION_QK_NORM)) return fail(FA_ERR_UNSUPPORTED, "attention: norms over all heads beside norms per head, keys as values, rotation or query temperature");
+        if ((l.attention & FA_ATTENTION_BIAS) && (!alone || (l.attention & (FA_ATTENTION_GATE | FA_ATTENTION_HEAD_GATE)))) return fail(FA_ERR_UNSUPPORTED, "attention: biases beside a gate or a second mixer");
         if ((l.attention & FA_ATTENTION_KEY_VALUES) && l.vdim != l.dim) return bad("keys as values need vdim = dim");
         if (l.rot_dim % 2 != 0 || l.rot_dim > l.dim) return bad("rot_dim must be even and at most dim");
         if (heads_form && l.kv_from >= 0) return fail(FA_ERR_UNSUPPORTED, "attention: an earlier layer's cache beside norms per head, keys as values or rotation");
@@ -857,12 +949,22 @@ fa_status check_layer(const fa_layered_config &c, uint32_t i) {
         if (!std::isfinite(l.left_scale) || !std::isfinite(l.right_scale)) return bad("bad scale of a mixer");
     }
     if (l.experts) {
-        if (l.experts > k::kMaxExperts || l.top > k::kMaxTop) return fail(FA_ERR_UNSUPPORTED, "sparse experts: more than 256, or more than 64 of them per token");
+        if (l.experts > k::kMaxExperts || l.identity >= l.experts || l.top > k::kMaxTop)
+            return fail(FA_ERR_UNSUPPORTED, "sparse experts: none or more than 256 of them, or more than 64 per token");
         if (l.top == 0 || l.top > l.experts || l.d_ffn == 0) return bad("top must be between 1 and experts, d_ffn positive");
-        if (c.norm != FA_NORM_OUTPUT) return fail(FA_ERR_UNSUPPORTED, "sparse experts: with norms at the sublayers' output only");
+        if (c.norm != FA_NORM_OUTPUT && c.norm != FA_NORM_INPUT_RMS) return fail(FA_ERR_UNSUPPORTED, "sparse experts: with RMS norms only");
+        if (l.glu != FA_GLU_CLAMPED && l.glu != FA_GLU_SILU) return bad("experts: unknown feed-forward");
+        if (l.route != FA_ROUTE_CHOSEN && l.route != FA_ROUTE_SCORED) return bad("unknown choice of experts");
+        if (l.route == FA_ROUTE_SCORED) {
+            if (!std::isfinite(l.route_scale)) return bad("bad scale of the experts' weights");
+            if (l.groups && (l.experts % l.groups != 0 || l.groups_kept == 0 || l.groups_kept > l.groups || l.top > l.experts / l.groups * l.groups_kept))
+                return bad("groups must be equal, and those kept hold at least `top` experts");
+        } else if (l.groups) {
+            return fail(FA_ERR_UNSUPPORTED, "groups of experts need scores");
+        }
         return FA_OK;
     }
-    if (l.glu != FA_GLU_CLAMPED && l.glu != FA_GLU_SILU) return bad("unknown gated linear unit");
+    if (l.glu != FA_GLU_CLAMPED && l.glu != FA_GLU_SILU && l.glu != FA_FFN_XIELU) return bad("unknown feed-forward");
     if (l.d_ffn && l.glu == FA_GLU_CLAMPED && !(l.ffn_limit >= 0.0f && std::isfinite(l.ffn_alpha))) return bad("bad feed-forward constants");
     return FA_OK;
 }
@@ -881,11 +983,11 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
     if (c.d_model > 16384) return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: d_model above 16384");
     if (c.dtype != FA_BF16 && c.dtype != FA_F32) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: dtype must be bf16 or f32");
     if (!std::isfinite(c.norm_eps) || c.norm_eps < 0.0f || !std::isfinite(c.logit_softcap)) return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad constants");
-    if (c.norm < FA_NORM_INPUT || c.norm > FA_NORM_BOTH || !std::isfinite(c.embed_scale) || !std::isfinite(c.position_base) || c.position_base < 0.0 ||
+    if (c.norm < FA_NORM_INPUT || c.norm > FA_NORM_INPUT_RMS || !std::isfinite(c.embed_scale) || !std::isfinite(c.position_base) || c.position_base < 0.0 ||
         !std::isfinite(c.logit_scale))
         return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: bad norm, embed_scale, position_base or logit_scale");
-    if (c.norm != FA_NORM_OUTPUT && (c.position_base > 0.0 || (c.embed_scale != 0.0f && c.embed_scale != 1.0f)))
-        return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: scaled or positioned embeddings need norms at the sublayers' output");
+    if (c.norm != FA_NORM_OUTPUT && c.norm != FA_NORM_INPUT_RMS && (c.position_base > 0.0 || (c.embed_scale != 0.0f && c.embed_scale != 1.0f)))
+        return fail(FA_ERR_UNSUPPORTED, "decoder_create_layered: scaled or positioned embeddings need RMS norms");
     if (c.block_size == 0 || (c.block_size & (c.block_size - 1)) != 0 || c.block_size > 256 || c.num_blocks == 0)
         return fail(FA_ERR_INVALID_ARGUMENT, "decoder_create_layered: block_size must be a power of two up to 256, num_blocks positive");
     if (c.max_blocks_per_seq == 0 || (uint64_t)c.max_blocks_per_seq * c.block_size > (uint64_t)INT32_MAX)
@@ -976,7 +1078,7 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             if (st == FA_OK) st = fa_upload_into(ctx, freq.data(), 2 * freq.size(), L->owned.back(), 0);
         }
         // what sublayer outputs pass on their way to the residual: a layer scale or a second norm
-        const char *post[3][2] = {{"ls1", "ls2"}, {nullptr, nullptr}, {"norm1b", "norm2b"}};
+        const char *post[4][2] = {{"ls1", "ls2"}, {nullptr, nullptr}, {"norm1b", "norm2b"}, {nullptr, nullptr}};
         const uint32_t max_ctx = (uint32_t)std::min<uint64_t>((uint64_t)c.max_blocks_per_seq * c.block_size, k::kWholeContext);
         auto rotation = [&](Mixer &m) {
             const Rotation r = rotation_of(m.cfg);
@@ -999,9 +1101,14 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 m.rank_at = pad_to(m.de.qkv(), 8);
                 m.lo = low_rank ? m.rank_at + pad_to(g.decay_rank, 8) + g.gate_rank : m.gate_at + ow;
                 m.hi = lightning ? 0 : low_rank ? g.heads : 2 * g.heads;
+            } else if (g.mixer == FA_MIXER_MINGRU) {
+                m.lo = ow;
+                m.hi = 2 * ow;
             } else if (g.mixer == FA_MIXER_ATTENTION) {
                 const bool own_kv = g.kv_from < 0;
                 m.hi = g.heads * g.dim + (own_kv ? g.kv_heads * g.dim + (g.attention & FA_ATTENTION_KEY_VALUES ? 0 : g.kv_heads * g.vdim) : 0);
+                m.head_gate_at = m.hi;
+                if (g.attention & FA_ATTENTION_HEAD_GATE) m.hi += g.heads;
                 m.lo = g.attention & FA_ATTENTION_GATE ? ow : 0;
             } else {
                 m.hi = g.q_rank + (g.kv_from < 0 ? g.kv_rank + g.rot_dim : 0) + (g.ungated ? 0 : g.heads);
@@ -1047,15 +1154,27 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 lin(m.prefix + "a", H, D, l.in, hi + H);
             }
         };
+        auto set_gated = [&](Mixer &m, const Layer &l) {
+            const uint32_t ow = m.out_width(), hi = l.lo + m.hi_at;
+            L->has_state = true;
+            m.z_bias = (float *)own(FA_F32, k::gated_pitch(ow));
+            m.u_bias = (float *)own(FA_F32, k::gated_pitch(ow));
+            lin(m.prefix + "z", ow, D, l.in, hi);
+            lin(m.prefix + "x", ow, D, l.in, hi + ow);
+            lin(m.prefix + "g", ow, D, l.in, m.lo_at);
+            vec(m.prefix + "z.b", ow, 0, m.z_bias);
+            vec(m.prefix + "x.b", ow, 0, m.u_bias);
+            m.state = (float *)own(FA_F32, (uint64_t)c.state_slots * k::gated_pitch(ow));
+        };
         auto set_attention = [&](Mixer &m, Layer &l) {
             const fa_layer_config &g = m.cfg;
             const uint32_t H = g.heads, hi = l.lo + m.hi_at;
             k::AttentionShape &a = m.at;
             a = k::AttentionShape{H, g.kv_heads, g.dim, g.vdim, 0, 0, g.scale, c.norm_eps, (uint64_t)c.num_blocks * c.block_size,
-                                  g.window ? std::min(g.window, k::kWholeContext) : k::kWholeContext, g.rot_dim, g.rot_interleaved ? 1u : 0u};
+                                  g.window ? std::min(g.window, k::kWholeContext) : k::kWholeContext, g.rot_dim, g.rot_interleaved ? 1u : 0u, g.q_temp, g.q_temp_every};
             k::attention_pad(a);
             const bool own_kv = g.kv_from < 0, bias = g.attention & FA_ATTENTION_BIAS, norms = g.attention & FA_ATTENTION_QK_NORM;
-            const uint32_t nq = H * g.dim, nk = own_kv ? g.kv_heads * g.dim : 0, nv = m.hi - nq - nk;
+            const uint32_t nq = H * g.dim, nk = own_kv ? g.kv_heads * g.dim : 0, nv = m.head_gate_at - nq - nk;
             if (bias) l.in_bias = (float *)own(FA_F32, pad_to(nq + nk + nv, 4));
             const std::pair<const char *, std::pair<uint32_t, uint32_t>> parts[3] = {{"q", {0, nq}}, {"k", {nq, nk}}, {"v", {nq + nk, nv}}};
             for (const auto &[name, at] : parts) {
@@ -1075,6 +1194,14 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
                 m.k_norm = norm("k.norm", g.dim);
             }
             if (g.attention & FA_ATTENTION_SINK) m.sink = norm("sink", H);
+            if (g.attention & FA_ATTENTION_SIGMOID) m.score_bias = norm("pb", H);
+            if (g.attention & FA_ATTENTION_HEAD_GATE) lin(m.prefix + "g", H, D, l.in, hi + m.head_gate_at);
+            if (g.distance != 0.0f) {
+                std::vector<float> slopes(H);
+                for (uint32_t h = 0; h < H; ++h) slopes[h] = (float)std::exp2(-(double)g.distance * (h + 1.0) / H);
+                m.slope = (float *)own(FA_F32, H);
+                if (st == FA_OK) st = fa_upload_into(ctx, slopes.data(), H, L->owned.back(), 0);
+            }
             if (g.attention & FA_ATTENTION_GATE) lin(m.prefix + "g", m.out_width(), D, l.in, m.lo_at + m.gate_at);
             if (g.rot_dim) rotation(m);
             if (own_kv) {
@@ -1185,6 +1312,7 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             l.out = weight(D, D, l.o_width);
             for (Mixer &m : l.mixers) {
                 if (recurrent(m.cfg)) set_recurrence(m, l);
+                else if (m.cfg.mixer == FA_MIXER_MINGRU) set_gated(m, l);
                 else if (m.cfg.mixer == FA_MIXER_ATTENTION) set_attention(m, l);
                 else set_latent(m, l);
                 lin(m.prefix + "o", D, m.out_width(), l.out, 0, 0, 0, m.o_at);
@@ -1204,19 +1332,38 @@ fa_status fa_decoder_create_layered(fa_context *ctx, const fa_layered_config *cf
             if (g.experts) {
                 l.router = weight(g.experts, g.experts, D);
                 lin(f + "router", g.experts, D, l.router, 0);
-                l.gate_up = weight(g.d_ffn, g.d_ffn, D, g.experts);
-                l.down = weight(D, D, g.d_ffn, g.experts);
+                if (g.route == FA_ROUTE_SCORED) {
+                    l.correction = (float *)own(FA_F32, g.experts);
+                    vec(f + "correction", g.experts, 0, l.correction);
+                }
+                const bool glu = g.glu == FA_GLU_SILU;
+                l.gate_up = weight(g.d_ffn, glu ? 2 * pad_to(g.d_ffn, 16) : g.d_ffn, D, l.lists());
+                l.down = weight(D, D, g.d_ffn, l.lists());
                 const auto one = [&](const k::LinearWeight &w, uint32_t e) {
                     k::LinearWeight t = w;
                     t.batches = 1;
                     t.w = (uint8_t *)w.w + (uint64_t)e * w.n_tiles * 16 * w.k_tiles * 32 * L->esz;
                     return t;
                 };
-                for (uint32_t e = 0; e < g.experts; ++e) {
+                for (uint32_t e = 0; e < l.lists(); ++e) {
                     const std::string x = f + "e" + std::to_string(e) + ".";
-                    lin(x + "up", g.d_ffn, D, one(l.gate_up, e), 0);
+                    if (glu) lin(x + "gate", g.d_ffn, D, one(l.gate_up, e), 0, 16, 32);
+                    if (glu) lin(x + "up", g.d_ffn, D, one(l.gate_up, e), 16, 16, 32);
+                    else lin(x + "up", g.d_ffn, D, one(l.gate_up, e), 0);
                     lin(x + "down", D, g.d_ffn, one(l.down, e), 0);
                 }
+            } else if (g.d_ffn && g.glu == FA_FFN_XIELU) {
+                l.gate_up = weight(g.d_ffn, g.d_ffn, D);
+                lin(f + "up", g.d_ffn, D, l.gate_up, 0);
+                l.down = weight(D, D, g.d_ffn);
+                lin(f + "down", D, g.d_ffn, l.down, 0);
+                l.act = (float *)own(FA_F32, 4);
+                float *act = l.act;
+                add(f + "act", 2, 0, [=](const void *src, int src_f32, hipStream_t s) {
+                    if (src_f32) (void)hipMemcpyAsync(act + 2, src, 8, hipMemcpyDeviceToDevice, s);
+                    else k::convert_bf16_to_f32((const uint16_t *)src, act + 2, 2, s);
+                    k::xielu_constants(act + 2, act, s);
+                });
             } else if (g.d_ffn) {
                 // gate and up alternate in tiles of 16 columns
                 l.gate_up = weight(g.d_ffn, 2 * pad_to(g.d_ffn, 16), D);

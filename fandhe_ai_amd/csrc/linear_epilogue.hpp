@@ -25,6 +25,8 @@ __device__ __forceinline__ float epilogue_value(const LinearEpilogue &ep, uint32
     } else if constexpr (MODE == LinearEpilogue::kSquaredRelu) {
         const float r = fmaxf(y, 0.0f);
         return r * r;
+    } else if constexpr (MODE == LinearEpilogue::kXielu) {
+        return (y > 0.0f ? ep.act[0] * y * y : ep.act[1] * (expm1f(y) - y)) + 0.5f * y;
     } else if constexpr (MODE == LinearEpilogue::kStore) {
         return y * ep.factor;
     } else {
@@ -41,7 +43,7 @@ __device__ __forceinline__ void epilogue_store1(const LinearEpilogue &ep, uint32
     if (MODE == LinearEpilogue::kStore && ep.bias) v += ep.bias[col];
     if constexpr (MODE == LinearEpilogue::kResidual) {
         float *o = (float *)ep.out + (uint64_t)row * ep.ld_out + col;
-        *o = *o + ep.scale[col] * v;
+        *o = *o + (ep.scale ? ep.scale[col] * v : v);
         return;
     }
     if (MODE == LinearEpilogue::kStore && col >= ep.n_lo) {
@@ -81,7 +83,7 @@ __device__ __forceinline__ void epilogue_store4(const LinearEpilogue &ep, uint32
     }
     if constexpr (MODE == LinearEpilogue::kResidual) {
         dev::v4f *p = (dev::v4f *)((float *)ep.out + o);
-        const dev::v4f r = *p, ls = *(const dev::v4f *)(ep.scale + col);
+        const dev::v4f r = *p, ls = ep.scale ? *(const dev::v4f *)(ep.scale + col) : dev::v4f{1.0f, 1.0f, 1.0f, 1.0f};
         *p = dev::v4f{r[0] + ls[0] * v[0], r[1] + ls[1] * v[1], r[2] + ls[2] * v[2], r[3] + ls[3] * v[3]};
     } else if (ep.out_f32) {
         *(dev::v4f *)((float *)ep.out + o) = dev::v4f{v[0], v[1], v[2], v[3]};

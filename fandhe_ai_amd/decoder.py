@@ -145,8 +145,8 @@ class Decoder:
 
 class LayeredDecoder(Decoder):
     """A decoder whose layers are described one by one (``fa_decoder_create_layered``): unquantized weights in bf16 or
-    f32, per layer one mixer or two side by side (gated delta rule or lightning attention with a recurrent state, attention,
-    latent or grouped-query, over the paged cache), and an optional feed-forward, dense or of sparse experts.  Sequences,
+    f32, per layer one mixer or two side by side (gated delta rule, lightning attention or a minimal gated recurrence with a
+    recurrent state, attention, latent or grouped-query, over the paged cache), and an optional feed-forward, dense or of sparse experts.  Sequences,
     steps, prompt passes and sampling are ``Decoder``'s."""
 
     takes_portions = True
@@ -157,7 +157,7 @@ class LayeredDecoder(Decoder):
         """layers: one dict of ``capi.LayerConfig`` fields per layer (``right``: such a dict, ``decay``: a list)."""
         self._ops = ops
         rows = (capi.LayerConfig * len(layers))(*[self._layer(l) for l in layers])
-        recurrent = any(m["mixer"] in (capi.MIXER_DELTA, capi.MIXER_LIGHTNING) for l in layers for m in (l, l.get("right") or l))
+        recurrent = any(m["mixer"] in (capi.MIXER_DELTA, capi.MIXER_LIGHTNING, capi.MIXER_MINGRU) for l in layers for m in (l, l.get("right") or l))
         slots = max_batch if state_slots is None else state_slots
         self.cfg = capi.LayeredConfig(len(layers), d_model, vocab, block_size, max_blocks_per_seq, num_blocks, max_batch,
                                       slots, norm_eps, logit_softcap, dtype, rows, norm, embed_scale, position_base, logit_scale)

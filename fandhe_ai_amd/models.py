@@ -230,8 +230,69 @@ def bubetar(config, shapes):
             "logit_softcap": config.get("logit_softcap") or 0.0, "logit_scale": 1.0 if scale is None else scale}
 
 
+# ---- Lugipel: minimal gated recurrences and windowed sigmoid attention, dense xIELU or sparse feed-forwards --------
+
+DISTANCE_SPAN = 8.0                                        # slopes of the distance bias fall to 2^-8 over the heads
+
+
+def _mingru(mx, where):
+    return {"mixer": capi.MIXER_MINGRU, "heads": 1, "dim": 1, "vdim": _entry(mx, "width", where), "kv_from": -1}
+
+
+def _sigmoid_attention(mx, where):
+    l = {key: _entry(mx, key, where) for key in ("heads", "kv_heads", "dim", "vdim", "scale")}
+    temp = _entry(mx, "q_temp", where)
+    every = _entry(temp, "every", where + " q_temp")
+    if every != int(every) or every < 1:
+        raise ConfigError("%s: q_temp.every must be a positive whole number" % where)
+    return dict(l, mixer=capi.MIXER_ATTENTION, attention=capi.ATTENTION_HEAD_NORM | capi.ATTENTION_SIGMOID | capi.ATTENTION_HEAD_GATE, kv_from=-1,
+                window=_entry(_entry(mx, "mask", where), "size", where + " mask"), distance=DISTANCE_SPAN,
+                q_temp=_entry(temp, "coef", where + " q_temp"), q_temp_every=int(every))
+
+
+def _scored_experts(mlp, where):
+    """SiLU GLU experts chosen by scores, some of whose router outputs return the input."""
+    router = _entry(mlp, "router", where)
+    identity, at = router.get("identity") or 0, where + " router"
+    l = {"d_ffn": _entry(_entry(mlp, "expert", where), "ff", where + " expert"), "experts": _entry(router, "experts", at) + identity,
+         "identity": identity, "top": _entry(router, "top", at), "glu": capi.GLU_SILU, "route": capi.ROUTE_SCORED,
+         "route_scale": _entry(router, "scale", at)}
+    if router.get("groups"):
+        l.update(groups=_entry(router["groups"], "count", at + " groups"), groups_kept=_entry(router["groups"], "keep", at + " groups"))
+    return l
+
+
+def lugipel_layers(config):
+    """config.json's layer list as ``capi.LayerConfig`` fields."""
+    out, mixers = [], {"mingru": _mingru, "attention": _sigmoid_attention}
+    for i, layer in enumerate(_entry(config, "layers", CONFIG_FILE)):
+        where = "layer %d" % i
+        kind, mlp = _entry(layer, "type", where), layer.get("mlp")
+        if kind not in mixers:
+            raise ConfigError("%s: unknown type %r" % (where, kind))
+        l = mixers[kind](_entry(layer, "mixer", where), where + " mixer")
+        if mlp is not None:
+            ff = _entry(mlp, "kind", where + " mlp")
+            if ff == "dense":
+                l.update(d_ffn=_entry(mlp, "ff", where + " mlp"), glu=capi.FFN_XIELU)
+            elif ff == "moe":
+                l.update(_scored_experts(mlp, where + " mlp"))
+            else:
+                raise ConfigError("%s: unknown feed-forward %r" % (where, ff))
+        out.append(l)
+    return out
+
+
+def lugipel(config):
+    """A Lugipel configuration as ``LayeredDecoder`` arguments."""
+    return {"d_model": _entry(config, "width", CONFIG_FILE), "vocab": _entry(config, "vocab", CONFIG_FILE), "layers": lugipel_layers(config),
+            "norm_eps": _entry(_entry(config, "norm", CONFIG_FILE), "eps", "norm"), "logit_softcap": 0.0, "norm": capi.NORM_INPUT_RMS,
+            "embed_scale": _entry(_entry(config, "embedding", CONFIG_FILE), "scale", "embedding"), "position_base": POSITION_BASE}
+
+
 # designs made of described layers: architecture name -> function(config, shapes of the weights) -> LayeredDecoder arguments
-LAYERED = {"Nugelix": lambda config, shapes: nugelix(config), "Zoferax": lambda config, shapes: zoferax(config), "Bubetar": bubetar}
+LAYERED = {"Nugelix": lambda config, shapes: nugelix(config), "Zoferax": lambda config, shapes: zoferax(config), "Bubetar": bubetar,
+           "Lugipel": lambda config, shapes: lugipel(config)}
 
 
 def build_layered(ops, config, dtype, capacity, shapes=None):
@@ -263,6 +324,7 @@ def install_weights(decoder, typed):
 @register("Nugelix")
 @register("Zoferax")
 @register("Bubetar")
+@register("Lugipel")
 def _layered(ops, config, weights, dtype, capacity):
     typed = st.load_safetensors_typed(weights)
     decoder = build_layered(ops, config, dtype, capacity, {n: t.shape for n, t in typed.items()})

@@ -565,26 +565,34 @@ fa_status fa_decoder_logits_buffer(fa_decoder *dec, fa_buffer **out);
 
 /* -------------------------------------------------------- layered decoders */
 /* A decoder whose layers are described one by one, on unquantized weights: per layer one mixer or two side by side (gated
- * delta rule or lightning attention with a recurrent state; latent attention or grouped-query attention over the paged
- * cache) and an optional feed-forward (a gated linear unit, or sparse experts).  No counterpart in the reference.  It is an
+ * delta rule, lightning attention or a minimal gated recurrence with a recurrent state; latent attention or grouped-query attention
+ * over the paged cache) and an optional feed-forward (dense, or sparse experts).  No counterpart in the reference.  It is an
  * fa_decoder: sequences, tokens, sampling, steps, prompt passes, verification and the read-outs are the calls above. */
-typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1, FA_MIXER_ATTENTION = 2, FA_MIXER_LIGHTNING = 3 } fa_mixer_kind;
+typedef enum { FA_MIXER_DELTA = 0, FA_MIXER_LATENT_ATTENTION = 1, FA_MIXER_ATTENTION = 2, FA_MIXER_LIGHTNING = 3,
+               FA_MIXER_MINGRU = 4 } fa_mixer_kind;
 /* How sublayers meet the residual stream x.  FA_NORM_INPUT: x += scale * f(layer_norm(x)), a layer scale per channel;
- * FA_NORM_OUTPUT: x += rms_norm(f(x)); FA_NORM_BOTH: x += layer_norm(f(layer_norm(x))).  The final norm is of the same
- * kind (layer norm for the last). */
-typedef enum { FA_NORM_INPUT = 0, FA_NORM_OUTPUT = 1, FA_NORM_BOTH = 2 } fa_norm_kind;
+ * FA_NORM_OUTPUT: x += rms_norm(f(x)); FA_NORM_BOTH: x += layer_norm(f(layer_norm(x))); FA_NORM_INPUT_RMS:
+ * x += f(rms_norm(x)).  The final norm is of the same kind (layer norm for FA_NORM_BOTH). */
+typedef enum { FA_NORM_INPUT = 0, FA_NORM_OUTPUT = 1, FA_NORM_BOTH = 2, FA_NORM_INPUT_RMS = 3 } fa_norm_kind;
 /* Attention: projections with biases; RMS norm of the whole query and key projections, over all heads at once; RMS norm per
  * head with a weight [dim] that the heads share (before the rotation), or without a weight; the projected keys are the
  * values (vdim = dim); the heads' outputs times the sigmoid of a further projection; a learned score per head that has no
- * key and no value and takes its share of the softmax. */
+ * key and no value and takes its share of the softmax; no softmax, the weight of a visible key being the sigmoid of its score
+ * plus a learned bias per head; the heads' outputs times the sigmoid of one number per head. */
 enum { FA_ATTENTION_BIAS = 1, FA_ATTENTION_QK_NORM = 2, FA_ATTENTION_HEAD_NORM = 4, FA_ATTENTION_HEAD_UNIT = 8, FA_ATTENTION_KEY_VALUES = 16,
-       FA_ATTENTION_GATE = 32, FA_ATTENTION_SINK = 64 };
-/* The feed-forward's gated linear unit.  Clamped: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + 1);
- * silu: gate sigmoid(gate) up. */
-typedef enum { FA_GLU_CLAMPED = 0, FA_GLU_SILU = 1 } fa_glu_kind;
+       FA_ATTENTION_GATE = 32, FA_ATTENTION_SINK = 64, FA_ATTENTION_SIGMOID = 128, FA_ATTENTION_HEAD_GATE = 256 };
+/* The feed-forward.  Clamped GLU: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + 1); silu GLU:
+ * gate sigmoid(gate) up; xIELU, without a gate, learned p and q: softplus(p) z^2 + z / 2 above 0, (1/2 + softplus(q)) (e^z - 1 - z) +
+ * z / 2 below. */
+typedef enum { FA_GLU_CLAMPED = 0, FA_GLU_SILU = 1, FA_FFN_XIELU = 2 } fa_glu_kind;
+/* The choice of experts from the router logits.  Chosen: the `top` largest logits, a softmax over those.  Scored: scores s = softmax over
+ * all router outputs; the `top` largest s + correction, taken from the groups_kept of `groups` neighbouring groups with the largest
+ * maxima; weights s / (sum of the chosen s + 1e-20) route_scale. */
+typedef enum { FA_ROUTE_CHOSEN = 0, FA_ROUTE_SCORED = 1 } fa_route_kind;
 typedef struct fa_layer_config {
     int32_t mixer;                /* fa_mixer_kind */
-    uint32_t heads, dim, vdim;    /* per head: query / key dims (latent attention: the unrotated part), value dims */
+    uint32_t heads, dim, vdim;    /* per head: query / key dims (latent attention: the unrotated part), value dims; minimal gated recurrence: heads 1,
+                                     vdim its width */
     uint32_t kv_heads, conv;      /* delta: q / k heads, taps of the short convolution (1..=16); attention: key / value heads */
     uint32_t q_rank, kv_rank;     /* latent attention: sizes of the two latents */
     uint32_t rot_dim, window;     /* rotated dims (even): latent attention's rotated part; attention: the first ones of every query and key
@@ -595,9 +603,9 @@ typedef struct fa_layer_config {
     uint32_t d_ffn;               /* 0: no feed-forward; with experts: size of one */
     float ffn_limit, ffn_alpha;   /* FA_GLU_CLAMPED */
     uint32_t attention;           /* attention: FA_ATTENTION_* */
-    uint32_t experts, top;        /* experts > 0 (up to 256): every token takes `top` (up to 64) of them, weighted by a softmax over their
-                                     router logits; an expert is W_down relu(W_up x)^2.  With FA_NORM_OUTPUT only */
-    int32_t glu;                  /* fa_glu_kind */
+    uint32_t experts, top;        /* experts > 0: every token takes `top` (up to 64) of the router's outputs (experts and identity experts,
+                                     up to 256).  With FA_NORM_OUTPUT and FA_NORM_INPUT_RMS */
+    int32_t glu;                  /* fa_glu_kind; experts: FA_GLU_SILU, or FA_GLU_CLAMPED for W_down relu(W_up x)^2 */
     uint32_t rot_interleaved;     /* pairs of the rotation: 0: i and i + rot_dim / 2, 1: 2i and 2i + 1 */
     /* rot_factor > 0: frequencies of fewer than rot_low turns within rot_original positions are divided by it, of more than
        rot_high turns kept, with a linear ramp between */
@@ -610,6 +618,14 @@ typedef struct fa_layer_config {
                                      unused); the outputs are added as left_scale, right_scale times each.  Tensors are then
                                      named mix.left.* and mix.right.* */
     float left_scale, right_scale;
+    /* attention: scores less 2^(-distance (h + 1) / heads) times the distance of the key, h from 0 (0: none); queries times
+       1 + q_temp ln(floor((position + 1) / q_temp_every) + 1) (0: one) */
+    float distance, q_temp;
+    uint32_t q_temp_every;
+    /* experts: how they are chosen; the router's last `identity` outputs stand for experts that return their input */
+    int32_t route;                /* fa_route_kind; the rest but identity: FA_ROUTE_SCORED */
+    uint32_t identity, groups, groups_kept;       /* groups 0: one */
+    float route_scale;
 } fa_layer_config;
 typedef struct {
     uint32_t n_layers, d_model, vocab;
@@ -621,7 +637,7 @@ typedef struct {
     const fa_layer_config *layers;        /* [n_layers], copied */
     int32_t norm;                 /* fa_norm_kind */
     float embed_scale;            /* factor of the embedding rows; 0: one */
-    double position_base;         /* FA_NORM_OUTPUT, above 0: sin(p base^(-2i / d_model)) is added to entry 2i of the embedding of position p, the
+    double position_base;         /* FA_NORM_OUTPUT and FA_NORM_INPUT_RMS, above 0: sin(p base^(-2i / d_model)) is added to entry 2i of the embedding of position p, the
                                      cosine to entry 2i + 1 */
     float logit_scale;            /* factor of the logits ahead of the soft cap; 0: one */
 } fa_layered_config;

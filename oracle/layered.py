@@ -2,7 +2,8 @@
 layer norm with layer scale, soft-capped head; grouped-query attention with normed projections, sparse experts, additive
 positions, norms on the sublayers' outputs; two mixers side by side, rotations of either layout with scaled frequencies, norms
 per head, output gates, sinks, lightning attention, the delta rule with a decay per channel, norms on both sides of a
-sublayer), one function per mechanism, in float64 and token by token.
+sublayer; minimal gated recurrence, attention with sigmoid weights, distance biases, query temperature and gates per head, xIELU
+feed-forward, experts in groups with identity experts), one function per mechanism, in float64 and token by token.
 
 TEST INFRASTRUCTURE ONLY: written from the equations, for whole sequences, without a cache, a batch or any code
 of the product; only tests and the smoke check may import it.
@@ -369,12 +370,137 @@ def forward_bubetar(config, w, tokens, layers_out=None):
     return softcap(layer_norm(x, w["final.norm"], eps) @ w["head"].T * config["logit_scale"], config["logit_softcap"])
 
 
+# ---- Lugipel ---------------------------------------------------------------------------------------------------
+
+def gated_recurrence(z, candidate):
+    """S <- (1 - z) S + z candidate, entry by entry; z, candidate [T, width] -> every S."""
+    S = np.zeros(z.shape[1])
+    out = np.empty_like(z)
+    for t in range(len(z)):
+        S = (1.0 - z[t]) * S + z[t] * candidate[t]
+        out[t] = S
+    return out
+
+
+def positive_candidate(u):
+    """u + 1/2 from zero on, the logistic function below: continuous and never negative."""
+    return np.where(u >= 0.0, u + 0.5, sigmoid(np.minimum(u, 0.0)))
+
+
+def mingru_mixer(h, w, p):
+    """The recurrence's gates read the current token only."""
+    z = sigmoid(h @ w[p + "z"].T + w[p + "z.b"])
+    S = gated_recurrence(z, positive_candidate(h @ w[p + "x"].T + w[p + "x.b"]))
+    return (S * silu(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def query_temperature(positions, coef, every):
+    """1 in the first `every` - 1 positions, growing with the logarithm of the number of whole blocks seen."""
+    return np.array([1.0 + coef * np.log(float((p + 1) // every) + 1.0) for p in positions])
+
+
+def distance_slopes(heads):
+    """Geometric from 2^(-8 / heads) down to 2^-8."""
+    return np.array([2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)])
+
+
+def sigmoid_attention(q, k, v, scale, window, slopes, bias):
+    """Weights sigmoid(q . k scale - slope (i - j) + bias), not normalized; position i sees the last `window` tokens."""
+    T, H = q.shape[:2]
+    share = H // k.shape[1]
+    out = np.empty((T, H, v.shape[2]))
+    for t in range(T):
+        j = np.arange(0 if window is None else max(0, t - window + 1), t + 1)
+        for h in range(H):
+            s = k[j, h // share] @ q[t, h] * scale - slopes[h] * (t - j) + bias[h]
+            out[t, h] = sigmoid(s) @ v[j, h // share]
+    return out
+
+
+def sigmoid_attention_mixer(h, w, p, mx, eps):
+    T, H, G, d = len(h), mx["heads"], mx["kv_heads"], mx["dim"]
+    q = rms_norm((h @ w[p + "q"].T).reshape(T, H, d), w[p + "q.norm"], eps)
+    k = rms_norm((h @ w[p + "k"].T).reshape(T, G, d), w[p + "k.norm"], eps)
+    q = q * query_temperature(range(T), mx["q_temp"]["coef"], mx["q_temp"]["every"])[:, None, None]
+    o = sigmoid_attention(q, k, (h @ w[p + "v"].T).reshape(T, G, mx["vdim"]), mx["scale"], mx["mask"]["size"], distance_slopes(H), w[p + "pb"])
+    return (o * sigmoid(h @ w[p + "g"].T)[:, :, None]).reshape(T, -1) @ w[p + "o"].T
+
+
+def xielu(z, p, q):
+    n = np.minimum(z, 0.0)
+    return np.where(z > 0.0, softplus(p) * z * z, (0.5 + softplus(q)) * (np.expm1(n) - n)) + 0.5 * z
+
+
+def xielu_forward(h, w, p):
+    return xielu(h @ w[p + "up"].T, *w[p + "act"]) @ w[p + "down"].T
+
+
+def grouped_choice(s, correction, top, groups, keep):
+    """The chosen experts of one row of scores, and how close the choice is: the least distance of a choice score, or of a
+    group's, to one on the other side."""
+    c = s + correction
+    size = len(c) // groups
+    best = c.reshape(groups, size).max(axis=1)
+    order = np.argsort(-best, kind="stable")
+    margin = best[order[keep - 1]] - best[order[keep]] if keep < groups else np.inf
+    allowed = np.repeat(np.isin(np.arange(groups), order[:keep]), size)
+    c = np.where(allowed, c, -np.inf)
+    order = np.argsort(-c, kind="stable")
+    if top < int(allowed.sum()):
+        margin = min(margin, c[order[top - 1]] - c[order[top]])
+    return order[:top], margin
+
+
+def route_scored(z, correction, router):
+    """Router logits [T, outputs] -> weights [T, outputs] and choice margins [T]."""
+    groups = router.get("groups") or {"count": 1, "keep": 1}
+    out, margins = np.zeros_like(z), np.empty(len(z))
+    for t, row in enumerate(z):
+        e = np.exp(row - row.max())
+        s = e / e.sum()
+        best, margins[t] = grouped_choice(s, correction, router["top"], groups["count"], groups["keep"])
+        out[t, best] = s[best] / (s[best].sum() + 1e-20) * router["scale"]
+    return out, margins
+
+
+def scored_experts(h, w, p, mlp, margins=None):
+    """Sparse SiLU GLU experts; the last router outputs belong to experts that return their input."""
+    router = mlp["router"]
+    g, m = route_scored(h @ w[p + "router"].T, w[p + "correction"], router)
+    if margins is not None:
+        margins.append(m)
+    n = router["experts"]
+    y = g[:, n:].sum(axis=1, keepdims=True) * h
+    for e in range(n):
+        rows = np.nonzero(g[:, e])[0]
+        y[rows] += g[rows, e:e + 1] * silu_glu(h[rows], w, p + "e%d." % e)
+    return y
+
+
+def forward_lugipel(config, w, tokens, layers_out=None, margins=None):
+    """RMS norms ahead of every sublayer, additive positions."""
+    eps = config["norm"]["eps"]
+    x = w["embed"][np.asarray(tokens, dtype=np.int64)] * config["embedding"]["scale"] + sinusoid(np.arange(len(tokens)), config["width"])
+    for i, layer in enumerate(config["layers"]):
+        p, mx = "l%d." % i, layer["mixer"]
+        h = rms_norm(x, w[p + "norm1"], eps)
+        x = x + (mingru_mixer(h, w, p + "mix.") if layer["type"] == "mingru" else sigmoid_attention_mixer(h, w, p + "mix.", mx, eps))
+        if layer["mlp"] is not None:
+            h = rms_norm(x, w[p + "norm2"], eps)
+            x = x + (xielu_forward(h, w, p + "mlp.") if layer["mlp"]["kind"] == "dense" else scored_experts(h, w, p + "mlp.", layer["mlp"], margins))
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return rms_norm(x, w["final.norm"], eps) @ w["head"].T
+
+
 def forward(config, weights, tokens, layers_out=None, margins=None):
     """Logits [T, vocab] of one whole sequence; layers_out (a list) receives the residual after every layer, margins (a
     list) the routing margins of every layer of sparse experts."""
     w = {n: np.asarray(a, dtype=np.float64) for n, a in weights.items()}
     if config["architecture"] == "Zoferax":
         return forward_zoferax(config, w, tokens, layers_out, margins)
+    if config["architecture"] == "Lugipel":
+        return forward_lugipel(config, w, tokens, layers_out, margins)
     if config["architecture"] == "Bubetar":
         return forward_bubetar(config, w, tokens, layers_out)
     eps = config["norm"]["eps"]
