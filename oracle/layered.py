@@ -437,9 +437,9 @@ def xielu_forward(h, w, p):
 
 def grouped_choice(s, correction, top, groups, keep):
     """The chosen experts of one row of scores, and how close the choice is: the least distance of a choice score, or of a
-    group's, to one on the other side."""
+    group's, to one on the other side, relative to the scores' spread."""
     c = s + correction
-    size = len(c) // groups
+    size, spread = len(c) // groups, s.std() + 1e-30
     best = c.reshape(groups, size).max(axis=1)
     order = np.argsort(-best, kind="stable")
     margin = best[order[keep - 1]] - best[order[keep]] if keep < groups else np.inf
@@ -448,7 +448,7 @@ def grouped_choice(s, correction, top, groups, keep):
     order = np.argsort(-c, kind="stable")
     if top < int(allowed.sum()):
         margin = min(margin, c[order[top - 1]] - c[order[top]])
-    return order[:top], margin
+    return order[:top], margin / spread
 
 
 def route_scored(z, correction, router):

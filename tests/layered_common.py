@@ -97,6 +97,30 @@ def bubetar(layers, width=76, vocab=131, eps=1e-5, softcap=12.0, scale=0.8, rank
             "_ranks": ranks}
 
 
+def sigmoid_attention(heads=6, kv_heads=2, dim=20, vdim=12, window=13, scale=None, coef=0.6, every=8, mlp=None):
+    mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": 1.5 * dim ** -0.5 if scale is None else scale, "mask": {"size": window},
+          "q_temp": {"coef": coef, "every": every}}
+    return {"type": "attention", "mixer": mx, "mlp": mlp}
+
+
+def mingru(width=52, mlp=None):
+    return {"type": "mingru", "mixer": {"width": width}, "mlp": mlp}
+
+
+def scored(n=6, identity=3, groups=(3, 2), top=3, ff=28, scale=1.6):
+    """groups: count and those kept; None for none."""
+    router = {"experts": n, "top": top, "scale": scale}
+    if identity:
+        router["identity"] = identity
+    if groups:
+        router["groups"] = {"count": groups[0], "keep": groups[1]}
+    return {"kind": "moe", "expert": {"ff": ff}, "router": router}
+
+
+def lugipel(layers, width=76, vocab=131, eps=1e-5, scale=1.7):
+    return {"architecture": "Lugipel", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps}, "embedding": {"scale": scale}}
+
+
 def bf16_round(a):
     u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
     return ((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32).view(np.float32)
@@ -147,7 +171,36 @@ def bubetar_shapes(cfg):
     return out
 
 
+def lugipel_shapes(cfg):
+    D = cfg["width"]
+    out = {"embed": (cfg["vocab"], D), "head": (cfg["vocab"], D), "final.norm": (D,)}
+    for i, l in enumerate(cfg["layers"]):
+        p, m, f, mx = "l%d." % i, "l%d.mix." % i, "l%d.mlp." % i, l["mixer"]
+        out[p + "norm1"] = (D,)
+        if l["type"] == "mingru":
+            wide = mx["width"]
+            out.update({m + "z": (wide, D), m + "z.b": (wide,), m + "x": (wide, D), m + "x.b": (wide,), m + "g": (wide, D), m + "o": (D, wide)})
+        else:
+            H, G, d, v = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+            out.update({m + "q": (H * d, D), m + "k": (G * d, D), m + "v": (G * v, D), m + "q.norm": (d,), m + "k.norm": (d,), m + "pb": (H,), m + "g": (H, D),
+                        m + "o": (D, H * v)})
+        if not l["mlp"]:
+            continue
+        out[p + "norm2"] = (D,)
+        if l["mlp"]["kind"] == "dense":
+            out.update({f + "up": (l["mlp"]["ff"], D), f + "down": (D, l["mlp"]["ff"]), f + "act": (2,)})
+        else:
+            r, ff = l["mlp"]["router"], l["mlp"]["expert"]["ff"]
+            n = r["experts"] + r.get("identity", 0)
+            out.update({f + "router": (n, D), f + "correction": (n,)})
+            for e in range(r["experts"]):
+                out.update({f + "e%d.gate" % e: (ff, D), f + "e%d.up" % e: (ff, D), f + "e%d.down" % e: (D, ff)})
+    return out
+
+
 def shapes(cfg):
+    if cfg["architecture"] == "Lugipel":
+        return lugipel_shapes(cfg)
     if cfg["architecture"] == "Bubetar":
         return bubetar_shapes(cfg)
     if cfg["architecture"] == "Zoferax":
@@ -190,6 +243,8 @@ def weights(cfg, seed=0):
             a = rng.normal(0, 0.6, shape)
         elif "norm" in leaf:
             a = 1.0 + 0.3 * rng.normal(size=shape)
+        elif leaf == "correction":
+            a = 0.15 * rng.normal(size=shape) - 0.1
         elif leaf in ("ls1", "ls2"):
             a = rng.uniform(0.3, 1.2, shape) * rng.choice([-1.0, 1.0], shape)
         elif leaf == "embed" or len(shape) == 1:               # also the projections' biases

@@ -313,11 +313,151 @@ def test_another_reading_of_a_bubetar_mechanism_exceeds_the_gpu_tests_tolerance(
     assert lc.error(oracle.forward(cfg, w, toks), good) > 30 * 2e-4
 
 
+# ---- Lugipel ---------------------------------------------------------------------------------------------------
+
+def test_gated_recurrence_closed_forms():
+    rng = np.random.default_rng(0)
+    c = rng.normal(size=(9, 3))
+    z = np.zeros((9, 3))
+    z[2], z[5:, 1] = 1.0, 0.5
+    S = oracle.gated_recurrence(z, c)
+    assert (S[:2] == 0.0).all() and np.allclose(S[2:5], c[2]) and np.allclose(S[-1, 0], c[2, 0])       # written once, kept
+    assert np.allclose(S[6, 1], 0.25 * c[2, 1] + 0.25 * c[5, 1] + 0.5 * c[6, 1])
+    u = oracle.positive_candidate(np.array([-40.0, -1e-9, 0.0, 2.0]))
+    assert np.allclose(u, [0.0, 0.5, 0.5, 2.5])
+
+
+def test_sigmoid_attention_sums_what_it_sees():
+    rng = np.random.default_rng(1)
+    q, k, v = rng.normal(size=(12, 4, 5)), rng.normal(size=(12, 2, 5)), rng.normal(size=(12, 2, 3))
+    slopes = oracle.distance_slopes(4)
+    assert np.allclose(slopes, [0.25, 0.0625, 1 / 64.0, 1 / 256.0]) and np.allclose(oracle.distance_slopes(1), [2.0 ** -8])
+    o = oracle.sigmoid_attention(q, k, v, 0.0, 4, 0.0 * slopes, np.full(4, 50.0))                       # every weight one
+    assert np.allclose(o[9, 1], v[6:10, 0].sum(axis=0)) and np.allclose(o[2, 3], v[:3, 1].sum(axis=0))
+    o = oracle.sigmoid_attention(q, k, v, 0.7, 1, slopes, np.zeros(4))
+    assert np.allclose(o[5, 2], v[5, 1] / (1.0 + np.exp(-0.7 * q[5, 2] @ k[5, 1])))
+    o = oracle.sigmoid_attention(q, 0.0 * k, v, 1.0, None, slopes, np.zeros(4))
+    assert np.allclose(o[7, 0], sum(v[j, 0] / (1.0 + np.exp(0.25 * (7 - j))) for j in range(8)))
+
+
+def test_query_temperature_steps_once_a_block_is_whole():
+    t = oracle.query_temperature(range(20), 0.5, 8)
+    assert (t[:7] == 1.0).all() and np.allclose(t[7:15], 1.0 + 0.5 * np.log(2.0)) and np.allclose(t[15:], 1.0 + 0.5 * np.log(3.0))
+
+
+def test_xielu_closed_forms():
+    p, q = np.log(np.expm1(0.8)), np.log(np.expm1(0.3))                # softplus gives 0.8 and 0.3
+    z = np.array([-2.0, -1e-6, 0.0, 1.5])
+    want = [0.8 * (np.exp(-2.0) + 1.0) - 1.0, -0.5e-6, 0.0, 0.8 * 2.25 + 0.75]
+    assert np.allclose(oracle.xielu(z, p, q), want)
+
+
+def test_experts_are_chosen_from_the_best_groups_by_corrected_scores():
+    s = np.array([0.30, 0.05, 0.20, 0.10, 0.25, 0.10])
+    none = np.zeros(6)
+    assert sorted(oracle.grouped_choice(s, none, 3, 1, 1)[0]) == [0, 2, 4]
+    assert sorted(oracle.grouped_choice(s, none, 3, 3, 2)[0]) == [0, 4, 5]          # the middle pair is left out
+    assert sorted(oracle.grouped_choice(s, none - 1.0, 4, 3, 2)[0]) == [0, 1, 4, 5]  # and stays out where all are negative
+    assert sorted(oracle.grouped_choice(s, np.array([-1.0, 0, 0, 1.0, 0, 0]), 2, 3, 1)[0]) == [2, 3]
+    z = np.log(s)[None]
+    g, _ = oracle.route_scored(z, np.array([-1.0, 0, 0, 1.0, 0, 0]), {"top": 2, "scale": 3.0, "groups": {"count": 3, "keep": 1}})
+    assert np.allclose(g, [[0, 0, 2.0, 1.0, 0, 0]])                                 # weights know no correction
+    rng = np.random.default_rng(2)
+    h = rng.normal(size=(4, 5))
+    w = {"m.router": np.zeros((3, 5)), "m.correction": np.array([0.0, 0.0, 1.0])}
+    w.update({"m.e%d.%s" % (e, n): rng.normal(size=(5, 5)) for e in (0, 1) for n in ("gate", "up", "down")})
+    y = oracle.scored_experts(h, w, "m.", {"router": {"experts": 2, "identity": 1, "top": 1, "scale": 0.5}})
+    assert np.allclose(y, 0.5 * h)
+
+
+def _lugipel():
+    layers = [lc.sigmoid_attention(mlp=lc.dense(40)), lc.mingru(mlp=lc.scored()), lc.sigmoid_attention(heads=4, window=9, mlp=lc.scored(5, 3, (4, 2), 3)), lc.mingru(30)]
+    cfg = lc.lugipel(layers)
+    return cfg, lc.weights(cfg, 5), lc.tokens(cfg, 40, 5)
+
+
+def _router(c, **change):
+    for l in c["layers"]:
+        if l["mlp"] and l["mlp"]["kind"] == "moe":
+            l["mlp"]["router"].update(change)
+
+
+LUGIPEL_MISTAKES = {
+    "embedding scale": lambda c: c["embedding"].update(scale=c["embedding"]["scale"] * 1.05),
+    "scores": lambda c: [m.update(scale=m["scale"] * 1.05) for m in _mixers(c, "attention")],
+    "window one longer": lambda c: [m["mask"].update(size=m["mask"]["size"] + 1) for m in _mixers(c, "attention")],
+    "window one shorter": lambda c: [m["mask"].update(size=m["mask"]["size"] - 1) for m in _mixers(c, "attention")],
+    "temperature": lambda c: [m["q_temp"].update(coef=m["q_temp"]["coef"] * 1.1) for m in _mixers(c, "attention")],
+    "temperature one position late": lambda c: [m["q_temp"].update(every=m["q_temp"]["every"] + 1) for m in _mixers(c, "attention")],
+    "experts' scale": lambda c: _router(c, scale=1.7),
+    "one expert fewer": lambda c: _router(c, top=2),
+    "all groups kept": lambda c: [l["mlp"]["router"]["groups"].update(keep=l["mlp"]["router"]["groups"]["count"]) for l in c["layers"][1:3]],
+    "no groups": lambda c: _router(c, groups=None),
+    "norm eps": lambda c: c["norm"].update(eps=0.05),
+    "feed-forward left out": lambda c: c["layers"][0].update(mlp=None),
+}
+
+
+@pytest.mark.parametrize("name", sorted(LUGIPEL_MISTAKES))
+def test_a_planted_mistake_in_a_lugipel_model_exceeds_the_gpu_tests_tolerance(name):
+    cfg, w, toks = _lugipel()
+    good = oracle.forward(cfg, w, toks)
+    wrong = copy.deepcopy(cfg)
+    LUGIPEL_MISTAKES[name](wrong)
+    assert lc.error(oracle.forward(wrong, w, toks), good) > 30 * 2e-4
+
+
+def _without_groups_forgotten(s, correction, top, groups, keep):
+    """Experts of the groups left out count as zero instead of minus infinity."""
+    c = s + correction
+    size = len(c) // groups
+    best = np.argsort(-c.reshape(groups, size).max(axis=1), kind="stable")[:keep]
+    c = np.where(np.repeat(np.isin(np.arange(groups), best), size), c, 0.0)
+    return np.argsort(-c, kind="stable")[:top], np.inf
+
+
+LUGIPEL_READINGS = {
+    "softmax": ("sigmoid_attention", lambda f: lambda q, k, v, s, w, m, b: oracle.sink_attention(q, k, v, s, w)),
+    "no distance": ("sigmoid_attention", lambda f: lambda q, k, v, s, w, m, b: f(q, k, v, s, w, 0 * m, b)),
+    "slopes of other heads": ("sigmoid_attention", lambda f: lambda q, k, v, s, w, m, b: f(q, k, v, s, w, m[::-1], b)),
+    "no bias per head": ("sigmoid_attention", lambda f: lambda q, k, v, s, w, m, b: f(q, k, v, s, w, m, 0 * b)),
+    "a scaled bias": ("sigmoid_attention", lambda f: lambda q, k, v, s, w, m, b: f(q, k, v, s, w, m, s * b)),
+    "weights that sum to one": ("sigmoid_attention", lambda f: lambda q, k, v, s, w, m, b: f(q, k, v, s, w, m, b) / f(q, k, np.ones_like(v), s, w, m, b)),
+    "temperature from the position before": ("query_temperature", lambda f: lambda p, c, e: f([i - 1 for i in p], c, e)),
+    "temperature that grows in between": ("query_temperature", lambda f: lambda p, c, e: np.array([1.0 + c * np.log((i + 1) / e + 1.0) for i in p])),
+    "keep and write exchanged": ("gated_recurrence", lambda f: lambda z, c: f(1.0 - z, c)),
+    "the state forgotten": ("gated_recurrence", lambda f: lambda z, c: np.concatenate([f(z[:20], c[:20]), f(z[20:], c[20:])])),
+    "a bare candidate": ("positive_candidate", lambda f: lambda u: u),
+    "a candidate without its half": ("positive_candidate", lambda f: lambda u: np.where(u >= 0.0, u, f(u))),
+    "corrected weights": ("route_scored", lambda f: lambda z, c, r: f(z + c, 0 * c, r)),
+    "groups left out count as zero": ("grouped_choice", lambda f: _without_groups_forgotten),
+    "activation of p and q exchanged": ("xielu", lambda f: lambda z, p, q: f(z, q, p)),
+    "activation without its half": ("xielu", lambda f: lambda z, p, q: f(z, p, q) - 0.5 * z),
+    "norms that take the mean off": ("rms_norm", lambda f: oracle.layer_norm),
+}
+
+
+@pytest.mark.parametrize("mistake", sorted(LUGIPEL_READINGS))
+def test_another_reading_of_a_lugipel_mechanism_exceeds_the_gpu_tests_tolerance(mistake, monkeypatch):
+    cfg, w, toks = _lugipel()
+    good = oracle.forward(cfg, w, toks)
+    name, change = LUGIPEL_READINGS[mistake]
+    monkeypatch.setattr(oracle, name, change(getattr(oracle, name)))
+    assert lc.error(oracle.forward(cfg, w, toks), good) > 30 * 2e-4
+
+
+@pytest.mark.parametrize("tensor", ["l0.mix.q.norm", "l0.mix.pb", "l0.mix.g", "l0.mlp.act", "l1.mix.z.b", "l1.mix.x.b", "l1.mlp.correction", "l3.mix.g", "final.norm"])
+def test_every_small_tensor_of_a_lugipel_model_counts(tensor):
+    cfg, w, toks = _lugipel()
+    wrong = dict(w, **{tensor: np.roll(w[tensor], 1, axis=0)})
+    assert lc.error(oracle.forward(cfg, wrong, toks), oracle.forward(cfg, w, toks)) > 30 * 2e-4
+
+
 # ---- configuration ---------------------------------------------------------------------------------------------
 
 def test_registry_picks_by_architecture_and_rejects_what_it_does_not_know(tmp_path):
     models = _fa().models
-    assert {"Nugelix", "Zoferax", "Bubetar", "LlamaForCausalLM"} <= set(models.ARCHITECTURES)
+    assert {"Nugelix", "Zoferax", "Bubetar", "Lugipel", "LlamaForCausalLM"} <= set(models.ARCHITECTURES)
     (tmp_path / "config.json").write_text(json.dumps({"architecture": "Nonesuch"}))
     with pytest.raises(models.ConfigError, match="unknown architecture"):
         models.load_model(None, str(tmp_path))
@@ -415,6 +555,41 @@ def test_bubetar_configuration_reads_every_size_and_names_what_is_missing():
     bad["layers"][0]["mixer"]["right"]["decay"].pop()
     with pytest.raises(models.ConfigError, match="decay"):
         models.bubetar(bad, shapes)
+
+
+def test_lugipel_configuration_reads_every_size_and_names_what_is_missing():
+    fa = _fa()
+    models, capi = fa.models, fa.capi
+    cfg = lc.lugipel([lc.sigmoid_attention(heads=12, kv_heads=4, dim=10, vdim=6, window=21, scale=0.25, coef=0.3, every=5, mlp=lc.dense(44)),
+                      lc.mingru(37, mlp=lc.scored(7, 5, (4, 3), 6, 18, 0.7)), lc.mingru(8, mlp=lc.scored(4, 0, None, 2, 9, 1.0)), lc.sigmoid_attention()], scale=2.5)
+    a = models.lugipel(cfg)
+    assert (a["d_model"], a["vocab"], a["norm"], a["embed_scale"], a["position_base"], a["norm_eps"]) == (76, 131, capi.NORM_INPUT_RMS, 2.5, 10000.0, 1e-5)
+    p, q, r, s = a["layers"]
+    assert (p["mixer"], p["heads"], p["kv_heads"], p["dim"], p["vdim"], p["scale"], p["window"]) == (capi.MIXER_ATTENTION, 12, 4, 10, 6, 0.25, 21)
+    assert p["attention"] == capi.ATTENTION_HEAD_NORM | capi.ATTENTION_SIGMOID | capi.ATTENTION_HEAD_GATE and p.get("rot_dim", 0) == 0
+    assert (p["distance"], p["q_temp"], p["q_temp_every"], p["d_ffn"], p["glu"]) == (8.0, 0.3, 5, 44, capi.FFN_XIELU)
+    assert (q["mixer"], q["heads"], q["vdim"]) == (capi.MIXER_MINGRU, 1, 37)
+    assert (q["experts"], q["identity"], q["top"], q["groups"], q["groups_kept"], q["d_ffn"], q["route_scale"]) == (12, 5, 6, 4, 3, 18, 0.7)
+    assert (q["route"], q["glu"]) == (capi.ROUTE_SCORED, capi.GLU_SILU)
+    assert (r["experts"], r["identity"], r["top"], r.get("groups", 0)) == (4, 0, 2, 0) and "d_ffn" not in s
+    for layer, path in ((0, ("mixer", "kv_heads")), (0, ("mixer", "q_temp", "every")), (0, ("mixer", "mask", "size")), (0, ("mlp", "ff")), (1, ("mixer", "width")),
+                        (1, ("mlp", "router", "scale")), (1, ("mlp", "router", "groups", "keep")), (1, ("mlp", "expert", "ff")), (2, ("type",)), (0, ("mlp", "kind"))):
+        bad = copy.deepcopy(cfg)
+        at = bad["layers"][layer]
+        for key in path[:-1]:
+            at = at[key]
+        del at[path[-1]]
+        with pytest.raises(models.ConfigError, match=path[-1]):
+            models.lugipel(bad)
+    for change in ({"type": "delta"}, {"mlp": {"kind": "glu", "ff": 3}}):
+        bad = copy.deepcopy(cfg)
+        bad["layers"][1].update(change)
+        with pytest.raises(models.ConfigError, match="unknown"):
+            models.lugipel(bad)
+    bad = copy.deepcopy(cfg)
+    bad["layers"][0]["mixer"]["q_temp"]["every"] = 2.5
+    with pytest.raises(models.ConfigError, match="every"):
+        models.lugipel(bad)
 
 
 # ---- batching on a fake decoder ---------------------------------------------------------------------------------
