@@ -105,7 +105,7 @@ def make_tables(rng, ctxs, extra_tokens, bs, num_blocks=None):
 
 
 # ------------------------------------------------------------------ layered decoders
-# Nugelix, Zoferax and Bubetar stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward
+# Nugelix, Zoferax, Bubetar and Lugipel stacks whose layers have a real model's sizes, and the W8A8 decoder of equal width, feed-forward
 # (of the experts: those one token takes) and depth.
 def _nugelix(width, heads, q_rank, window, ff, d_heads, d_kv_heads, repeat):
     latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff, "limit": 7.0},
@@ -143,11 +143,22 @@ def _bubetar(width, heads, kv_heads, q_rank, window, ff, repeat):
             "layers": (layers + [latent, latent]) * repeat}
 
 
+def _lugipel(width, heads, kv_heads, window, dense_ff, experts, identity, top, groups, ff, repeat):
+    dense, moe = {"kind": "dense", "ff": dense_ff}, {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "identity": identity, "top": top, "scale": 1.5,
+                                                     "groups": {"count": groups[0], "keep": groups[1]}}}
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "mask": {"size": window}, "q_temp": {"coef": 0.1, "every": 1024}, "scale": 128 ** -0.5}
+    layers = [("attention", mixer, dense), ("mingru", {"width": width}, moe), ("attention", mixer, moe), ("mingru", {"width": width}, moe)]
+    return {"architecture": "Lugipel", "width": width, "vocab": 32000, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+            "layers": [{"type": t, "mixer": m, "mlp": f} for t, m, f in layers] * repeat}
+
+
 LAYERED = {"large": dict(nugelix=_nugelix(4096, 32, 1536, 2048, 14336, 32, 16, 2), zoferax=_zoferax(4096, 32, 8, 128, 16, 4, 5376, 8, 3),
                          bubetar=_bubetar(4096, 32, 8, 1536, 2048, 14336, 2),
+                         lugipel=_lugipel(4096, 32, 8, 2048, 14336, 16, 4, 4, (5, 3), 3584, 2),
                          w8a8=dict(d_model=4096, n_heads=32, n_kv_heads=8, d_ffn=14336, n_layers=8, vocab=32000)),
            "small": dict(nugelix=_nugelix(2048, 16, 768, 1024, 8192, 16, 8, 2), zoferax=_zoferax(2048, 16, 4, 64, 16, 4, 3072, 8, 3),
                          bubetar=_bubetar(2048, 16, 4, 768, 1024, 8192, 2),
+                         lugipel=_lugipel(2048, 16, 4, 1024, 8192, 16, 4, 4, (5, 3), 2048, 2),
                          w8a8=dict(d_model=2048, n_heads=16, n_kv_heads=4, d_ffn=8192, n_layers=8, vocab=32000))}
 
 
@@ -158,20 +169,20 @@ def build_layered(fa, be, config, max_tokens, batch):
     made = {}                                                     # equal shapes hold equal values
     for name, shape in dec.tensors().items():
         n, leaf = int(np.prod(shape)), name.split(".")[-1]
-        kind = "one" if "norm" in leaf or leaf in ("ls1", "ls2") else "minus one" if leaf in ("A_log", "dt_bias") else "embed" if leaf == "embed" else "noise"
+        kind = "one" if "norm" in leaf or leaf in ("ls1", "ls2") else "minus one" if leaf in ("A_log", "dt_bias") else "zero" if leaf == "correction" else "few" if leaf == "pb" else "embed" if leaf == "embed" else "noise"
         if (shape, kind) not in made:
             if kind == "noise" and len(shape) == 2:
                 a = np.resize(noise, n).reshape(shape) * np.float32(shape[1] ** -0.5)
             elif kind in ("noise", "embed"):
                 a = np.resize(noise, n).reshape(shape)
             else:
-                a = np.full(shape, 1.0 if kind == "one" else -1.0, np.float32)
+                a = np.full(shape, {"one": 1.0, "minus one": -1.0, "zero": 0.0, "few": -8.0}[kind], np.float32)
             made[shape, kind] = (a.view(np.uint32) >> 16).astype(np.uint16)
         dec.set_tensor(name, made[shape, kind], bf16=True)
     return dec
 
 
-def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "zoferax", "bubetar", "w8a8")):
+def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1, 2048), (4, 2048)), steps=20, models=("nugelix", "zoferax", "bubetar", "lugipel", "w8a8")):
     """Decode and prompt throughput of layered stacks, and of the W8A8 decoder of equal width, feed-forward and depth."""
     lib = fa.capi.lib
     V = LAYERED[size]["w8a8"]["vocab"]
@@ -214,7 +225,7 @@ def bench_layered(fa, be, size, decode_batches=(1, 8, 32), ctx=4096, prompts=((1
             dec.set_sequences(t, [length] * b)
         return set_rows
 
-    for model in ("nugelix", "zoferax", "bubetar"):
+    for model in ("nugelix", "zoferax", "bubetar", "lugipel"):
         if model in models:
             dec = build_layered(fa, be, LAYERED[size][model], most * pages * 16, most)
             measure(model + " bf16", dec, rows_of(most * pages))
@@ -944,7 +955,7 @@ def main():
                     help="with --only layered: the sizes of the layered stacks (and of the W8A8 decoder beside them)")
     ap.add_argument("--layered-phase", choices=("all", "decode", "prompt"), default="all",
                     help="with --only layered: all, or one shape of one phase (for a kernel trace)")
-    ap.add_argument("--layered-model", choices=("all", "nugelix", "zoferax", "bubetar", "w8a8"), default="all", help="with --only layered: one of the decoders")
+    ap.add_argument("--layered-model", choices=("all", "nugelix", "zoferax", "bubetar", "lugipel", "w8a8"), default="all", help="with --only layered: one of the decoders")
     a = ap.parse_args()
     if a.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (--gpus 1); nothing here shards across devices")

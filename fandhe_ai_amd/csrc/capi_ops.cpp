@@ -15,7 +15,7 @@ namespace k {
 extern int g_gemm_f32_form, g_weight_prefetch, g_probe_plain_loads, g_rows_wide;
 extern int g_skinny_ksplit, g_skinny_ksplit_s, g_row_fusion;
 extern int g_rows_kernel;
-extern int g_linear_form, g_latent_form, g_latent_blocks, g_delta_form, g_attention_form, g_attention_blocks, g_route_form;
+extern int g_linear_form, g_latent_form, g_latent_blocks, g_delta_form, g_attention_form, g_attention_blocks, g_route_form, g_gated_lanes;
 extern int g_skinny_ntw, g_skinny_waves, g_skinny_astat, g_gemm_small_tiles, g_gemm_waves, g_gemm_ntb, g_gemm_split_fill;
 }
 int g_decode_waves = 0;
@@ -114,6 +114,7 @@ fa_status fa_set_tuning(int32_t key, int32_t value) {
         case 33: k::g_attention_form = value; return FA_OK;
         case 34: k::g_attention_blocks = value; return FA_OK;
         case 35: k::g_route_form = value; return FA_OK;
+        case 36: k::g_gated_lanes = value; return FA_OK;
     }
     return fail(FA_ERR_INVALID_ARGUMENT, "fa_set_tuning: unknown key");
 }

@@ -14,45 +14,55 @@ int g_route_form = 0;         // tuning: 1 the router in the residual update wha
 
 namespace {
 
+// The largest value of a row that is not taken yet (ties: the lower index), by one wavefront: value i of lane l is the row's
+// 64 i + l, bit i of `taken` says that it is out.  It is taken; false where none is left.
+template <int N>
+__device__ __forceinline__ bool take_largest(const float (&v)[N], uint32_t &taken, int lane, uint32_t *index, float *value) {
+    float best = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+        if (!(taken >> i & 1)) best = fmaxf(best, v[i]);
+    best = wave_max_dpp(best);
+    *value = best;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        const uint64_t there = __ballot(!(taken >> i & 1) && v[i] == best);
+        if (there) {
+            const int at = __builtin_ctzll(there);
+            *index = i * 64 + at;
+            if (lane == at) taken |= 1u << i;
+            return true;
+        }
+    }
+    return false;
+}
+
 // The experts of one row from its logits (LDS), by one wavefront: lane i < top returns with the i-th largest logit's expert in
 // `id` and its softmax weight in `weight`.  NaN logits come out as experts in order with NaN weights.
+template <int N>
 __device__ __forceinline__ void choose_experts(const float *logits, uint32_t experts, uint32_t top, int lane, uint32_t *id, float *weight) {
-    float v[kMaxExperts / 64];
+    float v[N];
     bool bad = false;
+    uint32_t taken = 0;
 #pragma unroll
-    for (uint32_t i = 0; i < kMaxExperts / 64; ++i) {
+    for (int i = 0; i < N; ++i) {
         const uint32_t e = i * 64 + lane;
         v[i] = e < experts ? logits[e] : -INFINITY;
+        if (e >= experts) taken |= 1u << i;
         bad = bad || v[i] != v[i];
         if (v[i] != v[i]) v[i] = -INFINITY;
     }
     bad = __any(bad);
-    uint32_t taken = 0;                              // bit i: this lane's value i has been chosen
     float mine = -INFINITY, first = 0.0f;
     *id = 0;
     for (uint32_t t = 0; t < top; ++t) {
-        float best = -INFINITY;
-        uint32_t at = 0xffffffffu;
-#pragma unroll
-        for (uint32_t i = 0; i < kMaxExperts / 64; ++i) {
-            const uint32_t e = i * 64 + lane;
-            if (e < experts && !(taken >> i & 1) && (at == 0xffffffffu || v[i] > best)) {
-                best = v[i];
-                at = e;
-            }
-        }
-        const float top_v = wave_max_dpp(at == 0xffffffffu ? -INFINITY : best);
-        uint32_t cand = at != 0xffffffffu && best == top_v ? at : 0xffffffffu;
-#pragma unroll
-        for (int off = 32; off > 0; off >>= 1) {
-            const uint32_t o = (uint32_t)__shfl_xor((int)cand, off, 64);
-            cand = o < cand ? o : cand;
-        }
-        if (t == 0) first = top_v;
-        if ((uint32_t)lane == cand % 64) taken |= 1u << (cand / 64);
+        uint32_t at = 0;
+        float value;
+        take_largest<N>(v, taken, lane, &at, &value);
+        if (t == 0) first = value;
         if ((uint32_t)lane == t) {
-            mine = top_v;
-            *id = cand;
+            mine = value;
+            *id = at;
         }
     }
     const float e = (uint32_t)lane < top ? expf(mine - first) : 0.0f;
@@ -61,91 +71,93 @@ __device__ __forceinline__ void choose_experts(const float *logits, uint32_t exp
 }
 
 // The scored choice: softmax over all outputs, the `top` largest s + correction out of the best groups.  Lane i < top returns with
-// the i-th chosen output in `id` and its weight in `weight`.  row: the logits (LDS), overwritten; open: LDS of the wavefront, a
-// flag per group.
-__device__ __forceinline__ void choose_scored(float *row, uint32_t *open, const RouteIo &io, int lane, uint32_t *id, float *weight) {
-    constexpr uint32_t N = kMaxExperts / 64;
+// the i-th chosen output in `id` and its weight in `weight`.  NaN: as above.
+template <int N>
+__device__ __forceinline__ void choose_scored(const float *logits, const RouteIo &io, int lane, uint32_t *id, float *weight) {
     float s[N], c[N], mx = -INFINITY, sum = 0.0f;
     bool bad = false;
 #pragma unroll
-    for (uint32_t i = 0; i < N; ++i) {
+    for (int i = 0; i < N; ++i) {
         const uint32_t e = i * 64 + lane;
-        s[i] = e < io.experts ? row[e] : -INFINITY;
+        s[i] = e < io.experts ? logits[e] : -INFINITY;
+        c[i] = e < io.experts ? io.correction[e] : 0.0f;
         bad = bad || s[i] != s[i];
         mx = fmaxf(mx, s[i]);
     }
     bad = __any(bad);
     mx = wave_max_dpp(mx);
 #pragma unroll
-    for (uint32_t i = 0; i < N; ++i) {
-        s[i] = i * 64 + lane < io.experts ? expf(s[i] - mx) : 0.0f;
+    for (int i = 0; i < N; ++i) {
+        s[i] = i * 64u + lane < io.experts ? expf(s[i] - mx) : 0.0f;
         sum += s[i];
     }
     sum = wave_sum_dpp(sum);
-    const uint32_t size = io.experts / io.groups;
-    const bool all = io.keep >= io.groups;
-#pragma unroll
-    for (uint32_t i = 0; i < N; ++i) {
-        const uint32_t e = i * 64 + lane;
-        s[i] /= sum;
-        c[i] = bad || e >= io.experts ? 0.0f : s[i] + io.correction[e];
-        if (!all && e < io.experts) row[e] = c[i];
-    }
-    if (!all) {
-        __builtin_amdgcn_wave_barrier();
-        float best[N];                               // of the groups lane, lane + 64, ..
-#pragma unroll
-        for (uint32_t i = 0; i < N; ++i) {
-            best[i] = -INFINITY;
-            const uint32_t g = i * 64 + lane;
-            if (g < io.groups)
-                for (uint32_t j = 0; j < size; ++j) best[i] = fmaxf(best[i], row[g * size + j]);
-        }
-        __builtin_amdgcn_wave_barrier();
-#pragma unroll
-        for (uint32_t i = 0; i < N; ++i)
-            if (i * 64 + lane < io.groups) row[i * 64 + lane] = best[i];
-        __builtin_amdgcn_wave_barrier();
-#pragma unroll
-        for (uint32_t i = 0; i < N; ++i) {
-            const uint32_t g = i * 64 + lane;
-            if (g >= io.groups) continue;
-            uint32_t ahead = 0;
-            for (uint32_t o = 0; o < io.groups; ++o) ahead += row[o] > best[i] || (row[o] == best[i] && o < g);
-            open[g] = ahead < io.keep;
-        }
-        __builtin_amdgcn_wave_barrier();
-    }
     uint32_t taken = 0;                              // bit i: this lane's value i cannot be chosen (any more)
 #pragma unroll
-    for (uint32_t i = 0; i < N; ++i) {
-        const uint32_t e = i * 64 + lane;
-        if (e >= io.experts || (!all && !open[e / size])) taken |= 1u << i;
+    for (int i = 0; i < N; ++i) {
+        s[i] /= sum;
+        c[i] = bad ? 0.0f : s[i] + c[i];
+        if (i * 64u + lane >= io.experts) taken |= 1u << i;
+    }
+    if (io.keep < io.groups) {
+        // a group's best, then the number of groups ahead of it: value i of lane l belongs to group 64 i + l
+        const uint32_t size = io.experts / io.groups;
+        float best[N];
+        uint32_t ahead[N];
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            best[i] = -INFINITY;
+            ahead[i] = 0;
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            uint32_t g = i * 64 / size, left = size - i * 64 % size;
+            const uint32_t n = io.experts > i * 64u ? (io.experts - i * 64 < 64 ? io.experts - i * 64 : 64) : 0;
+            for (uint32_t l = 0; l < n; ++l) {
+                const float v = lane_value(c[i], (int)l);
+#pragma unroll
+                for (int j = 0; j < N; ++j)
+                    if (j * 64u + lane == g) best[j] = fmaxf(best[j], v);
+                if (--left == 0) {
+                    ++g;
+                    left = size;
+                }
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            const uint32_t n = io.groups > i * 64u ? (io.groups - i * 64 < 64 ? io.groups - i * 64 : 64) : 0;
+            for (uint32_t l = 0; l < n; ++l) {
+                const float v = lane_value(best[i], (int)l);
+#pragma unroll
+                for (int j = 0; j < N; ++j) ahead[j] += v > best[j] || (v == best[j] && i * 64u + l < j * 64u + lane);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            const uint32_t g = (i * 64 + lane) / size;
+            uint32_t rank = 0;
+#pragma unroll
+            for (int j = 0; j < N; ++j) {
+                const uint32_t r = (uint32_t)__shfl((int)ahead[j], (int)(g % 64), 64);
+                if (g / 64 == (uint32_t)j) rank = r;
+            }
+            if (rank >= io.keep) taken |= 1u << i;
+        }
     }
     float mine = 0.0f;
     *id = 0;
     for (uint32_t t = 0; t < io.top; ++t) {
-        float best = -INFINITY, best_s = 0.0f;
         uint32_t at = 0xffffffffu;
+        float value, score = 0.0f;
+        if (take_largest<N>(c, taken, lane, &at, &value)) {
 #pragma unroll
-        for (uint32_t i = 0; i < N; ++i)
-            if (!(taken >> i & 1) && (at == 0xffffffffu || c[i] > best)) {
-                best = c[i];
-                best_s = s[i];
-                at = i * 64 + lane;
-            }
-        const float top_c = wave_max_dpp(best);
-        uint32_t cand = at != 0xffffffffu && best == top_c ? at : 0xffffffffu;
-#pragma unroll
-        for (int off = 32; off > 0; off >>= 1) {
-            const uint32_t o = (uint32_t)__shfl_xor((int)cand, off, 64);
-            cand = o < cand ? o : cand;
+            for (int i = 0; i < N; ++i)
+                if (at / 64 == (uint32_t)i) score = lane_value(s[i], (int)(at % 64));
         }
-        const float cand_s = __shfl(best_s, (int)(cand % 64), 64);
-        if ((uint32_t)lane == cand % 64) taken |= 1u << (cand / 64);
         if ((uint32_t)lane == t) {
-            mine = cand_s;
-            *id = cand;
+            mine = score;
+            *id = at;
         }
     }
     const float total = wave_sum_dpp(mine) + 1e-20f;
@@ -153,10 +165,12 @@ __device__ __forceinline__ void choose_scored(float *row, uint32_t *open, const 
 }
 
 // The experts of row r from its logits (LDS): gates stored; true in the lanes whose expert has a list.
-__device__ __forceinline__ bool choose_row(float *logits, uint32_t *open, const RouteIo &io, uint64_t r, bool store, int lane, uint32_t *id) {
+// N: values per lane.
+template <int N>
+__device__ __forceinline__ bool choose_row(const float *logits, const RouteIo &io, uint64_t r, bool store, int lane, uint32_t *id) {
     float w;
-    if (io.scored) choose_scored(logits, open, io, lane, id, &w);
-    else choose_experts(logits, io.experts, io.top, lane, id, &w);
+    if (io.scored) choose_scored<N>(logits, io, lane, id, &w);
+    else choose_experts<N>(logits, io.experts, io.top, lane, id, &w);
     const bool own = (uint32_t)lane < io.top, listed = own && *id < io.experts - io.identity;
     if (io.identity_gate) {
         const float sum = wave_sum_dpp(own && !listed ? w : 0.0f);
@@ -176,7 +190,6 @@ __global__ void __launch_bounds__(NT)
     constexpr bool LAYER = KIND == ResidualNorm::kBoth, INPUT = KIND == ResidualNorm::kInput;
     typedef float piece __attribute__((ext_vector_type(S)));
     __shared__ float smem[LAYER ? 4 : 1][NW], logits[ROUTE ? kMaxExperts : 1];
-    __shared__ uint32_t open[ROUTE ? kMaxExperts : 1];
     extern __shared__ __attribute__((aligned(16))) uint8_t hs_raw[];     // ROUTE: the row of hn
     const uint64_t r = blockIdx.x;
     const int tid = threadIdx.x;
@@ -350,7 +363,7 @@ __global__ void __launch_bounds__(NT)
         __syncthreads();
         if (wave == 0) {
             uint32_t id;
-            if (choose_row(logits, open, io, r, true, lane, &id)) {
+            if (io.experts <= 64 ? choose_row<1>(logits, io, r, true, lane, &id) : choose_row<kMaxExperts / 64>(logits, io, r, true, lane, &id)) {
                 const uint32_t at = atomicAdd(io.count + id, 1u);
                 if (at < io.pitch) io.list[(uint64_t)id * io.pitch + at] = (uint32_t)(r * io.top + lane);
             }
@@ -365,7 +378,7 @@ template <int ET>
 __global__ void __launch_bounds__(256)
     route_kernel(const uint16_t *__restrict__ h, uint64_t ld, uint32_t rows, RouteIo io) {
     extern __shared__ __attribute__((aligned(16))) float part[];         // [4][ET * 16][17]
-    __shared__ uint32_t cnt[kMaxExperts], base[kMaxExperts], open[4][kMaxExperts];
+    __shared__ uint32_t cnt[kMaxExperts], base[kMaxExperts];
     __shared__ float logits[16][ET * 16 + 1];
     const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), g = lane / 16, c = lane % 16;
     const uint32_t r0 = blockIdx.x * 16, row = r0 + c < rows ? r0 + c : rows - 1;
@@ -408,7 +421,7 @@ __global__ void __launch_bounds__(256)
     for (int q = 0; q < 4; ++q) {
         const uint32_t rr = wave * 4 + q;
         const bool there = r0 + rr < rows;
-        listed[q] = choose_row(logits[rr], open[wave], io, r0 + rr, there, lane, &id[q]) && there;
+        listed[q] = choose_row<(ET + 3) / 4>(logits[rr], io, r0 + rr, there, lane, &id[q]) && there;
         at[q] = listed[q] ? atomicAdd(&cnt[id[q]], 1u) : 0;
     }
     __syncthreads();

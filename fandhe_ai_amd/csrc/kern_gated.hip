@@ -8,6 +8,8 @@ namespace fa {
 namespace k {
 using namespace fa::dev;
 
+int g_gated_lanes = 0;        // tuning: threads across the channels of a block of the scan, 8 or 16
+
 namespace {
 
 // bf16 models: the native exponential and reciprocal (a few ulp); f32 models: the library's
@@ -45,8 +47,14 @@ __device__ __forceinline__ void token_step(const Piece<S> &z, const Piece<S> &u,
 #pragma unroll
     for (int e = 0; e < S; ++e) {
         const float c = u[e] >= 0.0f ? u[e] + 0.5f : logistic<FAST>(u[e]);
-        a[e] = logistic<FAST>(-z[e]);
-        b[e] = logistic<FAST>(z[e]) * c;
+        if constexpr (FAST) {                        // z = 1 / (1 + t), 1 - z = t z; t stays finite
+            const float t = exp2_fast(fminf(-z[e] * kLog2e, 120.0f)), w = __builtin_amdgcn_rcpf(1.0f + t);
+            a[e] = t * w;
+            b[e] = w * c;
+        } else {
+            a[e] = logistic<FAST>(-z[e]);
+            b[e] = logistic<FAST>(z[e]) * c;
+        }
     }
 }
 template <int S, bool FAST>
@@ -77,18 +85,19 @@ __global__ void __launch_bounds__(256) gated_step_kernel(GatedIo io, uint32_t wi
     store_piece<S>((T *)io.out + (uint64_t)r * io.ld_out + c, gated<S, FAST>(s, g, io.out_scale));
 }
 
-// Portions.  A block takes 16 S channels of a sequence and walks its rows in tiles of 128: thread (i, c) has four tokens
-// of S channels, composes them, and the tile's 32 thread rows are scanned inside their wavefronts and through LDS.
-constexpr int kScanWaves = 8, kScanTokens = 4, kScanTile = kScanWaves * 4 * kScanTokens;
-template <typename T, int S>
+// Portions.  A block takes LANES S channels of a sequence and walks its rows in tiles: thread (i, c) has four tokens of S
+// channels, composes them, and the tile's thread rows are scanned inside their wavefronts and through LDS.
+constexpr int kScanWaves = 8, kScanTokens = 4;
+template <typename T, int S, int LANES>
 __global__ void __launch_bounds__(kScanWaves * 64) gated_scan_kernel(GatedIo io, uint32_t width, RaggedRows rr) {
     constexpr bool FAST = sizeof(T) == 2;
+    constexpr int ROWS = 64 / LANES, kScanTile = kScanWaves * ROWS * kScanTokens;
     typedef Piece<S> P;
-    __shared__ P tot_a[2][kScanWaves][16], tot_b[2][kScanWaves][16];
+    __shared__ P tot_a[2][kScanWaves][LANES], tot_b[2][kScanWaves][LANES];
     const uint32_t q = blockIdx.y, row0 = rr.row_start[q], n = rr.row_start[q + 1] - row0;
     if (n == 0) return;
-    const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, lc = lane % 16, group = lane / 16;
-    const uint32_t c = (blockIdx.x * 16 + lc) * S;
+    const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, lc = lane % LANES, group = lane / LANES;
+    const uint32_t c = (blockIdx.x * LANES + lc) * S;
     const bool in = c < width;
     const uint32_t cc = in ? c : 0;
     float *state = io.state + (uint64_t)rr.state_slot[q] * gated_pitch(width) + cc;
@@ -98,7 +107,7 @@ __global__ void __launch_bounds__(kScanWaves * 64) gated_scan_kernel(GatedIo io,
     const P zb = *(const P *)(io.z_bias + cc), ub = *(const P *)(io.u_bias + cc);
     P carry = P(0.0f);
     if (rr.pos[row0] != 0) carry = *(const P *)state;
-    const uint32_t t_own = (wave * 4 + group) * kScanTokens;
+    const uint32_t t_own = (wave * ROWS + group) * kScanTokens;
     P z[kScanTokens], u[kScanTokens], g[kScanTokens];
     auto fetch = [&](uint32_t t0) {
 #pragma unroll
@@ -127,26 +136,26 @@ __global__ void __launch_bounds__(kScanWaves * 64) gated_scan_kernel(GatedIo io,
             A *= a[i];
         }
         if (t0 + kScanTile < n) fetch(t0 + kScanTile);
-        // inclusive over the wavefront's four thread rows
+        // inclusive over the wavefront's thread rows
 #pragma unroll
-        for (int off = 1; off < 4; off *= 2)
+        for (int off = 1; off < ROWS; off *= 2)
 #pragma unroll
             for (int e = 0; e < S; ++e) {
-                const float pa = __shfl_up(A[e], off * 16, 64), pb = __shfl_up(B[e], off * 16, 64);
+                const float pa = __shfl_up(A[e], off * LANES, 64), pb = __shfl_up(B[e], off * LANES, 64);
                 if (group >= off) {
                     B[e] = fmaf(A[e], pb, B[e]);
                     A[e] *= pa;
                 }
             }
-        if (group == 3) {
+        if (group == ROWS - 1) {
             tot_a[buf][wave][lc] = A;
             tot_b[buf][wave][lc] = B;
         }
         P ea, eb;                                    // of the thread rows before this one
 #pragma unroll
         for (int e = 0; e < S; ++e) {
-            ea[e] = __shfl_up(A[e], 16, 64);
-            eb[e] = __shfl_up(B[e], 16, 64);
+            ea[e] = __shfl_up(A[e], LANES, 64);
+            eb[e] = __shfl_up(B[e], LANES, 64);
             if (group == 0) {
                 ea[e] = 1.0f;
                 eb[e] = 0.0f;
@@ -170,26 +179,34 @@ __global__ void __launch_bounds__(kScanWaves * 64) gated_scan_kernel(GatedIo io,
             if (in && t0 + t_own + i < n) store_piece<S>(out + (uint64_t)(t0 + t_own + i) * io.ld_out, gated<S, FAST>(s, gs[i], io.out_scale));
         }
     }
-    if (in && tid < 16) *(P *)state = carry;
+    if (in && tid < LANES) *(P *)state = carry;
 }
 
+template <typename T, int S, int LANES>
+void launch_scan(uint32_t width, const GatedIo &io, const RaggedRows &rr, hipStream_t s) {
+    gated_scan_kernel<T, S, LANES><<<dim3((width + LANES * S - 1) / (LANES * S), rr.batch), kScanWaves * 64, 0, s>>>(io, width, rr);
+}
 template <typename T, int S>
-void launch_gated(uint32_t width, const GatedIo &io, const RaggedRows &rr, uint32_t max_new, hipStream_t s) {
+void launch_gated(uint32_t width, const GatedIo &io, const RaggedRows &rr, uint32_t max_new, int num_cus, hipStream_t s) {
+    // 16 lanes read longer pieces of a row; with too few blocks for the device, 8: half the steps in twice the blocks (us for 4 x 2048
+    // tokens, width 4096 / 2048, 16, 8, 4 lanes: 108, 127, 180 / 84, 58, 86)
+    const bool wide = g_gated_lanes ? g_gated_lanes == 16 : (uint64_t)((width + 16 * S - 1) / (16 * S)) * rr.batch >= (uint64_t)num_cus;
     if (max_new <= 1) gated_step_kernel<T, S><<<dim3((width + 256 * S - 1) / (256 * S), rr.rows), 256, 0, s>>>(io, width, rr);
-    else gated_scan_kernel<T, S><<<dim3((width + 16 * S - 1) / (16 * S), rr.batch), kScanWaves * 64, 0, s>>>(io, width, rr);
+    else if (wide) launch_scan<T, S, 16>(width, io, rr, s);
+    else launch_scan<T, S, 8>(width, io, rr, s);
 }
 
 }  // namespace
 
-void gated_mixer(uint32_t width, const GatedIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, hipStream_t s) {
+void gated_mixer(uint32_t width, const GatedIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, int num_cus, hipStream_t s) {
     if (rr.rows == 0) return;
     const bool vec = width % 4 == 0 && io.ld_zu % 4 == 0 && io.ld_gate % 4 == 0 && io.ld_out % 4 == 0;
     if (is_f32) {
-        if (vec) launch_gated<float, 4>(width, io, rr, max_new, s);
-        else launch_gated<float, 1>(width, io, rr, max_new, s);
+        if (vec) launch_gated<float, 4>(width, io, rr, max_new, num_cus, s);
+        else launch_gated<float, 1>(width, io, rr, max_new, num_cus, s);
     } else {
-        if (vec) launch_gated<uint16_t, 4>(width, io, rr, max_new, s);
-        else launch_gated<uint16_t, 1>(width, io, rr, max_new, s);
+        if (vec) launch_gated<uint16_t, 4>(width, io, rr, max_new, num_cus, s);
+        else launch_gated<uint16_t, 1>(width, io, rr, max_new, num_cus, s);
     }
 }
 

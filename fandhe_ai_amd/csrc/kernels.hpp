@@ -591,7 +591,7 @@ struct GatedIo {
 };
 constexpr uint32_t gated_pitch(uint32_t width) { return (width + 3) / 4 * 4; }
 // max_new: most new tokens of any sequence of the pass
-void gated_mixer(uint32_t width, const GatedIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, hipStream_t s);
+void gated_mixer(uint32_t width, const GatedIo &io, int is_f32, const RaggedRows &rr, uint32_t max_new, int num_cus, hipStream_t s);
 
 // act[0] = softplus(pq[0]), act[1] = 1/2 + softplus(pq[1]): what kXielu reads
 void xielu_constants(const float *pq, float *act, hipStream_t s);

@@ -389,7 +389,7 @@ void enqueue_gated(fa_context *ctx, LayeredState &L, Arena &a, const Layer &l, c
     io.out = element(L, a.o, m.o_at);
     io.ld_out = ld_o;
     io.out_scale = m.out_scale;
-    k::gated_mixer(m.cfg.vdim, io, L.is_f32, rr, max_new, ctx->stream);
+    k::gated_mixer(m.cfg.vdim, io, L.is_f32, rr, max_new, ctx->props.multiProcessorCount, ctx->stream);
 }
 
 // What an attention mixer does to its scores and to their result; y: its f32 columns
@@ -496,7 +496,13 @@ fa_status enqueue_layers(fa_context *ctx, fa_decoder *d, Arena &a, const k::Ragg
     const int f32 = L.is_f32;
     for (size_t i = 0; i < L.rotations.size(); ++i) k::rotation_table(rr.pos, a.cos_sin[i], M, L.rotations[i].dims, L.rotation_freq[i], s);
     if (L.cfg.norm == FA_NORM_BOTH) k::layernorm_rows(a.x, L.layers[0].norm1, a.hn, f32, M, D, ld_hn, eps, s);
-    if (L.cfg.norm == FA_NORM_INPUT_RMS) k::rmsnorm_rows(a.x, L.layers[0].norm1, a.hn, f32, M, D, ld_hn, eps, s);
+    if (L.cfg.norm == FA_NORM_INPUT_RMS) {
+        k::ResidualNorm rn;
+        rn.kind = k::ResidualNorm::kInput;
+        rn.next = L.layers[0].norm1;
+        rn.eps = eps;
+        k::residual_norm(rn, a.x, a.hn, f32, M, D, ld_hn, nullptr, s);
+    }
     for (size_t li = 0; li < L.layers.size(); ++li) {
         const Layer &l = L.layers[li];
         if (L.cfg.norm == FA_NORM_INPUT) k::layernorm_rows(a.x, l.norm1, a.hn, f32, M, D, ld_hn, eps, s);

@@ -120,7 +120,8 @@ fa_status fa_probe_l2_path(fa_context *ctx, const fa_buffer *cold, uint64_t cold
  * key 32: blocks per compute unit the key split of the absorbed form aims at;
  * key 33: grouped-query attention: 1: the plain kernel, 2: the few-rows kernel for every sequence, 3: the many-rows kernel
  *        for every sequence; key 34: blocks per compute unit its key split aims at;
- * key 35: routing of experts: 1: always in the residual update's launch, 2: always in a launch of its own. */
+ * key 35: routing of experts: 1: always in the residual update's launch, 2: always in a launch of its own.
+ * key 36: minimal gated recurrence: threads across the channels of a block of the scan, 8 or 16. */
 fa_status fa_set_tuning(int32_t key, int32_t value);
 
 /* What the context found when it was created: xcd_local = 1 when workgroups b and b + 8 of a launch were seen to

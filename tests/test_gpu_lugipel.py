@@ -104,7 +104,8 @@ def test_mechanism_prompt_then_decode(name, dtype):
 
 
 FORMS = {"attention plain": (33, 1), "attention few rows": (33, 2), "attention many rows": (33, 3), "attention, keys split further": (34, 8),
-         "experts streamed": (29, 4), "experts in tiles": (29, 5), "experts in large tiles": (29, 6), "routed with the norm": (35, 1), "routed apart": (35, 2)}
+         "experts streamed": (29, 4), "experts in tiles": (29, 5), "experts in large tiles": (29, 6), "routed with the norm": (35, 1), "routed apart": (35, 2),
+         "scan of 8 lanes": (36, 8), "scan of 16 lanes": (36, 16)}
 FORM_LAYERS = {
     "all": MECHANISMS["all"],
     "large sizes": [att(heads=12, kv_heads=3, dim=128, vdim=128, window=600, mlp=lc.scored(4, 2, (3, 2), 2, 272)), gru(260, mlp=lc.dense(520))],
@@ -357,7 +358,7 @@ def test_what_was_written_long_ago_is_read_back_from_the_state(width):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_gates_from_closed_to_open(dtype):
+def test_gates_from_closed_to_open(dtype, tune):
     """Channels that never write beside channels that keep nothing; candidates on both sides of zero."""
     cfg = lc.lugipel([gru(64), gru(90)])
     w = lc.weights(cfg, 14)
@@ -368,8 +369,10 @@ def test_gates_from_closed_to_open(dtype):
     toks = lc.tokens(cfg, 300, 14)
     want = oracle.forward(cfg, w, toks)
     dec = lc.make_decoder(ops(), cfg, w, dtype)
-    for sizes in ((300,), (130, 17), (12, 11), (1,)):
-        assert lc.error(portions_of(dec, toks, sizes), want) < tolerance(dtype), sizes
+    for lanes in (8, 16):
+        tune(36, lanes)
+        for sizes in ((300,), (130, 17), (12, 11), (1,)):
+            assert lc.error(portions_of(dec, toks, sizes), want) < tolerance(dtype), sizes
     dec.close()
 
 
