@@ -241,13 +241,16 @@ def _mingru(mx, where):
 
 def _sigmoid_attention(mx, where):
     l = {key: _entry(mx, key, where) for key in ("heads", "kv_heads", "dim", "vdim", "scale")}
-    temp = _entry(mx, "q_temp", where)
-    every = _entry(temp, "every", where + " q_temp")
-    if every != int(every) or every < 1:
-        raise ConfigError("%s: q_temp.every must be a positive whole number" % where)
-    return dict(l, mixer=capi.MIXER_ATTENTION, attention=capi.ATTENTION_HEAD_NORM | capi.ATTENTION_SIGMOID | capi.ATTENTION_HEAD_GATE, kv_from=-1,
-                window=_entry(_entry(mx, "mask", where), "size", where + " mask"), distance=DISTANCE_SPAN,
-                q_temp=_entry(temp, "coef", where + " q_temp"), q_temp_every=int(every))
+    l.update(mixer=capi.MIXER_ATTENTION, attention=capi.ATTENTION_HEAD_NORM | capi.ATTENTION_SIGMOID | capi.ATTENTION_HEAD_GATE, kv_from=-1,
+             distance=DISTANCE_SPAN)
+    if mx.get("mask") is not None:
+        l["window"] = _entry(mx["mask"], "size", where + " mask")
+    if mx.get("q_temp") is not None:
+        every = _entry(mx["q_temp"], "every", where + " q_temp")
+        if every != int(every) or every < 1:
+            raise ConfigError("%s: q_temp.every must be a positive whole number" % where)
+        l.update(q_temp=_entry(mx["q_temp"], "coef", where + " q_temp"), q_temp_every=int(every))
+    return l
 
 
 def _scored_experts(mlp, where):
@@ -257,7 +260,7 @@ def _scored_experts(mlp, where):
     l = {"d_ffn": _entry(_entry(mlp, "expert", where), "ff", where + " expert"), "experts": _entry(router, "experts", at) + identity,
          "identity": identity, "top": _entry(router, "top", at), "glu": capi.GLU_SILU, "route": capi.ROUTE_SCORED,
          "route_scale": _entry(router, "scale", at)}
-    if router.get("groups"):
+    if router.get("groups") is not None:
         l.update(groups=_entry(router["groups"], "count", at + " groups"), groups_kept=_entry(router["groups"], "keep", at + " groups"))
     return l
 

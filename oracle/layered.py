@@ -421,8 +421,10 @@ def sigmoid_attention_mixer(h, w, p, mx, eps):
     T, H, G, d = len(h), mx["heads"], mx["kv_heads"], mx["dim"]
     q = rms_norm((h @ w[p + "q"].T).reshape(T, H, d), w[p + "q.norm"], eps)
     k = rms_norm((h @ w[p + "k"].T).reshape(T, G, d), w[p + "k.norm"], eps)
-    q = q * query_temperature(range(T), mx["q_temp"]["coef"], mx["q_temp"]["every"])[:, None, None]
-    o = sigmoid_attention(q, k, (h @ w[p + "v"].T).reshape(T, G, mx["vdim"]), mx["scale"], mx["mask"]["size"], distance_slopes(H), w[p + "pb"])
+    if mx.get("q_temp"):
+        q = q * query_temperature(range(T), mx["q_temp"]["coef"], mx["q_temp"]["every"])[:, None, None]
+    window = mx["mask"]["size"] if mx.get("mask") else None
+    o = sigmoid_attention(q, k, (h @ w[p + "v"].T).reshape(T, G, mx["vdim"]), mx["scale"], window, distance_slopes(H), w[p + "pb"])
     return (o * sigmoid(h @ w[p + "g"].T)[:, :, None]).reshape(T, -1) @ w[p + "o"].T
 
 

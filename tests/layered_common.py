@@ -98,8 +98,11 @@ def bubetar(layers, width=76, vocab=131, eps=1e-5, softcap=12.0, scale=0.8, rank
 
 
 def sigmoid_attention(heads=6, kv_heads=2, dim=20, vdim=12, window=13, scale=None, coef=0.6, every=8, mlp=None):
-    mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": 1.5 * dim ** -0.5 if scale is None else scale, "mask": {"size": window},
-          "q_temp": {"coef": coef, "every": every}}
+    mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": 1.5 * dim ** -0.5 if scale is None else scale}
+    if window:
+        mx["mask"] = {"size": window}
+    if every:
+        mx["q_temp"] = {"coef": coef, "every": every}
     return {"type": "attention", "mixer": mx, "mlp": mlp}
 
 

@@ -64,7 +64,8 @@ MECHANISMS = {
     "window longer than the sequence": [att(window=4096)],
     "a negative scale": [att(scale=-0.4)],
     "temperature at every position": [att(every=1, coef=0.4)],
-    "no temperature": [att(coef=0.0)],
+    "no temperature": [att(coef=0.0), att(every=None)],
+    "no window": [att(window=None), att(heads=2, kv_heads=1, dim=64, vdim=64, window=None, every=None)],
     "a negative temperature": [att(every=3, coef=-0.3)],
     "recurrence": [gru()],
     "recurrence of one channel": [gru(1)],

@@ -590,6 +590,8 @@ def test_lugipel_configuration_reads_every_size_and_names_what_is_missing():
     bad["layers"][0]["mixer"]["q_temp"]["every"] = 2.5
     with pytest.raises(models.ConfigError, match="every"):
         models.lugipel(bad)
+    bare = models.lugipel_layers(lc.lugipel([lc.sigmoid_attention(window=None, every=None)]))[0]
+    assert bare.get("window", 0) == 0 and bare.get("q_temp", 0.0) == 0.0
 
 
 # ---- batching on a fake decoder ---------------------------------------------------------------------------------
